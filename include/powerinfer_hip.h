@@ -27,7 +27,7 @@ extern "C" {
 typedef void * pi_stream_t;
 
 /* element types: numeric values of enum ggml_type (ggml.h:333-355) */
-enum { PI_TYPE_F32 = 0, PI_TYPE_F16 = 1, PI_TYPE_Q4_0 = 2, PI_TYPE_I32 = 18 };
+enum { PI_TYPE_F32 = 0, PI_TYPE_F16 = 1, PI_TYPE_Q4_0 = 2, PI_TYPE_I32 = 18, PI_TYPE_BF16 = 30 };
 
 enum { PI_OK = 0, PI_E_ARG = -1, PI_E_HIP = -2, PI_E_UNSUPPORTED = -3, PI_E_STATE = -4 };
 
@@ -559,9 +559,72 @@ PI_API int pi_k_embed(int wtype, const void * table, int cols, const int32_t * t
 /* greedy sampling: *token_out = index of the first maximum (llama_sample_token_greedy, llama.cpp:8617-8631) */
 PI_API int pi_k_argmax(const float * logits, int n, int32_t * token_out, pi_stream_t stream);
 
+/* ---- operators of the models described layer by layer (pi_model_create_layers) ----------------------------------------------------
+ * `type` is the storage of activations and caches: PI_TYPE_BF16 (bf16 matrix cores, fp32 accumulation) or PI_TYPE_F32 (fp32 matrix
+ * cores and vector units; nothing is rounded below fp32).  Matrices are BF16 with their inner dimension padded with zeros to a multiple
+ * of 32 (ldw), vectors F32. */
+/* x[t] = rms_norm(table[tokens[t]]) * w */
+PI_API int pi_k_embed_norm(const void * table_bf16, int cols, const int32_t * tokens, int T, const float * w, float eps, float * x, pi_stream_t stream);
+/* two RMS norms of the same rows in one pass: out_a[t] = rms(x[t]) * wa, out_b[t] = rms(x[t]) * wb (wb, out_b may be NULL); rows of the
+ * outputs are ld values apart.  rows (optional): row t of the outputs is made from x[rows[t]].  ol != 0 (BF16, T <= 16): outputs in the
+ * operand layout of pi_k_gemm_bf16_ol over ld columns */
+PI_API int pi_k_norm_pair(int type, const float * x, const int32_t * rows, int T, int cols, float eps, const float * wa, void * out_a,
+                          const float * wb, void * out_b, int ld, int ol, pi_stream_t stream);
+/* y = alpha * W x for several groups at once: group g multiplies W + g * w_gs with its own rows of x.  off == NULL: every group takes
+ * the T rows x + g * x_gs + t * ldx into y + g * y_gs + t * ldy.  off != NULL (n_group + 1 offsets on the device): group g takes the
+ * places s in [off[g], off[g + 1]) of a list; input row = gather ? gather[s] / gather_div : s, output row = s; T bounds the places of one group.
+ * relu2: y = relu(.)^2.  y_f32: y is fp32 whatever `type` is.  Strides count elements. */
+typedef struct pi_group_gemm {
+    const void * W; size_t w_gs; int32_t rows, cols, ldw, n_group;
+    const void * x; size_t x_gs; int32_t ldx, T;
+    void * y; size_t y_gs; int32_t ldy, y_f32, relu2;
+    float alpha;
+    const int32_t * off, * gather; int32_t gather_div;
+} pi_group_gemm;
+PI_API int pi_k_group_gemm(int type, const pi_group_gemm * g, pi_stream_t stream);
+/* (cos, sin)[t][i] of the angles pos[t] * base^(-2i / dims), i < dims / 2 */
+PI_API int pi_k_rope_angles(const int32_t * pos, int T, int dims, double base, void * cs_float2, pi_stream_t stream);
+/* Behind the joint projection of a latent-attention layer, z [T][ldz] = per head [dim | rot_dim], then (own cells) [kv_rank | rot_dim]:
+ * the unrotated query parts to q_un [T][n_head][dim_ld], the rotated ones to q_lat [T][n_head][kd] behind rank_ld values, and
+ * (cache != NULL) the token's cell: normed latent, rotated key part behind rank_ld values, rows of kd values. */
+typedef struct pi_latent_prep {
+    const float * z; int32_t ldz, T, n_head, dim, dim_ld, rot_dim, kv_rank, rank_ld, kd;
+    const void * cs; const float * norm_w; float eps;
+    void * q_un, * q_lat, * cache; const int32_t * cell;
+} pi_latent_prep;
+PI_API int pi_k_latent_prep(int type, const pi_latent_prep * p, pi_stream_t stream);
+/* Attention over cached latents: query rows q_lat [(token, head)][kd] against the cells lists[seq][0 .. n_vis[token]) ; out_lat
+ * [(token, head)][rank_ld] = soft-max weighted latents, the denominator holding exp(sink[head]).  work [n_work]: {first token, first row
+ * among (tokens behind it) x heads, rows, sequence} - at most pi_k_latent_attn_rows rows each
+ * (PI_TYPE_F32: work [T] = each token's sequence, n_parts 1).  n_parts > 1: the cells of every item are
+ * split over that many workgroups and merged (scratch: pi_k_latent_attn_scratch_floats). */
+typedef struct pi_latent_attn {
+    const void * q_lat, * cache; const int32_t * lists; size_t list_ld; const int32_t * work, * n_vis;
+    int32_t n_work, T, n_head, kv_rank, rank_ld, kd, n_parts; float scale; const float * sink; float * scratch; void * out_lat;
+} pi_latent_attn;
+PI_API int    pi_k_latent_attn_rows(int type);
+PI_API int    pi_k_latent_attn_supported(int type, int rank_ld, int kd);
+PI_API size_t pi_k_latent_attn_scratch_floats(int T, int n_head, int rank_ld, int n_parts);
+PI_API int    pi_k_latent_attn(int type, const pi_latent_attn * p, pi_stream_t stream);
+/* rotates the shared key part (rot_dim values behind rank_ld) of cells by delta[cell] positions; cells with delta 0 are left alone */
+PI_API int pi_k_latent_shift(int type, void * cache, int n_cells, int kd, int rank_ld, int rot_dim, double base, const int32_t * delta, pi_stream_t stream);
+/* expert choice of T tokens from router logits z [T][n_expert] (see PI_FFN_MOE): ids, weights [T][n_top] by falling choice score */
+PI_API int pi_k_route(const float * z, int T, int n_expert, int n_top, int n_group, int n_keep, const float * bias, int32_t * ids, float * weights,
+                      pi_stream_t stream);
+/* pairs (token, choice) in expert order, tokens ascending: off [n_expert + 1], perm[place] = pair, inv[pair] = place */
+PI_API int pi_k_moe_sort(const int32_t * ids, int n_pairs, int n_expert, int32_t * off, int32_t * perm, int32_t * inv, pi_stream_t stream);
+/* out[t] = x[t] + (mix[t] + sum over k of weights[t][k] * y[inv[t][k]]); weights == NULL: out = x + mix.  keep (optional) receives a copy */
+PI_API int pi_k_moe_combine(const float * x, const float * mix, const float * y, const int32_t * inv, const float * weights, int n_top, int T, int cols,
+                            float * out, float * keep, pi_stream_t stream);
+/* BF16 matrices: out [rows][ld] = in [rows][cols] padded with zeros; out [n_mat][cols][ld] = each in [rows][cols] transposed, padded with zeros */
+PI_API int pi_k_pad_cols_bf16(const void * in, int64_t rows, int cols, void * out, int ld, pi_stream_t stream);
+PI_API int pi_k_transpose_pad_bf16(const void * in, int n_mat, int rows, int cols, void * out, int ld, pi_stream_t stream);
+/* lockstep decoding on shared cells: after tokens and positions have moved on, n_vis[t] += 1 and cell[t] = lists[seq[t]][n_vis[t] - 1] */
+PI_API int pi_k_cells_advance(int T, const int32_t * seq, const int32_t * lists, size_t list_ld, int32_t * n_vis, int32_t * cell, int32_t * step, pi_stream_t stream);
+
 /* ---- decode loop with resident weights ------------------------------------------------------------- */
 
-enum { PI_ARCH_LLAMA = 0, PI_ARCH_FALCON = 1 };
+enum { PI_ARCH_LLAMA = 0, PI_ARCH_FALCON = 1, PI_ARCH_LERASUN = 2 };
 
 /* the llama_hparams fields this path reads (llama.cpp:1207-1270) */
 typedef struct pi_hparams {
@@ -579,8 +642,45 @@ enum {
     PI_T_FFN_NORM, PI_T_FFN_GATE, PI_T_FFN_UP, PI_T_FFN_DOWN_T,
     PI_T_FC1, PI_T_FC2, PI_T_GPU_IDX, PI_T_GPU_BUCKET,
     PI_T_NEURON_RATE,
+    /* models created by pi_model_create_layers (matrices BF16, vectors F32): the norm behind the embedding (global), latent attention
+     * (query, joint latent + shared-key projection, its norm, per-head key / value expansions, sinks), router and stacked experts */
+    PI_T_EMBD_NORM,
+    PI_T_MIX_Q, PI_T_MIX_DKV, PI_T_MIX_DKV_NORM, PI_T_MIX_UK, PI_T_MIX_UV, PI_T_MIX_SINK,
+    PI_T_ROUTER, PI_T_ROUTER_BIAS, PI_T_EXPERT_UP, PI_T_EXPERT_DOWN,
     PI_T_COUNT
 };
+
+/*
+ * Models whose layers are described one by one.  A layer is  x + (mixer(norm_a(x)) + ffn(norm_b(x)))  (both of the same x, each part
+ * with its own RMS norm; tensors PI_T_ATTN_NORM and PI_T_FFN_NORM), or without the second part (PI_FFN_NONE).
+ *
+ * PI_MIXER_LATENT: multi-head attention over a cached low-rank latent.  PI_T_MIX_Q [n_head * (dim + rot_dim)][n_embd] gives each head
+ *   an unrotated and a rotated query part; PI_T_MIX_DKV [kv_rank + rot_dim][n_embd] gives the latent (RMS norm with PI_T_MIX_DKV_NORM
+ *   follows) and one rotated key part shared by the heads, which together are a cell of the layer's cache.  PI_T_MIX_UK
+ *   [n_head * dim][kv_rank] and PI_T_MIX_UV [n_head * vdim][kv_rank] expand a head's keys and values from the latent; scores are
+ *   multiplied by `scale`; PI_T_MIX_SINK [n_head] adds exp(sink) to each head's soft-max denominator; PI_T_WO [n_embd][n_head * vdim].
+ *   Rotation: neighbouring pairs, frequency rot_base^(-2i / rot_dim).  kv_from >= 0: the layer has no PI_T_MIX_DKV and reads the cells of
+ *   that (earlier) layer.
+ * PI_FFN_MOE: PI_T_ROUTER [n_expert][n_embd] and PI_T_ROUTER_BIAS [n_expert]; sigmoid scores, choice by score + bias inside the best
+ *   n_group_keep of n_group groups (a group counts the sum of its two best), weights = the chosen scores over their sum;
+ *   PI_T_EXPERT_UP [n_expert * expert_ff][n_embd] and PI_T_EXPERT_DOWN [n_expert * n_embd][expert_ff] hold the experts one behind the
+ *   other, activation relu(z)^2.
+ */
+enum { PI_MIXER_LATENT = 0 };
+enum { PI_FFN_NONE = 0, PI_FFN_MOE = 1 };
+typedef struct pi_layer_desc {
+    int32_t mixer, n_head, dim, rot_dim, vdim, kv_rank, kv_from;
+    float   scale;
+    double  rot_base;
+    int32_t ffn, n_expert, n_top, n_group, n_group_keep, expert_ff;
+} pi_layer_desc;
+typedef struct pi_layers_opts {
+    int32_t compute;         /* PI_TYPE_BF16: activations and caches in bf16, fp32 accumulation (residual, norms, router, scores in fp32);
+                              * PI_TYPE_F32: everything in fp32 */
+    float   logit_scale;     /* logits are multiplied by this */
+    float   norm_offset;     /* added to the weights of the model's own norms (1 for weights stored around zero); not to PI_T_MIX_DKV_NORM */
+    int32_t max_batch;       /* most tokens the step buffers hold; longer steps run in several passes (0: 2048) */
+} pi_layers_opts;
 
 /* The ggml_cuda_* boundary (include/ggml_backend_abi.h) keeps single-token nodes in a window until it knows whether they form a block
  * it computes in one launch: llm_build_ffn_sparse's sequence (llama.cpp:4652-4757), with every neuron on the device, becomes pi_k_gemv +
@@ -595,6 +695,11 @@ typedef struct pi_model pi_model;
 /* llama_load_model_from_file + llama_new_context_with_model (llama.cpp:9789, 9819) without the file
  * format: the caller hands over tensors one by one. */
 PI_API pi_model * pi_model_create(const pi_hparams * hp);
+/* the same for a model described layer by layer: hp->arch, n_embd, n_vocab, n_ctx and norm_eps are read, the rest comes from the
+ * descriptions.  Every pi_model_* call below works on such a model except the ones about sparse FFN rows (rest_on_gpu, capture of
+ * predictor logits, unions, time_section); its sequences live in one cache of shared cells (pi_model_kv_cells_init; pi_model_decode and
+ * pi_model_batch_init set one up with n_ctx cells per sequence where the caller has not). */
+PI_API pi_model * pi_model_create_layers(const pi_hparams * hp, const pi_layers_opts * opts, const pi_layer_desc * layers, int n_layer);
 PI_API void       pi_model_free(pi_model * m);
 
 /*
@@ -679,6 +784,13 @@ PI_API int pi_model_batch_kv_seq_cp(pi_model * m, int src, int dst, int p0, int 
 PI_API int pi_model_kv_cells_init(pi_model * m, int n_cells);
 PI_API int pi_model_kv_cells_decode(pi_model * m, const int32_t * tokens, const int32_t * positions, const uint32_t * seq_masks, int n_tokens,
                                     int32_t * next_tokens, float * logits_out);
+/* One step of any number of tokens: the next tokens of several sequences behind one another (portions of prompts and single decoded
+ * tokens alike; a sequence's tokens in ascending position).  want[n_want]: indices among the step's tokens whose next token (greedy)
+ * and, if logits_out != NULL, logits [n_want][n_vocab] are returned.  Models created by pi_model_create_layers take any free cells
+ * (a pool of n cells holds n tokens, however it was cut up before); the other models run the step in pieces of up to 16 tokens, which
+ * each need a run of free cells.  PI_E_STATE: not enough free cells; nothing has been evaluated or stored. */
+PI_API int pi_model_kv_cells_step(pi_model * m, const int32_t * tokens, const int32_t * positions, const uint32_t * seq_masks, int n_tokens,
+                                  const int32_t * want, int n_want, int32_t * next_tokens, float * logits_out);
 PI_API int pi_model_kv_cells_seq_rm(pi_model * m, int seq, int p0, int p1);
 PI_API int pi_model_kv_cells_seq_cp(pi_model * m, int src, int dst, int p0, int p1);
 PI_API int pi_model_kv_cells_seq_keep(pi_model * m, int seq);
@@ -701,6 +813,9 @@ PI_API int pi_model_batch_dense_layers(pi_model * m);
  * token loop then needs no host step and replays as a HIP graph.  Q4_0 layers at n_embd 4096; the VRAM split is unchanged. */
 PI_API int pi_model_set_rest_on_gpu(pi_model * m, int enable);
 PI_API int pi_model_set_capture(pi_model * m, int enable);
+/* with capture enabled, a model described layer by layer also keeps the residual stream behind every layer for the last pass of a step:
+ * out [n_layer][n_tokens][n_embd]; returns n_tokens or a negative error (out may be NULL) */
+PI_API int pi_model_get_streams(pi_model * m, float * out);
 PI_API int pi_model_get_capture(pi_model * m, float * ffn_out, float * pred_logits, int32_t * n_active, float * ffn_src);
 
 /*

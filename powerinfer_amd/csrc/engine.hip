@@ -23,7 +23,7 @@ namespace {
 size_t row_bytes(int type, int64_t ne0) {
     switch (type) {
         case PI_TYPE_F32: case PI_TYPE_I32: return (size_t)ne0 * 4;
-        case PI_TYPE_F16:  return (size_t)ne0 * 2;
+        case PI_TYPE_F16: case PI_TYPE_BF16: return (size_t)ne0 * 2;
         case PI_TYPE_Q4_0: return (size_t)(ne0 / 32) * 18;
         default: return 0;
     }
@@ -446,6 +446,7 @@ void pi_model_free(pi_model * m) {
     for (hipEvent_t e : m->ev_join) if (e) (void)hipEventDestroy(e);
     if (m->stream2) (void)hipStreamDestroy(m->stream2);
     if (m->cold) pi::cold_destroy(m->cold);
+    if (m->lay) pi::layers_destroy(m);
     pi::batch_destroy(m);
     if (m->ws) pi_workspace_destroy(m->ws);
     for (void * p : m->owned) pi_free(p);
@@ -457,6 +458,7 @@ void pi_model_free(pi_model * m) {
 int pi_model_set_tensor(pi_model * m, int layer, int kind, int type, const void * data, int64_t ne0, int64_t ne1, int on_device) {
     if (!m || !data || kind < 0 || kind >= PI_T_COUNT || ne0 <= 0 || ne1 <= 0) return pi::fail(PI_E_ARG, "pi_model_set_tensor: bad arguments");
     if (m->finalized) return pi::fail(PI_E_STATE, "pi_model_set_tensor: model already finalized");
+    if (kind == PI_T_EMBD_NORM) return upload_tensor(m, m->embd_norm, type, data, ne0, ne1, on_device);
     if (kind <= PI_T_OUTPUT) return upload_tensor(m, m->glob[kind], type, data, ne0, ne1, on_device);
     if (layer < 0 || layer >= m->hp.n_layer) return pi::fail(PI_E_ARG, "pi_model_set_tensor: layer out of range");
     Tensor & t = m->L(layer, kind);
@@ -556,6 +558,7 @@ int pi_model_finalize(pi_model * m) {
     const pi_hparams & hp = m->hp;
     const int d = hp.n_embd, ff = hp.n_ff, gqa = m->gqa;
     PI_HIP_TRY(hipStreamCreateWithFlags(&m->stream, hipStreamNonBlocking));
+    if (m->lay) return pi::layers_finalize(m);
     {
         const char * nb = getenv("PI_NO_BRANCH");          // PI_NO_BRANCH=1: Falcon layers run their two branches one after the other
         if (hp_arch_is_falcon(m) && !(nb && nb[0] == '1')) {
@@ -736,6 +739,7 @@ int pi_model_finalize(pi_model * m) {
 
 int pi_model_kv_clear(pi_model * m) {
     if (!m || !m->finalized) return pi::fail(PI_E_STATE, "pi_model_kv_clear: model not finalized");
+    if (m->lay) { if (KvCells * kv = pi::layers_cells(m)) kv->clear(); return PI_OK; }
     const size_t kv = (size_t)m->hp.n_layer * m->hp.n_head_kv * m->hp.n_ctx * m->hd;
     PI_HIP_TRY(hipStreamSynchronize(m->stream));
     PI_TRY(pi_memset(m->k_cache, 0, kv * 2));
@@ -747,16 +751,19 @@ int pi_model_kv_clear(pi_model * m) {
 
 int pi_model_kv_seq_rm(pi_model * m, int p0, int p1) {
     if (!m || !m->finalized) return pi::fail(PI_E_STATE, "pi_model_kv_seq_rm: model not finalized");
+    if (m->lay) return pi::layers_seq_edit(m, -1, p0, p1, 0, false);
     return pi::kv_edit(m, m->k_cache, m->v_cache, m->d_pos, m->kv_pos, p0, p1, 0, false);
 }
 
 int pi_model_kv_seq_shift(pi_model * m, int p0, int p1, int delta) {
     if (!m || !m->finalized) return pi::fail(PI_E_STATE, "pi_model_kv_seq_shift: model not finalized");
+    if (m->lay) return pi::layers_seq_edit(m, -1, p0, p1, delta, true);
     return pi::kv_edit(m, m->k_cache, m->v_cache, m->d_pos, m->kv_pos, p0, p1, delta, true);
 }
 
 int pi_model_decode(pi_model * m, const int32_t * tokens, int n_tokens, int n_past, float * logits_out) {
     if (!m || !m->finalized) return pi::fail(PI_E_STATE, "pi_model_decode: model not finalized");
+    if (m->lay) return pi::layers_decode(m, tokens, n_tokens, n_past, logits_out);
     if (!m->kv_pos.empty()) return pi::fail(PI_E_STATE, "pi_model_decode: the KV cells' positions are not contiguous (shift the cells behind a removed range first)");
     if (!tokens || n_tokens <= 0 || n_past < 0 || n_past + n_tokens > m->hp.n_ctx) return pi::fail(PI_E_ARG, "pi_model_decode: token range exceeds the context");
     for (int i = 0; i < n_tokens; ++i)
@@ -802,6 +809,7 @@ int pi_model_decode(pi_model * m, const int32_t * tokens, int n_tokens, int n_pa
 
 int pi_model_generate(pi_model * m, int n_steps, int32_t * out_tokens, float * ms_out) {
     if (!m || !m->finalized) return pi::fail(PI_E_STATE, "pi_model_generate: model not finalized");
+    if (m->lay) return pi::layers_generate(m, 1, n_steps, out_tokens, ms_out);
     if (n_steps <= 0 || n_steps > m->max_steps || !out_tokens) return pi::fail(PI_E_ARG, "pi_model_generate: bad step count");
     if (!m->kv_pos.empty()) return pi::fail(PI_E_STATE, "pi_model_generate: the KV cells' positions are not contiguous (shift the cells behind a removed range first)");
     int32_t pos = 0;
@@ -850,6 +858,7 @@ int pi_model_generate(pi_model * m, int n_steps, int32_t * out_tokens, float * m
 }
 
 int pi_model_time_section(pi_model * m, int section, int rounds, float * ms_total, int * launches) {
+    if (m && m->lay) return pi::fail(PI_E_UNSUPPORTED, "pi_model_time_section: about sparse FFN rows; this model has none");
     if (!m || !m->finalized || !ms_total || !launches || rounds <= 0) return pi::fail(PI_E_ARG, "pi_model_time_section: bad arguments");
     if (m->hybrid) return pi::fail(PI_E_UNSUPPORTED, "pi_model_time_section: not available for hybrid models");
     const pi_hparams & hp = m->hp;
@@ -944,6 +953,7 @@ int pi_model_set_capture(pi_model * m, int enable) {
 }
 
 int pi_model_get_capture(pi_model * m, float * ffn_out, float * pred_logits, int32_t * n_active, float * ffn_src) {
+    if (m && m->lay) return pi::fail(PI_E_UNSUPPORTED, "pi_model_get_capture: about sparse FFN rows; this model has none");
     if (!m || !m->finalized) return pi::fail(PI_E_STATE, "pi_model_get_capture: model not finalized");
     PI_HIP_TRY(hipStreamSynchronize(m->stream));
     if (ffn_out) PI_TRY(pi_memcpy_d2h(ffn_out, m->cap_ffn, sizeof(float) * (size_t)m->hp.n_layer * m->hp.n_embd));
@@ -965,6 +975,7 @@ int pi_model_get_capture(pi_model * m, float * ffn_out, float * pred_logits, int
 }
 
 int pi_model_step_active(pi_model * m, int32_t * per_step_total, int n_steps) {
+    if (m && m->lay) return pi::fail(PI_E_UNSUPPORTED, "pi_model_step_active: about sparse FFN rows; this model has none");
     if (!m || !m->finalized || !per_step_total || n_steps <= 0 || n_steps > m->max_steps) return pi::fail(PI_E_ARG, "pi_model_step_active: bad arguments");
     PI_HIP_TRY(hipStreamSynchronize(m->stream));
     return pi_memcpy_d2h(per_step_total, m->d_out_active, sizeof(int32_t) * n_steps);

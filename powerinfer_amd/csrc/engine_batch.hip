@@ -31,13 +31,10 @@ struct BatchState {
     __half *h16 = nullptr;                             //                     and the FFN's hidden vector
     // One KV cache whose cells are shared between sequences (llama_kv_cache, llama.cpp:1683-1848): a cell holds a position and a set of
     // sequence ids; K cells [n_layer][n_cells][n_embd_gqa] and transposed values [n_layer][n_embd_gqa][n_cells] as the reference lays them
-    // out.  Host side: the cells' positions (-1: free), sequence sets (bit s) and the ring's search start.
+    // out; the host side of it is kv.
     bool unified = false;
-    int n_cells = 0, head = 0, n_kv = 0;
-    std::vector<int32_t> cell_pos;
-    std::vector<uint32_t> cell_seq;
-    std::vector<int32_t> cell_delta;                   // position shifts not yet applied to the K rows
-    bool has_shift = false;
+    int n_cells = 0, n_kv = 0;
+    KvCells kv;
     int32_t * d_delta = nullptr;
     __half *cells_k = nullptr, *cells_v = nullptr;
     float *cells_mask = nullptr, *kq_scale = nullptr;  // device: [16][n_cells] mask rows of a step, 1 / sqrt(head size)
@@ -699,6 +696,7 @@ int pi_model_batch_dense_layers(pi_model * m) {
 int pi_model_batch_init(pi_model * m, int n_seq) {
     if (!m || !m->finalized) return pi::fail(PI_E_STATE, "pi_model_batch_init: model not finalized");
     if (n_seq < 1 || n_seq > 16) return pi::fail(PI_E_ARG, "pi_model_batch_init: 1 <= n_seq <= 16");
+    if (m->lay) return pi::layers_batch_init(m, n_seq);
     if (m->batch) return pi::fail(PI_E_STATE, "pi_model_batch_init: already initialised");
     if (!m->rope_table || !pi_k_attn_fused_supported(m->hd, m->hp.n_ctx)) return pi::fail(PI_E_UNSUPPORTED, "pi_model_batch_init: head size or context outside the fused attention kernel (pi_k_attn_fused_supported)");
     const bool q4_route = q4_steps_unsupported(m) == nullptr;
@@ -716,6 +714,7 @@ int pi_model_batch_init(pi_model * m, int n_seq) {
 }
 
 int pi_model_batch_decode(pi_model * m, const int32_t * tokens, const int32_t * positions, int32_t * next_tokens, float * logits_out) {
+    if (m && m->lay) return pi::layers_batch_decode(m, tokens, positions, next_tokens, logits_out);
     if (!m || !m->batch) return pi::fail(PI_E_STATE, "pi_model_batch_decode: pi_model_batch_init first");
     if (!tokens || !positions) return pi::fail(PI_E_ARG, "pi_model_batch_decode: null pointer");
     BatchState * b = m->batch;
@@ -737,6 +736,7 @@ int pi_model_batch_decode(pi_model * m, const int32_t * tokens, const int32_t * 
 }
 
 int pi_model_batch_generate(pi_model * m, int n_steps, int32_t * out_tokens, float * ms_out) {
+    if (m && m->lay) return pi::layers_generate(m, 0, n_steps, out_tokens, ms_out);
     if (!m || !m->batch) return pi::fail(PI_E_STATE, "pi_model_batch_generate: pi_model_batch_init first");
     BatchState * b = m->batch;
     if (n_steps <= 0 || n_steps > b->max_steps || !out_tokens) return pi::fail(PI_E_ARG, "pi_model_batch_generate: bad step count");
@@ -780,6 +780,7 @@ int pi_model_batch_generate(pi_model * m, int n_steps, int32_t * out_tokens, flo
 // so "copy" really copies: cells [p0, p1) of src become the same cells of dst, which must hold exactly p0 cells (a shared prompt
 // prefix is evaluated once and handed to the other sequences).
 int pi_model_batch_kv_seq_rm(pi_model * m, int seq, int p0, int p1) {
+    if (m && m->lay) return pi::layers_seq_edit(m, seq, p0, p1, 0, false);
     if (!m || !m->batch || seq < 0 || seq >= m->batch->n_seq) return pi::fail(PI_E_ARG, "pi_model_batch_kv_seq_rm: bad sequence");
     BatchState * b = m->batch;
     if ((int)b->kv_pos.size() != b->n_seq) b->kv_pos.resize(b->n_seq);
@@ -787,6 +788,7 @@ int pi_model_batch_kv_seq_rm(pi_model * m, int seq, int p0, int p1) {
 }
 
 int pi_model_batch_kv_seq_shift(pi_model * m, int seq, int p0, int p1, int delta) {
+    if (m && m->lay) return pi::layers_seq_edit(m, seq, p0, p1, delta, true);
     if (!m || !m->batch || seq < 0 || seq >= m->batch->n_seq) return pi::fail(PI_E_ARG, "pi_model_batch_kv_seq_shift: bad sequence");
     BatchState * b = m->batch;
     if ((int)b->kv_pos.size() != b->n_seq) b->kv_pos.resize(b->n_seq);
@@ -794,6 +796,7 @@ int pi_model_batch_kv_seq_shift(pi_model * m, int seq, int p0, int p1, int delta
 }
 
 int pi_model_batch_kv_seq_cp(pi_model * m, int src, int dst, int p0, int p1) {
+    if (m && m->lay) return pi::layers_seq_cp(m, src, dst, p0, p1);
     if (!m || !m->batch || src < 0 || dst < 0 || src >= m->batch->n_seq || dst >= m->batch->n_seq || src == dst)
         return pi::fail(PI_E_ARG, "pi_model_batch_kv_seq_cp: bad sequences");
     BatchState * b = m->batch;
@@ -822,6 +825,7 @@ int pi_model_batch_kv_seq_cp(pi_model * m, int src, int dst, int p0, int p1) {
 // ---- one KV cache with cells shared between sequences ----------------------------------------------------------------------------
 int pi_model_kv_cells_init(pi_model * m, int n_cells) {
     if (!m || !m->finalized) return pi::fail(PI_E_STATE, "pi_model_kv_cells_init: model not finalized");
+    if (m->lay) return pi::layers_cells_init(m, n_cells);
     if (m->cells) return pi::fail(PI_E_STATE, "pi_model_kv_cells_init: already initialised");
     if (n_cells < 32 || n_cells % 32) return pi::fail(PI_E_ARG, "pi_model_kv_cells_init: n_cells must be a multiple of 32, at least 32");
     const bool q4_route = q4_steps_unsupported(m) == nullptr;
@@ -832,9 +836,7 @@ int pi_model_kv_cells_init(pi_model * m, int n_cells) {
     if (!b) return PI_E_HIP;
     b->unified = true;
     b->n_cells = n_cells;
-    b->cell_pos.assign(n_cells, -1);
-    b->cell_seq.assign(n_cells, 0u);
-    b->cell_delta.assign(n_cells, 0);
+    b->kv.init(n_cells);
     const size_t per_layer = (size_t)n_cells * m->gqa;
     b->cells_k = m->alloc<__half>(per_layer * m->hp.n_layer); b->cells_v = m->alloc<__half>(per_layer * m->hp.n_layer);
     b->cells_mask = m->alloc<float>((size_t)16 * n_cells); b->kq_scale = m->alloc<float>(1); b->d_delta = m->alloc<int32_t>(n_cells);
@@ -848,23 +850,13 @@ int pi_model_kv_cells_init(pi_model * m, int n_cells) {
     return PI_OK;
 }
 
-// llama_kv_cache_find_slot (llama.cpp:1683-1730): n contiguous free cells, searched from the ring's head, wrapping once
-static bool cells_find_slot(BatchState * b, int n) {
-    const int n_ctx = b->n_cells;
-    if (n > n_ctx) return false;
-    int n_tested = 0;
-    while (true) {
-        if (b->head + n > n_ctx) { n_tested += n_ctx - b->head; b->head = 0; continue; }
-        bool found = true;
-        for (int i = 0; i < n; ++i)
-            if (b->cell_pos[b->head + i] >= 0) { found = false; b->head += i + 1; n_tested += i + 1; break; }
-        if (found) return true;
-        if (n_tested >= n_ctx) return false;
-    }
-}
-
 int pi_model_kv_cells_decode(pi_model * m, const int32_t * tokens, const int32_t * positions, const uint32_t * seq_masks, int n_tokens,
                              int32_t * next_tokens, float * logits_out) {
+    if (m && m->lay) {
+        std::vector<int32_t> all(n_tokens > 0 ? n_tokens : 0);
+        for (int t = 0; t < (int)all.size(); ++t) all[t] = t;
+        return pi::layers_step(m, tokens, positions, seq_masks, n_tokens, all.data(), n_tokens, next_tokens, logits_out);
+    }
     if (!m || !m->cells) return pi::fail(PI_E_STATE, "pi_model_kv_cells_decode: pi_model_kv_cells_init first");
     if (!tokens || !positions || !seq_masks || n_tokens < 1 || n_tokens > 16) return pi::fail(PI_E_ARG, "pi_model_kv_cells_decode: 1 <= n_tokens <= 16");
     BatchState * b = m->cells;
@@ -872,31 +864,27 @@ int pi_model_kv_cells_decode(pi_model * m, const int32_t * tokens, const int32_t
         if (tokens[t] < 0 || tokens[t] >= m->hp.n_vocab) return pi::fail(PI_E_ARG, "pi_model_kv_cells_decode: token id out of range");
         if (positions[t] < 0 || seq_masks[t] == 0) return pi::fail(PI_E_ARG, "pi_model_kv_cells_decode: a token needs a position and at least one sequence");
     }
-    if (!cells_find_slot(b, n_tokens)) return pi::fail(PI_E_STATE, "pi_model_kv_cells_decode: no run of free cells for the step (llama_kv_cache_find_slot failed)");
+    KvCells & kv = b->kv;
+    if (!kv.find_run(n_tokens)) return pi::fail(PI_E_STATE, "pi_model_kv_cells_decode: no run of free cells for the step (llama_kv_cache_find_slot failed)");
     for (int t = 0; t < n_tokens; ++t) {
-        b->slot[t] = b->head + t;
-        b->cell_pos[b->head + t] = positions[t];
-        b->cell_seq[b->head + t] |= seq_masks[t];
+        b->slot[t] = kv.head + t;
+        kv.take(kv.head + t, positions[t], seq_masks[t]);
     }
-    // the cells a step looks at: up to the last one in use, at least 32 (llama_kv_cache_cell_max, llama.cpp:1735-1743, 6842)
-    int cell_max = 0;
-    for (int i = b->n_cells - 1; i > 0; --i) if (b->cell_pos[i] >= 0 && b->cell_seq[i]) { cell_max = i + 1; break; }
-    b->n_kv = std::min(b->n_cells, std::max(32, cell_max));
+    b->n_kv = kv.n_kv();
     // mask rows (llama.cpp:6506-6531): a cell is hidden from token t unless it belongs to t's sequence and its position is not beyond t's
     std::vector<float> mask((size_t)n_tokens * b->n_cells, 0.0f);
     for (int t = 0; t < n_tokens; ++t) {
         const int seq = __builtin_ctz(seq_masks[t]);               // the reference masks by the token's first sequence id
         for (int i = 0; i < b->n_kv; ++i)
-            if (!(b->cell_seq[i] >> seq & 1u) || b->cell_pos[i] > positions[t]) mask[(size_t)t * b->n_cells + i] = -INFINITY;
+            if (!(kv.seq[i] >> seq & 1u) || kv.pos[i] > positions[t]) mask[(size_t)t * b->n_cells + i] = -INFINITY;
     }
     b->n_seq = n_tokens;
-    if (b->has_shift) {          // pending position shifts: the K rows are rotated ahead of the step's layers (llm_build_k_shift runs first in the graph)
-        PI_HIP_TRY(hipMemcpyAsync(b->d_delta, b->cell_delta.data(), sizeof(int32_t) * b->n_cells, hipMemcpyHostToDevice, m->stream));
+    if (kv.has_shift) {          // pending position shifts: the K rows are rotated ahead of the step's layers (llm_build_k_shift runs first in the graph)
+        PI_HIP_TRY(hipMemcpyAsync(b->d_delta, kv.delta.data(), sizeof(int32_t) * b->n_cells, hipMemcpyHostToDevice, m->stream));
         PI_HIP_TRY(hipStreamSynchronize(m->stream));
         PI_TRY(pi_k_k_shift_cells(b->cells_k, m->hp.n_layer, b->n_cells, m->hp.n_head_kv, m->hd, m->hp.arch == PI_ARCH_FALCON ? 2 : 0, m->theta_scale,
                                   m->freq_scale, b->d_delta, m->stream));
-        b->has_shift = false;
-        std::fill(b->cell_delta.begin(), b->cell_delta.end(), 0);
+        kv.shift_done();
     }
     PI_HIP_TRY(hipMemcpyAsync(b->d_tokens, tokens, sizeof(int32_t) * n_tokens, hipMemcpyHostToDevice, m->stream));
     PI_HIP_TRY(hipMemcpyAsync(b->d_pos, positions, sizeof(int32_t) * n_tokens, hipMemcpyHostToDevice, m->stream));
@@ -905,93 +893,94 @@ int pi_model_kv_cells_decode(pi_model * m, const int32_t * tokens, const int32_t
     PI_HIP_TRY(hipStreamSynchronize(m->stream));
     PI_TRY(batch_step(m, b));
     PI_HIP_TRY(hipStreamSynchronize(m->stream));
-    b->head += n_tokens;                                          // llama_decode moves the ring's head past the step's cells and wraps it
-    if (b->head >= b->n_cells) b->head = 0;                       // (llama.cpp:6936-6943)
+    kv.move_head(kv.head + n_tokens);
     if (next_tokens) PI_TRY(pi_memcpy_d2h(next_tokens, b->d_tokens, sizeof(int32_t) * n_tokens));
     if (logits_out) PI_TRY(pi_memcpy_d2h(logits_out, b->logits, sizeof(float) * (size_t)n_tokens * m->hp.n_vocab));
     return PI_OK;
 }
 
-// llama_kv_cache_seq_rm (llama.cpp:1757-1785): seq < 0 removes the range from every sequence; p1 < 0: to the end
+namespace {
+KvCells * cells_of(pi_model * m) { return !m ? nullptr : m->lay ? pi::layers_cells(m) : m->cells ? &m->cells->kv : nullptr; }
+}
+
 int pi_model_kv_cells_seq_rm(pi_model * m, int seq, int p0, int p1) {
-    if (!m || !m->cells || seq >= 32) return pi::fail(PI_E_ARG, "pi_model_kv_cells_seq_rm: bad arguments");
-    BatchState * b = m->cells;
-    int new_head = b->n_cells;
-    if (p0 < 0) p0 = 0;
-    if (p1 < 0) p1 = INT32_MAX;
-    for (int i = 0; i < b->n_cells; ++i) {
-        if (b->cell_pos[i] >= p0 && b->cell_pos[i] < p1) {
-            if (seq < 0) b->cell_seq[i] = 0;
-            else if (b->cell_seq[i] >> seq & 1u) b->cell_seq[i] &= ~(1u << seq);
-            else continue;
-            if (b->cell_seq[i] == 0) { b->cell_pos[i] = -1; if (new_head == b->n_cells) new_head = i; }
-        }
-    }
-    if (new_head != b->n_cells) b->head = new_head;
+    KvCells * kv = cells_of(m);
+    if (!kv || seq >= 32) return pi::fail(PI_E_ARG, "pi_model_kv_cells_seq_rm: bad arguments");
+    kv->seq_rm(seq, p0, p1);
     return PI_OK;
 }
 
-// llama_kv_cache_seq_cp (llama.cpp:1787-1803): the cells of src in [p0, p1) join dst as well; nothing is copied
 int pi_model_kv_cells_seq_cp(pi_model * m, int src, int dst, int p0, int p1) {
-    if (!m || !m->cells || src < 0 || dst < 0 || src >= 32 || dst >= 32) return pi::fail(PI_E_ARG, "pi_model_kv_cells_seq_cp: bad arguments");
-    BatchState * b = m->cells;
-    if (p0 < 0) p0 = 0;
-    if (p1 < 0) p1 = INT32_MAX;
-    b->head = 0;
-    for (int i = 0; i < b->n_cells; ++i)
-        if ((b->cell_seq[i] >> src & 1u) && b->cell_pos[i] >= p0 && b->cell_pos[i] < p1) b->cell_seq[i] |= 1u << dst;
+    KvCells * kv = cells_of(m);
+    if (!kv || src < 0 || dst < 0 || src >= 32 || dst >= 32) return pi::fail(PI_E_ARG, "pi_model_kv_cells_seq_cp: bad arguments");
+    kv->seq_cp(src, dst, p0, p1);
     return PI_OK;
 }
 
-// llama_kv_cache_seq_keep (llama.cpp:1805-1822)
 int pi_model_kv_cells_seq_keep(pi_model * m, int seq) {
-    if (!m || !m->cells || seq < 0 || seq >= 32) return pi::fail(PI_E_ARG, "pi_model_kv_cells_seq_keep: bad arguments");
-    BatchState * b = m->cells;
-    int new_head = b->n_cells;
-    for (int i = 0; i < b->n_cells; ++i) {
-        if (!(b->cell_seq[i] >> seq & 1u)) { b->cell_pos[i] = -1; b->cell_seq[i] = 0; if (new_head == b->n_cells) new_head = i; }
-        else b->cell_seq[i] = 1u << seq;
-    }
-    if (new_head != b->n_cells) b->head = new_head;
+    KvCells * kv = cells_of(m);
+    if (!kv || seq < 0 || seq >= 32) return pi::fail(PI_E_ARG, "pi_model_kv_cells_seq_keep: bad arguments");
+    kv->seq_keep(seq);
     return PI_OK;
 }
 
-// llama_kv_cache_seq_shift (llama.cpp:1824-1848): the positions move now, the K rows at the start of the next step
 int pi_model_kv_cells_seq_shift(pi_model * m, int seq, int p0, int p1, int delta) {
-    if (!m || !m->cells || seq < 0 || seq >= 32) return pi::fail(PI_E_ARG, "pi_model_kv_cells_seq_shift: bad arguments");
-    BatchState * b = m->cells;
-    int new_head = b->n_cells;
-    if (p0 < 0) p0 = 0;
-    if (p1 < 0) p1 = INT32_MAX;
-    for (int i = 0; i < b->n_cells; ++i) {
-        if ((b->cell_seq[i] >> seq & 1u) && b->cell_pos[i] >= p0 && b->cell_pos[i] < p1) {
-            b->has_shift = true;
-            b->cell_pos[i] += delta;
-            b->cell_delta[i] += delta;
-            if (b->cell_pos[i] < 0) { b->cell_pos[i] = -1; b->cell_seq[i] = 0; if (new_head == b->n_cells) new_head = i; }
-        }
-    }
-    b->head = new_head != b->n_cells ? new_head : 0;
+    KvCells * kv = cells_of(m);
+    if (!kv || seq < 0 || seq >= 32) return pi::fail(PI_E_ARG, "pi_model_kv_cells_seq_shift: bad arguments");
+    kv->seq_shift(seq, p0, p1, delta);
     return PI_OK;
 }
 
-// llama_kv_cache_clear (llama.cpp:1745-1751)
 int pi_model_kv_cells_clear(pi_model * m) {
-    if (!m || !m->cells) return pi::fail(PI_E_ARG, "pi_model_kv_cells_clear: bad arguments");
-    BatchState * b = m->cells;
-    std::fill(b->cell_pos.begin(), b->cell_pos.end(), -1);
-    std::fill(b->cell_seq.begin(), b->cell_seq.end(), 0u);
-    b->head = 0;
+    KvCells * kv = cells_of(m);
+    if (!kv) return pi::fail(PI_E_ARG, "pi_model_kv_cells_clear: bad arguments");
+    kv->clear();
     return PI_OK;
 }
 
 int pi_model_kv_cells_state(pi_model * m, int32_t * cell_pos, uint32_t * cell_seq, int32_t * head) {
-    if (!m || !m->cells) return pi::fail(PI_E_ARG, "pi_model_kv_cells_state: bad arguments");
-    BatchState * b = m->cells;
-    if (cell_pos) memcpy(cell_pos, b->cell_pos.data(), sizeof(int32_t) * b->n_cells);
-    if (cell_seq) memcpy(cell_seq, b->cell_seq.data(), sizeof(uint32_t) * b->n_cells);
-    if (head) *head = b->head;
-    return b->n_cells;
+    KvCells * kv = cells_of(m);
+    if (!kv) return pi::fail(PI_E_ARG, "pi_model_kv_cells_state: bad arguments");
+    if (cell_pos) memcpy(cell_pos, kv->pos.data(), sizeof(int32_t) * kv->n);
+    if (cell_seq) memcpy(cell_seq, kv->seq.data(), sizeof(uint32_t) * kv->n);
+    if (head) *head = kv->head;
+    return kv->n;
+}
+
+// a step of any length on the other models: pieces of up to 16 tokens.  The pool is checked first (a run per piece), so that a step
+// that does not fit leaves nothing behind.
+int pi_model_kv_cells_step(pi_model * m, const int32_t * tokens, const int32_t * positions, const uint32_t * seq_masks, int n_tokens,
+                           const int32_t * want, int n_want, int32_t * next_tokens, float * logits_out) {
+    if (m && m->lay) return pi::layers_step(m, tokens, positions, seq_masks, n_tokens, want, n_want, next_tokens, logits_out);
+    if (!m || !m->cells) return pi::fail(PI_E_STATE, "pi_model_kv_cells_step: pi_model_kv_cells_init first");
+    if (!tokens || !positions || !seq_masks || n_tokens < 1 || n_want < 0 || (n_want && !want)) return pi::fail(PI_E_ARG, "pi_model_kv_cells_step: bad arguments");
+    for (int w = 0; w < n_want; ++w) if (want[w] < 0 || want[w] >= n_tokens) return pi::fail(PI_E_ARG, "pi_model_kv_cells_step: a wanted place is outside the step");
+    for (int t = 0; t < n_tokens; ++t)
+        if (tokens[t] < 0 || tokens[t] >= m->hp.n_vocab || positions[t] < 0 || seq_masks[t] == 0) return pi::fail(PI_E_ARG, "pi_model_kv_cells_step: a token needs an id, a position and a sequence");
+    {
+        KvCells trial = m->cells->kv;
+        for (int t0 = 0; t0 < n_tokens; t0 += 16) {
+            const int T = std::min(16, n_tokens - t0);
+            if (!trial.find_run(T)) return pi::fail(PI_E_STATE, "pi_model_kv_cells_step: no run of free cells for the step");
+            for (int t = 0; t < T; ++t) trial.take(trial.head + t, positions[t0 + t], seq_masks[t0 + t]);
+            trial.move_head(trial.head + T);
+        }
+    }
+    const size_t V = m->hp.n_vocab;
+    std::vector<float> lg(logits_out ? 16 * V : 0);
+    int32_t nxt[16];
+    for (int t0 = 0; t0 < n_tokens; t0 += 16) {
+        const int T = std::min(16, n_tokens - t0);
+        bool any = false;
+        for (int w = 0; w < n_want; ++w) any = any || (want[w] >= t0 && want[w] < t0 + T);
+        PI_TRY(pi_model_kv_cells_decode(m, tokens + t0, positions + t0, seq_masks + t0, T, nxt, any && logits_out ? lg.data() : nullptr));
+        for (int w = 0; w < n_want; ++w) {
+            if (want[w] < t0 || want[w] >= t0 + T) continue;
+            if (next_tokens) next_tokens[w] = nxt[want[w] - t0];
+            if (logits_out) memcpy(logits_out + (size_t)w * V, lg.data() + (size_t)(want[w] - t0) * V, sizeof(float) * V);
+        }
+    }
+    return PI_OK;
 }
 
 int pi_model_batch_union(pi_model * m, int32_t * n_union_per_layer) {

@@ -3,6 +3,7 @@
 
 #include "../../include/powerinfer_hip.h"
 #include "cold_path.hpp"
+#include "kv_cells.hpp"
 
 #include <hip/hip_runtime.h>
 #include <hip/hip_fp16.h>
@@ -20,11 +21,14 @@ struct Tensor {
 
 
 struct BatchState;
+struct LayerState;
 
 struct pi_model {
     pi_hparams hp{};
     std::vector<Tensor> layers;           // [n_layer][PI_T_COUNT]
     Tensor glob[4];
+    Tensor embd_norm;                     // PI_T_EMBD_NORM
+    LayerState * lay = nullptr;           // models described layer by layer (engine_layers.hip); null: the sparse LLaMA / Falcon token loop
     std::vector<void *> owned;            // every device allocation made by the model
     bool finalized = false, hybrid = false;
     int hd = 0, gqa = 0, max_steps = 4096;
@@ -89,6 +93,20 @@ struct pi_model {
 };
 
 namespace pi {
+// models described layer by layer: what the pi_model_* entry points hand over to (engine_layers.hip)
+int  layers_finalize(pi_model * m);
+void layers_destroy(pi_model * m);
+KvCells * layers_cells(pi_model * m);
+int  layers_cells_init(pi_model * m, int n_cells);
+int  layers_step(pi_model * m, const int32_t * tokens, const int32_t * positions, const uint32_t * seq_masks, int n_tokens, const int32_t * want, int n_want,
+                 int32_t * next_tokens, float * logits_out);
+int  layers_decode(pi_model * m, const int32_t * tokens, int n_tokens, int n_past, float * logits_out);
+int  layers_batch_init(pi_model * m, int n_seq);
+int  layers_batch_decode(pi_model * m, const int32_t * tokens, const int32_t * positions, int32_t * next_tokens, float * logits_out);
+int  layers_generate(pi_model * m, int own, int n_steps, int32_t * out_tokens, float * ms_out);
+int  layers_seq_edit(pi_model * m, int seq /* -1: the model's own */, int p0, int p1, int delta, bool shift);
+int  layers_seq_cp(pi_model * m, int src, int dst, int p0, int p1);
+
 int  kv_edit(pi_model * m, __half * k_cache, __half * v_cache, int32_t * d_pos, std::vector<int32_t> & kv_pos, int p0, int p1, int delta, bool shift);
 void batch_destroy(pi_model * m);       // frees the batched-decoding state (graphs; device buffers belong to the model)
 bool prefill_supported(pi_model * m);   // F16 weights, every neuron on the GPU, shapes the multi-token kernels cover

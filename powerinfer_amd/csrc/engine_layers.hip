@@ -1,0 +1,790 @@
+// Models described layer by layer (pi_model_create_layers): weights in the operators' layouts, one pool of cache cells shared by all
+// sequences, steps of any mixture of prompt portions and single tokens, and the captured greedy loop.
+#include "engine_internal.hpp"
+#include "runtime.hpp"
+
+#include <math.h>
+#include <stdlib.h>
+#include <string.h>
+
+#include <algorithm>
+#include <vector>
+
+#define PI_TRY(expr) do { int _rc = (expr); if (_rc != PI_OK) return _rc; } while (0)
+
+namespace {
+
+constexpr int kOwnSeq = 31;              // the model's own sequence (pi_model_decode / pi_model_generate)
+constexpr int kHeadRows = 256;           // rows of logits held at a time
+constexpr int kMaxLockstep = 16;
+constexpr int kItemRows = 32;             // query rows of an attention work item
+constexpr int kAttnItems = 512;          // (work item, part) pairs a split attention aims at: two workgroups per compute unit
+
+int up_to(int v, int m) { return (v + m - 1) / m * m; }
+
+struct Layer {
+    pi_layer_desc d{};
+    int nq = 0, z_rows = 0, dim_ld = 0, rank_ld = 0, kd = 0, hv_ld = 0, ff_ld = 0, rot = 0, hc = 0;      // rot, hc: index among the model's rotations / head counts
+    bool own_kv = true;
+    const void *w_z = nullptr, *uk_t = nullptr, *uv = nullptr, *wo = nullptr, *router = nullptr, *up = nullptr, *down = nullptr;
+    const float *norm_a = nullptr, *norm_b = nullptr, *dkv_norm = nullptr, *sink = nullptr, *bias = nullptr;
+    void * cache = nullptr;
+};
+
+struct Rotation { int dims; double base; };
+
+// where a pass finds its tokens
+struct Step {
+    int T = 0;
+    const int32_t *tokens = nullptr, *pos = nullptr, *cell = nullptr, *n_vis = nullptr, *seq = nullptr;
+    struct Work { const int32_t * items = nullptr; int n = 0, parts = 1; };
+    std::vector<Work> work;               // attention work items, per distinct head count of the model
+};
+
+}  // namespace
+
+struct LayerState {
+    pi_layers_opts opts{};
+    std::vector<Layer> layers;
+    std::vector<Rotation> rots;
+    std::vector<int> head_counts;
+    int d_ld = 0, es = 2;
+    const float *embd_norm = nullptr, *out_norm = nullptr;
+    const void *embed = nullptr, *head = nullptr;
+    KvCells kv;
+    int32_t * lists = nullptr;                         // device [32][kv.n]: a sequence's cells in position order
+    std::vector<int32_t> list_cells[32], list_pos[32]; // the same on the host
+    int32_t * d_delta = nullptr;
+    // step buffers for `cap` tokens (one allocation)
+    int cap = 0;
+    unsigned char * arena = nullptr;
+    float *x = nullptr, *x2 = nullptr, *z = nullptr, *mix = nullptr, *rl = nullptr, *wts = nullptr, *y_exp = nullptr;
+    void *h_a = nullptr, *h_b = nullptr, *q_un = nullptr, *q_lat = nullptr, *o_lat = nullptr, *att = nullptr, *act = nullptr;
+    int32_t *ids = nullptr, *perm = nullptr, *inv = nullptr, *off = nullptr;
+    std::vector<float *> cs;                           // per rotation [cap][dims / 2] (cos, sin)
+    float * scratch = nullptr;                         // partial sums of a split attention
+    float * logits = nullptr; void * h_head = nullptr; int32_t * d_next = nullptr;
+    int32_t * h_in = nullptr, * d_in = nullptr; size_t in_cap = 0;       // a pass's integers: pinned host side and device side
+    float * streams = nullptr; size_t streams_cap = 0; int streams_T = 0;
+    // lockstep decoding and the greedy loop
+    int n_seq = 0;
+    int32_t last_tok[32], last_pos[32];
+    int32_t *g_tok = nullptr, *g_pos = nullptr, *g_cell = nullptr, *g_vis = nullptr, *g_seq = nullptr, *g_work = nullptr, *g_step = nullptr, *g_out = nullptr;
+    int max_steps = 4096;
+    hipGraph_t graph = nullptr; hipGraphExec_t exec = nullptr;
+    int graph_T = 0, graph_seq0 = -1; std::vector<int> graph_parts;
+};
+
+namespace {
+
+__global__ void cells_append_kernel(const int32_t * __restrict__ app, int n, int32_t * __restrict__ lists, size_t ld) {
+    const int i = blockIdx.x * blockDim.x + threadIdx.x;
+    if (i < n) lists[(size_t)app[3 * i] * ld + app[3 * i + 1]] = app[3 * i + 2];
+}
+
+bool bf16_mode(const LayerState * s) { return s->opts.compute == PI_TYPE_BF16; }
+
+void drop_graph(LayerState * s) {
+    if (s->exec) (void)hipGraphExecDestroy(s->exec);
+    if (s->graph) (void)hipGraphDestroy(s->graph);
+    s->exec = nullptr; s->graph = nullptr;
+}
+
+// ---- weights ---------------------------------------------------------------------------------------------------------------------
+int want_tensor(const Tensor & t, int type, int64_t ne0, int64_t ne1, const char * what) {
+    if (!t.dev || t.type != type || t.ne0 != ne0 || t.ne1 != ne1) {
+        char msg[160];
+        snprintf(msg, sizeof msg, "pi_model_finalize: %s must be %s of {%lld, %lld}", what, type == PI_TYPE_BF16 ? "BF16" : "F32", (long long)ne0, (long long)ne1);
+        return pi::fail(PI_E_ARG, msg);
+    }
+    return PI_OK;
+}
+
+void release(pi_model * m, Tensor & t) {
+    if (t.owned) for (auto & o : m->owned) if (o == t.dev) { pi_free(o); o = nullptr; }
+    t.owned = false; t.dev = nullptr;
+}
+
+// rows of ld values, the tensor itself when it has that pitch already
+int padded(pi_model * m, Tensor & t, int ld, const void ** out) {
+    if (t.ne0 == ld) { *out = t.dev; return PI_OK; }
+    uint16_t * p = m->alloc<uint16_t>((size_t)t.ne1 * ld);
+    if (!p) return PI_E_HIP;
+    PI_TRY(pi_k_pad_cols_bf16(t.dev, t.ne1, (int)t.ne0, p, ld, nullptr));
+    PI_TRY(pi_sync());
+    release(m, t);
+    *out = p;
+    return PI_OK;
+}
+
+// the weights of one of the model's norms with the offset of the design added
+int norm_weights(pi_model * m, const Tensor & t, float offset, const float ** out) {
+    std::vector<float> w((size_t)t.ne0);
+    PI_TRY(pi_memcpy_d2h(w.data(), t.dev, sizeof(float) * w.size()));
+    for (float & v : w) v += offset;
+    float * p = m->alloc<float>(w.size());
+    if (!p) return PI_E_HIP;
+    PI_TRY(pi_memcpy_h2d(p, w.data(), sizeof(float) * w.size()));
+    *out = p;
+    return PI_OK;
+}
+
+int layer_weights(pi_model * m, int il) {
+    LayerState * s = m->lay;
+    Layer & L = s->layers[il];
+    const pi_layer_desc & d = L.d;
+    const int D = m->hp.n_embd;
+    PI_TRY(want_tensor(m->L(il, PI_T_ATTN_NORM), PI_TYPE_F32, D, 1, "attn_norm"));
+    PI_TRY(norm_weights(m, m->L(il, PI_T_ATTN_NORM), s->opts.norm_offset, &L.norm_a));
+    Tensor & q = m->L(il, PI_T_MIX_Q); Tensor & dkv = m->L(il, PI_T_MIX_DKV);
+    PI_TRY(want_tensor(q, PI_TYPE_BF16, D, L.nq, "mix_q"));
+    if (L.own_kv) {
+        PI_TRY(want_tensor(dkv, PI_TYPE_BF16, D, d.kv_rank + d.rot_dim, "mix_dkv"));
+        PI_TRY(want_tensor(m->L(il, PI_T_MIX_DKV_NORM), PI_TYPE_F32, d.kv_rank, 1, "mix_dkv_norm"));
+        L.dkv_norm = (const float *)m->L(il, PI_T_MIX_DKV_NORM).dev;
+        // one matrix, so that one mat-mul gives the queries and the cell
+        uint16_t * w = m->alloc<uint16_t>((size_t)L.z_rows * s->d_ld);
+        if (!w) return PI_E_HIP;
+        PI_TRY(pi_k_pad_cols_bf16(q.dev, q.ne1, D, w, s->d_ld, nullptr));
+        PI_TRY(pi_k_pad_cols_bf16(dkv.dev, dkv.ne1, D, w + (size_t)L.nq * s->d_ld, s->d_ld, nullptr));
+        PI_TRY(pi_sync());
+        release(m, q); release(m, dkv);
+        L.w_z = w;
+    } else {
+        PI_TRY(padded(m, q, s->d_ld, &L.w_z));
+    }
+    Tensor & uk = m->L(il, PI_T_MIX_UK); Tensor & uv = m->L(il, PI_T_MIX_UV);
+    PI_TRY(want_tensor(uk, PI_TYPE_BF16, d.kv_rank, (int64_t)d.n_head * d.dim, "mix_uk"));
+    PI_TRY(want_tensor(uv, PI_TYPE_BF16, d.kv_rank, (int64_t)d.n_head * d.vdim, "mix_uv"));
+    uint16_t * ukt = m->alloc<uint16_t>((size_t)d.n_head * d.kv_rank * L.dim_ld);
+    if (!ukt) return PI_E_HIP;
+    PI_TRY(pi_k_transpose_pad_bf16(uk.dev, d.n_head, d.dim, d.kv_rank, ukt, L.dim_ld, nullptr));
+    PI_TRY(pi_sync());
+    release(m, uk);
+    L.uk_t = ukt;
+    PI_TRY(padded(m, uv, L.rank_ld, &L.uv));
+    PI_TRY(want_tensor(m->L(il, PI_T_MIX_SINK), PI_TYPE_F32, d.n_head, 1, "mix_sink"));
+    L.sink = (const float *)m->L(il, PI_T_MIX_SINK).dev;
+    PI_TRY(want_tensor(m->L(il, PI_T_WO), PI_TYPE_BF16, (int64_t)d.n_head * d.vdim, D, "wo"));
+    PI_TRY(padded(m, m->L(il, PI_T_WO), L.hv_ld, &L.wo));
+    if (d.ffn == PI_FFN_NONE) return PI_OK;
+    PI_TRY(want_tensor(m->L(il, PI_T_FFN_NORM), PI_TYPE_F32, D, 1, "ffn_norm"));
+    PI_TRY(norm_weights(m, m->L(il, PI_T_FFN_NORM), s->opts.norm_offset, &L.norm_b));
+    PI_TRY(want_tensor(m->L(il, PI_T_ROUTER), PI_TYPE_BF16, D, d.n_expert, "router"));
+    PI_TRY(want_tensor(m->L(il, PI_T_ROUTER_BIAS), PI_TYPE_F32, d.n_expert, 1, "router_bias"));
+    PI_TRY(want_tensor(m->L(il, PI_T_EXPERT_UP), PI_TYPE_BF16, D, (int64_t)d.n_expert * d.expert_ff, "expert_up"));
+    PI_TRY(want_tensor(m->L(il, PI_T_EXPERT_DOWN), PI_TYPE_BF16, d.expert_ff, (int64_t)d.n_expert * D, "expert_down"));
+    L.bias = (const float *)m->L(il, PI_T_ROUTER_BIAS).dev;
+    PI_TRY(padded(m, m->L(il, PI_T_ROUTER), s->d_ld, &L.router));
+    PI_TRY(padded(m, m->L(il, PI_T_EXPERT_UP), s->d_ld, &L.up));
+    PI_TRY(padded(m, m->L(il, PI_T_EXPERT_DOWN), L.ff_ld, &L.down));
+    return PI_OK;
+}
+
+// ---- step buffers ----------------------------------------------------------------------------------------------------------------
+int ensure_capacity(pi_model * m, int T) {
+    LayerState * s = m->lay;
+    if (T <= s->cap) return PI_OK;
+    int cap = 64;
+    while (cap < T) cap *= 2;
+    const size_t es = s->es, D = m->hp.n_embd;
+    size_t z = 0, qu = 0, ql = 0, ol = 0, at = 0, E = 0, top = 0, ff = 0;
+    for (const Layer & L : s->layers) {
+        const pi_layer_desc & d = L.d;
+        z = std::max(z, (size_t)L.z_rows); qu = std::max(qu, (size_t)d.n_head * L.dim_ld); ql = std::max(ql, (size_t)d.n_head * L.kd);
+        ol = std::max(ol, (size_t)d.n_head * L.rank_ld); at = std::max(at, (size_t)L.hv_ld);
+        if (d.ffn == PI_FFN_MOE) { E = std::max(E, (size_t)d.n_expert); top = std::max(top, (size_t)d.n_top); ff = std::max(ff, (size_t)d.n_top * L.ff_ld); }
+    }
+    PI_HIP_TRY(hipStreamSynchronize(m->stream));
+    drop_graph(s);
+    if (s->arena) { pi_free(s->arena); s->arena = nullptr; s->cap = 0; }
+    // carved twice: once to learn the size, once to hand out addresses
+    size_t used = 0;
+    auto carve = [&](auto *& p, size_t bytes) {
+        using P = std::remove_reference_t<decltype(p)>;
+        p = reinterpret_cast<P>(s->arena ? s->arena + used : nullptr);
+        used += (bytes + 255) / 256 * 256;
+    };
+    auto lay_out = [&]() {
+        used = 0;
+        const size_t n = cap;
+        carve(s->x, n * D * 4); carve(s->x2, n * D * 4); carve(s->mix, n * D * 4); carve(s->z, n * z * 4);
+        carve(s->h_a, n * s->d_ld * es); carve(s->h_b, n * s->d_ld * es);
+        carve(s->q_un, n * qu * es); carve(s->q_lat, n * ql * es); carve(s->o_lat, n * ol * es); carve(s->att, n * at * es);
+        carve(s->rl, n * E * 4); carve(s->wts, n * top * 4); carve(s->ids, n * top * 4); carve(s->perm, n * top * 4); carve(s->inv, n * top * 4);
+        carve(s->off, (E + 1) * 4); carve(s->act, n * ff * es); carve(s->y_exp, n * top * D * 4);
+        s->cs.resize(s->rots.size());
+        for (size_t r = 0; r < s->rots.size(); ++r) carve(s->cs[r], n * s->rots[r].dims * 4);
+    };
+    lay_out();
+    s->arena = (unsigned char *)pi_malloc(used);
+    if (!s->arena) return PI_E_HIP;
+    lay_out();
+    PI_TRY(pi_memset(s->arena, 0, used));           // the padding columns of the operands stay zero or finite from here on
+    PI_TRY(pi_sync());
+    s->cap = cap;
+    return PI_OK;
+}
+
+int ensure_inputs(pi_model * m, size_t n) {
+    LayerState * s = m->lay;
+    if (n <= s->in_cap) return PI_OK;
+    PI_HIP_TRY(hipStreamSynchronize(m->stream));
+    if (s->h_in) { (void)hipHostFree(s->h_in); s->h_in = nullptr; }
+    if (s->d_in) { pi_free(s->d_in); s->d_in = nullptr; }
+    s->in_cap = 0;
+    size_t c = 4096;
+    while (c < n) c *= 2;
+    PI_HIP_TRY(hipHostMalloc((void **)&s->h_in, c * 4, hipHostMallocDefault));
+    s->d_in = (int32_t *)pi_malloc(c * 4);
+    if (!s->d_in) return PI_E_HIP;
+    s->in_cap = c;
+    return PI_OK;
+}
+
+// ---- one pass over the layers ----------------------------------------------------------------------------------------------------
+int dense(LayerState * s, const void * W, int rows, int cols, const void * x, int ldx, int T, float * y, int ldy, float alpha, hipStream_t st) {
+    pi_group_gemm g{};
+    g.W = W; g.rows = rows; g.cols = cols; g.ldw = cols; g.n_group = 1; g.x = x; g.ldx = ldx; g.T = T; g.y = y; g.ldy = ldy; g.y_f32 = 1; g.alpha = alpha;
+    return pi_k_group_gemm(s->opts.compute, &g, st);
+}
+
+int mix_latent(pi_model * m, Layer & L, const Step & in) {
+    LayerState * s = m->lay;
+    const pi_layer_desc & d = L.d;
+    const int type = s->opts.compute, T = in.T;
+    hipStream_t st = m->stream;
+    Layer & src = L.own_kv ? L : s->layers[d.kv_from];
+    PI_TRY(dense(s, L.w_z, L.z_rows, s->d_ld, s->h_a, s->d_ld, T, s->z, L.z_rows, 1.0f, st));
+    pi_latent_prep p{};
+    p.z = s->z; p.ldz = L.z_rows; p.T = T; p.n_head = d.n_head; p.dim = d.dim; p.dim_ld = L.dim_ld; p.rot_dim = d.rot_dim; p.kv_rank = d.kv_rank;
+    p.rank_ld = L.rank_ld; p.kd = L.kd; p.cs = s->cs[L.rot]; p.norm_w = L.dkv_norm; p.eps = m->hp.norm_eps; p.q_un = s->q_un; p.q_lat = s->q_lat;
+    p.cache = L.own_kv ? L.cache : nullptr; p.cell = in.cell;
+    PI_TRY(pi_k_latent_prep(type, &p, st));
+    pi_group_gemm g{};                              // each head's query in latent coordinates
+    g.W = L.uk_t; g.w_gs = (size_t)d.kv_rank * L.dim_ld; g.rows = d.kv_rank; g.cols = L.dim_ld; g.ldw = L.dim_ld; g.n_group = d.n_head; g.alpha = 1.0f;
+    g.x = s->q_un; g.x_gs = L.dim_ld; g.ldx = d.n_head * L.dim_ld; g.T = T; g.y = s->q_lat; g.y_gs = L.kd; g.ldy = d.n_head * L.kd;
+    PI_TRY(pi_k_group_gemm(type, &g, st));
+    pi_latent_attn a{};
+    a.q_lat = s->q_lat; a.cache = src.cache; a.lists = s->lists; a.list_ld = s->kv.n; a.work = bf16_mode(s) ? in.work[L.hc].items : in.seq; a.n_vis = in.n_vis;
+    a.n_work = in.work[L.hc].n; a.T = T; a.n_head = d.n_head; a.kv_rank = d.kv_rank; a.rank_ld = L.rank_ld; a.kd = L.kd; a.n_parts = in.work[L.hc].parts; a.scale = d.scale;
+    a.sink = L.sink; a.scratch = s->scratch; a.out_lat = s->o_lat;
+    PI_TRY(pi_k_latent_attn(type, &a, st));
+    pi_group_gemm v{};                              // each head's value from its weighted latent
+    v.W = L.uv; v.w_gs = (size_t)d.vdim * L.rank_ld; v.rows = d.vdim; v.cols = L.rank_ld; v.ldw = L.rank_ld; v.n_group = d.n_head; v.alpha = 1.0f;
+    v.x = s->o_lat; v.x_gs = L.rank_ld; v.ldx = d.n_head * L.rank_ld; v.T = T; v.y = s->att; v.y_gs = d.vdim; v.ldy = L.hv_ld;
+    PI_TRY(pi_k_group_gemm(type, &v, st));
+    return dense(s, L.wo, m->hp.n_embd, L.hv_ld, s->att, L.hv_ld, T, s->mix, m->hp.n_embd, 1.0f, st);
+}
+
+int ffn_moe(pi_model * m, Layer & L, const Step & in) {
+    LayerState * s = m->lay;
+    const pi_layer_desc & d = L.d;
+    const int type = s->opts.compute, T = in.T, D = m->hp.n_embd;
+    hipStream_t st = m->stream;
+    PI_TRY(dense(s, L.router, d.n_expert, s->d_ld, s->h_b, s->d_ld, T, s->rl, d.n_expert, 1.0f, st));
+    PI_TRY(pi_k_route(s->rl, T, d.n_expert, d.n_top, d.n_group, d.n_group_keep, L.bias, s->ids, s->wts, st));
+    PI_TRY(pi_k_moe_sort(s->ids, T * d.n_top, d.n_expert, s->off, s->perm, s->inv, st));
+    pi_group_gemm g{};
+    g.W = L.up; g.w_gs = (size_t)d.expert_ff * s->d_ld; g.rows = d.expert_ff; g.cols = s->d_ld; g.ldw = s->d_ld; g.n_group = d.n_expert; g.alpha = 1.0f; g.relu2 = 1;
+    g.x = s->h_b; g.ldx = s->d_ld; g.T = T; g.y = s->act; g.ldy = L.ff_ld; g.off = s->off; g.gather = s->perm; g.gather_div = d.n_top;
+    PI_TRY(pi_k_group_gemm(type, &g, st));
+    pi_group_gemm w{};
+    w.W = L.down; w.w_gs = (size_t)D * L.ff_ld; w.rows = D; w.cols = L.ff_ld; w.ldw = L.ff_ld; w.n_group = d.n_expert; w.alpha = 1.0f;
+    w.x = s->act; w.ldx = L.ff_ld; w.T = T; w.y = s->y_exp; w.ldy = D; w.y_f32 = 1; w.off = s->off;
+    return pi_k_group_gemm(type, &w, st);
+}
+
+int pass_layers(pi_model * m, const Step & in) {
+    LayerState * s = m->lay;
+    const int type = s->opts.compute, T = in.T, D = m->hp.n_embd;
+    hipStream_t st = m->stream;
+    PI_TRY(pi_k_embed_norm(s->embed, D, in.tokens, T, s->embd_norm, m->hp.norm_eps, s->x, st));
+    for (size_t r = 0; r < s->rots.size(); ++r) PI_TRY(pi_k_rope_angles(in.pos, T, s->rots[r].dims, s->rots[r].base, s->cs[r], st));
+    for (size_t il = 0; il < s->layers.size(); ++il) {
+        Layer & L = s->layers[il];
+        const bool moe = L.d.ffn == PI_FFN_MOE;
+        PI_TRY(pi_k_norm_pair(type, s->x, nullptr, T, D, m->hp.norm_eps, L.norm_a, s->h_a, moe ? L.norm_b : nullptr, moe ? s->h_b : nullptr, s->d_ld, 0, st));
+        PI_TRY(mix_latent(m, L, in));
+        if (moe) PI_TRY(ffn_moe(m, L, in));
+        PI_TRY(pi_k_moe_combine(s->x, s->mix, s->y_exp, s->inv, moe ? s->wts : nullptr, moe ? L.d.n_top : 0, T, D, s->x2,
+                                s->streams_T ? s->streams + il * (size_t)s->streams_T * D : nullptr, st));
+        std::swap(s->x, s->x2);
+    }
+    return PI_OK;
+}
+
+// logits of `n` rows of the residual stream (rows: device indices, null: the first n) into s->logits
+int pass_head(pi_model * m, const int32_t * rows, int n) {
+    LayerState * s = m->lay;
+    const int D = m->hp.n_embd;
+    PI_TRY(pi_k_norm_pair(s->opts.compute, s->x, rows, n, D, m->hp.norm_eps, s->out_norm, s->h_head, nullptr, nullptr, s->d_ld, 0, m->stream));
+    return dense(s, s->head, m->hp.n_vocab, s->d_ld, s->h_head, s->d_ld, n, s->logits, m->hp.n_vocab, s->opts.logit_scale, m->stream);
+}
+
+int head_buffers(pi_model * m) {
+    LayerState * s = m->lay;
+    if (s->logits) return PI_OK;
+    s->h_head = m->alloc<unsigned char>((size_t)kHeadRows * s->d_ld * s->es);
+    s->d_next = m->alloc<int32_t>(kHeadRows);
+    s->logits = m->alloc<float>((size_t)kHeadRows * m->hp.n_vocab);
+    if (!s->h_head || !s->d_next || !s->logits) return PI_E_HIP;
+    return pi_memset(s->h_head, 0, (size_t)kHeadRows * s->d_ld * s->es);
+}
+
+// attention work items of n tokens' runs (consecutive tokens of one sequence with ascending cells): appended to `out`
+void work_items(const int32_t * seq, const int32_t * n_vis, int n, int n_head, std::vector<int32_t> & out) {
+    for (int t0 = 0; t0 < n;) {
+        int t1 = t0 + 1;
+        while (t1 < n && seq[t1] == seq[t0] && n_vis[t1] >= n_vis[t1 - 1]) ++t1;
+        const int rows = (t1 - t0) * n_head;
+        for (int r = 0; r < rows; r += kItemRows) { out.push_back(t0); out.push_back(r); out.push_back(std::min(kItemRows, rows - r)); out.push_back(seq[t0]); }
+        t0 = t1;
+    }
+}
+
+// how many workgroups share one work item's cells
+int choose_parts(LayerState * s, int n_work, int n_vis_max) {
+    if (!bf16_mode(s) || n_work <= 0) return 1;
+    const int tiles = (n_vis_max + 31) / 32;
+    return std::max(1, std::min({kAttnItems / n_work, tiles / 4, 64}));
+}
+
+// ---- cells -----------------------------------------------------------------------------------------------------------------------
+// the host's list of a sequence's cells, rebuilt after an edit; `app` receives what the device has to learn
+void refresh_list(LayerState * s, int q, std::vector<int32_t> & app) {
+    if (!(s->kv.edited >> q & 1u)) return;
+    s->kv.edited &= ~(1u << q);
+    std::vector<std::pair<int32_t, int32_t>> v;
+    for (int i = 0; i < s->kv.n; ++i) if (s->kv.pos[i] >= 0 && (s->kv.seq[i] >> q & 1u)) v.push_back({s->kv.pos[i], i});
+    std::sort(v.begin(), v.end());
+    s->list_cells[q].clear(); s->list_pos[q].clear();
+    for (size_t k = 0; k < v.size(); ++k) {
+        s->list_pos[q].push_back(v[k].first); s->list_cells[q].push_back(v[k].second);
+        app.push_back(q); app.push_back((int32_t)k); app.push_back(v[k].second);
+    }
+}
+
+int live_cells(LayerState * s, int q) {
+    int n = 0;
+    for (int i = 0; i < s->kv.n; ++i) n += s->kv.pos[i] >= 0 && (s->kv.seq[i] >> q & 1u) ? 1 : 0;
+    return n;
+}
+
+// takes the cell for sequences `mask` at position p; false: some sequence's list has to be rebuilt (the position is not behind its last)
+void take_cell(LayerState * s, int cell, int32_t p, uint32_t mask, std::vector<int32_t> & app) {
+    s->kv.take(cell, p, mask);
+    for (uint32_t b = mask; b; b &= b - 1) {
+        const int q = __builtin_ctz(b);
+        if (s->kv.edited >> q & 1u) continue;                      // rebuilt as a whole later
+        if (!s->list_pos[q].empty() && s->list_pos[q].back() >= p) { s->kv.edited |= 1u << q; continue; }
+        app.push_back(q); app.push_back((int32_t)s->list_pos[q].size()); app.push_back(cell);
+        s->list_pos[q].push_back(p); s->list_cells[q].push_back(cell);
+    }
+}
+
+int apply_shift(pi_model * m) {
+    LayerState * s = m->lay;
+    if (!s->kv.has_shift) return PI_OK;
+    PI_HIP_TRY(hipStreamSynchronize(m->stream));
+    PI_TRY(pi_memcpy_h2d(s->d_delta, s->kv.delta.data(), sizeof(int32_t) * s->kv.n));
+    for (Layer & L : s->layers)
+        if (L.own_kv) PI_TRY(pi_k_latent_shift(s->opts.compute, L.cache, s->kv.n, L.kd, L.rank_ld, L.d.rot_dim, L.d.rot_base, s->d_delta, m->stream));
+    PI_HIP_TRY(hipStreamSynchronize(m->stream));
+    s->kv.shift_done();
+    return PI_OK;
+}
+
+int upload_appends(pi_model * m, const std::vector<int32_t> & app) {
+    if (app.empty()) return PI_OK;
+    LayerState * s = m->lay;
+    PI_TRY(ensure_inputs(m, app.size()));
+    PI_HIP_TRY(hipStreamSynchronize(m->stream));                   // the staging buffer's last copy is done
+    memcpy(s->h_in, app.data(), app.size() * 4);
+    PI_HIP_TRY(hipMemcpyAsync(s->d_in, s->h_in, app.size() * 4, hipMemcpyHostToDevice, m->stream));
+    const int n = (int)(app.size() / 3);
+    hipLaunchKernelGGL(cells_append_kernel, dim3((n + 255) / 256), dim3(256), 0, m->stream, s->d_in, n, s->lists, (size_t)s->kv.n);
+    return pi::check_launch("cells_append");
+}
+
+}  // namespace
+
+namespace pi {
+
+KvCells * layers_cells(pi_model * m) { return m->lay->kv.n ? &m->lay->kv : nullptr; }
+
+int layers_cells_init(pi_model * m, int n_cells) {
+    LayerState * s = m->lay;
+    if (s->kv.n) return fail(PI_E_STATE, "pi_model_kv_cells_init: already initialised");
+    if (n_cells < 1) return fail(PI_E_ARG, "pi_model_kv_cells_init: at least one cell");
+    for (Layer & L : s->layers) {
+        if (!L.own_kv) continue;
+        L.cache = m->alloc<unsigned char>((size_t)n_cells * L.kd * s->es);
+        if (!L.cache) return PI_E_HIP;
+        PI_TRY(pi_memset(L.cache, 0, (size_t)n_cells * L.kd * s->es));
+    }
+    s->lists = m->alloc<int32_t>((size_t)32 * n_cells);
+    s->d_delta = m->alloc<int32_t>(n_cells);
+    if (!s->lists || !s->d_delta) return PI_E_HIP;
+    PI_TRY(pi_memset(s->lists, 0, sizeof(int32_t) * 32 * (size_t)n_cells));
+    PI_TRY(pi_sync());
+    s->kv.init(n_cells);
+    return PI_OK;
+}
+
+int layers_finalize(pi_model * m) {
+    LayerState * s = m->lay;
+    const int D = m->hp.n_embd;
+    PI_HIP_TRY(hipEventCreate(&m->ev0));
+    PI_HIP_TRY(hipEventCreate(&m->ev1));
+    s->es = bf16_mode(s) ? 2 : 4;
+    s->d_ld = up_to(D, 128);
+    PI_TRY(want_tensor(m->glob[PI_T_TOK_EMBD], PI_TYPE_BF16, D, m->hp.n_vocab, "tok_embd"));
+    PI_TRY(want_tensor(m->glob[PI_T_OUTPUT], PI_TYPE_BF16, D, m->hp.n_vocab, "output"));
+    PI_TRY(want_tensor(m->glob[PI_T_OUTPUT_NORM], PI_TYPE_F32, D, 1, "output_norm"));
+    PI_TRY(want_tensor(m->embd_norm, PI_TYPE_F32, D, 1, "embd_norm"));
+    s->embed = m->glob[PI_T_TOK_EMBD].dev;
+    PI_TRY(padded(m, m->glob[PI_T_OUTPUT], s->d_ld, &s->head));
+    PI_TRY(norm_weights(m, m->embd_norm, s->opts.norm_offset, &s->embd_norm));
+    PI_TRY(norm_weights(m, m->glob[PI_T_OUTPUT_NORM], s->opts.norm_offset, &s->out_norm));
+    size_t scratch = 0;
+    for (size_t il = 0; il < s->layers.size(); ++il) {
+        Layer & L = s->layers[il];
+        const pi_layer_desc & d = L.d;
+        L.own_kv = d.kv_from < 0;
+        L.nq = d.n_head * (d.dim + d.rot_dim);
+        L.z_rows = L.nq + (L.own_kv ? d.kv_rank + d.rot_dim : 0);
+        L.dim_ld = up_to(d.dim, 32); L.rank_ld = up_to(d.kv_rank, 32); L.kd = L.rank_ld + up_to(d.rot_dim, 32);
+        L.hv_ld = up_to(d.n_head * d.vdim, 128); L.ff_ld = d.ffn == PI_FFN_MOE ? up_to(d.expert_ff, 64) : 0;
+        if (!pi_k_latent_attn_supported(s->opts.compute, L.rank_ld, L.kd)) return fail(PI_E_UNSUPPORTED, "pi_model_finalize: latent sizes outside the attention kernels (rank up to 1024)");
+        size_t r = 0;
+        while (r < s->rots.size() && (s->rots[r].dims != d.rot_dim || s->rots[r].base != d.rot_base)) ++r;
+        if (r == s->rots.size()) s->rots.push_back({d.rot_dim, d.rot_base});
+        L.rot = (int)r;
+        size_t h = 0;
+        while (h < s->head_counts.size() && s->head_counts[h] != d.n_head) ++h;
+        if (h == s->head_counts.size()) s->head_counts.push_back(d.n_head);
+        L.hc = (int)h;
+        scratch = std::max(scratch, pi_k_latent_attn_scratch_floats(pi_k_latent_attn_rows(s->opts.compute) * kAttnItems, 1, L.rank_ld, 2) / 2);
+        PI_TRY(layer_weights(m, (int)il));
+    }
+    if (bf16_mode(s)) {
+        s->scratch = m->alloc<float>(scratch);
+        if (!s->scratch) return PI_E_HIP;
+    }
+    PI_TRY(head_buffers(m));
+    for (int32_t ** p : {&s->g_tok, &s->g_pos, &s->g_cell, &s->g_vis, &s->g_seq, &s->g_step}) {
+        *p = m->alloc<int32_t>(kMaxLockstep);
+        if (!*p) return PI_E_HIP;
+    }
+    size_t items = 0;
+    for (int h : s->head_counts) items += (size_t)kMaxLockstep * ((h + kItemRows - 1) / kItemRows);
+    s->g_work = m->alloc<int32_t>(4 * items);
+    s->g_out = m->alloc<int32_t>((size_t)s->max_steps * kMaxLockstep);
+    if (!s->g_work || !s->g_out) return PI_E_HIP;
+    PI_HIP_TRY(hipDeviceSynchronize());
+    m->finalized = true;
+    return PI_OK;
+}
+
+void layers_destroy(pi_model * m) {
+    LayerState * s = m->lay;
+    drop_graph(s);
+    if (s->arena) pi_free(s->arena);
+    if (s->h_in) (void)hipHostFree(s->h_in);
+    if (s->d_in) pi_free(s->d_in);
+    if (s->streams) pi_free(s->streams);
+    delete s;
+    m->lay = nullptr;
+}
+
+// One step: cells for every token (or PI_E_STATE with nothing changed), then passes of at most max_batch tokens.
+int layers_step(pi_model * m, const int32_t * tokens, const int32_t * positions, const uint32_t * seq_masks, int n_tokens, const int32_t * want, int n_want,
+                int32_t * next_tokens, float * logits_out) {
+    LayerState * s = m->lay;
+    if (!m->finalized || !s->kv.n) return fail(PI_E_STATE, "pi_model_kv_cells_step: pi_model_kv_cells_init first");
+    if (!tokens || !positions || !seq_masks || n_tokens < 1 || n_want < 0 || (n_want && !want)) return fail(PI_E_ARG, "pi_model_kv_cells_step: bad arguments");
+    for (int w = 0; w < n_want; ++w) if (want[w] < 0 || want[w] >= n_tokens) return fail(PI_E_ARG, "pi_model_kv_cells_step: a wanted place is outside the step");
+    for (int t = 0; t < n_tokens; ++t)
+        if (tokens[t] < 0 || tokens[t] >= m->hp.n_vocab || positions[t] < 0 || seq_masks[t] == 0) return fail(PI_E_ARG, "pi_model_kv_cells_step: a token needs an id, a position and a sequence");
+    std::vector<int32_t> cells(n_tokens), app;
+    if (!s->kv.find_free(n_tokens, cells.data())) return fail(PI_E_STATE, "pi_model_kv_cells_step: not enough free cells");
+    const int batch = s->opts.max_batch > 0 ? s->opts.max_batch : 2048;
+    PI_TRY(ensure_capacity(m, std::min(n_tokens, batch)));
+    PI_TRY(apply_shift(m));
+    for (int t = 0; t < n_tokens; ++t) for (uint32_t b = seq_masks[t]; b; b &= b - 1) refresh_list(s, __builtin_ctz(b), app);
+    for (int t = 0; t < n_tokens; ++t) take_cell(s, cells[t], positions[t], seq_masks[t], app);
+    s->kv.move_head(cells[n_tokens - 1] + 1);
+    for (int t = 0; t < n_tokens; ++t) for (uint32_t b = seq_masks[t]; b; b &= b - 1) refresh_list(s, __builtin_ctz(b), app);
+    PI_TRY(upload_appends(m, app));
+    std::vector<int32_t> vis(n_tokens), seq(n_tokens);
+    for (int t = 0; t < n_tokens; ++t) {
+        seq[t] = __builtin_ctz(seq_masks[t]);                    // a token attends the cells of its first sequence
+        const auto & lp = s->list_pos[seq[t]];
+        vis[t] = (int32_t)(std::upper_bound(lp.begin(), lp.end(), positions[t]) - lp.begin());
+    }
+    std::vector<int32_t> rows, place, items;
+    for (int t0 = 0; t0 < n_tokens; t0 += batch) {
+        const int T = std::min(batch, n_tokens - t0);
+        rows.clear(); place.clear(); items.clear();
+        for (int w = 0; w < n_want; ++w) if (want[w] >= t0 && want[w] < t0 + T) { rows.push_back(want[w] - t0); place.push_back(w); }
+        Step in;
+        in.T = T;
+        const int vmax = *std::max_element(vis.begin() + t0, vis.begin() + t0 + T);
+        std::vector<size_t> begin;
+        for (int h : s->head_counts) {
+            begin.push_back(items.size());
+            if (bf16_mode(s)) work_items(seq.data() + t0, vis.data() + t0, T, h, items);
+        }
+        begin.push_back(items.size());
+        const size_t n_in = (size_t)5 * T + items.size() + rows.size();
+        PI_TRY(ensure_inputs(m, n_in));
+        PI_HIP_TRY(hipStreamSynchronize(m->stream));
+        int32_t * h = s->h_in;
+        memcpy(h, tokens + t0, 4 * (size_t)T); memcpy(h + T, positions + t0, 4 * (size_t)T); memcpy(h + 2 * T, cells.data() + t0, 4 * (size_t)T);
+        memcpy(h + 3 * T, vis.data() + t0, 4 * (size_t)T); memcpy(h + 4 * T, seq.data() + t0, 4 * (size_t)T);
+        if (!items.empty()) memcpy(h + 5 * T, items.data(), 4 * items.size());
+        if (!rows.empty()) memcpy(h + 5 * T + items.size(), rows.data(), 4 * rows.size());
+        PI_HIP_TRY(hipMemcpyAsync(s->d_in, h, 4 * n_in, hipMemcpyHostToDevice, m->stream));
+        in.tokens = s->d_in; in.pos = s->d_in + T; in.cell = s->d_in + 2 * T; in.n_vis = s->d_in + 3 * T; in.seq = s->d_in + 4 * T;
+        for (size_t k = 0; k < s->head_counts.size(); ++k) {
+            Step::Work w;
+            w.items = s->d_in + 5 * T + begin[k];
+            w.n = bf16_mode(s) ? (int)(begin[k + 1] - begin[k]) / 4 : T;
+            w.parts = choose_parts(s, w.n, vmax);
+            in.work.push_back(w);
+        }
+        s->streams_T = 0;
+        if (m->capture) {
+            const size_t need = s->layers.size() * (size_t)T * m->hp.n_embd;
+            if (need > s->streams_cap) {
+                if (s->streams) pi_free(s->streams);
+                s->streams_cap = 0;
+                s->streams = (float *)pi_malloc(need * 4);
+                if (!s->streams) return PI_E_HIP;
+                s->streams_cap = need;
+            }
+            s->streams_T = T;
+        }
+        PI_TRY(pass_layers(m, in));
+        const int32_t * d_rows = s->d_in + 5 * T + items.size();
+        for (int r0 = 0; r0 < (int)rows.size(); r0 += kHeadRows) {
+            const int n = std::min(kHeadRows, (int)rows.size() - r0);
+            const size_t V = m->hp.n_vocab;
+            PI_TRY(pass_head(m, d_rows + r0, n));
+            if (next_tokens) for (int k = 0; k < n; ++k) PI_TRY(pi_k_argmax(s->logits + k * V, (int)V, s->d_next + k, m->stream));
+            PI_HIP_TRY(hipStreamSynchronize(m->stream));
+            std::vector<int32_t> nx(next_tokens ? n : 0);
+            if (next_tokens) PI_TRY(pi_memcpy_d2h(nx.data(), s->d_next, 4 * (size_t)n));
+            for (int k = 0; k < n; ) {                              // runs of places that follow one another leave in one copy
+                int e = k + 1;
+                while (e < n && place[r0 + e] == place[r0 + k] + (e - k)) ++e;
+                if (logits_out) PI_TRY(pi_memcpy_d2h(logits_out + (size_t)place[r0 + k] * V, s->logits + (size_t)k * V, sizeof(float) * V * (e - k)));
+                if (next_tokens) for (int j = k; j < e; ++j) next_tokens[place[r0 + j]] = nx[j];
+                k = e;
+            }
+        }
+    }
+    PI_HIP_TRY(hipStreamSynchronize(m->stream));
+    return PI_OK;
+}
+
+static int ensure_pool(pi_model * m, int64_t n) {
+    if (m->lay->kv.n) return PI_OK;
+    if (n > INT32_MAX) return fail(PI_E_ARG, "the cache pool is too large");
+    return layers_cells_init(m, (int)n);
+}
+
+// tokens at n_past .. of sequence q, behind exactly n_past cells (what lies at n_past and beyond is dropped first)
+static int continue_at(pi_model * m, int q, int n_past) {
+    LayerState * s = m->lay;
+    s->kv.seq_rm(q, n_past, -1);
+    std::vector<int32_t> app;
+    refresh_list(s, q, app);
+    PI_TRY(upload_appends(m, app));
+    const auto & lp = s->list_pos[q];
+    if ((int)lp.size() != n_past || (n_past && (lp.front() != 0 || lp.back() != n_past - 1))) return fail(PI_E_STATE, "the sequence's cells do not hold the positions 0 .. n_past - 1");
+    return PI_OK;
+}
+
+int layers_decode(pi_model * m, const int32_t * tokens, int n_tokens, int n_past, float * logits_out) {
+    LayerState * s = m->lay;
+    if (!tokens || n_tokens <= 0 || n_past < 0 || n_past + n_tokens > m->hp.n_ctx) return fail(PI_E_ARG, "pi_model_decode: token range exceeds the context");
+    PI_TRY(ensure_pool(m, m->hp.n_ctx));
+    PI_TRY(continue_at(m, kOwnSeq, n_past));
+    std::vector<int32_t> pos(n_tokens);
+    for (int i = 0; i < n_tokens; ++i) pos[i] = n_past + i;
+    const std::vector<uint32_t> mask(n_tokens, 1u << kOwnSeq);
+    const int32_t last = n_tokens - 1;
+    int32_t next = -1;
+    PI_TRY(layers_step(m, tokens, pos.data(), mask.data(), n_tokens, &last, 1, &next, logits_out));
+    s->last_tok[kOwnSeq] = next; s->last_pos[kOwnSeq] = n_past + n_tokens;
+    return next;
+}
+
+int layers_batch_init(pi_model * m, int n_seq) {
+    LayerState * s = m->lay;
+    if (s->n_seq) return fail(PI_E_STATE, "pi_model_batch_init: already initialised");
+    PI_TRY(ensure_pool(m, (int64_t)m->hp.n_ctx * (n_seq + 1)));
+    PI_TRY(ensure_capacity(m, n_seq));
+    s->n_seq = n_seq;
+    for (int q = 0; q < n_seq; ++q) { s->last_tok[q] = 0; s->last_pos[q] = 0; }
+    return PI_OK;
+}
+
+int layers_batch_decode(pi_model * m, const int32_t * tokens, const int32_t * positions, int32_t * next_tokens, float * logits_out) {
+    LayerState * s = m->lay;
+    if (!s->n_seq) return fail(PI_E_STATE, "pi_model_batch_decode: pi_model_batch_init first");
+    if (!tokens || !positions) return fail(PI_E_ARG, "pi_model_batch_decode: null pointer");
+    uint32_t mask[kMaxLockstep]; int32_t want[kMaxLockstep], next[kMaxLockstep];
+    for (int q = 0; q < s->n_seq; ++q) {
+        if (positions[q] < 0 || positions[q] >= m->hp.n_ctx) return fail(PI_E_ARG, "pi_model_batch_decode: position outside the context");
+        if (!s->list_pos[q].empty() && s->list_pos[q].back() >= positions[q]) PI_TRY(continue_at(m, q, positions[q]));
+        mask[q] = 1u << q; want[q] = q;
+    }
+    PI_TRY(layers_step(m, tokens, positions, mask, s->n_seq, want, s->n_seq, next, logits_out));
+    for (int q = 0; q < s->n_seq; ++q) {
+        s->last_tok[q] = next[q]; s->last_pos[q] = positions[q] + 1;
+        if (next_tokens) next_tokens[q] = next[q];
+    }
+    return PI_OK;
+}
+
+// the greedy loop of the model's own sequence (own) or of the lockstep sequences: one captured step, replayed
+int layers_generate(pi_model * m, int own, int n_steps, int32_t * out_tokens, float * ms_out) {
+    LayerState * s = m->lay;
+    const int T = own ? 1 : s->n_seq, q0 = own ? kOwnSeq : 0;
+    if (!T || !s->kv.n) return fail(PI_E_STATE, "pi_model_generate: decode a prompt first");
+    if (n_steps <= 0 || n_steps > s->max_steps || !out_tokens) return fail(PI_E_ARG, "pi_model_generate: bad step count");
+    std::vector<int32_t> tok(T), pos(T), vis(T), seq(T), cell(T), cells((size_t)n_steps * T), app;
+    PI_TRY(apply_shift(m));
+    for (int t = 0; t < T; ++t) {
+        seq[t] = q0 + t; tok[t] = s->last_tok[q0 + t]; pos[t] = s->last_pos[q0 + t];
+        refresh_list(s, q0 + t, app);
+        if (pos[t] + n_steps > m->hp.n_ctx) return fail(PI_E_ARG, "pi_model_generate: would run past the context");
+        if ((int)s->list_pos[q0 + t].size() != pos[t]) return fail(PI_E_STATE, "pi_model_generate: a sequence's cells do not end at its next position");
+    }
+    if (!s->kv.find_free(n_steps * T, cells.data())) return fail(PI_E_STATE, "pi_model_generate: not enough free cells");
+    for (int k = 0; k < n_steps; ++k)
+        for (int t = 0; t < T; ++t) take_cell(s, cells[(size_t)k * T + t], pos[t] + k, 1u << (q0 + t), app);
+    s->kv.move_head(cells.back() + 1);
+    PI_TRY(upload_appends(m, app));
+    PI_TRY(ensure_capacity(m, T));
+    for (int t = 0; t < T; ++t) { vis[t] = pos[t] + 1; cell[t] = cells[t]; }
+    std::vector<int32_t> items;
+    Step in;
+    in.T = T; in.tokens = s->g_tok; in.pos = s->g_pos; in.cell = s->g_cell; in.n_vis = s->g_vis; in.seq = s->g_seq;
+    std::vector<int> parts;
+    for (int h : s->head_counts) {
+        Step::Work w;
+        const size_t at = items.size();
+        if (bf16_mode(s)) work_items(seq.data(), vis.data(), T, h, items);
+        w.items = s->g_work + at;
+        w.n = bf16_mode(s) ? (int)(items.size() - at) / 4 : T;
+        w.parts = choose_parts(s, w.n, *std::max_element(pos.begin(), pos.end()) + n_steps);
+        in.work.push_back(w);
+        parts.push_back(w.parts);
+    }
+    PI_HIP_TRY(hipStreamSynchronize(m->stream));
+    const int32_t zero = 0;
+    PI_TRY(pi_memcpy_h2d(s->g_tok, tok.data(), 4 * T)); PI_TRY(pi_memcpy_h2d(s->g_pos, pos.data(), 4 * T)); PI_TRY(pi_memcpy_h2d(s->g_vis, vis.data(), 4 * T));
+    PI_TRY(pi_memcpy_h2d(s->g_seq, seq.data(), 4 * T)); PI_TRY(pi_memcpy_h2d(s->g_cell, cell.data(), 4 * T)); PI_TRY(pi_memcpy_h2d(s->g_step, &zero, 4));
+    if (!items.empty()) PI_TRY(pi_memcpy_h2d(s->g_work, items.data(), 4 * items.size()));
+    s->streams_T = 0;
+    float * const x0 = s->x, * const x20 = s->x2;
+    auto step = [&]() -> int {
+        s->x = x0; s->x2 = x20;                                    // every step starts on the same buffers, whatever the layer count
+        PI_TRY(pass_layers(m, in));
+        PI_TRY(pass_head(m, nullptr, T));
+        PI_TRY(pi_k_argmax_batch(s->logits, m->hp.n_vocab, T, s->g_tok, s->g_pos, s->g_step, s->g_out, s->max_steps, m->stream));
+        return pi_k_cells_advance(T, s->g_seq, s->lists, s->kv.n, s->g_vis, s->g_cell, s->g_step, m->stream);
+    };
+    const char * no_graph = getenv("PI_NO_GRAPH");
+    const bool use_graph = !(no_graph && no_graph[0] == '1');
+    if (use_graph && s->exec && (s->graph_T != T || s->graph_seq0 != q0 || s->graph_parts != parts)) drop_graph(s);
+    if (use_graph && !s->exec) {
+        PI_HIP_TRY(hipStreamBeginCapture(m->stream, hipStreamCaptureModeThreadLocal));
+        const int rc = step();
+        hipGraph_t g = nullptr;
+        const hipError_t e = hipStreamEndCapture(m->stream, &g);
+        if (rc != PI_OK) { if (g) (void)hipGraphDestroy(g); return rc; }
+        if (e != hipSuccess) return hip_fail(e, "hipStreamEndCapture");
+        s->graph = g;
+        PI_HIP_TRY(hipGraphInstantiate(&s->exec, g, nullptr, nullptr, 0));
+        s->graph_T = T; s->graph_seq0 = q0; s->graph_parts = parts;
+    }
+    PI_HIP_TRY(hipEventRecord(m->ev0, m->stream));
+    for (int k = 0; k < n_steps; ++k) {
+        if (use_graph) PI_HIP_TRY(hipGraphLaunch(s->exec, m->stream));
+        else PI_TRY(step());
+    }
+    PI_HIP_TRY(hipEventRecord(m->ev1, m->stream));
+    PI_HIP_TRY(hipStreamSynchronize(m->stream));
+    if (ms_out) PI_HIP_TRY(hipEventElapsedTime(ms_out, m->ev0, m->ev1));
+    PI_TRY(pi_memcpy_d2h(out_tokens, s->g_out, sizeof(int32_t) * (size_t)n_steps * T));
+    for (int t = 0; t < T; ++t) { s->last_tok[q0 + t] = out_tokens[(size_t)(n_steps - 1) * T + t]; s->last_pos[q0 + t] = pos[t] + n_steps; }
+    return PI_OK;
+}
+
+int layers_seq_edit(pi_model * m, int seq, int p0, int p1, int delta, bool shift) {
+    LayerState * s = m->lay;
+    if (seq < -1 || seq >= s->n_seq || !s->kv.n) return fail(PI_E_ARG, "KV edit: bad sequence");
+    const int q = seq < 0 ? kOwnSeq : seq;
+    if (shift) s->kv.seq_shift(q, p0, p1, delta); else s->kv.seq_rm(q, p0, p1);
+    const int n = live_cells(s, q);
+    s->last_pos[q] = n;
+    return n;
+}
+
+int layers_seq_cp(pi_model * m, int src, int dst, int p0, int p1) {
+    LayerState * s = m->lay;
+    if (src < 0 || dst < 0 || src >= s->n_seq || dst >= s->n_seq || src == dst) return fail(PI_E_ARG, "pi_model_batch_kv_seq_cp: bad sequences");
+    if (live_cells(s, dst) != std::max(p0, 0)) return fail(PI_E_UNSUPPORTED, "pi_model_batch_kv_seq_cp: the destination must hold exactly p0 cells");
+    s->kv.seq_cp(src, dst, p0, p1);                                // shared, not copied
+    s->last_pos[dst] = live_cells(s, dst);
+    return s->last_pos[dst];
+}
+
+}  // namespace pi
+
+extern "C" {
+
+pi_model * pi_model_create_layers(const pi_hparams * hp, const pi_layers_opts * opts, const pi_layer_desc * layers, int n_layer) {
+    const auto bad = [](const char * why) -> pi_model * { pi::set_error(why); return nullptr; };
+    if (!hp || !opts || !layers || n_layer <= 0 || hp->n_embd <= 0 || hp->n_vocab <= 0 || hp->n_ctx <= 0 || hp->arch != PI_ARCH_LERASUN ||
+        (opts->compute != PI_TYPE_BF16 && opts->compute != PI_TYPE_F32) || opts->max_batch < 0)
+        return bad("pi_model_create_layers: inconsistent hyper-parameters");
+    for (int il = 0; il < n_layer; ++il) {
+        const pi_layer_desc & d = layers[il];
+        if (d.mixer != PI_MIXER_LATENT || d.n_head <= 0 || d.dim <= 0 || d.rot_dim <= 0 || d.rot_dim % 2 || d.vdim <= 0 || d.kv_rank <= 0 || !(d.rot_base > 0.0))
+            return bad("pi_model_create_layers: a layer's mixer");
+        if (d.kv_from >= 0) {
+            if (d.kv_from >= il) return bad("pi_model_create_layers: kv_from must name an earlier layer");
+            const pi_layer_desc & o = layers[d.kv_from];
+            if (o.kv_from >= 0 || o.kv_rank != d.kv_rank || o.rot_dim != d.rot_dim || o.rot_base != d.rot_base)
+                return bad("pi_model_create_layers: kv_from must name a layer with cells of its own and the same latent and rotation");
+        }
+        if (d.ffn != PI_FFN_NONE && (d.ffn != PI_FFN_MOE || d.n_expert <= 0 || d.n_group <= 0 || d.n_expert % d.n_group || d.n_group_keep <= 0 || d.n_group_keep > d.n_group ||
+                                     d.n_top <= 0 || d.n_top > d.n_group_keep * (d.n_expert / d.n_group) || d.expert_ff <= 0))
+            return bad("pi_model_create_layers: a layer's experts");
+    }
+    if (pi_init(0) != PI_OK) return nullptr;
+    pi_model * m = new pi_model();
+    m->hp = *hp;
+    m->hp.n_layer = n_layer;
+    m->layers.resize((size_t)n_layer * PI_T_COUNT);
+    m->lay = new LayerState();
+    m->lay->opts = *opts;
+    for (int il = 0; il < n_layer; ++il) { Layer L; L.d = layers[il]; m->lay->layers.push_back(L); }
+    return m;
+}
+
+int pi_model_get_streams(pi_model * m, float * out) {
+    if (!m || !m->finalized || !m->lay || !m->capture || !m->lay->streams_T) return pi::fail(PI_E_STATE, "pi_model_get_streams: run a step with capture enabled first");
+    LayerState * s = m->lay;
+    PI_HIP_TRY(hipStreamSynchronize(m->stream));
+    if (out) PI_TRY(pi_memcpy_d2h(out, s->streams, sizeof(float) * s->layers.size() * (size_t)s->streams_T * m->hp.n_embd));
+    return s->streams_T;
+}
+
+}  // extern "C"

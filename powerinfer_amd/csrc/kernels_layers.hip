@@ -1,0 +1,335 @@
+// Operators of the models that are described layer by layer, apart from attention: embedding + norm, the pair of norms of a parallel
+// layer, grouped mat-muls (heads of a latent attention, experts), rotation angles, expert choice, and the sum that closes a layer.
+// Templated on the storage of activations: bf16 (matrix cores on bf16 operands, fp32 accumulation) or fp32.
+#include "layer_types.hpp"
+
+namespace {
+
+// ---------------------------------------------------------------------------------------------------------------------------------
+// norms
+// ---------------------------------------------------------------------------------------------------------------------------------
+// 1 / sqrt(mean(x^2) + eps) of a row the workgroup reads together (squares summed in fp64, fixed order)
+template <typename LD> __device__ float row_rms_scale(int cols, float eps, double * red, LD && ld) {
+    double s = 0.0;
+    for (int i = threadIdx.x; i < cols; i += blockDim.x) { const float v = ld(i); s += (double)v * (double)v; }
+    s = block_sum_f64(s, red);
+    return pi_inv_sqrt((float)(s / cols) + eps);
+}
+
+__global__ __launch_bounds__(256) void embed_norm_kernel(const uint16_t * __restrict__ table, int cols, const int32_t * __restrict__ tokens,
+                                                         const float * __restrict__ w, float eps, float * __restrict__ x) {
+    __shared__ double red[4];
+    const uint16_t * row = table + (size_t)tokens[blockIdx.x] * cols;
+    const float sc = row_rms_scale(cols, eps, red, [&](int i) { return bf16_to_f32(row[i]); });
+    for (int i = threadIdx.x; i < cols; i += blockDim.x) x[(size_t)blockIdx.x * cols + i] = bf16_to_f32(row[i]) * sc * w[i];
+}
+
+template <typename ST>
+__global__ __launch_bounds__(1024) void norm_pair_kernel(const float * __restrict__ x, const int32_t * __restrict__ rows, int cols, float eps,
+                                                        const float * __restrict__ wa, ST * __restrict__ out_a, const float * __restrict__ wb,
+                                                        ST * __restrict__ out_b, int ld, int ol) {
+    __shared__ double red[16];
+    const float * xt = x + (size_t)(rows ? rows[blockIdx.x] : blockIdx.x) * cols;
+    auto at = [&](int i) -> size_t { return ol ? pi_ol_index(blockIdx.x, i) : (size_t)blockIdx.x * ld + i; };
+    if (cols <= 4 * (int)blockDim.x) {              // one memory round trip: the row and both weight vectors are requested together
+        float xv[4], av[4], bv[4];
+        double s = 0.0;
+#pragma unroll
+        for (int k = 0; k < 4; ++k) {
+            const int i = threadIdx.x + k * blockDim.x;
+            xv[k] = i < cols ? xt[i] : 0.0f;
+            av[k] = i < cols ? wa[i] : 0.0f;
+            bv[k] = wb && i < cols ? wb[i] : 0.0f;
+            s += (double)xv[k] * (double)xv[k];
+        }
+        s = block_sum_f64(s, red);
+        const float sc = pi_inv_sqrt((float)(s / cols) + eps);
+#pragma unroll
+        for (int k = 0; k < 4; ++k) {
+            const int i = threadIdx.x + k * blockDim.x;
+            if (i < cols) {
+                out_a[at(i)] = to_st<ST>(xv[k] * sc * av[k]);
+                if (wb) out_b[at(i)] = to_st<ST>(xv[k] * sc * bv[k]);
+            }
+        }
+        return;
+    }
+    const float sc = row_rms_scale(cols, eps, red, [&](int i) { return xt[i]; });
+    for (int i = threadIdx.x; i < cols; i += blockDim.x) {
+        const float v = xt[i] * sc;
+        out_a[at(i)] = to_st<ST>(v * wa[i]);
+        if (wb) out_b[at(i)] = to_st<ST>(v * wb[i]);
+    }
+}
+
+// ---------------------------------------------------------------------------------------------------------------------------------
+// grouped mat-mul.  A workgroup of four waves owns 64 rows of one group's matrix x 32 of the group's tokens; each wave holds 16 rows in
+// the matrix cores' operand layout (lane l: row l % 16, eight consecutive columns 8 * (l / 16) of a 32-column step) against two token
+// tiles.  fp32 storage runs the same steps on v_mfma_f32_16x16x4_f32, eight per 32 columns.
+// ---------------------------------------------------------------------------------------------------------------------------------
+template <typename ST>
+__global__ __launch_bounds__(256) void group_gemm_kernel(pi_group_gemm g) {
+    const int grp = blockIdx.z;
+    const int lo = g.off ? g.off[grp] : 0, n = g.off ? g.off[grp + 1] - lo : g.T;
+    const int t0 = blockIdx.y * 32;
+    if (t0 >= n) return;
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, i = lane & 15, q = lane >> 4;
+    const int row0 = blockIdx.x * 64 + wave * 16;
+    if (row0 >= g.rows) return;
+    const uint16_t * W = (const uint16_t *)g.W + (size_t)grp * g.w_gs + (size_t)min(row0 + i, g.rows - 1) * g.ldw + q * 8;
+    const ST * xb = (const ST *)g.x + (g.off ? 0 : (size_t)grp * g.x_gs);
+    const ST * xp[2];
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+        const int t = min(t0 + u * 16 + i, n - 1);
+        const int xr = g.off ? (g.gather ? g.gather[lo + t] / g.gather_div : lo + t) : t;
+        xp[u] = xb + (size_t)xr * g.ldx + q * 8;
+    }
+    pi_f4 acc[2] = {pi_f4{0, 0, 0, 0}, pi_f4{0, 0, 0, 0}};
+    const bool two = t0 + 16 < n;
+#pragma unroll 4
+    for (int k = 0; k < g.cols; k += 32) {
+        const Frag<ST> a = frag_weights<ST>(W + k);
+        frag_mma(a, frag_load(xp[0] + k), acc[0]);
+        if (two) frag_mma(a, frag_load(xp[1] + k), acc[1]);
+    }
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+        const int t = t0 + u * 16 + i;
+        if (t >= n) continue;
+        const size_t yr = g.off ? (size_t)(lo + t) * g.ldy : (size_t)grp * g.y_gs + (size_t)t * g.ldy;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int row = row0 + 4 * q + r;
+            if (row >= g.rows) continue;
+            float v = acc[u][r] * g.alpha;
+            if (g.relu2) { v = fmaxf(v, 0.0f); v *= v; }
+            if (g.y_f32) ((float *)g.y)[yr + row] = v;
+            else ((ST *)g.y)[yr + row] = to_st<ST>(v);
+        }
+    }
+}
+
+// ---------------------------------------------------------------------------------------------------------------------------------
+// rotation angles: formed and reduced in fp64, so that the fp32 cosine and sine are right at any position
+// ---------------------------------------------------------------------------------------------------------------------------------
+__global__ void rope_angles_kernel(const int32_t * __restrict__ pos, int T, int dims, double base, float2 * __restrict__ cs) {
+    const int half = dims / 2, idx = blockIdx.x * blockDim.x + threadIdx.x;
+    if (idx >= T * half) return;
+    const int t = idx / half, i = idx % half;
+    double s, c;
+    sincos((double)pos[t] * pow(base, -2.0 * (double)i / (double)dims), &s, &c);
+    cs[idx] = make_float2((float)c, (float)s);
+}
+
+// ---------------------------------------------------------------------------------------------------------------------------------
+// expert choice, one wave per token: scores, choice scores and the groups' sums in LDS, arg-max passes over the lanes (the lower index
+// wins a tie)
+// ---------------------------------------------------------------------------------------------------------------------------------
+__device__ __forceinline__ void wave_argmax(float & v, int & i) {
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+        const float ov = __shfl_xor(v, o, PI_WAVE); const int oi = __shfl_xor(i, o, PI_WAVE);
+        if (ov > v || (ov == v && oi < i)) { v = ov; i = oi; }
+    }
+}
+
+__global__ __launch_bounds__(64) void route_kernel(const float * __restrict__ z, int E, int top, int G, int keep, const float * __restrict__ bias,
+                                                   int32_t * __restrict__ ids, float * __restrict__ weights) {
+    extern __shared__ float sm[];
+    float * sc = sm, * ch = sm + E, * gs = sm + 2 * E;        // [E] scores, [E] choice scores, [G] group sums
+    const int t = blockIdx.x, lane = threadIdx.x, size = E / G;
+    for (int e = lane; e < E; e += 64) {
+        const float s = 1.0f / (1.0f + expf(-z[(size_t)t * E + e]));
+        sc[e] = s;
+        ch[e] = s + bias[e];
+    }
+    __syncthreads();
+    if (keep < G) {
+        for (int g = lane; g < G; g += 64) {
+            float a = -INFINITY, b = -INFINITY;
+            for (int k = 0; k < size; ++k) {
+                const float v = ch[g * size + k];
+                if (v > a) { b = a; a = v; } else if (v > b) b = v;
+            }
+            gs[g] = size > 1 ? a + b : a;
+        }
+        __syncthreads();
+        // a group stays if fewer than `keep` groups come before it (larger sum, or the same sum and a lower index)
+        for (int g = lane; g < G; g += 64) {
+            int before = 0;
+            for (int o = 0; o < G; ++o) before += (gs[o] > gs[g] || (gs[o] == gs[g] && o < g)) ? 1 : 0;
+            if (before >= keep) for (int k = 0; k < size; ++k) ch[g * size + k] = -INFINITY;
+        }
+        __syncthreads();
+    }
+    float total = 0.0f;
+    for (int k = 0; k < top; ++k) {
+        float v = -INFINITY; int idx = E;
+        for (int e = lane; e < E; e += 64) {
+            const float c = ch[e];
+            if (c > v || (c == v && e < idx)) { v = c; idx = e; }
+        }
+        wave_argmax(v, idx);
+        if (idx >= E) idx = 0;                                 // not-a-number scores: any expert, never an index outside
+        const float s = sc[idx];
+        total += s;
+        if (lane == 0) { ids[(size_t)t * top + k] = idx; weights[(size_t)t * top + k] = s; ch[idx] = __int_as_float(0x7fc00000); }   // taken: compares false with everything
+        __syncthreads();
+    }
+    for (int k = lane; k < top; k += 64) weights[(size_t)t * top + k] = weights[(size_t)t * top + k] / (total + 1e-20f);
+}
+
+// pairs in expert order, one workgroup: thread e counts and places the pairs of expert e (and e + 1024, ...), reading the ids of a block
+// of pairs from LDS; pairs keep their order within an expert
+constexpr int kSortTile = 4096;
+__global__ __launch_bounds__(1024) void moe_sort_kernel(const int32_t * __restrict__ ids, int n, int E, int32_t * __restrict__ off, int32_t * __restrict__ perm,
+                                                        int32_t * __restrict__ inv) {
+    __shared__ int32_t tile[kSortTile];
+    __shared__ int sred[16];
+    int base = 0;
+    for (int e0 = 0; e0 < E; e0 += 1024) {
+        const int e = e0 + threadIdx.x;
+        int cnt = 0;
+        for (int p0 = 0; p0 < n; p0 += kSortTile) {
+            const int m = min(kSortTile, n - p0);
+            __syncthreads();
+            for (int p = threadIdx.x; p < m; p += 1024) tile[p] = ids[p0 + p];
+            __syncthreads();
+            if (e < E) for (int p = 0; p < m; ++p) cnt += tile[p] == e ? 1 : 0;
+        }
+        int tot;
+        int at = base + block_exclusive_scan_i32(cnt, &tot, sred);
+        if (e < E) off[e] = at;
+        for (int p0 = 0; p0 < n; p0 += kSortTile) {
+            const int m = min(kSortTile, n - p0);
+            __syncthreads();
+            for (int p = threadIdx.x; p < m; p += 1024) tile[p] = ids[p0 + p];
+            __syncthreads();
+            if (e < E) for (int p = 0; p < m; ++p) if (tile[p] == e) { perm[at] = p0 + p; inv[p0 + p] = at; ++at; }
+        }
+        base += tot;
+    }
+    if (threadIdx.x == 0) off[E] = base;
+}
+
+__global__ __launch_bounds__(256) void moe_combine_kernel(const float * __restrict__ x, const float * __restrict__ mix, const float * __restrict__ y,
+                                                          const int32_t * __restrict__ inv, const float * __restrict__ weights, int top, int cols,
+                                                          float * __restrict__ out, float * __restrict__ keep) {
+    const int t = blockIdx.y, c = blockIdx.x * 256 + threadIdx.x;
+    if (c >= cols) return;
+    const size_t o = (size_t)t * cols + c;
+    float s = 0.0f;
+    if (weights) for (int k = 0; k < top; ++k) s = fmaf(weights[(size_t)t * top + k], y[(size_t)inv[(size_t)t * top + k] * cols + c], s);
+    const float v = x[o] + (mix[o] + s);
+    out[o] = v;
+    if (keep) keep[o] = v;
+}
+
+__global__ void pad_cols_kernel(const uint16_t * __restrict__ in, int64_t rows, int cols, uint16_t * __restrict__ out, int ld) {
+    for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < rows * ld; i += (int64_t)gridDim.x * blockDim.x) {
+        const int64_t r = i / ld; const int c = (int)(i % ld);
+        out[i] = c < cols ? in[r * cols + c] : (uint16_t)0;
+    }
+}
+__global__ void transpose_pad_kernel(const uint16_t * __restrict__ in, int n_mat, int rows, int cols, uint16_t * __restrict__ out, int ld) {
+    const int64_t n = (int64_t)n_mat * cols * ld;
+    for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (int64_t)gridDim.x * blockDim.x) {
+        const int r = (int)(i % ld); const int64_t mc = i / ld;
+        const int64_t mat = mc / cols; const int c = (int)(mc % cols);
+        out[i] = r < rows ? in[(mat * rows + r) * cols + c] : (uint16_t)0;
+    }
+}
+
+__global__ void cells_advance_kernel(int T, const int32_t * __restrict__ seq, const int32_t * __restrict__ lists, size_t list_ld, int32_t * __restrict__ n_vis,
+                                     int32_t * __restrict__ cell, int32_t * step) {
+    const int t = threadIdx.x;
+    if (t < T) {
+        const int n = n_vis[t] + 1;
+        n_vis[t] = n;
+        cell[t] = lists[(size_t)seq[t] * list_ld + n - 1];
+    }
+    if (t == 0) *step += 1;
+}
+
+}  // namespace
+
+extern "C" {
+
+int pi_k_embed_norm(const void * table, int cols, const int32_t * tokens, int T, const float * w, float eps, float * x, pi_stream_t stream) {
+    if (!table || !tokens || !w || !x || cols <= 0 || T <= 0) return pi::fail(PI_E_ARG, "pi_k_embed_norm: bad arguments");
+    hipLaunchKernelGGL(embed_norm_kernel, dim3(T), dim3(256), 0, (hipStream_t)stream, (const uint16_t *)table, cols, tokens, w, eps, x);
+    return pi::check_launch("pi_k_embed_norm");
+}
+
+int pi_k_norm_pair(int type, const float * x, const int32_t * rows, int T, int cols, float eps, const float * wa, void * out_a,
+                   const float * wb, void * out_b, int ld, int ol, pi_stream_t stream) {
+    if (!x || !wa || !out_a || (wb && !out_b) || T <= 0 || cols <= 0 || ld < cols) return pi::fail(PI_E_ARG, "pi_k_norm_pair: bad arguments");
+    if (ol && (type != PI_TYPE_BF16 || T > kBtMaxT || ld % 8)) return pi::fail(PI_E_ARG, "pi_k_norm_pair: operand layout needs BF16, T <= 16, ld % 8 == 0");
+    const int block = cols > 2048 ? 1024 : cols > 512 ? 512 : 256;
+    if (type == PI_TYPE_BF16)
+        hipLaunchKernelGGL(norm_pair_kernel<bf16>, dim3(T), dim3(block), 0, (hipStream_t)stream, x, rows, cols, eps, wa, (bf16 *)out_a, wb, (bf16 *)out_b, ld, ol);
+    else if (type == PI_TYPE_F32)
+        hipLaunchKernelGGL(norm_pair_kernel<float>, dim3(T), dim3(block), 0, (hipStream_t)stream, x, rows, cols, eps, wa, (float *)out_a, wb, (float *)out_b, ld, 0);
+    else return pi::fail(PI_E_UNSUPPORTED, "pi_k_norm_pair: type");
+    return pi::check_launch("pi_k_norm_pair");
+}
+
+int pi_k_group_gemm(int type, const pi_group_gemm * g, pi_stream_t stream) {
+    if (!g || !g->W || !g->x || !g->y || g->rows <= 0 || g->cols <= 0 || g->cols % 32 || g->ldw < g->cols || g->ldw % 8 || g->ldx < g->cols || g->ldx % 8 ||
+        g->ldy < g->rows || g->T <= 0 || g->n_group <= 0 || g->n_group > 65535 || (g->gather && g->gather_div <= 0) || g->w_gs % 8 || g->x_gs % 8)
+        return pi::fail(PI_E_ARG, "pi_k_group_gemm: bad arguments");
+    const dim3 grid((g->rows + 63) / 64, (g->T + 31) / 32, g->n_group);
+    if (grid.y > 65535) return pi::fail(PI_E_ARG, "pi_k_group_gemm: too many tokens");
+    if (type == PI_TYPE_BF16) hipLaunchKernelGGL(group_gemm_kernel<bf16>, grid, dim3(256), 0, (hipStream_t)stream, *g);
+    else if (type == PI_TYPE_F32) hipLaunchKernelGGL(group_gemm_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream, *g);
+    else return pi::fail(PI_E_UNSUPPORTED, "pi_k_group_gemm: type");
+    return pi::check_launch("pi_k_group_gemm");
+}
+
+int pi_k_rope_angles(const int32_t * pos, int T, int dims, double base, void * cs, pi_stream_t stream) {
+    if (!pos || !cs || T <= 0 || dims <= 0 || dims % 2 || !(base > 0.0)) return pi::fail(PI_E_ARG, "pi_k_rope_angles: bad arguments");
+    hipLaunchKernelGGL(rope_angles_kernel, dim3((T * (dims / 2) + 63) / 64), dim3(64), 0, (hipStream_t)stream, pos, T, dims, base, (float2 *)cs);
+    return pi::check_launch("pi_k_rope_angles");
+}
+
+int pi_k_route(const float * z, int T, int n_expert, int n_top, int n_group, int n_keep, const float * bias, int32_t * ids, float * weights, pi_stream_t stream) {
+    if (!z || !bias || !ids || !weights || T <= 0 || n_expert <= 0 || n_expert > 8192 || n_top <= 0 || n_group <= 0 || n_expert % n_group || n_keep <= 0 || n_keep > n_group ||
+        n_top > n_keep * (n_expert / n_group))
+        return pi::fail(PI_E_ARG, "pi_k_route: bad arguments");
+    hipLaunchKernelGGL(route_kernel, dim3(T), dim3(64), sizeof(float) * (2 * n_expert + n_group), (hipStream_t)stream, z, n_expert, n_top, n_group, n_keep, bias, ids, weights);
+    return pi::check_launch("pi_k_route");
+}
+
+int pi_k_moe_sort(const int32_t * ids, int n_pairs, int n_expert, int32_t * off, int32_t * perm, int32_t * inv, pi_stream_t stream) {
+    if (!ids || !off || !perm || !inv || n_pairs <= 0 || n_expert <= 0) return pi::fail(PI_E_ARG, "pi_k_moe_sort: bad arguments");
+    hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(1024), 0, (hipStream_t)stream, ids, n_pairs, n_expert, off, perm, inv);
+    return pi::check_launch("pi_k_moe_sort");
+}
+
+int pi_k_moe_combine(const float * x, const float * mix, const float * y, const int32_t * inv, const float * weights, int n_top, int T, int cols,
+                     float * out, float * keep, pi_stream_t stream) {
+    if (!x || !mix || !out || T <= 0 || T > 65535 || cols <= 0 || (weights && (!y || !inv || n_top <= 0))) return pi::fail(PI_E_ARG, "pi_k_moe_combine: bad arguments");
+    hipLaunchKernelGGL(moe_combine_kernel, dim3((cols + 255) / 256, T), dim3(256), 0, (hipStream_t)stream, x, mix, y, inv, weights, n_top, cols, out, keep);
+    return pi::check_launch("pi_k_moe_combine");
+}
+
+int pi_k_pad_cols_bf16(const void * in, int64_t rows, int cols, void * out, int ld, pi_stream_t stream) {
+    if (!in || !out || rows <= 0 || cols <= 0 || ld < cols) return pi::fail(PI_E_ARG, "pi_k_pad_cols_bf16: bad arguments");
+    hipLaunchKernelGGL(pad_cols_kernel, dim3(4096), dim3(256), 0, (hipStream_t)stream, (const uint16_t *)in, rows, cols, (uint16_t *)out, ld);
+    return pi::check_launch("pi_k_pad_cols_bf16");
+}
+
+int pi_k_transpose_pad_bf16(const void * in, int n_mat, int rows, int cols, void * out, int ld, pi_stream_t stream) {
+    if (!in || !out || n_mat <= 0 || rows <= 0 || cols <= 0 || ld < rows) return pi::fail(PI_E_ARG, "pi_k_transpose_pad_bf16: bad arguments");
+    hipLaunchKernelGGL(transpose_pad_kernel, dim3(4096), dim3(256), 0, (hipStream_t)stream, (const uint16_t *)in, n_mat, rows, cols, (uint16_t *)out, ld);
+    return pi::check_launch("pi_k_transpose_pad_bf16");
+}
+
+int pi_k_cells_advance(int T, const int32_t * seq, const int32_t * lists, size_t list_ld, int32_t * n_vis, int32_t * cell, int32_t * step, pi_stream_t stream) {
+    if (T <= 0 || T > 64 || !seq || !lists || !n_vis || !cell || !step) return pi::fail(PI_E_ARG, "pi_k_cells_advance: bad arguments");
+    hipLaunchKernelGGL(cells_advance_kernel, dim3(1), dim3(64), 0, (hipStream_t)stream, T, seq, lists, list_ld, n_vis, cell, step);
+    return pi::check_launch("pi_k_cells_advance");
+}
+
+}  // extern "C"

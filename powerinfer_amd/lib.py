@@ -11,7 +11,8 @@ import numpy as np
 HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(HERE, "libpowerinfer_hip.so")
 
-F32, F16, Q4_0, I32 = 0, 1, 2, 18
+F32, F16, Q4_0, I32, BF16 = 0, 1, 2, 18, 30
+MIXER_LATENT, FFN_NONE, FFN_MOE = 0, 0, 1
 EPI_NONE, EPI_RELU, EPI_ADD, EPI_ADD2 = 0, 1, 2, 3
 NORM_NONE, NORM_RMS, NORM_LAYER = 0, 1, 2
 
@@ -20,6 +21,24 @@ _vp, _i, _f, _sz, _u64 = C.c_void_p, C.c_int, C.c_float, C.c_size_t, C.c_uint64
 
 class Norm(C.Structure):
     _fields_ = [("kind", C.c_int32), ("eps", C.c_float), ("w", C.c_void_p), ("b", C.c_void_p)]
+
+
+class GroupGemm(C.Structure):
+    _fields_ = [("W", _vp), ("w_gs", _sz), ("rows", C.c_int32), ("cols", C.c_int32), ("ldw", C.c_int32), ("n_group", C.c_int32),
+                ("x", _vp), ("x_gs", _sz), ("ldx", C.c_int32), ("T", C.c_int32),
+                ("y", _vp), ("y_gs", _sz), ("ldy", C.c_int32), ("y_f32", C.c_int32), ("relu2", C.c_int32),
+                ("alpha", _f), ("off", _vp), ("gather", _vp), ("gather_div", C.c_int32)]
+
+
+class LatentPrep(C.Structure):
+    _fields_ = [("z", _vp)] + [(n, C.c_int32) for n in ("ldz", "T", "n_head", "dim", "dim_ld", "rot_dim", "kv_rank", "rank_ld", "kd")] + [
+        ("cs", _vp), ("norm_w", _vp), ("eps", _f), ("q_un", _vp), ("q_lat", _vp), ("cache", _vp), ("cell", _vp)]
+
+
+class LatentAttn(C.Structure):
+    _fields_ = [("q_lat", _vp), ("cache", _vp), ("lists", _vp), ("list_ld", _sz), ("work", _vp), ("n_vis", _vp)] + [
+        (n, C.c_int32) for n in ("n_work", "T", "n_head", "kv_rank", "rank_ld", "kd", "n_parts")] + [
+        ("scale", _f), ("sink", _vp), ("scratch", _vp), ("out_lat", _vp)]
 
 
 class PiError(RuntimeError):
@@ -142,6 +161,22 @@ _SIGS = {
     "pi_k_attn_fused": (_i, [_vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _vp, _vp, _vp]),
     "pi_k_embed": (_i, [_i, _vp, _i, _vp, _vp, _vp]),
     "pi_k_argmax": (_i, [_vp, _i, _vp, _vp]),
+    "pi_k_embed_norm": (_i, [_vp, _i, _vp, _i, _vp, _f, _vp, _vp]),
+    "pi_k_norm_pair": (_i, [_i, _vp, _vp, _i, _i, _f, _vp, _vp, _vp, _vp, _i, _i, _vp]),
+    "pi_k_group_gemm": (_i, [_i, C.POINTER(GroupGemm), _vp]),
+    "pi_k_rope_angles": (_i, [_vp, _i, _i, C.c_double, _vp, _vp]),
+    "pi_k_latent_prep": (_i, [_i, C.POINTER(LatentPrep), _vp]),
+    "pi_k_latent_attn_rows": (_i, [_i]),
+    "pi_k_latent_attn_supported": (_i, [_i, _i, _i]),
+    "pi_k_latent_attn_scratch_floats": (_sz, [_i, _i, _i, _i]),
+    "pi_k_latent_attn": (_i, [_i, C.POINTER(LatentAttn), _vp]),
+    "pi_k_latent_shift": (_i, [_i, _vp, _i, _i, _i, _i, C.c_double, _vp, _vp]),
+    "pi_k_route": (_i, [_vp, _i, _i, _i, _i, _i, _vp, _vp, _vp, _vp]),
+    "pi_k_moe_sort": (_i, [_vp, _i, _i, _vp, _vp, _vp, _vp]),
+    "pi_k_moe_combine": (_i, [_vp, _vp, _vp, _vp, _vp, _i, _i, _i, _vp, _vp, _vp]),
+    "pi_k_pad_cols_bf16": (_i, [_vp, C.c_int64, _i, _vp, _i, _vp]),
+    "pi_k_transpose_pad_bf16": (_i, [_vp, _i, _i, _i, _vp, _i, _vp]),
+    "pi_k_cells_advance": (_i, [_i, _vp, _vp, _sz, _vp, _vp, _vp, _vp]),
 }
 
 

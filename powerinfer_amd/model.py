@@ -7,14 +7,16 @@ import numpy as np
 from . import lib as pl
 from .lib import check
 
-ARCH = {"llama": 0, "falcon": 1}
+ARCH = {"llama": 0, "falcon": 1, "lerasun": 2}
 
 # tensor roles, same order as the enum in include/powerinfer_hip.h
 KINDS = ["tok_embd", "output_norm", "output_norm_b", "output",
          "attn_norm", "attn_norm_b", "attn_norm_2", "attn_norm_2_b",
          "wq", "wk", "wv", "wqkv", "wo",
          "ffn_norm", "ffn_gate", "ffn_up", "ffn_down_t",
-         "fc1", "fc2", "gpu_idx", "gpu_bucket", "neuron_rate"]
+         "fc1", "fc2", "gpu_idx", "gpu_bucket", "neuron_rate",
+         "embd_norm", "mix_q", "mix_dkv", "mix_dkv_norm", "mix_uk", "mix_uv", "mix_sink",
+         "router", "router_bias", "expert_up", "expert_down"]
 KIND = {k: i for i, k in enumerate(KINDS)}
 
 
@@ -24,8 +26,22 @@ class HParamsC(C.Structure):
                 ("norm_eps", C.c_float), ("rope_freq_base", C.c_float), ("sparse_threshold", C.c_float), ("rope_freq_scale", C.c_float)]
 
 
+class LayerDescC(C.Structure):
+    _fields_ = [(n, C.c_int32) for n in ("mixer", "n_head", "dim", "rot_dim", "vdim", "kv_rank", "kv_from")] + [
+        ("scale", C.c_float), ("rot_base", C.c_double)] + [
+        (n, C.c_int32) for n in ("ffn", "n_expert", "n_top", "n_group", "n_group_keep", "expert_ff")]
+
+
+class LayersOptsC(C.Structure):
+    _fields_ = [("compute", C.c_int32), ("logit_scale", C.c_float), ("norm_offset", C.c_float), ("max_batch", C.c_int32)]
+
+
 def _declare(L):
     vp, i = C.c_void_p, C.c_int
+    L.pi_model_create_layers.restype = vp
+    L.pi_model_create_layers.argtypes = [C.POINTER(HParamsC), C.POINTER(LayersOptsC), C.POINTER(LayerDescC), i]
+    L.pi_model_get_streams.restype, L.pi_model_get_streams.argtypes = i, [vp, vp]
+    L.pi_model_kv_cells_step.restype, L.pi_model_kv_cells_step.argtypes = i, [vp, vp, vp, vp, i, vp, i, vp, vp]
     L.pi_model_create.restype, L.pi_model_create.argtypes = vp, [C.POINTER(HParamsC)]
     L.pi_model_free.restype, L.pi_model_free.argtypes = None, [vp]
     L.pi_model_set_tensor.restype, L.pi_model_set_tensor.argtypes = i, [vp, i, i, i, vp, C.c_int64, C.c_int64, i]
@@ -59,7 +75,7 @@ def _declare(L):
     L.pi_model_time_section.restype, L.pi_model_time_section.argtypes = i, [vp, i, i, C.POINTER(C.c_float), C.POINTER(C.c_int)]
 
 
-ENGINE_SYMBOLS = ["pi_model_create", "pi_model_free", "pi_model_set_tensor", "pi_model_finalize", "pi_model_kv_clear",
+ENGINE_SYMBOLS = ["pi_model_create", "pi_model_create_layers", "pi_model_get_streams", "pi_model_kv_cells_step", "pi_model_free", "pi_model_set_tensor", "pi_model_finalize", "pi_model_kv_clear",
                   "pi_model_kv_seq_rm", "pi_model_kv_seq_shift",
                   "pi_model_decode", "pi_model_generate", "pi_model_set_capture", "pi_model_get_capture", "pi_model_set_rest_on_gpu",
                   "pi_model_step_active", "pi_model_time_section",
@@ -79,6 +95,8 @@ def _type_of(a, hint):
         return pl.I32
     if a.dtype == np.uint8:
         return pl.Q4_0
+    if a.dtype == np.uint16:                     # bf16 bit patterns
+        return pl.BF16
     raise TypeError(f"{hint}: unsupported dtype {a.dtype}")
 
 
@@ -252,6 +270,20 @@ class Model:
                                               logits.ctypes.data_as(C.c_void_p) if want_logits else None), "pi_model_kv_cells_decode")
         return nxt, logits
 
+    def kv_cells_step(self, tokens, positions, masks, want, want_logits=True, want_next=True):
+        """One step of any number of tokens (several sequences behind one another).  masks[t]: the bit set of the sequences token t's cell
+        belongs to; want: indices of the tokens whose next token / logits are returned.  Returns (next tokens or None, logits or None)."""
+        tokens, positions = np.ascontiguousarray(tokens, np.int32), np.ascontiguousarray(positions, np.int32)
+        masks, want = np.ascontiguousarray(masks, np.uint32), np.ascontiguousarray(want, np.int32)
+        if not tokens.size == positions.size == masks.size:
+            raise pl.PiError("kv_cells_step: one position and one sequence set per token")
+        nxt = np.empty(want.size, np.int32) if want_next else None
+        logits = np.empty((want.size, self.hp.n_vocab), np.float32) if want_logits else None
+        p = lambda a: a.ctypes.data_as(C.c_void_p) if a is not None and a.size else None  # noqa: E731
+        check(self.L.pi_model_kv_cells_step(self.h, p(tokens), p(positions), p(masks), int(tokens.size), p(want), int(want.size), p(nxt), p(logits)),
+              "pi_model_kv_cells_step")
+        return nxt, logits
+
     def kv_cells_seq_rm(self, seq, p0, p1):
         check(self.L.pi_model_kv_cells_seq_rm(self.h, seq, p0, p1), "pi_model_kv_cells_seq_rm")
 
@@ -299,3 +331,34 @@ class Model:
             self.close()
         except Exception:
             pass
+
+
+class LayerModel(Model):
+    """A model described layer by layer (pi_model_create_layers); every entry point of Model that is not about sparse FFN rows works on it."""
+
+    def __init__(self, arch, descs, n_embd, n_vocab, n_ctx, norm_eps, compute=pl.BF16, logit_scale=1.0, norm_offset=0.0, max_batch=0):
+        from .synth import HParams
+        self.L = pl.init()
+        _declare(self.L)
+        self.hp = HParams(arch=arch, n_embd=n_embd, n_layer=len(descs), n_vocab=n_vocab, n_ctx=n_ctx, norm_eps=norm_eps)
+        self.descs = descs
+        c = HParamsC(arch=ARCH[arch], n_embd=n_embd, n_layer=len(descs), n_vocab=n_vocab, n_ctx=n_ctx, norm_eps=norm_eps)
+        o = LayersOptsC(compute, logit_scale, norm_offset, max_batch)
+        arr = (LayerDescC * len(descs))(*[LayerDescC(**d) for d in descs])
+        self.h = self.L.pi_model_create_layers(C.byref(c), C.byref(o), arr, len(descs))
+        if not self.h:
+            raise pl.PiError("pi_model_create_layers: " + self.L.pi_last_error().decode())
+        self._keep, self.n_seq = [], 0
+
+    def release_host(self):
+        """Everything has been copied to the device: the host arrays may go."""
+        self._keep = []
+
+    def get_streams(self):
+        """The residual stream behind every layer for the last pass of a step, [n_layer][n_tokens][n_embd] (capture enabled)."""
+        n = self.L.pi_model_get_streams(self.h, None)
+        if n < 0:
+            check(n, "pi_model_get_streams")
+        out = np.empty((self.hp.n_layer, n, self.hp.n_embd), np.float32)
+        check(min(self.L.pi_model_get_streams(self.h, out.ctypes.data_as(C.c_void_p)), 0), "pi_model_get_streams")
+        return out
