@@ -298,8 +298,134 @@ def bench_batched(args):
     print(json.dumps(out), flush=True)
 
 
+# shapes of --design lerasun: layers like those of a real model of that width, and the existing model of equal width they run beside
+DESIGN_SHAPES = {
+    2048: dict(heads=16, dim=128, rot=64, vdim=128, rank=512, experts=64, top=6, groups=8, keep=4, ff=1408, layers=8,
+               beside=("llama-7b", dict(n_embd=2048, n_head=16, n_head_kv=16, n_ff=5632, n_rank=512))),
+    4096: dict(heads=32, dim=128, rot=64, vdim=128, rank=512, experts=64, top=6, groups=8, keep=4, ff=1408, layers=8, beside=("llama-7b", {})),
+    5120: dict(heads=128, dim=128, rot=64, vdim=128, rank=512, experts=160, top=6, groups=8, keep=3, ff=1536, layers=4, beside=("llama-13b", {})),
+}
+
+
+def build_lerasun_on_device(width, sh, n_ctx, keep):
+    """Random-init weights of a Lerasun shape generated in HBM; every second layer reads the cells of the one before it."""
+    from powerinfer_amd import lib as pl
+    from powerinfer_amd.lerasun import NORM_OFFSET
+    from powerinfer_amd.model import LayerModel
+    L = pl.init()
+    H, V = sh["heads"], 32000
+    descs = [dict(mixer=pl.MIXER_LATENT, n_head=H, dim=sh["dim"], rot_dim=sh["rot"], vdim=sh["vdim"], kv_rank=sh["rank"], kv_from=i - 1 if i % 2 else -1,
+                  scale=(sh["dim"] + sh["rot"]) ** -0.5, rot_base=10000.0, ffn=pl.FFN_MOE, n_expert=sh["experts"], n_top=sh["top"], n_group=sh["groups"],
+                  n_group_keep=sh["keep"], expert_ff=sh["ff"]) for i in range(sh["layers"])]
+    m = LayerModel("lerasun", descs, n_embd=width, n_vocab=V, n_ctx=n_ctx, norm_eps=1e-6, norm_offset=NORM_OFFSET)
+    seed = [7]
+
+    def put(layer, kind, rows, cols):
+        seed[0] += 1
+        buf = pl.DevBuf(rows * cols * 2)
+        pl.check(L.pi_fill_normal_bf16(buf.ptr, rows * cols, seed[0], 0.02, None), "fill")
+        m.set_tensor_device(layer, kind, buf.ptr, pl.BF16, cols, rows)
+        keep.append(buf)
+
+    zero = np.zeros(width, np.float32)
+    put(-1, "tok_embd", V, width)
+    put(-1, "output", V, width)
+    m.set_tensor(-1, "embd_norm", zero)
+    m.set_tensor(-1, "output_norm", zero)
+    for i, d in enumerate(descs):
+        m.set_tensor(i, "attn_norm", zero)
+        m.set_tensor(i, "ffn_norm", zero)
+        put(i, "mix_q", H * (sh["dim"] + sh["rot"]), width)
+        if d["kv_from"] < 0:
+            put(i, "mix_dkv", sh["rank"] + sh["rot"], width)
+            m.set_tensor(i, "mix_dkv_norm", np.ones(sh["rank"], np.float32))
+        put(i, "mix_uk", H * sh["dim"], sh["rank"])
+        put(i, "mix_uv", H * sh["vdim"], sh["rank"])
+        m.set_tensor(i, "mix_sink", np.zeros(H, np.float32))
+        put(i, "wo", width, H * sh["vdim"])
+        put(i, "router", sh["experts"], width)
+        m.set_tensor(i, "router_bias", np.zeros(sh["experts"], np.float32))
+        put(i, "expert_up", sh["experts"] * sh["ff"], width)
+        put(i, "expert_down", sh["experts"] * width, sh["ff"])
+    pl.sync()
+    m.finalize()
+    return m
+
+
+def time_prefill_and_decode(m, n_prompt, steps, warmup):
+    """(prompt seconds, seconds per decoded token) of one sequence: the prompt through Model.decode (second pass timed), then the greedy loop."""
+    from powerinfer_amd import lib as pl
+    toks = np.random.default_rng(3).integers(0, m.hp.n_vocab, n_prompt).astype(np.int32)
+    m.decode(toks, 0, want_logits=False)
+    m.kv_clear()
+    pl.sync()
+    t0 = time.perf_counter()
+    m.decode(toks, 0, want_logits=False)
+    pl.sync()
+    t1 = time.perf_counter()
+    m.generate(max(warmup, 1))
+    pl.sync()
+    t2 = time.perf_counter()
+    m.generate(steps)
+    pl.sync()
+    return t1 - t0, (time.perf_counter() - t2) / steps
+
+
+def time_lockstep(m, n_seq, n_prompt, steps, warmup):
+    from powerinfer_amd import lib as pl
+    m.batch_init(n_seq)
+    toks = np.random.default_rng(5).integers(0, m.hp.n_vocab, (n_prompt, n_seq)).astype(np.int32)
+    for p in range(n_prompt):
+        m.batch_decode(toks[p], np.full(n_seq, p, np.int32), want_logits=False)
+    m.batch_generate(max(warmup, 1))
+    pl.sync()
+    t0 = time.perf_counter()
+    m.batch_generate(steps)
+    pl.sync()
+    return (time.perf_counter() - t0) / steps
+
+
+def bench_design(args):
+    """Prefill and decode of the Lerasun design at sizes like a real model's, beside the sparse LLaMA engine at equal width and depth."""
+    from powerinfer_amd import lib as pl, synth
+    pl.init()
+    n_prompt, steps, lock_prompt = (2048 if args.prompt == 64 else args.prompt), min(args.steps, 128), 128
+    n_ctx = n_prompt + steps + args.warmup + 8
+    rows = []
+    for width in ([args.design_width] if args.design_width else sorted(DESIGN_SHAPES)):
+        sh = DESIGN_SHAPES[width]
+        row = {"width": width, "n_layer": sh["layers"], **{k: v for k, v in sh.items() if k not in ("beside", "layers")}}
+        for who in ("lerasun", "beside"):
+            if args.design_only and who != args.design_only:
+                continue
+            keep = []
+            if who == "lerasun":
+                m = build_lerasun_on_device(width, sh, n_ctx, keep)
+            else:
+                name, over = sh["beside"]
+                hp = synth.hparams(name, n_layer=sh["layers"], n_ctx=n_ctx, seed=1, **over)
+                m = build_synthetic_on_device(hp, keep)
+            pre, dec = time_prefill_and_decode(m, n_prompt, steps, args.warmup)
+            lock = time_lockstep(m, 16, lock_prompt, steps, args.warmup)
+            row[who] = {"prefill_tok_per_s": round(n_prompt / pre, 1), "prefill_ms": round(pre * 1e3, 3), "decode_ms_per_token": round(dec * 1e3, 4),
+                        "decode_tok_per_s": round(1 / dec, 1), "lockstep16_ms_per_step": round(lock * 1e3, 4), "lockstep16_tok_per_s": round(16 / lock, 1)}
+            m.close()
+            for b in keep:
+                b.free()
+            print(f"# width {width} {who}: {row[who]}", file=sys.stderr, flush=True)
+        rows.append(row)
+    best = rows[-1].get("lerasun") or rows[-1].get("beside")
+    print(json.dumps({"metric": "decode tok/s, batch 1, Lerasun layers (bf16)", "value": best["decode_tok_per_s"], "unit": "tokens/s", "n_gpus": 1, "steps": steps,
+                      "warmup": args.warmup, "ms_per_step": best["decode_ms_per_token"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16",
+                      "data": "synthetic", "config": {"model": "lerasun", "prompt_tokens": n_prompt, "lockstep_prompt_tokens": lock_prompt, "device": pl.device_name()},
+                      "sizes": rows}), flush=True)
+
+
 def main():
     ap = argparse.ArgumentParser()
+    ap.add_argument("--design", choices=["lerasun"], default=None, help="instead of the default workload: prefill and decode of this design beside the closest existing model")
+    ap.add_argument("--design-width", type=int, default=None, choices=sorted(DESIGN_SHAPES), help="one size of --design only")
+    ap.add_argument("--design-only", choices=["lerasun", "beside"], default=None, help="one side of --design only")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=256)
     ap.add_argument("--warmup", type=int, default=8)
@@ -330,6 +456,8 @@ def main():
         sys.exit("bench.py: this build runs the token loop on ONE GPU; --gpus must be 1 "
                  "(more GPUs would split the FFN by neuron and attention by head, one [n_embd] exchange per layer)")
 
+    if args.design:
+        return bench_design(args)
     from powerinfer_amd import lib as pl, synth
     if args.pmc_probe:
         hp = synth.hparams("llama-7b", n_layer=4, n_ctx=64, seed=1)

@@ -49,6 +49,7 @@ PI_API int          pi_sync(void);
 /* deterministic N(0, std^2) fill rounded to fp16 (synthetic weights generated in HBM); row_bias, if
  * not NULL, holds one fp32 per row of `cols` elements that is added before rounding */
 PI_API int          pi_fill_normal_f16(void * dptr, size_t n, uint64_t seed, float std, const float * row_bias, int cols, pi_stream_t stream);
+PI_API int          pi_fill_normal_bf16(void * dptr, size_t n, uint64_t seed, float std, pi_stream_t stream);       /* the same values rounded to bf16 */
 /* the same values (rounded to fp16 first) quantised to Q4_0 blocks of 32 as quantize_row_q4_0_reference does
  * (ggml-quants.c:428-463); n_weights % 32 == 0, dptr receives n_weights / 32 * 18 bytes */
 PI_API int          pi_fill_normal_q4_0(void * dptr, size_t n_weights, uint64_t seed, float std, pi_stream_t stream);
@@ -292,6 +293,8 @@ PI_API int pi_k_sparse_axpy_dense(const void * down_t_f16, int cols, int ff, con
 PI_API int pi_k_norm_round_f16(const float * x, int T, int cols, const pi_norm * norm, void * out_f16, void * out_plain_f16, pi_stream_t stream);
 PI_API int pi_k_gemm_f16(const void * W_f16, int rows, int cols, const void * xn_f16, int T, int epilogue,
                          const float * add1, const float * add2, float * y, void * y_f16, pi_stream_t stream);
+PI_API int pi_k_gemm_bf16(const void * W_bf16, int rows, int cols, const void * xn_bf16, int T, int epilogue,
+                          const float * add1, const float * add2, float * y, void * y_bf16, pi_stream_t stream);      /* bf16 weights and activations */
 PI_API int pi_k_batch_predictor_fc2(const void * fc2_f16, int ff, int r, const void * hidden_f16, int T, float threshold, float * logits,
                                     pi_workspace * ws, pi_stream_t stream);
 /* the union list and count alone, from the flags pi_k_batch_predictor_fc2 left in the workspace */
@@ -315,6 +318,8 @@ PI_API int pi_k_batch_sparse_ffn(const float * logits, int T, int ff, float thre
 PI_API int pi_k_norm_round_f16_ol(const float * x, int T, int cols, const pi_norm * norm, void * out_ol, void * out_plain_ol, pi_stream_t stream);
 PI_API int pi_k_gemm_f16_ol(const void * W_f16, int rows, int cols, const void * xn_ol, int T, int epilogue,
                             const float * add1, const float * add2, float * y, void * y_ol, pi_stream_t stream);
+PI_API int pi_k_gemm_bf16_ol(const void * W_bf16, int rows, int cols, const void * xn_ol, int T, int epilogue,
+                             const float * add1, const float * add2, float * y, void * y_ol, pi_stream_t stream);      /* bf16 weights and activations */
 PI_API int pi_k_batch_predictor_fc2_ol(const void * fc2_f16, int ff, int r, const void * hidden_ol, int T, float threshold, float * logits,
                                        pi_workspace * ws, pi_stream_t stream);
 PI_API int pi_k_batch_sparse_ffn_ol(const float * logits, int T, int ff, float threshold,
@@ -333,6 +338,8 @@ PI_API int pi_k_batch_sparse_ffn_ol(const float * logits, int T, int ff, float t
  * contiguous). */
 PI_API int pi_k_gemm_tile_f16(const void * W_f16, int rows, int cols, const void * xn_f16, int T, int epilogue,
                               const float * add1, const float * add2, float * y, void * y_f16, int tile, pi_stream_t stream);
+PI_API int pi_k_gemm_tile_bf16(const void * W_bf16, int rows, int cols, const void * xn_bf16, int T, int epilogue,
+                               const float * add1, const float * add2, float * y, void * y_bf16, int tile, pi_stream_t stream);
 /* Steps of up to 16 tokens on Q4_0 weights with the CPU path's arithmetic (ggml_vec_dot_q4_0_q8_0, ggml-quants.c:2512-2650; in the reference's
  * CUDA backend the mul_mat_q tiles and dequantize_mul_mat_batch_sparse, ggml-cuda.cu:3524-4308, 4757-4830): one integer matrix-core
  * instruction per pair of a Q4_0 weight block and a Q8_0 activation block gives the exact int32 sum, scaled by d_w * d_x in fp32.
@@ -430,6 +437,8 @@ PI_API pi_gemm_lib * pi_gemm_lib_create(size_t workspace_bytes);
 PI_API int           pi_gemm_lib_destroy(pi_gemm_lib * g);
 PI_API int pi_gemm_lib_f16(pi_gemm_lib * g, const void * W_f16, int rows, int cols, const void * xn_f16, int T, int epilogue,
                            const float * add1, const float * add2, float * y, void * y_f16, pi_stream_t stream);
+PI_API int pi_gemm_lib_bf16(pi_gemm_lib * g, const void * W_bf16, int rows, int cols, const void * xn_bf16, int T, int epilogue,
+                            const float * add1, const float * add2, float * y, void * y_bf16, pi_stream_t stream);
 
 /* The two sparse operators of a step AS OPERATORS, for a host that runs the predictor itself and hands over its output idx [T][ff]
  * (the reference's mul_mat_batch_sparse and axpy at batch size > 1, ggml-cuda.cu:6994-7034, 8787-8814): T <= 16, F16 rows, cols % 256 == 0.
@@ -580,8 +589,11 @@ typedef struct pi_group_gemm {
     void * y; size_t y_gs; int32_t ldy, y_f32, relu2;
     float alpha;
     const int32_t * off, * gather; int32_t gather_div;
+    const int32_t * tiles, * n_tiles; int32_t max_tiles;      /* pi_k_group_gemm_tile with off: pi_k_moe_sort's list and an upper bound of its length */
 } pi_group_gemm;
 PI_API int pi_k_group_gemm(int type, const pi_group_gemm * g, pi_stream_t stream);
+/* the same for many tokens, bf16, both operands tiled through LDS (cols % 64 == 0); tile_n 64 or 128 tokens per tile, as given to pi_k_moe_sort */
+PI_API int pi_k_group_gemm_tile(const pi_group_gemm * g, int tile_n, pi_stream_t stream);
 /* (cos, sin)[t][i] of the angles pos[t] * base^(-2i / dims), i < dims / 2 */
 PI_API int pi_k_rope_angles(const int32_t * pos, int T, int dims, double base, void * cs_float2, pi_stream_t stream);
 /* Behind the joint projection of a latent-attention layer, z [T][ldz] = per head [dim | rot_dim], then (own cells) [kv_rank | rot_dim]:
@@ -611,11 +623,14 @@ PI_API int pi_k_latent_shift(int type, void * cache, int n_cells, int kd, int ra
 /* expert choice of T tokens from router logits z [T][n_expert] (see PI_FFN_MOE): ids, weights [T][n_top] by falling choice score */
 PI_API int pi_k_route(const float * z, int T, int n_expert, int n_top, int n_group, int n_keep, const float * bias, int32_t * ids, float * weights,
                       pi_stream_t stream);
-/* pairs (token, choice) in expert order, tokens ascending: off [n_expert + 1], perm[place] = pair, inv[pair] = place */
-PI_API int pi_k_moe_sort(const int32_t * ids, int n_pairs, int n_expert, int32_t * off, int32_t * perm, int32_t * inv, pi_stream_t stream);
-/* out[t] = x[t] + (mix[t] + sum over k of weights[t][k] * y[inv[t][k]]); weights == NULL: out = x + mix.  keep (optional) receives a copy */
-PI_API int pi_k_moe_combine(const float * x, const float * mix, const float * y, const int32_t * inv, const float * weights, int n_top, int T, int cols,
-                            float * out, float * keep, pi_stream_t stream);
+/* pairs (token, choice) in expert order: off [n_expert + 1], perm[place] = pair, inv[pair] = place.  tiles (optional): {expert, first
+ * place} of every group of up to tile_n pairs of one expert; *n_tiles of them, at most n_pairs / tile_n + n_expert */
+PI_API int pi_k_moe_sort(const int32_t * ids, int n_pairs, int n_expert, int32_t * off, int32_t * perm, int32_t * inv, int tile_n, int32_t * tiles,
+                         int32_t * n_tiles, pi_stream_t stream);
+/* out[t] = x[t] + (mix[t] + sum over k of weights[t][k] * y[inv[t][k]]), y of the given type; weights == NULL: out = x + mix.  keep
+ * (optional) receives a copy */
+PI_API int pi_k_moe_combine(int type, const float * x, const float * mix, const void * y, const int32_t * inv, const float * weights, int n_top, int T,
+                            int cols, float * out, float * keep, pi_stream_t stream);
 /* BF16 matrices: out [rows][ld] = in [rows][cols] padded with zeros; out [n_mat][cols][ld] = each in [rows][cols] transposed, padded with zeros */
 PI_API int pi_k_pad_cols_bf16(const void * in, int64_t rows, int cols, void * out, int ld, pi_stream_t stream);
 PI_API int pi_k_transpose_pad_bf16(const void * in, int n_mat, int rows, int cols, void * out, int ld, pi_stream_t stream);

@@ -52,15 +52,16 @@ struct LayerState {
     const float *embd_norm = nullptr, *out_norm = nullptr;
     const void *embed = nullptr, *head = nullptr;
     KvCells kv;
+    bool auto_pool = false;                            // sized by the engine (decode, batch_init), not by the caller
     int32_t * lists = nullptr;                         // device [32][kv.n]: a sequence's cells in position order
     std::vector<int32_t> list_cells[32], list_pos[32]; // the same on the host
     int32_t * d_delta = nullptr;
     // step buffers for `cap` tokens (one allocation)
     int cap = 0;
     unsigned char * arena = nullptr;
-    float *x = nullptr, *x2 = nullptr, *z = nullptr, *mix = nullptr, *rl = nullptr, *wts = nullptr, *y_exp = nullptr;
-    void *h_a = nullptr, *h_b = nullptr, *q_un = nullptr, *q_lat = nullptr, *o_lat = nullptr, *att = nullptr, *act = nullptr;
-    int32_t *ids = nullptr, *perm = nullptr, *inv = nullptr, *off = nullptr;
+    float *x = nullptr, *x2 = nullptr, *z = nullptr, *mix = nullptr, *rl = nullptr, *wts = nullptr;
+    void *h_a = nullptr, *h_b = nullptr, *q_un = nullptr, *q_lat = nullptr, *o_lat = nullptr, *att = nullptr, *act = nullptr, *y_exp = nullptr;
+    int32_t *ids = nullptr, *perm = nullptr, *inv = nullptr, *off = nullptr, *tiles = nullptr, *n_tiles = nullptr;
     std::vector<float *> cs;                           // per rotation [cap][dims / 2] (cos, sin)
     float * scratch = nullptr;                         // partial sums of a split attention
     float * logits = nullptr; void * h_head = nullptr; int32_t * d_next = nullptr;
@@ -117,11 +118,11 @@ int padded(pi_model * m, Tensor & t, int ld, const void ** out) {
     return PI_OK;
 }
 
-// the weights of one of the model's norms with the offset of the design added
-int norm_weights(pi_model * m, const Tensor & t, float offset, const float ** out) {
+// the weights of one of the model's norms with the offset of the design added, times a factor (the logit scale rides on the last norm)
+int norm_weights(pi_model * m, const Tensor & t, float offset, float factor, const float ** out) {
     std::vector<float> w((size_t)t.ne0);
     PI_TRY(pi_memcpy_d2h(w.data(), t.dev, sizeof(float) * w.size()));
-    for (float & v : w) v += offset;
+    for (float & v : w) v = (v + offset) * factor;
     float * p = m->alloc<float>(w.size());
     if (!p) return PI_E_HIP;
     PI_TRY(pi_memcpy_h2d(p, w.data(), sizeof(float) * w.size()));
@@ -135,7 +136,7 @@ int layer_weights(pi_model * m, int il) {
     const pi_layer_desc & d = L.d;
     const int D = m->hp.n_embd;
     PI_TRY(want_tensor(m->L(il, PI_T_ATTN_NORM), PI_TYPE_F32, D, 1, "attn_norm"));
-    PI_TRY(norm_weights(m, m->L(il, PI_T_ATTN_NORM), s->opts.norm_offset, &L.norm_a));
+    PI_TRY(norm_weights(m, m->L(il, PI_T_ATTN_NORM), s->opts.norm_offset, 1.0f, &L.norm_a));
     Tensor & q = m->L(il, PI_T_MIX_Q); Tensor & dkv = m->L(il, PI_T_MIX_DKV);
     PI_TRY(want_tensor(q, PI_TYPE_BF16, D, L.nq, "mix_q"));
     if (L.own_kv) {
@@ -169,7 +170,7 @@ int layer_weights(pi_model * m, int il) {
     PI_TRY(padded(m, m->L(il, PI_T_WO), L.hv_ld, &L.wo));
     if (d.ffn == PI_FFN_NONE) return PI_OK;
     PI_TRY(want_tensor(m->L(il, PI_T_FFN_NORM), PI_TYPE_F32, D, 1, "ffn_norm"));
-    PI_TRY(norm_weights(m, m->L(il, PI_T_FFN_NORM), s->opts.norm_offset, &L.norm_b));
+    PI_TRY(norm_weights(m, m->L(il, PI_T_FFN_NORM), s->opts.norm_offset, 1.0f, &L.norm_b));
     PI_TRY(want_tensor(m->L(il, PI_T_ROUTER), PI_TYPE_BF16, D, d.n_expert, "router"));
     PI_TRY(want_tensor(m->L(il, PI_T_ROUTER_BIAS), PI_TYPE_F32, d.n_expert, 1, "router_bias"));
     PI_TRY(want_tensor(m->L(il, PI_T_EXPERT_UP), PI_TYPE_BF16, D, (int64_t)d.n_expert * d.expert_ff, "expert_up"));
@@ -212,7 +213,8 @@ int ensure_capacity(pi_model * m, int T) {
         carve(s->h_a, n * s->d_ld * es); carve(s->h_b, n * s->d_ld * es);
         carve(s->q_un, n * qu * es); carve(s->q_lat, n * ql * es); carve(s->o_lat, n * ol * es); carve(s->att, n * at * es);
         carve(s->rl, n * E * 4); carve(s->wts, n * top * 4); carve(s->ids, n * top * 4); carve(s->perm, n * top * 4); carve(s->inv, n * top * 4);
-        carve(s->off, (E + 1) * 4); carve(s->act, n * ff * es); carve(s->y_exp, n * top * D * 4);
+        carve(s->off, (E + 1) * 4); carve(s->act, n * ff * es); carve(s->y_exp, n * top * D * es);
+        carve(s->tiles, (n * top / 64 + E + 1) * 8); carve(s->n_tiles, 4);
         s->cs.resize(s->rots.size());
         for (size_t r = 0; r < s->rots.size(); ++r) carve(s->cs[r], n * s->rots[r].dims * 4);
     };
@@ -243,10 +245,31 @@ int ensure_inputs(pi_model * m, size_t n) {
 }
 
 // ---- one pass over the layers ----------------------------------------------------------------------------------------------------
-int dense(LayerState * s, const void * W, int rows, int cols, const void * x, int ldx, int T, float * y, int ldy, float alpha, hipStream_t st) {
-    pi_group_gemm g{};
-    g.W = W; g.rows = rows; g.cols = cols; g.ldw = cols; g.n_group = 1; g.x = x; g.ldx = ldx; g.T = T; g.y = y; g.ldy = ldy; g.y_f32 = 1; g.alpha = alpha;
-    return pi_k_group_gemm(s->opts.compute, &g, st);
+// y [T][rows] = W x, x rows of `cols` values.  bf16: the mat-muls the other models run (steps of up to 16 tokens, LDS tiles, and
+// hipBLASLt plans for large products)
+int dense(pi_model * m, const void * W, int rows, int cols, const void * x, int T, float * y) {
+    LayerState * s = m->lay;
+    hipStream_t st = m->stream;
+    if (!bf16_mode(s)) {
+        pi_group_gemm g{};
+        g.W = W; g.rows = rows; g.cols = cols; g.ldw = cols; g.n_group = 1; g.x = x; g.ldx = cols; g.T = T; g.y = y; g.ldy = rows; g.y_f32 = 1; g.alpha = 1.0f;
+        return pi_k_group_gemm(s->opts.compute, &g, st);
+    }
+    if (T <= 16) return pi_k_gemm_bf16(W, rows, cols, x, T, PI_EPI_NONE, nullptr, nullptr, y, nullptr, st);
+    const char * own = getenv("PI_PREFILL_GEMM");
+    if (T >= 256 && rows >= 1024 && cols >= 1024 && !(own && !strcmp(own, "own"))) {
+        if (!m->gemm_lib) {
+            m->gemm_lib = pi_gemm_lib_create((size_t)64 << 20);
+            if (!m->gemm_lib) return PI_E_HIP;
+        }
+        const int rc = pi_gemm_lib_bf16(m->gemm_lib, W, rows, cols, x, T, PI_EPI_NONE, nullptr, nullptr, y, nullptr, st);
+        if (rc != PI_E_UNSUPPORTED) return rc;
+    }
+    return pi_k_gemm_tile_bf16(W, rows, cols, x, T, PI_EPI_NONE, nullptr, nullptr, y, nullptr, 0, st);
+}
+
+int grouped(LayerState * s, const pi_group_gemm & g, int tile_n, hipStream_t st) {
+    return bf16_mode(s) && g.T > 16 ? pi_k_group_gemm_tile(&g, tile_n, st) : pi_k_group_gemm(s->opts.compute, &g, st);
 }
 
 int mix_latent(pi_model * m, Layer & L, const Step & in) {
@@ -255,7 +278,7 @@ int mix_latent(pi_model * m, Layer & L, const Step & in) {
     const int type = s->opts.compute, T = in.T;
     hipStream_t st = m->stream;
     Layer & src = L.own_kv ? L : s->layers[d.kv_from];
-    PI_TRY(dense(s, L.w_z, L.z_rows, s->d_ld, s->h_a, s->d_ld, T, s->z, L.z_rows, 1.0f, st));
+    PI_TRY(dense(m, L.w_z, L.z_rows, s->d_ld, s->h_a, T, s->z));
     pi_latent_prep p{};
     p.z = s->z; p.ldz = L.z_rows; p.T = T; p.n_head = d.n_head; p.dim = d.dim; p.dim_ld = L.dim_ld; p.rot_dim = d.rot_dim; p.kv_rank = d.kv_rank;
     p.rank_ld = L.rank_ld; p.kd = L.kd; p.cs = s->cs[L.rot]; p.norm_w = L.dkv_norm; p.eps = m->hp.norm_eps; p.q_un = s->q_un; p.q_lat = s->q_lat;
@@ -264,7 +287,7 @@ int mix_latent(pi_model * m, Layer & L, const Step & in) {
     pi_group_gemm g{};                              // each head's query in latent coordinates
     g.W = L.uk_t; g.w_gs = (size_t)d.kv_rank * L.dim_ld; g.rows = d.kv_rank; g.cols = L.dim_ld; g.ldw = L.dim_ld; g.n_group = d.n_head; g.alpha = 1.0f;
     g.x = s->q_un; g.x_gs = L.dim_ld; g.ldx = d.n_head * L.dim_ld; g.T = T; g.y = s->q_lat; g.y_gs = L.kd; g.ldy = d.n_head * L.kd;
-    PI_TRY(pi_k_group_gemm(type, &g, st));
+    PI_TRY(grouped(s, g, T > 64 ? 128 : 64, st));
     pi_latent_attn a{};
     a.q_lat = s->q_lat; a.cache = src.cache; a.lists = s->lists; a.list_ld = s->kv.n; a.work = bf16_mode(s) ? in.work[L.hc].items : in.seq; a.n_vis = in.n_vis;
     a.n_work = in.work[L.hc].n; a.T = T; a.n_head = d.n_head; a.kv_rank = d.kv_rank; a.rank_ld = L.rank_ld; a.kd = L.kd; a.n_parts = in.work[L.hc].parts; a.scale = d.scale;
@@ -273,26 +296,28 @@ int mix_latent(pi_model * m, Layer & L, const Step & in) {
     pi_group_gemm v{};                              // each head's value from its weighted latent
     v.W = L.uv; v.w_gs = (size_t)d.vdim * L.rank_ld; v.rows = d.vdim; v.cols = L.rank_ld; v.ldw = L.rank_ld; v.n_group = d.n_head; v.alpha = 1.0f;
     v.x = s->o_lat; v.x_gs = L.rank_ld; v.ldx = d.n_head * L.rank_ld; v.T = T; v.y = s->att; v.y_gs = d.vdim; v.ldy = L.hv_ld;
-    PI_TRY(pi_k_group_gemm(type, &v, st));
-    return dense(s, L.wo, m->hp.n_embd, L.hv_ld, s->att, L.hv_ld, T, s->mix, m->hp.n_embd, 1.0f, st);
+    PI_TRY(grouped(s, v, T > 64 ? 128 : 64, st));
+    return dense(m, L.wo, m->hp.n_embd, L.hv_ld, s->att, T, s->mix);
 }
 
 int ffn_moe(pi_model * m, Layer & L, const Step & in) {
     LayerState * s = m->lay;
     const pi_layer_desc & d = L.d;
-    const int type = s->opts.compute, T = in.T, D = m->hp.n_embd;
+    const int T = in.T, D = m->hp.n_embd;
     hipStream_t st = m->stream;
-    PI_TRY(dense(s, L.router, d.n_expert, s->d_ld, s->h_b, s->d_ld, T, s->rl, d.n_expert, 1.0f, st));
+    PI_TRY(dense(m, L.router, d.n_expert, s->d_ld, s->h_b, T, s->rl));
     PI_TRY(pi_k_route(s->rl, T, d.n_expert, d.n_top, d.n_group, d.n_group_keep, L.bias, s->ids, s->wts, st));
-    PI_TRY(pi_k_moe_sort(s->ids, T * d.n_top, d.n_expert, s->off, s->perm, s->inv, st));
+    const int tile_n = (long long)T * d.n_top > 96LL * d.n_expert ? 128 : 64;       // tokens per tile, by the tokens an expert has on average
+    PI_TRY(pi_k_moe_sort(s->ids, T * d.n_top, d.n_expert, s->off, s->perm, s->inv, tile_n, s->tiles, s->n_tiles, st));
     pi_group_gemm g{};
     g.W = L.up; g.w_gs = (size_t)d.expert_ff * s->d_ld; g.rows = d.expert_ff; g.cols = s->d_ld; g.ldw = s->d_ld; g.n_group = d.n_expert; g.alpha = 1.0f; g.relu2 = 1;
     g.x = s->h_b; g.ldx = s->d_ld; g.T = T; g.y = s->act; g.ldy = L.ff_ld; g.off = s->off; g.gather = s->perm; g.gather_div = d.n_top;
-    PI_TRY(pi_k_group_gemm(type, &g, st));
+    g.tiles = s->tiles; g.n_tiles = s->n_tiles; g.max_tiles = T * d.n_top / tile_n + d.n_expert;
+    PI_TRY(grouped(s, g, tile_n, st));
     pi_group_gemm w{};
     w.W = L.down; w.w_gs = (size_t)D * L.ff_ld; w.rows = D; w.cols = L.ff_ld; w.ldw = L.ff_ld; w.n_group = d.n_expert; w.alpha = 1.0f;
-    w.x = s->act; w.ldx = L.ff_ld; w.T = T; w.y = s->y_exp; w.ldy = D; w.y_f32 = 1; w.off = s->off;
-    return pi_k_group_gemm(type, &w, st);
+    w.x = s->act; w.ldx = L.ff_ld; w.T = T; w.y = s->y_exp; w.ldy = D; w.off = s->off; w.tiles = s->tiles; w.n_tiles = s->n_tiles; w.max_tiles = g.max_tiles;
+    return grouped(s, w, tile_n, st);
 }
 
 int pass_layers(pi_model * m, const Step & in) {
@@ -307,7 +332,7 @@ int pass_layers(pi_model * m, const Step & in) {
         PI_TRY(pi_k_norm_pair(type, s->x, nullptr, T, D, m->hp.norm_eps, L.norm_a, s->h_a, moe ? L.norm_b : nullptr, moe ? s->h_b : nullptr, s->d_ld, 0, st));
         PI_TRY(mix_latent(m, L, in));
         if (moe) PI_TRY(ffn_moe(m, L, in));
-        PI_TRY(pi_k_moe_combine(s->x, s->mix, s->y_exp, s->inv, moe ? s->wts : nullptr, moe ? L.d.n_top : 0, T, D, s->x2,
+        PI_TRY(pi_k_moe_combine(type, s->x, s->mix, s->y_exp, s->inv, moe ? s->wts : nullptr, moe ? L.d.n_top : 0, T, D, s->x2,
                                 s->streams_T ? s->streams + il * (size_t)s->streams_T * D : nullptr, st));
         std::swap(s->x, s->x2);
     }
@@ -319,7 +344,7 @@ int pass_head(pi_model * m, const int32_t * rows, int n) {
     LayerState * s = m->lay;
     const int D = m->hp.n_embd;
     PI_TRY(pi_k_norm_pair(s->opts.compute, s->x, rows, n, D, m->hp.norm_eps, s->out_norm, s->h_head, nullptr, nullptr, s->d_ld, 0, m->stream));
-    return dense(s, s->head, m->hp.n_vocab, s->d_ld, s->h_head, s->d_ld, n, s->logits, m->hp.n_vocab, s->opts.logit_scale, m->stream);
+    return dense(m, s->head, m->hp.n_vocab, s->d_ld, s->h_head, n, s->logits);
 }
 
 int head_buffers(pi_model * m) {
@@ -413,23 +438,38 @@ namespace pi {
 
 KvCells * layers_cells(pi_model * m) { return m->lay->kv.n ? &m->lay->kv : nullptr; }
 
-int layers_cells_init(pi_model * m, int n_cells) {
+// caches and lists for n_cells cells; what earlier cells hold is kept
+static int resize_pool(pi_model * m, int n_cells) {
     LayerState * s = m->lay;
-    if (s->kv.n) return fail(PI_E_STATE, "pi_model_kv_cells_init: already initialised");
-    if (n_cells < 1) return fail(PI_E_ARG, "pi_model_kv_cells_init: at least one cell");
+    PI_HIP_TRY(hipStreamSynchronize(m->stream));
+    drop_graph(s);
+    auto give_back = [&](void * p) { for (auto & o : m->owned) if (p && o == p) { pi_free(o); o = nullptr; } };
     for (Layer & L : s->layers) {
         if (!L.own_kv) continue;
-        L.cache = m->alloc<unsigned char>((size_t)n_cells * L.kd * s->es);
-        if (!L.cache) return PI_E_HIP;
-        PI_TRY(pi_memset(L.cache, 0, (size_t)n_cells * L.kd * s->es));
+        const size_t row = (size_t)L.kd * s->es;
+        unsigned char * c = m->alloc<unsigned char>(n_cells * row);
+        if (!c) return PI_E_HIP;
+        PI_TRY(pi_memset(c, 0, n_cells * row));
+        if (L.cache) PI_TRY(pi_memcpy_d2d(c, L.cache, s->kv.n * row));
+        PI_TRY(pi_sync());
+        give_back(L.cache);
+        L.cache = c;
     }
+    give_back(s->lists); give_back(s->d_delta);
     s->lists = m->alloc<int32_t>((size_t)32 * n_cells);
     s->d_delta = m->alloc<int32_t>(n_cells);
     if (!s->lists || !s->d_delta) return PI_E_HIP;
     PI_TRY(pi_memset(s->lists, 0, sizeof(int32_t) * 32 * (size_t)n_cells));
     PI_TRY(pi_sync());
-    s->kv.init(n_cells);
+    if (s->kv.n) s->kv.grow(n_cells); else s->kv.init(n_cells);
     return PI_OK;
+}
+
+int layers_cells_init(pi_model * m, int n_cells) {
+    if (!m->finalized) return fail(PI_E_STATE, "pi_model_kv_cells_init: model not finalized");
+    if (m->lay->kv.n) return fail(PI_E_STATE, "pi_model_kv_cells_init: already initialised");
+    if (n_cells < 1) return fail(PI_E_ARG, "pi_model_kv_cells_init: at least one cell");
+    return resize_pool(m, n_cells);
 }
 
 int layers_finalize(pi_model * m) {
@@ -445,8 +485,8 @@ int layers_finalize(pi_model * m) {
     PI_TRY(want_tensor(m->embd_norm, PI_TYPE_F32, D, 1, "embd_norm"));
     s->embed = m->glob[PI_T_TOK_EMBD].dev;
     PI_TRY(padded(m, m->glob[PI_T_OUTPUT], s->d_ld, &s->head));
-    PI_TRY(norm_weights(m, m->embd_norm, s->opts.norm_offset, &s->embd_norm));
-    PI_TRY(norm_weights(m, m->glob[PI_T_OUTPUT_NORM], s->opts.norm_offset, &s->out_norm));
+    PI_TRY(norm_weights(m, m->embd_norm, s->opts.norm_offset, 1.0f, &s->embd_norm));
+    PI_TRY(norm_weights(m, m->glob[PI_T_OUTPUT_NORM], s->opts.norm_offset, s->opts.logit_scale, &s->out_norm));
     size_t scratch = 0;
     for (size_t il = 0; il < s->layers.size(); ++il) {
         Layer & L = s->layers[il];
@@ -454,7 +494,7 @@ int layers_finalize(pi_model * m) {
         L.own_kv = d.kv_from < 0;
         L.nq = d.n_head * (d.dim + d.rot_dim);
         L.z_rows = L.nq + (L.own_kv ? d.kv_rank + d.rot_dim : 0);
-        L.dim_ld = up_to(d.dim, 32); L.rank_ld = up_to(d.kv_rank, 32); L.kd = L.rank_ld + up_to(d.rot_dim, 32);
+        L.dim_ld = up_to(d.dim, 64); L.rank_ld = up_to(d.kv_rank, 64); L.kd = L.rank_ld + up_to(d.rot_dim, 32);
         L.hv_ld = up_to(d.n_head * d.vdim, 128); L.ff_ld = d.ffn == PI_FFN_MOE ? up_to(d.expert_ff, 64) : 0;
         if (!pi_k_latent_attn_supported(s->opts.compute, L.rank_ld, L.kd)) return fail(PI_E_UNSUPPORTED, "pi_model_finalize: latent sizes outside the attention kernels (rank up to 1024)");
         size_t r = 0;
@@ -590,9 +630,11 @@ int layers_step(pi_model * m, const int32_t * tokens, const int32_t * positions,
 }
 
 static int ensure_pool(pi_model * m, int64_t n) {
-    if (m->lay->kv.n) return PI_OK;
-    if (n > INT32_MAX) return fail(PI_E_ARG, "the cache pool is too large");
-    return layers_cells_init(m, (int)n);
+    LayerState * s = m->lay;
+    if (s->kv.n && (!s->auto_pool || s->kv.n >= n)) return PI_OK;      // a pool the caller has sized stays as it is
+    if (n > INT32_MAX / 2) return fail(PI_E_ARG, "the cache pool is too large");
+    s->auto_pool = true;
+    return resize_pool(m, (int)n);
 }
 
 // tokens at n_past .. of sequence q, behind exactly n_past cells (what lies at n_past and beyond is dropped first)

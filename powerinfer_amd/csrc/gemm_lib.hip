@@ -14,7 +14,7 @@
 namespace {
 
 struct Plan {
-    int rows, cols, T;
+    int rows, cols, T, el;                // el: PI_TYPE_F16 or PI_TYPE_BF16 operands
     bool with_c;
     uint64_t last_use;
     hipblasLtMatmulDesc_t op;
@@ -23,13 +23,14 @@ struct Plan {
 };
 
 // y = relu(y) | y += add2, and the fp16 copy, in one pass over the result
-__global__ void gemm_lib_post_kernel(float * __restrict__ y, const float * __restrict__ add2, __half * __restrict__ y16, int relu, size_t n) {
+template <typename EL>
+__global__ void gemm_lib_post_kernel(float * __restrict__ y, const float * __restrict__ add2, EL * __restrict__ y16, int relu, size_t n) {
     for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (size_t)gridDim.x * blockDim.x) {
         float v = y[i];
         if (relu) v = fmaxf(v, 0.0f);
         if (add2) v = __fadd_rn(v, add2[i]);
         if (relu || add2) y[i] = v;
-        if (y16) y16[i] = __float2half_rn(v);
+        if (y16) y16[i] = (EL)v;
     }
 }
 
@@ -65,19 +66,20 @@ static void destroy_plan(Plan & p) {
 
 // A plan is used only to enqueue its product (the descriptors are read at enqueue time), so evicting one between two calls is safe.
 // Prompt remainders of every length ask for their own plans: a server would otherwise run into the cap after a few dozen prompts.
-static int make_plan(pi_gemm_lib * g, int rows, int cols, int T, bool with_c, Plan ** out) {
+static int make_plan(pi_gemm_lib * g, int el, int rows, int cols, int T, bool with_c, Plan ** out) {
+    const hipDataType dt = el == PI_TYPE_BF16 ? HIP_R_16BF : HIP_R_16F;
     for (Plan & p : g->plans)
-        if (p.rows == rows && p.cols == cols && p.T == T && p.with_c == with_c) { p.last_use = ++g->clock; *out = &p; return PI_OK; }
+        if (p.el == el && p.rows == rows && p.cols == cols && p.T == T && p.with_c == with_c) { p.last_use = ++g->clock; *out = &p; return PI_OK; }
     Plan p{};
-    p.rows = rows; p.cols = cols; p.T = T; p.with_c = with_c;
+    p.rows = rows; p.cols = cols; p.T = T; p.el = el; p.with_c = with_c;
     const auto build = [&]() -> int {
         // column-major view: D (rows x T, ld rows) = W^T-as-stored (cols x rows, ld cols) transposed  x  xn-as-stored (cols x T, ld cols)
         PI_LT_TRY(hipblasLtMatmulDescCreate(&p.op, HIPBLAS_COMPUTE_32F, HIP_R_32F));
         const hipblasOperation_t ta = HIPBLAS_OP_T, tb = HIPBLAS_OP_N;
         PI_LT_TRY(hipblasLtMatmulDescSetAttribute(p.op, HIPBLASLT_MATMUL_DESC_TRANSA, &ta, sizeof ta));
         PI_LT_TRY(hipblasLtMatmulDescSetAttribute(p.op, HIPBLASLT_MATMUL_DESC_TRANSB, &tb, sizeof tb));
-        PI_LT_TRY(hipblasLtMatrixLayoutCreate(&p.a, HIP_R_16F, cols, rows, cols));
-        PI_LT_TRY(hipblasLtMatrixLayoutCreate(&p.b, HIP_R_16F, cols, T, cols));
+        PI_LT_TRY(hipblasLtMatrixLayoutCreate(&p.a, dt, cols, rows, cols));
+        PI_LT_TRY(hipblasLtMatrixLayoutCreate(&p.b, dt, cols, T, cols));
         PI_LT_TRY(hipblasLtMatrixLayoutCreate(&p.c, HIP_R_32F, rows, T, rows));
         hipblasLtMatmulPreference_t pref;
         PI_LT_TRY(hipblasLtMatmulPreferenceCreate(&pref));
@@ -86,7 +88,7 @@ static int make_plan(pi_gemm_lib * g, int rows, int cols, int T, bool with_c, Pl
         int found = 0;
         if (hs == HIPBLAS_STATUS_SUCCESS) hs = hipblasLtMatmulAlgoGetHeuristic(g->handle, p.op, p.a, p.b, p.c, p.c, pref, 1, &p.heur, &found);
         (void)hipblasLtMatmulPreferenceDestroy(pref);
-        if (hs != HIPBLAS_STATUS_SUCCESS || found < 1) return pi::fail(PI_E_UNSUPPORTED, "pi_gemm_lib_f16: hipBLASLt offers no kernel for this shape");
+        if (hs != HIPBLAS_STATUS_SUCCESS || found < 1) return pi::fail(PI_E_UNSUPPORTED, "pi_gemm_lib: hipBLASLt offers no kernel for this shape");
         return PI_OK;
     };
     const int rc = build();
@@ -101,6 +103,30 @@ static int make_plan(pi_gemm_lib * g, int rows, int cols, int T, bool with_c, Pl
         destroy_plan(g->plans[victim]);
         g->plans[victim] = p;
         *out = &g->plans[victim];
+    }
+    return PI_OK;
+}
+
+template <typename EL>
+static int gemm_lib_run(int el, pi_gemm_lib * g, const void * W_f16, int rows, int cols, const void * xn_f16, int T, int epilogue,
+                    const float * add1, const float * add2, float * y, void * y_f16, pi_stream_t stream) {
+    if (!g || !W_f16 || !xn_f16 || !y || rows <= 0 || cols <= 0 || T <= 0) return pi::fail(PI_E_ARG, "pi_gemm_lib: bad arguments");
+    if (epilogue < PI_EPI_NONE || epilogue > PI_EPI_ADD2) return pi::fail(PI_E_ARG, "pi_gemm_lib: unknown epilogue");
+    if ((epilogue >= PI_EPI_ADD && !add1) || (epilogue == PI_EPI_ADD2 && !add2)) return pi::fail(PI_E_ARG, "pi_gemm_lib: residual operand missing");
+    const bool with_c = epilogue >= PI_EPI_ADD;
+    Plan * p = nullptr;
+    PI_TRY(make_plan(g, el, rows, cols, T, with_c, &p));
+    const float alpha = 1.0f, beta = with_c ? 1.0f : 0.0f;
+    hipStream_t st = (hipStream_t)stream;
+    PI_LT_TRY(hipblasLtMatmul(g->handle, p->op, &alpha, W_f16, p->a, xn_f16, p->b, &beta, with_c ? (const void *)add1 : (const void *)y, p->c, y, p->c,
+                              &p->heur.algo, g->ws, g->ws_bytes, st));
+    const bool relu = epilogue == PI_EPI_RELU;
+    if (relu || epilogue == PI_EPI_ADD2 || y_f16) {
+        const size_t n = (size_t)rows * T;
+        size_t blocks = (n + 255) / 256;
+        if (blocks > 4096) blocks = 4096;
+        hipLaunchKernelGGL(gemm_lib_post_kernel<EL>, dim3((unsigned)blocks), dim3(256), 0, st, y, epilogue == PI_EPI_ADD2 ? add2 : nullptr, (EL *)y_f16, relu ? 1 : 0, n);
+        return pi::check_launch("pi_gemm_lib");
     }
     return PI_OK;
 }
@@ -130,25 +156,12 @@ int pi_gemm_lib_destroy(pi_gemm_lib * g) {
 
 int pi_gemm_lib_f16(pi_gemm_lib * g, const void * W_f16, int rows, int cols, const void * xn_f16, int T, int epilogue,
                     const float * add1, const float * add2, float * y, void * y_f16, pi_stream_t stream) {
-    if (!g || !W_f16 || !xn_f16 || !y || rows <= 0 || cols <= 0 || T <= 0) return pi::fail(PI_E_ARG, "pi_gemm_lib_f16: bad arguments");
-    if (epilogue < PI_EPI_NONE || epilogue > PI_EPI_ADD2) return pi::fail(PI_E_ARG, "pi_gemm_lib_f16: unknown epilogue");
-    if ((epilogue >= PI_EPI_ADD && !add1) || (epilogue == PI_EPI_ADD2 && !add2)) return pi::fail(PI_E_ARG, "pi_gemm_lib_f16: residual operand missing");
-    const bool with_c = epilogue >= PI_EPI_ADD;
-    Plan * p = nullptr;
-    PI_TRY(make_plan(g, rows, cols, T, with_c, &p));
-    const float alpha = 1.0f, beta = with_c ? 1.0f : 0.0f;
-    hipStream_t st = (hipStream_t)stream;
-    PI_LT_TRY(hipblasLtMatmul(g->handle, p->op, &alpha, W_f16, p->a, xn_f16, p->b, &beta, with_c ? (const void *)add1 : (const void *)y, p->c, y, p->c,
-                              &p->heur.algo, g->ws, g->ws_bytes, st));
-    const bool relu = epilogue == PI_EPI_RELU;
-    if (relu || epilogue == PI_EPI_ADD2 || y_f16) {
-        const size_t n = (size_t)rows * T;
-        size_t blocks = (n + 255) / 256;
-        if (blocks > 4096) blocks = 4096;
-        hipLaunchKernelGGL(gemm_lib_post_kernel, dim3((unsigned)blocks), dim3(256), 0, st, y, epilogue == PI_EPI_ADD2 ? add2 : nullptr, (__half *)y_f16, relu ? 1 : 0, n);
-        return pi::check_launch("pi_gemm_lib_f16");
-    }
-    return PI_OK;
+    return gemm_lib_run<__half>(PI_TYPE_F16, g, W_f16, rows, cols, xn_f16, T, epilogue, add1, add2, y, y_f16, stream);
+}
+
+int pi_gemm_lib_bf16(pi_gemm_lib * g, const void * W_bf16, int rows, int cols, const void * xn_bf16, int T, int epilogue,
+                     const float * add1, const float * add2, float * y, void * y_bf16, pi_stream_t stream) {
+    return gemm_lib_run<__bf16>(PI_TYPE_BF16, g, W_bf16, rows, cols, xn_bf16, T, epilogue, add1, add2, y, y_bf16, stream);
 }
 
 }  // extern "C"

@@ -1,7 +1,6 @@
 // Steps of several tokens: 2..16 sequences in lockstep or a prompt chunk of one sequence.  Dense and sparse mat-muls on the matrix
 // cores, the union of the tokens' active rows, norm + rounding passes, Q4_0 expansion and row assembly for prompt chunks.
-#include "kernels_common.hpp"
-#include <type_traits>
+#include "gemm_tile.hpp"
 
 namespace {
 
@@ -110,10 +109,10 @@ __global__ __launch_bounds__(1024) void norm_round_f16_kernel(const float * __re
 // activation fragment once per 32-column step and uses it for its RT row tiles (the activations of a step are 16 x cols
 // fp16, as many bytes per row tile as the weights, so re-reading them per tile would double the L2 -> CU traffic);
 // 16 weight loads of 16 B per lane are in flight.
-template <int RT>
-__global__ __launch_bounds__(kBlock) void gemm_t16_f16_kernel(const __half * __restrict__ W, const __half * __restrict__ xn, int T, int rows, int cols,
+template <typename EL, int RT>
+__global__ __launch_bounds__(kBlock) void gemm_t16_kernel(const EL * __restrict__ W, const EL * __restrict__ xn, int T, int rows, int cols,
                                                               int epi, const float * __restrict__ add1, const float * __restrict__ add2, float * __restrict__ y,
-                                                              __half * __restrict__ y16, float thr, unsigned char * __restrict__ row_any, int lay) {
+                                                              EL * __restrict__ y16, float thr, unsigned char * __restrict__ row_any, int lay) {
     // lay bit 0: xn in the operand layout (pi_ol_index); bit 1: y16 in the operand layout (the next mat-mul's input)
     __shared__ float cs[kWavesPerBlock][16][17];
     constexpr int SU = 16 / RT;                     // steps per batch of loads
@@ -122,13 +121,13 @@ __global__ __launch_bounds__(kBlock) void gemm_t16_f16_kernel(const __half * __r
     const int row0 = blockIdx.x * 16 * RT;
     const int tok = i < T ? i : T - 1;
     const int kw = cols / kWavesPerBlock;
-    const __half * ap[RT];
+    const EL * ap[RT];
 #pragma unroll
     for (int rt = 0; rt < RT; ++rt) {
         const int row = row0 + rt * 16 + i < rows ? row0 + rt * 16 + i : rows - 1;
         ap[rt] = W + (size_t)row * cols + wave * kw + g * 8;
     }
-    const __half * bp = (lay & 1) ? xn + ((size_t)(wave * kw / 32) * 64 + g * 16 + i) * 8 : xn + (size_t)tok * cols + wave * kw + g * 8;
+    const EL * bp = (lay & 1) ? xn + ((size_t)(wave * kw / 32) * 64 + g * 16 + i) * 8 : xn + (size_t)tok * cols + wave * kw + g * 8;
     const int bstep = (lay & 1) ? 512 : 32;        // halves from one 32-column step's fragment to the next
     pi_f4 acc[RT];
 #pragma unroll
@@ -148,7 +147,7 @@ __global__ __launch_bounds__(kBlock) void gemm_t16_f16_kernel(const __half * __r
             if (s0 + u < steps) {
 #pragma unroll
                 for (int rt = 0; rt < RT; ++rt)
-                    acc[rt] = __builtin_amdgcn_mfma_f32_16x16x32_f16(__builtin_bit_cast(pi_h8, a[u][rt]), __builtin_bit_cast(pi_h8, b[u]), acc[rt], 0, 0, 0);
+                    acc[rt] = mma16<EL>(a[u][rt], b[u], acc[rt]);
             }
     }
     const int rr = threadIdx.x >> 4, t = threadIdx.x & 15;
@@ -169,7 +168,7 @@ __global__ __launch_bounds__(kBlock) void gemm_t16_f16_kernel(const __half * __r
             else if (epi == PI_EPI_ADD) sum = __fadd_rn(sum, add1[o]);
             else if (epi == PI_EPI_ADD2) sum = __fadd_rn(__fadd_rn(sum, add1[o]), add2[o]);
             y[o] = sum;
-            if (y16) y16[(lay & 2) ? pi_ol_index(t, row) : o] = __float2half_rn(sum);
+            if (y16) y16[(lay & 2) ? pi_ol_index(t, row) : o] = to_el<EL>(sum);
             act = !(sum < thr);
         }
         if (row_any) {      // predictor logits: is the row active for at least one token of the step?  (16 lanes = 16 tokens of a row)
@@ -185,10 +184,10 @@ __global__ __launch_bounds__(kBlock) void gemm_t16_f16_kernel(const __half * __r
 // row stride (conflict-free both ways) and reads it back in operand layout.  No workgroup barrier is involved: the
 // buffer belongs to one wave and LDS operations of a wave complete in order.  Two 256-column tiles of loads are in flight.
 constexpr int kGlStride = 512 + 16;               // bytes per LDS row: 256 fp16 + one 16-byte pad
-template <int RT, int NW>
-__global__ __launch_bounds__(64 * NW) void gemm_t16_lds_f16_kernel(const __half * __restrict__ W, const __half * __restrict__ xn, int T, int rows, int cols,
+template <typename EL, int RT, int NW>
+__global__ __launch_bounds__(64 * NW) void gemm_t16_lds_kernel(const EL * __restrict__ W, const EL * __restrict__ xn, int T, int rows, int cols,
                                                                   int epi, const float * __restrict__ add1, const float * __restrict__ add2, float * __restrict__ y,
-                                                                  __half * __restrict__ y16, float thr, unsigned char * __restrict__ row_any, int lay) {
+                                                                  EL * __restrict__ y16, float thr, unsigned char * __restrict__ row_any, int lay) {
     __shared__ __align__(16) unsigned char tile[NW][16 * kGlStride];
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     const int i = lane & 15, g = lane >> 4;
@@ -196,7 +195,7 @@ __global__ __launch_bounds__(64 * NW) void gemm_t16_lds_f16_kernel(const __half 
     const int row0 = blockIdx.x * 16 * RT;
     const int tok = i < T ? i : T - 1;
     // the 256-column super-steps of a row are dealt round-robin to the NW waves: wave w takes steps w, w + NW, ...
-    const __half * bp = (lay & 1) ? xn + (g * 16 + i) * 8 : xn + (size_t)tok * cols + g * 8;
+    const EL * bp = (lay & 1) ? xn + (g * 16 + i) * 8 : xn + (size_t)tok * cols + g * 8;
     const int bstep = (lay & 1) ? 512 : 32;        // halves from one 32-column step's fragment to the next
     unsigned char * mytile = tile[wave];
     pi_f4 acc[RT];
@@ -233,7 +232,7 @@ __global__ __launch_bounds__(64 * NW) void gemm_t16_lds_f16_kernel(const __half 
 #pragma unroll
                     for (int st = 0; st < 8; ++st) {
                         const pi_u32x4 a = *reinterpret_cast<const pi_u32x4 *>(mytile + i * kGlStride + (4 * st + g) * 16);
-                        acc[rt] = __builtin_amdgcn_mfma_f32_16x16x32_f16(__builtin_bit_cast(pi_h8, a), __builtin_bit_cast(pi_h8, b[st]), acc[rt], 0, 0, 0);
+                        acc[rt] = mma16<EL>(a, b[st], acc[rt]);
                     }
                 }
             }
@@ -261,7 +260,7 @@ __global__ __launch_bounds__(64 * NW) void gemm_t16_lds_f16_kernel(const __half 
             else if (epi == PI_EPI_ADD) sum = __fadd_rn(sum, add1[o]);
             else if (epi == PI_EPI_ADD2) sum = __fadd_rn(__fadd_rn(sum, add1[o]), add2[o]);
             y[o] = sum;
-            if (y16) y16[(lay & 2) ? pi_ol_index(t, row) : o] = __float2half_rn(sum);
+            if (y16) y16[(lay & 2) ? pi_ol_index(t, row) : o] = to_el<EL>(sum);
             act = !(sum < thr);
         }
         if (row_any) {
@@ -271,130 +270,28 @@ __global__ __launch_bounds__(64 * NW) void gemm_t16_lds_f16_kernel(const __half 
     }
 }
 
-// ---------------------------------------------------------------------------------------------------
-// Prompt chunks of any length on the matrix cores with both operands staged in LDS: y[t][row] = epi(W[row] . xn[t]).
-// A workgroup of four waves owns BM weight rows x BN tokens; the reduction dimension advances 64 columns at a time through two
-// LDS stages, and two more stages travel in registers as 16-byte global loads (one stage of MFMAs lasts about 0.2 us, less than a
-// trip to HBM); one barrier per stage.  Both operands are stored row by row with the reduction dimension contiguous, which is
-// the matrix cores' operand layout (eight consecutive columns per lane), so a fragment is one ds_read_b128.  A row is 128 bytes;
-// its eight 16-byte pieces are stored at piece ^ (row & 7), so that the 16 rows a quarter wave reads the same piece of, and the
-// eight pieces of a row that eight neighbouring lanes write, fall on different banks (the bank-conflict counter reads 0; with
-// rows padded to 144 bytes instead it read a third of the LDS cycles).  A wave computes (BM/2) x (BN/2) outputs as 16 x 16
-// tiles; per 32-column step it reads BM/32 + BN/32 fragments for (BM/32) * (BN/32) MFMAs.  Workgroups are numbered so that the
-// token tiles of one row tile run on the same XCD back to back: the row tile's weights cross HBM once and are re-read from that
-// XCD's L2.  cols % 64 == 0; rows and T need not fill the tiles (requests past the edge re-read the last row, results are not
-// stored).
-// ---------------------------------------------------------------------------------------------------
-constexpr int kGtBK = 64;                        // columns per stage
-constexpr int kGtRow = kGtBK * 2;                // bytes per LDS row
-template <int BM, int BN, int WGM = 2, int WGN = 2>      // output tile and the waves' grid over it (WGM x WGN waves)
-__global__ __launch_bounds__(64 * WGM * WGN, (WGM * WGN > 4 ? 1 : BM + BN <= 192 ? 3 : 2)) void gemm_tile_f16_kernel(const __half * __restrict__ W, const __half * __restrict__ xn, int T, int rows, int cols,
+// the dense mat-mul of a prompt chunk: y[t][row] = epi(W[row] . xn[t]) in the tiles of GemmTile
+template <typename EL, int BM, int BN, int WGM = 2, int WGN = 2>
+__global__ __launch_bounds__(64 * WGM * WGN, (WGM * WGN > 4 ? 1 : BM + BN <= 192 ? 3 : 2)) void gemm_tile_kernel(const EL * __restrict__ W, const EL * __restrict__ xn, int T, int rows, int cols,
                                                                   int nx, int ny, int epi, const float * __restrict__ add1, const float * __restrict__ add2,
-                                                                  float * __restrict__ y, __half * __restrict__ y16) {
-    constexpr int kThreads = 64 * WGM * WGN;
-    constexpr int WM = BM / WGM, WN = BN / WGN, MT = WM / 16, NT = WN / 16;
-    constexpr int ACH = BM * kGtBK * 2 / 16 / kThreads, BCH = BN * kGtBK * 2 / 16 / kThreads;  // 16-byte chunks per thread and stage
-    static_assert(WM % 16 == 0 && WN % 16 == 0 && ACH * kThreads * 16 == BM * kGtBK * 2 && BCH * kThreads * 16 == BN * kGtBK * 2, "tile does not divide among the waves");
+                                                                  float * __restrict__ y, EL * __restrict__ y16) {
+    using Tile = GemmTile<EL, BM, BN, WGM, WGN>;
+    constexpr int WM = Tile::WM, WN = Tile::WN, MT = Tile::MT, NT = Tile::NT;
     extern __shared__ __align__(16) unsigned char smem[];
-    unsigned char * sa = smem;                                     // [2][BM][kGtRow]
-    unsigned char * sb = smem + 2 * BM * kGtRow;                   // [2][BN][kGtRow]
     // workgroup -> (row tile, token tile): XCD x takes row tiles x, x + 8, ... and walks each one's token tiles in turn
     const int xcd = blockIdx.x % 8, slot = blockIdx.x / 8;
     const int tx = (slot / ny) * 8 + xcd, ty = slot % ny;
     if (tx >= nx) return;
     const int row0 = tx * BM, tok0 = ty * BN;
-    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, i = lane & 15, g = lane >> 4;
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, i = lane & 15, g = lane >> 4;
     const int wm = wave % WGM, wn = wave / WGM;
-    auto lds_off = [](int r, int kc) { return r * kGtRow + ((kc ^ (r & 7)) * 16); };
-    const __half * ga[ACH]; const __half * gb[BCH];
-    int la[ACH], lb[BCH];
+    const EL * ga[Tile::ACH]; const EL * gb[Tile::BCH];
 #pragma unroll
-    for (int j = 0; j < ACH; ++j) {
-        const int kc = tid % 8, r = j * (kThreads / 8) + tid / 8;
-        const int rr = row0 + r < rows ? row0 + r : rows - 1;
-        ga[j] = W + (size_t)rr * cols + kc * 8; la[j] = lds_off(r, kc);
-    }
+    for (int j = 0; j < Tile::ACH; ++j) ga[j] = W + (size_t)min(row0 + Tile::chunk_row(j), rows - 1) * cols + Tile::chunk_col();
 #pragma unroll
-    for (int j = 0; j < BCH; ++j) {
-        const int kc = tid % 8, r = j * (kThreads / 8) + tid / 8;
-        const int tt = tok0 + r < T ? tok0 + r : T - 1;
-        gb[j] = xn + (size_t)tt * cols + kc * 8; lb[j] = lds_off(r, kc);
-    }
+    for (int j = 0; j < Tile::BCH; ++j) gb[j] = xn + (size_t)min(tok0 + Tile::chunk_row(j), T - 1) * cols + Tile::chunk_col();
     pi_f4 acc[MT][NT];
-#pragma unroll
-    for (int m = 0; m < MT; ++m)
-#pragma unroll
-        for (int n = 0; n < NT; ++n) acc[m][n] = pi_f4{0.0f, 0.0f, 0.0f, 0.0f};
-    // Two column stages travel in registers while a third is being multiplied: stage kt sits in LDS half kt & 1, stages kt + 1 and
-    // kt + 2 are in flight (one stage of MFMAs is about 0.2 us, less than a trip to HBM).
-    pi_u32x4 ra[2][ACH], rb[2][BCH];
-    const int nk = cols / kGtBK;
-    auto fetch = [&](auto slot, int kt) {
-        constexpr int S = decltype(slot)::value;
-#pragma unroll
-        for (int j = 0; j < ACH; ++j) ra[S][j] = pi_ld16(ga[j] + (size_t)kt * kGtBK);
-#pragma unroll
-        for (int j = 0; j < BCH; ++j) rb[S][j] = pi_ld16(gb[j] + (size_t)kt * kGtBK);
-    };
-    auto stash = [&](auto slot) {              // registers of slot S -> LDS half S
-        constexpr int S = decltype(slot)::value;
-        unsigned char * na = sa + S * BM * kGtRow; unsigned char * nb = sb + S * BN * kGtRow;
-#pragma unroll
-        for (int j = 0; j < ACH; ++j) *reinterpret_cast<pi_u32x4 *>(na + la[j]) = ra[S][j];
-#pragma unroll
-        for (int j = 0; j < BCH; ++j) *reinterpret_cast<pi_u32x4 *>(nb + lb[j]) = rb[S][j];
-    };
-    const std::integral_constant<int, 0> c0; const std::integral_constant<int, 1> c1;
-    // every fetch and stash below is unconditional (past the last stage the last one is fetched again and stashed where nobody
-    // reads): the count of loads in flight is then the same on every path, and the waits name exactly the loads they need
-    const int last = nk - 1;
-    fetch(c0, 0);
-    fetch(c1, min(1, last));
-    stash(c0);
-    fetch(c0, min(2, last));
-    __syncthreads();
-    // the lane's two pieces (columns 8g.. of each 32-column step) of fragment row i: every 16-row tile starts on a multiple of 8
-    const int koff[2] = {(g ^ (i & 7)) * 16, ((4 + g) ^ (i & 7)) * 16};
-    const int frag_a = (wm * WM + i) * kGtRow, frag_b = (wn * WN + i) * kGtRow;
-    // The fragments of a stage's first 32 columns are read while the previous stage's second 32 are multiplied, those of its second
-    // 32 while its first are: every LDS read has a block of MFMAs between its issue and its use.
-    pi_u32x4 f0a[MT], f0b[NT], f1a[MT], f1b[NT];
-    auto frags = [&](auto par, auto half, pi_u32x4 * fa, pi_u32x4 * fb) {
-        constexpr int P = decltype(par)::value, KS = decltype(half)::value;
-        const unsigned char * ca = sa + P * BM * kGtRow + frag_a + koff[KS];
-        const unsigned char * cb = sb + P * BN * kGtRow + frag_b + koff[KS];
-#pragma unroll
-        for (int m = 0; m < MT; ++m) fa[m] = *reinterpret_cast<const pi_u32x4 *>(ca + m * 16 * kGtRow);
-#pragma unroll
-        for (int n = 0; n < NT; ++n) fb[n] = *reinterpret_cast<const pi_u32x4 *>(cb + n * 16 * kGtRow);
-    };
-    auto mfmas = [&](const pi_u32x4 * fa, const pi_u32x4 * fb) {
-#pragma unroll
-        for (int m = 0; m < MT; ++m)
-#pragma unroll
-            for (int n = 0; n < NT; ++n)
-                acc[m][n] = __builtin_amdgcn_mfma_f32_16x16x32_f16(__builtin_bit_cast(pi_h8, fa[m]), __builtin_bit_cast(pi_h8, fb[n]), acc[m][n], 0, 0, 0);
-    };
-    frags(c0, c0, f0a, f0b);
-    auto step = [&](auto par, int kt) {
-        constexpr int P = decltype(par)::value;
-        const std::integral_constant<int, P ^ 1> other;
-        frags(par, c1, f1a, f1b);
-        __builtin_amdgcn_sched_barrier(0);
-        mfmas(f0a, f0b);
-        stash(other);
-        fetch(other, min(kt + 3, last));
-        __builtin_amdgcn_sched_barrier(0);
-        __syncthreads();
-        __builtin_amdgcn_sched_barrier(0);
-        frags(other, c0, f0a, f0b);           // past the last stage: the re-stashed last stage, read and not used
-        __builtin_amdgcn_sched_barrier(0);
-        mfmas(f1a, f1b);
-        __builtin_amdgcn_sched_barrier(0);
-    };
-    int kt = 0;
-    for (; kt + 1 < nk; kt += 2) { step(c0, kt); step(c1, kt + 1); }
-    if (kt < nk) step(c0, kt);
+    Tile::run(smem, ga, gb, cols / kGtBK, acc);
     // acc[m][n][r] = y[token tok0 + wn*WN + n*16 + i][row row0 + wm*WM + m*16 + 4g + r]: four consecutive rows per lane
 #pragma unroll
     for (int m = 0; m < MT; ++m)
@@ -416,8 +313,8 @@ __global__ __launch_bounds__(64 * WGM * WGN, (WGM * WGN > 4 ? 1 : BM + BN <= 192
                 }
                 *reinterpret_cast<float4 *>(y + o) = make_float4(v[0], v[1], v[2], v[3]);
                 if (y16) {
-                    __half2 h2[2] = {__floats2half2_rn(v[0], v[1]), __floats2half2_rn(v[2], v[3])};
-                    *reinterpret_cast<uint2 *>(y16 + o) = *reinterpret_cast<const uint2 *>(h2);
+                    EL h4[4] = {to_el<EL>(v[0]), to_el<EL>(v[1]), to_el<EL>(v[2]), to_el<EL>(v[3])};
+                    *reinterpret_cast<uint2 *>(y16 + o) = __builtin_bit_cast(uint2, h4);
                 }
             } else {
                 for (int r = 0; r < 4 && row + r < rows; ++r) {
@@ -426,7 +323,7 @@ __global__ __launch_bounds__(64 * WGM * WGN, (WGM * WGN > 4 ? 1 : BM + BN <= 192
                     else if (epi == PI_EPI_ADD) s = __fadd_rn(s, add1[o + r]);
                     else if (epi == PI_EPI_ADD2) s = __fadd_rn(__fadd_rn(s, add1[o + r]), add2[o + r]);
                     y[o + r] = s;
-                    if (y16) y16[o + r] = __float2half_rn(s);
+                    if (y16) y16[o + r] = to_el<EL>(s);
                 }
             }
         }
@@ -1119,7 +1016,10 @@ int pi_k_norm_q8_round_f16(const float * x, int T, int cols, const pi_norm * nor
     return pi::check_launch("pi_k_norm_q8_round_f16");
 }
 
+}  // extern "C"
+
 // lay bit 0: xn_f16 in the operand layout of the step's activations (pi_ol_index), bit 1: y_f16 written in it
+template <typename EL>
 static int gemm_launch(const char * who, const void * W, int rows, int cols, const void * xn_f16, int T, int epilogue, const float * add1, const float * add2,
                        float * y, void * y_f16, float thr, unsigned char * row_any, pi_stream_t stream, int lay = 0) {
     if (!W || !xn_f16 || !y || rows <= 0) return pi::fail(PI_E_ARG, who);
@@ -1128,10 +1028,10 @@ static int gemm_launch(const char * who, const void * W, int rows, int cols, con
         return pi::fail(PI_E_ARG, "batched mat-mul: bad epilogue arguments");
     // row tiles per wave: enough workgroups to fill the chip first, then as few reads of the activations as possible
     const int rt = rows >= 16384 ? 4 : rows >= 5120 ? 2 : 1;      // (two tiles already at 5120 rows: the activations, re-read per row tile, are what limits one tile per wave)
-#define PI_GEMM_T16(RT) hipLaunchKernelGGL((gemm_t16_f16_kernel<RT>), dim3((rows + 16 * RT - 1) / (16 * RT)), dim3(kBlock), 0, (hipStream_t)stream, \
-                       (const __half *)W, (const __half *)xn_f16, T, rows, cols, epilogue, add1, add2, y, (__half *)y_f16, thr, row_any, lay)
-#define PI_GEMM_LDS(RT, NW) hipLaunchKernelGGL((gemm_t16_lds_f16_kernel<RT, NW>), dim3((rows + 16 * RT - 1) / (16 * RT)), dim3(64 * NW), 0, (hipStream_t)stream, \
-                       (const __half *)W, (const __half *)xn_f16, T, rows, cols, epilogue, add1, add2, y, (__half *)y_f16, thr, row_any, lay)
+#define PI_GEMM_T16(RT) hipLaunchKernelGGL((gemm_t16_kernel<EL, RT>), dim3((rows + 16 * RT - 1) / (16 * RT)), dim3(kBlock), 0, (hipStream_t)stream, \
+                       (const EL *)W, (const EL *)xn_f16, T, rows, cols, epilogue, add1, add2, y, (EL *)y_f16, thr, row_any, lay)
+#define PI_GEMM_LDS(RT, NW) hipLaunchKernelGGL((gemm_t16_lds_kernel<EL, RT, NW>), dim3((rows + 16 * RT - 1) / (16 * RT)), dim3(64 * NW), 0, (hipStream_t)stream, \
+                       (const EL *)W, (const EL *)xn_f16, T, rows, cols, epilogue, add1, add2, y, (EL *)y_f16, thr, row_any, lay)
     if (cols % 256 == 0) {
         // waves per workgroup: when every workgroup has a compute unit to itself (at most one per unit), eight waves keep twice
         // the loads in flight per unit; with more workgroups than units the chip is full with four
@@ -1146,16 +1046,31 @@ static int gemm_launch(const char * who, const void * W, int rows, int cols, con
     return pi::check_launch(who);
 }
 
+extern "C" {
+
 int pi_k_gemm_f16(const void * W, int rows, int cols, const void * xn_f16, int T, int epilogue, const float * add1, const float * add2,
                   float * y, void * y_f16, pi_stream_t stream) {
-    return gemm_launch("pi_k_gemm_f16", W, rows, cols, xn_f16, T, epilogue, add1, add2, y, y_f16, 0.0f, nullptr, stream);
+    return gemm_launch<__half>("pi_k_gemm_f16", W, rows, cols, xn_f16, T, epilogue, add1, add2, y, y_f16, 0.0f, nullptr, stream);
 }
 
 int pi_k_gemm_f16_ol(const void * W, int rows, int cols, const void * xn_ol, int T, int epilogue, const float * add1, const float * add2,
                      float * y, void * y_ol, pi_stream_t stream) {
     if (y_ol && rows % 8) return pi::fail(PI_E_ARG, "pi_k_gemm_f16_ol: rows % 8 == 0 required for the fp16 copy in the operand layout");
-    return gemm_launch("pi_k_gemm_f16_ol", W, rows, cols, xn_ol, T, epilogue, add1, add2, y, y_ol, 0.0f, nullptr, stream, 3);
+    return gemm_launch<__half>("pi_k_gemm_f16_ol", W, rows, cols, xn_ol, T, epilogue, add1, add2, y, y_ol, 0.0f, nullptr, stream, 3);
 }
+
+int pi_k_gemm_bf16(const void * W, int rows, int cols, const void * xn_bf16, int T, int epilogue, const float * add1, const float * add2,
+                   float * y, void * y_bf16, pi_stream_t stream) {
+    return gemm_launch<__bf16>("pi_k_gemm_bf16", W, rows, cols, xn_bf16, T, epilogue, add1, add2, y, y_bf16, 0.0f, nullptr, stream);
+}
+
+int pi_k_gemm_bf16_ol(const void * W, int rows, int cols, const void * xn_ol, int T, int epilogue, const float * add1, const float * add2,
+                      float * y, void * y_ol, pi_stream_t stream) {
+    if (y_ol && rows % 8) return pi::fail(PI_E_ARG, "pi_k_gemm_bf16_ol: rows % 8 == 0 required for the bf16 copy in the operand layout");
+    return gemm_launch<__bf16>("pi_k_gemm_bf16_ol", W, rows, cols, xn_ol, T, epilogue, add1, add2, y, y_ol, 0.0f, nullptr, stream, 3);
+}
+
+}  // extern "C"
 
 // Output tiles the kernel is built for (weight rows x tokens per workgroup); the first two run eight waves, one workgroup per unit.
 constexpr int kGtNShapes = 7;
@@ -1176,26 +1091,27 @@ static int gt_choose(int rows, int T, int n_cu) {
     return best;
 }
 
-int pi_k_gemm_tile_f16(const void * W, int rows, int cols, const void * xn_f16, int T, int epilogue, const float * add1, const float * add2,
+template <typename EL>
+static int gemm_tile_launch(const void * W, int rows, int cols, const void * xn_f16, int T, int epilogue, const float * add1, const float * add2,
                        float * y, void * y_f16, int tile, pi_stream_t stream) {
-    if (!W || !xn_f16 || !y || rows <= 0 || T <= 0) return pi::fail(PI_E_ARG, "pi_k_gemm_tile_f16: null pointer or empty shape");
-    if (cols <= 0 || cols % kGtBK) return pi::fail(PI_E_ARG, "pi_k_gemm_tile_f16: cols % 64 == 0 required");
+    if (!W || !xn_f16 || !y || rows <= 0 || T <= 0) return pi::fail(PI_E_ARG, "pi_k_gemm_tile: null pointer or empty shape");
+    if (cols <= 0 || cols % kGtBK) return pi::fail(PI_E_ARG, "pi_k_gemm_tile: cols % 64 == 0 required");
     if (epilogue < 0 || epilogue > PI_EPI_ADD2 || (epilogue >= PI_EPI_ADD && !add1) || (epilogue == PI_EPI_ADD2 && !add2))
-        return pi::fail(PI_E_ARG, "pi_k_gemm_tile_f16: bad epilogue arguments");
+        return pi::fail(PI_E_ARG, "pi_k_gemm_tile: bad epilogue arguments");
     if ((((uintptr_t)W | (uintptr_t)xn_f16 | (uintptr_t)y | (uintptr_t)add1 | (uintptr_t)add2) & 15) != 0 || ((uintptr_t)y_f16 & 7) != 0)
-        return pi::fail(PI_E_ARG, "pi_k_gemm_tile_f16: operands must be 16-byte aligned");
+        return pi::fail(PI_E_ARG, "pi_k_gemm_tile: operands must be 16-byte aligned");
     hipStream_t st = (hipStream_t)stream;
     int shape = -1;
     if (tile == 0) shape = gt_choose(rows, T, pi::compute_units());
     else for (int s = 0; s < kGtNShapes; ++s) if (tile == kGtShapes[s][0] * 1000 + kGtShapes[s][1]) shape = s;
-    if (shape < 0) return pi::fail(PI_E_ARG, "pi_k_gemm_tile_f16: tile must be 0 or one of 256128, 192128, 128128, 96128, 128064, 64128, 64064");
+    if (shape < 0) return pi::fail(PI_E_ARG, "pi_k_gemm_tile: tile must be 0 or one of 256128, 192128, 128128, 96128, 128064, 64128, 64064");
 #define PI_GEMM_TILE(BM, BN, WGM, WGN) do {                                                                                               \
         const int nx = (rows + BM - 1) / BM, ny = (T + BN - 1) / BN;                                                                      \
-        const size_t sh = (size_t)2 * (BM + BN) * kGtRow;                                                                                 \
+        const size_t sh = GemmTile<EL, BM, BN, WGM, WGN>::kLds;                                                                                 \
         static bool raised = false;                                                                                                       \
-        if (!raised && sh > 64 * 1024) { PI_HIP_TRY(hipFuncSetAttribute((const void *)gemm_tile_f16_kernel<BM, BN, WGM, WGN>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)sh)); raised = true; } \
-        hipLaunchKernelGGL((gemm_tile_f16_kernel<BM, BN, WGM, WGN>), dim3(8 * ((nx + 7) / 8) * ny), dim3(64 * WGM * WGN), sh, st, (const __half *)W, (const __half *)xn_f16, T, rows, cols,   \
-                           nx, ny, epilogue, add1, add2, y, (__half *)y_f16);                                                             \
+        if (!raised && sh > 64 * 1024) { PI_HIP_TRY(hipFuncSetAttribute((const void *)gemm_tile_kernel<EL, BM, BN, WGM, WGN>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)sh)); raised = true; } \
+        hipLaunchKernelGGL((gemm_tile_kernel<EL, BM, BN, WGM, WGN>), dim3(8 * ((nx + 7) / 8) * ny), dim3(64 * WGM * WGN), sh, st, (const EL *)W, (const EL *)xn_f16, T, rows, cols,   \
+                           nx, ny, epilogue, add1, add2, y, (EL *)y_f16);                                                             \
     } while (0)
     switch (shape) {
         case 0: PI_GEMM_TILE(256, 128, 4, 2); break;
@@ -1207,8 +1123,21 @@ int pi_k_gemm_tile_f16(const void * W, int rows, int cols, const void * xn_f16, 
         default: PI_GEMM_TILE(64, 64, 2, 2); break;
     }
 #undef PI_GEMM_TILE
-    return pi::check_launch("pi_k_gemm_tile_f16");
+    return pi::check_launch("pi_k_gemm_tile");
 }
+
+extern "C" {
+
+int pi_k_gemm_tile_f16(const void * W, int rows, int cols, const void * xn_f16, int T, int epilogue, const float * add1, const float * add2,
+                       float * y, void * y_f16, int tile, pi_stream_t stream) {
+    return gemm_tile_launch<__half>(W, rows, cols, xn_f16, T, epilogue, add1, add2, y, y_f16, tile, stream);
+}
+
+int pi_k_gemm_tile_bf16(const void * W, int rows, int cols, const void * xn_bf16, int T, int epilogue, const float * add1, const float * add2,
+                        float * y, void * y_bf16, int tile, pi_stream_t stream) {
+    return gemm_tile_launch<__bf16>(W, rows, cols, xn_bf16, T, epilogue, add1, add2, y, y_bf16, tile, stream);
+}
+
 int pi_k_ffn_h_f16(const float * up, const float * gate, const float * logits, float threshold, int T, int ff, void * h_f16, pi_stream_t stream) {
     if (!up || !logits || !h_f16 || T <= 0 || ff <= 0) return pi::fail(PI_E_ARG, "pi_k_ffn_h_f16: bad arguments");
     hipLaunchKernelGGL(ffn_h_f16_kernel, dim3(1024), dim3(256), 0, (hipStream_t)stream, up, gate, logits, threshold, (size_t)T * ff, (__half *)h_f16, 0);
@@ -1293,13 +1222,13 @@ int pi_k_transpose_f16(const void * in, int rows, int cols, void * out, pi_strea
 int pi_k_batch_predictor_fc2(const void * fc2_f16, int ff, int r, const void * hidden_f16, int T, float threshold, float * logits,
                              pi_workspace * ws, pi_stream_t stream) {
     if (!ws || ff > ws->max_ff) return pi::fail(PI_E_ARG, "pi_k_batch_predictor_fc2: ff exceeds the workspace");
-    return gemm_launch("pi_k_batch_predictor_fc2", fc2_f16, ff, r, hidden_f16, T, PI_EPI_NONE, nullptr, nullptr, logits, nullptr, threshold, ws->row_any, stream);
+    return gemm_launch<__half>("pi_k_batch_predictor_fc2", fc2_f16, ff, r, hidden_f16, T, PI_EPI_NONE, nullptr, nullptr, logits, nullptr, threshold, ws->row_any, stream);
 }
 
 int pi_k_batch_predictor_fc2_ol(const void * fc2_f16, int ff, int r, const void * hidden_ol, int T, float threshold, float * logits,
                                 pi_workspace * ws, pi_stream_t stream) {
     if (!ws || ff > ws->max_ff) return pi::fail(PI_E_ARG, "pi_k_batch_predictor_fc2_ol: ff exceeds the workspace");
-    return gemm_launch("pi_k_batch_predictor_fc2_ol", fc2_f16, ff, r, hidden_ol, T, PI_EPI_NONE, nullptr, nullptr, logits, nullptr, threshold, ws->row_any, stream, 1);
+    return gemm_launch<__half>("pi_k_batch_predictor_fc2_ol", fc2_f16, ff, r, hidden_ol, T, PI_EPI_NONE, nullptr, nullptr, logits, nullptr, threshold, ws->row_any, stream, 1);
 }
 
 static int batch_sparse_ffn(const float * logits, int T, int ff, float threshold, const void * up_f16, const void * gate_f16, const void * down_t_f16,

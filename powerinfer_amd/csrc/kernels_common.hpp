@@ -185,7 +185,20 @@ __device__ __forceinline__ float apply_epilogue(float v, int epi, const float * 
 
 // shapes and operand types the step kernels and their callers agree on
 typedef _Float16 pi_h8 __attribute__((ext_vector_type(8)));
+typedef __bf16   pi_b8 __attribute__((ext_vector_type(8)));
 typedef float    pi_f4 __attribute__((ext_vector_type(4)));
+
+// the 16 x 16 x 32 matrix-core product and the storage conversion of the two 16-bit element types the mat-muls exist for
+template <typename EL> __device__ __forceinline__ pi_f4 mma16(const pi_u32x4 & a, const pi_u32x4 & b, pi_f4 c);
+template <> __device__ __forceinline__ pi_f4 mma16<__half>(const pi_u32x4 & a, const pi_u32x4 & b, pi_f4 c) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_f16(__builtin_bit_cast(pi_h8, a), __builtin_bit_cast(pi_h8, b), c, 0, 0, 0);
+}
+template <> __device__ __forceinline__ pi_f4 mma16<__bf16>(const pi_u32x4 & a, const pi_u32x4 & b, pi_f4 c) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(pi_b8, a), __builtin_bit_cast(pi_b8, b), c, 0, 0, 0);
+}
+template <typename EL> __device__ __forceinline__ EL to_el(float v);                 // round to nearest even
+template <> __device__ __forceinline__ __half to_el<__half>(float v) { return __float2half_rn(v); }
+template <> __device__ __forceinline__ __bf16 to_el<__bf16>(float v) { return (__bf16)v; }
 constexpr int kBtMaxT = 16;
 constexpr int kChunkMaxT = 512;           // longest chunk of the attention, embedding and elementwise kernels of a prompt chunk
 constexpr int kBmGroups = 32;

@@ -552,6 +552,16 @@ __global__ void fill_normal_f16_kernel(__half * __restrict__ p, size_t n, uint64
     }
 }
 
+// the same values rounded to bf16
+__global__ void fill_normal_bf16_kernel(__bf16 * __restrict__ p, size_t n, uint64_t seed, float std) {
+    for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (size_t)gridDim.x * blockDim.x) {
+        const uint64_t r = mix64(seed * 0xD1342543DE82EF95ull + i);
+        const float u1 = ((uint32_t)(r >> 32) + 1.0f) * (1.0f / 4294967296.0f);
+        const float u2 = (uint32_t)r * (1.0f / 4294967296.0f);
+        p[i] = (__bf16)(sqrtf(-2.0f * logf(u1)) * cosf(6.28318530718f * u2) * std);
+    }
+}
+
 // N(0, std^2) values quantised to Q4_0 exactly as quantize_row_q4_0_reference does (ggml-quants.c:428-463): the
 // element of largest magnitude (first one wins) sets d = max / -8, q = min(15, (int)(x / d + 8.5)).  One thread per block.
 __global__ void fill_normal_q4_0_kernel(pi_block_q4_0 * __restrict__ p, size_t n_blocks, uint64_t seed, float std) {
@@ -744,6 +754,15 @@ int pi_fill_normal_f16(void * dptr, size_t n, uint64_t seed, float std, const fl
     if (blocks > 65536) blocks = 65536;
     hipLaunchKernelGGL(fill_normal_f16_kernel, dim3((unsigned)blocks), dim3(256), 0, (hipStream_t)stream, (__half *)dptr, n, seed, std, row_bias, cols);
     return pi::check_launch("pi_fill_normal_f16");
+}
+
+int pi_fill_normal_bf16(void * dptr, size_t n, uint64_t seed, float std, pi_stream_t stream) {
+    if (!dptr) return pi::fail(PI_E_ARG, "pi_fill_normal_bf16: null pointer");
+    if (n == 0) return PI_OK;
+    size_t blocks = (n + 255) / 256;
+    if (blocks > 65536) blocks = 65536;
+    hipLaunchKernelGGL(fill_normal_bf16_kernel, dim3((unsigned)blocks), dim3(256), 0, (hipStream_t)stream, (__bf16 *)dptr, n, seed, std);
+    return pi::check_launch("pi_fill_normal_bf16");
 }
 
 int pi_fill_normal_q4_0(void * dptr, size_t n_weights, uint64_t seed, float std, pi_stream_t stream) {

@@ -1,6 +1,7 @@
 // Operators of the models that are described layer by layer, apart from attention: embedding + norm, the pair of norms of a parallel
 // layer, grouped mat-muls (heads of a latent attention, experts), rotation angles, expert choice, and the sum that closes a layer.
 // Templated on the storage of activations: bf16 (matrix cores on bf16 operands, fp32 accumulation) or fp32.
+#include "gemm_tile.hpp"
 #include "layer_types.hpp"
 
 namespace {
@@ -87,7 +88,6 @@ __global__ __launch_bounds__(256) void group_gemm_kernel(pi_group_gemm g) {
     }
     pi_f4 acc[2] = {pi_f4{0, 0, 0, 0}, pi_f4{0, 0, 0, 0}};
     const bool two = t0 + 16 < n;
-#pragma unroll 4
     for (int k = 0; k < g.cols; k += 32) {
         const Frag<ST> a = frag_weights<ST>(W + k);
         frag_mma(a, frag_load(xp[0] + k), acc[0]);
@@ -180,47 +180,128 @@ __global__ __launch_bounds__(64) void route_kernel(const float * __restrict__ z,
     for (int k = lane; k < top; k += 64) weights[(size_t)t * top + k] = weights[(size_t)t * top + k] / (total + 1e-20f);
 }
 
-// pairs in expert order, one workgroup: thread e counts and places the pairs of expert e (and e + 1024, ...), reading the ids of a block
-// of pairs from LDS; pairs keep their order within an expert
-constexpr int kSortTile = 4096;
+// Pairs in expert order, one workgroup with the experts' counters in LDS: counts, their prefix sums, places.  The order of the pairs
+// within an expert is free (every row of the grouped products is computed on its own).  tiles (optional): {expert, first place} of
+// every group of up to tile_n pairs of one expert, n_tiles of them - the token tiles of the grouped products.
 __global__ __launch_bounds__(1024) void moe_sort_kernel(const int32_t * __restrict__ ids, int n, int E, int32_t * __restrict__ off, int32_t * __restrict__ perm,
-                                                        int32_t * __restrict__ inv) {
-    __shared__ int32_t tile[kSortTile];
+                                                        int32_t * __restrict__ inv, int tile_n, int2 * __restrict__ tiles, int32_t * __restrict__ n_tiles) {
+    extern __shared__ int cnt[];
     __shared__ int sred[16];
-    int base = 0;
+    for (int e = threadIdx.x; e < E; e += 1024) cnt[e] = 0;
+    __syncthreads();
+    for (int p = threadIdx.x; p < n; p += 1024) atomicAdd(&cnt[ids[p]], 1);
+    __syncthreads();
+    int base = 0, tbase = 0;
     for (int e0 = 0; e0 < E; e0 += 1024) {
-        const int e = e0 + threadIdx.x;
-        int cnt = 0;
-        for (int p0 = 0; p0 < n; p0 += kSortTile) {
-            const int m = min(kSortTile, n - p0);
-            __syncthreads();
-            for (int p = threadIdx.x; p < m; p += 1024) tile[p] = ids[p0 + p];
-            __syncthreads();
-            if (e < E) for (int p = 0; p < m; ++p) cnt += tile[p] == e ? 1 : 0;
+        const int e = e0 + threadIdx.x, c = e < E ? cnt[e] : 0;
+        int tot, ttot;
+        const int at = base + block_exclusive_scan_i32(c, &tot, sred);
+        const int nt = tiles ? (c + tile_n - 1) / tile_n : 0;
+        const int ta = tbase + block_exclusive_scan_i32(nt, &ttot, sred);
+        if (e < E) {
+            off[e] = at;
+            cnt[e] = at;
+            for (int k = 0; k < nt; ++k) tiles[ta + k] = make_int2(e, at + k * tile_n);
         }
-        int tot;
-        int at = base + block_exclusive_scan_i32(cnt, &tot, sred);
-        if (e < E) off[e] = at;
-        for (int p0 = 0; p0 < n; p0 += kSortTile) {
-            const int m = min(kSortTile, n - p0);
-            __syncthreads();
-            for (int p = threadIdx.x; p < m; p += 1024) tile[p] = ids[p0 + p];
-            __syncthreads();
-            if (e < E) for (int p = 0; p < m; ++p) if (tile[p] == e) { perm[at] = p0 + p; inv[p0 + p] = at; ++at; }
-        }
-        base += tot;
+        base += tot; tbase += ttot;
     }
-    if (threadIdx.x == 0) off[E] = base;
+    if (threadIdx.x == 0) { off[E] = base; if (tiles) *n_tiles = tbase; }
+    __syncthreads();
+    for (int p = threadIdx.x; p < n; p += 1024) {
+        const int at = atomicAdd(&cnt[ids[p]], 1);
+        perm[at] = p;
+        inv[p] = at;
+    }
 }
 
-__global__ __launch_bounds__(256) void moe_combine_kernel(const float * __restrict__ x, const float * __restrict__ mix, const float * __restrict__ y,
+// ---------------------------------------------------------------------------------------------------------------------------------
+// grouped mat-mul of prompt portions (bf16): GemmTile per (group, token tile, row tile).  Token tiles come from moe_sort's list
+// (g.tiles) or, without a list, every group has ceil(T / BN) of them.  The units are dealt out so that an XCD works through a
+// contiguous range of them: the row tiles of a token tile, and the token tiles of a group, share that XCD's L2.
+// ---------------------------------------------------------------------------------------------------------------------------------
+template <int BM, int BN, int WGM, int WGN>
+__global__ __launch_bounds__(64 * WGM * WGN, (WGM * WGN > 4 ? 1 : BM + BN <= 192 ? 3 : 2)) void group_tile_kernel(pi_group_gemm g, int nx, int max_units) {
+    using Tile = GemmTile<bf16, BM, BN, WGM, WGN>;
+    constexpr int WM = Tile::WM, WN = Tile::WN, MT = Tile::MT, NT = Tile::NT;
+    extern __shared__ __align__(16) unsigned char smem[];
+    const int tt = (g.T + BN - 1) / BN;                       // token tiles of a group without a list
+    const int units = g.off ? *g.n_tiles * nx : max_units;
+    const int per = (units + 7) / 8, unit = (int)(blockIdx.x % 8) * per + (int)blockIdx.x / 8;
+    if ((int)blockIdx.x / 8 >= per || unit >= units) return;
+    const int tx = unit % nx, ty = unit / nx;
+    int grp, lo, n;                                           // group, first token (place), tokens from there on
+    if (g.off) {
+        const int2 t = reinterpret_cast<const int2 *>(g.tiles)[ty];
+        grp = t.x; lo = t.y; n = g.off[grp + 1] - lo;
+    } else {
+        grp = ty / tt; lo = (ty % tt) * BN; n = g.T - lo;
+    }
+    n = min(n, BN);
+    const int row0 = tx * BM;
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, i = lane & 15, q = lane >> 4;
+    const int wm = wave % WGM, wn = wave / WGM;
+    const bf16 * W = (const bf16 *)g.W + (size_t)grp * g.w_gs;
+    const bf16 * x = (const bf16 *)g.x + (g.off ? 0 : (size_t)grp * g.x_gs);
+    const bf16 * ga[Tile::ACH]; const bf16 * gb[Tile::BCH];
+#pragma unroll
+    for (int j = 0; j < Tile::ACH; ++j) ga[j] = W + (size_t)min(row0 + Tile::chunk_row(j), g.rows - 1) * g.ldw + Tile::chunk_col();
+#pragma unroll
+    for (int j = 0; j < Tile::BCH; ++j) {
+        const int s = lo + min(Tile::chunk_row(j), n - 1);
+        gb[j] = x + (size_t)(g.gather ? g.gather[s] / g.gather_div : s) * g.ldx + Tile::chunk_col();
+    }
+    pi_f4 acc[MT][NT];
+    Tile::run(smem, ga, gb, g.cols / kGtBK, acc);
+#pragma unroll
+    for (int m = 0; m < MT; ++m)
+#pragma unroll
+        for (int nn = 0; nn < NT; ++nn) {
+            const int row = row0 + wm * WM + m * 16 + 4 * q, tok = wn * WN + nn * 16 + i;
+            if (tok >= n || row >= g.rows) continue;
+            const size_t o = (g.off ? 0 : (size_t)grp * g.y_gs) + (size_t)(lo + tok) * g.ldy + row;
+            float v[4];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                v[r] = acc[m][nn][r] * g.alpha;
+                if (g.relu2) { v[r] = fmaxf(v[r], 0.0f); v[r] *= v[r]; }
+            }
+            const bool quad = row + 4 <= g.rows && (o & 3) == 0;
+            if (g.y_f32) {
+                float * y = (float *)g.y + o;
+                if (quad) *reinterpret_cast<float4 *>(y) = make_float4(v[0], v[1], v[2], v[3]);
+                else for (int r = 0; r < 4 && row + r < g.rows; ++r) y[r] = v[r];
+            } else {
+                bf16 * y = (bf16 *)g.y + o;
+                bf16 b[4] = {(bf16)v[0], (bf16)v[1], (bf16)v[2], (bf16)v[3]};
+                if (quad) *reinterpret_cast<uint2 *>(y) = __builtin_bit_cast(uint2, b);
+                else for (int r = 0; r < 4 && row + r < g.rows; ++r) y[r] = b[r];
+            }
+        }
+}
+
+template <int BM, int BN, int WGM, int WGN> int launch_group_tile(const pi_group_gemm & g, hipStream_t st) {
+    using Tile = GemmTile<bf16, BM, BN, WGM, WGN>;
+    static bool raised = false;
+    if (!raised && Tile::kLds > 64 * 1024) {
+        PI_HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void *>(&group_tile_kernel<BM, BN, WGM, WGN>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)Tile::kLds));
+        raised = true;
+    }
+    const int nx = (g.rows + BM - 1) / BM;
+    const long long units = (long long)nx * (g.off ? g.max_tiles : (long long)g.n_group * ((g.T + BN - 1) / BN));
+    if (units > (1 << 30)) return pi::fail(PI_E_ARG, "pi_k_group_gemm_tile: too many tiles");
+    hipLaunchKernelGGL((group_tile_kernel<BM, BN, WGM, WGN>), dim3((unsigned)((units + 7) / 8 * 8)), dim3(64 * WGM * WGN), Tile::kLds, st, g, nx, (int)units);
+    return pi::check_launch("pi_k_group_gemm_tile");
+}
+
+template <typename ST>
+__global__ __launch_bounds__(256) void moe_combine_kernel(const float * __restrict__ x, const float * __restrict__ mix, const ST * __restrict__ y,
                                                           const int32_t * __restrict__ inv, const float * __restrict__ weights, int top, int cols,
                                                           float * __restrict__ out, float * __restrict__ keep) {
     const int t = blockIdx.y, c = blockIdx.x * 256 + threadIdx.x;
     if (c >= cols) return;
     const size_t o = (size_t)t * cols + c;
     float s = 0.0f;
-    if (weights) for (int k = 0; k < top; ++k) s = fmaf(weights[(size_t)t * top + k], y[(size_t)inv[(size_t)t * top + k] * cols + c], s);
+    if (weights) for (int k = 0; k < top; ++k) s = fmaf(weights[(size_t)t * top + k], from_st(y[(size_t)inv[(size_t)t * top + k] * cols + c]), s);
     const float v = x[o] + (mix[o] + s);
     out[o] = v;
     if (keep) keep[o] = v;
@@ -301,16 +382,30 @@ int pi_k_route(const float * z, int T, int n_expert, int n_top, int n_group, int
     return pi::check_launch("pi_k_route");
 }
 
-int pi_k_moe_sort(const int32_t * ids, int n_pairs, int n_expert, int32_t * off, int32_t * perm, int32_t * inv, pi_stream_t stream) {
-    if (!ids || !off || !perm || !inv || n_pairs <= 0 || n_expert <= 0) return pi::fail(PI_E_ARG, "pi_k_moe_sort: bad arguments");
-    hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(1024), 0, (hipStream_t)stream, ids, n_pairs, n_expert, off, perm, inv);
+int pi_k_moe_sort(const int32_t * ids, int n_pairs, int n_expert, int32_t * off, int32_t * perm, int32_t * inv, int tile_n, int32_t * tiles, int32_t * n_tiles,
+                  pi_stream_t stream) {
+    if (!ids || !off || !perm || !inv || n_pairs <= 0 || n_expert <= 0 || n_expert > 8192 || (tiles && (tile_n <= 0 || !n_tiles))) return pi::fail(PI_E_ARG, "pi_k_moe_sort: bad arguments");
+    hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(1024), sizeof(int) * n_expert, (hipStream_t)stream, ids, n_pairs, n_expert, off, perm, inv, tile_n, (int2 *)tiles, n_tiles);
     return pi::check_launch("pi_k_moe_sort");
 }
 
-int pi_k_moe_combine(const float * x, const float * mix, const float * y, const int32_t * inv, const float * weights, int n_top, int T, int cols,
+int pi_k_group_gemm_tile(const pi_group_gemm * g, int tile_n, pi_stream_t stream) {
+    if (!g || !g->W || !g->x || !g->y || g->rows <= 0 || g->cols <= 0 || g->cols % kGtBK || g->ldw < g->cols || g->ldw % 8 || g->ldx < g->cols || g->ldx % 8 ||
+        g->ldy < g->rows || g->T <= 0 || g->n_group <= 0 || (g->gather && g->gather_div <= 0) || g->w_gs % 8 || g->x_gs % 8 || (g->off && (!g->tiles || !g->n_tiles || g->max_tiles <= 0)))
+        return pi::fail(PI_E_ARG, "pi_k_group_gemm_tile: bad arguments");
+    if ((((uintptr_t)g->W | (uintptr_t)g->x | (uintptr_t)g->y) & 15) != 0) return pi::fail(PI_E_ARG, "pi_k_group_gemm_tile: operands must be 16-byte aligned");
+    hipStream_t st = (hipStream_t)stream;
+    if (tile_n == 128) return launch_group_tile<128, 128, 2, 2>(*g, st);
+    if (tile_n == 64) return g->rows <= 64 ? launch_group_tile<64, 64, 2, 2>(*g, st) : launch_group_tile<128, 64, 2, 2>(*g, st);
+    return pi::fail(PI_E_ARG, "pi_k_group_gemm_tile: tile_n must be 64 or 128");
+}
+
+int pi_k_moe_combine(int type, const float * x, const float * mix, const void * y, const int32_t * inv, const float * weights, int n_top, int T, int cols,
                      float * out, float * keep, pi_stream_t stream) {
     if (!x || !mix || !out || T <= 0 || T > 65535 || cols <= 0 || (weights && (!y || !inv || n_top <= 0))) return pi::fail(PI_E_ARG, "pi_k_moe_combine: bad arguments");
-    hipLaunchKernelGGL(moe_combine_kernel, dim3((cols + 255) / 256, T), dim3(256), 0, (hipStream_t)stream, x, mix, y, inv, weights, n_top, cols, out, keep);
+    const dim3 grid((cols + 255) / 256, T);
+    if (type == PI_TYPE_BF16) hipLaunchKernelGGL(moe_combine_kernel<bf16>, grid, dim3(256), 0, (hipStream_t)stream, x, mix, (const bf16 *)y, inv, weights, n_top, cols, out, keep);
+    else hipLaunchKernelGGL(moe_combine_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream, x, mix, (const float *)y, inv, weights, n_top, cols, out, keep);
     return pi::check_launch("pi_k_moe_combine");
 }
 

@@ -20,6 +20,11 @@ struct KvCells {
         pos.assign(n, -1); seq.assign(n, 0u); delta.assign(n, 0);
         edited = ~0u;
     }
+    void grow(int n_cells) {                       // further free cells behind the ones there are
+        n = n_cells;
+        pos.resize(n, -1); seq.resize(n, 0u); delta.resize(n, 0);
+        edited = ~0u;
+    }
     void take(int cell, int32_t p, uint32_t seqs) {
         if (pos[cell] < 0) ++n_used;
         pos[cell] = p;

@@ -5,7 +5,6 @@
 namespace {
 
 typedef __bf16 bf16;
-typedef __bf16 pi_b8 __attribute__((ext_vector_type(8)));
 
 __device__ __forceinline__ float bf16_to_f32(uint16_t b) { return __uint_as_float((uint32_t)b << 16); }
 template <typename ST> __device__ __forceinline__ ST to_st(float v) { return (ST)v; }           // bf16: round to nearest even
@@ -33,7 +32,7 @@ template <> __device__ __forceinline__ Frag<float> frag_weights<float>(const uin
     return f;
 }
 __device__ __forceinline__ pi_f4 mfma_bf16(const pi_u32x4 & a, const pi_u32x4 & b, pi_f4 c) {
-    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(pi_b8, a), __builtin_bit_cast(pi_b8, b), c, 0, 0, 0);
+    return mma16<bf16>(a, b, c);
 }
 __device__ __forceinline__ void frag_mma(const Frag<bf16> & a, const Frag<bf16> & b, pi_f4 & c) { c = mfma_bf16(a.v, b.v, c); }
 // the k index within a step is free as long as both operands agree: instruction j takes columns 8 g + j of the four lane groups

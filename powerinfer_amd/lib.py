@@ -27,7 +27,8 @@ class GroupGemm(C.Structure):
     _fields_ = [("W", _vp), ("w_gs", _sz), ("rows", C.c_int32), ("cols", C.c_int32), ("ldw", C.c_int32), ("n_group", C.c_int32),
                 ("x", _vp), ("x_gs", _sz), ("ldx", C.c_int32), ("T", C.c_int32),
                 ("y", _vp), ("y_gs", _sz), ("ldy", C.c_int32), ("y_f32", C.c_int32), ("relu2", C.c_int32),
-                ("alpha", _f), ("off", _vp), ("gather", _vp), ("gather_div", C.c_int32)]
+                ("alpha", _f), ("off", _vp), ("gather", _vp), ("gather_div", C.c_int32),
+                ("tiles", _vp), ("n_tiles", _vp), ("max_tiles", C.c_int32)]
 
 
 class LatentPrep(C.Structure):
@@ -62,6 +63,7 @@ _SIGS = {
     "pi_memcpy_d2d": (_i, [_vp, _vp, _sz]),
     "pi_sync": (_i, []),
     "pi_fill_normal_f16": (_i, [_vp, _sz, _u64, _f, _vp, _i, _vp]),
+    "pi_fill_normal_bf16": (_i, [_vp, _sz, _u64, _f, _vp]),
     "pi_fill_normal_q4_0": (_i, [_vp, _sz, _u64, _f, _vp]),
     "pi_event_create": (_vp, []),
     "pi_event_record": (_i, [_vp, _vp]),
@@ -100,10 +102,12 @@ _SIGS = {
     "pi_k_sparse_axpy_dense": (_i, [_vp, _i, _i, _vp, _vp, _i, _vp, _vp, _vp, _vp, _vp]),
     "pi_k_norm_round_f16": (_i, [_vp, _i, _i, C.POINTER(Norm), _vp, _vp, _vp]),
     "pi_k_gemm_f16": (_i, [_vp, _i, _i, _vp, _i, _i, _vp, _vp, _vp, _vp, _vp]),
+    "pi_k_gemm_bf16": (_i, [_vp, _i, _i, _vp, _i, _i, _vp, _vp, _vp, _vp, _vp]),
     "pi_k_batch_predictor_fc2": (_i, [_vp, _i, _i, _vp, _i, _f, _vp, _vp, _vp]),
     "pi_k_batch_sparse_ffn": (_i, [_vp, _i, _i, _f, _vp, _vp, _vp, _i, _vp, _i, _vp, _vp, _vp, _vp, _vp, _vp, _vp]),
     "pi_k_norm_round_f16_ol": (_i, [_vp, _i, _i, C.POINTER(Norm), _vp, _vp, _vp]),
     "pi_k_gemm_f16_ol": (_i, [_vp, _i, _i, _vp, _i, _i, _vp, _vp, _vp, _vp, _vp]),
+    "pi_k_gemm_bf16_ol": (_i, [_vp, _i, _i, _vp, _i, _i, _vp, _vp, _vp, _vp, _vp]),
     "pi_k_batch_predictor_fc2_ol": (_i, [_vp, _i, _i, _vp, _i, _f, _vp, _vp, _vp]),
     "pi_k_batch_sparse_ffn_ol": (_i, [_vp, _i, _i, _f, _vp, _vp, _vp, _i, _vp, _i, _vp, _vp, _vp, _vp, _vp, _vp, _vp]),
     "pi_k_batch_union_count": (_i, [_i, _vp, _vp, _vp, _vp]),
@@ -113,6 +117,7 @@ _SIGS = {
     "pi_k_gemm_q4_t16": (_i, [_vp, _vp, _i, _i, _vp, _vp, _vp, _i, _i, _vp, _vp, _vp, _vp]),
     "pi_k_batch_sparse_ffn_q4": (_i, [_vp, _i, _i, _f, _vp, _vp, _vp, _vp, _vp, _vp, _i, _vp, _vp, _vp, _i, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp]),
     "pi_k_gemm_tile_f16": (_i, [_vp, _i, _i, _vp, _i, _i, _vp, _vp, _vp, _vp, _i, _vp]),
+    "pi_k_gemm_tile_bf16": (_i, [_vp, _i, _i, _vp, _i, _i, _vp, _vp, _vp, _vp, _i, _vp]),
     "pi_k_ffn_h_f16": (_i, [_vp, _vp, _vp, _f, _i, _i, _vp, _vp]),
     "pi_k_transpose_f16": (_i, [_vp, _i, _i, _vp, _vp]),
     "pi_k_norm_q8_round_f16": (_i, [_vp, _i, _i, C.POINTER(Norm), _vp, _vp, _vp]),
@@ -135,6 +140,7 @@ _SIGS = {
     "pi_gemm_lib_create": (_vp, [C.c_size_t]),
     "pi_gemm_lib_destroy": (_i, [_vp]),
     "pi_gemm_lib_f16": (_i, [_vp, _vp, _i, _i, _vp, _i, _i, _vp, _vp, _vp, _vp, _vp]),
+    "pi_gemm_lib_bf16": (_i, [_vp, _vp, _i, _i, _vp, _i, _i, _vp, _vp, _vp, _vp, _vp]),
     "pi_k_batch_sparse_mul_mat": (_i, [_vp, _i, _i, _vp, _i, _vp, _f, _vp, _vp, _vp, _vp, _vp]),
     "pi_k_batch_sparse_axpy": (_i, [_vp, _i, _i, _vp, _vp, _i, _f, _vp, _vp, _vp, _vp, _vp]),
     "pi_k_attn_split_supported": (_i, [_i, _i, _i]),
@@ -164,6 +170,7 @@ _SIGS = {
     "pi_k_embed_norm": (_i, [_vp, _i, _vp, _i, _vp, _f, _vp, _vp]),
     "pi_k_norm_pair": (_i, [_i, _vp, _vp, _i, _i, _f, _vp, _vp, _vp, _vp, _i, _i, _vp]),
     "pi_k_group_gemm": (_i, [_i, C.POINTER(GroupGemm), _vp]),
+    "pi_k_group_gemm_tile": (_i, [C.POINTER(GroupGemm), _i, _vp]),
     "pi_k_rope_angles": (_i, [_vp, _i, _i, C.c_double, _vp, _vp]),
     "pi_k_latent_prep": (_i, [_i, C.POINTER(LatentPrep), _vp]),
     "pi_k_latent_attn_rows": (_i, [_i]),
@@ -172,8 +179,8 @@ _SIGS = {
     "pi_k_latent_attn": (_i, [_i, C.POINTER(LatentAttn), _vp]),
     "pi_k_latent_shift": (_i, [_i, _vp, _i, _i, _i, _i, C.c_double, _vp, _vp]),
     "pi_k_route": (_i, [_vp, _i, _i, _i, _i, _i, _vp, _vp, _vp, _vp]),
-    "pi_k_moe_sort": (_i, [_vp, _i, _i, _vp, _vp, _vp, _vp]),
-    "pi_k_moe_combine": (_i, [_vp, _vp, _vp, _vp, _vp, _i, _i, _i, _vp, _vp, _vp]),
+    "pi_k_moe_sort": (_i, [_vp, _i, _i, _vp, _vp, _vp, _i, _vp, _vp, _vp]),
+    "pi_k_moe_combine": (_i, [_i, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _vp, _vp, _vp]),
     "pi_k_pad_cols_bf16": (_i, [_vp, C.c_int64, _i, _vp, _i, _vp]),
     "pi_k_transpose_pad_bf16": (_i, [_vp, _i, _i, _i, _vp, _i, _vp]),
     "pi_k_cells_advance": (_i, [_i, _vp, _vp, _sz, _vp, _vp, _vp, _vp]),
