@@ -320,6 +320,9 @@ PI_API int pi_k_gemm_f16_ol(const void * W_f16, int rows, int cols, const void *
                             const float * add1, const float * add2, float * y, void * y_ol, pi_stream_t stream);
 PI_API int pi_k_gemm_bf16_ol(const void * W_bf16, int rows, int cols, const void * xn_ol, int T, int epilogue,
                              const float * add1, const float * add2, float * y, void * y_ol, pi_stream_t stream);      /* bf16 weights and activations */
+/* y = W xn and y2 = W2 xn2 in one launch (cols % 256 == 0), bf16, operand layout */
+PI_API int pi_k_gemm_bf16_ol_two(const void * W, int rows, const void * xn_ol, float * y, const void * W2, int rows2, const void * xn2_ol, float * y2,
+                                 int cols, int T, pi_stream_t stream);
 PI_API int pi_k_batch_predictor_fc2_ol(const void * fc2_f16, int ff, int r, const void * hidden_ol, int T, float threshold, float * logits,
                                        pi_workspace * ws, pi_stream_t stream);
 PI_API int pi_k_batch_sparse_ffn_ol(const float * logits, int T, int ff, float threshold,
@@ -631,6 +634,24 @@ PI_API int pi_k_moe_sort(const int32_t * ids, int n_pairs, int n_expert, int32_t
  * (optional) receives a copy */
 PI_API int pi_k_moe_combine(int type, const float * x, const float * mix, const void * y, const int32_t * inv, const float * weights, int n_top, int T,
                             int cols, float * out, float * keep, pi_stream_t stream);
+/* Steps of up to 16 tokens (bf16; pi_k_layer_step_supported).  pi_k_latent_step: pi_k_latent_prep, the absorbed queries (uk_t
+ * [n_head][kv_rank][dim_ld]; p->q_un is not used) and, with ids != NULL, pi_k_route in one launch.  pi_k_latent_value_step: the merge of
+ * a split attention (or its whole result) and the value expansion, att [T][ld_att]; pi_k_latent_attn_parts leaves the parts unmerged.
+ * pi_k_expert_up_step: act [T * top][ld_act] = weight * relu(up[e] x)^2 for every (token, choice).  pi_k_layer_out_step: what closes the
+ * layer, out = x + (wo att + sum over the pairs of a token of down[e] act[pair]); ids == NULL: no experts. */
+typedef struct pi_layer_out {
+    const float * x; const void * wo, * att; int32_t rows, ld_att, T;
+    const void * down, * act; const int32_t * ids; int32_t ld_act, top, n_expert;
+    float * out, * keep;
+} pi_layer_out;
+PI_API int pi_k_layer_step_supported(int T, int n_expert, int n_top);
+PI_API int pi_k_latent_step(const pi_latent_prep * p, const void * uk_t, const float * z_router, int n_expert, int n_top, int n_group, int n_keep, const float * bias,
+                            int32_t * ids, float * weights, pi_stream_t stream);
+PI_API int pi_k_latent_attn_parts(const pi_latent_attn * p, pi_stream_t stream);
+PI_API int pi_k_latent_value_step(const pi_latent_attn * p, const void * uv, int vdim, void * att, int ld_att, pi_stream_t stream);
+PI_API int pi_k_expert_up_step(const void * up, int n_expert, int ff, int cols, const void * x_ol, const int32_t * ids, const float * weights, int T, int top, void * act,
+                               int ld_act, pi_stream_t stream);
+PI_API int pi_k_layer_out_step(const pi_layer_out * a, pi_stream_t stream);
 /* BF16 matrices: out [rows][ld] = in [rows][cols] padded with zeros; out [n_mat][cols][ld] = each in [rows][cols] transposed, padded with zeros */
 PI_API int pi_k_pad_cols_bf16(const void * in, int64_t rows, int cols, void * out, int ld, pi_stream_t stream);
 PI_API int pi_k_transpose_pad_bf16(const void * in, int n_mat, int rows, int cols, void * out, int ld, pi_stream_t stream);

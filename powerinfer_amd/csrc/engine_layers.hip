@@ -272,6 +272,26 @@ int grouped(LayerState * s, const pi_group_gemm & g, int tile_n, hipStream_t st)
     return bf16_mode(s) && g.T > 16 ? pi_k_group_gemm_tile(&g, tile_n, st) : pi_k_group_gemm(s->opts.compute, &g, st);
 }
 
+pi_latent_prep prep_args(pi_model * m, const Layer & L, const Step & in) {
+    LayerState * s = m->lay;
+    const pi_layer_desc & d = L.d;
+    pi_latent_prep p{};
+    p.z = s->z; p.ldz = L.z_rows; p.T = in.T; p.n_head = d.n_head; p.dim = d.dim; p.dim_ld = L.dim_ld; p.rot_dim = d.rot_dim; p.kv_rank = d.kv_rank;
+    p.rank_ld = L.rank_ld; p.kd = L.kd; p.cs = s->cs[L.rot]; p.norm_w = L.dkv_norm; p.eps = m->hp.norm_eps; p.q_un = s->q_un; p.q_lat = s->q_lat;
+    p.cache = L.own_kv ? L.cache : nullptr; p.cell = in.cell;
+    return p;
+}
+
+pi_latent_attn attn_args(pi_model * m, const Layer & L, const Layer & src, const Step & in) {
+    LayerState * s = m->lay;
+    const pi_layer_desc & d = L.d;
+    pi_latent_attn a{};
+    a.q_lat = s->q_lat; a.cache = src.cache; a.lists = s->lists; a.list_ld = s->kv.n; a.work = bf16_mode(s) ? in.work[L.hc].items : in.seq; a.n_vis = in.n_vis;
+    a.n_work = in.work[L.hc].n; a.T = in.T; a.n_head = d.n_head; a.kv_rank = d.kv_rank; a.rank_ld = L.rank_ld; a.kd = L.kd; a.n_parts = in.work[L.hc].parts; a.scale = d.scale;
+    a.sink = L.sink; a.scratch = s->scratch; a.out_lat = s->o_lat;
+    return a;
+}
+
 int mix_latent(pi_model * m, Layer & L, const Step & in) {
     LayerState * s = m->lay;
     const pi_layer_desc & d = L.d;
@@ -279,19 +299,13 @@ int mix_latent(pi_model * m, Layer & L, const Step & in) {
     hipStream_t st = m->stream;
     Layer & src = L.own_kv ? L : s->layers[d.kv_from];
     PI_TRY(dense(m, L.w_z, L.z_rows, s->d_ld, s->h_a, T, s->z));
-    pi_latent_prep p{};
-    p.z = s->z; p.ldz = L.z_rows; p.T = T; p.n_head = d.n_head; p.dim = d.dim; p.dim_ld = L.dim_ld; p.rot_dim = d.rot_dim; p.kv_rank = d.kv_rank;
-    p.rank_ld = L.rank_ld; p.kd = L.kd; p.cs = s->cs[L.rot]; p.norm_w = L.dkv_norm; p.eps = m->hp.norm_eps; p.q_un = s->q_un; p.q_lat = s->q_lat;
-    p.cache = L.own_kv ? L.cache : nullptr; p.cell = in.cell;
+    const pi_latent_prep p = prep_args(m, L, in);
     PI_TRY(pi_k_latent_prep(type, &p, st));
     pi_group_gemm g{};                              // each head's query in latent coordinates
     g.W = L.uk_t; g.w_gs = (size_t)d.kv_rank * L.dim_ld; g.rows = d.kv_rank; g.cols = L.dim_ld; g.ldw = L.dim_ld; g.n_group = d.n_head; g.alpha = 1.0f;
     g.x = s->q_un; g.x_gs = L.dim_ld; g.ldx = d.n_head * L.dim_ld; g.T = T; g.y = s->q_lat; g.y_gs = L.kd; g.ldy = d.n_head * L.kd;
     PI_TRY(grouped(s, g, T > 64 ? 128 : 64, st));
-    pi_latent_attn a{};
-    a.q_lat = s->q_lat; a.cache = src.cache; a.lists = s->lists; a.list_ld = s->kv.n; a.work = bf16_mode(s) ? in.work[L.hc].items : in.seq; a.n_vis = in.n_vis;
-    a.n_work = in.work[L.hc].n; a.T = T; a.n_head = d.n_head; a.kv_rank = d.kv_rank; a.rank_ld = L.rank_ld; a.kd = L.kd; a.n_parts = in.work[L.hc].parts; a.scale = d.scale;
-    a.sink = L.sink; a.scratch = s->scratch; a.out_lat = s->o_lat;
+    const pi_latent_attn a = attn_args(m, L, src, in);
     PI_TRY(pi_k_latent_attn(type, &a, st));
     pi_group_gemm v{};                              // each head's value from its weighted latent
     v.W = L.uv; v.w_gs = (size_t)d.vdim * L.rank_ld; v.rows = d.vdim; v.cols = L.rank_ld; v.ldw = L.rank_ld; v.n_group = d.n_head; v.alpha = 1.0f;
@@ -320,6 +334,29 @@ int ffn_moe(pi_model * m, Layer & L, const Step & in) {
     return grouped(s, w, tile_n, st);
 }
 
+// a layer of a step of up to 16 tokens (bf16): seven launches
+int step_layer(pi_model * m, Layer & L, const Step & in, float * keep) {
+    LayerState * s = m->lay;
+    const pi_layer_desc & d = L.d;
+    const int T = in.T, D = m->hp.n_embd;
+    const bool moe = d.ffn == PI_FFN_MOE;
+    hipStream_t st = m->stream;
+    Layer & src = L.own_kv ? L : s->layers[d.kv_from];
+    PI_TRY(pi_k_norm_pair(PI_TYPE_BF16, s->x, nullptr, T, D, m->hp.norm_eps, L.norm_a, s->h_a, moe ? L.norm_b : nullptr, moe ? s->h_b : nullptr, s->d_ld, 1, st));
+    if (moe) PI_TRY(pi_k_gemm_bf16_ol_two(L.w_z, L.z_rows, s->h_a, s->z, L.router, d.n_expert, s->h_b, s->rl, s->d_ld, T, st));
+    else     PI_TRY(pi_k_gemm_bf16_ol(L.w_z, L.z_rows, s->d_ld, s->h_a, T, PI_EPI_NONE, nullptr, nullptr, s->z, nullptr, st));
+    const pi_latent_prep p = prep_args(m, L, in);
+    PI_TRY(pi_k_latent_step(&p, L.uk_t, s->rl, d.n_expert, d.n_top, d.n_group, d.n_group_keep, L.bias, moe ? s->ids : nullptr, s->wts, st));
+    const pi_latent_attn a = attn_args(m, L, src, in);
+    PI_TRY(pi_k_latent_attn_parts(&a, st));
+    PI_TRY(pi_k_latent_value_step(&a, L.uv, d.vdim, s->att, L.hv_ld, st));
+    if (moe) PI_TRY(pi_k_expert_up_step(L.up, d.n_expert, d.expert_ff, s->d_ld, s->h_b, s->ids, s->wts, T, d.n_top, s->act, L.ff_ld, st));
+    pi_layer_out o{};
+    o.x = s->x; o.wo = L.wo; o.att = s->att; o.rows = D; o.ld_att = L.hv_ld; o.T = T; o.out = s->x2; o.keep = keep;
+    if (moe) { o.down = L.down; o.act = s->act; o.ids = s->ids; o.ld_act = L.ff_ld; o.top = d.n_top; o.n_expert = d.n_expert; }
+    return pi_k_layer_out_step(&o, st);
+}
+
 int pass_layers(pi_model * m, const Step & in) {
     LayerState * s = m->lay;
     const int type = s->opts.compute, T = in.T, D = m->hp.n_embd;
@@ -329,11 +366,16 @@ int pass_layers(pi_model * m, const Step & in) {
     for (size_t il = 0; il < s->layers.size(); ++il) {
         Layer & L = s->layers[il];
         const bool moe = L.d.ffn == PI_FFN_MOE;
+        float * keep = s->streams_T ? s->streams + il * (size_t)s->streams_T * D : nullptr;
+        if (bf16_mode(s) && pi_k_layer_step_supported(T, moe ? L.d.n_expert : 0, moe ? L.d.n_top : 0)) {
+            PI_TRY(step_layer(m, L, in, keep));
+            std::swap(s->x, s->x2);
+            continue;
+        }
         PI_TRY(pi_k_norm_pair(type, s->x, nullptr, T, D, m->hp.norm_eps, L.norm_a, s->h_a, moe ? L.norm_b : nullptr, moe ? s->h_b : nullptr, s->d_ld, 0, st));
         PI_TRY(mix_latent(m, L, in));
         if (moe) PI_TRY(ffn_moe(m, L, in));
-        PI_TRY(pi_k_moe_combine(type, s->x, s->mix, s->y_exp, s->inv, moe ? s->wts : nullptr, moe ? L.d.n_top : 0, T, D, s->x2,
-                                s->streams_T ? s->streams + il * (size_t)s->streams_T * D : nullptr, st));
+        PI_TRY(pi_k_moe_combine(type, s->x, s->mix, s->y_exp, s->inv, moe ? s->wts : nullptr, moe ? L.d.n_top : 0, T, D, s->x2, keep, st));
         std::swap(s->x, s->x2);
     }
     return PI_OK;
@@ -343,7 +385,9 @@ int pass_layers(pi_model * m, const Step & in) {
 int pass_head(pi_model * m, const int32_t * rows, int n) {
     LayerState * s = m->lay;
     const int D = m->hp.n_embd;
-    PI_TRY(pi_k_norm_pair(s->opts.compute, s->x, rows, n, D, m->hp.norm_eps, s->out_norm, s->h_head, nullptr, nullptr, s->d_ld, 0, m->stream));
+    const bool ol = bf16_mode(s) && n <= 16;
+    PI_TRY(pi_k_norm_pair(s->opts.compute, s->x, rows, n, D, m->hp.norm_eps, s->out_norm, s->h_head, nullptr, nullptr, s->d_ld, ol, m->stream));
+    if (ol) return pi_k_gemm_bf16_ol(s->head, m->hp.n_vocab, s->d_ld, s->h_head, n, PI_EPI_NONE, nullptr, nullptr, s->logits, nullptr, m->stream);
     return dense(m, s->head, m->hp.n_vocab, s->d_ld, s->h_head, n, s->logits);
 }
 
@@ -478,7 +522,7 @@ int layers_finalize(pi_model * m) {
     PI_HIP_TRY(hipEventCreate(&m->ev0));
     PI_HIP_TRY(hipEventCreate(&m->ev1));
     s->es = bf16_mode(s) ? 2 : 4;
-    s->d_ld = up_to(D, 128);
+    s->d_ld = up_to(D, 256);
     PI_TRY(want_tensor(m->glob[PI_T_TOK_EMBD], PI_TYPE_BF16, D, m->hp.n_vocab, "tok_embd"));
     PI_TRY(want_tensor(m->glob[PI_T_OUTPUT], PI_TYPE_BF16, D, m->hp.n_vocab, "output"));
     PI_TRY(want_tensor(m->glob[PI_T_OUTPUT_NORM], PI_TYPE_F32, D, 1, "output_norm"));

@@ -184,15 +184,23 @@ __global__ __launch_bounds__(kBlock) void gemm_t16_kernel(const EL * __restrict_
 // row stride (conflict-free both ways) and reads it back in operand layout.  No workgroup barrier is involved: the
 // buffer belongs to one wave and LDS operations of a wave complete in order.  Two 256-column tiles of loads are in flight.
 constexpr int kGlStride = 512 + 16;               // bytes per LDS row: 256 fp16 + one 16-byte pad
+// a second matrix of the same width with its own input and output (no epilogue) in the same launch; rows 0: none
+struct SecondGemm { const void * W; const void * x; int rows; float * y; };
 template <typename EL, int RT, int NW>
 __global__ __launch_bounds__(64 * NW) void gemm_t16_lds_kernel(const EL * __restrict__ W, const EL * __restrict__ xn, int T, int rows, int cols,
                                                                   int epi, const float * __restrict__ add1, const float * __restrict__ add2, float * __restrict__ y,
-                                                                  EL * __restrict__ y16, float thr, unsigned char * __restrict__ row_any, int lay) {
+                                                                  EL * __restrict__ y16, float thr, unsigned char * __restrict__ row_any, int lay, SecondGemm two) {
+    const int n_first = (rows + 16 * RT - 1) / (16 * RT);
+    int bx = blockIdx.x;
+    if (bx >= n_first) {                                // the workgroups behind the first matrix take the second one
+        bx -= n_first;
+        W = (const EL *)two.W; xn = (const EL *)two.x; rows = two.rows; y = two.y;
+    }
     __shared__ __align__(16) unsigned char tile[NW][16 * kGlStride];
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     const int i = lane & 15, g = lane >> 4;
     const int lr = lane >> 5, lc = lane & 31;           // load role: row within the pair, 16-byte chunk within the 512-byte row piece
-    const int row0 = blockIdx.x * 16 * RT;
+    const int row0 = bx * 16 * RT;
     const int tok = i < T ? i : T - 1;
     // the 256-column super-steps of a row are dealt round-robin to the NW waves: wave w takes steps w, w + NW, ...
     const EL * bp = (lay & 1) ? xn + (g * 16 + i) * 8 : xn + (size_t)tok * cols + g * 8;
@@ -1021,7 +1029,7 @@ int pi_k_norm_q8_round_f16(const float * x, int T, int cols, const pi_norm * nor
 // lay bit 0: xn_f16 in the operand layout of the step's activations (pi_ol_index), bit 1: y_f16 written in it
 template <typename EL>
 static int gemm_launch(const char * who, const void * W, int rows, int cols, const void * xn_f16, int T, int epilogue, const float * add1, const float * add2,
-                       float * y, void * y_f16, float thr, unsigned char * row_any, pi_stream_t stream, int lay = 0) {
+                       float * y, void * y_f16, float thr, unsigned char * row_any, pi_stream_t stream, int lay = 0, SecondGemm two = {nullptr, nullptr, 0, nullptr}) {
     if (!W || !xn_f16 || !y || rows <= 0) return pi::fail(PI_E_ARG, who);
     if (T < 1 || T > kBtMaxT || cols <= 0 || cols % 128) return pi::fail(PI_E_ARG, "batched mat-mul: 1 <= T <= 16 and cols % 128 == 0 required");
     if (epilogue < 0 || epilogue > PI_EPI_ADD2 || (epilogue >= PI_EPI_ADD && !add1) || (epilogue == PI_EPI_ADD2 && !add2))
@@ -1030,8 +1038,8 @@ static int gemm_launch(const char * who, const void * W, int rows, int cols, con
     const int rt = rows >= 16384 ? 4 : rows >= 5120 ? 2 : 1;      // (two tiles already at 5120 rows: the activations, re-read per row tile, are what limits one tile per wave)
 #define PI_GEMM_T16(RT) hipLaunchKernelGGL((gemm_t16_kernel<EL, RT>), dim3((rows + 16 * RT - 1) / (16 * RT)), dim3(kBlock), 0, (hipStream_t)stream, \
                        (const EL *)W, (const EL *)xn_f16, T, rows, cols, epilogue, add1, add2, y, (EL *)y_f16, thr, row_any, lay)
-#define PI_GEMM_LDS(RT, NW) hipLaunchKernelGGL((gemm_t16_lds_kernel<EL, RT, NW>), dim3((rows + 16 * RT - 1) / (16 * RT)), dim3(64 * NW), 0, (hipStream_t)stream, \
-                       (const EL *)W, (const EL *)xn_f16, T, rows, cols, epilogue, add1, add2, y, (EL *)y_f16, thr, row_any, lay)
+#define PI_GEMM_LDS(RT, NW) hipLaunchKernelGGL((gemm_t16_lds_kernel<EL, RT, NW>), dim3((rows + 16 * RT - 1) / (16 * RT) + (two.rows + 16 * RT - 1) / (16 * RT)), dim3(64 * NW), 0, (hipStream_t)stream, \
+                       (const EL *)W, (const EL *)xn_f16, T, rows, cols, epilogue, add1, add2, y, (EL *)y_f16, thr, row_any, lay, two)
     if (cols % 256 == 0) {
         // waves per workgroup: when every workgroup has a compute unit to itself (at most one per unit), eight waves keep twice
         // the loads in flight per unit; with more workgroups than units the chip is full with four
@@ -1040,6 +1048,7 @@ static int gemm_launch(const char * who, const void * W, int rows, int cols, con
         if (rtl == 2) { if (wide) PI_GEMM_LDS(2, 8); else PI_GEMM_LDS(2, 4); }
         else { if (wide) PI_GEMM_LDS(1, 8); else PI_GEMM_LDS(1, 4); }
     }
+    else if (two.rows) return pi::fail(PI_E_ARG, "batched mat-mul: two matrices in one launch need cols % 256 == 0");
     else if (rt == 4) PI_GEMM_T16(4); else if (rt == 2) PI_GEMM_T16(2); else PI_GEMM_T16(1);
 #undef PI_GEMM_LDS
 #undef PI_GEMM_T16
@@ -1068,6 +1077,13 @@ int pi_k_gemm_bf16_ol(const void * W, int rows, int cols, const void * xn_ol, in
                       float * y, void * y_ol, pi_stream_t stream) {
     if (y_ol && rows % 8) return pi::fail(PI_E_ARG, "pi_k_gemm_bf16_ol: rows % 8 == 0 required for the bf16 copy in the operand layout");
     return gemm_launch<__bf16>("pi_k_gemm_bf16_ol", W, rows, cols, xn_ol, T, epilogue, add1, add2, y, y_ol, 0.0f, nullptr, stream, 3);
+}
+
+int pi_k_gemm_bf16_ol_two(const void * W, int rows, const void * xn_ol, float * y, const void * W2, int rows2, const void * xn2_ol, float * y2, int cols, int T,
+                          pi_stream_t stream) {
+    if (!W2 || !xn2_ol || !y2 || rows2 <= 0 || cols % 256) return pi::fail(PI_E_ARG, "pi_k_gemm_bf16_ol_two: bad arguments (cols % 256 == 0)");
+    return gemm_launch<__bf16>("pi_k_gemm_bf16_ol_two", W, rows, cols, xn_ol, T, PI_EPI_NONE, nullptr, nullptr, y, nullptr, 0.0f, nullptr, stream, 3,
+                               SecondGemm{W2, xn2_ol, rows2, y2});
 }
 
 }  // extern "C"

@@ -322,21 +322,35 @@ int pi_k_latent_attn_supported(int type, int rank_ld, int kd) {
 
 size_t pi_k_latent_attn_scratch_floats(int T, int n_head, int rank_ld, int n_parts) { return n_parts > 1 ? (size_t)T * n_head * n_parts * (rank_ld + 2) : 0; }
 
-int pi_k_latent_attn(int type, const pi_latent_attn * p, pi_stream_t stream) {
+static int attn_bf16(const pi_latent_attn * p, hipStream_t st) {
+    if (p->rank_ld <= 128 && p->kd <= 256) return launch_attn<2, 2, 4>(p, st);
+    if (p->rank_ld <= 256 && p->kd <= 384) return launch_attn<2, 4, 6>(p, st);
+    if (p->rank_ld <= 512 && p->kd <= 640) return launch_attn<2, 8, 10>(p, st);
+    return launch_attn<2, 16, 18>(p, st);
+}
+
+static int attn_check(int type, const pi_latent_attn * p) {
     if (!p || !p->q_lat || !p->cache || !p->lists || !p->work || !p->n_vis || !p->sink || !p->out_lat || p->n_work <= 0 || p->T <= 0 || p->n_head <= 0 ||
         p->n_parts <= 0 || p->n_parts > 65535 || (p->n_parts > 1 && !p->scratch) || p->kv_rank > p->rank_ld)
         return pi::fail(PI_E_ARG, "pi_k_latent_attn: bad arguments");
     if (!pi_k_latent_attn_supported(type, p->rank_ld, p->kd)) return pi::fail(PI_E_UNSUPPORTED, "pi_k_latent_attn: latent sizes (rank up to 1024)");
+    return PI_OK;
+}
+
+int pi_k_latent_attn_parts(const pi_latent_attn * p, pi_stream_t stream) {
+    const int rc = attn_check(PI_TYPE_BF16, p);
+    return rc != PI_OK ? rc : attn_bf16(p, (hipStream_t)stream);
+}
+
+int pi_k_latent_attn(int type, const pi_latent_attn * p, pi_stream_t stream) {
+    int rc = attn_check(type, p);
+    if (rc != PI_OK) return rc;
     hipStream_t st = (hipStream_t)stream;
     if (type == PI_TYPE_F32) {
         hipLaunchKernelGGL(latent_attn_f32_kernel, dim3(p->T * p->n_head), dim3(256), sizeof(float) * (p->kd + kLfCells) + sizeof(int) * kLfCells, st, *p);
         return pi::check_launch("pi_k_latent_attn");
     }
-    int rc;
-    if (p->rank_ld <= 128 && p->kd <= 256) rc = launch_attn<2, 2, 4>(p, st);
-    else if (p->rank_ld <= 256 && p->kd <= 384) rc = launch_attn<2, 4, 6>(p, st);
-    else if (p->rank_ld <= 512 && p->kd <= 640) rc = launch_attn<2, 8, 10>(p, st);
-    else rc = launch_attn<2, 16, 18>(p, st);
+    rc = attn_bf16(p, st);
     if (rc != PI_OK || p->n_parts == 1) return rc;
     hipLaunchKernelGGL(latent_merge_kernel, dim3(p->T * p->n_head), dim3(128), 0, st, *p);
     return pi::check_launch("pi_k_latent_attn merge");

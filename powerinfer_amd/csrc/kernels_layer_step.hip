@@ -1,0 +1,326 @@
+// Steps of up to 16 tokens of a model described layer by layer (bf16), as few launches as its dependencies allow: everything behind
+// the joint projection (absorbed queries, rotation, cells, expert choice) in one, the merge of a split attention with the value
+// expansion in one, the experts' first matrices in one, and one for what closes a layer - attention output and the experts' second
+// matrices as a single long dot product per row, plus the residual.
+#include "layer_types.hpp"
+#include "route.hpp"
+
+namespace {
+
+// Behind the joint projection: per head the absorbed query (64 latent rows a workgroup), per token the rotated query parts, the cell,
+// and the expert choice.
+__global__ __launch_bounds__(256) void latent_step_kernel(pi_latent_prep p, const uint16_t * __restrict__ uk_t, RouteArgs r, int n_absorb) {
+    extern __shared__ __align__(16) float sm[];
+    __shared__ double red[4];
+    const int hd = p.dim + p.rot_dim, half = p.rot_dim / 2, tid = threadIdx.x;
+    int b = blockIdx.x;
+    if (b < n_absorb) {                                       // a head's query in latent coordinates: 64 rows of W_uk^T against the step's tokens
+        const int tiles = (p.kv_rank + 63) / 64, h = b / tiles, wave = tid >> 6, lane = tid & 63, i = lane & 15, g = lane >> 4;
+        const int row0 = (b % tiles) * 64 + wave * 16;
+        if (row0 >= p.kv_rank) return;
+        const uint16_t * W = uk_t + ((size_t)h * p.kv_rank + min(row0 + i, p.kv_rank - 1)) * p.dim_ld + g * 8;
+        const float * z = p.z + (size_t)min(i, p.T - 1) * p.ldz + h * hd;
+        pi_f4 acc = pi_f4{0, 0, 0, 0};
+        for (int k = 0; k < p.dim_ld; k += 32) {
+            const pi_u32x4 a = pi_ld16(W + k);
+            bf16 q[8];
+#pragma unroll
+            for (int j = 0; j < 8; ++j) { const int c = k + g * 8 + j; q[j] = (bf16)(c < p.dim ? z[c] : 0.0f); }
+            acc = mma16<bf16>(a, __builtin_bit_cast(pi_u32x4, q), acc);
+        }
+        if (i >= p.T) return;
+        bf16 * o = (bf16 *)p.q_lat + ((size_t)i * p.n_head + h) * p.kd + row0 + 4 * g;
+#pragma unroll
+        for (int k = 0; k < 4; ++k) if (row0 + 4 * g + k < p.kv_rank) o[k] = (bf16)acc[k];
+        return;
+    }
+    b -= n_absorb;
+    const int kinds = 1 + (p.cache ? 1 : 0) + (r.ids ? 1 : 0), t = b / kinds, what = b % kinds;
+    const float * z = p.z + (size_t)t * p.ldz;
+    const float2 * cs = (const float2 *)p.cs + (size_t)t * half;
+    if (what == 0) {                                          // rotated query parts
+        for (int e = tid; e < p.n_head * half; e += 256) {
+            const int h = e / half, i = e % half;
+            const float u = z[h * hd + p.dim + 2 * i], v = z[h * hd + p.dim + 2 * i + 1];
+            bf16 * o = (bf16 *)p.q_lat + ((size_t)t * p.n_head + h) * p.kd + p.rank_ld + 2 * i;
+            o[0] = (bf16)(u * cs[i].x - v * cs[i].y);
+            o[1] = (bf16)(v * cs[i].x + u * cs[i].y);
+        }
+    } else if (what == 1 && p.cache) {                        // the token's cell
+        const float * c = z + p.n_head * hd;
+        bf16 * cell = (bf16 *)p.cache + (size_t)p.cell[t] * p.kd;
+        double s = 0.0;
+        for (int i = tid; i < p.kv_rank; i += 256) { const float v = c[i]; s += (double)v * (double)v; }
+        s = block_sum_f64(s, red);
+        const float sc = pi_inv_sqrt((float)(s / p.kv_rank) + p.eps);
+        for (int i = tid; i < p.kv_rank; i += 256) cell[i] = (bf16)(c[i] * sc * p.norm_w[i]);
+        for (int i = tid; i < half; i += 256) {
+            const float u = c[p.kv_rank + 2 * i], v = c[p.kv_rank + 2 * i + 1];
+            cell[p.rank_ld + 2 * i] = (bf16)(u * cs[i].x - v * cs[i].y);
+            cell[p.rank_ld + 2 * i + 1] = (bf16)(v * cs[i].x + u * cs[i].y);
+        }
+    } else if (tid < 64) {                                    // the token's experts
+        route_token(r, t, sm);
+    }
+}
+
+// ---------------------------------------------------------------------------------------------------------------------------------
+// the parts of a split attention merged (fixed order, the sink in the denominator) and the head's values expanded from the result:
+// a workgroup owns 64 value rows of one head, for all tokens of the step
+// ---------------------------------------------------------------------------------------------------------------------------------
+__global__ __launch_bounds__(256) void latent_value_kernel(pi_latent_attn p, const uint16_t * __restrict__ uv, int vdim, bf16 * __restrict__ att, int ld_att) {
+    extern __shared__ __align__(16) unsigned char smem[];
+    const int h = blockIdx.x, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, i = lane & 15, g = lane >> 4;
+    const int ld = p.rank_ld + 8;
+    bf16 * ol = reinterpret_cast<bf16 *>(smem);               // [T][ld]
+    float * f = reinterpret_cast<float *>(smem + (size_t)p.T * ld * 2 + (size_t)(p.T * ld * 2) % 16);      // [T][n_parts] factor of each part
+    const int row0 = blockIdx.y * 64 + wave * 16;
+    // the value matrix does not depend on the attention: its first fragments are requested ahead of everything else
+    const uint16_t * W = uv + ((size_t)h * vdim + min(row0 + i, vdim - 1)) * p.rank_ld + g * 8;
+    pi_u32x4 w0[4];
+#pragma unroll
+    for (int k = 0; k < 4; ++k) w0[k] = k * 32 < p.rank_ld ? pi_ld_stream(W + k * 32) : pi_u32x4{0, 0, 0, 0};
+    if (p.n_parts == 1) {
+        for (int c = tid; c < p.T * (p.rank_ld / 8); c += 256) {
+            const int t = c / (p.rank_ld / 8), k = (c % (p.rank_ld / 8)) * 8;
+            *reinterpret_cast<pi_u32x4 *>(ol + t * ld + k) = pi_ld16((const uint16_t *)p.out_lat + ((size_t)t * p.n_head + h) * p.rank_ld + k);
+        }
+    } else {
+        const float * ml = p.scratch + (size_t)p.T * p.n_head * p.n_parts * p.rank_ld;
+        const float sink = p.sink[h];
+        for (int t = wave; t < p.T; t += 4) {                 // a wave per token: n_parts <= 64 lanes
+            const float2 v = lane < p.n_parts ? reinterpret_cast<const float2 *>(ml)[((size_t)t * p.n_head + h) * p.n_parts + lane] : make_float2(-INFINITY, 0.0f);
+            const float m = fmaxf(pi_wave_max(v.x), sink);
+            const float e = v.x == -INFINITY ? 0.0f : expf(v.x - m);
+            const float l = pi_wave_sum(e * v.y) + expf(sink - m);
+            if (lane < p.n_parts) f[t * p.n_parts + lane] = e / l;
+        }
+        __syncthreads();
+        for (int c = tid; c < p.T * (p.rank_ld / 4); c += 256) {
+            const int t = c / (p.rank_ld / 4), k = (c % (p.rank_ld / 4)) * 4;
+            const float * a = p.scratch + ((size_t)t * p.n_head + h) * p.n_parts * p.rank_ld + k;
+            float4 s = make_float4(0, 0, 0, 0);
+#pragma unroll 8
+            for (int q = 0; q < p.n_parts; ++q) {
+                const float4 v = *reinterpret_cast<const float4 *>(a + (size_t)q * p.rank_ld);
+                const float w = f[t * p.n_parts + q];
+                s.x = fmaf(w, v.x, s.x); s.y = fmaf(w, v.y, s.y); s.z = fmaf(w, v.z, s.z); s.w = fmaf(w, v.w, s.w);
+            }
+            bf16 o[4] = {(bf16)s.x, (bf16)s.y, (bf16)s.z, (bf16)s.w};
+            *reinterpret_cast<pi_u32x2 *>(ol + t * ld + k) = __builtin_bit_cast(pi_u32x2, o);
+        }
+    }
+    __syncthreads();
+    if (row0 >= vdim) return;
+    const bf16 * x = ol + min(i, p.T - 1) * ld + g * 8;
+    pi_f4 acc = pi_f4{0, 0, 0, 0};
+#pragma unroll
+    for (int k = 0; k < 4; ++k)
+        if (k * 32 < p.rank_ld) acc = mma16<bf16>(w0[k], *reinterpret_cast<const pi_u32x4 *>(x + k * 32), acc);
+#pragma unroll 4
+    for (int k = 128; k < p.rank_ld; k += 32) acc = mma16<bf16>(pi_ld_stream(W + k), *reinterpret_cast<const pi_u32x4 *>(x + k), acc);
+    if (i >= p.T) return;
+    bf16 * o = att + (size_t)i * ld_att + h * vdim + row0 + 4 * g;
+#pragma unroll
+    for (int k = 0; k < 4; ++k) if (row0 + 4 * g + k < vdim) o[k] = (bf16)acc[k];
+}
+
+// ---------------------------------------------------------------------------------------------------------------------------------
+// Weight rows streamed past the step's tokens: a wave reads 2 rows x 512 B per load (16 rows x 256 columns in eight), passes them
+// through its own LDS buffer into the matrix cores' operand layout (as gemm_t16_lds_kernel does) and multiplies.  Columns beyond the
+// end of a row are not read (the last piece of the row is read again) and meet zeros.
+// ---------------------------------------------------------------------------------------------------------------------------------
+constexpr int kWsStride = 512 + 16;
+struct WaveStream {
+    unsigned char * tile;
+    int lane, i, g, lr, lc;
+    __device__ __forceinline__ WaveStream(unsigned char * t) : tile(t), lane(threadIdx.x & 63), i(lane & 15), g(lane >> 4), lr(lane >> 5), lc(lane & 31) {}
+    // rows row0 .. row0 + 15 (clamped to rows), columns c0 .. c0 + 255 of a matrix of `cols` (a multiple of 32) columns
+    __device__ __forceinline__ void load(pi_u32x4 (&ld)[8], const bf16 * W, size_t ldw, int row0, int rows, int c0, int cols) const {
+        const int c = min(c0 + lc * 8, cols - 8);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) ld[j] = pi_ld_stream(W + (size_t)min(row0 + 2 * j + lr, rows - 1) * ldw + c);
+    }
+    __device__ __forceinline__ void multiply(const pi_u32x4 (&ld)[8], const pi_u32x4 (&b)[8], pi_f4 & acc) const {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) *reinterpret_cast<pi_u32x4 *>(tile + (2 * j + lr) * kWsStride + lc * 16) = ld[j];
+#pragma unroll
+        for (int st = 0; st < 8; ++st) acc = mma16<bf16>(*reinterpret_cast<const pi_u32x4 *>(tile + i * kWsStride + (4 * st + g) * 16), b[st], acc);
+    }
+};
+
+// The step's distinct experts in LDS: expert[k] in order of first appearance, slot[k][t] = token t's pair with it or -1.
+constexpr int kStepPairs = 256, kStepExperts = 2048;
+struct StepExperts {
+    int first[kStepExperts];
+    int expert[kStepPairs], rank[kStepPairs], sred[16];
+    int16_t slot[kStepPairs][16];
+};
+__device__ int step_experts(StepExperts & s, const int32_t * __restrict__ ids, int n, int top, int E) {
+    const int tid = threadIdx.x, e = tid < n ? ids[tid] : 0;
+    for (int k = tid; k < E; k += blockDim.x) s.first[k] = n;
+    for (int k = tid; k < n * 8; k += blockDim.x) reinterpret_cast<int *>(s.slot)[k] = -1;
+    __syncthreads();
+    if (tid < n) atomicMin(&s.first[e], tid);
+    __syncthreads();
+    const int lead = tid < n ? s.first[e] : -1, own = lead == tid ? 1 : 0;
+    int total;
+    const int rank = block_exclusive_scan_i32(own, &total, s.sred);
+    if (own) { s.expert[rank] = e; s.rank[tid] = rank; }
+    __syncthreads();
+    if (tid < n) s.slot[s.rank[lead]][tid / top] = (int16_t)tid;
+    __syncthreads();
+    return total;
+}
+
+// ---------------------------------------------------------------------------------------------------------------------------------
+// first matrices of the step's experts: workgroup (row tile, pair) works for the pair's expert if no earlier pair has the same one, for
+// every token that chose it; act[pair] = weight * relu(z)^2
+// ---------------------------------------------------------------------------------------------------------------------------------
+template <int NW>
+__global__ __launch_bounds__(64 * NW) void expert_up_step_kernel(const bf16 * __restrict__ up, int ff, int cols, const bf16 * __restrict__ x_ol, const int32_t * __restrict__ ids,
+                                                                 const float * __restrict__ weights, int T, int top, bf16 * __restrict__ act, int ld_act) {
+    __shared__ __align__(16) unsigned char tiles[NW][16 * kWsStride];
+    const int p = blockIdx.y, e = ids[p], tid = threadIdx.x, wave = tid >> 6;
+    if (T > 1 && __syncthreads_or(tid < p && ids[tid] == e)) return;            // p < 64 * NW: checked by the launcher
+    const WaveStream ws(tiles[wave]);
+    const int row0 = blockIdx.x * 16, n_ss = (cols + 255) / 256;
+    const bf16 * W = up + (size_t)e * ff * cols;
+    pi_u32x4 ld[2][8];
+    pi_f4 acc = pi_f4{0, 0, 0, 0};
+    if (wave < n_ss) ws.load(ld[0], W, cols, row0, ff, wave * 256, cols);
+    if (wave + NW < n_ss) ws.load(ld[1], W, cols, row0, ff, (wave + NW) * 256, cols);
+    for (int s0 = wave; s0 < n_ss; s0 += 2 * NW) {
+#pragma unroll
+        for (int b = 0; b < 2; ++b) {
+            const int ss = s0 + b * NW;
+            if (ss < n_ss) {
+                pi_u32x4 x[8];
+#pragma unroll
+                for (int st = 0; st < 8; ++st) x[st] = ss * 256 + st * 32 < cols ? pi_ld16(x_ol + ((size_t)(ss * 8 + st) * 64 + ws.g * 16 + ws.i) * 8) : pi_u32x4{0, 0, 0, 0};
+                ws.multiply(ld[b], x, acc);
+                if (ss + 2 * NW < n_ss) ws.load(ld[b], W, cols, row0, ff, (ss + 2 * NW) * 256, cols);
+            }
+        }
+    }
+    float (*cs)[17] = reinterpret_cast<float (*)[17]>(tiles[wave]);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) cs[4 * ws.g + r][ws.i] = acc[r];
+    __syncthreads();
+    if (tid >= 256) return;
+    const int rr = tid >> 4, t = tid & 15, row = row0 + rr;
+    if (row >= ff || t >= T) return;
+    float v = 0.0f;
+#pragma unroll
+    for (int w = 0; w < NW; ++w) v += reinterpret_cast<float (*)[17]>(tiles[w])[rr][t];
+    v = fmaxf(v, 0.0f);
+    for (int k = 0; k < top; ++k)
+        if (ids[t * top + k] == e) act[(size_t)(t * top + k) * ld_act + row] = (bf16)(weights[t * top + k] * v * v);
+}
+
+// ---------------------------------------------------------------------------------------------------------------------------------
+// what closes a layer: out[t] = x[t] + (W_o att[t] + sum over the token's experts of W_down[e] act[pair]), 16 rows a workgroup.  The
+// pieces of 256 columns of W_o and of every expert of the step form one list that the waves take in turn.
+// ---------------------------------------------------------------------------------------------------------------------------------
+template <int NW>
+__global__ __launch_bounds__(64 * NW) void layer_out_step_kernel(pi_layer_out a) {
+    __shared__ __align__(16) unsigned char tiles[NW][16 * kWsStride];
+    __shared__ StepExperts se;
+    const int tid = threadIdx.x, wave = tid >> 6;
+    const WaveStream ws(tiles[wave]);
+    const int row0 = blockIdx.x * 16, n_o = (a.ld_att + 255) / 256, n_e = a.ids ? (a.ld_act + 255) / 256 : 1;
+    const int tok = min(ws.i, a.T - 1);
+    const bf16 * wo = (const bf16 *)a.wo, * down = (const bf16 *)a.down;
+    pi_u32x4 ld[2][8];
+    pi_f4 acc = pi_f4{0, 0, 0, 0};
+    auto load = [&](pi_u32x4 (&l)[8], int ss) {
+        if (ss < n_o) { ws.load(l, wo, a.ld_att, row0, a.rows, ss * 256, a.ld_att); return; }
+        const int k = (ss - n_o) / n_e, c = (ss - n_o) % n_e;
+        ws.load(l, down + (size_t)se.expert[k] * a.rows * a.ld_act, a.ld_act, row0, a.rows, c * 256, a.ld_act);
+    };
+    // the attention's pieces are requested before the experts are known
+    if (wave < n_o) load(ld[0], wave);
+    if (wave + NW < n_o) load(ld[1], wave + NW);
+    const int n_exp = a.ids ? step_experts(se, a.ids, a.T * a.top, a.top, a.n_expert) : 0, n_ss = n_o + n_exp * n_e;
+    if (wave >= n_o && wave < n_ss) load(ld[0], wave);
+    if (wave + NW >= n_o && wave + NW < n_ss) load(ld[1], wave + NW);
+    for (int s0 = wave; s0 < n_ss; s0 += 2 * NW) {
+#pragma unroll
+        for (int b = 0; b < 2; ++b) {
+            const int ss = s0 + b * NW;
+            if (ss < n_ss) {
+                const bool att = ss < n_o;
+                const int k = att ? 0 : (ss - n_o) / n_e, c = (att ? ss : (ss - n_o) % n_e) * 256, cols = att ? a.ld_att : a.ld_act;
+                const int pair = att ? 0 : se.slot[k][ws.i];
+                const bf16 * xp = att ? (const bf16 *)a.att + (size_t)tok * a.ld_att : (const bf16 *)a.act + (size_t)max(pair, 0) * a.ld_act;
+                pi_u32x4 x[8];
+#pragma unroll
+                for (int st = 0; st < 8; ++st) x[st] = c + st * 32 < cols && pair >= 0 ? pi_ld16(xp + c + st * 32 + ws.g * 8) : pi_u32x4{0, 0, 0, 0};
+                ws.multiply(ld[b], x, acc);
+                if (ss + 2 * NW < n_ss) load(ld[b], ss + 2 * NW);
+            }
+        }
+    }
+    float (*cs)[17] = reinterpret_cast<float (*)[17]>(tiles[wave]);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) cs[4 * ws.g + r][ws.i] = acc[r];
+    __syncthreads();
+    if (tid >= 256) return;
+    const int t = tid >> 4, row = row0 + (tid & 15);
+    if (row >= a.rows || t >= a.T) return;
+    float v = 0.0f;
+#pragma unroll
+    for (int w = 0; w < NW; ++w) v += reinterpret_cast<float (*)[17]>(tiles[w])[tid & 15][t];
+    v += a.x[(size_t)t * a.rows + row];
+    a.out[(size_t)t * a.rows + row] = v;
+    if (a.keep) a.keep[(size_t)t * a.rows + row] = v;
+}
+
+}  // namespace
+
+extern "C" {
+
+int pi_k_layer_step_supported(int T, int n_expert, int n_top) { return T >= 1 && T <= kBtMaxT && n_expert <= kStepExperts && T * n_top <= kStepPairs; }
+
+int pi_k_latent_step(const pi_latent_prep * p, const void * uk_t, const float * z_router, int n_expert, int n_top, int n_group, int n_keep, const float * bias,
+                     int32_t * ids, float * weights, pi_stream_t stream) {
+    if (!p || !p->z || !p->q_lat || !p->cs || !uk_t || p->T <= 0 || p->T > kBtMaxT || p->n_head <= 0 || p->dim <= 0 || p->dim_ld % 32 || p->dim_ld < p->dim || p->rot_dim <= 0 ||
+        p->rot_dim % 2 || p->kv_rank <= 0 || p->rank_ld < p->kv_rank || p->kd < p->rank_ld + p->rot_dim || (p->cache && (!p->cell || !p->norm_w)) ||
+        p->ldz < p->n_head * (p->dim + p->rot_dim) + (p->cache ? p->kv_rank + p->rot_dim : 0))
+        return pi::fail(PI_E_ARG, "pi_k_latent_step: bad arguments");
+    if (ids && (!z_router || !bias || !weights || n_expert <= 0 || n_expert > kStepExperts || n_group <= 0 || n_expert % n_group || n_keep <= 0 || n_keep > n_group || n_top <= 0 ||
+                n_top > n_keep * (n_expert / n_group)))
+        return pi::fail(PI_E_ARG, "pi_k_latent_step: bad routing arguments");
+    const int n_absorb = p->n_head * ((p->kv_rank + 63) / 64), kinds = 1 + (p->cache ? 1 : 0) + (ids ? 1 : 0);
+    hipLaunchKernelGGL(latent_step_kernel, dim3(n_absorb + p->T * kinds), dim3(256), ids ? route_lds_bytes(n_expert, n_group) : 0, (hipStream_t)stream, *p, (const uint16_t *)uk_t,
+                       RouteArgs{z_router, n_expert, n_top, n_group, n_keep, bias, ids, weights}, n_absorb);
+    return pi::check_launch("pi_k_latent_step");
+}
+
+int pi_k_latent_value_step(const pi_latent_attn * p, const void * uv, int vdim, void * att, int ld_att, pi_stream_t stream) {
+    if (!p || !uv || !att || p->T <= 0 || p->T > kBtMaxT || p->n_head <= 0 || vdim <= 0 || p->rank_ld <= 0 || p->rank_ld % 64 || p->rank_ld > 1024 || ld_att < p->n_head * vdim || !p->sink ||
+        p->n_parts <= 0 || p->n_parts > 64 || (p->n_parts == 1 ? !p->out_lat : !p->scratch))
+        return pi::fail(PI_E_ARG, "pi_k_latent_value_step: bad arguments");
+    const size_t lds = (size_t)p->T * (p->rank_ld + 8) * 2 + 16 + sizeof(float) * p->T * p->n_parts;
+    hipLaunchKernelGGL(latent_value_kernel, dim3(p->n_head, (vdim + 63) / 64), dim3(256), lds, (hipStream_t)stream, *p, (const uint16_t *)uv, vdim, (bf16 *)att, ld_att);
+    return pi::check_launch("pi_k_latent_value_step");
+}
+
+int pi_k_expert_up_step(const void * up, int n_expert, int ff, int cols, const void * x_ol, const int32_t * ids, const float * weights, int T, int top, void * act, int ld_act,
+                        pi_stream_t stream) {
+    if (!up || !x_ol || !ids || !weights || !act || n_expert <= 0 || ff <= 0 || cols <= 0 || cols % 32 || T <= 0 || T > kBtMaxT || top <= 0 || T * top > kStepPairs || ld_act < ff)
+        return pi::fail(PI_E_ARG, "pi_k_expert_up_step: bad arguments");
+    hipLaunchKernelGGL(expert_up_step_kernel<4>, dim3((ff + 15) / 16, T * top), dim3(256), 0, (hipStream_t)stream, (const bf16 *)up, ff, cols, (const bf16 *)x_ol, ids, weights, T, top,
+                       (bf16 *)act, ld_act);
+    return pi::check_launch("pi_k_expert_up_step");
+}
+
+int pi_k_layer_out_step(const pi_layer_out * a, pi_stream_t stream) {
+    if (!a || !a->x || !a->wo || !a->att || !a->out || a->rows <= 0 || a->T <= 0 || a->T > kBtMaxT || a->ld_att <= 0 || a->ld_att % 32 ||
+        (a->ids && (!a->down || !a->act || a->ld_act <= 0 || a->ld_act % 32 || a->top <= 0 || a->T * a->top > kStepPairs || a->n_expert <= 0 || a->n_expert > kStepExperts)))
+        return pi::fail(PI_E_ARG, "pi_k_layer_out_step: bad arguments");
+    hipLaunchKernelGGL(layer_out_step_kernel<8>, dim3((a->rows + 15) / 16), dim3(512), 0, (hipStream_t)stream, *a);
+    return pi::check_launch("pi_k_layer_out_step");
+}
+
+}  // extern "C"

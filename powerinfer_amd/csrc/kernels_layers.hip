@@ -3,6 +3,7 @@
 // Templated on the storage of activations: bf16 (matrix cores on bf16 operands, fp32 accumulation) or fp32.
 #include "gemm_tile.hpp"
 #include "layer_types.hpp"
+#include "route.hpp"
 
 namespace {
 
@@ -122,62 +123,10 @@ __global__ void rope_angles_kernel(const int32_t * __restrict__ pos, int T, int 
     cs[idx] = make_float2((float)c, (float)s);
 }
 
-// ---------------------------------------------------------------------------------------------------------------------------------
-// expert choice, one wave per token: scores, choice scores and the groups' sums in LDS, arg-max passes over the lanes (the lower index
-// wins a tie)
-// ---------------------------------------------------------------------------------------------------------------------------------
-__device__ __forceinline__ void wave_argmax(float & v, int & i) {
-#pragma unroll
-    for (int o = 32; o > 0; o >>= 1) {
-        const float ov = __shfl_xor(v, o, PI_WAVE); const int oi = __shfl_xor(i, o, PI_WAVE);
-        if (ov > v || (ov == v && oi < i)) { v = ov; i = oi; }
-    }
-}
-
-__global__ __launch_bounds__(64) void route_kernel(const float * __restrict__ z, int E, int top, int G, int keep, const float * __restrict__ bias,
-                                                   int32_t * __restrict__ ids, float * __restrict__ weights) {
+// expert choice, one wave per token
+__global__ __launch_bounds__(64) void route_kernel(RouteArgs r) {
     extern __shared__ float sm[];
-    float * sc = sm, * ch = sm + E, * gs = sm + 2 * E;        // [E] scores, [E] choice scores, [G] group sums
-    const int t = blockIdx.x, lane = threadIdx.x, size = E / G;
-    for (int e = lane; e < E; e += 64) {
-        const float s = 1.0f / (1.0f + expf(-z[(size_t)t * E + e]));
-        sc[e] = s;
-        ch[e] = s + bias[e];
-    }
-    __syncthreads();
-    if (keep < G) {
-        for (int g = lane; g < G; g += 64) {
-            float a = -INFINITY, b = -INFINITY;
-            for (int k = 0; k < size; ++k) {
-                const float v = ch[g * size + k];
-                if (v > a) { b = a; a = v; } else if (v > b) b = v;
-            }
-            gs[g] = size > 1 ? a + b : a;
-        }
-        __syncthreads();
-        // a group stays if fewer than `keep` groups come before it (larger sum, or the same sum and a lower index)
-        for (int g = lane; g < G; g += 64) {
-            int before = 0;
-            for (int o = 0; o < G; ++o) before += (gs[o] > gs[g] || (gs[o] == gs[g] && o < g)) ? 1 : 0;
-            if (before >= keep) for (int k = 0; k < size; ++k) ch[g * size + k] = -INFINITY;
-        }
-        __syncthreads();
-    }
-    float total = 0.0f;
-    for (int k = 0; k < top; ++k) {
-        float v = -INFINITY; int idx = E;
-        for (int e = lane; e < E; e += 64) {
-            const float c = ch[e];
-            if (c > v || (c == v && e < idx)) { v = c; idx = e; }
-        }
-        wave_argmax(v, idx);
-        if (idx >= E) idx = 0;                                 // not-a-number scores: any expert, never an index outside
-        const float s = sc[idx];
-        total += s;
-        if (lane == 0) { ids[(size_t)t * top + k] = idx; weights[(size_t)t * top + k] = s; ch[idx] = __int_as_float(0x7fc00000); }   // taken: compares false with everything
-        __syncthreads();
-    }
-    for (int k = lane; k < top; k += 64) weights[(size_t)t * top + k] = weights[(size_t)t * top + k] / (total + 1e-20f);
+    route_token(r, blockIdx.x, sm);
 }
 
 // Pairs in expert order, one workgroup with the experts' counters in LDS: counts, their prefix sums, places.  The order of the pairs
@@ -375,10 +324,10 @@ int pi_k_rope_angles(const int32_t * pos, int T, int dims, double base, void * c
 }
 
 int pi_k_route(const float * z, int T, int n_expert, int n_top, int n_group, int n_keep, const float * bias, int32_t * ids, float * weights, pi_stream_t stream) {
-    if (!z || !bias || !ids || !weights || T <= 0 || n_expert <= 0 || n_expert > 8192 || n_top <= 0 || n_group <= 0 || n_expert % n_group || n_keep <= 0 || n_keep > n_group ||
+    if (!z || !bias || !ids || !weights || T <= 0 || n_expert <= 0 || n_expert > 4096 || n_top <= 0 || n_group <= 0 || n_expert % n_group || n_keep <= 0 || n_keep > n_group ||
         n_top > n_keep * (n_expert / n_group))
         return pi::fail(PI_E_ARG, "pi_k_route: bad arguments");
-    hipLaunchKernelGGL(route_kernel, dim3(T), dim3(64), sizeof(float) * (2 * n_expert + n_group), (hipStream_t)stream, z, n_expert, n_top, n_group, n_keep, bias, ids, weights);
+    hipLaunchKernelGGL(route_kernel, dim3(T), dim3(64), route_lds_bytes(n_expert, n_group), (hipStream_t)stream, RouteArgs{z, n_expert, n_top, n_group, n_keep, bias, ids, weights});
     return pi::check_launch("pi_k_route");
 }
 

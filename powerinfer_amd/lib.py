@@ -42,6 +42,12 @@ class LatentAttn(C.Structure):
         ("scale", _f), ("sink", _vp), ("scratch", _vp), ("out_lat", _vp)]
 
 
+class LayerOut(C.Structure):
+    _fields_ = [("x", _vp), ("wo", _vp), ("att", _vp), ("rows", C.c_int32), ("ld_att", C.c_int32), ("T", C.c_int32),
+                ("down", _vp), ("act", _vp), ("ids", _vp), ("ld_act", C.c_int32), ("top", C.c_int32), ("n_expert", C.c_int32),
+                ("out", _vp), ("keep", _vp)]
+
+
 class PiError(RuntimeError):
     pass
 
@@ -181,6 +187,13 @@ _SIGS = {
     "pi_k_route": (_i, [_vp, _i, _i, _i, _i, _i, _vp, _vp, _vp, _vp]),
     "pi_k_moe_sort": (_i, [_vp, _i, _i, _vp, _vp, _vp, _i, _vp, _vp, _vp]),
     "pi_k_moe_combine": (_i, [_i, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _vp, _vp, _vp]),
+    "pi_k_gemm_bf16_ol_two": (_i, [_vp, _i, _vp, _vp, _vp, _i, _vp, _vp, _i, _i, _vp]),
+    "pi_k_layer_step_supported": (_i, [_i, _i, _i]),
+    "pi_k_latent_step": (_i, [C.POINTER(LatentPrep), _vp, _vp, _i, _i, _i, _i, _vp, _vp, _vp, _vp]),
+    "pi_k_latent_attn_parts": (_i, [C.POINTER(LatentAttn), _vp]),
+    "pi_k_latent_value_step": (_i, [C.POINTER(LatentAttn), _vp, _i, _vp, _i, _vp]),
+    "pi_k_expert_up_step": (_i, [_vp, _i, _i, _i, _vp, _vp, _vp, _i, _i, _vp, _i, _vp]),
+    "pi_k_layer_out_step": (_i, [C.POINTER(LayerOut), _vp]),
     "pi_k_pad_cols_bf16": (_i, [_vp, C.c_int64, _i, _vp, _i, _vp]),
     "pi_k_transpose_pad_bf16": (_i, [_vp, _i, _i, _i, _vp, _i, _vp]),
     "pi_k_cells_advance": (_i, [_i, _vp, _vp, _sz, _vp, _vp, _vp, _vp]),
