@@ -621,6 +621,15 @@ PI_API int    pi_k_latent_attn_rows(int type);
 PI_API int    pi_k_latent_attn_supported(int type, int rank_ld, int kd);
 PI_API size_t pi_k_latent_attn_scratch_floats(int T, int n_head, int rank_ld, int n_parts);
 PI_API int    pi_k_latent_attn(int type, const pi_latent_attn * p, pi_stream_t stream);
+/* The same attention for a long run of tokens tok0 .. tok0 + T - 1 of one sequence (ascending n_vis), bf16, over expanded keys [cell][n_head * dim]
+ * and values [cell][n_head * vdim] of the cells list[0 .. n_vis of the last token): att rows get each head's values (pi_k_latent_prep's
+ * q_un and the rotated parts of q_lat are the queries; the shared rotated key part is read from the cells). */
+typedef struct pi_latent_expanded {
+    const void * q_un, * q_lat, * keys, * values, * cache; const int32_t * list, * n_vis; const float * sink; void * att;
+    int32_t tok0, T, n_head, dim, dim_ld, rot_dim, vdim, rank_ld, kd, ld_att; float scale;
+} pi_latent_expanded;
+PI_API int pi_k_latent_expanded_supported(int dim, int rot_dim, int vdim);
+PI_API int pi_k_latent_attn_expanded(const pi_latent_expanded * p, pi_stream_t stream);
 /* rotates the shared key part (rot_dim values behind rank_ld) of cells by delta[cell] positions; cells with delta 0 are left alone */
 PI_API int pi_k_latent_shift(int type, void * cache, int n_cells, int kd, int rank_ld, int rot_dim, double base, const int32_t * delta, pi_stream_t stream);
 /* expert choice of T tokens from router logits z [T][n_expert] (see PI_FFN_MOE): ids, weights [T][n_top] by falling choice score */

@@ -17,6 +17,7 @@ namespace {
 constexpr int kOwnSeq = 31;              // the model's own sequence (pi_model_decode / pi_model_generate)
 constexpr int kHeadRows = 256;           // rows of logits held at a time
 constexpr int kMaxLockstep = 16;
+constexpr long long kExpandedValues = 1LL << 29;      // most expanded key and value numbers of one run (1 GiB)
 constexpr int kItemRows = 32;             // query rows of an attention work item
 constexpr int kAttnItems = 512;          // (work item, part) pairs a split attention aims at: two workgroups per compute unit
 
@@ -24,30 +25,37 @@ int up_to(int v, int m) { return (v + m - 1) / m * m; }
 
 struct Layer {
     pi_layer_desc d{};
-    int nq = 0, z_rows = 0, dim_ld = 0, rank_ld = 0, kd = 0, hv_ld = 0, ff_ld = 0, rot = 0, hc = 0;      // rot, hc: index among the model's rotations / head counts
+    int nq = 0, z_rows = 0, dim_ld = 0, rank_ld = 0, kd = 0, hv_ld = 0, ff_ld = 0, rot = 0, hc = 0;      // rot, hc: index among the model's rotations / kinds of heads
     bool own_kv = true;
-    const void *w_z = nullptr, *uk_t = nullptr, *uv = nullptr, *wo = nullptr, *router = nullptr, *up = nullptr, *down = nullptr;
+    const void *w_z = nullptr, *uk = nullptr, *uk_t = nullptr, *uv = nullptr, *wo = nullptr, *router = nullptr, *up = nullptr, *down = nullptr;
     const float *norm_a = nullptr, *norm_b = nullptr, *dkv_norm = nullptr, *sink = nullptr, *bias = nullptr;
     void * cache = nullptr;
 };
 
 struct Rotation { int dims; double base; };
+struct HeadKind { int n_head, dim, rot_dim, vdim, rank_ld, kd; };
 
 // where a pass finds its tokens
 struct Step {
     int T = 0;
     const int32_t *tokens = nullptr, *pos = nullptr, *cell = nullptr, *n_vis = nullptr, *seq = nullptr;
     struct Work { const int32_t * items = nullptr; int n = 0, parts = 1; };
-    std::vector<Work> work;               // attention work items, per distinct head count of the model
+    struct Run { int tok0, T, seq, n_cells; };
+    // per kind of latent head (distinct sizes of the model's layers): the tokens that attend in latent space as work items, and the long
+    // runs that attend over expanded keys and values
+    std::vector<Work> work;
+    std::vector<std::vector<Run>> runs;
 };
 
 }  // namespace
+
+typedef uint16_t bf16_t;                 // bit patterns
 
 struct LayerState {
     pi_layers_opts opts{};
     std::vector<Layer> layers;
     std::vector<Rotation> rots;
-    std::vector<int> head_counts;
+    std::vector<HeadKind> kinds;
     int d_ld = 0, es = 2;
     const float *embd_norm = nullptr, *out_norm = nullptr;
     const void *embed = nullptr, *head = nullptr;
@@ -63,6 +71,7 @@ struct LayerState {
     void *h_a = nullptr, *h_b = nullptr, *q_un = nullptr, *q_lat = nullptr, *o_lat = nullptr, *att = nullptr, *act = nullptr, *y_exp = nullptr;
     int32_t *ids = nullptr, *perm = nullptr, *inv = nullptr, *off = nullptr, *tiles = nullptr, *n_tiles = nullptr;
     std::vector<float *> cs;                           // per rotation [cap][dims / 2] (cos, sin)
+    bf16_t * expanded = nullptr; size_t expanded_cap = 0;      // keys and values of a long run's cells
     float * scratch = nullptr;                         // partial sums of a split attention
     float * logits = nullptr; void * h_head = nullptr; int32_t * d_next = nullptr;
     int32_t * h_in = nullptr, * d_in = nullptr; size_t in_cap = 0;       // a pass's integers: pinned host side and device side
@@ -161,8 +170,8 @@ int layer_weights(pi_model * m, int il) {
     if (!ukt) return PI_E_HIP;
     PI_TRY(pi_k_transpose_pad_bf16(uk.dev, d.n_head, d.dim, d.kv_rank, ukt, L.dim_ld, nullptr));
     PI_TRY(pi_sync());
-    release(m, uk);
     L.uk_t = ukt;
+    PI_TRY(padded(m, uk, L.rank_ld, &L.uk));         // as it is, for the expanded keys of long prompt portions
     PI_TRY(padded(m, uv, L.rank_ld, &L.uv));
     PI_TRY(want_tensor(m->L(il, PI_T_MIX_SINK), PI_TYPE_F32, d.n_head, 1, "mix_sink"));
     L.sink = (const float *)m->L(il, PI_T_MIX_SINK).dev;
@@ -244,6 +253,22 @@ int ensure_inputs(pi_model * m, size_t n) {
     return PI_OK;
 }
 
+// room for the expanded keys and values of a pass's longest run
+int ensure_expanded(pi_model * m, const Step & in) {
+    LayerState * s = m->lay;
+    size_t need = 0;
+    for (size_t k = 0; k < in.runs.size(); ++k)
+        for (const Step::Run & r : in.runs[k]) need = std::max(need, (size_t)r.n_cells * s->kinds[k].n_head * (s->kinds[k].dim + s->kinds[k].vdim) + 128);
+    if (need <= s->expanded_cap) return PI_OK;
+    PI_HIP_TRY(hipStreamSynchronize(m->stream));
+    if (s->expanded) { pi_free(s->expanded); s->expanded = nullptr; s->expanded_cap = 0; }
+    need += need / 4;                                              // a prompt that grows portion by portion asks again less often
+    s->expanded = (bf16_t *)pi_malloc(need * sizeof(bf16_t));
+    if (!s->expanded) return PI_E_HIP;
+    s->expanded_cap = need;
+    return PI_OK;
+}
+
 // ---- one pass over the layers ----------------------------------------------------------------------------------------------------
 // y [T][rows] = W x, x rows of `cols` values.  bf16: the mat-muls the other models run (steps of up to 16 tokens, LDS tiles, and
 // hipBLASLt plans for large products)
@@ -292,15 +317,11 @@ pi_latent_attn attn_args(pi_model * m, const Layer & L, const Layer & src, const
     return a;
 }
 
-int mix_latent(pi_model * m, Layer & L, const Step & in) {
+int attend_latent(pi_model * m, const Layer & L, const Layer & src, const Step & in) {
     LayerState * s = m->lay;
     const pi_layer_desc & d = L.d;
     const int type = s->opts.compute, T = in.T;
     hipStream_t st = m->stream;
-    Layer & src = L.own_kv ? L : s->layers[d.kv_from];
-    PI_TRY(dense(m, L.w_z, L.z_rows, s->d_ld, s->h_a, T, s->z));
-    const pi_latent_prep p = prep_args(m, L, in);
-    PI_TRY(pi_k_latent_prep(type, &p, st));
     pi_group_gemm g{};                              // each head's query in latent coordinates
     g.W = L.uk_t; g.w_gs = (size_t)d.kv_rank * L.dim_ld; g.rows = d.kv_rank; g.cols = L.dim_ld; g.ldw = L.dim_ld; g.n_group = d.n_head; g.alpha = 1.0f;
     g.x = s->q_un; g.x_gs = L.dim_ld; g.ldx = d.n_head * L.dim_ld; g.T = T; g.y = s->q_lat; g.y_gs = L.kd; g.ldy = d.n_head * L.kd;
@@ -310,7 +331,41 @@ int mix_latent(pi_model * m, Layer & L, const Step & in) {
     pi_group_gemm v{};                              // each head's value from its weighted latent
     v.W = L.uv; v.w_gs = (size_t)d.vdim * L.rank_ld; v.rows = d.vdim; v.cols = L.rank_ld; v.ldw = L.rank_ld; v.n_group = d.n_head; v.alpha = 1.0f;
     v.x = s->o_lat; v.x_gs = L.rank_ld; v.ldx = d.n_head * L.rank_ld; v.T = T; v.y = s->att; v.y_gs = d.vdim; v.ldy = L.hv_ld;
-    PI_TRY(grouped(s, v, T > 64 ? 128 : 64, st));
+    return grouped(s, v, T > 64 ? 128 : 64, st);
+}
+
+// one long run over the expanded keys and values of its cells
+int attend_expanded(pi_model * m, const Layer & L, const Layer & src, const Step & in, const Step::Run & r) {
+    LayerState * s = m->lay;
+    const pi_layer_desc & d = L.d;
+    hipStream_t st = m->stream;
+    const int32_t * list = s->lists + (size_t)r.seq * s->kv.n;
+    const size_t nk = (size_t)d.n_head * d.dim, nv = (size_t)d.n_head * d.vdim, keys = ((size_t)r.n_cells * nk + 127) / 128 * 128;
+    bf16_t * k = s->expanded, * v = s->expanded + keys;
+    pi_group_gemm g{};
+    g.W = L.uk; g.rows = (int)nk; g.cols = L.rank_ld; g.ldw = L.rank_ld; g.n_group = 1; g.x = src.cache; g.ldx = L.kd; g.T = r.n_cells; g.y = k; g.ldy = (int)nk;
+    g.alpha = 1.0f; g.gather = list; g.gather_div = 1;
+    PI_TRY(pi_k_group_gemm_tile(&g, 128, st));
+    g.W = L.uv; g.rows = (int)nv; g.y = v; g.ldy = (int)nv;
+    PI_TRY(pi_k_group_gemm_tile(&g, 128, st));
+    pi_latent_expanded a{};
+    a.q_un = s->q_un; a.q_lat = s->q_lat; a.keys = k; a.values = v; a.cache = src.cache; a.list = list; a.n_vis = in.n_vis; a.sink = L.sink; a.att = s->att;
+    a.tok0 = r.tok0; a.T = r.T; a.n_head = d.n_head; a.dim = d.dim; a.dim_ld = L.dim_ld; a.rot_dim = d.rot_dim; a.vdim = d.vdim; a.rank_ld = L.rank_ld; a.kd = L.kd;
+    a.ld_att = L.hv_ld; a.scale = d.scale;
+    return pi_k_latent_attn_expanded(&a, st);
+}
+
+int mix_latent(pi_model * m, Layer & L, const Step & in) {
+    LayerState * s = m->lay;
+    const pi_layer_desc & d = L.d;
+    const int type = s->opts.compute, T = in.T;
+    hipStream_t st = m->stream;
+    Layer & src = L.own_kv ? L : s->layers[d.kv_from];
+    PI_TRY(dense(m, L.w_z, L.z_rows, s->d_ld, s->h_a, T, s->z));
+    const pi_latent_prep p = prep_args(m, L, in);
+    PI_TRY(pi_k_latent_prep(type, &p, st));
+    if (in.work[L.hc].n > 0) PI_TRY(attend_latent(m, L, src, in));
+    if (bf16_mode(s)) for (const Step::Run & r : in.runs[L.hc]) PI_TRY(attend_expanded(m, L, src, in, r));
     return dense(m, L.wo, m->hp.n_embd, L.hv_ld, s->att, T, s->mix);
 }
 
@@ -347,10 +402,15 @@ int step_layer(pi_model * m, Layer & L, const Step & in, float * keep) {
     else     PI_TRY(pi_k_gemm_bf16_ol(L.w_z, L.z_rows, s->d_ld, s->h_a, T, PI_EPI_NONE, nullptr, nullptr, s->z, nullptr, st));
     const pi_latent_prep p = prep_args(m, L, in);
     PI_TRY(pi_k_latent_step(&p, L.uk_t, s->rl, d.n_expert, d.n_top, d.n_group, d.n_group_keep, L.bias, moe ? s->ids : nullptr, s->wts, st));
+    // the experts' first matrices do not wait for the attention: in the captured loop they run beside it on the second stream
+    const bool fork = moe && m->building_graph;
+    hipStream_t st2 = fork ? m->stream2 : st;
+    if (fork) { PI_HIP_TRY(hipEventRecord(m->ev_fork[0], st)); PI_HIP_TRY(hipStreamWaitEvent(st2, m->ev_fork[0], 0)); }
+    if (moe) PI_TRY(pi_k_expert_up_step(L.up, d.n_expert, d.expert_ff, s->d_ld, s->h_b, s->ids, s->wts, T, d.n_top, s->act, L.ff_ld, st2));
     const pi_latent_attn a = attn_args(m, L, src, in);
     PI_TRY(pi_k_latent_attn_parts(&a, st));
     PI_TRY(pi_k_latent_value_step(&a, L.uv, d.vdim, s->att, L.hv_ld, st));
-    if (moe) PI_TRY(pi_k_expert_up_step(L.up, d.n_expert, d.expert_ff, s->d_ld, s->h_b, s->ids, s->wts, T, d.n_top, s->act, L.ff_ld, st));
+    if (fork) { PI_HIP_TRY(hipEventRecord(m->ev_join[0], st2)); PI_HIP_TRY(hipStreamWaitEvent(st, m->ev_join[0], 0)); }
     pi_layer_out o{};
     o.x = s->x; o.wo = L.wo; o.att = s->att; o.rows = D; o.ld_att = L.hv_ld; o.T = T; o.out = s->x2; o.keep = keep;
     if (moe) { o.down = L.down; o.act = s->act; o.ids = s->ids; o.ld_act = L.ff_ld; o.top = d.n_top; o.n_expert = d.n_expert; }
@@ -401,13 +461,23 @@ int head_buffers(pi_model * m) {
     return pi_memset(s->h_head, 0, (size_t)kHeadRows * s->d_ld * s->es);
 }
 
-// attention work items of n tokens' runs (consecutive tokens of one sequence with ascending cells): appended to `out`
-void work_items(const int32_t * seq, const int32_t * n_vis, int n, int n_head, std::vector<int32_t> & out) {
+// Tokens fall into runs (consecutive, of one sequence, with ascending cells).  A long run pays for expanding its cells' keys and values:
+// per (token, cell) pair and head the latent form multiplies kd + rank_ld numbers, the expanded one dim + rot_dim + vdim, and an
+// expansion costs rank_ld * (dim + vdim) per cell and head.
+bool worth_expanding(const HeadKind & h, int T, int n_cells) {
+    const long long latent = (long long)h.kd + h.rank_ld, expanded = (long long)h.dim + h.rot_dim + h.vdim;
+    return pi_k_latent_expanded_supported(h.dim, h.rot_dim, h.vdim) && T >= 64 && T * (latent - expanded) > (long long)h.rank_ld * (h.dim + h.vdim) &&
+           (long long)n_cells * h.n_head * (h.dim + h.vdim) <= kExpandedValues;
+}
+
+// work items {first token, first row, rows, sequence} of the tokens that attend in latent space, appended to `out`; long runs to `runs`
+void work_items(const int32_t * seq, const int32_t * n_vis, int n, const HeadKind & h, std::vector<int32_t> & out, std::vector<Step::Run> * runs) {
     for (int t0 = 0; t0 < n;) {
         int t1 = t0 + 1;
         while (t1 < n && seq[t1] == seq[t0] && n_vis[t1] >= n_vis[t1 - 1]) ++t1;
-        const int rows = (t1 - t0) * n_head;
-        for (int r = 0; r < rows; r += kItemRows) { out.push_back(t0); out.push_back(r); out.push_back(std::min(kItemRows, rows - r)); out.push_back(seq[t0]); }
+        const int rows = (t1 - t0) * h.n_head;
+        if (runs && worth_expanding(h, t1 - t0, n_vis[t1 - 1])) runs->push_back({t0, t1 - t0, seq[t0], n_vis[t1 - 1]});
+        else for (int r = 0; r < rows; r += kItemRows) { out.push_back(t0); out.push_back(r); out.push_back(std::min(kItemRows, rows - r)); out.push_back(seq[t0]); }
         t0 = t1;
     }
 }
@@ -416,7 +486,7 @@ void work_items(const int32_t * seq, const int32_t * n_vis, int n, int n_head, s
 int choose_parts(LayerState * s, int n_work, int n_vis_max) {
     if (!bf16_mode(s) || n_work <= 0) return 1;
     const int tiles = (n_vis_max + 31) / 32;
-    return std::max(1, std::min({kAttnItems / n_work, tiles / 4, 64}));
+    return std::max(1, std::min({kAttnItems / n_work, tiles, 64}));
 }
 
 // ---- cells -----------------------------------------------------------------------------------------------------------------------
@@ -521,6 +591,10 @@ int layers_finalize(pi_model * m) {
     const int D = m->hp.n_embd;
     PI_HIP_TRY(hipEventCreate(&m->ev0));
     PI_HIP_TRY(hipEventCreate(&m->ev1));
+    PI_HIP_TRY(hipStreamCreateWithFlags(&m->stream2, hipStreamNonBlocking));
+    m->ev_fork.assign(1, nullptr); m->ev_join.assign(1, nullptr);
+    PI_HIP_TRY(hipEventCreateWithFlags(&m->ev_fork[0], hipEventDisableTiming));
+    PI_HIP_TRY(hipEventCreateWithFlags(&m->ev_join[0], hipEventDisableTiming));
     s->es = bf16_mode(s) ? 2 : 4;
     s->d_ld = up_to(D, 256);
     PI_TRY(want_tensor(m->glob[PI_T_TOK_EMBD], PI_TYPE_BF16, D, m->hp.n_vocab, "tok_embd"));
@@ -546,8 +620,9 @@ int layers_finalize(pi_model * m) {
         if (r == s->rots.size()) s->rots.push_back({d.rot_dim, d.rot_base});
         L.rot = (int)r;
         size_t h = 0;
-        while (h < s->head_counts.size() && s->head_counts[h] != d.n_head) ++h;
-        if (h == s->head_counts.size()) s->head_counts.push_back(d.n_head);
+        const HeadKind hk{d.n_head, d.dim, d.rot_dim, d.vdim, L.rank_ld, L.kd};
+        while (h < s->kinds.size() && memcmp(&s->kinds[h], &hk, sizeof hk)) ++h;
+        if (h == s->kinds.size()) s->kinds.push_back(hk);
         L.hc = (int)h;
         scratch = std::max(scratch, pi_k_latent_attn_scratch_floats(pi_k_latent_attn_rows(s->opts.compute) * kAttnItems, 1, L.rank_ld, 2) / 2);
         PI_TRY(layer_weights(m, (int)il));
@@ -562,7 +637,7 @@ int layers_finalize(pi_model * m) {
         if (!*p) return PI_E_HIP;
     }
     size_t items = 0;
-    for (int h : s->head_counts) items += (size_t)kMaxLockstep * ((h + kItemRows - 1) / kItemRows);
+    for (const HeadKind & h : s->kinds) items += (size_t)kMaxLockstep * ((h.n_head + kItemRows - 1) / kItemRows);
     s->g_work = m->alloc<int32_t>(4 * items);
     s->g_out = m->alloc<int32_t>((size_t)s->max_steps * kMaxLockstep);
     if (!s->g_work || !s->g_out) return PI_E_HIP;
@@ -578,6 +653,7 @@ void layers_destroy(pi_model * m) {
     if (s->h_in) (void)hipHostFree(s->h_in);
     if (s->d_in) pi_free(s->d_in);
     if (s->streams) pi_free(s->streams);
+    if (s->expanded) pi_free(s->expanded);
     delete s;
     m->lay = nullptr;
 }
@@ -616,9 +692,10 @@ int layers_step(pi_model * m, const int32_t * tokens, const int32_t * positions,
         in.T = T;
         const int vmax = *std::max_element(vis.begin() + t0, vis.begin() + t0 + T);
         std::vector<size_t> begin;
-        for (int h : s->head_counts) {
+        for (const HeadKind & h : s->kinds) {
             begin.push_back(items.size());
-            if (bf16_mode(s)) work_items(seq.data() + t0, vis.data() + t0, T, h, items);
+            in.runs.emplace_back();
+            if (bf16_mode(s)) work_items(seq.data() + t0, vis.data() + t0, T, h, items, T > 16 ? &in.runs.back() : nullptr);
         }
         begin.push_back(items.size());
         const size_t n_in = (size_t)5 * T + items.size() + rows.size();
@@ -631,7 +708,7 @@ int layers_step(pi_model * m, const int32_t * tokens, const int32_t * positions,
         if (!rows.empty()) memcpy(h + 5 * T + items.size(), rows.data(), 4 * rows.size());
         PI_HIP_TRY(hipMemcpyAsync(s->d_in, h, 4 * n_in, hipMemcpyHostToDevice, m->stream));
         in.tokens = s->d_in; in.pos = s->d_in + T; in.cell = s->d_in + 2 * T; in.n_vis = s->d_in + 3 * T; in.seq = s->d_in + 4 * T;
-        for (size_t k = 0; k < s->head_counts.size(); ++k) {
+        for (size_t k = 0; k < s->kinds.size(); ++k) {
             Step::Work w;
             w.items = s->d_in + 5 * T + begin[k];
             w.n = bf16_mode(s) ? (int)(begin[k + 1] - begin[k]) / 4 : T;
@@ -650,6 +727,7 @@ int layers_step(pi_model * m, const int32_t * tokens, const int32_t * positions,
             }
             s->streams_T = T;
         }
+        PI_TRY(ensure_expanded(m, in));
         PI_TRY(pass_layers(m, in));
         const int32_t * d_rows = s->d_in + 5 * T + items.size();
         for (int r0 = 0; r0 < (int)rows.size(); r0 += kHeadRows) {
@@ -761,10 +839,10 @@ int layers_generate(pi_model * m, int own, int n_steps, int32_t * out_tokens, fl
     Step in;
     in.T = T; in.tokens = s->g_tok; in.pos = s->g_pos; in.cell = s->g_cell; in.n_vis = s->g_vis; in.seq = s->g_seq;
     std::vector<int> parts;
-    for (int h : s->head_counts) {
+    for (const HeadKind & h : s->kinds) {
         Step::Work w;
         const size_t at = items.size();
-        if (bf16_mode(s)) work_items(seq.data(), vis.data(), T, h, items);
+        if (bf16_mode(s)) work_items(seq.data(), vis.data(), T, h, items, nullptr);
         w.items = s->g_work + at;
         w.n = bf16_mode(s) ? (int)(items.size() - at) / 4 : T;
         w.parts = choose_parts(s, w.n, *std::max_element(pos.begin(), pos.end()) + n_steps);
@@ -790,7 +868,9 @@ int layers_generate(pi_model * m, int own, int n_steps, int32_t * out_tokens, fl
     if (use_graph && s->exec && (s->graph_T != T || s->graph_seq0 != q0 || s->graph_parts != parts)) drop_graph(s);
     if (use_graph && !s->exec) {
         PI_HIP_TRY(hipStreamBeginCapture(m->stream, hipStreamCaptureModeThreadLocal));
+        m->building_graph = true;
         const int rc = step();
+        m->building_graph = false;
         hipGraph_t g = nullptr;
         const hipError_t e = hipStreamEndCapture(m->stream, &g);
         if (rc != PI_OK) { if (g) (void)hipGraphDestroy(g); return rc; }

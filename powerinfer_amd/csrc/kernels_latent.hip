@@ -59,13 +59,13 @@ constexpr int kLaRows = 32;
 // B operand of 32 cells x 16 columns from LDS rows of `stride` bytes: lane (column i, cells 8 g ..) - two transposing reads, in each of
 // which sixteen lanes fetch 4 cells x 16 columns and swap them so that every lane ends up with its column's four cells
 typedef short pi_s4 __attribute__((ext_vector_type(4)));
+__device__ __forceinline__ pi_s4 tr_read(const unsigned char * q) {
+    return __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) pi_s4 *)(__attribute__((address_space(3))) void *)q);
+}
 __device__ __forceinline__ pi_u32x4 frag_cells(const unsigned char * rows, int stride, int col) {
     const int lane = threadIdx.x & 63, g = lane >> 4, li = lane & 15;
     const unsigned char * a = rows + (8 * g + (li >> 2)) * stride + (col + (li & 3) * 4) * 2;
-    auto rd = [](const unsigned char * q) {
-        return __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) pi_s4 *)(__attribute__((address_space(3))) void *)q);
-    };
-    const pi_u32x2 lo = __builtin_bit_cast(pi_u32x2, rd(a)), hi = __builtin_bit_cast(pi_u32x2, rd(a + 4 * stride));
+    const pi_u32x2 lo = __builtin_bit_cast(pi_u32x2, tr_read(a)), hi = __builtin_bit_cast(pi_u32x2, tr_read(a + 4 * stride));
     return pi_u32x4{lo.x, lo.y, hi.x, hi.y};
 }
 
@@ -265,6 +265,156 @@ __global__ __launch_bounds__(256) void latent_attn_f32_kernel(pi_latent_attn p) 
     for (int j = 0; j < 4; ++j) { const int k = tid + 256 * j; if (k < p.rank_ld) ((float *)p.out_lat)[(size_t)blockIdx.x * p.rank_ld + k] = acc[j] / l; }
 }
 
+// ---------------------------------------------------------------------------------------------------------------------------------
+// Long prompt portions: keys and values of the visible cells are expanded once (two mat-muls over the cells' latents) and a portion's
+// tokens attend to them head by head.  A workgroup owns 128 tokens of one head; a wave owns 32 of them as columns: scores are formed
+// transposed (keys x tokens), so that a lane's scores belong to one token, its soft-max needs two shuffles, and its weights are already
+// the column operand of the second product (values^T x weights) - which key a slot of that product's inner dimension stands for is free,
+// so the value operand is read in the order the scores came out.  64 keys at a time through LDS, the next 64 in registers.
+// ---------------------------------------------------------------------------------------------------------------------------------
+constexpr int kXKeys = 64, kXTok = 128;
+template <int KS, int VT>              // 32-column steps of a key row (unrotated | rotated, zero padded); 16-column tiles of a value row
+__global__ __launch_bounds__(256, 2) void latent_expanded_attn_kernel(pi_latent_expanded p, int n_qt, int hp) {
+    constexpr int KROW = KS * 64 + 16, VROW = VT * 32 + 16, KP = KS * 4 * kXKeys / 256, VP = VT * 2 * kXKeys / 256;      // bytes per LDS row; pieces per thread
+    __shared__ __align__(16) unsigned char ks[kXKeys * KROW];
+    __shared__ __align__(16) unsigned char vs[kXKeys * VROW];
+    const int xcd = blockIdx.x % 8, slot = blockIdx.x / 8, h = xcd + 8 * (slot % hp), qt = n_qt - 1 - slot / hp;            // the longest tiles first; a head stays on one XCD
+    if (h >= p.n_head) return;
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, i = lane & 15, g = lane >> 4;
+    const int q0 = qt * kXTok, dk = p.dim + p.rot_dim;
+    // the tokens of this lane (column i of two tiles) and the cells they see
+    int nv[2], tok[2];
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+        const int t = q0 + wave * 32 + u * 16 + i;
+        tok[u] = p.tok0 + min(t, p.T - 1);
+        nv[u] = t < p.T ? p.n_vis[tok[u]] : 0;
+    }
+    const int n_keys = p.n_vis[p.tok0 + min(q0 + kXTok, p.T) - 1], n_all = p.n_vis[p.tok0 + q0];          // the most and the fewest cells a token here sees
+    pi_u32x4 qf[2][KS];
+#pragma unroll
+    for (int u = 0; u < 2; ++u)
+#pragma unroll
+        for (int s = 0; s < KS; ++s) {
+            const int c = s * 32 + g * 8;
+            const bf16 * src = c < p.dim ? (const bf16 *)p.q_un + ((size_t)tok[u] * p.n_head + h) * p.dim_ld + c
+                                         : (const bf16 *)p.q_lat + ((size_t)tok[u] * p.n_head + h) * p.kd + p.rank_ld + (c - p.dim);
+            qf[u][s] = c < dk ? pi_ld16(src) : pi_u32x4{0, 0, 0, 0};
+        }
+    pi_u32x4 kr[KP], vr[VP];
+    auto fetch = [&](int k0) {
+#pragma unroll
+        for (int j = 0; j < KP; ++j) {
+            const int e = tid + 256 * j, key = min(k0 + e / (KS * 4), n_keys - 1), c = (e % (KS * 4)) * 8;
+            const bf16 * src = c < p.dim ? (const bf16 *)p.keys + ((size_t)key * p.n_head + h) * p.dim + c
+                                         : (const bf16 *)p.cache + (size_t)p.list[key] * p.kd + p.rank_ld + (c - p.dim);
+            kr[j] = c < dk ? pi_ld16(src) : pi_u32x4{0, 0, 0, 0};
+        }
+#pragma unroll
+        for (int j = 0; j < VP; ++j) {
+            const int e = tid + 256 * j, key = min(k0 + e / (VT * 2), n_keys - 1), c = (e % (VT * 2)) * 8;
+            vr[j] = c < p.vdim ? pi_ld16((const bf16 *)p.values + ((size_t)key * p.n_head + h) * p.vdim + c) : pi_u32x4{0, 0, 0, 0};
+        }
+    };
+    fetch(0);
+    float m[2] = {-INFINITY, -INFINITY}, l[2] = {0.0f, 0.0f};
+    pi_f4 o[2][VT];
+#pragma unroll
+    for (int u = 0; u < 2; ++u)
+#pragma unroll
+        for (int v = 0; v < VT; ++v) o[u][v] = pi_f4{0, 0, 0, 0};
+    for (int k0 = 0; k0 < n_keys; k0 += kXKeys) {
+        __syncthreads();
+#pragma unroll
+        for (int j = 0; j < KP; ++j) { const int e = tid + 256 * j; *reinterpret_cast<pi_u32x4 *>(ks + (e / (KS * 4)) * KROW + (e % (KS * 4)) * 16) = kr[j]; }
+#pragma unroll
+        for (int j = 0; j < VP; ++j) { const int e = tid + 256 * j; *reinterpret_cast<pi_u32x4 *>(vs + (e / (VT * 2)) * VROW + (e % (VT * 2)) * 16) = vr[j]; }
+        __syncthreads();
+        if (k0 + kXKeys < n_keys) fetch(k0 + kXKeys);
+        pi_f4 s[2][4];
+#pragma unroll
+        for (int kt = 0; kt < 4; ++kt) {
+            s[0][kt] = s[1][kt] = pi_f4{0, 0, 0, 0};
+#pragma unroll
+            for (int c = 0; c < KS; ++c) {
+                const pi_u32x4 a = *reinterpret_cast<const pi_u32x4 *>(ks + (kt * 16 + i) * KROW + c * 64 + g * 16);
+                s[0][kt] = mfma_bf16(a, qf[0][c], s[0][kt]);
+                s[1][kt] = mfma_bf16(a, qf[1][c], s[1][kt]);
+            }
+        }
+        pi_u32x4 pb[2][2];                             // weights as the column operand: [token tile][32 keys]
+#pragma unroll
+        for (int u = 0; u < 2; ++u) {
+            float mx = -INFINITY;
+            const bool edge = k0 + kXKeys > n_all;
+#pragma unroll
+            for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    float v = s[u][kt][r] * p.scale;
+                    if (edge && k0 + kt * 16 + 4 * g + r >= nv[u]) v = -INFINITY;
+                    s[u][kt][r] = v;
+                    mx = fmaxf(mx, v);
+                }
+            mx = fmaxf(mx, __shfl_xor(mx, 16, PI_WAVE));
+            mx = fmaxf(mx, __shfl_xor(mx, 32, PI_WAVE));
+            const float mn = fmaxf(m[u], mx), base = mn == -INFINITY ? 0.0f : mn;
+            const float a = expf(m[u] - base);         // 0 while nothing has been seen
+            m[u] = mn;
+            float sum = 0.0f;
+            bf16 w[16];
+#pragma unroll
+            for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) { const float e = expf(s[u][kt][r] - base); sum += e; w[kt * 4 + r] = (bf16)e; }
+            l[u] = l[u] * a + sum;
+#pragma unroll
+            for (int v = 0; v < VT; ++v) { o[u][v][0] *= a; o[u][v][1] *= a; o[u][v][2] *= a; o[u][v][3] *= a; }
+#pragma unroll
+            for (int k = 0; k < 2; ++k) {
+                bf16 b[8];
+#pragma unroll
+                for (int j = 0; j < 8; ++j) b[j] = w[k * 8 + j];
+                pb[u][k] = __builtin_bit_cast(pi_u32x4, b);
+            }
+        }
+        // slot (g, j) of a 32-key step: key 4 g + j of its first 16 (j < 4) or of its second 16 - two transposing reads
+#pragma unroll
+        for (int k = 0; k < 2; ++k)
+#pragma unroll
+            for (int v = 0; v < VT; ++v) {
+                const unsigned char * a = vs + (k * 32 + 4 * g + (i >> 2)) * VROW + (v * 16 + (i & 3) * 4) * 2;
+                const pi_u32x2 lo = __builtin_bit_cast(pi_u32x2, tr_read(a)), hi = __builtin_bit_cast(pi_u32x2, tr_read(a + 16 * VROW));
+                const pi_u32x4 f{lo.x, lo.y, hi.x, hi.y};
+                o[0][v] = mfma_bf16(f, pb[0][k], o[0][v]);
+                o[1][v] = mfma_bf16(f, pb[1][k], o[1][v]);
+            }
+    }
+    const float sink = p.sink[h];
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+        float sum = l[u];
+        sum += __shfl_xor(sum, 16, PI_WAVE);
+        sum += __shfl_xor(sum, 32, PI_WAVE);
+        const float mf = fmaxf(m[u], sink), a = m[u] == -INFINITY ? 0.0f : expf(m[u] - mf), f = a / (sum * a + expf(sink - mf));
+        if (q0 + wave * 32 + u * 16 + i >= p.T) continue;
+        bf16 * out = (bf16 *)p.att + (size_t)tok[u] * p.ld_att + h * p.vdim;
+#pragma unroll
+        for (int v = 0; v < VT; ++v) {
+            const int c = v * 16 + 4 * g;
+            if (c >= p.vdim) continue;                 // vdim % 8 == 0: four columns at a time
+            bf16 b[4] = {(bf16)(o[u][v][0] * f), (bf16)(o[u][v][1] * f), (bf16)(o[u][v][2] * f), (bf16)(o[u][v][3] * f)};
+            *reinterpret_cast<pi_u32x2 *>(out + c) = __builtin_bit_cast(pi_u32x2, b);
+        }
+    }
+}
+
+template <int KS, int VT> int launch_expanded(const pi_latent_expanded * p, hipStream_t st) {
+    const int n_qt = (p->T + kXTok - 1) / kXTok, hp = (p->n_head + 7) / 8;
+    hipLaunchKernelGGL((latent_expanded_attn_kernel<KS, VT>), dim3(8 * hp * n_qt), dim3(256), 0, st, *p, n_qt, hp);
+    return pi::check_launch("pi_k_latent_attn_expanded");
+}
+
 template <typename ST>
 __global__ void latent_shift_kernel(ST * __restrict__ cache, int kd, int rank_ld, int rot_dim, double base, const int32_t * __restrict__ delta) {
     const int c = blockIdx.x, d = delta[c];
@@ -354,6 +504,21 @@ int pi_k_latent_attn(int type, const pi_latent_attn * p, pi_stream_t stream) {
     if (rc != PI_OK || p->n_parts == 1) return rc;
     hipLaunchKernelGGL(latent_merge_kernel, dim3(p->T * p->n_head), dim3(128), 0, st, *p);
     return pi::check_launch("pi_k_latent_attn merge");
+}
+
+int pi_k_latent_expanded_supported(int dim, int rot_dim, int vdim) {
+    return dim > 0 && rot_dim > 0 && vdim > 0 && dim % 8 == 0 && rot_dim % 8 == 0 && vdim % 8 == 0 && dim + rot_dim <= 256 && vdim <= 128;
+}
+
+int pi_k_latent_attn_expanded(const pi_latent_expanded * p, pi_stream_t stream) {
+    if (!p || !p->q_un || !p->q_lat || !p->keys || !p->values || !p->cache || !p->list || !p->n_vis || !p->sink || !p->att || p->T <= 0 || p->tok0 < 0 || p->n_head <= 0 ||
+        p->dim_ld < p->dim || p->dim_ld % 8 || p->kd % 8 || p->rank_ld % 8 || p->kd < p->rank_ld + p->rot_dim || p->ld_att % 8 || p->ld_att < p->n_head * p->vdim)
+        return pi::fail(PI_E_ARG, "pi_k_latent_attn_expanded: bad arguments");
+    if (!pi_k_latent_expanded_supported(p->dim, p->rot_dim, p->vdim)) return pi::fail(PI_E_UNSUPPORTED, "pi_k_latent_attn_expanded: head sizes");
+    const int dk = p->dim + p->rot_dim;
+    hipStream_t st = (hipStream_t)stream;
+    if (p->vdim <= 64) return dk <= 128 ? launch_expanded<4, 4>(p, st) : dk <= 192 ? launch_expanded<6, 4>(p, st) : launch_expanded<8, 4>(p, st);
+    return dk <= 128 ? launch_expanded<4, 8>(p, st) : dk <= 192 ? launch_expanded<6, 8>(p, st) : launch_expanded<8, 8>(p, st);
 }
 
 int pi_k_latent_shift(int type, void * cache, int n_cells, int kd, int rank_ld, int rot_dim, double base, const int32_t * delta, pi_stream_t stream) {

@@ -42,6 +42,11 @@ class LatentAttn(C.Structure):
         ("scale", _f), ("sink", _vp), ("scratch", _vp), ("out_lat", _vp)]
 
 
+class LatentExpanded(C.Structure):
+    _fields_ = [(n, _vp) for n in ("q_un", "q_lat", "keys", "values", "cache", "list", "n_vis", "sink", "att")] + [
+        (n, C.c_int32) for n in ("tok0", "T", "n_head", "dim", "dim_ld", "rot_dim", "vdim", "rank_ld", "kd", "ld_att")] + [("scale", _f)]
+
+
 class LayerOut(C.Structure):
     _fields_ = [("x", _vp), ("wo", _vp), ("att", _vp), ("rows", C.c_int32), ("ld_att", C.c_int32), ("T", C.c_int32),
                 ("down", _vp), ("act", _vp), ("ids", _vp), ("ld_act", C.c_int32), ("top", C.c_int32), ("n_expert", C.c_int32),
@@ -183,6 +188,8 @@ _SIGS = {
     "pi_k_latent_attn_supported": (_i, [_i, _i, _i]),
     "pi_k_latent_attn_scratch_floats": (_sz, [_i, _i, _i, _i]),
     "pi_k_latent_attn": (_i, [_i, C.POINTER(LatentAttn), _vp]),
+    "pi_k_latent_expanded_supported": (_i, [_i, _i, _i]),
+    "pi_k_latent_attn_expanded": (_i, [C.POINTER(LatentExpanded), _vp]),
     "pi_k_latent_shift": (_i, [_i, _vp, _i, _i, _i, _i, C.c_double, _vp, _vp]),
     "pi_k_route": (_i, [_vp, _i, _i, _i, _i, _i, _vp, _vp, _vp, _vp]),
     "pi_k_moe_sort": (_i, [_vp, _i, _i, _vp, _vp, _vp, _i, _vp, _vp, _vp]),
