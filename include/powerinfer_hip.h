@@ -644,9 +644,9 @@ PI_API int pi_k_moe_sort(const int32_t * ids, int n_pairs, int n_expert, int32_t
 PI_API int pi_k_moe_combine(int type, const float * x, const float * mix, const void * y, const int32_t * inv, const float * weights, int n_top, int T,
                             int cols, float * out, float * keep, pi_stream_t stream);
 /* Steps of up to 16 tokens (bf16; pi_k_layer_step_supported).  pi_k_latent_step: pi_k_latent_prep, the absorbed queries (uk_t
- * [n_head][kv_rank][dim_ld]; p->q_un is not used) and, with ids != NULL, pi_k_route in one launch.  pi_k_latent_value_step: the merge of
- * a split attention (or its whole result) and the value expansion, att [T][ld_att]; pi_k_latent_attn_parts leaves the parts unmerged.
- * pi_k_expert_up_step: act [T * top][ld_act] = weight * relu(up[e] x)^2 for every (token, choice).  pi_k_layer_out_step: what closes the
+ * [n_head][kv_rank][dim_ld]; p->q_un is not used) and, with ids != NULL, pi_k_route in one launch.  pi_k_value_up_step: the merge of
+ * a split attention (or its whole result) and the value expansion, att [T][ld_att] - pi_k_latent_attn_parts leaves the parts unmerged -
+ * and, with ids != NULL, act [T * top][ld_act] = weight * relu(up[e] x)^2 for every (token, choice).  pi_k_layer_out_step: what closes the
  * layer, out = x + (wo att + sum over the pairs of a token of down[e] act[pair]); ids == NULL: no experts. */
 typedef struct pi_layer_out {
     const float * x; const void * wo, * att; int32_t rows, ld_att, T;
@@ -657,9 +657,8 @@ PI_API int pi_k_layer_step_supported(int T, int n_expert, int n_top);
 PI_API int pi_k_latent_step(const pi_latent_prep * p, const void * uk_t, const float * z_router, int n_expert, int n_top, int n_group, int n_keep, const float * bias,
                             int32_t * ids, float * weights, pi_stream_t stream);
 PI_API int pi_k_latent_attn_parts(const pi_latent_attn * p, pi_stream_t stream);
-PI_API int pi_k_latent_value_step(const pi_latent_attn * p, const void * uv, int vdim, void * att, int ld_att, pi_stream_t stream);
-PI_API int pi_k_expert_up_step(const void * up, int n_expert, int ff, int cols, const void * x_ol, const int32_t * ids, const float * weights, int T, int top, void * act,
-                               int ld_act, pi_stream_t stream);
+PI_API int pi_k_value_up_step(const pi_latent_attn * p, const void * uv, int vdim, void * att, int ld_att, const void * up, int n_expert, int ff, int cols,
+                              const void * x_ol, const int32_t * ids, const float * weights, int top, void * act, int ld_act, pi_stream_t stream);
 PI_API int pi_k_layer_out_step(const pi_layer_out * a, pi_stream_t stream);
 /* BF16 matrices: out [rows][ld] = in [rows][cols] padded with zeros; out [n_mat][cols][ld] = each in [rows][cols] transposed, padded with zeros */
 PI_API int pi_k_pad_cols_bf16(const void * in, int64_t rows, int cols, void * out, int ld, pi_stream_t stream);

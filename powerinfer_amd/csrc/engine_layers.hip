@@ -389,7 +389,7 @@ int ffn_moe(pi_model * m, Layer & L, const Step & in) {
     return grouped(s, w, tile_n, st);
 }
 
-// a layer of a step of up to 16 tokens (bf16): seven launches
+// a layer of a step of up to 16 tokens (bf16): six launches
 int step_layer(pi_model * m, Layer & L, const Step & in, float * keep) {
     LayerState * s = m->lay;
     const pi_layer_desc & d = L.d;
@@ -402,15 +402,9 @@ int step_layer(pi_model * m, Layer & L, const Step & in, float * keep) {
     else     PI_TRY(pi_k_gemm_bf16_ol(L.w_z, L.z_rows, s->d_ld, s->h_a, T, PI_EPI_NONE, nullptr, nullptr, s->z, nullptr, st));
     const pi_latent_prep p = prep_args(m, L, in);
     PI_TRY(pi_k_latent_step(&p, L.uk_t, s->rl, d.n_expert, d.n_top, d.n_group, d.n_group_keep, L.bias, moe ? s->ids : nullptr, s->wts, st));
-    // the experts' first matrices do not wait for the attention: in the captured loop they run beside it on the second stream
-    const bool fork = moe && m->building_graph;
-    hipStream_t st2 = fork ? m->stream2 : st;
-    if (fork) { PI_HIP_TRY(hipEventRecord(m->ev_fork[0], st)); PI_HIP_TRY(hipStreamWaitEvent(st2, m->ev_fork[0], 0)); }
-    if (moe) PI_TRY(pi_k_expert_up_step(L.up, d.n_expert, d.expert_ff, s->d_ld, s->h_b, s->ids, s->wts, T, d.n_top, s->act, L.ff_ld, st2));
     const pi_latent_attn a = attn_args(m, L, src, in);
     PI_TRY(pi_k_latent_attn_parts(&a, st));
-    PI_TRY(pi_k_latent_value_step(&a, L.uv, d.vdim, s->att, L.hv_ld, st));
-    if (fork) { PI_HIP_TRY(hipEventRecord(m->ev_join[0], st2)); PI_HIP_TRY(hipStreamWaitEvent(st, m->ev_join[0], 0)); }
+    PI_TRY(pi_k_value_up_step(&a, L.uv, d.vdim, s->att, L.hv_ld, L.up, d.n_expert, d.expert_ff, s->d_ld, s->h_b, moe ? s->ids : nullptr, s->wts, d.n_top, s->act, L.ff_ld, st));
     pi_layer_out o{};
     o.x = s->x; o.wo = L.wo; o.att = s->att; o.rows = D; o.ld_att = L.hv_ld; o.T = T; o.out = s->x2; o.keep = keep;
     if (moe) { o.down = L.down; o.act = s->act; o.ids = s->ids; o.ld_act = L.ff_ld; o.top = d.n_top; o.n_expert = d.n_expert; }
@@ -591,10 +585,6 @@ int layers_finalize(pi_model * m) {
     const int D = m->hp.n_embd;
     PI_HIP_TRY(hipEventCreate(&m->ev0));
     PI_HIP_TRY(hipEventCreate(&m->ev1));
-    PI_HIP_TRY(hipStreamCreateWithFlags(&m->stream2, hipStreamNonBlocking));
-    m->ev_fork.assign(1, nullptr); m->ev_join.assign(1, nullptr);
-    PI_HIP_TRY(hipEventCreateWithFlags(&m->ev_fork[0], hipEventDisableTiming));
-    PI_HIP_TRY(hipEventCreateWithFlags(&m->ev_join[0], hipEventDisableTiming));
     s->es = bf16_mode(s) ? 2 : 4;
     s->d_ld = up_to(D, 256);
     PI_TRY(want_tensor(m->glob[PI_T_TOK_EMBD], PI_TYPE_BF16, D, m->hp.n_vocab, "tok_embd"));
@@ -868,9 +858,7 @@ int layers_generate(pi_model * m, int own, int n_steps, int32_t * out_tokens, fl
     if (use_graph && s->exec && (s->graph_T != T || s->graph_seq0 != q0 || s->graph_parts != parts)) drop_graph(s);
     if (use_graph && !s->exec) {
         PI_HIP_TRY(hipStreamBeginCapture(m->stream, hipStreamCaptureModeThreadLocal));
-        m->building_graph = true;
         const int rc = step();
-        m->building_graph = false;
         hipGraph_t g = nullptr;
         const hipError_t e = hipStreamEndCapture(m->stream, &g);
         if (rc != PI_OK) { if (g) (void)hipGraphDestroy(g); return rc; }

@@ -81,7 +81,8 @@ __global__ __launch_bounds__(256) void latent_attn_bf16_kernel(pi_latent_attn p)
     float * row_m = reinterpret_cast<float *>(ps + R * (NC + 8)), * row_l = row_m + R, * row_a = row_l + R;
     int * row_n = reinterpret_cast<int *>(row_a + R);
     const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, i = lane & 15, g = lane >> 4;
-    const int tok0 = p.work[4 * blockIdx.x], first = p.work[4 * blockIdx.x + 1], rows = min(p.work[4 * blockIdx.x + 2], R), seq = p.work[4 * blockIdx.x + 3];
+    const int4 item = reinterpret_cast<const int4 *>(p.work)[blockIdx.x];
+    const int tok0 = item.x, first = item.y, rows = min(item.z, R), seq = item.w;
     const size_t qrow0 = (size_t)tok0 * p.n_head + first;        // row of q_lat / out_lat of this workgroup's first row
     const int32_t * list = p.lists + (size_t)seq * p.list_ld;
     const int n_all = p.n_vis[tok0 + (first + rows - 1) / p.n_head];                       // cells of the last row's token: the most of all
@@ -98,11 +99,16 @@ __global__ __launch_bounds__(256) void latent_attn_bf16_kernel(pi_latent_attn p)
         for (int j = 0; j < PF; ++j)
             if (pn[j] < NC) pre[j] = pi_ld16(cache + (size_t)list[min(cb + pn[j], n_all - 1)] * p.kd + pc[j]);
     };
+    // the query rows travel with the first cells: as many pieces per thread as a cell tile has (R == NC rows)
+    static_assert(R == NC, "query and cell tiles share the piece layout");
+    pi_u32x4 qr[PF];
+#pragma unroll
+    for (int j = 0; j < PF; ++j)
+        if (pn[j] < R) qr[j] = pi_ld16((const uint16_t *)p.q_lat + (qrow0 + min(pn[j], rows - 1)) * p.kd + pc[j]);
     if (c0 < c1) fetch(c0);
-    for (int c = tid; c < R * pieces; c += 256) {
-        const int r = c / pieces, k = (c % pieces) * 8;
-        *reinterpret_cast<pi_u32x4 *>(qs + r * stride + k * 2) = pi_ld16((const uint16_t *)p.q_lat + (qrow0 + min(r, rows - 1)) * p.kd + k);
-    }
+#pragma unroll
+    for (int j = 0; j < PF; ++j)
+        if (pn[j] < R) *reinterpret_cast<pi_u32x4 *>(qs + pn[j] * stride + pc[j] * 2) = qr[j];
     if (tid < R) { row_m[tid] = -INFINITY; row_l[tid] = 0.0f; row_n[tid] = tid < rows ? p.n_vis[tok0 + (first + tid) / p.n_head] : 0; }
     pi_f4 acc[RT][VT];
 #pragma unroll

@@ -1,6 +1,6 @@
 // Steps of up to 16 tokens of a model described layer by layer (bf16), as few launches as its dependencies allow: everything behind
 // the joint projection (absorbed queries, rotation, cells, expert choice) in one, the merge of a split attention with the value
-// expansion in one, the experts' first matrices in one, and one for what closes a layer - attention output and the experts' second
+// expansion together with the experts' first matrices in one, and one for what closes a layer - attention output and the experts' second
 // matrices as a single long dot product per row, plus the residual.
 #include "layer_types.hpp"
 #include "route.hpp"
@@ -68,18 +68,21 @@ __global__ __launch_bounds__(256) void latent_step_kernel(pi_latent_prep p, cons
 // the parts of a split attention merged (fixed order, the sink in the denominator) and the head's values expanded from the result:
 // a workgroup owns 64 value rows of one head, for all tokens of the step
 // ---------------------------------------------------------------------------------------------------------------------------------
-__global__ __launch_bounds__(256) void latent_value_kernel(pi_latent_attn p, const uint16_t * __restrict__ uv, int vdim, bf16 * __restrict__ att, int ld_att) {
-    extern __shared__ __align__(16) unsigned char smem[];
-    const int h = blockIdx.x, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, i = lane & 15, g = lane >> 4;
+__host__ __device__ inline size_t value_lds_bytes(int T, int rank_ld, int n_parts) {
+    return (size_t)T * (rank_ld + 8) * 2 + sizeof(float) * (((size_t)T * n_parts + 3) / 4 * 4 + 4 * (size_t)rank_ld);
+}
+__device__ void latent_value(const pi_latent_attn & p, const uint16_t * __restrict__ uv, int vdim, bf16 * __restrict__ att, int ld_att, int h, int rt, unsigned char * smem) {
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, i = lane & 15, g = lane >> 4;
     const int ld = p.rank_ld + 8;
     bf16 * ol = reinterpret_cast<bf16 *>(smem);               // [T][ld]
-    float * f = reinterpret_cast<float *>(smem + (size_t)p.T * ld * 2 + (size_t)(p.T * ld * 2) % 16);      // [T][n_parts] factor of each part
-    const int row0 = blockIdx.y * 64 + wave * 16;
+    float * f = reinterpret_cast<float *>(ol + p.T * ld);     // [T][n_parts] factor of each part
+    float * ws = f + (p.T * p.n_parts + 3) / 4 * 4;           // [4][rank_ld] the waves' sums
+    const int row0 = rt * 64 + wave * 16;
     // the value matrix does not depend on the attention: its first fragments are requested ahead of everything else
     const uint16_t * W = uv + ((size_t)h * vdim + min(row0 + i, vdim - 1)) * p.rank_ld + g * 8;
-    pi_u32x4 w0[4];
+    pi_u32x4 w0[8];
 #pragma unroll
-    for (int k = 0; k < 4; ++k) w0[k] = k * 32 < p.rank_ld ? pi_ld_stream(W + k * 32) : pi_u32x4{0, 0, 0, 0};
+    for (int k = 0; k < 8; ++k) w0[k] = k * 32 < p.rank_ld ? pi_ld_stream(W + k * 32) : pi_u32x4{0, 0, 0, 0};
     if (p.n_parts == 1) {
         for (int c = tid; c < p.T * (p.rank_ld / 8); c += 256) {
             const int t = c / (p.rank_ld / 8), k = (c % (p.rank_ld / 8)) * 8;
@@ -96,18 +99,25 @@ __global__ __launch_bounds__(256) void latent_value_kernel(pi_latent_attn p, con
             if (lane < p.n_parts) f[t * p.n_parts + lane] = e / l;
         }
         __syncthreads();
-        for (int c = tid; c < p.T * (p.rank_ld / 4); c += 256) {
-            const int t = c / (p.rank_ld / 4), k = (c % (p.rank_ld / 4)) * 4;
-            const float * a = p.scratch + ((size_t)t * p.n_head + h) * p.n_parts * p.rank_ld + k;
-            float4 s = make_float4(0, 0, 0, 0);
-#pragma unroll 8
-            for (int q = 0; q < p.n_parts; ++q) {
-                const float4 v = *reinterpret_cast<const float4 *>(a + (size_t)q * p.rank_ld);
-                const float w = f[t * p.n_parts + q];
-                s.x = fmaf(w, v.x, s.x); s.y = fmaf(w, v.y, s.y); s.z = fmaf(w, v.z, s.z); s.w = fmaf(w, v.w, s.w);
+        for (int t = 0; t < p.T; ++t) {                       // a wave takes every fourth part, a lane four columns of a 256-column piece
+            const float * a = p.scratch + ((size_t)t * p.n_head + h) * p.n_parts * p.rank_ld;
+            for (int c = lane * 4; c < p.rank_ld; c += 256) {
+                float4 s = make_float4(0, 0, 0, 0);
+                for (int q0 = wave; q0 < p.n_parts; q0 += 32) {
+                    float4 v[8];
+#pragma unroll
+                    for (int u = 0; u < 8; ++u) v[u] = *reinterpret_cast<const float4 *>(a + (size_t)min(q0 + 4 * u, p.n_parts - 1) * p.rank_ld + c);
+#pragma unroll
+                    for (int u = 0; u < 8; ++u) {
+                        const float w = q0 + 4 * u < p.n_parts ? f[t * p.n_parts + q0 + 4 * u] : 0.0f;
+                        s.x = fmaf(w, v[u].x, s.x); s.y = fmaf(w, v[u].y, s.y); s.z = fmaf(w, v[u].z, s.z); s.w = fmaf(w, v[u].w, s.w);
+                    }
+                }
+                *reinterpret_cast<float4 *>(ws + wave * p.rank_ld + c) = s;
             }
-            bf16 o[4] = {(bf16)s.x, (bf16)s.y, (bf16)s.z, (bf16)s.w};
-            *reinterpret_cast<pi_u32x2 *>(ol + t * ld + k) = __builtin_bit_cast(pi_u32x2, o);
+            __syncthreads();
+            for (int c = tid; c < p.rank_ld; c += 256) ol[t * ld + c] = (bf16)(ws[c] + ws[p.rank_ld + c] + ws[2 * p.rank_ld + c] + ws[3 * p.rank_ld + c]);
+            __syncthreads();
         }
     }
     __syncthreads();
@@ -115,10 +125,14 @@ __global__ __launch_bounds__(256) void latent_value_kernel(pi_latent_attn p, con
     const bf16 * x = ol + min(i, p.T - 1) * ld + g * 8;
     pi_f4 acc = pi_f4{0, 0, 0, 0};
 #pragma unroll
-    for (int k = 0; k < 4; ++k)
+    for (int k = 0; k < 8; ++k)
         if (k * 32 < p.rank_ld) acc = mma16<bf16>(w0[k], *reinterpret_cast<const pi_u32x4 *>(x + k * 32), acc);
-#pragma unroll 4
-    for (int k = 128; k < p.rank_ld; k += 32) acc = mma16<bf16>(pi_ld_stream(W + k), *reinterpret_cast<const pi_u32x4 *>(x + k), acc);
+    for (int k0 = 256; k0 < p.rank_ld; k0 += 256) {
+#pragma unroll
+        for (int k = 0; k < 8; ++k) w0[k] = k0 + k * 32 < p.rank_ld ? pi_ld_stream(W + k0 + k * 32) : pi_u32x4{0, 0, 0, 0};
+#pragma unroll
+        for (int k = 0; k < 8; ++k) if (k0 + k * 32 < p.rank_ld) acc = mma16<bf16>(w0[k], *reinterpret_cast<const pi_u32x4 *>(x + k0 + k * 32), acc);
+    }
     if (i >= p.T) return;
     bf16 * o = att + (size_t)i * ld_att + h * vdim + row0 + 4 * g;
 #pragma unroll
@@ -177,14 +191,17 @@ __device__ int step_experts(StepExperts & s, const int32_t * __restrict__ ids, i
 // first matrices of the step's experts: workgroup (row tile, pair) works for the pair's expert if no earlier pair has the same one, for
 // every token that chose it; act[pair] = weight * relu(z)^2
 // ---------------------------------------------------------------------------------------------------------------------------------
-template <int NW>
-__global__ __launch_bounds__(64 * NW) void expert_up_step_kernel(const bf16 * __restrict__ up, int ff, int cols, const bf16 * __restrict__ x_ol, const int32_t * __restrict__ ids,
-                                                                 const float * __restrict__ weights, int T, int top, bf16 * __restrict__ act, int ld_act) {
-    __shared__ __align__(16) unsigned char tiles[NW][16 * kWsStride];
-    const int p = blockIdx.y, e = ids[p], tid = threadIdx.x, wave = tid >> 6;
-    if (T > 1 && __syncthreads_or(tid < p && ids[tid] == e)) return;            // p < 64 * NW: checked by the launcher
+struct ExpertUp { const bf16 * up; int ff, cols; const bf16 * x_ol; const int32_t * ids; const float * weights; int T, top; bf16 * act; int ld_act; };
+constexpr int kUpLds = 4 * 16 * kWsStride;
+__device__ void expert_up(const ExpertUp & a, int tile, int p, unsigned char * smem) {
+    constexpr int NW = 4;
+    unsigned char (*tiles)[16 * kWsStride] = reinterpret_cast<unsigned char (*)[16 * kWsStride]>(smem);
+    const bf16 * up = a.up, * x_ol = a.x_ol; const int32_t * ids = a.ids;
+    const int ff = a.ff, cols = a.cols, T = a.T, top = a.top;
+    const int e = ids[p], tid = threadIdx.x, wave = tid >> 6;
+    if (T > 1 && __syncthreads_or(tid < p && ids[tid] == e)) return;            // p < 256: checked by the launcher
     const WaveStream ws(tiles[wave]);
-    const int row0 = blockIdx.x * 16, n_ss = (cols + 255) / 256;
+    const int row0 = tile * 16, n_ss = (cols + 255) / 256;
     const bf16 * W = up + (size_t)e * ff * cols;
     pi_u32x4 ld[2][8];
     pi_f4 acc = pi_f4{0, 0, 0, 0};
@@ -215,7 +232,16 @@ __global__ __launch_bounds__(64 * NW) void expert_up_step_kernel(const bf16 * __
     for (int w = 0; w < NW; ++w) v += reinterpret_cast<float (*)[17]>(tiles[w])[rr][t];
     v = fmaxf(v, 0.0f);
     for (int k = 0; k < top; ++k)
-        if (ids[t * top + k] == e) act[(size_t)(t * top + k) * ld_act + row] = (bf16)(weights[t * top + k] * v * v);
+        if (ids[t * top + k] == e) a.act[(size_t)(t * top + k) * a.ld_act + row] = (bf16)(a.weights[t * top + k] * v * v);
+}
+
+// both in one launch: the value expansion of the attention branch hides behind the experts' weights
+__global__ __launch_bounds__(256) void value_and_up_kernel(pi_latent_attn p, const uint16_t * __restrict__ uv, int vdim, bf16 * __restrict__ att, int ld_att, int n_rt, int n_value,
+                                                           ExpertUp u, int n_up_tiles) {
+    extern __shared__ __align__(16) unsigned char smem[];
+    const int b = blockIdx.x;
+    if (b < n_value) latent_value(p, uv, vdim, att, ld_att, b / n_rt, b % n_rt, smem);
+    else expert_up(u, (b - n_value) % n_up_tiles, (b - n_value) / n_up_tiles, smem);
 }
 
 // ---------------------------------------------------------------------------------------------------------------------------------
@@ -297,22 +323,21 @@ int pi_k_latent_step(const pi_latent_prep * p, const void * uk_t, const float * 
     return pi::check_launch("pi_k_latent_step");
 }
 
-int pi_k_latent_value_step(const pi_latent_attn * p, const void * uv, int vdim, void * att, int ld_att, pi_stream_t stream) {
+int pi_k_value_up_step(const pi_latent_attn * p, const void * uv, int vdim, void * att, int ld_att, const void * up, int n_expert, int ff, int cols, const void * x_ol,
+                       const int32_t * ids, const float * weights, int top, void * act, int ld_act, pi_stream_t stream) {
     if (!p || !uv || !att || p->T <= 0 || p->T > kBtMaxT || p->n_head <= 0 || vdim <= 0 || p->rank_ld <= 0 || p->rank_ld % 64 || p->rank_ld > 1024 || ld_att < p->n_head * vdim || !p->sink ||
         p->n_parts <= 0 || p->n_parts > 64 || (p->n_parts == 1 ? !p->out_lat : !p->scratch))
-        return pi::fail(PI_E_ARG, "pi_k_latent_value_step: bad arguments");
-    const size_t lds = (size_t)p->T * (p->rank_ld + 8) * 2 + 16 + sizeof(float) * p->T * p->n_parts;
-    hipLaunchKernelGGL(latent_value_kernel, dim3(p->n_head, (vdim + 63) / 64), dim3(256), lds, (hipStream_t)stream, *p, (const uint16_t *)uv, vdim, (bf16 *)att, ld_att);
-    return pi::check_launch("pi_k_latent_value_step");
-}
-
-int pi_k_expert_up_step(const void * up, int n_expert, int ff, int cols, const void * x_ol, const int32_t * ids, const float * weights, int T, int top, void * act, int ld_act,
-                        pi_stream_t stream) {
-    if (!up || !x_ol || !ids || !weights || !act || n_expert <= 0 || ff <= 0 || cols <= 0 || cols % 32 || T <= 0 || T > kBtMaxT || top <= 0 || T * top > kStepPairs || ld_act < ff)
-        return pi::fail(PI_E_ARG, "pi_k_expert_up_step: bad arguments");
-    hipLaunchKernelGGL(expert_up_step_kernel<4>, dim3((ff + 15) / 16, T * top), dim3(256), 0, (hipStream_t)stream, (const bf16 *)up, ff, cols, (const bf16 *)x_ol, ids, weights, T, top,
-                       (bf16 *)act, ld_act);
-    return pi::check_launch("pi_k_expert_up_step");
+        return pi::fail(PI_E_ARG, "pi_k_value_up_step: bad arguments");
+    if (ids && (!up || !x_ol || !weights || !act || n_expert <= 0 || ff <= 0 || cols <= 0 || cols % 32 || top <= 0 || p->T * top > kStepPairs || ld_act < ff))
+        return pi::fail(PI_E_ARG, "pi_k_value_up_step: bad expert arguments");
+    const int n_rt = (vdim + 63) / 64, n_value = p->n_head * n_rt, n_up_tiles = ids ? (ff + 15) / 16 : 1, n_up = ids ? n_up_tiles * p->T * top : 0;
+    size_t lds = value_lds_bytes(p->T, p->rank_ld, p->n_parts);
+    if (ids && lds < (size_t)kUpLds) lds = kUpLds;
+    static bool raised = false;
+    if (!raised) { PI_HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void *>(&value_and_up_kernel), hipFuncAttributeMaxDynamicSharedMemorySize, 96 * 1024)); raised = true; }
+    hipLaunchKernelGGL(value_and_up_kernel, dim3(n_value + n_up), dim3(256), lds, (hipStream_t)stream, *p, (const uint16_t *)uv, vdim, (bf16 *)att, ld_att, n_rt, n_value,
+                       ExpertUp{(const bf16 *)up, ff, cols, (const bf16 *)x_ol, ids, weights, p->T, top, (bf16 *)act, ld_act}, n_up_tiles);
+    return pi::check_launch("pi_k_value_up_step");
 }
 
 int pi_k_layer_out_step(const pi_layer_out * a, pi_stream_t stream) {

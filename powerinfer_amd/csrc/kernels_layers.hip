@@ -18,12 +18,29 @@ template <typename LD> __device__ float row_rms_scale(int cols, float eps, doubl
     return pi_inv_sqrt((float)(s / cols) + eps);
 }
 
-__global__ __launch_bounds__(256) void embed_norm_kernel(const uint16_t * __restrict__ table, int cols, const int32_t * __restrict__ tokens,
-                                                         const float * __restrict__ w, float eps, float * __restrict__ x) {
-    __shared__ double red[4];
+__global__ __launch_bounds__(1024) void embed_norm_kernel(const uint16_t * __restrict__ table, int cols, const int32_t * __restrict__ tokens,
+                                                          const float * __restrict__ w, float eps, float * __restrict__ x) {
+    __shared__ double red[16];
     const uint16_t * row = table + (size_t)tokens[blockIdx.x] * cols;
+    float * out = x + (size_t)blockIdx.x * cols;
+    if (cols <= 8 * (int)blockDim.x) {              // row and weights requested together, kept in registers
+        float v[8], wv[8];
+        double s = 0.0;
+#pragma unroll
+        for (int k = 0; k < 8; ++k) {
+            const int i = threadIdx.x + k * blockDim.x;
+            v[k] = i < cols ? bf16_to_f32(row[i]) : 0.0f;
+            wv[k] = i < cols ? w[i] : 0.0f;
+            s += (double)v[k] * (double)v[k];
+        }
+        s = block_sum_f64(s, red);
+        const float sc = pi_inv_sqrt((float)(s / cols) + eps);
+#pragma unroll
+        for (int k = 0; k < 8; ++k) { const int i = threadIdx.x + k * blockDim.x; if (i < cols) out[i] = v[k] * sc * wv[k]; }
+        return;
+    }
     const float sc = row_rms_scale(cols, eps, red, [&](int i) { return bf16_to_f32(row[i]); });
-    for (int i = threadIdx.x; i < cols; i += blockDim.x) x[(size_t)blockIdx.x * cols + i] = bf16_to_f32(row[i]) * sc * w[i];
+    for (int i = threadIdx.x; i < cols; i += blockDim.x) out[i] = bf16_to_f32(row[i]) * sc * w[i];
 }
 
 template <typename ST>
@@ -288,7 +305,7 @@ extern "C" {
 
 int pi_k_embed_norm(const void * table, int cols, const int32_t * tokens, int T, const float * w, float eps, float * x, pi_stream_t stream) {
     if (!table || !tokens || !w || !x || cols <= 0 || T <= 0) return pi::fail(PI_E_ARG, "pi_k_embed_norm: bad arguments");
-    hipLaunchKernelGGL(embed_norm_kernel, dim3(T), dim3(256), 0, (hipStream_t)stream, (const uint16_t *)table, cols, tokens, w, eps, x);
+    hipLaunchKernelGGL(embed_norm_kernel, dim3(T), dim3(cols > 2048 ? 1024 : 256), 0, (hipStream_t)stream, (const uint16_t *)table, cols, tokens, w, eps, x);
     return pi::check_launch("pi_k_embed_norm");
 }
 

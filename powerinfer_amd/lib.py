@@ -198,8 +198,7 @@ _SIGS = {
     "pi_k_layer_step_supported": (_i, [_i, _i, _i]),
     "pi_k_latent_step": (_i, [C.POINTER(LatentPrep), _vp, _vp, _i, _i, _i, _i, _vp, _vp, _vp, _vp]),
     "pi_k_latent_attn_parts": (_i, [C.POINTER(LatentAttn), _vp]),
-    "pi_k_latent_value_step": (_i, [C.POINTER(LatentAttn), _vp, _i, _vp, _i, _vp]),
-    "pi_k_expert_up_step": (_i, [_vp, _i, _i, _i, _vp, _vp, _vp, _i, _i, _vp, _i, _vp]),
+    "pi_k_value_up_step": (_i, [C.POINTER(LatentAttn), _vp, _i, _vp, _i, _vp, _i, _i, _i, _vp, _vp, _vp, _i, _vp, _i, _vp]),
     "pi_k_layer_out_step": (_i, [C.POINTER(LayerOut), _vp]),
     "pi_k_pad_cols_bf16": (_i, [_vp, C.c_int64, _i, _vp, _i, _vp]),
     "pi_k_transpose_pad_bf16": (_i, [_vp, _i, _i, _i, _vp, _i, _vp]),
