@@ -752,13 +752,17 @@ static int ensure_pool(pi_model * m, int64_t n) {
 // tokens at n_past .. of sequence q, behind exactly n_past cells (what lies at n_past and beyond is dropped first)
 static int continue_at(pi_model * m, int q, int n_past) {
     LayerState * s = m->lay;
-    s->kv.seq_rm(q, n_past, -1);
     std::vector<int32_t> app;
     refresh_list(s, q, app);
     PI_TRY(upload_appends(m, app));
     const auto & lp = s->list_pos[q];
-    if ((int)lp.size() != n_past || (n_past && (lp.front() != 0 || lp.back() != n_past - 1))) return fail(PI_E_STATE, "the sequence's cells do not hold the positions 0 .. n_past - 1");
-    return PI_OK;
+    const int before = (int)(std::lower_bound(lp.begin(), lp.end(), n_past) - lp.begin());
+    if (before != n_past || (n_past && (lp[0] != 0 || lp[n_past - 1] != n_past - 1))) return fail(PI_E_STATE, "the sequence's cells do not hold the positions 0 .. n_past - 1");
+    if ((int)lp.size() == before) return PI_OK;
+    s->kv.seq_rm(q, n_past, -1);
+    app.clear();
+    refresh_list(s, q, app);
+    return upload_appends(m, app);
 }
 
 int layers_decode(pi_model * m, const int32_t * tokens, int n_tokens, int n_past, float * logits_out) {

@@ -64,9 +64,9 @@ def latent_attention(h, pos, c, k_rot, kpos, t, cfg):
 
 
 def route(h, w_router, correction, top, groups, keep):
-    """(chosen expert ids [n, top] by falling choice score, their weights)."""
+    """(chosen expert ids [n, top] by falling choice score, their weights).  route.margins: per token, how far the closest decision was."""
     s = 1.0 / (1.0 + np.exp(-(h @ w_router.T)))
-    ids, wts = [], []
+    ids, wts, margins = [], [], []
     for row in s:
         choice = row + correction
         size = choice.size // groups
@@ -75,9 +75,16 @@ def route(h, w_router, correction, top, groups, keep):
         open_ = np.full(choice.size, -np.inf)
         for g in kept:
             open_[g * size:(g + 1) * size] = choice[g * size:(g + 1) * size]
-        e = np.argsort(-open_, kind="stable")[:top]
+        order = np.argsort(-open_, kind="stable")
+        e = order[:top]
+        gaps = [open_[order[top - 1]] - open_[order[top]]] if top < choice.size else [np.inf]
+        if keep < groups:
+            by = np.sort(best)[::-1]
+            gaps.append(by[keep - 1] - by[keep])
+        margins.append(min(gaps))
         ids.append(e)
         wts.append(row[e] / (row[e].sum() + 1e-20))
+    route.margins = np.asarray(margins)
     return np.asarray(ids), np.asarray(wts)
 
 
@@ -107,6 +114,7 @@ class PlainModel:
         self.kv = {}
         self.n = 0
         self.streams = []
+        self.margins = np.empty(0)                   # closest routing decision of every token so far
 
     def _mix(self, i, h, pos):
         m, p = self.c["layers"][i]["mixer"], f"l{i}.mix."
@@ -135,11 +143,14 @@ class PlainModel:
         self.n += len(tokens)
         x = rms_norm_zero(self.t["embed"][np.asarray(tokens)], self.t["embed.norm"], eps)
         self.streams = []
+        margins = np.full(len(tokens), np.inf)
         for i in range(len(self.c["layers"])):
             a = rms_norm_zero(x, self.t[f"l{i}.norm1"], eps)
             y = self._mix(i, a, pos)
             if self.c["layers"][i]["mlp"] is not None:
                 y = y + self._ff(i, rms_norm_zero(x, self.t[f"l{i}.norm2"], eps))
+                margins = np.minimum(margins, getattr(route, "margins", margins))
             x = x + y
             self.streams.append(x)
+        self.margins = np.concatenate([self.margins, margins])
         return rms_norm_zero(x, self.t["final.norm"], eps) @ self.t["head"].T * self.c["logit_scale"]
