@@ -91,24 +91,40 @@ __global__ __launch_bounds__(256) void latent_attn_bf16_kernel(pi_latent_attn p)
     // thread's pieces of a cell tile
     pi_u32x4 pre[PF];
     int pn[PF], pc[PF];
+    const int step_n = 256 / pieces, step_c = 256 - step_n * pieces;
 #pragma unroll
-    for (int j = 0; j < PF; ++j) { const int c = tid + 256 * j; pn[j] = c / pieces; pc[j] = (c % pieces) * 8; }
+    for (int j = 0; j < PF; ++j) {                   // piece tid + 256 j: row and place within it, by carrying instead of dividing
+        if (j == 0) { pn[0] = tid / pieces; pc[0] = tid - pn[0] * pieces; continue; }
+        const int c = pc[j - 1] + step_c, over = c >= pieces ? 1 : 0;
+        pc[j] = c - (over ? pieces : 0);
+        pn[j] = pn[j - 1] + step_n + over;
+    }
+    // pieces past the tile repeat its last row: loads and stores stay unconditional (a guarded load makes the compiler wait for all of
+    // them one by one), and what is stored twice is the same
+#pragma unroll
+    for (int j = 0; j < PF; ++j) { pn[j] = min(pn[j], NC - 1); pc[j] *= 8; }
     const uint16_t * cache = (const uint16_t *)p.cache;
-    auto fetch = [&](int cb) {
+    // a tile's cells are looked up one tile before its rows are requested, the rows one tile before they are used
+    int idx[PF];
+    auto look_up = [&](int cb) {
 #pragma unroll
-        for (int j = 0; j < PF; ++j)
-            if (pn[j] < NC) pre[j] = pi_ld16(cache + (size_t)list[min(cb + pn[j], n_all - 1)] * p.kd + pc[j]);
+        for (int j = 0; j < PF; ++j) idx[j] = list[min(cb + pn[j], n_all - 1)];
     };
+    auto fetch = [&]() {
+#pragma unroll
+        for (int j = 0; j < PF; ++j) pre[j] = pi_ld16(cache + (size_t)idx[j] * p.kd + pc[j]);
+    };
+    if (c0 < c1) look_up(c0);
     // the query rows travel with the first cells: as many pieces per thread as a cell tile has (R == NC rows)
     static_assert(R == NC, "query and cell tiles share the piece layout");
     pi_u32x4 qr[PF];
 #pragma unroll
     for (int j = 0; j < PF; ++j)
-        if (pn[j] < R) qr[j] = pi_ld16((const uint16_t *)p.q_lat + (qrow0 + min(pn[j], rows - 1)) * p.kd + pc[j]);
-    if (c0 < c1) fetch(c0);
+        qr[j] = pi_ld16((const uint16_t *)p.q_lat + (qrow0 + min(pn[j], rows - 1)) * p.kd + pc[j]);
+    if (c0 < c1) { fetch(); look_up(c0 + NC); }
 #pragma unroll
     for (int j = 0; j < PF; ++j)
-        if (pn[j] < R) *reinterpret_cast<pi_u32x4 *>(qs + pn[j] * stride + pc[j] * 2) = qr[j];
+        *reinterpret_cast<pi_u32x4 *>(qs + pn[j] * stride + pc[j] * 2) = qr[j];
     if (tid < R) { row_m[tid] = -INFINITY; row_l[tid] = 0.0f; row_n[tid] = tid < rows ? p.n_vis[tok0 + (first + tid) / p.n_head] : 0; }
     pi_f4 acc[RT][VT];
 #pragma unroll
@@ -120,16 +136,37 @@ __global__ __launch_bounds__(256) void latent_attn_bf16_kernel(pi_latent_attn p)
         __syncthreads();                                         // the previous tile's readers are done (first pass: nothing to wait for)
 #pragma unroll
         for (int j = 0; j < PF; ++j)
-            if (pn[j] < NC) *reinterpret_cast<pi_u32x4 *>(ks + pn[j] * stride + pc[j] * 2) = pre[j];
+            *reinterpret_cast<pi_u32x4 *>(ks + pn[j] * stride + pc[j] * 2) = pre[j];
         __syncthreads();
-        if (cb + NC < c1) fetch(cb + NC);
+        fetch();                                                 // past the last tile: rows of the last cell, not used
+        look_up(cb + 2 * NC);
         // scores: RT x 2 pairs of (row tile, cell tile) over four waves
         for (int pr = wave; pr < RT * 2; pr += 4) {
             const int rt = pr >> 1, ct = pr & 1;
-            pi_f4 s = pi_f4{0, 0, 0, 0};
+            pi_f4 s = pi_f4{0, 0, 0, 0}, s2 = s;
             const unsigned char * qa = qs + (rt * 16 + i) * stride + g * 16, * kb = ks + (ct * 16 + i) * stride + g * 16;
-            for (int k = 0; k < p.kd * 2; k += 64)
+            // four 32-column steps at a time: their operands are read while the previous four are multiplied
+            const int n4 = p.kd / 128;
+            pi_u32x4 fa[2][4], fb[2][4];
+            auto read4 = [&](pi_u32x4 (&a)[4], pi_u32x4 (&b)[4], int k) {
+#pragma unroll
+                for (int u = 0; u < 4; ++u) { a[u] = *reinterpret_cast<const pi_u32x4 *>(qa + k * 256 + u * 64); b[u] = *reinterpret_cast<const pi_u32x4 *>(kb + k * 256 + u * 64); }
+            };
+            auto mul4 = [&](const pi_u32x4 (&a)[4], const pi_u32x4 (&b)[4]) {
+                s = mfma_bf16(a[0], b[0], s); s2 = mfma_bf16(a[1], b[1], s2); s = mfma_bf16(a[2], b[2], s); s2 = mfma_bf16(a[3], b[3], s2);
+            };
+            if (n4 > 0) read4(fa[0], fb[0], 0);
+            for (int k = 0; k < n4; k += 2) {
+                if (k + 1 < n4) read4(fa[1], fb[1], k + 1);
+                mul4(fa[0], fb[0]);
+                if (k + 1 < n4) {
+                    if (k + 2 < n4) read4(fa[0], fb[0], k + 2);
+                    mul4(fa[1], fb[1]);
+                }
+            }
+            for (int k = n4 * 256; k < p.kd * 2; k += 64)
                 s = mfma_bf16(*reinterpret_cast<const pi_u32x4 *>(qa + k), *reinterpret_cast<const pi_u32x4 *>(kb + k), s);
+            s += s2;
             const int cell = cb + ct * 16 + i;
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
@@ -193,21 +230,32 @@ __global__ __launch_bounds__(256) void latent_attn_bf16_kernel(pi_latent_attn p)
         }
     }
     __syncthreads();
+    // the sums leave through LDS (queries and cells are done with), so that the stores are whole lines and the code is short
+    float * os = reinterpret_cast<float *>(smem);                // [R][rank_ld]
 #pragma unroll
     for (int rt = 0; rt < RT; ++rt)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            const int row = rt * 16 + 4 * g + r;
-            if (row >= rows) continue;
-            const float f = whole ? row_a[row] : 1.0f;
+        for (int v = 0; v < VT; ++v) {
+            const int col = (wave * VT + v) * 16 + i;
+            if (col >= p.rank_ld) continue;
+            float * d = os + (rt * 16 + 4 * g) * p.rank_ld + col;
 #pragma unroll
-            for (int v = 0; v < VT; ++v) {
-                const int col = (wave * VT + v) * 16 + i;
-                if (col >= p.rank_ld) continue;
-                if (whole) ((bf16 *)p.out_lat)[(qrow0 + row) * p.rank_ld + col] = (bf16)(acc[rt][v][r] * f);
-                else p.scratch[((qrow0 + row) * p.n_parts + part) * p.rank_ld + col] = acc[rt][v][r];
+            for (int r = 0; r < 4; ++r) d[r * p.rank_ld] = acc[rt][v][r];
+        }
+    __syncthreads();
+    const int quads = p.rank_ld / 4;
+    for (int r = wave; r < rows; r += 4) {                       // a wave per row
+        const float f = whole ? row_a[r] : 1.0f;
+        for (int c = lane; c < quads; c += 64) {
+            const float4 v = *reinterpret_cast<const float4 *>(os + r * p.rank_ld + c * 4);
+            if (whole) {
+                const bf16 b[4] = {(bf16)(v.x * f), (bf16)(v.y * f), (bf16)(v.z * f), (bf16)(v.w * f)};
+                *reinterpret_cast<pi_u32x2 *>((bf16 *)p.out_lat + (qrow0 + r) * p.rank_ld + c * 4) = __builtin_bit_cast(pi_u32x2, b);
+            } else {
+                *reinterpret_cast<float4 *>(p.scratch + ((qrow0 + r) * p.n_parts + part) * p.rank_ld + c * 4) = v;
             }
         }
+    }
 }
 
 // the parts of one row and the sink: fixed order
@@ -313,13 +361,13 @@ __global__ __launch_bounds__(256, 2) void latent_expanded_attn_kernel(pi_latent_
         for (int j = 0; j < KP; ++j) {
             const int e = tid + 256 * j, key = min(k0 + e / (KS * 4), n_keys - 1), c = (e % (KS * 4)) * 8;
             const bf16 * src = c < p.dim ? (const bf16 *)p.keys + ((size_t)key * p.n_head + h) * p.dim + c
-                                         : (const bf16 *)p.cache + (size_t)p.list[key] * p.kd + p.rank_ld + (c - p.dim);
-            kr[j] = c < dk ? pi_ld16(src) : pi_u32x4{0, 0, 0, 0};
+                                         : (const bf16 *)p.cache + (size_t)p.list[key] * p.kd + p.rank_ld + (min(c, dk - 8) - p.dim);
+            kr[j] = pi_ld16(src);                      // (unconditional loads: past the end of a row its last piece, zeroed on the way to LDS)
         }
 #pragma unroll
         for (int j = 0; j < VP; ++j) {
-            const int e = tid + 256 * j, key = min(k0 + e / (VT * 2), n_keys - 1), c = (e % (VT * 2)) * 8;
-            vr[j] = c < p.vdim ? pi_ld16((const bf16 *)p.values + ((size_t)key * p.n_head + h) * p.vdim + c) : pi_u32x4{0, 0, 0, 0};
+            const int e = tid + 256 * j, key = min(k0 + e / (VT * 2), n_keys - 1), c = min((e % (VT * 2)) * 8, p.vdim - 8);
+            vr[j] = pi_ld16((const bf16 *)p.values + ((size_t)key * p.n_head + h) * p.vdim + c);
         }
     };
     fetch(0);
@@ -332,11 +380,11 @@ __global__ __launch_bounds__(256, 2) void latent_expanded_attn_kernel(pi_latent_
     for (int k0 = 0; k0 < n_keys; k0 += kXKeys) {
         __syncthreads();
 #pragma unroll
-        for (int j = 0; j < KP; ++j) { const int e = tid + 256 * j; *reinterpret_cast<pi_u32x4 *>(ks + (e / (KS * 4)) * KROW + (e % (KS * 4)) * 16) = kr[j]; }
+        for (int j = 0; j < KP; ++j) { const int e = tid + 256 * j; *reinterpret_cast<pi_u32x4 *>(ks + (e / (KS * 4)) * KROW + (e % (KS * 4)) * 16) = (e % (KS * 4)) * 8 < dk ? kr[j] : pi_u32x4{0, 0, 0, 0}; }
 #pragma unroll
         for (int j = 0; j < VP; ++j) { const int e = tid + 256 * j; *reinterpret_cast<pi_u32x4 *>(vs + (e / (VT * 2)) * VROW + (e % (VT * 2)) * 16) = vr[j]; }
         __syncthreads();
-        if (k0 + kXKeys < n_keys) fetch(k0 + kXKeys);
+        fetch(k0 + kXKeys);
         pi_f4 s[2][4];
 #pragma unroll
         for (int kt = 0; kt < 4; ++kt) {

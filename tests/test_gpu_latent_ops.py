@@ -167,7 +167,7 @@ def test_sorted_experts_and_combine(t, T, E, top, tile):
     assert np.abs(got - want).max() <= tol(t) * np.abs(want).max() and np.array_equal(got, keep.download(np.float32).reshape(T, D))
 
 
-@pytest.mark.parametrize("E,top,G,keep", [(8, 2, 4, 3), (6, 2, 3, 1), (64, 6, 8, 4), (5, 5, 1, 1), (160, 6, 8, 3), (4, 2, 4, 2), (300, 8, 1, 1)])
+@pytest.mark.parametrize("E,top,G,keep", [(10, 2, 5, 3), (6, 2, 3, 1), (64, 6, 8, 4), (5, 5, 1, 1), (160, 6, 8, 3), (4, 2, 4, 2), (300, 8, 1, 1)])
 def test_route(E, top, G, keep):
     L, rng = pl.init(), np.random.default_rng(E)
     T = 33
@@ -307,7 +307,7 @@ def test_sinks_of_any_size(t):
         assert np.abs(got - want).max() < (2e-2 if t == pl.BF16 else 1e-5) * max(np.abs(want).max(), 1e-3)
 
 
-@pytest.mark.parametrize("H,dim,rot,vdim,rank,T,start", [(2, 32, 16, 32, 64, 64, 0), (3, 64, 32, 64, 128, 130, 0), (9, 128, 64, 128, 64, 200, 77), (4, 160, 96, 72, 96, 70, 190), (5, 40, 8, 24, 40, 129, 63)])
+@pytest.mark.parametrize("H,dim,rot,vdim,rank,T,start", [(2, 32, 16, 32, 64, 64, 0), (3, 64, 48, 56, 120, 130, 0), (9, 128, 64, 128, 64, 200, 77), (4, 160, 96, 72, 96, 70, 190), (5, 40, 8, 24, 40, 129, 63)])
 def test_expanded_attention(H, dim, rot, vdim, rank, T, start):
     """A long run over expanded keys and values against the plain form and against the latent form."""
     L, t = pl.init(), pl.BF16
