@@ -612,14 +612,15 @@ PI_API int pi_k_latent_prep(int type, const pi_latent_prep * p, pi_stream_t stre
  * [(token, head)][rank_ld] = soft-max weighted latents, the denominator holding exp(sink[head]).  work [n_work]: {first token, first row
  * among (tokens behind it) x heads, rows, sequence} - at most pi_k_latent_attn_rows rows each
  * (PI_TYPE_F32: work [T] = each token's sequence, n_parts 1).  n_parts > 1: the cells of every item are
- * split over that many workgroups and merged (scratch: pi_k_latent_attn_scratch_floats). */
+ * split over that many workgroups and merged (scratch: pi_k_latent_attn_scratch_floats of n_work * pi_k_latent_attn_rows rows;
+ * pi_k_latent_attn_parts: of T * n_head rows). */
 typedef struct pi_latent_attn {
     const void * q_lat, * cache; const int32_t * lists; size_t list_ld; const int32_t * work, * n_vis;
     int32_t n_work, T, n_head, kv_rank, rank_ld, kd, n_parts; float scale; const float * sink; float * scratch; void * out_lat;
 } pi_latent_attn;
 PI_API int    pi_k_latent_attn_rows(int type);
 PI_API int    pi_k_latent_attn_supported(int type, int rank_ld, int kd);
-PI_API size_t pi_k_latent_attn_scratch_floats(int T, int n_head, int rank_ld, int n_parts);
+PI_API size_t pi_k_latent_attn_scratch_floats(int rows, int rank_ld, int n_parts);
 PI_API int    pi_k_latent_attn(int type, const pi_latent_attn * p, pi_stream_t stream);
 /* The same attention for a long run of tokens tok0 .. tok0 + T - 1 of one sequence (ascending n_vis), bf16, over expanded keys [cell][n_head * dim]
  * and values [cell][n_head * vdim] of the cells list[0 .. n_vis of the last token): att rows get each head's values (pi_k_latent_prep's

@@ -614,7 +614,7 @@ int layers_finalize(pi_model * m) {
         while (h < s->kinds.size() && memcmp(&s->kinds[h], &hk, sizeof hk)) ++h;
         if (h == s->kinds.size()) s->kinds.push_back(hk);
         L.hc = (int)h;
-        scratch = std::max(scratch, pi_k_latent_attn_scratch_floats(pi_k_latent_attn_rows(s->opts.compute) * kAttnItems, 1, L.rank_ld, 2) / 2);
+        scratch = std::max(scratch, pi_k_latent_attn_scratch_floats(kItemRows * kAttnItems / 2, L.rank_ld, 2));      // items x parts <= kAttnItems
         PI_TRY(layer_weights(m, (int)il));
     }
     if (bf16_mode(s)) {

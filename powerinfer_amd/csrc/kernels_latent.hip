@@ -69,8 +69,9 @@ __device__ __forceinline__ pi_u32x4 frag_cells(const unsigned char * rows, int s
     return pi_u32x4{lo.x, lo.y, hi.x, hi.y};
 }
 
+// by_item: parts are kept per work item (row = item * rows per item + row of the item) instead of per (token, head)
 template <int RT, int VT, int PF>      // row tiles; latent-column tiles per wave; 16-byte pieces of a cell tile per thread
-__global__ __launch_bounds__(256) void latent_attn_bf16_kernel(pi_latent_attn p) {
+__global__ __launch_bounds__(256) void latent_attn_bf16_kernel(pi_latent_attn p, int by_item) {
     constexpr int R = 16 * RT, NC = kLaCells, TPR = 256 / R, CPT = NC / TPR;      // threads per row and cells per thread of the soft-max
     extern __shared__ __align__(16) unsigned char smem[];
     const int stride = p.kd * 2 + 16, pieces = p.kd / 8;
@@ -84,6 +85,7 @@ __global__ __launch_bounds__(256) void latent_attn_bf16_kernel(pi_latent_attn p)
     const int4 item = reinterpret_cast<const int4 *>(p.work)[blockIdx.x];
     const int tok0 = item.x, first = item.y, rows = min(item.z, R), seq = item.w;
     const size_t qrow0 = (size_t)tok0 * p.n_head + first;        // row of q_lat / out_lat of this workgroup's first row
+    const size_t srow0 = by_item ? (size_t)blockIdx.x * R : qrow0;                         // and of the parts it leaves
     const int32_t * list = p.lists + (size_t)seq * p.list_ld;
     const int n_all = p.n_vis[tok0 + (first + rows - 1) / p.n_head];                       // cells of the last row's token: the most of all
     const int tiles = (n_all + NC - 1) / NC, part = blockIdx.y;
@@ -223,8 +225,8 @@ __global__ __launch_bounds__(256) void latent_attn_bf16_kernel(pi_latent_attn p)
             const float sink = p.sink[(first + tid) % p.n_head], m = fmaxf(row_m[tid], sink), a = row_m[tid] == -INFINITY ? 0.0f : expf(row_m[tid] - m);
             row_a[tid] = a / (row_l[tid] * a + expf(sink - m));
         } else {
-            float * ml = p.scratch + (size_t)p.T * p.n_head * p.n_parts * p.rank_ld;
-            const size_t o = ((qrow0 + tid) * p.n_parts + part) * 2;
+            float * ml = p.scratch + (by_item ? (size_t)p.n_work * R : (size_t)p.T * p.n_head) * p.n_parts * p.rank_ld;
+            const size_t o = ((srow0 + tid) * p.n_parts + part) * 2;
             ml[o] = row_m[tid];
             ml[o + 1] = row_l[tid];
         }
@@ -252,17 +254,20 @@ __global__ __launch_bounds__(256) void latent_attn_bf16_kernel(pi_latent_attn p)
                 const bf16 b[4] = {(bf16)(v.x * f), (bf16)(v.y * f), (bf16)(v.z * f), (bf16)(v.w * f)};
                 *reinterpret_cast<pi_u32x2 *>((bf16 *)p.out_lat + (qrow0 + r) * p.rank_ld + c * 4) = __builtin_bit_cast(pi_u32x2, b);
             } else {
-                *reinterpret_cast<float4 *>(p.scratch + ((qrow0 + r) * p.n_parts + part) * p.rank_ld + c * 4) = v;
+                *reinterpret_cast<float4 *>(p.scratch + ((srow0 + r) * p.n_parts + part) * p.rank_ld + c * 4) = v;
             }
         }
     }
 }
 
-// the parts of one row and the sink: fixed order
+// the parts of one row of a work item and the sink: fixed order
 __global__ __launch_bounds__(128) void latent_merge_kernel(pi_latent_attn p) {
-    const size_t row = blockIdx.x;
-    const float * ml = p.scratch + (size_t)p.T * p.n_head * p.n_parts * p.rank_ld + row * p.n_parts * 2;
-    const float * acc = p.scratch + row * p.n_parts * p.rank_ld;
+    const int4 item = reinterpret_cast<const int4 *>(p.work)[blockIdx.x / kLaRows];
+    const int r = blockIdx.x % kLaRows;
+    if (r >= item.z) return;
+    const size_t row = (size_t)item.x * p.n_head + item.y + r, srow = blockIdx.x;
+    const float * ml = p.scratch + (size_t)p.n_work * kLaRows * p.n_parts * p.rank_ld + srow * p.n_parts * 2;
+    const float * acc = p.scratch + srow * p.n_parts * p.rank_ld;
     const float sink = p.sink[row % p.n_head];
     float m = sink;
     for (int s = 0; s < p.n_parts; ++s) m = fmaxf(m, ml[2 * s]);
@@ -488,14 +493,14 @@ size_t attn_lds(int rt, int kd) {
     return (size_t)(R + kLaCells) * stride + 4 * (size_t)(R * (kLaCells + 1) + (R * (kLaCells + 1)) % 4) + 2 * (size_t)R * (kLaCells + 8) + 16 * (size_t)R;
 }
 
-template <int RT, int VT, int PF> int launch_attn(const pi_latent_attn * p, hipStream_t st) {
+template <int RT, int VT, int PF> int launch_attn(const pi_latent_attn * p, int by_item, hipStream_t st) {
     const size_t lds = attn_lds(RT, p->kd);
     static bool raised = false;
     if (!raised) {
         PI_HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void *>(&latent_attn_bf16_kernel<RT, VT, PF>), hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024));
         raised = true;
     }
-    hipLaunchKernelGGL((latent_attn_bf16_kernel<RT, VT, PF>), dim3(p->n_work, p->n_parts), dim3(256), lds, st, *p);
+    hipLaunchKernelGGL((latent_attn_bf16_kernel<RT, VT, PF>), dim3(p->n_work, p->n_parts), dim3(256), lds, st, *p, by_item);
     return pi::check_launch("pi_k_latent_attn");
 }
 
@@ -524,13 +529,13 @@ int pi_k_latent_attn_supported(int type, int rank_ld, int kd) {
     return type == PI_TYPE_F32 ? kd <= 8192 : (kd <= 1152 && attn_lds(kLaRows / 16, kd) <= 160 * 1024);
 }
 
-size_t pi_k_latent_attn_scratch_floats(int T, int n_head, int rank_ld, int n_parts) { return n_parts > 1 ? (size_t)T * n_head * n_parts * (rank_ld + 2) : 0; }
+size_t pi_k_latent_attn_scratch_floats(int rows, int rank_ld, int n_parts) { return n_parts > 1 ? (size_t)rows * n_parts * (rank_ld + 2) : 0; }
 
-static int attn_bf16(const pi_latent_attn * p, hipStream_t st) {
-    if (p->rank_ld <= 128 && p->kd <= 256) return launch_attn<2, 2, 4>(p, st);
-    if (p->rank_ld <= 256 && p->kd <= 384) return launch_attn<2, 4, 6>(p, st);
-    if (p->rank_ld <= 512 && p->kd <= 640) return launch_attn<2, 8, 10>(p, st);
-    return launch_attn<2, 16, 18>(p, st);
+static int attn_bf16(const pi_latent_attn * p, int by_item, hipStream_t st) {
+    if (p->rank_ld <= 128 && p->kd <= 256) return launch_attn<2, 2, 4>(p, by_item, st);
+    if (p->rank_ld <= 256 && p->kd <= 384) return launch_attn<2, 4, 6>(p, by_item, st);
+    if (p->rank_ld <= 512 && p->kd <= 640) return launch_attn<2, 8, 10>(p, by_item, st);
+    return launch_attn<2, 16, 18>(p, by_item, st);
 }
 
 static int attn_check(int type, const pi_latent_attn * p) {
@@ -543,7 +548,7 @@ static int attn_check(int type, const pi_latent_attn * p) {
 
 int pi_k_latent_attn_parts(const pi_latent_attn * p, pi_stream_t stream) {
     const int rc = attn_check(PI_TYPE_BF16, p);
-    return rc != PI_OK ? rc : attn_bf16(p, (hipStream_t)stream);
+    return rc != PI_OK ? rc : attn_bf16(p, 0, (hipStream_t)stream);
 }
 
 int pi_k_latent_attn(int type, const pi_latent_attn * p, pi_stream_t stream) {
@@ -554,9 +559,9 @@ int pi_k_latent_attn(int type, const pi_latent_attn * p, pi_stream_t stream) {
         hipLaunchKernelGGL(latent_attn_f32_kernel, dim3(p->T * p->n_head), dim3(256), sizeof(float) * (p->kd + kLfCells) + sizeof(int) * kLfCells, st, *p);
         return pi::check_launch("pi_k_latent_attn");
     }
-    rc = attn_bf16(p, st);
+    rc = attn_bf16(p, 1, st);
     if (rc != PI_OK || p->n_parts == 1) return rc;
-    hipLaunchKernelGGL(latent_merge_kernel, dim3(p->T * p->n_head), dim3(128), 0, st, *p);
+    hipLaunchKernelGGL(latent_merge_kernel, dim3(p->n_work * kLaRows), dim3(128), 0, st, *p);
     return pi::check_launch("pi_k_latent_attn merge");
 }
 

@@ -7,6 +7,7 @@
 
 namespace {
 
+constexpr int kRopePerWg = 512;           // rotated query pairs of a workgroup
 // Behind the joint projection: per head the absorbed query (64 latent rows a workgroup), per token the rotated query parts, the cell,
 // and the expert choice.
 __global__ __launch_bounds__(256) void latent_step_kernel(pi_latent_prep p, const uint16_t * __restrict__ uk_t, RouteArgs r, int n_absorb) {
@@ -20,13 +21,33 @@ __global__ __launch_bounds__(256) void latent_step_kernel(pi_latent_prep p, cons
         if (row0 >= p.kv_rank) return;
         const uint16_t * W = uk_t + ((size_t)h * p.kv_rank + min(row0 + i, p.kv_rank - 1)) * p.dim_ld + g * 8;
         const float * z = p.z + (size_t)min(i, p.T - 1) * p.ldz + h * hd;
+        const bool whole = p.dim % 8 == 0 && hd % 4 == 0 && p.ldz % 4 == 0;        // eight columns are two 16-byte loads
         pi_f4 acc = pi_f4{0, 0, 0, 0};
-        for (int k = 0; k < p.dim_ld; k += 32) {
-            const pi_u32x4 a = pi_ld16(W + k);
-            bf16 q[8];
+        for (int k0 = 0; k0 < p.dim_ld; k0 += 128) {          // four steps requested together, unguarded; what is past the end is zeroed
+            pi_u32x4 w[4];
+            float q[4][8];
 #pragma unroll
-            for (int j = 0; j < 8; ++j) { const int c = k + g * 8 + j; q[j] = (bf16)(c < p.dim ? z[c] : 0.0f); }
-            acc = mma16<bf16>(a, __builtin_bit_cast(pi_u32x4, q), acc);
+            for (int s = 0; s < 4; ++s) w[s] = pi_ld16(W + min(k0 + s * 32, p.dim_ld - 32));
+            if (whole) {
+#pragma unroll
+                for (int s = 0; s < 4; ++s) {
+                    const float4 * zp = reinterpret_cast<const float4 *>(z + min(k0 + s * 32 + g * 8, p.dim - 8));
+                    const float4 a = zp[0], c = zp[1];
+                    q[s][0] = a.x; q[s][1] = a.y; q[s][2] = a.z; q[s][3] = a.w; q[s][4] = c.x; q[s][5] = c.y; q[s][6] = c.z; q[s][7] = c.w;
+                }
+            } else {
+#pragma unroll
+                for (int s = 0; s < 4; ++s)
+#pragma unroll
+                    for (int j = 0; j < 8; ++j) q[s][j] = z[min(k0 + s * 32 + g * 8 + j, p.dim - 1)];
+            }
+#pragma unroll
+            for (int s = 0; s < 4; ++s) {
+                bf16 v[8];
+#pragma unroll
+                for (int j = 0; j < 8; ++j) v[j] = (bf16)(k0 + s * 32 + g * 8 + j < p.dim ? q[s][j] : 0.0f);
+                acc = mma16<bf16>(w[s], __builtin_bit_cast(pi_u32x4, v), acc);
+            }
         }
         if (i >= p.T) return;
         bf16 * o = (bf16 *)p.q_lat + ((size_t)i * p.n_head + h) * p.kd + row0 + 4 * g;
@@ -35,18 +56,26 @@ __global__ __launch_bounds__(256) void latent_step_kernel(pi_latent_prep p, cons
         return;
     }
     b -= n_absorb;
-    const int kinds = 1 + (p.cache ? 1 : 0) + (r.ids ? 1 : 0), t = b / kinds, what = b % kinds;
+    const int n_rope = (p.n_head * half + kRopePerWg - 1) / kRopePerWg, kinds = n_rope + (p.cache ? 1 : 0) + (r.ids ? 1 : 0), t = b / kinds, what = b % kinds;
     const float * z = p.z + (size_t)t * p.ldz;
     const float2 * cs = (const float2 *)p.cs + (size_t)t * half;
-    if (what == 0) {                                          // rotated query parts
-        for (int e = tid; e < p.n_head * half; e += 256) {
-            const int h = e / half, i = e % half;
-            const float u = z[h * hd + p.dim + 2 * i], v = z[h * hd + p.dim + 2 * i + 1];
-            bf16 * o = (bf16 *)p.q_lat + ((size_t)t * p.n_head + h) * p.kd + p.rank_ld + 2 * i;
-            o[0] = (bf16)(u * cs[i].x - v * cs[i].y);
-            o[1] = (bf16)(v * cs[i].x + u * cs[i].y);
+    if (what < n_rope) {                                      // rotated query parts
+        float u[kRopePerWg / 256], v[kRopePerWg / 256];
+        const int e0 = what * kRopePerWg + tid, last = p.n_head * half - 1;
+#pragma unroll
+        for (int k = 0; k < kRopePerWg / 256; ++k) {
+            const int e = min(e0 + k * 256, last), h = e / half, i = e - h * half;
+            u[k] = z[h * hd + p.dim + 2 * i]; v[k] = z[h * hd + p.dim + 2 * i + 1];
         }
-    } else if (what == 1 && p.cache) {                        // the token's cell
+#pragma unroll
+        for (int k = 0; k < kRopePerWg / 256; ++k) {
+            const int e = e0 + k * 256, h = e / half, i = e - h * half;
+            if (e > last) continue;
+            bf16 * o = (bf16 *)p.q_lat + ((size_t)t * p.n_head + h) * p.kd + p.rank_ld + 2 * i;
+            o[0] = (bf16)(u[k] * cs[i].x - v[k] * cs[i].y);
+            o[1] = (bf16)(v[k] * cs[i].x + u[k] * cs[i].y);
+        }
+    } else if (what == n_rope && p.cache) {                        // the token's cell
         const float * c = z + p.n_head * hd;
         bf16 * cell = (bf16 *)p.cache + (size_t)p.cell[t] * p.kd;
         double s = 0.0;
@@ -59,7 +88,7 @@ __global__ __launch_bounds__(256) void latent_step_kernel(pi_latent_prep p, cons
             cell[p.rank_ld + 2 * i] = (bf16)(u * cs[i].x - v * cs[i].y);
             cell[p.rank_ld + 2 * i + 1] = (bf16)(v * cs[i].x + u * cs[i].y);
         }
-    } else if (tid < 64) {                                    // the token's experts
+    } else {                                                  // the token's experts
         route_token(r, t, sm);
     }
 }
@@ -166,18 +195,18 @@ struct WaveStream {
 // The step's distinct experts in LDS: expert[k] in order of first appearance, slot[k][t] = token t's pair with it or -1.
 constexpr int kStepPairs = 256, kStepExperts = 2048;
 struct StepExperts {
-    int first[kStepExperts];
     int expert[kStepPairs], rank[kStepPairs], sred[16];
     int16_t slot[kStepPairs][16];
 };
-__device__ int step_experts(StepExperts & s, const int32_t * __restrict__ ids, int n, int top, int E) {
+// first: kStepExperts ints of LDS
+__device__ int step_experts(StepExperts & s, int * first, const int32_t * __restrict__ ids, int n, int top, int E) {
     const int tid = threadIdx.x, e = tid < n ? ids[tid] : 0;
-    for (int k = tid; k < E; k += blockDim.x) s.first[k] = n;
+    for (int k = tid; k < E; k += blockDim.x) first[k] = n;
     for (int k = tid; k < n * 8; k += blockDim.x) reinterpret_cast<int *>(s.slot)[k] = -1;
     __syncthreads();
-    if (tid < n) atomicMin(&s.first[e], tid);
+    if (tid < n) atomicMin(&first[e], tid);
     __syncthreads();
-    const int lead = tid < n ? s.first[e] : -1, own = lead == tid ? 1 : 0;
+    const int lead = tid < n ? first[e] : -1, own = lead == tid ? 1 : 0;
     int total;
     const int rank = block_exclusive_scan_i32(own, &total, s.sred);
     if (own) { s.expert[rank] = e; s.rank[tid] = rank; }
@@ -252,6 +281,9 @@ template <int NW>
 __global__ __launch_bounds__(64 * NW) void layer_out_step_kernel(pi_layer_out a) {
     __shared__ __align__(16) unsigned char tiles[NW][16 * kWsStride];
     __shared__ StepExperts se;
+    __shared__ int first[kStepExperts];
+    // (eight waves: the workgroup's LDS exceeds half a compute unit's, so that no two share one while others idle)
+    static_assert(NW < 8 || sizeof(tiles) + sizeof(se) + sizeof(first) > 80 * 1024, "one workgroup per compute unit");
     const int tid = threadIdx.x, wave = tid >> 6;
     const WaveStream ws(tiles[wave]);
     const int row0 = blockIdx.x * 16, n_o = (a.ld_att + 255) / 256, n_e = a.ids ? (a.ld_act + 255) / 256 : 1;
@@ -267,7 +299,7 @@ __global__ __launch_bounds__(64 * NW) void layer_out_step_kernel(pi_layer_out a)
     // the attention's pieces are requested before the experts are known
     if (wave < n_o) load(ld[0], wave);
     if (wave + NW < n_o) load(ld[1], wave + NW);
-    const int n_exp = a.ids ? step_experts(se, a.ids, a.T * a.top, a.top, a.n_expert) : 0, n_ss = n_o + n_exp * n_e;
+    const int n_exp = a.ids ? step_experts(se, first, a.ids, a.T * a.top, a.top, a.n_expert) : 0, n_ss = n_o + n_exp * n_e;
     if (wave >= n_o && wave < n_ss) load(ld[0], wave);
     if (wave + NW >= n_o && wave + NW < n_ss) load(ld[1], wave + NW);
     for (int s0 = wave; s0 < n_ss; s0 += 2 * NW) {
@@ -317,8 +349,8 @@ int pi_k_latent_step(const pi_latent_prep * p, const void * uk_t, const float * 
     if (ids && (!z_router || !bias || !weights || n_expert <= 0 || n_expert > kStepExperts || n_group <= 0 || n_expert % n_group || n_keep <= 0 || n_keep > n_group || n_top <= 0 ||
                 n_top > n_keep * (n_expert / n_group)))
         return pi::fail(PI_E_ARG, "pi_k_latent_step: bad routing arguments");
-    const int n_absorb = p->n_head * ((p->kv_rank + 63) / 64), kinds = 1 + (p->cache ? 1 : 0) + (ids ? 1 : 0);
-    hipLaunchKernelGGL(latent_step_kernel, dim3(n_absorb + p->T * kinds), dim3(256), ids ? route_lds_bytes(n_expert, n_group) : 0, (hipStream_t)stream, *p, (const uint16_t *)uk_t,
+    const int n_absorb = p->n_head * ((p->kv_rank + 63) / 64), kinds = (p->n_head * (p->rot_dim / 2) + kRopePerWg - 1) / kRopePerWg + (p->cache ? 1 : 0) + (ids ? 1 : 0);
+    hipLaunchKernelGGL(latent_step_kernel, dim3(n_absorb + p->T * kinds), dim3(256), ids ? route_lds_bytes(n_expert, n_group, n_top) : 0, (hipStream_t)stream, *p, (const uint16_t *)uk_t,
                        RouteArgs{z_router, n_expert, n_top, n_group, n_keep, bias, ids, weights}, n_absorb);
     return pi::check_launch("pi_k_latent_step");
 }
@@ -344,7 +376,10 @@ int pi_k_layer_out_step(const pi_layer_out * a, pi_stream_t stream) {
     if (!a || !a->x || !a->wo || !a->att || !a->out || a->rows <= 0 || a->T <= 0 || a->T > kBtMaxT || a->ld_att <= 0 || a->ld_att % 32 ||
         (a->ids && (!a->down || !a->act || a->ld_act <= 0 || a->ld_act % 32 || a->top <= 0 || a->T * a->top > kStepPairs || a->n_expert <= 0 || a->n_expert > kStepExperts)))
         return pi::fail(PI_E_ARG, "pi_k_layer_out_step: bad arguments");
-    hipLaunchKernelGGL(layer_out_step_kernel<8>, dim3((a->rows + 15) / 16), dim3(512), 0, (hipStream_t)stream, *a);
+    // eight waves a workgroup when every workgroup has a compute unit to itself, four (and several workgroups a unit) beyond
+    const int n = (a->rows + 15) / 16;
+    if (n <= pi::compute_units() ) hipLaunchKernelGGL(layer_out_step_kernel<8>, dim3(n), dim3(512), 0, (hipStream_t)stream, *a);
+    else hipLaunchKernelGGL(layer_out_step_kernel<4>, dim3(n), dim3(256), 0, (hipStream_t)stream, *a);
     return pi::check_launch("pi_k_layer_out_step");
 }
 

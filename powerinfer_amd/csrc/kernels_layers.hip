@@ -140,9 +140,9 @@ __global__ void rope_angles_kernel(const int32_t * __restrict__ pos, int T, int 
     cs[idx] = make_float2((float)c, (float)s);
 }
 
-// expert choice, one wave per token
-__global__ __launch_bounds__(64) void route_kernel(RouteArgs r) {
-    extern __shared__ float sm[];
+// expert choice, one workgroup per token
+__global__ __launch_bounds__(256) void route_kernel(RouteArgs r) {
+    extern __shared__ __align__(16) float sm[];
     route_token(r, blockIdx.x, sm);
 }
 
@@ -263,14 +263,32 @@ template <typename ST>
 __global__ __launch_bounds__(256) void moe_combine_kernel(const float * __restrict__ x, const float * __restrict__ mix, const ST * __restrict__ y,
                                                           const int32_t * __restrict__ inv, const float * __restrict__ weights, int top, int cols,
                                                           float * __restrict__ out, float * __restrict__ keep) {
-    const int t = blockIdx.y, c = blockIdx.x * 256 + threadIdx.x;
-    if (c >= cols) return;
-    const size_t o = (size_t)t * cols + c;
-    float s = 0.0f;
-    if (weights) for (int k = 0; k < top; ++k) s = fmaf(weights[(size_t)t * top + k], from_st(y[(size_t)inv[(size_t)t * top + k] * cols + c]), s);
-    const float v = x[o] + (mix[o] + s);
-    out[o] = v;
-    if (keep) keep[o] = v;
+    const int t = blockIdx.y, c0 = (blockIdx.x * 256 + threadIdx.x) * 4;
+    if (c0 >= cols) return;
+    if ((cols & 3) == 0) {                           // four columns a thread
+        const size_t o = (size_t)t * cols + c0;
+        float s[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+        if (weights) for (int k = 0; k < top; ++k) {
+            const float w = weights[(size_t)t * top + k];
+            struct alignas(4 * sizeof(ST)) Quad { ST v[4]; };
+            const Quad q = *reinterpret_cast<const Quad *>(y + (size_t)inv[(size_t)t * top + k] * cols + c0);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) s[j] = fmaf(w, from_st(q.v[j]), s[j]);
+        }
+        const float4 a = *reinterpret_cast<const float4 *>(x + o), b = *reinterpret_cast<const float4 *>(mix + o);
+        const float4 v = make_float4(a.x + (b.x + s[0]), a.y + (b.y + s[1]), a.z + (b.z + s[2]), a.w + (b.w + s[3]));
+        *reinterpret_cast<float4 *>(out + o) = v;
+        if (keep) *reinterpret_cast<float4 *>(keep + o) = v;
+        return;
+    }
+    for (int c = c0; c < min(c0 + 4, cols); ++c) {
+        const size_t o = (size_t)t * cols + c;
+        float s = 0.0f;
+        if (weights) for (int k = 0; k < top; ++k) s = fmaf(weights[(size_t)t * top + k], from_st(y[(size_t)inv[(size_t)t * top + k] * cols + c]), s);
+        const float v = x[o] + (mix[o] + s);
+        out[o] = v;
+        if (keep) keep[o] = v;
+    }
 }
 
 __global__ void pad_cols_kernel(const uint16_t * __restrict__ in, int64_t rows, int cols, uint16_t * __restrict__ out, int ld) {
@@ -294,7 +312,7 @@ __global__ void cells_advance_kernel(int T, const int32_t * __restrict__ seq, co
     if (t < T) {
         const int n = n_vis[t] + 1;
         n_vis[t] = n;
-        cell[t] = lists[(size_t)seq[t] * list_ld + n - 1];
+        cell[t] = lists[(size_t)seq[t] * list_ld + min((size_t)n, list_ld) - 1];        // (behind the last step of a full pool: not used)
     }
     if (t == 0) *step += 1;
 }
@@ -344,7 +362,7 @@ int pi_k_route(const float * z, int T, int n_expert, int n_top, int n_group, int
     if (!z || !bias || !ids || !weights || T <= 0 || n_expert <= 0 || n_expert > 4096 || n_top <= 0 || n_group <= 0 || n_expert % n_group || n_keep <= 0 || n_keep > n_group ||
         n_top > n_keep * (n_expert / n_group))
         return pi::fail(PI_E_ARG, "pi_k_route: bad arguments");
-    hipLaunchKernelGGL(route_kernel, dim3(T), dim3(64), route_lds_bytes(n_expert, n_group), (hipStream_t)stream, RouteArgs{z, n_expert, n_top, n_group, n_keep, bias, ids, weights});
+    hipLaunchKernelGGL(route_kernel, dim3(T), dim3(n_expert > 128 ? 256 : n_expert > 64 ? 128 : 64), route_lds_bytes(n_expert, n_group, n_top), (hipStream_t)stream, RouteArgs{z, n_expert, n_top, n_group, n_keep, bias, ids, weights});
     return pi::check_launch("pi_k_route");
 }
 
@@ -369,7 +387,7 @@ int pi_k_group_gemm_tile(const pi_group_gemm * g, int tile_n, pi_stream_t stream
 int pi_k_moe_combine(int type, const float * x, const float * mix, const void * y, const int32_t * inv, const float * weights, int n_top, int T, int cols,
                      float * out, float * keep, pi_stream_t stream) {
     if (!x || !mix || !out || T <= 0 || T > 65535 || cols <= 0 || (weights && (!y || !inv || n_top <= 0))) return pi::fail(PI_E_ARG, "pi_k_moe_combine: bad arguments");
-    const dim3 grid((cols + 255) / 256, T);
+    const dim3 grid((cols + 1023) / 1024, T);
     if (type == PI_TYPE_BF16) hipLaunchKernelGGL(moe_combine_kernel<bf16>, grid, dim3(256), 0, (hipStream_t)stream, x, mix, (const bf16 *)y, inv, weights, n_top, cols, out, keep);
     else hipLaunchKernelGGL(moe_combine_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream, x, mix, (const float *)y, inv, weights, n_top, cols, out, keep);
     return pi::check_launch("pi_k_moe_combine");

@@ -186,7 +186,7 @@ _SIGS = {
     "pi_k_latent_prep": (_i, [_i, C.POINTER(LatentPrep), _vp]),
     "pi_k_latent_attn_rows": (_i, [_i]),
     "pi_k_latent_attn_supported": (_i, [_i, _i, _i]),
-    "pi_k_latent_attn_scratch_floats": (_sz, [_i, _i, _i, _i]),
+    "pi_k_latent_attn_scratch_floats": (_sz, [_i, _i, _i]),
     "pi_k_latent_attn": (_i, [_i, C.POINTER(LatentAttn), _vp]),
     "pi_k_latent_expanded_supported": (_i, [_i, _i, _i]),
     "pi_k_latent_attn_expanded": (_i, [C.POINTER(LatentExpanded), _vp]),

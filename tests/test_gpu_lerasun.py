@@ -179,6 +179,23 @@ def test_long_steps_run_in_passes(compute):
     m.close()
 
 
+@pytest.mark.parametrize("compute", [pl.BF16, pl.F32])
+def test_a_decoded_token_beside_a_long_prompt(compute):
+    """A token far into its sequence (its cells split over workgroups) in one batch with a long run on expanded keys and values."""
+    orc = Oracle(even_config)
+    m = model(orc, compute, n_ctx=1024)
+    st = serve.Stepper(m, 760)
+    a, b = tokens(orc.cfg, 340, 1), tokens(orc.cfg, 400, 2)
+    st.run([("a", a[:330], [])])
+    got, _ = st.run([("a", a[330:331], [0]), ("b", b[:399], list(range(399)))])
+    check(got[:1], orc.logits(a)[330:331], compute)
+    check(got[1:], orc.logits(b)[:399], compute)
+    got, _ = st.run([("b", b[399:], [0]), ("a", a[331:], list(range(9)))])
+    check(got[:1], orc.logits(b)[399:], compute)
+    check(got[1:], orc.logits(a)[331:], compute)
+    m.close()
+
+
 def test_far_keys_in_prompts_and_decoding():
     """One layer in which token 32 + k looks for token 42 + k and for nothing else: that key decides the result hundreds of tokens back, at
     the first positions, at edges of 32- and 64-cell tiles - and not at all one position before it appears."""
