@@ -724,7 +724,7 @@ int layers_step(pi_model * m, const int32_t * tokens, const int32_t * positions,
             const int n = std::min(kHeadRows, (int)rows.size() - r0);
             const size_t V = m->hp.n_vocab;
             PI_TRY(pass_head(m, d_rows + r0, n));
-            if (next_tokens) for (int k = 0; k < n; ++k) PI_TRY(pi_k_argmax(s->logits + k * V, (int)V, s->d_next + k, m->stream));
+            if (next_tokens) for (int k = 0; k < n; k += 16) PI_TRY(pi_k_argmax_batch(s->logits + k * V, (int)V, std::min(16, n - k), s->d_next + k, nullptr, nullptr, nullptr, 0, m->stream));
             PI_HIP_TRY(hipStreamSynchronize(m->stream));
             std::vector<int32_t> nx(next_tokens ? n : 0);
             if (next_tokens) PI_TRY(pi_memcpy_d2h(nx.data(), s->d_next, 4 * (size_t)n));
