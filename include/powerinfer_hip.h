@@ -577,15 +577,24 @@ PI_API int pi_k_argmax(const float * logits, int n, int32_t * token_out, pi_stre
  * of 32 (ldw), vectors F32. */
 /* x[t] = rms_norm(table[tokens[t]]) * w */
 PI_API int pi_k_embed_norm(const void * table_bf16, int cols, const int32_t * tokens, int T, const float * w, float eps, float * x, pi_stream_t stream);
+/* x[t] = table[tokens[t]] * scale + bigram[row], row = (prev[t] * mul_prev + tokens[t] * mul_cur) mod buckets, or `buckets` where prev[t] < 0
+ * (bigram [buckets + 1][cols] may be NULL).  x0 (optional) receives a copy; carry != 0: prev[t] = tokens[t] afterwards */
+PI_API int pi_k_embed_bigram(const void * table_bf16, int cols, const int32_t * tokens, int32_t * prev, int T, float scale, const void * bigram_bf16,
+                             int32_t buckets, int64_t mul_prev, int64_t mul_cur, int carry, float * x, float * x0, pi_stream_t stream);
 /* two RMS norms of the same rows in one pass: out_a[t] = rms(x[t]) * wa, out_b[t] = rms(x[t]) * wb (wb, out_b may be NULL); rows of the
  * outputs are ld values apart.  rows (optional): row t of the outputs is made from x[rows[t]].  ol != 0 (BF16, T <= 16): outputs in the
  * operand layout of pi_k_gemm_bf16_ol over ld columns */
 PI_API int pi_k_norm_pair(int type, const float * x, const int32_t * rows, int T, int cols, float eps, const float * wa, void * out_a,
                           const float * wb, void * out_b, int ld, int ol, pi_stream_t stream);
+/* out[t] = layer_norm(x[t]) * w (no bias), out and ol as above; before that, and kept in x: x[t] += x0[t] (optional) and x[t] += step (optional,
+ * one row for every token) */
+PI_API int pi_k_layer_norm(int type, float * x, const int32_t * rows, int T, int cols, float eps, const float * w, const float * x0, const float * step,
+                           void * out, int ld, int ol, pi_stream_t stream);
 /* y = alpha * W x for several groups at once: group g multiplies W + g * w_gs with its own rows of x.  off == NULL: every group takes
  * the T rows x + g * x_gs + t * ldx into y + g * y_gs + t * ldy.  off != NULL (n_group + 1 offsets on the device): group g takes the
  * places s in [off[g], off[g + 1]) of a list; input row = gather ? gather[s] / gather_div : s, output row = s; T bounds the places of one group.
- * relu2: y = relu(.)^2.  y_f32: y is fp32 whatever `type` is.  Strides count elements. */
+ * relu2: y = relu(.)^2.  glu: rows 2 j and 2 j + 1 of W are gate and up row j, y has rows / 2 columns: the clamped GLU
+ * (pi_ffn_front).  y_f32: y is fp32 whatever `type` is.  Strides count elements. */
 typedef struct pi_group_gemm {
     const void * W; size_t w_gs; int32_t rows, cols, ldw, n_group;
     const void * x; size_t x_gs; int32_t ldx, T;
@@ -593,6 +602,7 @@ typedef struct pi_group_gemm {
     float alpha;
     const int32_t * off, * gather; int32_t gather_div;
     const int32_t * tiles, * n_tiles; int32_t max_tiles;      /* pi_k_group_gemm_tile with off: pi_k_moe_sort's list and an upper bound of its length */
+    int32_t glu; float glu_limit, glu_gain;
 } pi_group_gemm;
 PI_API int pi_k_group_gemm(int type, const pi_group_gemm * g, pi_stream_t stream);
 /* the same for many tokens, bf16, both operands tiled through LDS (cols % 64 == 0); tile_n 64 or 128 tokens per tile, as given to pi_k_moe_sort */
@@ -633,6 +643,62 @@ PI_API int pi_k_latent_expanded_supported(int dim, int rot_dim, int vdim);
 PI_API int pi_k_latent_attn_expanded(const pi_latent_expanded * p, pi_stream_t stream);
 /* rotates the shared key part (rot_dim values behind rank_ld) of cells by delta[cell] positions; cells with delta 0 are left alone */
 PI_API int pi_k_latent_shift(int type, void * cache, int n_cells, int kd, int rank_ld, int rot_dim, double base, const int32_t * delta, pi_stream_t stream);
+/* What a layer with one norm computes of its feed-forward straight from the joint projection z [T][ldz]: the clamped GLU of the rows at
+ * off_glu (gate and up row by row: g = min(z[2 j], limit), u = clamp(z[2 j + 1], -limit, limit), y = g * sigmoid(gain * g) * (u + 1)) times
+ * sigmoid(z[off_score]) (off_score < 0: times one) into act [T][ld_act], ff of them (0: none) and zeros up to ff_ld; and the choice of n_top
+ * of n_expert experts (0: none) from the logits at off_router: the largest logits (the lower index of a tie), weights their soft-max. */
+typedef struct pi_ffn_front {
+    int32_t off_glu, ff, ff_ld, off_score; float limit, gain; void * act; int32_t ld_act;
+    int32_t off_router, n_expert, n_top; int32_t * ids; float * weights;
+} pi_ffn_front;
+/* Grouped-query attention, behind the joint projection z [T][ldz] of its layer: queries at 0 (n_head x dim), keys at off_k (n_kv x dim), values at
+ * off_v (n_kv x vdim; off_v == off_k: the values are the keys as projected).  Queries and keys are rotated (pairs i, i + rot_dim / 2 of the
+ * first rot_dim values; cs as pi_k_rope_angles makes it) and, with unit != 0, divided by their root mean square; queries go to
+ * q [T][n_head][hd], the token's cell is n_kv rows [key | value] of hd values each, padded with zeros (pi_k_gqa_head_ld).  front (optional)
+ * runs in the same launch. */
+typedef struct pi_gqa_prep {
+    const float * z; int32_t ldz, T, n_head, n_kv, dim, vdim, rot_dim, off_k, off_v, hd, unit;
+    const void * cs; float eps; void * q, * cache; const int32_t * cell;
+} pi_gqa_prep;
+PI_API int pi_k_gqa_head_ld(int type, int dim, int vdim);                    /* hd for a head size, 0: not supported */
+PI_API int pi_k_gqa_prep(int type, const pi_gqa_prep * p, const pi_ffn_front * front, pi_stream_t stream);
+/* The attention itself.  bf16: work [n_work] = {first token, first row among (tokens behind it) x (n_head / n_kv), rows, sequence} of at most
+ * pi_k_gqa_rows(wide) rows; query row r sees the cells lists[seq][0 .. n_vis[its token]).  n_parts > 1: the cells are split over that many
+ * workgroups, partial sums in scratch (pi_k_gqa_scratch_floats).  fp32: work [T] = each token's sequence.  sink: score of an entry of the
+ * soft-max without a value (-INFINITY: none).  att [T][ld_att] gets n_head x vdim values per token.  pi_k_gqa_attn merges the parts,
+ * pi_k_gqa_attn_parts leaves them to pi_k_mix_up_step. */
+typedef struct pi_gqa_attn {
+    const void * q, * cache; const int32_t * lists; size_t list_ld; const int32_t * work, * n_vis;
+    int32_t n_work, T, n_head, n_kv, dim, vdim, hd, n_parts, wide; float scale, sink; float * scratch; void * att; int32_t ld_att;
+} pi_gqa_attn;
+PI_API int    pi_k_gqa_rows(int wide);
+PI_API size_t pi_k_gqa_scratch_floats(int n_work, int wide, int n_kv, int hd, int n_parts);
+PI_API int    pi_k_gqa_attn(int type, const pi_gqa_attn * p, pi_stream_t stream);
+PI_API int    pi_k_gqa_attn_parts(const pi_gqa_attn * p, pi_stream_t stream);
+/* rotates the key parts of cells by delta[cell] positions */
+PI_API int pi_k_gqa_shift(int type, void * cache, int n_cells, int n_kv, int hd, int rot_dim, double base, const int32_t * delta, pi_stream_t stream);
+/* Linear attention with a constant decay per head over a fp32 state [slot][n_head][dim][vdim], behind the joint projection z [T][ldz]: q = silu(z) at 0
+ * (n_head x dim), k = silu at off_k, v = silu at off_v (n_head x vdim); S = decay S + k v^T, o = S^T q.  runs [n_runs] = {first token, tokens,
+ * slot, 1 if the state starts at zero}: the consecutive tokens of one sequence.  o [T][n_head * vdim] fp32.
+ * pi_k_linear_step walks every run token by token; front (optional) runs in the same launch.
+ * pi_k_linear_prep + pi_k_linear_chunks (bf16) do the same for long runs in chunks of pi_k_linear_chunk() tokens: q, k [T][n_head][dim_ld] and
+ * v [T][n_head][vdim_ld] in bf16 (dim_ld a multiple of 32, vdim_ld of 64), then the states before every chunk (as sums of two bf16) into
+ * states (pi_k_linear_states_bytes) and the outputs.  chunks [n_chunks] = {first token, tokens, 1 if nothing lies before it}, a run's chunks
+ * behind one another; run r of `runs` begins with chunk first_chunk[r].  powers [n_head][chunk + 1]: decay^0 .. decay^chunk. */
+typedef struct pi_linear {
+    const float * z; int32_t ldz, T, n_head, dim, vdim, off_k, off_v;
+    const float * decay, * powers; float * state; const int32_t * runs; int32_t n_runs; float * o;
+    void * q, * k, * v, * states; int32_t dim_ld, vdim_ld, n_chunks; const int32_t * chunks, * first_chunk;
+} pi_linear;
+PI_API int    pi_k_linear_chunk(void);
+PI_API int    pi_k_linear_supported(int dim, int vdim);
+PI_API size_t pi_k_linear_states_bytes(int n_chunks, int n_head, int dim_ld, int vdim_ld);
+PI_API int    pi_k_linear_step(int type, const pi_linear * p, const pi_ffn_front * front, pi_stream_t stream);
+PI_API int    pi_k_linear_prep(int type, const pi_linear * p, const pi_ffn_front * front, pi_stream_t stream);
+PI_API int    pi_k_linear_chunks(const pi_linear * p, pi_stream_t stream);
+/* att[t][0 .. n) = rms_norm(o[t]) * w * sigmoid(z[t][off_gate ..]), o [T][n] */
+typedef struct pi_gate_norm { const float * o, * z, * w; int32_t ldz, off_gate, n, T; float eps; void * att; int32_t ld_att; } pi_gate_norm;
+PI_API int pi_k_gate_norm(int type, const pi_gate_norm * p, pi_stream_t stream);
 /* expert choice of T tokens from router logits z [T][n_expert] (see PI_FFN_MOE): ids, weights [T][n_top] by falling choice score */
 PI_API int pi_k_route(const float * z, int T, int n_expert, int n_top, int n_group, int n_keep, const float * bias, int32_t * ids, float * weights,
                       pi_stream_t stream);
@@ -661,15 +727,22 @@ PI_API int pi_k_latent_attn_parts(const pi_latent_attn * p, pi_stream_t stream);
 PI_API int pi_k_value_up_step(const pi_latent_attn * p, const void * uv, int vdim, void * att, int ld_att, const void * up, int n_expert, int ff, int cols,
                               const void * x_ol, const int32_t * ids, const float * weights, int top, void * act, int ld_act, pi_stream_t stream);
 PI_API int pi_k_layer_out_step(const pi_layer_out * a, pi_stream_t stream);
+/* Steps of up to 16 tokens (bf16): the merge of a split grouped-query attention (attn, n_parts > 1) or the gated norm of a linear attention
+ * (gate), and, with ids != NULL, act [T * top][ld_act] = weight * clamped GLU of up[e] x (up [n_expert * 2 * ff][cols], gate and up rows in
+ * turn) for every (token, choice), in one launch. */
+PI_API int pi_k_mix_up_step(const pi_gqa_attn * attn, const pi_gate_norm * gate, const void * up, int n_expert, int ff, int cols, float limit, float gain,
+                            const void * x_ol, int T, const int32_t * ids, const float * weights, int top, void * act, int ld_act, pi_stream_t stream);
 /* BF16 matrices: out [rows][ld] = in [rows][cols] padded with zeros; out [n_mat][cols][ld] = each in [rows][cols] transposed, padded with zeros */
 PI_API int pi_k_pad_cols_bf16(const void * in, int64_t rows, int cols, void * out, int ld, pi_stream_t stream);
+/* row r of in [rows][cols] becomes columns col0 .. col0 + width - 1 (zeros behind cols) of row row0 + r * row_step of out [..][ld] */
+PI_API int pi_k_place_bf16(const void * in, int64_t rows, int cols, void * out, int ld, int col0, int width, int64_t row0, int row_step, pi_stream_t stream);
 PI_API int pi_k_transpose_pad_bf16(const void * in, int n_mat, int rows, int cols, void * out, int ld, pi_stream_t stream);
 /* lockstep decoding on shared cells: after tokens and positions have moved on, n_vis[t] += 1 and cell[t] = lists[seq[t]][n_vis[t] - 1] */
 PI_API int pi_k_cells_advance(int T, const int32_t * seq, const int32_t * lists, size_t list_ld, int32_t * n_vis, int32_t * cell, int32_t * step, pi_stream_t stream);
 
 /* ---- decode loop with resident weights ------------------------------------------------------------- */
 
-enum { PI_ARCH_LLAMA = 0, PI_ARCH_FALCON = 1, PI_ARCH_LERASUN = 2 };
+enum { PI_ARCH_LLAMA = 0, PI_ARCH_FALCON = 1, PI_ARCH_LERASUN = 2, PI_ARCH_PIBALORN = 3 };
 
 /* the llama_hparams fields this path reads (llama.cpp:1207-1270) */
 typedef struct pi_hparams {
@@ -692,12 +765,21 @@ enum {
     PI_T_EMBD_NORM,
     PI_T_MIX_Q, PI_T_MIX_DKV, PI_T_MIX_DKV_NORM, PI_T_MIX_UK, PI_T_MIX_UV, PI_T_MIX_SINK,
     PI_T_ROUTER, PI_T_ROUTER_BIAS, PI_T_EXPERT_UP, PI_T_EXPERT_DOWN,
+    /* bigram table and the loop's step vectors (global); key, value and gate projections, the norm behind a linear attention (F32), its
+     * decays (F32); gate matrices of the experts; the dense or shared feed-forward and the shared one's score row */
+    PI_T_BIGRAM, PI_T_LOOP_STEP,
+    PI_T_MIX_K, PI_T_MIX_V, PI_T_MIX_G, PI_T_MIX_NORM, PI_T_MIX_DECAY,
+    PI_T_EXPERT_GATE, PI_T_GLU_GATE, PI_T_GLU_UP, PI_T_GLU_DOWN, PI_T_SHARED_SCORE,
     PI_T_COUNT
 };
 
 /*
- * Models whose layers are described one by one.  A layer is  x + (mixer(norm_a(x)) + ffn(norm_b(x)))  (both of the same x, each part
- * with its own RMS norm; tensors PI_T_ATTN_NORM and PI_T_FFN_NORM), or without the second part (PI_FFN_NONE).
+ * Models whose layers are described one by one.  A layer is  x + (mixer(norm_a(x)) + ffn(norm_b(x)))  (both of the same x; tensors
+ * PI_T_ATTN_NORM and PI_T_FFN_NORM), or without the second part (PI_FFN_NONE).  PI_MIXER_LATENT layers have two RMS norms, layers with
+ * the other mixers one layer norm (weight, no bias) that both parts share; a model has layers of one of the two families.
+ *
+ * Layers loop_start .. loop_stop - 1 run loop_times times in a row (each pass with a cache or state of its own).  Before every pass but the
+ * first the embedding is added to the residual stream, before every pass row t of PI_T_LOOP_STEP [loop_times][n_embd].
  *
  * PI_MIXER_LATENT: multi-head attention over a cached low-rank latent.  PI_T_MIX_Q [n_head * (dim + rot_dim)][n_embd] gives each head
  *   an unrotated and a rotated query part; PI_T_MIX_DKV [kv_rank + rot_dim][n_embd] gives the latent (RMS norm with PI_T_MIX_DKV_NORM
@@ -710,14 +792,26 @@ enum {
  *   n_group_keep of n_group groups (a group counts the sum of its two best), weights = the chosen scores over their sum;
  *   PI_T_EXPERT_UP [n_expert * expert_ff][n_embd] and PI_T_EXPERT_DOWN [n_expert * n_embd][expert_ff] hold the experts one behind the
  *   other, activation relu(z)^2.
+ *
+ * PI_MIXER_GROUPED: grouped-query attention of n_head query heads on n_kv_head key / value heads (PI_T_MIX_Q, PI_T_MIX_K, PI_T_WO; PI_T_MIX_V,
+ *   or, values_are_keys, the keys as projected).  Rotation of the first rot_dim values of a head, value i paired with i + rot_dim / 2,
+ *   frequency rot_base^(-2i / rot_dim); unit_qk: queries and keys are divided by their root mean square afterwards; scores times
+ *   `scale`; sink: the soft-max has one more entry, of this score and without a value (-INFINITY: none).
+ * PI_MIXER_LINEAR: linear attention with the decay PI_T_MIX_DECAY [n_head] (pi_linear; PI_T_MIX_Q, _K [n_head * dim], _V [n_head * vdim]), its output
+ *   RMS-normed over all heads with PI_T_MIX_NORM, times sigmoid(PI_T_MIX_G h), through PI_T_WO.
+ * PI_FFN_GLU: PI_T_GLU_GATE, _UP [glu_ff][n_embd], _DOWN [n_embd][glu_ff], the clamped GLU with glu_limit and glu_gain (pi_ffn_front).
+ * PI_FFN_GLU_MOE: PI_T_ROUTER; the n_top largest logits, weights their soft-max; PI_T_EXPERT_GATE, _UP, _DOWN as above with expert_limit;
+ *   glu_ff > 0: beside them a shared one (PI_T_GLU_*, glu_limit) that every token uses times sigmoid(PI_T_SHARED_SCORE [1][n_embd] h).
  */
-enum { PI_MIXER_LATENT = 0 };
-enum { PI_FFN_NONE = 0, PI_FFN_MOE = 1 };
+enum { PI_MIXER_LATENT = 0, PI_MIXER_GROUPED = 1, PI_MIXER_LINEAR = 2 };
+enum { PI_FFN_NONE = 0, PI_FFN_MOE = 1, PI_FFN_GLU = 2, PI_FFN_GLU_MOE = 3 };
 typedef struct pi_layer_desc {
     int32_t mixer, n_head, dim, rot_dim, vdim, kv_rank, kv_from;
     float   scale;
     double  rot_base;
     int32_t ffn, n_expert, n_top, n_group, n_group_keep, expert_ff;
+    int32_t n_kv_head, values_are_keys, unit_qk; float sink;
+    int32_t glu_ff; float glu_limit, expert_limit, glu_gain;
 } pi_layer_desc;
 typedef struct pi_layers_opts {
     int32_t compute;         /* PI_TYPE_BF16: activations and caches in bf16, fp32 accumulation (residual, norms, router, scores in fp32);
@@ -725,6 +819,12 @@ typedef struct pi_layers_opts {
     float   logit_scale;     /* logits are multiplied by this */
     float   norm_offset;     /* added to the weights of the model's own norms (1 for weights stored around zero); not to PI_T_MIX_DKV_NORM */
     int32_t max_batch;       /* most tokens the step buffers hold; longer steps run in several passes (0: 2048) */
+    /* models of the PI_MIXER_GROUPED / PI_MIXER_LINEAR family: embedding = table row * embed_scale + a row of PI_T_BIGRAM [buckets + 1][n_embd]
+     * (pi_k_embed_bigram; bigram_buckets 0: none), and the loop (loop_times 0: none) */
+    float   embed_scale;
+    int32_t bigram_buckets; int64_t bigram_mul_prev, bigram_mul_cur;
+    int32_t loop_start, loop_stop, loop_times;
+    int32_t n_slots;         /* sequences whose recurrent states there is room for at the start (0: 4; grows when more are live) */
 } pi_layers_opts;
 
 /* The ggml_cuda_* boundary (include/ggml_backend_abi.h) keeps single-token nodes in a window until it knows whether they form a block
@@ -859,7 +959,7 @@ PI_API int pi_model_batch_dense_layers(pi_model * m);
 PI_API int pi_model_set_rest_on_gpu(pi_model * m, int enable);
 PI_API int pi_model_set_capture(pi_model * m, int enable);
 /* with capture enabled, a model described layer by layer also keeps the residual stream behind every layer for the last pass of a step:
- * out [n_layer][n_tokens][n_embd]; returns n_tokens or a negative error (out may be NULL) */
+ * out [layer runs][n_tokens][n_embd] (a layer inside the loop counts once per pass); returns n_tokens or a negative error (out may be NULL) */
 PI_API int pi_model_get_streams(pi_model * m, float * out);
 PI_API int pi_model_get_capture(pi_model * m, float * ffn_out, float * pred_logits, int32_t * n_active, float * ffn_src);
 

@@ -459,6 +459,8 @@ int pi_model_set_tensor(pi_model * m, int layer, int kind, int type, const void 
     if (!m || !data || kind < 0 || kind >= PI_T_COUNT || ne0 <= 0 || ne1 <= 0) return pi::fail(PI_E_ARG, "pi_model_set_tensor: bad arguments");
     if (m->finalized) return pi::fail(PI_E_STATE, "pi_model_set_tensor: model already finalized");
     if (kind == PI_T_EMBD_NORM) return upload_tensor(m, m->embd_norm, type, data, ne0, ne1, on_device);
+    if (kind == PI_T_BIGRAM) return upload_tensor(m, m->bigram, type, data, ne0, ne1, on_device);
+    if (kind == PI_T_LOOP_STEP) return upload_tensor(m, m->loop_step, type, data, ne0, ne1, on_device);
     if (kind <= PI_T_OUTPUT) return upload_tensor(m, m->glob[kind], type, data, ne0, ne1, on_device);
     if (layer < 0 || layer >= m->hp.n_layer) return pi::fail(PI_E_ARG, "pi_model_set_tensor: layer out of range");
     Tensor & t = m->L(layer, kind);

@@ -906,6 +906,7 @@ KvCells * cells_of(pi_model * m) { return !m ? nullptr : m->lay ? pi::layers_cel
 int pi_model_kv_cells_seq_rm(pi_model * m, int seq, int p0, int p1) {
     KvCells * kv = cells_of(m);
     if (!kv || seq >= 32) return pi::fail(PI_E_ARG, "pi_model_kv_cells_seq_rm: bad arguments");
+    if (m->lay) PI_TRY(pi::layers_edit_allowed(m, [&](KvCells & c) { c.seq_rm(seq, p0, p1); }));
     kv->seq_rm(seq, p0, p1);
     return PI_OK;
 }
@@ -913,6 +914,7 @@ int pi_model_kv_cells_seq_rm(pi_model * m, int seq, int p0, int p1) {
 int pi_model_kv_cells_seq_cp(pi_model * m, int src, int dst, int p0, int p1) {
     KvCells * kv = cells_of(m);
     if (!kv || src < 0 || dst < 0 || src >= 32 || dst >= 32) return pi::fail(PI_E_ARG, "pi_model_kv_cells_seq_cp: bad arguments");
+    if (m->lay) PI_TRY(pi::layers_copy_state(m, src, dst, p0, p1));
     kv->seq_cp(src, dst, p0, p1);
     return PI_OK;
 }
@@ -927,6 +929,7 @@ int pi_model_kv_cells_seq_keep(pi_model * m, int seq) {
 int pi_model_kv_cells_seq_shift(pi_model * m, int seq, int p0, int p1, int delta) {
     KvCells * kv = cells_of(m);
     if (!kv || seq < 0 || seq >= 32) return pi::fail(PI_E_ARG, "pi_model_kv_cells_seq_shift: bad arguments");
+    if (m->lay) PI_TRY(pi::layers_edit_allowed(m, nullptr));
     kv->seq_shift(seq, p0, p1, delta);
     return PI_OK;
 }

@@ -8,6 +8,7 @@
 #include <hip/hip_runtime.h>
 #include <hip/hip_fp16.h>
 
+#include <functional>
 #include <unordered_map>
 #include <vector>
 
@@ -27,7 +28,7 @@ struct pi_model {
     pi_hparams hp{};
     std::vector<Tensor> layers;           // [n_layer][PI_T_COUNT]
     Tensor glob[4];
-    Tensor embd_norm;                     // PI_T_EMBD_NORM
+    Tensor embd_norm, bigram, loop_step;  // PI_T_EMBD_NORM, PI_T_BIGRAM, PI_T_LOOP_STEP
     LayerState * lay = nullptr;           // models described layer by layer (engine_layers.hip); null: the sparse LLaMA / Falcon token loop
     std::vector<void *> owned;            // every device allocation made by the model
     bool finalized = false, hybrid = false;
@@ -105,6 +106,8 @@ int  layers_batch_init(pi_model * m, int n_seq);
 int  layers_batch_decode(pi_model * m, const int32_t * tokens, const int32_t * positions, int32_t * next_tokens, float * logits_out);
 int  layers_generate(pi_model * m, int own, int n_steps, int32_t * out_tokens, float * ms_out);
 int  layers_seq_edit(pi_model * m, int seq /* -1: the model's own */, int p0, int p1, int delta, bool shift);
+int  layers_edit_allowed(pi_model * m, const std::function<void(KvCells &)> & edit);
+int  layers_copy_state(pi_model * m, int src, int dst, int p0, int p1);
 int  layers_seq_cp(pi_model * m, int src, int dst, int p0, int p1);
 
 int  kv_edit(pi_model * m, __half * k_cache, __half * v_cache, int32_t * d_pos, std::vector<int32_t> & kv_pos, int p0, int p1, int delta, bool shift);

@@ -20,20 +20,33 @@ constexpr int kMaxLockstep = 16;
 constexpr long long kExpandedValues = 1LL << 29;      // most expanded key and value numbers of one run (1 GiB)
 constexpr int kItemRows = 32;             // query rows of an attention work item
 constexpr int kAttnItems = 512;          // (work item, part) pairs a split attention aims at: two workgroups per compute unit
+constexpr int kWideRows = 64;            // query rows from which a run of grouped-query attention takes the wide work items
+constexpr int kLinearChunked = 17;       // tokens from which a run of linear attention is worked in chunks
 
 int up_to(int v, int m) { return (v + m - 1) / m * m; }
 
 struct Layer {
     pi_layer_desc d{};
     int nq = 0, z_rows = 0, dim_ld = 0, rank_ld = 0, kd = 0, hv_ld = 0, ff_ld = 0, rot = 0, hc = 0;      // rot, hc: index among the model's rotations / kinds of heads
+    int off_k = 0, off_v = 0, off_g = 0, off_glu = 0, off_score = -1, off_router = 0;      // rows of the joint projection (layers with one norm)
+    int hd = 0, vdim_ld = 0, glu_ld = 0, close_ld = 0;
     bool own_kv = true;
     const void *w_z = nullptr, *uk = nullptr, *uk_t = nullptr, *uv = nullptr, *wo = nullptr, *router = nullptr, *up = nullptr, *down = nullptr;
     const float *norm_a = nullptr, *norm_b = nullptr, *dkv_norm = nullptr, *sink = nullptr, *bias = nullptr;
-    void * cache = nullptr;
+    const float *mix_norm = nullptr, *decay = nullptr, *powers = nullptr;
+    // one per pass of the loop the layer is part of
+    std::vector<void *> cache;                         // cells
+    std::vector<float *> state;                        // [slots][n_head][dim][vdim]
+    size_t cell_values() const { return d.mixer == PI_MIXER_GROUPED ? (size_t)d.n_kv_head * 2 * hd : d.mixer == PI_MIXER_LATENT && own_kv ? (size_t)kd : 0; }
+    size_t state_floats() const { return d.mixer == PI_MIXER_LINEAR ? (size_t)d.n_head * d.dim * d.vdim : 0; }
+    bool moe() const { return d.ffn == PI_FFN_MOE || d.ffn == PI_FFN_GLU_MOE; }
 };
 
+struct LayerRun { int layer, pass; bool starts; };     // starts: a pass of the loop begins with it
+
 struct Rotation { int dims; double base; };
-struct HeadKind { int n_head, dim, rot_dim, vdim, rank_ld, kd; };
+// n_head: of a work item's rows - all heads on a latent, the heads of a group otherwise (n_kv groups, kd values of a key row)
+struct HeadKind { int mixer, n_head, n_kv, dim, rot_dim, vdim, rank_ld, kd; };
 
 // where a pass finds its tokens
 struct Step {
@@ -45,6 +58,12 @@ struct Step {
     // runs that attend over expanded keys and values
     std::vector<Work> work;
     std::vector<std::vector<Run>> runs;
+    // grouped-query attention: the long runs as wide work items (per kind); linear attention: the runs walked token by token and in chunks;
+    // prev: each token's predecessor (carry: the embedding moves it on, for a captured step)
+    std::vector<Work> wide;
+    int32_t * prev = nullptr; bool carry = false;
+    const int32_t *lin = nullptr, *lin_long = nullptr, *lin_first = nullptr, *lin_chunks = nullptr;
+    int n_lin = 0, n_lin_long = 0, n_lin_chunks = 0;
 };
 
 }  // namespace
@@ -58,8 +77,13 @@ struct LayerState {
     std::vector<HeadKind> kinds;
     int d_ld = 0, es = 2;
     const float *embd_norm = nullptr, *out_norm = nullptr;
-    const void *embed = nullptr, *head = nullptr;
+    const void *embed = nullptr, *head = nullptr, *bigram = nullptr;
+    const float * loop_step = nullptr;                 // [loop_times][n_embd]
+    std::vector<LayerRun> order;                       // the layer runs of a step
+    bool one_norm = false, recurrent = false;
+    int n_slots = 0, slot_of[32];                      // slots of recurrent states; -1: the sequence has none
     KvCells kv;
+    std::vector<int32_t> cell_tok;                     // the token of every cell
     bool auto_pool = false;                            // sized by the engine (decode, batch_init), not by the caller
     int32_t * lists = nullptr;                         // device [32][kv.n]: a sequence's cells in position order
     std::vector<int32_t> list_cells[32], list_pos[32]; // the same on the host
@@ -67,7 +91,8 @@ struct LayerState {
     // step buffers for `cap` tokens (one allocation)
     int cap = 0;
     unsigned char * arena = nullptr;
-    float *x = nullptr, *x2 = nullptr, *z = nullptr, *mix = nullptr, *rl = nullptr, *wts = nullptr;
+    float *x = nullptr, *x2 = nullptr, *x0 = nullptr, *z = nullptr, *mix = nullptr, *rl = nullptr, *wts = nullptr, *lin_o = nullptr;
+    void *lin_q = nullptr, *lin_k = nullptr, *lin_v = nullptr, *lin_states = nullptr;
     void *h_a = nullptr, *h_b = nullptr, *q_un = nullptr, *q_lat = nullptr, *o_lat = nullptr, *att = nullptr, *act = nullptr, *y_exp = nullptr;
     int32_t *ids = nullptr, *perm = nullptr, *inv = nullptr, *off = nullptr, *tiles = nullptr, *n_tiles = nullptr;
     std::vector<float *> cs;                           // per rotation [cap][dims / 2] (cos, sin)
@@ -79,7 +104,7 @@ struct LayerState {
     // lockstep decoding and the greedy loop
     int n_seq = 0;
     int32_t last_tok[32], last_pos[32];
-    int32_t *g_tok = nullptr, *g_pos = nullptr, *g_cell = nullptr, *g_vis = nullptr, *g_seq = nullptr, *g_work = nullptr, *g_step = nullptr, *g_out = nullptr;
+    int32_t *g_tok = nullptr, *g_pos = nullptr, *g_cell = nullptr, *g_vis = nullptr, *g_seq = nullptr, *g_work = nullptr, *g_step = nullptr, *g_out = nullptr, *g_prev = nullptr, *g_lin = nullptr;
     int max_steps = 4096;
     hipGraph_t graph = nullptr; hipGraphExec_t exec = nullptr;
     int graph_T = 0, graph_seq0 = -1; std::vector<int> graph_parts;
@@ -137,6 +162,108 @@ int norm_weights(pi_model * m, const Tensor & t, float offset, float factor, con
     PI_TRY(pi_memcpy_h2d(p, w.data(), sizeof(float) * w.size()));
     *out = p;
     return PI_OK;
+}
+
+// a matrix of the tensor's rows inside a larger one: rows row0, row0 + step, .., columns col0 .. col0 + width - 1
+int place(pi_model * m, Tensor & t, uint16_t * out, int ld, int col0, int width, int64_t row0, int step) {
+    PI_TRY(pi_k_place_bf16(t.dev, t.ne1, (int)t.ne0, out, ld, col0, width, row0, step, nullptr));
+    PI_TRY(pi_sync());
+    release(m, t);
+    return PI_OK;
+}
+
+uint16_t * zeroed(pi_model * m, size_t n) {
+    uint16_t * p = m->alloc<uint16_t>(n);
+    return p && pi_memset(p, 0, n * 2) == PI_OK ? p : nullptr;
+}
+
+// A layer with one norm: everything that reads the normed input is one matrix - the mixer's projections, gate and up rows of the dense or
+// shared feed-forward (in turn), its score row, the router - and what closes the layer is one as well, [W_o | W_down].
+int one_norm_weights(pi_model * m, int il) {
+    LayerState * s = m->lay;
+    Layer & L = s->layers[il];
+    const pi_layer_desc & d = L.d;
+    const int D = m->hp.n_embd, hv = d.n_head * d.vdim;
+    const auto want = [&](int kind, int64_t ne0, int64_t ne1, const char * what) { return want_tensor(m->L(il, kind), PI_TYPE_BF16, ne0, ne1, what); };
+    PI_TRY(want_tensor(m->L(il, PI_T_ATTN_NORM), PI_TYPE_F32, D, 1, "attn_norm"));
+    PI_TRY(norm_weights(m, m->L(il, PI_T_ATTN_NORM), s->opts.norm_offset, 1.0f, &L.norm_a));
+    uint16_t * z = zeroed(m, (size_t)L.z_rows * s->d_ld);
+    if (!z) return PI_E_HIP;
+    L.w_z = z;
+    const auto rows = [&](int kind, int64_t n, int off, int step, const char * what) -> int {
+        PI_TRY(want(kind, D, n, what));
+        return place(m, m->L(il, kind), z, s->d_ld, 0, s->d_ld, off, step);
+    };
+    PI_TRY(rows(PI_T_MIX_Q, (int64_t)d.n_head * d.dim, 0, 1, "mix_q"));
+    PI_TRY(rows(PI_T_MIX_K, (int64_t)(d.mixer == PI_MIXER_GROUPED ? d.n_kv_head : d.n_head) * d.dim, L.off_k, 1, "mix_k"));
+    if (L.off_v != L.off_k) PI_TRY(rows(PI_T_MIX_V, (int64_t)(d.mixer == PI_MIXER_GROUPED ? d.n_kv_head : d.n_head) * d.vdim, L.off_v, 1, "mix_v"));
+    if (d.mixer == PI_MIXER_LINEAR) {
+        PI_TRY(rows(PI_T_MIX_G, hv, L.off_g, 1, "mix_g"));
+        PI_TRY(want_tensor(m->L(il, PI_T_MIX_NORM), PI_TYPE_F32, hv, 1, "mix_norm"));
+        PI_TRY(want_tensor(m->L(il, PI_T_MIX_DECAY), PI_TYPE_F32, d.n_head, 1, "mix_decay"));
+        L.mix_norm = (const float *)m->L(il, PI_T_MIX_NORM).dev;
+        L.decay = (const float *)m->L(il, PI_T_MIX_DECAY).dev;
+        const int C = pi_k_linear_chunk();
+        std::vector<float> dec(d.n_head), pw((size_t)d.n_head * (C + 1));
+        PI_TRY(pi_memcpy_d2h(dec.data(), L.decay, sizeof(float) * dec.size()));
+        for (int h = 0; h < d.n_head; ++h) {
+            double v = 1.0;
+            for (int k = 0; k <= C; ++k, v *= dec[h]) pw[(size_t)h * (C + 1) + k] = (float)v;
+        }
+        float * p = m->alloc<float>(pw.size());
+        if (!p) return PI_E_HIP;
+        PI_TRY(pi_memcpy_h2d(p, pw.data(), sizeof(float) * pw.size()));
+        L.powers = p;
+    }
+    uint16_t * close = zeroed(m, (size_t)D * L.close_ld);
+    if (!close) return PI_E_HIP;
+    L.wo = close;
+    PI_TRY(want(PI_T_WO, hv, D, "wo"));
+    PI_TRY(place(m, m->L(il, PI_T_WO), close, L.close_ld, 0, L.hv_ld, 0, 1));
+    if (d.glu_ff > 0) {
+        PI_TRY(rows(PI_T_GLU_GATE, d.glu_ff, L.off_glu, 2, "glu_gate"));
+        PI_TRY(rows(PI_T_GLU_UP, d.glu_ff, L.off_glu + 1, 2, "glu_up"));
+        PI_TRY(want(PI_T_GLU_DOWN, d.glu_ff, D, "glu_down"));
+        PI_TRY(place(m, m->L(il, PI_T_GLU_DOWN), close, L.close_ld, L.hv_ld, L.glu_ld, 0, 1));
+        if (L.off_score >= 0) PI_TRY(rows(PI_T_SHARED_SCORE, 1, L.off_score, 1, "shared_score"));
+    }
+    if (d.ffn != PI_FFN_GLU_MOE) return PI_OK;
+    PI_TRY(rows(PI_T_ROUTER, d.n_expert, L.off_router, 1, "router"));
+    const int64_t ne = (int64_t)d.n_expert * d.expert_ff;
+    uint16_t * up = zeroed(m, (size_t)2 * ne * s->d_ld);
+    if (!up) return PI_E_HIP;
+    PI_TRY(want(PI_T_EXPERT_GATE, D, ne, "expert_gate"));
+    PI_TRY(want(PI_T_EXPERT_UP, D, ne, "expert_up"));
+    PI_TRY(want(PI_T_EXPERT_DOWN, d.expert_ff, (int64_t)d.n_expert * D, "expert_down"));
+    PI_TRY(place(m, m->L(il, PI_T_EXPERT_GATE), up, s->d_ld, 0, s->d_ld, 0, 2));
+    PI_TRY(place(m, m->L(il, PI_T_EXPERT_UP), up, s->d_ld, 0, s->d_ld, 1, 2));
+    L.up = up;
+    return padded(m, m->L(il, PI_T_EXPERT_DOWN), L.ff_ld, &L.down);
+}
+
+// sizes and places that follow from the description of a layer with one norm
+void one_norm_sizes(Layer & L) {
+    const pi_layer_desc & d = L.d;
+    int at = 0;
+    const auto take = [&](int n) { const int o = at; at = up_to(at + n, 16); return o; };
+    take(d.n_head * d.dim);
+    if (d.mixer == PI_MIXER_GROUPED) {
+        L.off_k = take(d.n_kv_head * d.dim);
+        L.off_v = d.values_are_keys ? L.off_k : take(d.n_kv_head * d.vdim);
+    } else {
+        L.off_k = take(d.n_head * d.dim);
+        L.off_v = take(d.n_head * d.vdim);
+        L.off_g = take(d.n_head * d.vdim);
+        L.dim_ld = up_to(d.dim, 32); L.vdim_ld = up_to(d.vdim, 64);
+    }
+    if (d.glu_ff > 0) {
+        L.off_glu = take(2 * d.glu_ff);
+        if (d.ffn == PI_FFN_GLU_MOE) L.off_score = take(1);
+    }
+    if (d.ffn == PI_FFN_GLU_MOE) L.off_router = take(d.n_expert);
+    L.z_rows = at;
+    L.hv_ld = up_to(d.n_head * d.vdim, 128); L.glu_ld = d.glu_ff > 0 ? up_to(d.glu_ff, 64) : 0; L.close_ld = L.hv_ld + L.glu_ld;
+    L.ff_ld = d.ffn == PI_FFN_GLU_MOE ? up_to(d.expert_ff, 64) : 0;
 }
 
 int layer_weights(pi_model * m, int il) {
@@ -198,9 +325,23 @@ int ensure_capacity(pi_model * m, int T) {
     int cap = 64;
     while (cap < T) cap *= 2;
     const size_t es = s->es, D = m->hp.n_embd;
-    size_t z = 0, qu = 0, ql = 0, ol = 0, at = 0, E = 0, top = 0, ff = 0;
+    size_t z = 0, qu = 0, ql = 0, ol = 0, at = 0, E = 0, top = 0, ff = 0, lq = 0, lv = 0, lo = 0, ls = 0;
+    const size_t chunks = s->recurrent && bf16_mode(s) ? (size_t)cap / pi_k_linear_chunk() + 32 : 0;        // every run of a pass ends with a part of one
     for (const Layer & L : s->layers) {
         const pi_layer_desc & d = L.d;
+        if (s->one_norm) {
+            z = std::max(z, (size_t)L.z_rows); at = std::max(at, (size_t)L.close_ld);
+            if (d.mixer == PI_MIXER_GROUPED) ql = std::max(ql, (size_t)d.n_head * L.hd);
+            else {
+                lo = std::max(lo, (size_t)d.n_head * d.vdim);
+                if (chunks) {
+                    lq = std::max(lq, (size_t)d.n_head * L.dim_ld); lv = std::max(lv, (size_t)d.n_head * L.vdim_ld);
+                    ls = std::max(ls, pi_k_linear_states_bytes((int)chunks, d.n_head, L.dim_ld, L.vdim_ld));
+                }
+            }
+            if (L.moe()) { E = std::max(E, (size_t)d.n_expert); top = std::max(top, (size_t)d.n_top); ff = std::max(ff, (size_t)d.n_top * L.ff_ld); }
+            continue;
+        }
         z = std::max(z, (size_t)L.z_rows); qu = std::max(qu, (size_t)d.n_head * L.dim_ld); ql = std::max(ql, (size_t)d.n_head * L.kd);
         ol = std::max(ol, (size_t)d.n_head * L.rank_ld); at = std::max(at, (size_t)L.hv_ld);
         if (d.ffn == PI_FFN_MOE) { E = std::max(E, (size_t)d.n_expert); top = std::max(top, (size_t)d.n_top); ff = std::max(ff, (size_t)d.n_top * L.ff_ld); }
@@ -224,6 +365,8 @@ int ensure_capacity(pi_model * m, int T) {
         carve(s->rl, n * E * 4); carve(s->wts, n * top * 4); carve(s->ids, n * top * 4); carve(s->perm, n * top * 4); carve(s->inv, n * top * 4);
         carve(s->off, (E + 1) * 4); carve(s->act, n * ff * es); carve(s->y_exp, n * top * D * es);
         carve(s->tiles, (n * top / 64 + E + 1) * 8); carve(s->n_tiles, 4);
+        carve(s->x0, s->opts.loop_times > 0 ? n * D * 4 : 0);
+        carve(s->lin_o, n * lo * 4); carve(s->lin_q, n * lq * 2); carve(s->lin_k, n * lq * 2); carve(s->lin_v, n * lv * 2); carve(s->lin_states, ls);
         s->cs.resize(s->rots.size());
         for (size_t r = 0; r < s->rots.size(); ++r) carve(s->cs[r], n * s->rots[r].dims * 4);
     };
@@ -303,7 +446,7 @@ pi_latent_prep prep_args(pi_model * m, const Layer & L, const Step & in) {
     pi_latent_prep p{};
     p.z = s->z; p.ldz = L.z_rows; p.T = in.T; p.n_head = d.n_head; p.dim = d.dim; p.dim_ld = L.dim_ld; p.rot_dim = d.rot_dim; p.kv_rank = d.kv_rank;
     p.rank_ld = L.rank_ld; p.kd = L.kd; p.cs = s->cs[L.rot]; p.norm_w = L.dkv_norm; p.eps = m->hp.norm_eps; p.q_un = s->q_un; p.q_lat = s->q_lat;
-    p.cache = L.own_kv ? L.cache : nullptr; p.cell = in.cell;
+    p.cache = L.own_kv ? L.cache[0] : nullptr; p.cell = in.cell;
     return p;
 }
 
@@ -311,7 +454,7 @@ pi_latent_attn attn_args(pi_model * m, const Layer & L, const Layer & src, const
     LayerState * s = m->lay;
     const pi_layer_desc & d = L.d;
     pi_latent_attn a{};
-    a.q_lat = s->q_lat; a.cache = src.cache; a.lists = s->lists; a.list_ld = s->kv.n; a.work = bf16_mode(s) ? in.work[L.hc].items : in.seq; a.n_vis = in.n_vis;
+    a.q_lat = s->q_lat; a.cache = src.cache[0]; a.lists = s->lists; a.list_ld = s->kv.n; a.work = bf16_mode(s) ? in.work[L.hc].items : in.seq; a.n_vis = in.n_vis;
     a.n_work = in.work[L.hc].n; a.T = in.T; a.n_head = d.n_head; a.kv_rank = d.kv_rank; a.rank_ld = L.rank_ld; a.kd = L.kd; a.n_parts = in.work[L.hc].parts; a.scale = d.scale;
     a.sink = L.sink; a.scratch = s->scratch; a.out_lat = s->o_lat;
     return a;
@@ -343,13 +486,13 @@ int attend_expanded(pi_model * m, const Layer & L, const Layer & src, const Step
     const size_t nk = (size_t)d.n_head * d.dim, nv = (size_t)d.n_head * d.vdim, keys = ((size_t)r.n_cells * nk + 127) / 128 * 128;
     bf16_t * k = s->expanded, * v = s->expanded + keys;
     pi_group_gemm g{};
-    g.W = L.uk; g.rows = (int)nk; g.cols = L.rank_ld; g.ldw = L.rank_ld; g.n_group = 1; g.x = src.cache; g.ldx = L.kd; g.T = r.n_cells; g.y = k; g.ldy = (int)nk;
+    g.W = L.uk; g.rows = (int)nk; g.cols = L.rank_ld; g.ldw = L.rank_ld; g.n_group = 1; g.x = src.cache[0]; g.ldx = L.kd; g.T = r.n_cells; g.y = k; g.ldy = (int)nk;
     g.alpha = 1.0f; g.gather = list; g.gather_div = 1;
     PI_TRY(pi_k_group_gemm_tile(&g, 128, st));
     g.W = L.uv; g.rows = (int)nv; g.y = v; g.ldy = (int)nv;
     PI_TRY(pi_k_group_gemm_tile(&g, 128, st));
     pi_latent_expanded a{};
-    a.q_un = s->q_un; a.q_lat = s->q_lat; a.keys = k; a.values = v; a.cache = src.cache; a.list = list; a.n_vis = in.n_vis; a.sink = L.sink; a.att = s->att;
+    a.q_un = s->q_un; a.q_lat = s->q_lat; a.keys = k; a.values = v; a.cache = src.cache[0]; a.list = list; a.n_vis = in.n_vis; a.sink = L.sink; a.att = s->att;
     a.tok0 = r.tok0; a.T = r.T; a.n_head = d.n_head; a.dim = d.dim; a.dim_ld = L.dim_ld; a.rot_dim = d.rot_dim; a.vdim = d.vdim; a.rank_ld = L.rank_ld; a.kd = L.kd;
     a.ld_att = L.hv_ld; a.scale = d.scale;
     return pi_k_latent_attn_expanded(&a, st);
@@ -369,24 +512,114 @@ int mix_latent(pi_model * m, Layer & L, const Step & in) {
     return dense(m, L.wo, m->hp.n_embd, L.hv_ld, s->att, T, s->mix);
 }
 
-int ffn_moe(pi_model * m, Layer & L, const Step & in) {
+// the experts of the chosen pairs (s->ids): relu^2 or, with a gate, clamped GLU in between; s->y_exp holds a row per pair, in expert order
+int experts(pi_model * m, Layer & L, const void * h, const Step & in) {
     LayerState * s = m->lay;
     const pi_layer_desc & d = L.d;
-    const int T = in.T, D = m->hp.n_embd;
+    const int T = in.T, D = m->hp.n_embd, per = d.ffn == PI_FFN_GLU_MOE ? 2 : 1;
     hipStream_t st = m->stream;
-    PI_TRY(dense(m, L.router, d.n_expert, s->d_ld, s->h_b, T, s->rl));
-    PI_TRY(pi_k_route(s->rl, T, d.n_expert, d.n_top, d.n_group, d.n_group_keep, L.bias, s->ids, s->wts, st));
     const int tile_n = (long long)T * d.n_top > 96LL * d.n_expert ? 128 : 64;       // tokens per tile, by the tokens an expert has on average
     PI_TRY(pi_k_moe_sort(s->ids, T * d.n_top, d.n_expert, s->off, s->perm, s->inv, tile_n, s->tiles, s->n_tiles, st));
     pi_group_gemm g{};
-    g.W = L.up; g.w_gs = (size_t)d.expert_ff * s->d_ld; g.rows = d.expert_ff; g.cols = s->d_ld; g.ldw = s->d_ld; g.n_group = d.n_expert; g.alpha = 1.0f; g.relu2 = 1;
-    g.x = s->h_b; g.ldx = s->d_ld; g.T = T; g.y = s->act; g.ldy = L.ff_ld; g.off = s->off; g.gather = s->perm; g.gather_div = d.n_top;
+    g.W = L.up; g.w_gs = (size_t)per * d.expert_ff * s->d_ld; g.rows = per * d.expert_ff; g.cols = s->d_ld; g.ldw = s->d_ld; g.n_group = d.n_expert; g.alpha = 1.0f;
+    if (per == 2) { g.glu = 1; g.glu_limit = d.expert_limit; g.glu_gain = d.glu_gain; }
+    else g.relu2 = 1;
+    g.x = h; g.ldx = s->d_ld; g.T = T; g.y = s->act; g.ldy = L.ff_ld; g.off = s->off; g.gather = s->perm; g.gather_div = d.n_top;
     g.tiles = s->tiles; g.n_tiles = s->n_tiles; g.max_tiles = T * d.n_top / tile_n + d.n_expert;
     PI_TRY(grouped(s, g, tile_n, st));
     pi_group_gemm w{};
     w.W = L.down; w.w_gs = (size_t)D * L.ff_ld; w.rows = D; w.cols = L.ff_ld; w.ldw = L.ff_ld; w.n_group = d.n_expert; w.alpha = 1.0f;
     w.x = s->act; w.ldx = L.ff_ld; w.T = T; w.y = s->y_exp; w.ldy = D; w.off = s->off; w.tiles = s->tiles; w.n_tiles = s->n_tiles; w.max_tiles = g.max_tiles;
     return grouped(s, w, tile_n, st);
+}
+
+int ffn_moe(pi_model * m, Layer & L, const Step & in) {
+    LayerState * s = m->lay;
+    const pi_layer_desc & d = L.d;
+    PI_TRY(dense(m, L.router, d.n_expert, s->d_ld, s->h_b, in.T, s->rl));
+    PI_TRY(pi_k_route(s->rl, in.T, d.n_expert, d.n_top, d.n_group, d.n_group_keep, L.bias, s->ids, s->wts, m->stream));
+    return experts(m, L, s->h_b, in);
+}
+
+// grouped-query attention over one list of work items
+pi_gqa_attn gqa_args(pi_model * m, const Layer & L, int pass, const Step & in, const Step::Work & w, int wide) {
+    LayerState * s = m->lay;
+    const pi_layer_desc & d = L.d;
+    pi_gqa_attn a{};
+    a.q = s->q_lat; a.cache = L.cache[pass]; a.lists = s->lists; a.list_ld = s->kv.n; a.work = bf16_mode(s) ? w.items : in.seq; a.n_vis = in.n_vis; a.n_work = w.n; a.T = in.T;
+    a.n_head = d.n_head; a.n_kv = d.n_kv_head; a.dim = d.dim; a.vdim = d.vdim; a.hd = L.hd; a.n_parts = w.parts; a.wide = wide; a.scale = d.scale; a.sink = d.sink;
+    a.scratch = s->scratch; a.att = s->att; a.ld_att = L.close_ld;
+    return a;
+}
+
+pi_linear linear_args(pi_model * m, const Layer & L, int pass, const Step & in) {
+    LayerState * s = m->lay;
+    const pi_layer_desc & d = L.d;
+    pi_linear p{};
+    p.z = s->z; p.ldz = L.z_rows; p.T = in.T; p.n_head = d.n_head; p.dim = d.dim; p.vdim = d.vdim; p.off_k = L.off_k; p.off_v = L.off_v; p.decay = L.decay; p.powers = L.powers;
+    p.state = L.state[pass]; p.runs = in.lin; p.n_runs = in.n_lin; p.o = s->lin_o; p.q = s->lin_q; p.k = s->lin_k; p.v = s->lin_v; p.states = s->lin_states;
+    p.dim_ld = L.dim_ld; p.vdim_ld = L.vdim_ld;
+    return p;
+}
+
+// A layer with one norm.  Steps of up to 16 tokens (bf16): norm, joint projection, what lies behind it (queries and cells or the state's step,
+// beside the dense or shared feed-forward's activation and the choice of experts), attention, merge or gated norm beside the experts'
+// first matrices, and what closes the layer.  Longer steps run the same parts one by one.
+int one_norm_layer(pi_model * m, Layer & L, const LayerRun & r, const Step & in, float * keep) {
+    LayerState * s = m->lay;
+    const pi_layer_desc & d = L.d;
+    const int T = in.T, D = m->hp.n_embd, type = s->opts.compute;
+    const bool moe = L.moe(), step = bf16_mode(s) && pi_k_layer_step_supported(T, moe ? d.n_expert : 0, moe ? d.n_top : 0), linear = d.mixer == PI_MIXER_LINEAR;
+    hipStream_t st = m->stream;
+    PI_TRY(pi_k_layer_norm(type, s->x, nullptr, T, D, m->hp.norm_eps, L.norm_a, r.starts && r.pass > 0 ? s->x0 : nullptr, r.starts ? s->loop_step + (size_t)r.pass * D : nullptr,
+                           s->h_a, s->d_ld, step, st));
+    if (step) PI_TRY(pi_k_gemm_bf16_ol(L.w_z, L.z_rows, s->d_ld, s->h_a, T, PI_EPI_NONE, nullptr, nullptr, s->z, nullptr, st));
+    else PI_TRY(dense(m, L.w_z, L.z_rows, s->d_ld, s->h_a, T, s->z));
+    pi_ffn_front f{};
+    f.off_glu = L.off_glu; f.ff = d.glu_ff; f.ff_ld = L.glu_ld; f.off_score = L.off_score; f.limit = d.glu_limit; f.gain = d.glu_gain;
+    f.act = (unsigned char *)s->att + (size_t)L.hv_ld * s->es; f.ld_act = L.close_ld; f.off_router = L.off_router; f.n_expert = moe ? d.n_expert : 0; f.n_top = d.n_top;
+    f.ids = s->ids; f.weights = s->wts;
+    pi_gqa_attn parts{};
+    pi_gate_norm gate{};
+    if (linear) {
+        pi_linear p = linear_args(m, L, r.pass, in);
+        if (in.n_lin_long == 0) PI_TRY(pi_k_linear_step(type, &p, &f, st));
+        else {
+            PI_TRY(pi_k_linear_prep(type, &p, &f, st));
+            if (in.n_lin > 0) PI_TRY(pi_k_linear_step(type, &p, nullptr, st));
+            p.runs = in.lin_long; p.n_runs = in.n_lin_long; p.chunks = in.lin_chunks; p.n_chunks = in.n_lin_chunks; p.first_chunk = in.lin_first;
+            PI_TRY(pi_k_linear_chunks(&p, st));
+        }
+        gate.o = s->lin_o; gate.z = s->z; gate.w = L.mix_norm; gate.ldz = L.z_rows; gate.off_gate = L.off_g; gate.n = d.n_head * d.vdim; gate.T = T; gate.eps = m->hp.norm_eps;
+        gate.att = s->att; gate.ld_att = L.close_ld;
+        if (!step) PI_TRY(pi_k_gate_norm(type, &gate, st));
+    } else {
+        pi_gqa_prep p{};
+        p.z = s->z; p.ldz = L.z_rows; p.T = T; p.n_head = d.n_head; p.n_kv = d.n_kv_head; p.dim = d.dim; p.vdim = d.vdim; p.rot_dim = d.rot_dim; p.off_k = L.off_k; p.off_v = L.off_v;
+        p.hd = L.hd; p.unit = d.unit_qk; p.cs = L.rot >= 0 ? s->cs[L.rot] : s->x; p.eps = m->hp.norm_eps; p.q = s->q_lat; p.cache = L.cache[r.pass]; p.cell = in.cell;
+        PI_TRY(pi_k_gqa_prep(type, &p, &f, st));
+        if (bf16_mode(s) && in.wide[L.hc].n > 0) {
+            const pi_gqa_attn a = gqa_args(m, L, r.pass, in, in.wide[L.hc], 1);
+            PI_TRY(pi_k_gqa_attn(type, &a, st));
+        }
+        if (in.work[L.hc].n > 0) {
+            const pi_gqa_attn a = gqa_args(m, L, r.pass, in, in.work[L.hc], 0);
+            if (step) { PI_TRY(pi_k_gqa_attn_parts(&a, st)); if (a.n_parts > 1) parts = a; }
+            else PI_TRY(pi_k_gqa_attn(type, &a, st));
+        }
+    }
+    if (step) {
+        if (moe || linear || parts.n_parts > 1)
+            PI_TRY(pi_k_mix_up_step(parts.n_parts > 1 ? &parts : nullptr, linear ? &gate : nullptr, L.up, d.n_expert, d.expert_ff, s->d_ld, d.expert_limit, d.glu_gain, s->h_a, T,
+                                    moe ? s->ids : nullptr, s->wts, d.n_top, s->act, L.ff_ld, st));
+        pi_layer_out o{};
+        o.x = s->x; o.wo = L.wo; o.att = s->att; o.rows = D; o.ld_att = L.close_ld; o.T = T; o.out = s->x2; o.keep = keep;
+        if (moe) { o.down = L.down; o.act = s->act; o.ids = s->ids; o.ld_act = L.ff_ld; o.top = d.n_top; o.n_expert = d.n_expert; }
+        return pi_k_layer_out_step(&o, st);
+    }
+    PI_TRY(dense(m, L.wo, D, L.close_ld, s->att, T, s->mix));
+    if (moe) PI_TRY(experts(m, L, s->h_a, in));
+    return pi_k_moe_combine(type, s->x, s->mix, s->y_exp, s->inv, moe ? s->wts : nullptr, moe ? d.n_top : 0, T, D, s->x2, keep, st);
 }
 
 // a layer of a step of up to 16 tokens (bf16): six launches
@@ -415,12 +648,19 @@ int pass_layers(pi_model * m, const Step & in) {
     LayerState * s = m->lay;
     const int type = s->opts.compute, T = in.T, D = m->hp.n_embd;
     hipStream_t st = m->stream;
-    PI_TRY(pi_k_embed_norm(s->embed, D, in.tokens, T, s->embd_norm, m->hp.norm_eps, s->x, st));
+    if (s->one_norm) PI_TRY(pi_k_embed_bigram(s->embed, D, in.tokens, in.prev, T, s->opts.embed_scale, s->bigram, s->opts.bigram_buckets, s->opts.bigram_mul_prev, s->opts.bigram_mul_cur,
+                                              in.carry, s->x, s->opts.loop_times > 0 ? s->x0 : nullptr, st));
+    else PI_TRY(pi_k_embed_norm(s->embed, D, in.tokens, T, s->embd_norm, m->hp.norm_eps, s->x, st));
     for (size_t r = 0; r < s->rots.size(); ++r) PI_TRY(pi_k_rope_angles(in.pos, T, s->rots[r].dims, s->rots[r].base, s->cs[r], st));
-    for (size_t il = 0; il < s->layers.size(); ++il) {
-        Layer & L = s->layers[il];
-        const bool moe = L.d.ffn == PI_FFN_MOE;
-        float * keep = s->streams_T ? s->streams + il * (size_t)s->streams_T * D : nullptr;
+    for (size_t k = 0; k < s->order.size(); ++k) {
+        Layer & L = s->layers[s->order[k].layer];
+        const bool moe = L.moe();
+        float * keep = s->streams_T ? s->streams + k * (size_t)s->streams_T * D : nullptr;
+        if (s->one_norm) {
+            PI_TRY(one_norm_layer(m, L, s->order[k], in, keep));
+            std::swap(s->x, s->x2);
+            continue;
+        }
         if (bf16_mode(s) && pi_k_layer_step_supported(T, moe ? L.d.n_expert : 0, moe ? L.d.n_top : 0)) {
             PI_TRY(step_layer(m, L, in, keep));
             std::swap(s->x, s->x2);
@@ -440,7 +680,8 @@ int pass_head(pi_model * m, const int32_t * rows, int n) {
     LayerState * s = m->lay;
     const int D = m->hp.n_embd;
     const bool ol = bf16_mode(s) && n <= 16;
-    PI_TRY(pi_k_norm_pair(s->opts.compute, s->x, rows, n, D, m->hp.norm_eps, s->out_norm, s->h_head, nullptr, nullptr, s->d_ld, ol, m->stream));
+    if (s->one_norm) PI_TRY(pi_k_layer_norm(s->opts.compute, s->x, rows, n, D, m->hp.norm_eps, s->out_norm, nullptr, nullptr, s->h_head, s->d_ld, ol, m->stream));
+    else PI_TRY(pi_k_norm_pair(s->opts.compute, s->x, rows, n, D, m->hp.norm_eps, s->out_norm, s->h_head, nullptr, nullptr, s->d_ld, ol, m->stream));
     if (ol) return pi_k_gemm_bf16_ol(s->head, m->hp.n_vocab, s->d_ld, s->h_head, n, PI_EPI_NONE, nullptr, nullptr, s->logits, nullptr, m->stream);
     return dense(m, s->head, m->hp.n_vocab, s->d_ld, s->h_head, n, s->logits);
 }
@@ -476,6 +717,21 @@ void work_items(const int32_t * seq, const int32_t * n_vis, int n, const HeadKin
     }
 }
 
+// the same for grouped-query attention: runs of at least kWideRows rows as wide items (where the caller takes them)
+void gqa_items(const int32_t * seq, const int32_t * n_vis, int n, int per, std::vector<int32_t> & narrow, std::vector<int32_t> * wide) {
+    for (int t0 = 0; t0 < n;) {
+        int t1 = t0 + 1;
+        while (t1 < n && seq[t1] == seq[t0] && n_vis[t1] >= n_vis[t1 - 1]) ++t1;
+        const int rows = (t1 - t0) * per;
+        const bool w = wide && rows >= kWideRows;
+        const int step = pi_k_gqa_rows(w);
+        for (int r = 0; r < rows; r += step) { const int32_t item[4] = {t0, r, std::min(step, rows - r), seq[t0]}; (w ? *wide : narrow).insert((w ? *wide : narrow).end(), item, item + 4); }
+        t0 = t1;
+    }
+}
+
+int gqa_parts(int n_groups, int n_vis_max, int cells) { return n_groups <= 0 ? 1 : std::max(1, std::min({kAttnItems / n_groups, (n_vis_max + cells - 1) / cells, 64})); }
+
 // how many workgroups share one work item's cells
 int choose_parts(LayerState * s, int n_work, int n_vis_max) {
     if (!bf16_mode(s) || n_work <= 0) return 1;
@@ -505,8 +761,9 @@ int live_cells(LayerState * s, int q) {
 }
 
 // takes the cell for sequences `mask` at position p; false: some sequence's list has to be rebuilt (the position is not behind its last)
-void take_cell(LayerState * s, int cell, int32_t p, uint32_t mask, std::vector<int32_t> & app) {
+void take_cell(LayerState * s, int cell, int32_t p, uint32_t mask, int32_t tok, std::vector<int32_t> & app) {
     s->kv.take(cell, p, mask);
+    s->cell_tok[cell] = tok;
     for (uint32_t b = mask; b; b &= b - 1) {
         const int q = __builtin_ctz(b);
         if (s->kv.edited >> q & 1u) continue;                      // rebuilt as a whole later
@@ -521,11 +778,66 @@ int apply_shift(pi_model * m) {
     if (!s->kv.has_shift) return PI_OK;
     PI_HIP_TRY(hipStreamSynchronize(m->stream));
     PI_TRY(pi_memcpy_h2d(s->d_delta, s->kv.delta.data(), sizeof(int32_t) * s->kv.n));
-    for (Layer & L : s->layers)
-        if (L.own_kv) PI_TRY(pi_k_latent_shift(s->opts.compute, L.cache, s->kv.n, L.kd, L.rank_ld, L.d.rot_dim, L.d.rot_base, s->d_delta, m->stream));
+    for (Layer & L : s->layers) {
+        if (L.d.mixer == PI_MIXER_GROUPED)
+            for (void * c : L.cache) PI_TRY(pi_k_gqa_shift(s->opts.compute, c, s->kv.n, L.d.n_kv_head, L.hd, L.d.rot_dim, L.d.rot_base, s->d_delta, m->stream));
+        else if (L.cell_values()) PI_TRY(pi_k_latent_shift(s->opts.compute, L.cache[0], s->kv.n, L.kd, L.rank_ld, L.d.rot_dim, L.d.rot_base, s->d_delta, m->stream));
+    }
     PI_HIP_TRY(hipStreamSynchronize(m->stream));
     s->kv.shift_done();
     return PI_OK;
+}
+
+// ---- slots of recurrent states ----------------------------------------------------------------------------------------------------
+int resize_slots(pi_model * m, int n) {
+    LayerState * s = m->lay;
+    PI_HIP_TRY(hipStreamSynchronize(m->stream));
+    drop_graph(s);
+    for (Layer & L : s->layers)
+        for (float *& st : L.state) {
+            const size_t one = L.state_floats();
+            float * p = m->alloc<float>(n * one);
+            if (!p) return PI_E_HIP;
+            PI_TRY(pi_memset(p, 0, n * one * 4));
+            if (st) PI_TRY(pi_memcpy_d2d(p, st, s->n_slots * one * 4));
+            PI_TRY(pi_sync());
+            for (auto & o : m->owned) if (st && o == st) { pi_free(o); o = nullptr; }
+            st = p;
+        }
+    s->n_slots = n;
+    return PI_OK;
+}
+
+// the sequence's slot; one of a sequence without cells (other than those of `keep`) is taken, or there will be more of them
+int take_slot(pi_model * m, int q, uint32_t keep) {
+    LayerState * s = m->lay;
+    if (s->slot_of[q] >= 0) return PI_OK;
+    std::vector<char> used(s->n_slots, 0);
+    for (int o = 0; o < 32; ++o) {
+        if (s->slot_of[o] < 0) continue;
+        if (!(keep >> o & 1u) && live_cells(s, o) == 0) s->slot_of[o] = -1;
+        else used[s->slot_of[o]] = 1;
+    }
+    int k = 0;
+    while (k < s->n_slots && used[k]) ++k;
+    if (k == s->n_slots) PI_TRY(resize_slots(m, std::max(4, 2 * s->n_slots)));
+    s->slot_of[q] = k;
+    return PI_OK;
+}
+
+// a recurrent state holds all of a sequence's tokens: true if the edit leaves every sequence whole or empty
+template <typename F> bool keeps_whole(LayerState * s, F && edit) {
+    KvCells trial = s->kv;
+    edit(trial);
+    for (int q = 0; q < 32; ++q) {
+        int before = 0, after = 0;
+        for (int i = 0; i < s->kv.n; ++i) {
+            before += s->kv.pos[i] >= 0 && (s->kv.seq[i] >> q & 1u);
+            after += trial.pos[i] >= 0 && (trial.seq[i] >> q & 1u);
+        }
+        if (after != before && after != 0) return false;
+    }
+    return true;
 }
 
 int upload_appends(pi_model * m, const std::vector<int32_t> & app) {
@@ -553,16 +865,19 @@ static int resize_pool(pi_model * m, int n_cells) {
     drop_graph(s);
     auto give_back = [&](void * p) { for (auto & o : m->owned) if (p && o == p) { pi_free(o); o = nullptr; } };
     for (Layer & L : s->layers) {
-        if (!L.own_kv) continue;
-        const size_t row = (size_t)L.kd * s->es;
-        unsigned char * c = m->alloc<unsigned char>(n_cells * row);
-        if (!c) return PI_E_HIP;
-        PI_TRY(pi_memset(c, 0, n_cells * row));
-        if (L.cache) PI_TRY(pi_memcpy_d2d(c, L.cache, s->kv.n * row));
-        PI_TRY(pi_sync());
-        give_back(L.cache);
-        L.cache = c;
+        const size_t row = L.cell_values() * s->es;
+        if (!row) continue;
+        for (void *& old : L.cache) {
+            unsigned char * c = m->alloc<unsigned char>(n_cells * row);
+            if (!c) return PI_E_HIP;
+            PI_TRY(pi_memset(c, 0, n_cells * row));
+            if (old) PI_TRY(pi_memcpy_d2d(c, old, s->kv.n * row));
+            PI_TRY(pi_sync());
+            give_back(old);
+            old = c;
+        }
     }
+    s->cell_tok.resize(n_cells, -1);
     give_back(s->lists); give_back(s->d_delta);
     s->lists = m->alloc<int32_t>((size_t)32 * n_cells);
     s->d_delta = m->alloc<int32_t>(n_cells);
@@ -590,30 +905,59 @@ int layers_finalize(pi_model * m) {
     PI_TRY(want_tensor(m->glob[PI_T_TOK_EMBD], PI_TYPE_BF16, D, m->hp.n_vocab, "tok_embd"));
     PI_TRY(want_tensor(m->glob[PI_T_OUTPUT], PI_TYPE_BF16, D, m->hp.n_vocab, "output"));
     PI_TRY(want_tensor(m->glob[PI_T_OUTPUT_NORM], PI_TYPE_F32, D, 1, "output_norm"));
-    PI_TRY(want_tensor(m->embd_norm, PI_TYPE_F32, D, 1, "embd_norm"));
     s->embed = m->glob[PI_T_TOK_EMBD].dev;
     PI_TRY(padded(m, m->glob[PI_T_OUTPUT], s->d_ld, &s->head));
-    PI_TRY(norm_weights(m, m->embd_norm, s->opts.norm_offset, 1.0f, &s->embd_norm));
+    if (!s->one_norm) {
+        PI_TRY(want_tensor(m->embd_norm, PI_TYPE_F32, D, 1, "embd_norm"));
+        PI_TRY(norm_weights(m, m->embd_norm, s->opts.norm_offset, 1.0f, &s->embd_norm));
+    }
+    if (s->opts.bigram_buckets > 0) {
+        PI_TRY(want_tensor(m->bigram, PI_TYPE_BF16, D, (int64_t)s->opts.bigram_buckets + 1, "bigram"));
+        s->bigram = m->bigram.dev;
+    }
+    if (s->opts.loop_times > 0) {
+        PI_TRY(want_tensor(m->loop_step, PI_TYPE_F32, D, s->opts.loop_times, "loop_step"));
+        s->loop_step = (const float *)m->loop_step.dev;
+    }
     PI_TRY(norm_weights(m, m->glob[PI_T_OUTPUT_NORM], s->opts.norm_offset, s->opts.logit_scale, &s->out_norm));
     size_t scratch = 0;
     for (size_t il = 0; il < s->layers.size(); ++il) {
         Layer & L = s->layers[il];
         const pi_layer_desc & d = L.d;
+        const auto rotation = [&]() {
+            size_t r = 0;
+            while (r < s->rots.size() && (s->rots[r].dims != d.rot_dim || s->rots[r].base != d.rot_base)) ++r;
+            if (r == s->rots.size()) s->rots.push_back({d.rot_dim, d.rot_base});
+            L.rot = (int)r;
+        };
+        const auto kind = [&](const HeadKind & hk) {
+            size_t h = 0;
+            while (h < s->kinds.size() && memcmp(&s->kinds[h], &hk, sizeof hk)) ++h;
+            if (h == s->kinds.size()) s->kinds.push_back(hk);
+            L.hc = (int)h;
+        };
+        if (s->one_norm) {
+            one_norm_sizes(L);
+            if (d.mixer == PI_MIXER_GROUPED) {
+                L.hd = pi_k_gqa_head_ld(s->opts.compute, d.dim, d.vdim);
+                if (!L.hd) return fail(PI_E_UNSUPPORTED, "pi_model_finalize: head sizes outside the attention kernels (up to 256)");
+                if (d.rot_dim > 0) rotation(); else L.rot = -1;
+                kind(HeadKind{d.mixer, d.n_head / d.n_kv_head, d.n_kv_head, 0, 0, 0, 0, L.hd});
+                scratch = std::max(scratch, pi_k_gqa_scratch_floats(kAttnItems, 1, 1, L.hd, 2) / 2);      // items x groups x parts <= kAttnItems
+            } else if (!pi_k_linear_supported(d.dim, d.vdim)) {
+                return fail(PI_E_UNSUPPORTED, "pi_model_finalize: head sizes outside the linear attention's kernels (up to 256)");
+            }
+            PI_TRY(one_norm_weights(m, (int)il));
+            continue;
+        }
         L.own_kv = d.kv_from < 0;
         L.nq = d.n_head * (d.dim + d.rot_dim);
         L.z_rows = L.nq + (L.own_kv ? d.kv_rank + d.rot_dim : 0);
         L.dim_ld = up_to(d.dim, 64); L.rank_ld = up_to(d.kv_rank, 64); L.kd = L.rank_ld + up_to(d.rot_dim, 32);
         L.hv_ld = up_to(d.n_head * d.vdim, 128); L.ff_ld = d.ffn == PI_FFN_MOE ? up_to(d.expert_ff, 64) : 0;
         if (!pi_k_latent_attn_supported(s->opts.compute, L.rank_ld, L.kd)) return fail(PI_E_UNSUPPORTED, "pi_model_finalize: latent sizes outside the attention kernels (rank up to 1024)");
-        size_t r = 0;
-        while (r < s->rots.size() && (s->rots[r].dims != d.rot_dim || s->rots[r].base != d.rot_base)) ++r;
-        if (r == s->rots.size()) s->rots.push_back({d.rot_dim, d.rot_base});
-        L.rot = (int)r;
-        size_t h = 0;
-        const HeadKind hk{d.n_head, d.dim, d.rot_dim, d.vdim, L.rank_ld, L.kd};
-        while (h < s->kinds.size() && memcmp(&s->kinds[h], &hk, sizeof hk)) ++h;
-        if (h == s->kinds.size()) s->kinds.push_back(hk);
-        L.hc = (int)h;
+        rotation();
+        kind(HeadKind{d.mixer, d.n_head, 1, d.dim, d.rot_dim, d.vdim, L.rank_ld, L.kd});
         scratch = std::max(scratch, pi_k_latent_attn_scratch_floats(kItemRows * kAttnItems / 2, L.rank_ld, 2));      // items x parts <= kAttnItems
         PI_TRY(layer_weights(m, (int)il));
     }
@@ -622,12 +966,15 @@ int layers_finalize(pi_model * m) {
         if (!s->scratch) return PI_E_HIP;
     }
     PI_TRY(head_buffers(m));
-    for (int32_t ** p : {&s->g_tok, &s->g_pos, &s->g_cell, &s->g_vis, &s->g_seq, &s->g_step}) {
+    if (s->recurrent) PI_TRY(resize_slots(m, s->opts.n_slots > 0 ? s->opts.n_slots : 4));
+    s->g_lin = m->alloc<int32_t>(4 * kMaxLockstep);
+    if (!s->g_lin) return PI_E_HIP;
+    for (int32_t ** p : {&s->g_tok, &s->g_pos, &s->g_cell, &s->g_vis, &s->g_seq, &s->g_step, &s->g_prev}) {
         *p = m->alloc<int32_t>(kMaxLockstep);
         if (!*p) return PI_E_HIP;
     }
     size_t items = 0;
-    for (const HeadKind & h : s->kinds) items += (size_t)kMaxLockstep * ((h.n_head + kItemRows - 1) / kItemRows);
+    for (const HeadKind & h : s->kinds) items += (size_t)kMaxLockstep * ((h.n_head + 15) / 16);      // (16: the smaller of the two kinds of items)
     s->g_work = m->alloc<int32_t>(4 * items);
     s->g_out = m->alloc<int32_t>((size_t)s->max_steps * kMaxLockstep);
     if (!s->g_work || !s->g_out) return PI_E_HIP;
@@ -663,17 +1010,33 @@ int layers_step(pi_model * m, const int32_t * tokens, const int32_t * positions,
     PI_TRY(ensure_capacity(m, std::min(n_tokens, batch)));
     PI_TRY(apply_shift(m));
     for (int t = 0; t < n_tokens; ++t) for (uint32_t b = seq_masks[t]; b; b &= b - 1) refresh_list(s, __builtin_ctz(b), app);
-    for (int t = 0; t < n_tokens; ++t) take_cell(s, cells[t], positions[t], seq_masks[t], app);
+    uint32_t fresh = 0;                                          // recurrent models: sequences whose state starts at zero
+    if (s->recurrent) {
+        uint32_t met = 0;
+        const char * why = nullptr;
+        for (int t = 0; t < n_tokens && !why; ++t) {
+            const int q = __builtin_ctz(seq_masks[t]);
+            if (seq_masks[t] & (seq_masks[t] - 1)) why = "pi_model_kv_cells_step: a token of several sequences in a model with recurrent states";
+            else if (t && seq_masks[t] == seq_masks[t - 1]) { if (positions[t] <= positions[t - 1]) why = "pi_model_kv_cells_step: a recurrent state takes its tokens in order"; }
+            else if (met >> q & 1u) why = "pi_model_kv_cells_step: a sequence's tokens follow one another in a step";
+            else if (!s->list_pos[q].empty() && s->list_pos[q].back() >= positions[t]) why = "pi_model_kv_cells_step: a recurrent state takes its tokens in order";
+            else { met |= 1u << q; if (s->list_pos[q].empty()) fresh |= 1u << q; }
+        }
+        if (why) { PI_TRY(upload_appends(m, app)); return fail(PI_E_UNSUPPORTED, why); }
+        for (uint32_t b = met; b; b &= b - 1) PI_TRY(take_slot(m, __builtin_ctz(b), met));
+    }
+    for (int t = 0; t < n_tokens; ++t) take_cell(s, cells[t], positions[t], seq_masks[t], tokens[t], app);
     s->kv.move_head(cells[n_tokens - 1] + 1);
     for (int t = 0; t < n_tokens; ++t) for (uint32_t b = seq_masks[t]; b; b &= b - 1) refresh_list(s, __builtin_ctz(b), app);
     PI_TRY(upload_appends(m, app));
-    std::vector<int32_t> vis(n_tokens), seq(n_tokens);
+    std::vector<int32_t> vis(n_tokens), seq(n_tokens), prev(n_tokens, -1);
     for (int t = 0; t < n_tokens; ++t) {
         seq[t] = __builtin_ctz(seq_masks[t]);                    // a token attends the cells of its first sequence
         const auto & lp = s->list_pos[seq[t]];
         vis[t] = (int32_t)(std::upper_bound(lp.begin(), lp.end(), positions[t]) - lp.begin());
+        if (vis[t] >= 2) prev[t] = s->cell_tok[s->list_cells[seq[t]][vis[t] - 2]];
     }
-    std::vector<int32_t> rows, place, items;
+    std::vector<int32_t> rows, place, items, wide, lin;
     for (int t0 = 0; t0 < n_tokens; t0 += batch) {
         const int T = std::min(batch, n_tokens - t0);
         rows.clear(); place.clear(); items.clear();
@@ -681,33 +1044,70 @@ int layers_step(pi_model * m, const int32_t * tokens, const int32_t * positions,
         Step in;
         in.T = T;
         const int vmax = *std::max_element(vis.begin() + t0, vis.begin() + t0 + T);
-        std::vector<size_t> begin;
+        std::vector<size_t> begin, begin_wide;
+        wide.clear(); lin.clear();
         for (const HeadKind & h : s->kinds) {
             begin.push_back(items.size());
+            begin_wide.push_back(wide.size());
             in.runs.emplace_back();
-            if (bf16_mode(s)) work_items(seq.data() + t0, vis.data() + t0, T, h, items, T > 16 ? &in.runs.back() : nullptr);
+            if (h.mixer == PI_MIXER_GROUPED) { if (bf16_mode(s)) gqa_items(seq.data() + t0, vis.data() + t0, T, h.n_head, items, T > 16 ? &wide : nullptr); }
+            else if (bf16_mode(s)) work_items(seq.data() + t0, vis.data() + t0, T, h, items, T > 16 ? &in.runs.back() : nullptr);
         }
         begin.push_back(items.size());
-        const size_t n_in = (size_t)5 * T + items.size() + rows.size();
+        begin_wide.push_back(wide.size());
+        items.insert(items.end(), wide.begin(), wide.end());
+        const size_t at_lin = items.size();
+        if (s->recurrent) {                                       // runs walked token by token, long runs, their first chunks, the chunks
+            std::vector<int32_t> lng, first, chunks;
+            const int C = pi_k_linear_chunk();
+            for (int a = 0; a < T;) {
+                int b = a + 1;
+                while (b < T && seq[t0 + b] == seq[t0 + a]) ++b;
+                const int q = seq[t0 + a], new_state = fresh >> q & 1u;
+                const int32_t run[4] = {a, b - a, s->slot_of[q], new_state};
+                fresh &= ~(1u << q);                              // a later pass of this step goes on
+                const bool chunked = bf16_mode(s) && b - a >= kLinearChunked;
+                (chunked ? lng : lin).insert((chunked ? lng : lin).end(), run, run + 4);
+                if (chunked) {
+                    first.push_back((int32_t)(chunks.size() / 3));
+                    for (int c = a; c < b; c += C) { const int32_t ch[3] = {c, std::min(C, b - c), new_state && c == a}; chunks.insert(chunks.end(), ch, ch + 3); }
+                }
+                a = b;
+            }
+            in.n_lin = (int)lin.size() / 4; in.n_lin_long = (int)lng.size() / 4; in.n_lin_chunks = (int)chunks.size() / 3;
+            items.insert(items.end(), lin.begin(), lin.end());
+            items.insert(items.end(), lng.begin(), lng.end());
+            items.insert(items.end(), first.begin(), first.end());
+            items.insert(items.end(), chunks.begin(), chunks.end());
+        }
+        const size_t n_in = (size_t)8 * T + items.size() + rows.size();
         PI_TRY(ensure_inputs(m, n_in));
         PI_HIP_TRY(hipStreamSynchronize(m->stream));
         int32_t * h = s->h_in;
         memcpy(h, tokens + t0, 4 * (size_t)T); memcpy(h + T, positions + t0, 4 * (size_t)T); memcpy(h + 2 * T, cells.data() + t0, 4 * (size_t)T);
         memcpy(h + 3 * T, vis.data() + t0, 4 * (size_t)T); memcpy(h + 4 * T, seq.data() + t0, 4 * (size_t)T);
-        if (!items.empty()) memcpy(h + 5 * T, items.data(), 4 * items.size());
-        if (!rows.empty()) memcpy(h + 5 * T + items.size(), rows.data(), 4 * rows.size());
+        memcpy(h + 5 * T, prev.data() + t0, 4 * (size_t)T);      // (the items behind start on a multiple of 16 bytes)
+        if (!items.empty()) memcpy(h + 8 * T, items.data(), 4 * items.size());
+        if (!rows.empty()) memcpy(h + 8 * T + items.size(), rows.data(), 4 * rows.size());
         PI_HIP_TRY(hipMemcpyAsync(s->d_in, h, 4 * n_in, hipMemcpyHostToDevice, m->stream));
-        in.tokens = s->d_in; in.pos = s->d_in + T; in.cell = s->d_in + 2 * T; in.n_vis = s->d_in + 3 * T; in.seq = s->d_in + 4 * T;
+        in.tokens = s->d_in; in.pos = s->d_in + T; in.cell = s->d_in + 2 * T; in.n_vis = s->d_in + 3 * T; in.seq = s->d_in + 4 * T; in.prev = s->d_in + 5 * T;
+        in.lin = s->d_in + 8 * T + at_lin; in.lin_long = in.lin + 4 * in.n_lin; in.lin_first = in.lin_long + 4 * in.n_lin_long; in.lin_chunks = in.lin_first + in.n_lin_long;
         for (size_t k = 0; k < s->kinds.size(); ++k) {
             Step::Work w;
-            w.items = s->d_in + 5 * T + begin[k];
+            w.items = s->d_in + 8 * T + begin[k];
             w.n = bf16_mode(s) ? (int)(begin[k + 1] - begin[k]) / 4 : T;
-            w.parts = choose_parts(s, w.n, vmax);
+            const HeadKind & hk = s->kinds[k];
+            w.parts = hk.mixer == PI_MIXER_GROUPED ? (bf16_mode(s) ? gqa_parts(w.n * hk.n_kv, vmax, 128) : 1) : choose_parts(s, w.n, vmax);
             in.work.push_back(w);
+            Step::Work wd;
+            wd.items = s->d_in + 8 * T + begin.back() + begin_wide[k];
+            wd.n = (int)(begin_wide[k + 1] - begin_wide[k]) / 4;
+            wd.parts = gqa_parts(wd.n * hk.n_kv, vmax, 512);
+            in.wide.push_back(wd);
         }
         s->streams_T = 0;
         if (m->capture) {
-            const size_t need = s->layers.size() * (size_t)T * m->hp.n_embd;
+            const size_t need = s->order.size() * (size_t)T * m->hp.n_embd;
             if (need > s->streams_cap) {
                 if (s->streams) pi_free(s->streams);
                 s->streams_cap = 0;
@@ -719,7 +1119,7 @@ int layers_step(pi_model * m, const int32_t * tokens, const int32_t * positions,
         }
         PI_TRY(ensure_expanded(m, in));
         PI_TRY(pass_layers(m, in));
-        const int32_t * d_rows = s->d_in + 5 * T + items.size();
+        const int32_t * d_rows = s->d_in + 8 * T + items.size();
         for (int r0 = 0; r0 < (int)rows.size(); r0 += kHeadRows) {
             const int n = std::min(kHeadRows, (int)rows.size() - r0);
             const size_t V = m->hp.n_vocab;
@@ -759,6 +1159,7 @@ static int continue_at(pi_model * m, int q, int n_past) {
     const int before = (int)(std::lower_bound(lp.begin(), lp.end(), n_past) - lp.begin());
     if (before != n_past || (n_past && (lp[0] != 0 || lp[n_past - 1] != n_past - 1))) return fail(PI_E_STATE, "the sequence's cells do not hold the positions 0 .. n_past - 1");
     if ((int)lp.size() == before) return PI_OK;
+    if (s->recurrent && before > 0) return fail(PI_E_UNSUPPORTED, "a model with recurrent states cannot go back to an earlier position");
     s->kv.seq_rm(q, n_past, -1);
     app.clear();
     refresh_list(s, q, app);
@@ -814,17 +1215,23 @@ int layers_generate(pi_model * m, int own, int n_steps, int32_t * out_tokens, fl
     const int T = own ? 1 : s->n_seq, q0 = own ? kOwnSeq : 0;
     if (!T || !s->kv.n) return fail(PI_E_STATE, "pi_model_generate: decode a prompt first");
     if (n_steps <= 0 || n_steps > s->max_steps || !out_tokens) return fail(PI_E_ARG, "pi_model_generate: bad step count");
-    std::vector<int32_t> tok(T), pos(T), vis(T), seq(T), cell(T), cells((size_t)n_steps * T), app;
+    std::vector<int32_t> tok(T), pos(T), vis(T), seq(T), cell(T), prev(T), lin(4 * T), cells((size_t)n_steps * T), app;
     PI_TRY(apply_shift(m));
     for (int t = 0; t < T; ++t) {
         seq[t] = q0 + t; tok[t] = s->last_tok[q0 + t]; pos[t] = s->last_pos[q0 + t];
         refresh_list(s, q0 + t, app);
         if (pos[t] + n_steps > m->hp.n_ctx) return fail(PI_E_ARG, "pi_model_generate: would run past the context");
         if ((int)s->list_pos[q0 + t].size() != pos[t]) return fail(PI_E_STATE, "pi_model_generate: a sequence's cells do not end at its next position");
+        prev[t] = pos[t] ? s->cell_tok[s->list_cells[q0 + t].back()] : -1;
+        if (s->recurrent) {
+            PI_TRY(take_slot(m, q0 + t, ((1u << T) - 1) << q0));
+            if (pos[t] == 0)
+                for (Layer & L : s->layers) for (float * st : L.state) PI_TRY(pi_memset(st + s->slot_of[q0 + t] * L.state_floats(), 0, L.state_floats() * 4));
+        }
     }
     if (!s->kv.find_free(n_steps * T, cells.data())) return fail(PI_E_STATE, "pi_model_generate: not enough free cells");
     for (int k = 0; k < n_steps; ++k)
-        for (int t = 0; t < T; ++t) take_cell(s, cells[(size_t)k * T + t], pos[t] + k, 1u << (q0 + t), app);
+        for (int t = 0; t < T; ++t) take_cell(s, cells[(size_t)k * T + t], pos[t] + k, 1u << (q0 + t), k ? -1 : tok[t], app);
     s->kv.move_head(cells.back() + 1);
     PI_TRY(upload_appends(m, app));
     PI_TRY(ensure_capacity(m, T));
@@ -836,14 +1243,23 @@ int layers_generate(pi_model * m, int own, int n_steps, int32_t * out_tokens, fl
     for (const HeadKind & h : s->kinds) {
         Step::Work w;
         const size_t at = items.size();
-        if (bf16_mode(s)) work_items(seq.data(), vis.data(), T, h, items, nullptr);
+        const int vmax = *std::max_element(pos.begin(), pos.end()) + n_steps;
+        if (bf16_mode(s)) { if (h.mixer == PI_MIXER_GROUPED) gqa_items(seq.data(), vis.data(), T, h.n_head, items, nullptr); else work_items(seq.data(), vis.data(), T, h, items, nullptr); }
         w.items = s->g_work + at;
         w.n = bf16_mode(s) ? (int)(items.size() - at) / 4 : T;
-        w.parts = choose_parts(s, w.n, *std::max_element(pos.begin(), pos.end()) + n_steps);
+        w.parts = h.mixer == PI_MIXER_GROUPED ? (bf16_mode(s) ? gqa_parts(w.n * h.n_kv, vmax, 128) : 1) : choose_parts(s, w.n, vmax);
         in.work.push_back(w);
+        in.wide.emplace_back();
         parts.push_back(w.parts);
     }
     PI_HIP_TRY(hipStreamSynchronize(m->stream));
+    if (s->recurrent) {
+        for (int t = 0; t < T; ++t) { lin[4 * t] = t; lin[4 * t + 1] = 1; lin[4 * t + 2] = s->slot_of[q0 + t]; lin[4 * t + 3] = 0; }
+        in.lin = s->g_lin; in.n_lin = T;
+        PI_TRY(pi_memcpy_h2d(s->g_lin, lin.data(), 16 * T));
+    }
+    in.prev = s->g_prev; in.carry = true;
+    PI_TRY(pi_memcpy_h2d(s->g_prev, prev.data(), 4 * T));
     const int32_t zero = 0;
     PI_TRY(pi_memcpy_h2d(s->g_tok, tok.data(), 4 * T)); PI_TRY(pi_memcpy_h2d(s->g_pos, pos.data(), 4 * T)); PI_TRY(pi_memcpy_h2d(s->g_vis, vis.data(), 4 * T));
     PI_TRY(pi_memcpy_h2d(s->g_seq, seq.data(), 4 * T)); PI_TRY(pi_memcpy_h2d(s->g_cell, cell.data(), 4 * T)); PI_TRY(pi_memcpy_h2d(s->g_step, &zero, 4));
@@ -880,14 +1296,42 @@ int layers_generate(pi_model * m, int own, int n_steps, int32_t * out_tokens, fl
     PI_HIP_TRY(hipStreamSynchronize(m->stream));
     if (ms_out) PI_HIP_TRY(hipEventElapsedTime(ms_out, m->ev0, m->ev1));
     PI_TRY(pi_memcpy_d2h(out_tokens, s->g_out, sizeof(int32_t) * (size_t)n_steps * T));
+    for (int k = 1; k < n_steps; ++k) for (int t = 0; t < T; ++t) s->cell_tok[cells[(size_t)k * T + t]] = out_tokens[(size_t)(k - 1) * T + t];
     for (int t = 0; t < T; ++t) { s->last_tok[q0 + t] = out_tokens[(size_t)(n_steps - 1) * T + t]; s->last_pos[q0 + t] = pos[t] + n_steps; }
     return PI_OK;
+}
+
+// a recurrent state cannot lose or move some of its tokens: edits that leave a sequence neither whole nor empty are refused (edit empty: any)
+int layers_edit_allowed(pi_model * m, const std::function<void(KvCells &)> & edit) {
+    LayerState * s = m->lay;
+    if (!s->recurrent || (edit && keeps_whole(s, edit))) return PI_OK;
+    return fail(PI_E_UNSUPPORTED, "KV edit: a model with recurrent states cannot drop or move part of a sequence");
+}
+
+// before the cells of src in [p0, p1) become dst's as well: its states do, if that is all of src and dst is empty
+int layers_copy_state(pi_model * m, int src, int dst, int p0, int p1) {
+    LayerState * s = m->lay;
+    if (!s->recurrent || src == dst) return PI_OK;
+    int all = 0, taken = 0;
+    for (int i = 0; i < s->kv.n; ++i) {
+        if (s->kv.pos[i] < 0 || !(s->kv.seq[i] >> src & 1u)) continue;
+        ++all;
+        taken += s->kv.pos[i] >= std::max(p0, 0) && (p1 < 0 || s->kv.pos[i] < p1);
+    }
+    if (taken == 0) return PI_OK;
+    if (taken != all || live_cells(s, dst) != 0 || s->slot_of[src] < 0) return fail(PI_E_UNSUPPORTED, "KV edit: a model with recurrent states copies whole sequences into empty ones");
+    PI_TRY(take_slot(m, dst, 1u << dst));
+    PI_HIP_TRY(hipStreamSynchronize(m->stream));
+    for (Layer & L : s->layers)
+        for (float * st : L.state) PI_TRY(pi_memcpy_d2d(st + s->slot_of[dst] * L.state_floats(), st + s->slot_of[src] * L.state_floats(), L.state_floats() * 4));
+    return pi_sync();
 }
 
 int layers_seq_edit(pi_model * m, int seq, int p0, int p1, int delta, bool shift) {
     LayerState * s = m->lay;
     if (seq < -1 || seq >= s->n_seq || !s->kv.n) return fail(PI_E_ARG, "KV edit: bad sequence");
     const int q = seq < 0 ? kOwnSeq : seq;
+    PI_TRY(shift ? layers_edit_allowed(m, nullptr) : layers_edit_allowed(m, [&](KvCells & kv) { kv.seq_rm(q, p0, p1); }));
     if (shift) s->kv.seq_shift(q, p0, p1, delta); else s->kv.seq_rm(q, p0, p1);
     const int n = live_cells(s, q);
     s->last_pos[q] = n;
@@ -898,6 +1342,7 @@ int layers_seq_cp(pi_model * m, int src, int dst, int p0, int p1) {
     LayerState * s = m->lay;
     if (src < 0 || dst < 0 || src >= s->n_seq || dst >= s->n_seq || src == dst) return fail(PI_E_ARG, "pi_model_batch_kv_seq_cp: bad sequences");
     if (live_cells(s, dst) != std::max(p0, 0)) return fail(PI_E_UNSUPPORTED, "pi_model_batch_kv_seq_cp: the destination must hold exactly p0 cells");
+    PI_TRY(layers_copy_state(m, src, dst, p0, p1));
     s->kv.seq_cp(src, dst, p0, p1);                                // shared, not copied
     s->last_pos[dst] = live_cells(s, dst);
     return s->last_pos[dst];
@@ -909,12 +1354,25 @@ extern "C" {
 
 pi_model * pi_model_create_layers(const pi_hparams * hp, const pi_layers_opts * opts, const pi_layer_desc * layers, int n_layer) {
     const auto bad = [](const char * why) -> pi_model * { pi::set_error(why); return nullptr; };
-    if (!hp || !opts || !layers || n_layer <= 0 || hp->n_embd <= 0 || hp->n_vocab <= 0 || hp->n_ctx <= 0 || hp->arch != PI_ARCH_LERASUN ||
+    if (!hp || !opts || !layers || n_layer <= 0 || hp->n_embd <= 0 || hp->n_vocab <= 0 || hp->n_ctx <= 0 || (hp->arch != PI_ARCH_LERASUN && hp->arch != PI_ARCH_PIBALORN) ||
         (opts->compute != PI_TYPE_BF16 && opts->compute != PI_TYPE_F32) || opts->max_batch < 0)
         return bad("pi_model_create_layers: inconsistent hyper-parameters");
+    const bool one_norm = layers[0].mixer != PI_MIXER_LATENT;
     for (int il = 0; il < n_layer; ++il) {
         const pi_layer_desc & d = layers[il];
-        if (d.mixer != PI_MIXER_LATENT || d.n_head <= 0 || d.dim <= 0 || d.rot_dim <= 0 || d.rot_dim % 2 || d.vdim <= 0 || d.kv_rank <= 0 || !(d.rot_base > 0.0))
+        if ((d.mixer != PI_MIXER_LATENT) != one_norm) return bad("pi_model_create_layers: layers of one and of two norms in one model");
+        if (one_norm) {
+            if ((d.mixer != PI_MIXER_GROUPED && d.mixer != PI_MIXER_LINEAR) || d.n_head <= 0 || d.dim <= 0 || d.vdim <= 0) return bad("pi_model_create_layers: a layer's mixer");
+            if (d.mixer == PI_MIXER_GROUPED && (d.n_kv_head <= 0 || d.n_head % d.n_kv_head || d.rot_dim < 0 || d.rot_dim % 2 || d.rot_dim > d.dim || (d.rot_dim && !(d.rot_base > 0.0)) ||
+                                                (d.values_are_keys && d.vdim != d.dim)))
+                return bad("pi_model_create_layers: a layer's grouped-query attention");
+            if (d.ffn != PI_FFN_NONE && d.ffn != PI_FFN_GLU && d.ffn != PI_FFN_GLU_MOE) return bad("pi_model_create_layers: a layer's feed-forward");
+            if (d.glu_ff < 0 || (d.ffn == PI_FFN_GLU) > (d.glu_ff > 0) || (d.ffn == PI_FFN_NONE && d.glu_ff) ||
+                (d.ffn == PI_FFN_GLU_MOE && (d.n_expert <= 0 || d.n_expert > 4096 || d.n_top <= 0 || d.n_top > d.n_expert || d.expert_ff <= 0)))
+                return bad("pi_model_create_layers: a layer's experts");
+            continue;
+        }
+        if (d.n_head <= 0 || d.dim <= 0 || d.rot_dim <= 0 || d.rot_dim % 2 || d.vdim <= 0 || d.kv_rank <= 0 || !(d.rot_base > 0.0))
             return bad("pi_model_create_layers: a layer's mixer");
         if (d.kv_from >= 0) {
             if (d.kv_from >= il) return bad("pi_model_create_layers: kv_from must name an earlier layer");
@@ -926,6 +1384,9 @@ pi_model * pi_model_create_layers(const pi_hparams * hp, const pi_layers_opts * 
                                      d.n_top <= 0 || d.n_top > d.n_group_keep * (d.n_expert / d.n_group) || d.expert_ff <= 0))
             return bad("pi_model_create_layers: a layer's experts");
     }
+    if (opts->loop_times < 0 || (opts->loop_times > 0 && (!one_norm || opts->loop_start < 0 || opts->loop_start >= opts->loop_stop || opts->loop_stop > n_layer)) || opts->bigram_buckets < 0 ||
+        (opts->bigram_buckets && (!one_norm || opts->bigram_mul_prev < 0 || opts->bigram_mul_cur < 0)))
+        return bad("pi_model_create_layers: the loop or the bigram table");
     if (pi_init(0) != PI_OK) return nullptr;
     pi_model * m = new pi_model();
     m->hp = *hp;
@@ -933,7 +1394,21 @@ pi_model * pi_model_create_layers(const pi_hparams * hp, const pi_layers_opts * 
     m->layers.resize((size_t)n_layer * PI_T_COUNT);
     m->lay = new LayerState();
     m->lay->opts = *opts;
-    for (int il = 0; il < n_layer; ++il) { Layer L; L.d = layers[il]; m->lay->layers.push_back(L); }
+    LayerState * s = m->lay;
+    s->one_norm = one_norm;
+    std::fill(s->slot_of, s->slot_of + 32, -1);
+    const int lo = opts->loop_times > 0 ? opts->loop_start : n_layer, hi = opts->loop_times > 0 ? opts->loop_stop : n_layer;
+    for (int il = 0; il < n_layer; ++il) {
+        Layer L;
+        L.d = layers[il];
+        const int passes = il >= lo && il < hi ? opts->loop_times : 1;
+        if (L.d.mixer == PI_MIXER_LINEAR) { L.state.resize(passes, nullptr); s->recurrent = true; }
+        else if (L.d.mixer == PI_MIXER_GROUPED || L.d.kv_from < 0) L.cache.resize(passes, nullptr);
+        s->layers.push_back(L);
+    }
+    for (int il = 0; il < lo; ++il) s->order.push_back({il, 0, false});
+    for (int t = 0; t < opts->loop_times; ++t) for (int il = lo; il < hi; ++il) s->order.push_back({il, t, il == lo});
+    for (int il = hi; il < n_layer; ++il) s->order.push_back({il, 0, false});
     return m;
 }
 
@@ -941,7 +1416,7 @@ int pi_model_get_streams(pi_model * m, float * out) {
     if (!m || !m->finalized || !m->lay || !m->capture || !m->lay->streams_T) return pi::fail(PI_E_STATE, "pi_model_get_streams: run a step with capture enabled first");
     LayerState * s = m->lay;
     PI_HIP_TRY(hipStreamSynchronize(m->stream));
-    if (out) PI_TRY(pi_memcpy_d2h(out, s->streams, sizeof(float) * s->layers.size() * (size_t)s->streams_T * m->hp.n_embd));
+    if (out) PI_TRY(pi_memcpy_d2h(out, s->streams, sizeof(float) * s->order.size() * (size_t)s->streams_T * m->hp.n_embd));
     return s->streams_T;
 }
 

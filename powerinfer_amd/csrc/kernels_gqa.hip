@@ -1,0 +1,408 @@
+// Grouped-query attention on cells that lie anywhere in the pool: lists[seq] names a sequence's cells in position order.  A cell of a
+// layer is, per key / value head, one row [key | value] of 2 * hd values, so that what a head reads of a cell is contiguous.
+#include "mixers.hpp"
+
+namespace {
+
+// ---------------------------------------------------------------------------------------------------------------------------------
+// behind the joint projection: a wave per head - rotation, division by the root mean square, query row or cell
+// ---------------------------------------------------------------------------------------------------------------------------------
+constexpr int kGqaMaxDim = 256;
+template <typename ST>
+__global__ __launch_bounds__(256) void gqa_prep_kernel(pi_gqa_prep p, pi_ffn_front f, int n_heads4, int per) {
+    extern __shared__ __align__(16) float sm[];
+    const int t = blockIdx.x / per, b = blockIdx.x % per;
+    if (b >= n_heads4) { front_block<ST>(f, p.z, p.ldz, t, b - n_heads4, sm); return; }
+    const int head = b * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63, half = p.rot_dim / 2;
+    if (head >= p.n_head + p.n_kv) return;
+    const bool key = head >= p.n_head;
+    const int g = head - p.n_head;
+    const float * z = p.z + (size_t)t * p.ldz, * src = key ? z + p.off_k + g * p.dim : z + head * p.dim;
+    const float2 * cs = (const float2 *)p.cs + (size_t)t * half;
+    constexpr int J = kGqaMaxDim / 64;
+    float x[J];
+    float ss = 0.0f;
+#pragma unroll
+    for (int j = 0; j < J; ++j) {
+        const int e = lane + 64 * j;
+        float v = 0.0f;
+        if (e < p.dim) {
+            v = src[e];
+            if (e < half) { const float2 c = cs[e]; v = v * c.x - src[e + half] * c.y; }
+            else if (e < 2 * half) { const float2 c = cs[e - half]; v = v * c.x + src[e - half] * c.y; }
+        }
+        x[j] = v;
+        ss = fmaf(v, v, ss);
+    }
+    float sc = 1.0f;
+    if (p.unit) sc = pi_inv_sqrt(pi_wave_sum(ss) / (float)p.dim + p.eps);
+    ST * row = key ? (ST *)p.cache + ((size_t)p.cell[t] * p.n_kv + g) * 2 * p.hd : (ST *)p.q + ((size_t)t * p.n_head + head) * p.hd;
+#pragma unroll
+    for (int j = 0; j < J; ++j) { const int e = lane + 64 * j; if (e < p.hd) row[e] = to_st<ST>(x[j] * sc); }      // (zeros behind dim)
+    if (key) {
+        const float * v = z + p.off_v + g * p.vdim;
+#pragma unroll
+        for (int j = 0; j < J; ++j) { const int e = lane + 64 * j; if (e < p.hd) row[p.hd + e] = to_st<ST>(e < p.vdim ? v[e] : 0.0f); }
+    }
+}
+
+// ---------------------------------------------------------------------------------------------------------------------------------
+// bf16 attention on the matrix cores.  Scores are formed transposed (keys x query rows), so that a lane's scores belong to one row, its
+// soft-max needs two shuffles, and its weights are already the column operand of the second product (values^T x weights) - which key a
+// slot of that product's inner dimension stands for is free, so the value operand is read (transposed, ds_read_tr16) in the order the
+// scores came out.  Query rows are (token, head of the group) pairs, heads innermost: the rows of a token share its cells.
+//   WIDE: 128 rows, 32 per wave, against 64 cells at a time (long runs).
+//   else: 16 rows, the same in every wave, against 128 cells at a time, 32 per wave; the waves' sums are merged at the end.
+// ---------------------------------------------------------------------------------------------------------------------------------
+typedef short pi_s4 __attribute__((ext_vector_type(4)));
+__device__ __forceinline__ pi_s4 tr_read(const unsigned char * q) {
+    return __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) pi_s4 *)(__attribute__((address_space(3))) void *)q);
+}
+
+template <int KS, bool WIDE> constexpr size_t gqa_lds() { return (size_t)2 * (WIDE ? 64 : 128) * (KS * 64 + 16); }
+
+template <int KS, bool WIDE>      // 32-column steps of a key or value row
+__global__ __launch_bounds__(256, WIDE && KS <= 4 ? 2 : 1) void gqa_attn_kernel(pi_gqa_attn p) {
+    constexpr int VT = 2 * KS, NK = WIDE ? 64 : 128, R = WIDE ? 128 : 16, U = WIDE ? 2 : 1, KT = WIDE ? 4 : 2, ROW = KS * 64 + 16, NKK = NK / 32, HD = KS * 32;
+    extern __shared__ __align__(16) unsigned char smem[];
+    unsigned char * ks = smem, * vs = smem + NK * ROW;
+    const int g = blockIdx.x % p.n_kv, item_index = p.n_work - 1 - (int)blockIdx.x / p.n_kv, part = blockIdx.y;      // the last items see the most cells
+    const int4 item = reinterpret_cast<const int4 *>(p.work)[item_index];
+    const int tok0 = item.x, first = item.y, rows = min(item.z, R), per = p.n_head / p.n_kv;
+    const int32_t * list = p.lists + (size_t)item.w * p.list_ld;
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, i = lane & 15, gq = lane >> 4;
+    const int n_keys = p.n_vis[tok0 + (first + rows - 1) / per], n_all = p.n_vis[tok0 + first / per];       // the most and the fewest cells a row here sees
+    const int tiles = (n_keys + NK - 1) / NK;
+    const int c0 = (int)((long long)tiles * part / p.n_parts) * NK, c1 = min((int)((long long)tiles * (part + 1) / p.n_parts) * NK, n_keys);
+    // the thread's pieces of a tile: eight threads share a cell's row
+    const int sub = tid % 8, key0 = tid / 8;
+    const uint16_t * cache = (const uint16_t *)p.cache + (size_t)g * 2 * HD + sub * 8;
+    int idx[NKK];
+    pi_u32x4 pre[NKK][KS];
+    auto look_up = [&](int cb) {
+#pragma unroll
+        for (int k = 0; k < NKK; ++k) idx[k] = list[min(cb + key0 + 32 * k, n_keys - 1)];
+    };
+    auto fetch = [&]() {
+#pragma unroll
+        for (int k = 0; k < NKK; ++k)
+#pragma unroll
+            for (int j = 0; j < KS; ++j) pre[k][j] = pi_ld16(cache + (size_t)idx[k] * p.n_kv * 2 * HD + j * 64);
+    };
+    if (c0 < c1) look_up(c0);
+    int row[U], tok[U], head[U], nv[U];
+    pi_u32x4 qf[U][KS];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+        row[u] = (WIDE ? wave * 32 : 0) + u * 16 + i;
+        const int rr = first + min(row[u], rows - 1);
+        tok[u] = tok0 + rr / per;
+        head[u] = g * per + rr % per;
+        nv[u] = row[u] < rows ? p.n_vis[tok[u]] : 0;
+#pragma unroll
+        for (int s = 0; s < KS; ++s) qf[u][s] = pi_ld16((const uint16_t *)p.q + ((size_t)tok[u] * p.n_head + head[u]) * HD + s * 32 + gq * 8);
+    }
+    if (c0 < c1) { fetch(); look_up(c0 + NK); }
+    float m[U], l[U];
+    pi_f4 o[U][VT];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+        m[u] = -INFINITY; l[u] = 0.0f;
+#pragma unroll
+        for (int v = 0; v < VT; ++v) o[u][v] = pi_f4{0, 0, 0, 0};
+    }
+    const int kb = WIDE ? 0 : wave * 32;                         // this wave's cells of a tile
+    for (int cb = c0; cb < c1; cb += NK) {
+        __syncthreads();
+#pragma unroll
+        for (int k = 0; k < NKK; ++k)
+#pragma unroll
+            for (int j = 0; j < KS; ++j) {
+                const int c = sub + 8 * j;
+                *reinterpret_cast<pi_u32x4 *>((c < 4 * KS ? ks + c * 16 : vs + (c - 4 * KS) * 16) + (key0 + 32 * k) * ROW) = pre[k][j];
+            }
+        __syncthreads();
+        fetch();                                                 // past the last tile: rows of the last cell, not used
+        look_up(cb + 2 * NK);
+        pi_f4 s[U][KT];
+#pragma unroll
+        for (int kt = 0; kt < KT; ++kt) {
+#pragma unroll
+            for (int u = 0; u < U; ++u) s[u][kt] = pi_f4{0, 0, 0, 0};
+#pragma unroll
+            for (int c = 0; c < KS; ++c) {
+                const pi_u32x4 a = *reinterpret_cast<const pi_u32x4 *>(ks + (kb + kt * 16 + i) * ROW + c * 64 + gq * 16);
+#pragma unroll
+                for (int u = 0; u < U; ++u) s[u][kt] = mfma_bf16(a, qf[u][c], s[u][kt]);
+            }
+        }
+        pi_u32x4 pb[U][KT / 2];                                  // weights as the column operand
+        const bool edge = cb + NK > n_all;
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            float mx = -INFINITY;
+#pragma unroll
+            for (int kt = 0; kt < KT; ++kt)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    float v = s[u][kt][r] * p.scale;
+                    if (edge && cb + kb + kt * 16 + 4 * gq + r >= nv[u]) v = -INFINITY;
+                    s[u][kt][r] = v;
+                    mx = fmaxf(mx, v);
+                }
+            mx = fmaxf(mx, __shfl_xor(mx, 16, PI_WAVE));
+            mx = fmaxf(mx, __shfl_xor(mx, 32, PI_WAVE));
+            const float mn = fmaxf(m[u], mx), base = mn == -INFINITY ? 0.0f : mn;
+            const float a = expf(m[u] - base);                   // 0 while nothing has been seen
+            m[u] = mn;
+            float sum = 0.0f;
+            bf16 w[4 * KT];
+#pragma unroll
+            for (int kt = 0; kt < KT; ++kt)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) { const float e = expf(s[u][kt][r] - base); sum += e; w[kt * 4 + r] = (bf16)e; }
+            l[u] = l[u] * a + sum;
+#pragma unroll
+            for (int v = 0; v < VT; ++v) { o[u][v][0] *= a; o[u][v][1] *= a; o[u][v][2] *= a; o[u][v][3] *= a; }
+#pragma unroll
+            for (int k = 0; k < KT / 2; ++k) {
+                bf16 b[8];
+#pragma unroll
+                for (int j = 0; j < 8; ++j) b[j] = w[k * 8 + j];
+                pb[u][k] = __builtin_bit_cast(pi_u32x4, b);
+            }
+        }
+        // slot (gq, j) of a 32-cell step: cell 4 gq + j of its first 16 (j < 4) or of its second 16 - two transposing reads
+#pragma unroll
+        for (int k = 0; k < KT / 2; ++k)
+#pragma unroll
+            for (int v = 0; v < VT; ++v) {
+                const unsigned char * a = vs + (kb + k * 32 + 4 * gq + (i >> 2)) * ROW + (v * 16 + (i & 3) * 4) * 2;
+                const pi_u32x2 lo = __builtin_bit_cast(pi_u32x2, tr_read(a)), hi = __builtin_bit_cast(pi_u32x2, tr_read(a + 16 * ROW));
+                const pi_u32x4 fr{lo.x, lo.y, hi.x, hi.y};
+#pragma unroll
+                for (int u = 0; u < U; ++u) o[u][v] = mfma_bf16(fr, pb[u][k], o[u][v]);
+            }
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u) { l[u] += __shfl_xor(l[u], 16, PI_WAVE); l[u] += __shfl_xor(l[u], 32, PI_WAVE); }
+    const bool whole = p.n_parts == 1, quads = ((p.vdim | p.ld_att) & 3) == 0;
+    const size_t srow0 = ((size_t)item_index * p.n_kv + g) * R;
+    float2 * ml = reinterpret_cast<float2 *>(p.scratch + (size_t)p.n_work * p.n_kv * R * p.n_parts * HD);
+    if (WIDE) {
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            if (row[u] >= rows) continue;
+            if (!whole) {
+                float * acc = p.scratch + ((srow0 + row[u]) * p.n_parts + part) * HD;
+#pragma unroll
+                for (int v = 0; v < VT; ++v) *reinterpret_cast<pi_f4 *>(acc + v * 16 + 4 * gq) = o[u][v];
+                if (gq == 0) ml[(srow0 + row[u]) * p.n_parts + part] = make_float2(m[u], l[u]);
+                continue;
+            }
+            const float mf = fmaxf(m[u], p.sink), a = m[u] == -INFINITY ? 0.0f : expf(m[u] - mf), f = a / (l[u] * a + expf(p.sink - mf));
+            bf16 * out = (bf16 *)p.att + (size_t)tok[u] * p.ld_att + head[u] * p.vdim;
+#pragma unroll
+            for (int v = 0; v < VT; ++v) {
+                const int c = v * 16 + 4 * gq;
+                const float w[4] = {o[u][v][0] * f, o[u][v][1] * f, o[u][v][2] * f, o[u][v][3] * f};
+                if (c < p.vdim) store4(out + c, w, quads && c + 4 <= p.vdim, p.vdim - c);
+            }
+        }
+        return;
+    }
+    // merge of the waves' sums
+    __syncthreads();
+    constexpr int OLD = HD + 4;
+    float * os = reinterpret_cast<float *>(smem);                // [4][16][OLD]
+    float2 * wm = reinterpret_cast<float2 *>(os + 4 * 16 * OLD); // [4][16]
+#pragma unroll
+    for (int v = 0; v < VT; ++v) *reinterpret_cast<pi_f4 *>(os + (wave * 16 + i) * OLD + v * 16 + 4 * gq) = o[0][v];
+    if (gq == 0) wm[wave * 16 + i] = make_float2(m[0], l[0]);
+    __syncthreads();
+    const int r = tid >> 4, cl = tid & 15;
+    if (r >= rows) return;
+    float mm = -INFINITY, f[4], sum = 0.0f;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) mm = fmaxf(mm, wm[w * 16 + r].x);
+#pragma unroll
+    for (int w = 0; w < 4; ++w) { const float2 x = wm[w * 16 + r]; f[w] = x.x == -INFINITY ? 0.0f : expf(x.x - mm); sum += f[w] * x.y; }
+    float fin = 1.0f;
+    if (whole) {
+        const float mf = fmaxf(mm, p.sink), a = mm == -INFINITY ? 0.0f : expf(mm - mf);
+        fin = a / (sum * a + expf(p.sink - mf));
+    } else if (cl == 0) ml[(srow0 + r) * p.n_parts + part] = make_float2(mm, sum);
+    const int rr = first + r;
+    bf16 * out = (bf16 *)p.att + (size_t)(tok0 + rr / per) * p.ld_att + (g * per + rr % per) * p.vdim;
+    float * acc = p.scratch + ((srow0 + r) * p.n_parts + part) * HD;
+    for (int c = cl * 4; c < HD; c += 64) {
+        float v[4] = {0, 0, 0, 0};
+#pragma unroll
+        for (int w = 0; w < 4; ++w) {
+            const pi_f4 x = *reinterpret_cast<const pi_f4 *>(os + (w * 16 + r) * OLD + c);
+#pragma unroll
+            for (int k = 0; k < 4; ++k) v[k] = fmaf(f[w], x[k], v[k]);
+        }
+        if (whole) {
+#pragma unroll
+            for (int k = 0; k < 4; ++k) v[k] *= fin;
+            if (c < p.vdim) store4(out + c, v, quads && c + 4 <= p.vdim, p.vdim - c);
+        } else {
+            *reinterpret_cast<float4 *>(acc + c) = make_float4(v[0], v[1], v[2], v[3]);
+        }
+    }
+}
+
+__global__ __launch_bounds__(256) void gqa_merge_kernel(pi_gqa_attn p) {
+    const int R4 = gqa_rows(p.wide) / 4, wg = blockIdx.x;
+    gqa_merge_row(p, wg / R4 / p.n_kv, wg / R4 % p.n_kv, (wg % R4) * 4 + (threadIdx.x >> 6));
+}
+
+// fp32: one workgroup per (token, head), 64 cells at a time (a wave per cell for the scores, a thread per column for the sum)
+constexpr int kGfCells = 64;
+__global__ __launch_bounds__(256) void gqa_attn_f32_kernel(pi_gqa_attn p) {
+    __shared__ float q[kGqaMaxDim], s[kGfCells];
+    __shared__ int idx[kGfCells];
+    const int t = blockIdx.x / p.n_head, h = blockIdx.x % p.n_head, g = h / (p.n_head / p.n_kv), tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+    const int n = p.n_vis[t];
+    const int32_t * list = p.lists + (size_t)p.work[t] * p.list_ld;
+    const float * cache = (const float *)p.cache + (size_t)g * 2 * p.hd;
+    const size_t cell_ld = (size_t)p.n_kv * 2 * p.hd;
+    for (int k = tid; k < p.dim; k += 256) q[k] = ((const float *)p.q)[(size_t)blockIdx.x * p.hd + k];
+    const bool sink = p.sink != -INFINITY;
+    float m = p.sink, l = sink ? 1.0f : 0.0f, acc = 0.0f;              // the sink is the soft-max's first entry: weight exp(0), no value
+    for (int c0 = 0; c0 < n; c0 += kGfCells) {
+        const int nc = min(kGfCells, n - c0);
+        __syncthreads();
+        for (int c = tid; c < nc; c += 256) idx[c] = list[c0 + c];
+        __syncthreads();
+        for (int c = wave; c < nc; c += 4) {
+            const float * row = cache + idx[c] * cell_ld;
+            float d = 0.0f;
+            for (int k = lane; k < p.dim; k += 64) d = fmaf(q[k], row[k], d);
+            d = pi_wave_sum(d);
+            if (lane == 0) s[c] = d * p.scale;
+        }
+        __syncthreads();
+        float mn = m;
+        for (int c = 0; c < nc; ++c) mn = fmaxf(mn, s[c]);
+        const float a = m == -INFINITY ? 0.0f : expf(m - mn);
+        l *= a;
+        acc *= a;
+        for (int c = 0; c < nc; ++c) {
+            const float w = expf(s[c] - mn);
+            l += w;
+            if (tid < p.vdim) acc = fmaf(w, cache[idx[c] * cell_ld + p.hd + tid], acc);
+        }
+        m = mn;
+    }
+    if (tid < p.vdim) ((float *)p.att)[(size_t)t * p.ld_att + h * p.vdim + tid] = acc / l;
+}
+
+template <typename ST>
+__global__ void gqa_shift_kernel(ST * __restrict__ cache, int n_kv, int hd, int rot_dim, double base, const int32_t * __restrict__ delta) {
+    const int c = blockIdx.x, d = delta[c], half = rot_dim / 2;
+    if (d == 0) return;
+    for (int e = threadIdx.x; e < n_kv * half; e += blockDim.x) {
+        const int g = e / half, i = e % half;
+        double sn, cn;
+        sincos((double)d * pow(base, -2.0 * (double)i / (double)rot_dim), &sn, &cn);
+        ST * r = cache + ((size_t)c * n_kv + g) * 2 * hd + i;
+        const float u = from_st(r[0]), v = from_st(r[half]);
+        r[0] = to_st<ST>(u * (float)cn - v * (float)sn);
+        r[half] = to_st<ST>(v * (float)cn + u * (float)sn);
+    }
+}
+
+template <int KS, bool WIDE> int launch_gqa(const pi_gqa_attn * p, hipStream_t st) {
+    constexpr size_t tile = gqa_lds<KS, WIDE>(), merge = WIDE ? 0 : sizeof(float) * (4 * 16 * (KS * 32 + 4) + 2 * 4 * 16), lds = tile > merge ? tile : merge;
+    static bool raised = false;
+    if (!raised && lds > 64 * 1024) {
+        PI_HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void *>(&gqa_attn_kernel<KS, WIDE>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
+        raised = true;
+    }
+    hipLaunchKernelGGL((gqa_attn_kernel<KS, WIDE>), dim3(p->n_work * p->n_kv, p->n_parts), dim3(256), lds, st, *p);
+    return pi::check_launch("pi_k_gqa_attn");
+}
+
+int gqa_check(int type, const pi_gqa_attn * p) {
+    if (!p || !p->q || !p->cache || !p->lists || !p->work || !p->n_vis || !p->att || p->T <= 0 || p->n_head <= 0 || p->n_kv <= 0 || p->n_head % p->n_kv || p->dim <= 0 || p->vdim <= 0 ||
+        p->hd < p->dim || p->hd < p->vdim || p->ld_att < p->n_head * p->vdim || p->hd != pi_k_gqa_head_ld(type, p->dim, p->vdim) || p->n_parts <= 0)
+        return pi::fail(PI_E_ARG, "pi_k_gqa_attn: bad arguments");
+    if (type == PI_TYPE_BF16 && (p->n_work <= 0 || (long long)p->n_work * p->n_kv > (1 << 30) || p->n_parts > 64 || (p->n_parts > 1 && !p->scratch)))
+        return pi::fail(PI_E_ARG, "pi_k_gqa_attn: bad work arguments");
+    return PI_OK;
+}
+
+template <bool WIDE> int gqa_bf16(const pi_gqa_attn * p, hipStream_t st) {
+    switch (p->hd) {
+        case 32: return launch_gqa<1, WIDE>(p, st);
+        case 64: return launch_gqa<2, WIDE>(p, st);
+        case 96: return launch_gqa<3, WIDE>(p, st);
+        case 128: return launch_gqa<4, WIDE>(p, st);
+        case 192: return launch_gqa<6, WIDE>(p, st);
+        default: return launch_gqa<8, WIDE>(p, st);
+    }
+}
+
+}  // namespace
+
+extern "C" {
+
+int pi_k_gqa_head_ld(int type, int dim, int vdim) {
+    const int d = dim > vdim ? dim : vdim;
+    if (dim <= 0 || vdim <= 0 || d > kGqaMaxDim) return 0;
+    if (type == PI_TYPE_F32) return (d + 31) / 32 * 32;
+    return d <= 128 ? (d + 31) / 32 * 32 : d <= 192 ? 192 : 256;
+}
+
+int pi_k_gqa_prep(int type, const pi_gqa_prep * p, const pi_ffn_front * front, pi_stream_t stream) {
+    const pi_ffn_front f = front ? *front : pi_ffn_front{};
+    if (!p || !p->z || !p->cs || !p->q || !p->cache || !p->cell || p->T <= 0 || p->n_head <= 0 || p->n_kv <= 0 || p->n_head % p->n_kv || p->rot_dim < 0 || p->rot_dim % 2 || p->rot_dim > p->dim ||
+        p->hd != pi_k_gqa_head_ld(type, p->dim, p->vdim) || p->hd <= 0 || p->off_k < p->n_head * p->dim || p->off_k + p->n_kv * p->dim > p->ldz || p->off_v < 0 ||
+        p->off_v + p->n_kv * p->vdim > p->ldz || !front_ok(f, p->ldz))
+        return pi::fail(PI_E_ARG, "pi_k_gqa_prep: bad arguments");
+    const int n4 = (p->n_head + p->n_kv + 3) / 4, per = n4 + front_blocks(f);
+    if ((long long)per * p->T > (1 << 30)) return pi::fail(PI_E_ARG, "pi_k_gqa_prep: too many tokens");
+    if (type == PI_TYPE_BF16) hipLaunchKernelGGL(gqa_prep_kernel<bf16>, dim3(per * p->T), dim3(256), front_lds_bytes(f), (hipStream_t)stream, *p, f, n4, per);
+    else if (type == PI_TYPE_F32) hipLaunchKernelGGL(gqa_prep_kernel<float>, dim3(per * p->T), dim3(256), front_lds_bytes(f), (hipStream_t)stream, *p, f, n4, per);
+    else return pi::fail(PI_E_UNSUPPORTED, "pi_k_gqa_prep: type");
+    return pi::check_launch("pi_k_gqa_prep");
+}
+
+int pi_k_gqa_rows(int wide) { return gqa_rows(wide); }
+
+size_t pi_k_gqa_scratch_floats(int n_work, int wide, int n_kv, int hd, int n_parts) {
+    return n_parts > 1 ? (size_t)n_work * gqa_rows(wide) * n_kv * n_parts * (hd + 2) : 0;
+}
+
+int pi_k_gqa_attn_parts(const pi_gqa_attn * p, pi_stream_t stream) {
+    const int rc = gqa_check(PI_TYPE_BF16, p);
+    if (rc != PI_OK) return rc;
+    return p->wide ? gqa_bf16<true>(p, (hipStream_t)stream) : gqa_bf16<false>(p, (hipStream_t)stream);
+}
+
+int pi_k_gqa_attn(int type, const pi_gqa_attn * p, pi_stream_t stream) {
+    if (type == PI_TYPE_F32) {
+        const int rc = gqa_check(type, p);
+        if (rc != PI_OK) return rc;
+        hipLaunchKernelGGL(gqa_attn_f32_kernel, dim3(p->T * p->n_head), dim3(256), 0, (hipStream_t)stream, *p);
+        return pi::check_launch("pi_k_gqa_attn");
+    }
+    if (type != PI_TYPE_BF16) return pi::fail(PI_E_UNSUPPORTED, "pi_k_gqa_attn: type");
+    const int rc = pi_k_gqa_attn_parts(p, stream);
+    if (rc != PI_OK || p->n_parts == 1) return rc;
+    hipLaunchKernelGGL(gqa_merge_kernel, dim3(p->n_work * p->n_kv * (gqa_rows(p->wide) / 4)), dim3(256), 0, (hipStream_t)stream, *p);
+    return pi::check_launch("pi_k_gqa_attn merge");
+}
+
+int pi_k_gqa_shift(int type, void * cache, int n_cells, int n_kv, int hd, int rot_dim, double base, const int32_t * delta, pi_stream_t stream) {
+    if (!cache || !delta || n_cells <= 0 || n_kv <= 0 || hd <= 0 || rot_dim < 0 || rot_dim % 2 || rot_dim > hd) return pi::fail(PI_E_ARG, "pi_k_gqa_shift: bad arguments");
+    if (rot_dim == 0) return PI_OK;
+    if (type == PI_TYPE_BF16) hipLaunchKernelGGL(gqa_shift_kernel<bf16>, dim3(n_cells), dim3(64), 0, (hipStream_t)stream, (bf16 *)cache, n_kv, hd, rot_dim, base, delta);
+    else if (type == PI_TYPE_F32) hipLaunchKernelGGL(gqa_shift_kernel<float>, dim3(n_cells), dim3(64), 0, (hipStream_t)stream, (float *)cache, n_kv, hd, rot_dim, base, delta);
+    else return pi::fail(PI_E_UNSUPPORTED, "pi_k_gqa_shift: type");
+    return pi::check_launch("pi_k_gqa_shift");
+}
+
+}  // extern "C"

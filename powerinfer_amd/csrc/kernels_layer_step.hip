@@ -3,6 +3,7 @@
 // expansion together with the experts' first matrices in one, and one for what closes a layer - attention output and the experts' second
 // matrices as a single long dot product per row, plus the residual.
 #include "layer_types.hpp"
+#include "mixers.hpp"
 #include "route.hpp"
 
 namespace {
@@ -218,9 +219,9 @@ __device__ int step_experts(StepExperts & s, int * first, const int32_t * __rest
 
 // ---------------------------------------------------------------------------------------------------------------------------------
 // first matrices of the step's experts: workgroup (row tile, pair) works for the pair's expert if no earlier pair has the same one, for
-// every token that chose it; act[pair] = weight * relu(z)^2
+// every token that chose it; act[pair] = weight * relu(z)^2, or (glu: rows of gate and up in turn, ff of both together) weight * clamped GLU
 // ---------------------------------------------------------------------------------------------------------------------------------
-struct ExpertUp { const bf16 * up; int ff, cols; const bf16 * x_ol; const int32_t * ids; const float * weights; int T, top; bf16 * act; int ld_act; };
+struct ExpertUp { const bf16 * up; int ff, cols; const bf16 * x_ol; const int32_t * ids; const float * weights; int T, top; bf16 * act; int ld_act; int glu = 0; float limit = 0.0f, gain = 0.0f; };
 constexpr int kUpLds = 4 * 16 * kWsStride;
 __device__ void expert_up(const ExpertUp & a, int tile, int p, unsigned char * smem) {
     constexpr int NW = 4;
@@ -256,6 +257,16 @@ __device__ void expert_up(const ExpertUp & a, int tile, int p, unsigned char * s
     if (tid >= 256) return;
     const int rr = tid >> 4, t = tid & 15, row = row0 + rr;
     if (row >= ff || t >= T) return;
+    if (a.glu) {
+        if (rr & 1) return;
+        float g = 0.0f, u = 0.0f;
+#pragma unroll
+        for (int w = 0; w < NW; ++w) { g += reinterpret_cast<float (*)[17]>(tiles[w])[rr][t]; u += reinterpret_cast<float (*)[17]>(tiles[w])[rr + 1][t]; }
+        const float y = clamped_glu(g, u, a.limit, a.gain);
+        for (int k = 0; k < top; ++k)
+            if (ids[t * top + k] == e) a.act[(size_t)(t * top + k) * a.ld_act + row / 2] = (bf16)(a.weights[t * top + k] * y);
+        return;
+    }
     float v = 0.0f;
 #pragma unroll
     for (int w = 0; w < NW; ++w) v += reinterpret_cast<float (*)[17]>(tiles[w])[rr][t];
@@ -271,6 +282,21 @@ __global__ __launch_bounds__(256) void value_and_up_kernel(pi_latent_attn p, con
     const int b = blockIdx.x;
     if (b < n_value) latent_value(p, uv, vdim, att, ld_att, b / n_rt, b % n_rt, smem);
     else expert_up(u, (b - n_value) % n_up_tiles, (b - n_value) / n_up_tiles, smem);
+}
+
+// the merge of a split grouped-query attention (four rows a workgroup) or the gated norm of a linear attention (a token a workgroup) beside
+// the experts' first matrices
+__global__ __launch_bounds__(256) void mix_and_up_kernel(pi_gqa_attn p, pi_gate_norm gn, int n_merge, int n_gate, ExpertUp u, int n_up_tiles) {
+    extern __shared__ __align__(16) unsigned char smem[];
+    int b = blockIdx.x;
+    if (b < n_gate) { gate_norm_token<bf16>(gn, b, reinterpret_cast<double *>(smem)); return; }
+    b -= n_gate;
+    if (b < n_merge) {
+        const int r4 = gqa_rows(p.wide) / 4;
+        gqa_merge_row(p, b / r4 / p.n_kv, b / r4 % p.n_kv, (b % r4) * 4 + (threadIdx.x >> 6));
+        return;
+    }
+    expert_up(u, (b - n_merge) % n_up_tiles, (b - n_merge) / n_up_tiles, smem);
 }
 
 // ---------------------------------------------------------------------------------------------------------------------------------
@@ -370,6 +396,23 @@ int pi_k_value_up_step(const pi_latent_attn * p, const void * uv, int vdim, void
     hipLaunchKernelGGL(value_and_up_kernel, dim3(n_value + n_up), dim3(256), lds, (hipStream_t)stream, *p, (const uint16_t *)uv, vdim, (bf16 *)att, ld_att, n_rt, n_value,
                        ExpertUp{(const bf16 *)up, ff, cols, (const bf16 *)x_ol, ids, weights, p->T, top, (bf16 *)act, ld_act}, n_up_tiles);
     return pi::check_launch("pi_k_value_up_step");
+}
+
+int pi_k_mix_up_step(const pi_gqa_attn * attn, const pi_gate_norm * gate, const void * up, int n_expert, int ff, int cols, float limit, float gain, const void * x_ol, int T,
+                     const int32_t * ids, const float * weights, int top, void * act, int ld_act, pi_stream_t stream) {
+    const pi_gqa_attn p = attn ? *attn : pi_gqa_attn{};
+    const pi_gate_norm g = gate ? *gate : pi_gate_norm{};
+    if (T <= 0 || T > kBtMaxT || (attn && (!p.att || !p.scratch || !p.work || p.n_parts <= 1 || p.n_parts > 64 || p.n_work <= 0 || p.n_kv <= 0 || p.n_head % p.n_kv || p.vdim <= 0 || p.hd < p.vdim)) ||
+        (gate && (!gate_norm_ok(g) || g.T != T)))
+        return pi::fail(PI_E_ARG, "pi_k_mix_up_step: bad arguments");
+    if (ids && (!up || !x_ol || !weights || !act || n_expert <= 0 || ff <= 0 || cols <= 0 || cols % 32 || top <= 0 || T * top > kStepPairs || ld_act < ff))
+        return pi::fail(PI_E_ARG, "pi_k_mix_up_step: bad expert arguments");
+    const int n_merge = attn ? p.n_work * p.n_kv * (gqa_rows(p.wide) / 4) : 0, n_gate = gate ? g.T : 0, n_up_tiles = ids ? (2 * ff + 15) / 16 : 1, n_up = ids ? n_up_tiles * T * top : 0;
+    if (n_merge + n_gate + n_up == 0) return PI_OK;
+    ExpertUp u{(const bf16 *)up, 2 * ff, cols, (const bf16 *)x_ol, ids, weights, T, top, (bf16 *)act, ld_act};
+    u.glu = 1; u.limit = limit; u.gain = gain;
+    hipLaunchKernelGGL(mix_and_up_kernel, dim3(n_merge + n_gate + n_up), dim3(256), ids ? kUpLds : 256, (hipStream_t)stream, p, g, n_merge, n_gate, u, n_up_tiles);
+    return pi::check_launch("pi_k_mix_up_step");
 }
 
 int pi_k_layer_out_step(const pi_layer_out * a, pi_stream_t stream) {

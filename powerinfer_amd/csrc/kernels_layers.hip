@@ -3,6 +3,7 @@
 // Templated on the storage of activations: bf16 (matrix cores on bf16 operands, fp32 accumulation) or fp32.
 #include "gemm_tile.hpp"
 #include "layer_types.hpp"
+#include "mixers.hpp"
 #include "route.hpp"
 
 namespace {
@@ -81,6 +82,78 @@ __global__ __launch_bounds__(1024) void norm_pair_kernel(const float * __restric
     }
 }
 
+__global__ __launch_bounds__(256) void embed_bigram_kernel(const uint16_t * __restrict__ table, int cols, const int32_t * __restrict__ tokens, int32_t * prev, float scale,
+                                                           const uint16_t * __restrict__ bigram, int buckets, long long mul_prev, long long mul_cur, int carry,
+                                                           float * __restrict__ x, float * __restrict__ x0) {
+    const int t = blockIdx.x, tok = tokens[t], before = prev[t];
+    const uint16_t * a = table + (size_t)tok * cols, * b = nullptr;
+    if (bigram) b = bigram + (size_t)(before < 0 ? buckets : (int)(((long long)before * mul_prev + (long long)tok * mul_cur) % buckets)) * cols;
+    for (int i = threadIdx.x; i < cols; i += 256) {
+        const float v = bf16_to_f32(a[i]) * scale + (b ? bf16_to_f32(b[i]) : 0.0f);
+        x[(size_t)t * cols + i] = v;
+        if (x0) x0[(size_t)t * cols + i] = v;
+    }
+    if (carry) {
+        __syncthreads();                               // every thread has read prev[t]
+        if (threadIdx.x == 0) prev[t] = tok;
+    }
+}
+
+// layer norm, two passes over the row (held in registers where it fits); x0, step: added to the residual stream first
+template <typename ST>
+__global__ __launch_bounds__(1024) void layer_norm_kernel(float * __restrict__ x, const int32_t * __restrict__ rows, int cols, float eps, const float * __restrict__ w,
+                                                         const float * __restrict__ x0, const float * __restrict__ step, ST * __restrict__ out, int ld, int ol) {
+    __shared__ double red[16];
+    const size_t base = (size_t)(rows ? rows[blockIdx.x] : blockIdx.x) * cols;
+    float * xt = x + base;
+    auto at = [&](int i) -> size_t { return ol ? pi_ol_index(blockIdx.x, i) : (size_t)blockIdx.x * ld + i; };
+    const bool adds = x0 || step;
+    if (cols <= 4 * (int)blockDim.x) {
+        float xv[4], wv[4];
+        double s = 0.0;
+#pragma unroll
+        for (int k = 0; k < 4; ++k) {
+            const int i = threadIdx.x + k * blockDim.x;
+            xv[k] = i < cols ? xt[i] : 0.0f;
+            wv[k] = i < cols ? w[i] : 0.0f;
+            if (x0 && i < cols) xv[k] += x0[base + i];
+            if (step && i < cols) xv[k] += step[i];
+            s += (double)xv[k];
+        }
+        const float mean = (float)(block_sum_f64(s, red) / cols);
+        s = 0.0;
+#pragma unroll
+        for (int k = 0; k < 4; ++k) {
+            const int i = threadIdx.x + k * blockDim.x;
+            if (i < cols) {
+                if (adds) xt[i] = xv[k];
+                xv[k] -= mean;
+                s += (double)xv[k] * (double)xv[k];
+            }
+        }
+        const float sc = pi_inv_sqrt((float)(block_sum_f64(s, red) / cols) + eps);
+#pragma unroll
+        for (int k = 0; k < 4; ++k) {
+            const int i = threadIdx.x + k * blockDim.x;
+            if (i < cols) out[at(i)] = to_st<ST>(xv[k] * sc * wv[k]);
+        }
+        return;
+    }
+    double s = 0.0;
+    for (int i = threadIdx.x; i < cols; i += blockDim.x) {
+        float v = xt[i];
+        if (x0) v += x0[base + i];
+        if (step) v += step[i];
+        if (adds) xt[i] = v;                           // (read back below by the thread that wrote it)
+        s += (double)v;
+    }
+    const float mean = (float)(block_sum_f64(s, red) / cols);
+    s = 0.0;
+    for (int i = threadIdx.x; i < cols; i += blockDim.x) { const float v = xt[i] - mean; s += (double)v * (double)v; }
+    const float sc = pi_inv_sqrt((float)(block_sum_f64(s, red) / cols) + eps);
+    for (int i = threadIdx.x; i < cols; i += blockDim.x) out[at(i)] = to_st<ST>((xt[i] - mean) * sc * w[i]);
+}
+
 // ---------------------------------------------------------------------------------------------------------------------------------
 // grouped mat-mul.  A workgroup of four waves owns 64 rows of one group's matrix x 32 of the group's tokens; each wave holds 16 rows in
 // the matrix cores' operand layout (lane l: row l % 16, eight consecutive columns 8 * (l / 16) of a 32-column step) against two token
@@ -116,6 +189,17 @@ __global__ __launch_bounds__(256) void group_gemm_kernel(pi_group_gemm g) {
         const int t = t0 + u * 16 + i;
         if (t >= n) continue;
         const size_t yr = g.off ? (size_t)(lo + t) * g.ldy : (size_t)grp * g.y_gs + (size_t)t * g.ldy;
+        if (g.glu) {                                   // rows in (gate, up) pairs: a lane holds two of them
+#pragma unroll
+            for (int r = 0; r < 4; r += 2) {
+                const int row = row0 + 4 * q + r;
+                if (row >= g.rows) continue;
+                const float v = clamped_glu(acc[u][r] * g.alpha, acc[u][r + 1] * g.alpha, g.glu_limit, g.glu_gain);
+                if (g.y_f32) ((float *)g.y)[yr + row / 2] = v;
+                else ((ST *)g.y)[yr + row / 2] = to_st<ST>(v);
+            }
+            continue;
+        }
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
             const int row = row0 + 4 * q + r;
@@ -224,6 +308,23 @@ __global__ __launch_bounds__(64 * WGM * WGN, (WGM * WGN > 4 ? 1 : BM + BN <= 192
         for (int nn = 0; nn < NT; ++nn) {
             const int row = row0 + wm * WM + m * 16 + 4 * q, tok = wn * WN + nn * 16 + i;
             if (tok >= n || row >= g.rows) continue;
+            if (g.glu) {                               // rows in (gate, up) pairs: a lane holds two of them
+                const size_t o = (g.off ? 0 : (size_t)grp * g.y_gs) + (size_t)(lo + tok) * g.ldy + row / 2;
+                const float a = clamped_glu(acc[m][nn][0] * g.alpha, acc[m][nn][1] * g.alpha, g.glu_limit, g.glu_gain);
+                const float b = clamped_glu(acc[m][nn][2] * g.alpha, acc[m][nn][3] * g.alpha, g.glu_limit, g.glu_gain);
+                const bool two = row + 4 <= g.rows;
+                if (g.y_f32) {
+                    ((float *)g.y)[o] = a;
+                    if (two) ((float *)g.y)[o + 1] = b;
+                } else if (two && (o & 1) == 0) {
+                    const bf16 v[2] = {(bf16)a, (bf16)b};
+                    *reinterpret_cast<uint32_t *>((bf16 *)g.y + o) = __builtin_bit_cast(uint32_t, v);
+                } else {
+                    ((bf16 *)g.y)[o] = (bf16)a;
+                    if (two) ((bf16 *)g.y)[o + 1] = (bf16)b;
+                }
+                continue;
+            }
             const size_t o = (g.off ? 0 : (size_t)grp * g.y_gs) + (size_t)(lo + tok) * g.ldy + row;
             float v[4];
 #pragma unroll
@@ -297,6 +398,12 @@ __global__ void pad_cols_kernel(const uint16_t * __restrict__ in, int64_t rows, 
         out[i] = c < cols ? in[r * cols + c] : (uint16_t)0;
     }
 }
+__global__ void place_kernel(const uint16_t * __restrict__ in, int64_t rows, int cols, uint16_t * __restrict__ out, int ld, int col0, int width, int64_t row0, int row_step) {
+    for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < rows * width; i += (int64_t)gridDim.x * blockDim.x) {
+        const int64_t r = i / width; const int c = (int)(i % width);
+        out[(size_t)(row0 + r * row_step) * ld + col0 + c] = c < cols ? in[r * cols + c] : (uint16_t)0;
+    }
+}
 __global__ void transpose_pad_kernel(const uint16_t * __restrict__ in, int n_mat, int rows, int cols, uint16_t * __restrict__ out, int ld) {
     const int64_t n = (int64_t)n_mat * cols * ld;
     for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (int64_t)gridDim.x * blockDim.x) {
@@ -327,6 +434,25 @@ int pi_k_embed_norm(const void * table, int cols, const int32_t * tokens, int T,
     return pi::check_launch("pi_k_embed_norm");
 }
 
+int pi_k_embed_bigram(const void * table, int cols, const int32_t * tokens, int32_t * prev, int T, float scale, const void * bigram, int32_t buckets, int64_t mul_prev,
+                      int64_t mul_cur, int carry, float * x, float * x0, pi_stream_t stream) {
+    if (!table || !tokens || !prev || !x || cols <= 0 || T <= 0 || (bigram && buckets <= 0)) return pi::fail(PI_E_ARG, "pi_k_embed_bigram: bad arguments");
+    hipLaunchKernelGGL(embed_bigram_kernel, dim3(T), dim3(256), 0, (hipStream_t)stream, (const uint16_t *)table, cols, tokens, prev, scale, (const uint16_t *)bigram, buckets,
+                       (long long)mul_prev, (long long)mul_cur, carry, x, x0);
+    return pi::check_launch("pi_k_embed_bigram");
+}
+
+int pi_k_layer_norm(int type, float * x, const int32_t * rows, int T, int cols, float eps, const float * w, const float * x0, const float * step, void * out, int ld, int ol,
+                    pi_stream_t stream) {
+    if (!x || !w || !out || T <= 0 || cols <= 0 || ld < cols || (rows && (x0 || step))) return pi::fail(PI_E_ARG, "pi_k_layer_norm: bad arguments");
+    if (ol && (type != PI_TYPE_BF16 || T > kBtMaxT || ld % 8)) return pi::fail(PI_E_ARG, "pi_k_layer_norm: operand layout needs BF16, T <= 16, ld % 8 == 0");
+    const int block = cols > 2048 ? 1024 : cols > 512 ? 512 : 256;
+    if (type == PI_TYPE_BF16) hipLaunchKernelGGL(layer_norm_kernel<bf16>, dim3(T), dim3(block), 0, (hipStream_t)stream, x, rows, cols, eps, w, x0, step, (bf16 *)out, ld, ol);
+    else if (type == PI_TYPE_F32) hipLaunchKernelGGL(layer_norm_kernel<float>, dim3(T), dim3(block), 0, (hipStream_t)stream, x, rows, cols, eps, w, x0, step, (float *)out, ld, 0);
+    else return pi::fail(PI_E_UNSUPPORTED, "pi_k_layer_norm: type");
+    return pi::check_launch("pi_k_layer_norm");
+}
+
 int pi_k_norm_pair(int type, const float * x, const int32_t * rows, int T, int cols, float eps, const float * wa, void * out_a,
                    const float * wb, void * out_b, int ld, int ol, pi_stream_t stream) {
     if (!x || !wa || !out_a || (wb && !out_b) || T <= 0 || cols <= 0 || ld < cols) return pi::fail(PI_E_ARG, "pi_k_norm_pair: bad arguments");
@@ -342,7 +468,7 @@ int pi_k_norm_pair(int type, const float * x, const int32_t * rows, int T, int c
 
 int pi_k_group_gemm(int type, const pi_group_gemm * g, pi_stream_t stream) {
     if (!g || !g->W || !g->x || !g->y || g->rows <= 0 || g->cols <= 0 || g->cols % 32 || g->ldw < g->cols || g->ldw % 8 || g->ldx < g->cols || g->ldx % 8 ||
-        g->ldy < g->rows || g->T <= 0 || g->n_group <= 0 || g->n_group > 65535 || (g->gather && g->gather_div <= 0) || g->w_gs % 8 || g->x_gs % 8)
+        g->ldy < (g->glu ? g->rows / 2 : g->rows) || (g->glu && (g->rows % 2 || g->relu2)) || g->T <= 0 || g->n_group <= 0 || g->n_group > 65535 || (g->gather && g->gather_div <= 0) || g->w_gs % 8 || g->x_gs % 8)
         return pi::fail(PI_E_ARG, "pi_k_group_gemm: bad arguments");
     const dim3 grid((g->rows + 63) / 64, (g->T + 31) / 32, g->n_group);
     if (grid.y > 65535) return pi::fail(PI_E_ARG, "pi_k_group_gemm: too many tokens");
@@ -375,7 +501,7 @@ int pi_k_moe_sort(const int32_t * ids, int n_pairs, int n_expert, int32_t * off,
 
 int pi_k_group_gemm_tile(const pi_group_gemm * g, int tile_n, pi_stream_t stream) {
     if (!g || !g->W || !g->x || !g->y || g->rows <= 0 || g->cols <= 0 || g->cols % kGtBK || g->ldw < g->cols || g->ldw % 8 || g->ldx < g->cols || g->ldx % 8 ||
-        g->ldy < g->rows || g->T <= 0 || g->n_group <= 0 || (g->gather && g->gather_div <= 0) || g->w_gs % 8 || g->x_gs % 8 || (g->off && (!g->tiles || !g->n_tiles || g->max_tiles <= 0)))
+        g->ldy < (g->glu ? g->rows / 2 : g->rows) || (g->glu && (g->rows % 2 || g->relu2)) || g->T <= 0 || g->n_group <= 0 || (g->gather && g->gather_div <= 0) || g->w_gs % 8 || g->x_gs % 8 || (g->off && (!g->tiles || !g->n_tiles || g->max_tiles <= 0)))
         return pi::fail(PI_E_ARG, "pi_k_group_gemm_tile: bad arguments");
     if ((((uintptr_t)g->W | (uintptr_t)g->x | (uintptr_t)g->y) & 15) != 0) return pi::fail(PI_E_ARG, "pi_k_group_gemm_tile: operands must be 16-byte aligned");
     hipStream_t st = (hipStream_t)stream;
@@ -397,6 +523,12 @@ int pi_k_pad_cols_bf16(const void * in, int64_t rows, int cols, void * out, int 
     if (!in || !out || rows <= 0 || cols <= 0 || ld < cols) return pi::fail(PI_E_ARG, "pi_k_pad_cols_bf16: bad arguments");
     hipLaunchKernelGGL(pad_cols_kernel, dim3(4096), dim3(256), 0, (hipStream_t)stream, (const uint16_t *)in, rows, cols, (uint16_t *)out, ld);
     return pi::check_launch("pi_k_pad_cols_bf16");
+}
+
+int pi_k_place_bf16(const void * in, int64_t rows, int cols, void * out, int ld, int col0, int width, int64_t row0, int row_step, pi_stream_t stream) {
+    if (!in || !out || rows <= 0 || cols <= 0 || width < cols || col0 < 0 || col0 + width > ld || row0 < 0 || row_step <= 0) return pi::fail(PI_E_ARG, "pi_k_place_bf16: bad arguments");
+    hipLaunchKernelGGL(place_kernel, dim3(4096), dim3(256), 0, (hipStream_t)stream, (const uint16_t *)in, rows, cols, (uint16_t *)out, ld, col0, width, row0, row_step);
+    return pi::check_launch("pi_k_place_bf16");
 }
 
 int pi_k_transpose_pad_bf16(const void * in, int n_mat, int rows, int cols, void * out, int ld, pi_stream_t stream) {

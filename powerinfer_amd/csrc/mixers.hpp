@@ -1,0 +1,128 @@
+// Pieces of a layer that several launches hold: the clamped GLU, what a layer with one norm computes of its feed-forward straight from the
+// joint projection, the merge of a split grouped-query attention, and the gated norm behind a linear attention.
+#pragma once
+#include "layer_types.hpp"
+#include "route.hpp"
+
+namespace {
+
+__device__ __forceinline__ float sigmoid_f32(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float silu_f32(float z) { return z * sigmoid_f32(z); }
+__device__ __forceinline__ float clamped_glu(float g, float u, float limit, float gain) {
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+    return g * sigmoid_f32(gain * g) * (u + 1.0f);
+}
+
+// four values of activation storage in one store where the place allows it
+template <typename ST> __device__ __forceinline__ void store4(ST * p, const float (&v)[4], bool whole, int n) {
+    if (whole) {
+        struct alignas(4 * sizeof(ST)) Quad { ST v[4]; } q{{to_st<ST>(v[0]), to_st<ST>(v[1]), to_st<ST>(v[2]), to_st<ST>(v[3])}};
+        *reinterpret_cast<Quad *>(p) = q;
+    } else {
+        for (int r = 0; r < 4 && r < n; ++r) p[r] = to_st<ST>(v[r]);
+    }
+}
+
+// ---- pi_ffn_front: blocks of 256 threads, front_glu_blocks of them and one more for the choice of experts per token -----------------
+constexpr int kFrontGlu = 1024;           // values of a workgroup
+__host__ __device__ inline int front_glu_blocks(const pi_ffn_front & f) { return f.ff > 0 ? (f.ff_ld + kFrontGlu - 1) / kFrontGlu : 0; }
+__host__ __device__ inline int front_blocks(const pi_ffn_front & f) { return front_glu_blocks(f) + (f.n_expert > 0 ? 1 : 0); }
+inline size_t front_lds_bytes(const pi_ffn_front & f) { return f.n_expert > 0 ? route_lds_bytes(f.n_expert, 1, f.n_top) : 0; }
+inline bool front_ok(const pi_ffn_front & f, int ldz) {
+    if (f.ff > 0 && (!f.act || f.off_glu < 0 || f.off_glu + 2 * f.ff > ldz || f.off_score >= ldz || f.ff_ld < f.ff || f.ff_ld % 4 || f.ld_act < f.ff_ld)) return false;
+    return f.n_expert <= 0 || (f.ids && f.weights && f.off_router >= 0 && f.off_router + f.n_expert <= ldz && f.n_expert <= 4096 && f.n_top > 0 && f.n_top <= f.n_expert);
+}
+template <typename ST> __device__ void front_block(const pi_ffn_front & f, const float * __restrict__ z, int ldz, int t, int b, float * sm) {
+    const float * row = z + (size_t)t * ldz;
+    if (b == front_glu_blocks(f)) {
+        route_token(RouteArgs{z + f.off_router, f.n_expert, f.n_top, 1, 1, nullptr, f.ids, f.weights, ldz, true}, t, sm);
+        return;
+    }
+    const int j0 = b * kFrontGlu + threadIdx.x * 4;
+    if (j0 >= f.ff_ld) return;
+    const float * g = row + f.off_glu + 2 * j0;
+    float v[4], w[8];
+    if (j0 + 4 <= f.ff && ((f.off_glu | ldz) & 3) == 0) {
+        const float4 a = reinterpret_cast<const float4 *>(g)[0], c = reinterpret_cast<const float4 *>(g)[1];
+        w[0] = a.x; w[1] = a.y; w[2] = a.z; w[3] = a.w; w[4] = c.x; w[5] = c.y; w[6] = c.z; w[7] = c.w;
+    } else {
+#pragma unroll
+        for (int k = 0; k < 8; ++k) w[k] = j0 + k / 2 < f.ff ? g[k] : 0.0f;
+    }
+    const float s = f.off_score >= 0 ? sigmoid_f32(row[f.off_score]) : 1.0f;
+#pragma unroll
+    for (int k = 0; k < 4; ++k) v[k] = j0 + k < f.ff ? s * clamped_glu(w[2 * k], w[2 * k + 1], f.limit, f.gain) : 0.0f;
+    ST * o = (ST *)f.act + (size_t)t * f.ld_act + j0;
+    store4(o, v, ((uintptr_t)o & (4 * sizeof(ST) - 1)) == 0, 4);
+}
+
+// ---- grouped-query attention: the parts of one row of a work item, by one wave (fixed order, the sink in the denominator) -------------
+__host__ __device__ inline int gqa_rows(int wide) { return wide ? 128 : 16; }
+__device__ void gqa_merge_row(const pi_gqa_attn & p, int item_index, int g, int r) {
+    const int lane = threadIdx.x & 63, per = p.n_head / p.n_kv, R = gqa_rows(p.wide);
+    const int4 item = reinterpret_cast<const int4 *>(p.work)[item_index];
+    if (r >= item.z) return;
+    const size_t srow = ((size_t)item_index * p.n_kv + g) * R + r;
+    const float * acc = p.scratch + srow * p.n_parts * p.hd;
+    const float2 ml = lane < p.n_parts ? reinterpret_cast<const float2 *>(p.scratch + (size_t)p.n_work * p.n_kv * R * p.n_parts * p.hd)[srow * p.n_parts + lane]
+                                       : make_float2(-INFINITY, 0.0f);
+    const float m = fmaxf(pi_wave_max(ml.x), p.sink);
+    const float e = ml.x == -INFINITY ? 0.0f : expf(ml.x - m);
+    const float l = pi_wave_sum(e * ml.y) + expf(p.sink - m);
+    const float f = e / l;
+    const int rr = item.y + r, head = g * per + rr % per;
+    bf16 * out = (bf16 *)p.att + (size_t)(item.x + rr / per) * p.ld_att + head * p.vdim;
+    for (int c0 = 0; c0 < p.vdim; c0 += 64) {            // (every lane stays in the loop: the factors are passed between lanes)
+        const int c = min(c0 + lane, p.hd - 1);
+        float v = 0.0f;
+        for (int s0 = 0; s0 < p.n_parts; s0 += 8) {
+            float a[8];
+#pragma unroll
+            for (int u = 0; u < 8; ++u) a[u] = acc[(size_t)min(s0 + u, p.n_parts - 1) * p.hd + c];
+#pragma unroll
+            for (int u = 0; u < 8; ++u) {
+                const float w = __shfl(f, min(s0 + u, PI_WAVE - 1), PI_WAVE);
+                if (s0 + u < p.n_parts) v = fmaf(w, a[u], v);
+            }
+        }
+        if (c0 + lane < p.vdim) out[c0 + lane] = (bf16)v;
+    }
+}
+
+// ---- gated norm of one token by one workgroup ------------------------------------------------------------------------------------------
+template <typename ST> __device__ void gate_norm_token(const pi_gate_norm & p, int t, double * red) {
+    const float * o = p.o + (size_t)t * p.n, * g = p.z + (size_t)t * p.ldz + p.off_gate;
+    ST * out = (ST *)p.att + (size_t)t * p.ld_att;
+    constexpr int K = 16;
+    const int nt = blockDim.x;
+    if (p.n <= K * nt) {                              // one memory round trip: everything requested together, kept in registers
+        float v[K], gv[K], wv[K];
+        double s = 0.0;
+#pragma unroll
+        for (int k = 0; k < K; ++k) {
+            const int i = min((int)threadIdx.x + k * nt, p.n - 1);
+            v[k] = o[i]; gv[k] = g[i]; wv[k] = p.w[i];
+        }
+#pragma unroll
+        for (int k = 0; k < K; ++k) if ((int)threadIdx.x + k * nt < p.n) s += (double)v[k] * (double)v[k];
+        s = block_sum_f64(s, red);
+        const float sc = pi_inv_sqrt((float)(s / p.n) + p.eps);
+#pragma unroll
+        for (int k = 0; k < K; ++k) {
+            const int i = threadIdx.x + k * nt;
+            if (i < p.n) out[i] = to_st<ST>(v[k] * sc * wv[k] * sigmoid_f32(gv[k]));
+        }
+        return;
+    }
+    double s = 0.0;
+    for (int i = threadIdx.x; i < p.n; i += nt) s += (double)o[i] * (double)o[i];
+    s = block_sum_f64(s, red);
+    const float sc = pi_inv_sqrt((float)(s / p.n) + p.eps);
+    for (int i = threadIdx.x; i < p.n; i += nt) out[i] = to_st<ST>(o[i] * sc * p.w[i] * sigmoid_f32(g[i]));
+}
+inline bool gate_norm_ok(const pi_gate_norm & p) {
+    return p.o && p.z && p.w && p.att && p.n > 0 && p.T > 0 && p.off_gate >= 0 && p.off_gate + p.n <= p.ldz && p.ld_att >= p.n;
+}
+
+}  // namespace

@@ -4,7 +4,9 @@
 
 namespace {
 
-struct RouteArgs { const float * z; int E, top, G, keep; const float * bias; int32_t * ids; float * weights; };
+// soft: the experts with the largest logits, their weights the soft-max over them; else sigmoid scores, a bias on the choice and groups.
+// ldz: values between the tokens' rows of z (0: E)
+struct RouteArgs { const float * z; int E, top, G, keep; const float * bias; int32_t * ids; float * weights; int ldz = 0; bool soft = false; };
 
 __host__ __device__ inline size_t route_lds_bytes(int E, int G, int top) { return sizeof(float) * (size_t)(2 * ((E + 3) / 4 * 4) + (G > top ? G : top)); }
 
@@ -13,11 +15,12 @@ __host__ __device__ inline size_t route_lds_bytes(int E, int G, int top) { retur
 __device__ void route_token(const RouteArgs & r, int t, float * sm) {
     const int E = r.E, E4 = (E + 3) / 4 * 4, G = r.G, tid = threadIdx.x, nt = blockDim.x, size = E / G;
     float * sc = sm, * ch = sm + E4, * gs = sm + 2 * E4;
+    const float * z = r.z + (size_t)t * (r.ldz ? r.ldz : E);
     for (int e = tid; e < E4; e += nt) {
         float s = 0.0f, c = -INFINITY;
         if (e < E) {
-            s = 1.0f / (1.0f + expf(-r.z[(size_t)t * E + e]));
-            c = s + r.bias[e];
+            s = r.soft ? z[e] : 1.0f / (1.0f + expf(-z[e]));
+            c = r.soft ? s : s + r.bias[e];
             if (!(c == c)) c = -INFINITY;                      // not a number: never chosen over a number
         }
         sc[e] = s;
@@ -62,6 +65,12 @@ __device__ void route_token(const RouteArgs & r, int t, float * sm) {
     }
     __syncthreads();
     float total = 0.0f;
+    if (r.soft) {
+        const float m = gs[0];                                 // rank 0 holds the largest
+        for (int k = 0; k < r.top; ++k) total += expf(gs[k] - m);
+        for (int k = tid; k < r.top; k += nt) r.weights[(size_t)t * r.top + k] = expf(gs[k] - m) / total;
+        return;
+    }
     for (int k = 0; k < r.top; ++k) total += gs[k];
     for (int k = tid; k < r.top; k += nt) r.weights[(size_t)t * r.top + k] = gs[k] / (total + 1e-20f);
 }

@@ -12,7 +12,8 @@ HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(HERE, "libpowerinfer_hip.so")
 
 F32, F16, Q4_0, I32, BF16 = 0, 1, 2, 18, 30
-MIXER_LATENT, FFN_NONE, FFN_MOE = 0, 0, 1
+MIXER_LATENT, MIXER_GROUPED, MIXER_LINEAR = 0, 1, 2
+FFN_NONE, FFN_MOE, FFN_GLU, FFN_GLU_MOE = 0, 1, 2, 3
 EPI_NONE, EPI_RELU, EPI_ADD, EPI_ADD2 = 0, 1, 2, 3
 NORM_NONE, NORM_RMS, NORM_LAYER = 0, 1, 2
 
@@ -28,7 +29,7 @@ class GroupGemm(C.Structure):
                 ("x", _vp), ("x_gs", _sz), ("ldx", C.c_int32), ("T", C.c_int32),
                 ("y", _vp), ("y_gs", _sz), ("ldy", C.c_int32), ("y_f32", C.c_int32), ("relu2", C.c_int32),
                 ("alpha", _f), ("off", _vp), ("gather", _vp), ("gather_div", C.c_int32),
-                ("tiles", _vp), ("n_tiles", _vp), ("max_tiles", C.c_int32)]
+                ("tiles", _vp), ("n_tiles", _vp), ("max_tiles", C.c_int32), ("glu", C.c_int32), ("glu_limit", _f), ("glu_gain", _f)]
 
 
 class LatentPrep(C.Structure):
@@ -45,6 +46,32 @@ class LatentAttn(C.Structure):
 class LatentExpanded(C.Structure):
     _fields_ = [(n, _vp) for n in ("q_un", "q_lat", "keys", "values", "cache", "list", "n_vis", "sink", "att")] + [
         (n, C.c_int32) for n in ("tok0", "T", "n_head", "dim", "dim_ld", "rot_dim", "vdim", "rank_ld", "kd", "ld_att")] + [("scale", _f)]
+
+
+class FfnFront(C.Structure):
+    _fields_ = [(n, C.c_int32) for n in ("off_glu", "ff", "ff_ld", "off_score")] + [("limit", _f), ("gain", _f), ("act", _vp)] + [
+        (n, C.c_int32) for n in ("ld_act", "off_router", "n_expert", "n_top")] + [("ids", _vp), ("weights", _vp)]
+
+
+class GqaPrep(C.Structure):
+    _fields_ = [("z", _vp)] + [(n, C.c_int32) for n in ("ldz", "T", "n_head", "n_kv", "dim", "vdim", "rot_dim", "off_k", "off_v", "hd", "unit")] + [
+        ("cs", _vp), ("eps", _f), ("q", _vp), ("cache", _vp), ("cell", _vp)]
+
+
+class GqaAttn(C.Structure):
+    _fields_ = [("q", _vp), ("cache", _vp), ("lists", _vp), ("list_ld", _sz), ("work", _vp), ("n_vis", _vp)] + [
+        (n, C.c_int32) for n in ("n_work", "T", "n_head", "n_kv", "dim", "vdim", "hd", "n_parts", "wide")] + [
+        ("scale", _f), ("sink", _f), ("scratch", _vp), ("att", _vp), ("ld_att", C.c_int32)]
+
+
+class Linear(C.Structure):
+    _fields_ = [("z", _vp)] + [(n, C.c_int32) for n in ("ldz", "T", "n_head", "dim", "vdim", "off_k", "off_v")] + [
+        ("decay", _vp), ("powers", _vp), ("state", _vp), ("runs", _vp), ("n_runs", C.c_int32), ("o", _vp), ("q", _vp), ("k", _vp), ("v", _vp), ("states", _vp)] + [
+        (n, C.c_int32) for n in ("dim_ld", "vdim_ld", "n_chunks")] + [("chunks", _vp), ("first_chunk", _vp)]
+
+
+class GateNorm(C.Structure):
+    _fields_ = [("o", _vp), ("z", _vp), ("w", _vp)] + [(n, C.c_int32) for n in ("ldz", "off_gate", "n", "T")] + [("eps", _f), ("att", _vp), ("ld_att", C.c_int32)]
 
 
 class LayerOut(C.Structure):
@@ -200,6 +227,24 @@ _SIGS = {
     "pi_k_latent_attn_parts": (_i, [C.POINTER(LatentAttn), _vp]),
     "pi_k_value_up_step": (_i, [C.POINTER(LatentAttn), _vp, _i, _vp, _i, _vp, _i, _i, _i, _vp, _vp, _vp, _i, _vp, _i, _vp]),
     "pi_k_layer_out_step": (_i, [C.POINTER(LayerOut), _vp]),
+    "pi_k_embed_bigram": (_i, [_vp, _i, _vp, _vp, _i, _f, _vp, C.c_int32, C.c_int64, C.c_int64, _i, _vp, _vp, _vp]),
+    "pi_k_layer_norm": (_i, [_i, _vp, _vp, _i, _i, _f, _vp, _vp, _vp, _vp, _i, _i, _vp]),
+    "pi_k_gqa_head_ld": (_i, [_i, _i, _i]),
+    "pi_k_gqa_prep": (_i, [_i, C.POINTER(GqaPrep), C.POINTER(FfnFront), _vp]),
+    "pi_k_gqa_rows": (_i, [_i]),
+    "pi_k_gqa_scratch_floats": (_sz, [_i, _i, _i, _i, _i]),
+    "pi_k_gqa_attn": (_i, [_i, C.POINTER(GqaAttn), _vp]),
+    "pi_k_gqa_attn_parts": (_i, [C.POINTER(GqaAttn), _vp]),
+    "pi_k_gqa_shift": (_i, [_i, _vp, _i, _i, _i, _i, C.c_double, _vp, _vp]),
+    "pi_k_linear_chunk": (_i, []),
+    "pi_k_linear_supported": (_i, [_i, _i]),
+    "pi_k_linear_states_bytes": (_sz, [_i, _i, _i, _i]),
+    "pi_k_linear_step": (_i, [_i, C.POINTER(Linear), C.POINTER(FfnFront), _vp]),
+    "pi_k_linear_prep": (_i, [_i, C.POINTER(Linear), C.POINTER(FfnFront), _vp]),
+    "pi_k_linear_chunks": (_i, [C.POINTER(Linear), _vp]),
+    "pi_k_gate_norm": (_i, [_i, C.POINTER(GateNorm), _vp]),
+    "pi_k_mix_up_step": (_i, [C.POINTER(GqaAttn), C.POINTER(GateNorm), _vp, _i, _i, _i, _f, _f, _vp, _i, _vp, _vp, _i, _vp, _i, _vp]),
+    "pi_k_place_bf16": (_i, [_vp, C.c_int64, _i, _vp, _i, _i, _i, C.c_int64, _i, _vp]),
     "pi_k_pad_cols_bf16": (_i, [_vp, C.c_int64, _i, _vp, _i, _vp]),
     "pi_k_transpose_pad_bf16": (_i, [_vp, _i, _i, _i, _vp, _i, _vp]),
     "pi_k_cells_advance": (_i, [_i, _vp, _vp, _sz, _vp, _vp, _vp, _vp]),

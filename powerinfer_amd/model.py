@@ -7,7 +7,7 @@ import numpy as np
 from . import lib as pl
 from .lib import check
 
-ARCH = {"llama": 0, "falcon": 1, "lerasun": 2}
+ARCH = {"llama": 0, "falcon": 1, "lerasun": 2, "pibalorn": 3}
 
 # tensor roles, same order as the enum in include/powerinfer_hip.h
 KINDS = ["tok_embd", "output_norm", "output_norm_b", "output",
@@ -16,7 +16,9 @@ KINDS = ["tok_embd", "output_norm", "output_norm_b", "output",
          "ffn_norm", "ffn_gate", "ffn_up", "ffn_down_t",
          "fc1", "fc2", "gpu_idx", "gpu_bucket", "neuron_rate",
          "embd_norm", "mix_q", "mix_dkv", "mix_dkv_norm", "mix_uk", "mix_uv", "mix_sink",
-         "router", "router_bias", "expert_up", "expert_down"]
+         "router", "router_bias", "expert_up", "expert_down",
+         "bigram", "loop_step", "mix_k", "mix_v", "mix_g", "mix_norm", "mix_decay",
+         "expert_gate", "glu_gate", "glu_up", "glu_down", "shared_score"]
 KIND = {k: i for i, k in enumerate(KINDS)}
 
 
@@ -29,11 +31,14 @@ class HParamsC(C.Structure):
 class LayerDescC(C.Structure):
     _fields_ = [(n, C.c_int32) for n in ("mixer", "n_head", "dim", "rot_dim", "vdim", "kv_rank", "kv_from")] + [
         ("scale", C.c_float), ("rot_base", C.c_double)] + [
-        (n, C.c_int32) for n in ("ffn", "n_expert", "n_top", "n_group", "n_group_keep", "expert_ff")]
+        (n, C.c_int32) for n in ("ffn", "n_expert", "n_top", "n_group", "n_group_keep", "expert_ff", "n_kv_head", "values_are_keys", "unit_qk")] + [
+        ("sink", C.c_float), ("glu_ff", C.c_int32), ("glu_limit", C.c_float), ("expert_limit", C.c_float), ("glu_gain", C.c_float)]
 
 
 class LayersOptsC(C.Structure):
-    _fields_ = [("compute", C.c_int32), ("logit_scale", C.c_float), ("norm_offset", C.c_float), ("max_batch", C.c_int32)]
+    _fields_ = [("compute", C.c_int32), ("logit_scale", C.c_float), ("norm_offset", C.c_float), ("max_batch", C.c_int32),
+                ("embed_scale", C.c_float), ("bigram_buckets", C.c_int32), ("bigram_mul_prev", C.c_int64), ("bigram_mul_cur", C.c_int64),
+                ("loop_start", C.c_int32), ("loop_stop", C.c_int32), ("loop_times", C.c_int32), ("n_slots", C.c_int32)]
 
 
 def _declare(L):
@@ -336,14 +341,17 @@ class Model:
 class LayerModel(Model):
     """A model described layer by layer (pi_model_create_layers); every entry point of Model that is not about sparse FFN rows works on it."""
 
-    def __init__(self, arch, descs, n_embd, n_vocab, n_ctx, norm_eps, compute=pl.BF16, logit_scale=1.0, norm_offset=0.0, max_batch=0):
+    def __init__(self, arch, descs, n_embd, n_vocab, n_ctx, norm_eps, compute=pl.BF16, logit_scale=1.0, norm_offset=0.0, max_batch=0, **opts):
+        """opts: further fields of pi_layers_opts (embedding, bigram table, loop)."""
         from .synth import HParams
         self.L = pl.init()
         _declare(self.L)
         self.hp = HParams(arch=arch, n_embd=n_embd, n_layer=len(descs), n_vocab=n_vocab, n_ctx=n_ctx, norm_eps=norm_eps)
         self.descs = descs
         c = HParamsC(arch=ARCH[arch], n_embd=n_embd, n_layer=len(descs), n_vocab=n_vocab, n_ctx=n_ctx, norm_eps=norm_eps)
-        o = LayersOptsC(compute, logit_scale, norm_offset, max_batch)
+        o = LayersOptsC(compute=compute, logit_scale=logit_scale, norm_offset=norm_offset, max_batch=max_batch, **opts)
+        looped = (opts.get("loop_stop", 0) - opts.get("loop_start", 0)) if opts.get("loop_times", 0) else 0
+        self.n_runs = len(descs) + looped * (opts.get("loop_times", 0) - 1)       # layers of a step, those of the loop once per pass
         arr = (LayerDescC * len(descs))(*[LayerDescC(**d) for d in descs])
         self.h = self.L.pi_model_create_layers(C.byref(c), C.byref(o), arr, len(descs))
         if not self.h:
@@ -355,10 +363,10 @@ class LayerModel(Model):
         self._keep = []
 
     def get_streams(self):
-        """The residual stream behind every layer for the last pass of a step, [n_layer][n_tokens][n_embd] (capture enabled)."""
+        """The residual stream behind every layer run for the last pass of a step, [n_runs][n_tokens][n_embd] (capture enabled)."""
         n = self.L.pi_model_get_streams(self.h, None)
         if n < 0:
             check(n, "pi_model_get_streams")
-        out = np.empty((self.hp.n_layer, n, self.hp.n_embd), np.float32)
+        out = np.empty((self.n_runs, n, self.hp.n_embd), np.float32)
         check(min(self.L.pi_model_get_streams(self.h, out.ctypes.data_as(C.c_void_p)), 0), "pi_model_get_streams")
         return out

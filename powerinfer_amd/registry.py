@@ -15,7 +15,12 @@ def _lerasun(config, tensors, **kw):
     return lerasun.build(config, tensors, **kw)
 
 
-FOLDERS = {"Lerasun": _lerasun}
+def _pibalorn(config, tensors, **kw):
+    from . import pibalorn
+    return pibalorn.build(config, tensors, **kw)
+
+
+FOLDERS = {"Lerasun": _lerasun, "Pibalorn": _pibalorn}
 
 
 def load_model(path, dtype="bfloat16", n_ctx=4096, max_batch=0):
