@@ -352,6 +352,70 @@ def build_lerasun_on_device(width, sh, n_ctx, keep):
     return m
 
 
+# shapes of --design pibalorn: six layers of which two run twice (eight layer runs), attention and linear attention in turn, beside Lerasun of
+# equal width, depth and experts
+PIBALORN_SHAPES = {
+    2048: dict(heads=16, kv_heads=4, dim=128, lin_heads=16, lin_dim=128, dense_ff=5632, experts=64, top=6, ff=1408, shared_ff=2816, beside=2048),
+    4096: dict(heads=32, kv_heads=8, dim=128, lin_heads=32, lin_dim=128, dense_ff=11008, experts=64, top=6, ff=1408, shared_ff=2816, beside=4096),
+    5120: dict(heads=40, kv_heads=8, dim=128, lin_heads=40, lin_dim=128, dense_ff=13824, experts=160, top=6, ff=1536, shared_ff=3072, beside=5120),
+}
+
+
+def build_pibalorn_on_device(width, sh, n_ctx, keep):
+    """Random-init weights of a Pibalorn shape generated in HBM."""
+    from powerinfer_amd import lib as pl, pibalorn
+    from powerinfer_amd.model import LayerModel
+    L = pl.init()
+    V, H, LH, dim = 32000, sh["heads"], sh["lin_heads"], sh["dim"]
+    dense = {"kind": "dense", "ff": sh["dense_ff"], "limit": 7.0}
+    moe = {"kind": "moe", "router": {"experts": sh["experts"], "top": sh["top"]}, "expert": {"ff": sh["ff"], "limit": 7.0}, "shared": {"ff": sh["shared_ff"], "limit": 7.0}}
+    att = {"type": "attention", "mixer": {"heads": H, "kv_heads": sh["kv_heads"], "dim": dim, "vdim": dim, "rot": {"dims": dim, "base": 10000.0}, "scale": dim ** -0.5}}
+    lin = {"type": "lightning", "mixer": {"heads": LH, "dim": sh["lin_dim"], "vdim": sh["lin_dim"], "decay": np.exp(-2.0 ** -np.linspace(0, 8, LH)).tolist()}}
+    cfg = {"width": width, "vocab": V, "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0, "bigram": {"buckets": 9973, "mul_prev": 31, "mul_cur": 7}}, "loop": {"start": 2, "stop": 4, "times": 2},
+           "layers": [dict(att, mlp=dense), dict(lin, mlp=moe), dict(att, mlp=moe), dict(lin, mlp=moe), dict(att, mlp=moe), dict(lin, mlp=moe)]}
+    descs = pibalorn.layer_descs(cfg)
+    m = LayerModel("pibalorn", descs, n_embd=width, n_vocab=V, n_ctx=n_ctx, norm_eps=1e-6, **pibalorn.model_opts(cfg))
+    seed = [7]
+
+    def put(layer, kind, rows, cols):
+        seed[0] += 1
+        buf = pl.DevBuf(rows * cols * 2)
+        pl.check(L.pi_fill_normal_bf16(buf.ptr, rows * cols, seed[0], 0.02, None), "fill")
+        m.set_tensor_device(layer, kind, buf.ptr, pl.BF16, cols, rows)
+        keep.append(buf)
+
+    one = np.ones(width, np.float32)
+    put(-1, "tok_embd", V, width)
+    put(-1, "output", V, width)
+    put(-1, "bigram", 9974, width)
+    m.set_tensor(-1, "output_norm", one)
+    m.set_tensor(-1, "loop_step", np.zeros((2, width), np.float32))
+    for i, (d, ly) in enumerate(zip(descs, cfg["layers"])):
+        m.set_tensor(i, "attn_norm", one)
+        hd, hv = d["n_head"] * d["dim"], d["n_head"] * d["vdim"]
+        put(i, "mix_q", hd, width)
+        if d["mixer"] == pl.MIXER_GROUPED:
+            put(i, "mix_k", d["n_kv_head"] * d["dim"], width)
+        else:
+            put(i, "mix_k", hd, width)
+            put(i, "mix_v", hv, width)
+            put(i, "mix_g", hv, width)
+            m.set_tensor(i, "mix_norm", np.ones(hv, np.float32))
+            m.set_tensor(i, "mix_decay", np.asarray(ly["mixer"]["decay"], np.float32))
+        put(i, "wo", width, hv)
+        for k, rows, cols in (("glu_gate", d["glu_ff"], width), ("glu_up", d["glu_ff"], width), ("glu_down", width, d["glu_ff"])):
+            put(i, k, rows, cols)
+        if d["ffn"] == pl.FFN_GLU_MOE:
+            E, ff = d["n_expert"], d["expert_ff"]
+            put(i, "router", E, width)
+            put(i, "shared_score", 1, width)
+            for k, rows, cols in (("expert_gate", E * ff, width), ("expert_up", E * ff, width), ("expert_down", E * width, ff)):
+                put(i, k, rows, cols)
+    pl.sync()
+    m.finalize()
+    return m
+
+
 def time_prefill_and_decode(m, n_prompt, steps, warmup):
     """(prompt seconds, seconds per decoded token) of one sequence: the prompt through Model.decode (second pass timed), then the greedy loop."""
     from powerinfer_amd import lib as pl
@@ -386,21 +450,27 @@ def time_lockstep(m, n_seq, n_prompt, steps, warmup):
 
 
 def bench_design(args):
-    """Prefill and decode of the Lerasun design at sizes like a real model's, beside the sparse LLaMA engine at equal width and depth."""
+    """Prefill and decode of a design described layer by layer at sizes like a real model's, beside the closest existing model at equal width
+    and depth: the sparse LLaMA engine for Lerasun, Lerasun for Pibalorn."""
     from powerinfer_amd import lib as pl, synth
     pl.init()
     n_prompt, steps, lock_prompt = (2048 if args.prompt == 64 else args.prompt), min(args.steps, 128), 128
     n_ctx = n_prompt + steps + args.warmup + 8
+    shapes = DESIGN_SHAPES if args.design == "lerasun" else PIBALORN_SHAPES
     rows = []
-    for width in ([args.design_width] if args.design_width else sorted(DESIGN_SHAPES)):
-        sh = DESIGN_SHAPES[width]
-        row = {"width": width, "n_layer": sh["layers"], **{k: v for k, v in sh.items() if k not in ("beside", "layers")}}
-        for who in ("lerasun", "beside"):
-            if args.design_only and who != args.design_only:
+    for width in ([args.design_width] if args.design_width else sorted(shapes)):
+        sh = shapes[width]
+        row = {"width": width, "n_layer": sh.get("layers", 8), **{k: v for k, v in sh.items() if k not in ("beside", "layers")}}
+        for who in (args.design, "beside"):
+            if args.design_only and (args.design_only == "beside") != (who == "beside"):
                 continue
             keep = []
-            if who == "lerasun":
+            if who == "pibalorn":
+                m = build_pibalorn_on_device(width, sh, n_ctx, keep)
+            elif who == "lerasun":
                 m = build_lerasun_on_device(width, sh, n_ctx, keep)
+            elif args.design == "pibalorn":
+                m = build_lerasun_on_device(width, dict(DESIGN_SHAPES[sh["beside"]], layers=8), n_ctx, keep)
             else:
                 name, over = sh["beside"]
                 hp = synth.hparams(name, n_layer=sh["layers"], n_ctx=n_ctx, seed=1, **over)
@@ -414,18 +484,18 @@ def bench_design(args):
                 b.free()
             print(f"# width {width} {who}: {row[who]}", file=sys.stderr, flush=True)
         rows.append(row)
-    best = rows[-1].get("lerasun") or rows[-1].get("beside")
-    print(json.dumps({"metric": "decode tok/s, batch 1, Lerasun layers (bf16)", "value": best["decode_tok_per_s"], "unit": "tokens/s", "n_gpus": 1, "steps": steps,
+    best = rows[-1].get(args.design) or rows[-1].get("beside")
+    print(json.dumps({"metric": f"decode tok/s, batch 1, {args.design.capitalize()} layers (bf16)", "value": best["decode_tok_per_s"], "unit": "tokens/s", "n_gpus": 1, "steps": steps,
                       "warmup": args.warmup, "ms_per_step": best["decode_ms_per_token"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16",
-                      "data": "synthetic", "config": {"model": "lerasun", "prompt_tokens": n_prompt, "lockstep_prompt_tokens": lock_prompt, "device": pl.device_name()},
+                      "data": "synthetic", "config": {"model": args.design, "prompt_tokens": n_prompt, "lockstep_prompt_tokens": lock_prompt, "device": pl.device_name()},
                       "sizes": rows}), flush=True)
 
 
 def main():
     ap = argparse.ArgumentParser()
-    ap.add_argument("--design", choices=["lerasun"], default=None, help="instead of the default workload: prefill and decode of this design beside the closest existing model")
+    ap.add_argument("--design", choices=["lerasun", "pibalorn"], default=None, help="instead of the default workload: prefill and decode of this design beside the closest existing model")
     ap.add_argument("--design-width", type=int, default=None, choices=sorted(DESIGN_SHAPES), help="one size of --design only")
-    ap.add_argument("--design-only", choices=["lerasun", "beside"], default=None, help="one side of --design only")
+    ap.add_argument("--design-only", choices=["design", "beside"], default=None, help="one side of --design only")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=256)
     ap.add_argument("--warmup", type=int, default=8)

@@ -262,7 +262,7 @@ void one_norm_sizes(Layer & L) {
     }
     if (d.ffn == PI_FFN_GLU_MOE) L.off_router = take(d.n_expert);
     L.z_rows = at;
-    L.hv_ld = up_to(d.n_head * d.vdim, 128); L.glu_ld = d.glu_ff > 0 ? up_to(d.glu_ff, 64) : 0; L.close_ld = L.hv_ld + L.glu_ld;
+    L.hv_ld = up_to(d.n_head * d.vdim, 128); L.glu_ld = d.glu_ff > 0 ? up_to(d.glu_ff, 128) : 0; L.close_ld = L.hv_ld + L.glu_ld;
     L.ff_ld = d.ffn == PI_FFN_GLU_MOE ? up_to(d.expert_ff, 64) : 0;
 }
 
