@@ -462,7 +462,7 @@ def bench_design(args):
         sh = shapes[width]
         row = {"width": width, "n_layer": sh.get("layers", 8), **{k: v for k, v in sh.items() if k not in ("beside", "layers")}}
         for who in (args.design, "beside"):
-            if args.design_only and (args.design_only == "beside") != (who == "beside"):
+            if args.design_only and who != args.design_only:
                 continue
             keep = []
             if who == "pibalorn":
@@ -495,7 +495,7 @@ def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--design", choices=["lerasun", "pibalorn"], default=None, help="instead of the default workload: prefill and decode of this design beside the closest existing model")
     ap.add_argument("--design-width", type=int, default=None, choices=sorted(DESIGN_SHAPES), help="one size of --design only")
-    ap.add_argument("--design-only", choices=["design", "beside"], default=None, help="one side of --design only")
+    ap.add_argument("--design-only", choices=["lerasun", "pibalorn", "beside"], default=None, help="one side of --design only")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=256)
     ap.add_argument("--warmup", type=int, default=8)

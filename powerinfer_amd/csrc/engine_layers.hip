@@ -829,15 +829,13 @@ int take_slot(pi_model * m, int q, uint32_t keep) {
 template <typename F> bool keeps_whole(LayerState * s, F && edit) {
     KvCells trial = s->kv;
     edit(trial);
-    for (int q = 0; q < 32; ++q) {
-        int before = 0, after = 0;
-        for (int i = 0; i < s->kv.n; ++i) {
-            before += s->kv.pos[i] >= 0 && (s->kv.seq[i] >> q & 1u);
-            after += trial.pos[i] >= 0 && (trial.seq[i] >> q & 1u);
-        }
-        if (after != before && after != 0) return false;
+    uint32_t lost = 0, left = 0;                                  // sequences that lose a cell, and that keep one
+    for (int i = 0; i < s->kv.n; ++i) {
+        const uint32_t before = s->kv.pos[i] >= 0 ? s->kv.seq[i] : 0u, after = trial.pos[i] >= 0 ? trial.seq[i] : 0u;
+        lost |= before & ~after;
+        left |= after;
     }
-    return true;
+    return (lost & left) == 0;
 }
 
 int upload_appends(pi_model * m, const std::vector<int32_t> & app) {

@@ -88,10 +88,28 @@ __global__ __launch_bounds__(256) void embed_bigram_kernel(const uint16_t * __re
     const int t = blockIdx.x, tok = tokens[t], before = prev[t];
     const uint16_t * a = table + (size_t)tok * cols, * b = nullptr;
     if (bigram) b = bigram + (size_t)(before < 0 ? buckets : (int)(((long long)before * mul_prev + (long long)tok * mul_cur) % buckets)) * cols;
-    for (int i = threadIdx.x; i < cols; i += 256) {
-        const float v = bf16_to_f32(a[i]) * scale + (b ? bf16_to_f32(b[i]) : 0.0f);
-        x[(size_t)t * cols + i] = v;
-        if (x0) x0[(size_t)t * cols + i] = v;
+    float * o = x + (size_t)t * cols, * o0 = x0 ? x0 + (size_t)t * cols : nullptr;
+    if ((cols & 7) == 0) {
+        for (int i = threadIdx.x * 8; i < cols; i += 2048) {
+            const pi_u32x4 u = pi_ld16(a + i), w = b ? pi_ld16(b + i) : pi_u32x4{0, 0, 0, 0};
+            float v[8];
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                v[2 * j] = __uint_as_float(u[j] << 16) * scale + __uint_as_float(w[j] << 16);
+                v[2 * j + 1] = __uint_as_float(u[j] & 0xffff0000u) * scale + __uint_as_float(w[j] & 0xffff0000u);
+            }
+#pragma unroll
+            for (int j = 0; j < 8; j += 4) {
+                *reinterpret_cast<float4 *>(o + i + j) = make_float4(v[j], v[j + 1], v[j + 2], v[j + 3]);
+                if (o0) *reinterpret_cast<float4 *>(o0 + i + j) = make_float4(v[j], v[j + 1], v[j + 2], v[j + 3]);
+            }
+        }
+    } else {
+        for (int i = threadIdx.x; i < cols; i += 256) {
+            const float v = bf16_to_f32(a[i]) * scale + (b ? bf16_to_f32(b[i]) : 0.0f);
+            o[i] = v;
+            if (o0) o0[i] = v;
+        }
     }
     if (carry) {
         __syncthreads();                               // every thread has read prev[t]

@@ -74,28 +74,37 @@ __global__ __launch_bounds__(256) void linear_step_kernel(pi_linear p, pi_ffn_fr
     }
 }
 
-// silu of the projections as bf16 operands, rows padded with zeros: a block covers 1024 values of a token's [q | k | v]
-constexpr int kLinPrep = 1024;
+// silu of the projections as bf16 operands, rows padded with zeros: a block covers 4096 values of a token's [q | k | v], a thread four of
+// every 1024
+constexpr int kLinPrep = 4096;
 __global__ __launch_bounds__(256) void linear_prep_kernel(pi_linear p, pi_ffn_front f, int n_val, int per) {
     extern __shared__ __align__(16) float sm[];
     const int t = blockIdx.x / per, b = blockIdx.x % per;
     if (b >= n_val) { front_block<bf16>(f, p.z, p.ldz, t, b - n_val, sm); return; }
-    const int nq = p.n_head * p.dim_ld, e = b * kLinPrep + threadIdx.x * 4;
-    if (e >= 2 * nq + p.n_head * p.vdim_ld) return;
-    const int what = e < nq ? 0 : e < 2 * nq ? 1 : 2, k = e - what * nq, ld = what == 2 ? p.vdim_ld : p.dim_ld, dim = what == 2 ? p.vdim : p.dim, h = k / ld, r = k % ld;
-    const float * z = p.z + (size_t)t * p.ldz + (what == 0 ? 0 : what == 1 ? p.off_k : p.off_v) + h * dim + r;
-    float v[4];
-    if (r + 4 <= dim && ((uintptr_t)z & 15) == 0) {
-        const float4 a = *reinterpret_cast<const float4 *>(z);
-        v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w;
-    } else {
+    const int nq = p.n_head * p.dim_ld, all = 2 * nq + p.n_head * p.vdim_ld;
+    constexpr int Q = kLinPrep / 1024;
+    float v[Q][4];
+    bf16 * o[Q];
 #pragma unroll
-        for (int j = 0; j < 4; ++j) v[j] = r + j < dim ? z[j] : 0.0f;
+    for (int i = 0; i < Q; ++i) {
+        const int e = min(b * kLinPrep + i * 1024 + (int)threadIdx.x * 4, all - 4);      // past the end: the last four again, the same values
+        const int what = e < nq ? 0 : e < 2 * nq ? 1 : 2, k = e - what * nq, ld = what == 2 ? p.vdim_ld : p.dim_ld, dim = what == 2 ? p.vdim : p.dim, h = k / ld, r = k % ld;
+        const float * z = p.z + (size_t)t * p.ldz + (what == 0 ? 0 : what == 1 ? p.off_k : p.off_v) + h * dim + r;
+        o[i] = (bf16 *)(what == 0 ? p.q : what == 1 ? p.k : p.v) + (size_t)t * p.n_head * ld + k;
+        if (r + 4 <= dim && ((uintptr_t)z & 15) == 0) {
+            const float4 a = *reinterpret_cast<const float4 *>(z);
+            v[i][0] = a.x; v[i][1] = a.y; v[i][2] = a.z; v[i][3] = a.w;
+        } else {
+#pragma unroll
+            for (int j = 0; j < 4; ++j) v[i][j] = r + j < dim ? z[j] : 0.0f;
+        }
     }
 #pragma unroll
-    for (int j = 0; j < 4; ++j) v[j] = silu_f32(v[j]);                      // (silu(0) = 0)
-    bf16 * o = (bf16 *)(what == 0 ? p.q : what == 1 ? p.k : p.v) + (size_t)t * p.n_head * ld + k;
-    store4(o, v, true, 4);
+    for (int i = 0; i < Q; ++i) {
+#pragma unroll
+        for (int j = 0; j < 4; ++j) v[i][j] = silu_f32(v[i][j]);            // (silu(0) = 0)
+        store4(o[i], v[i], true, 4);
+    }
 }
 
 // ---------------------------------------------------------------------------------------------------------------------------------

@@ -49,7 +49,7 @@ def model_opts(config):
     if b:
         out.update(bigram_buckets=b["buckets"], bigram_mul_prev=b["mul_prev"], bigram_mul_cur=b["mul_cur"])
     loop = config.get("loop")
-    if loop:
+    if loop and loop["stop"] > loop["start"]:
         out.update(loop_start=loop["start"], loop_stop=loop["stop"], loop_times=loop["times"])
     return out
 
