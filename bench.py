@@ -371,7 +371,7 @@ def build_pibalorn_on_device(width, sh, n_ctx, keep):
     moe = {"kind": "moe", "router": {"experts": sh["experts"], "top": sh["top"]}, "expert": {"ff": sh["ff"], "limit": 7.0}, "shared": {"ff": sh["shared_ff"], "limit": 7.0}}
     att = {"type": "attention", "mixer": {"heads": H, "kv_heads": sh["kv_heads"], "dim": dim, "vdim": dim, "rot": {"dims": dim, "base": 10000.0}, "scale": dim ** -0.5}}
     lin = {"type": "lightning", "mixer": {"heads": LH, "dim": sh["lin_dim"], "vdim": sh["lin_dim"], "decay": np.exp(-2.0 ** -np.linspace(0, 8, LH)).tolist()}}
-    cfg = {"width": width, "vocab": V, "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0, "bigram": {"buckets": 9973, "mul_prev": 31, "mul_cur": 7}}, "loop": {"start": 2, "stop": 4, "times": 2},
+    cfg = {"width": width, "vocab": V, "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0, "bigram": {"buckets": 9973, "mul_prev": 29, "mul_cur": 13}}, "loop": {"start": 2, "stop": 4, "times": 2},
            "layers": [dict(att, mlp=dense), dict(lin, mlp=moe), dict(att, mlp=moe), dict(lin, mlp=moe), dict(att, mlp=moe), dict(lin, mlp=moe)]}
     descs = pibalorn.layer_descs(cfg)
     m = LayerModel("pibalorn", descs, n_embd=width, n_vocab=V, n_ctx=n_ctx, norm_eps=1e-6, **pibalorn.model_opts(cfg))

@@ -4,11 +4,11 @@ import numpy as np
 from powerinfer_amd.checkpoint import bf16_bits, bf16_floats
 
 
-def dense(ff, limit=1.5):
+def dense(ff, limit=1.4):
     return {"kind": "dense", "ff": ff, "limit": limit}
 
 
-def moe(experts, top, ff, limit=2.0, shared=None):
+def moe(experts, top, ff, limit=1.8, shared=None):
     """shared: None, or (ff, limit)."""
     out = {"kind": "moe", "router": {"experts": experts, "top": top}, "expert": {"ff": ff, "limit": limit}}
     if shared:
@@ -25,7 +25,7 @@ def lightning(heads, dim, vdim, decay, mlp=None):
     return {"type": "lightning", "mixer": {"heads": heads, "dim": dim, "vdim": vdim, "decay": list(decay)}, "mlp": mlp}
 
 
-def config(width, vocab, layers, loop=None, eps=1e-5, scale=3.0, bigram=(97, 31, 7)):
+def config(width, vocab, layers, loop=None, eps=1e-5, scale=3.0, bigram=(97, 29, 13)):
     """loop: None, or (start, stop, times); bigram: (buckets, mul_prev, mul_cur)."""
     c = {"architecture": "Pibalorn", "width": width, "vocab": vocab, "layers": layers, "norm": {"eps": eps},
          "embedding": {"scale": scale, "bigram": dict(zip(("buckets", "mul_prev", "mul_cur"), bigram))}}
@@ -50,8 +50,8 @@ def odd_config():
 def even_config():
     return config(192, 200, [
         attention(8, 2, 64, mlp=dense(256)),
-        lightning(4, 64, 64, (0.999, 0.98, 0.9, 0.5), mlp=moe(16, 4, 48, shared=(64, 1.2))),
-        attention(6, 3, 32, base=50000.0, mlp=moe(12, 2, 64, 1.3, (32, 2.0))),
+        lightning(4, 64, 64, (0.999, 0.98, 0.9, 0.5), mlp=moe(18, 5, 48, shared=(64, 1.2))),
+        attention(6, 3, 32, base=50000.0, mlp=moe(12, 2, 64, 1.3, (32, 1.7))),
         lightning(2, 128, 128, (0.995, 0.6), mlp=moe(8, 1, 32)),
     ], loop=(1, 3, 2))
 

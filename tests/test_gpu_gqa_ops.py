@@ -21,7 +21,7 @@ def filled(cls, **kw):
     return s
 
 
-@pytest.mark.parametrize("cols,buckets,muls", [(64, 11, (31, 7)), (300, 1, (3, 5)), (1000, 50, (1 << 33, 1000003))])
+@pytest.mark.parametrize("cols,buckets,muls", [(64, 11, (29, 13)), (300, 1, (3, 5)), (1000, 50, (1 << 33, 1000003))])
 def test_embed_bigram(cols, buckets, muls):
     L, rng = pl.init(), np.random.default_rng(cols)
     table, bg = rounded(rng.standard_normal((40000, cols)))[:40000], rounded(rng.standard_normal((buckets + 1, cols)))
@@ -107,7 +107,7 @@ def prepped(q, k, v, pos, m, eps):
 
 
 @pytest.mark.parametrize("t", TYPES)
-@pytest.mark.parametrize("H,G,dim,vdim,rot,unit,ff,E,top", [(6, 3, 96, 96, 96, 1, 0, 0, 0), (5, 1, 17, 17, 6, 1, 30, 5, 2), (4, 2, 128, 64, 32, 0, 2100, 0, 0), (3, 3, 256, 256, 0, 1, 7, 300, 8),
+@pytest.mark.parametrize("H,G,dim,vdim,rot,unit,ff,E,top", [(6, 2, 96, 96, 96, 1, 0, 0, 0), (5, 1, 17, 17, 6, 1, 30, 5, 2), (4, 2, 128, 64, 32, 0, 2100, 0, 0), (3, 3, 256, 256, 0, 1, 7, 300, 8),
                                                             (8, 2, 40, 72, 40, 1, 0, 64, 6)])
 def test_gqa_prep_and_front(t, H, G, dim, vdim, rot, unit, ff, E, top):
     L, rng = pl.init(), np.random.default_rng(dim)
@@ -187,7 +187,7 @@ def attend(t, rng, seqs, H, G, dim, vdim, parts, wide, scale, sink, spike=()):
     return got[:, :H * vdim].reshape(T, H, vdim), want
 
 
-SHAPES = [(6, 3, 96, 96), (5, 1, 17, 17), (4, 4, 32, 20), (8, 1, 64, 64), (16, 2, 128, 128), (3, 3, 130, 130), (40, 2, 40, 64), (2, 1, 256, 250)]
+SHAPES = [(6, 2, 96, 96), (5, 1, 17, 17), (4, 4, 32, 20), (8, 1, 64, 64), (16, 2, 128, 128), (3, 3, 130, 130), (40, 2, 40, 64), (2, 1, 256, 250)]
 
 
 @pytest.mark.parametrize("t,parts,wide", [(pl.F32, 1, 0), (pl.BF16, 1, 0), (pl.BF16, 5, 0), (pl.BF16, 64, 0), (pl.BF16, 1, 1), (pl.BF16, 3, 1)])

@@ -60,7 +60,7 @@ def close(got, want, limit):
     return np.abs(got - want).max() <= limit * np.abs(want).max()
 
 
-SHAPES = [(3, 20, 36, (1.0, 0.5, 0.03)), (2, 64, 64, (0.999, 0.6)), (5, 33, 9, (0.999, 0.9, 0.0, 0.7, 0.97)), (1, 128, 128, (0.98,)), (2, 256, 70, (0.9, 1.0)), (2, 90, 256, (0.99, 0.5)),
+SHAPES = [(3, 20, 36, (1.0, 0.5, 0.03)), (4, 64, 64, (0.997, 0.7, 0.95, 0.4)), (5, 33, 9, (0.999, 0.9, 0.0, 0.7, 0.97)), (1, 128, 128, (0.98,)), (2, 256, 70, (0.9, 1.0)), (2, 90, 256, (0.99, 0.5)),
           (1, 1, 1, (0.9,))]
 
 
@@ -88,8 +88,8 @@ def test_chunks(H, dim, vdim, decay, runs):
 def test_chunks_and_steps_agree_closely():
     """The same tokens in chunks and one by one: what fp32 numbers lose as sums of two bf16 is far below bf16's own rounding."""
     runs, rng = [(150, 0, False)], lambda: np.random.default_rng(9)
-    a, _, sa, _ = run(pl.BF16, rng(), runs, 2, 64, 64, (0.999, 1.0), True)
-    b, _, sb, _ = run(pl.BF16, rng(), runs, 2, 64, 64, (0.999, 1.0), False)
+    a, _, sa, _ = run(pl.BF16, rng(), runs, 3, 64, 64, (0.999, 1.0, 0.8), True)
+    b, _, sb, _ = run(pl.BF16, rng(), runs, 3, 64, 64, (0.999, 1.0, 0.8), False)
     assert close(a, b, 3e-5) and close(sa, sb, 3e-5)
 
 

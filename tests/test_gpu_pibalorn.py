@@ -443,7 +443,7 @@ def test_bad_models_are_refused():
     with pytest.raises(pl.PiError, match="mix_g"):
         pibalorn.build(cfg, bad)
     for spoil, why in ((lambda c: c["layers"][0]["mixer"].update(kv_heads=3), "grouped-query"), (lambda c: c["loop"].update(stop=9), "loop"),
-                       (lambda c: c["layers"][1]["mlp"]["router"].update(top=17), "experts"), (lambda c: c["layers"][0]["mixer"]["rot"].update(dims=66), "grouped-query")):
+                       (lambda c: c["layers"][1]["mlp"]["router"].update(top=19), "experts"), (lambda c: c["layers"][0]["mixer"]["rot"].update(dims=66), "grouped-query")):
         c = even_config()
         spoil(c)
         with pytest.raises(pl.PiError, match=why):
