@@ -127,8 +127,8 @@ def test_a_mistake_in_a_mechanism_shows(monkeypatch, name):
     e = row_errors(run(), good)
     if "first token" in name:
         assert e[0] > 0.05
-    elif "decay" in name:                                   # the less a token weighs among those before it, the smaller the difference
-        assert e.max() > 0.2 and np.median(e) > 1e-3
+    elif "decay" in name:                                   # a factor per head, which the norm behind the heads takes out in part
+        assert np.median(e) > 5e-3
     elif "lost" in name:
         assert (e[:20] == 0).all() and e[20:].max() > 0.1
     else:
