@@ -650,54 +650,86 @@ PI_API int pi_k_latent_shift(int type, void * cache, int n_cells, int kd, int ra
 typedef struct pi_ffn_front {
     int32_t off_glu, ff, ff_ld, off_score; float limit, gain; void * act; int32_t ld_act;
     int32_t off_router, n_expert, n_top; int32_t * ids; float * weights;
+    int32_t plain_up;                                            /* y = g * sigmoid(gain * g) * u, without the one */
 } pi_ffn_front;
+/* the same by itself, over T rows of z */
+PI_API int pi_k_ffn_front(int type, const float * z, int ldz, int T, const pi_ffn_front * front, pi_stream_t stream);
 /* Grouped-query attention, behind the joint projection z [T][ldz] of its layer: queries at 0 (n_head x dim), keys at off_k (n_kv x dim), values at
  * off_v (n_kv x vdim; off_v == off_k: the values are the keys as projected).  Queries and keys are rotated (pairs i, i + rot_dim / 2 of the
- * first rot_dim values; cs as pi_k_rope_angles makes it) and, with unit != 0, divided by their root mean square; queries go to
- * q [T][n_head][hd], the token's cell is n_kv rows [key | value] of hd values each, padded with zeros (pi_k_gqa_head_ld).  front (optional)
- * runs in the same launch. */
+ * first rot_dim values, with rot_pairs != 0 pairs 2 i, 2 i + 1; cs as pi_k_rope_angles makes it) and, with unit != 0, divided by their root
+ * mean square; queries go to q [T][n_head][hd], the token's cell is n_kv rows [key | value] of hd values each, padded with zeros
+ * (pi_k_gqa_head_ld).  q_norm, k_norm (optional, [dim], both or none; unit 0): RMS norm of every head with these weights ahead of the
+ * rotation; unit_v: values are divided by their root mean square; temp (optional, [n_head]): factor of a head's queries.  front (optional) runs in the
+ * same launch. */
 typedef struct pi_gqa_prep {
     const float * z; int32_t ldz, T, n_head, n_kv, dim, vdim, rot_dim, off_k, off_v, hd, unit;
     const void * cs; float eps; void * q, * cache; const int32_t * cell;
+    int32_t rot_pairs, unit_v; const float * q_norm, * k_norm, * temp;
 } pi_gqa_prep;
 PI_API int pi_k_gqa_head_ld(int type, int dim, int vdim);                    /* hd for a head size, 0: not supported */
 PI_API int pi_k_gqa_prep(int type, const pi_gqa_prep * p, const pi_ffn_front * front, pi_stream_t stream);
 /* The attention itself.  bf16: work [n_work] = {first token, first row among (tokens behind it) x (n_head / n_kv), rows, sequence} of at most
  * pi_k_gqa_rows(wide) rows; query row r sees the cells lists[seq][0 .. n_vis[its token]).  n_parts > 1: the cells are split over that many
  * workgroups, partial sums in scratch (pi_k_gqa_scratch_floats).  fp32: work [T] = each token's sequence.  sink: score of an entry of the
- * soft-max without a value (-INFINITY: none).  att [T][ld_att] gets n_head x vdim values per token.  pi_k_gqa_attn merges the parts,
- * pi_k_gqa_attn_parts leaves them to pi_k_mix_up_step. */
+ * soft-max without a value (-INFINITY: none).  window > 0: a token sees the last `window` of those cells only; first (optional, [T]): it sees
+ * the cells from first[token] on instead (ascending along a run).  att [T][ld_att] gets n_head x vdim values per token, times out_scale.
+ * pi_k_gqa_attn merges the parts, pi_k_gqa_attn_parts leaves them to pi_k_mix_up_step. */
 typedef struct pi_gqa_attn {
     const void * q, * cache; const int32_t * lists; size_t list_ld; const int32_t * work, * n_vis;
     int32_t n_work, T, n_head, n_kv, dim, vdim, hd, n_parts, wide; float scale, sink; float * scratch; void * att; int32_t ld_att;
+    float out_scale; int32_t window; const int32_t * first;
 } pi_gqa_attn;
 PI_API int    pi_k_gqa_rows(int wide);
 PI_API size_t pi_k_gqa_scratch_floats(int n_work, int wide, int n_kv, int hd, int n_parts);
 PI_API int    pi_k_gqa_attn(int type, const pi_gqa_attn * p, pi_stream_t stream);
 PI_API int    pi_k_gqa_attn_parts(const pi_gqa_attn * p, pi_stream_t stream);
-/* rotates the key parts of cells by delta[cell] positions */
-PI_API int pi_k_gqa_shift(int type, void * cache, int n_cells, int n_kv, int hd, int rot_dim, double base, const int32_t * delta, pi_stream_t stream);
-/* Linear attention with a constant decay per head over a fp32 state [slot][n_head][dim][vdim], behind the joint projection z [T][ldz]: q = silu(z) at 0
- * (n_head x dim), k = silu at off_k, v = silu at off_v (n_head x vdim); S = decay S + k v^T, o = S^T q.  runs [n_runs] = {first token, tokens,
- * slot, 1 if the state starts at zero}: the consecutive tokens of one sequence.  o [T][n_head * vdim] fp32.
- * pi_k_linear_step walks every run token by token; front (optional) runs in the same launch.
+/* rotates the key parts of cells by delta[cell] positions (pairs != 0: neighbouring values are a pair) */
+PI_API int pi_k_gqa_shift(int type, void * cache, int n_cells, int n_kv, int hd, int rot_dim, double base, int pairs, const int32_t * delta, pi_stream_t stream);
+/* Linear attention over a fp32 state [slot][n_head][dim][vdim] (slot_ld floats per slot, 0: exactly these), behind the joint projection
+ * z [T][ldz]: q at off_q (n_head x dim), k at off_k, v at off_v (n_head x vdim); silu of each, or with plain != 0 the projections themselves and
+ * q times q_scale.  decay_kind says what becomes of the state:
+ *   PI_DECAY_CONST  S = d S + k v^T with d = decay[head], o = S^T q
+ *   PI_DECAY_KEYED  S = diag(a) S + k v^T with a decay per key channel and token, a = sigmoid(u)^(1 / tau), u = a2 z[off_a ..] + a2_b;
+ *                   a2 [n_head * dim][rank_ld] bf16, rank_ld a multiple of 8
+ *   PI_DECAY_GATED  exponential gates per head with a running maximum: i = cap tanh((z[off_i + head] + i_b) / cap),
+ *                   f = log sigmoid(cap tanh((z[off_f + head] + f_b) / cap)), m' = max(f + m, i), S = exp(f + m - m') S + exp(i - m') k v^T, the sum n of
+ *                   keys likewise, o = S^T q and den [T][n_head] = max(|n . q|, exp(-m')) + 1e-6, by which o has still to be divided.
+ *                   Behind a slot's S follow n [n_head][dim] and pi_k_linear_copies(vdim) copies of m per head (pi_k_linear_slot_floats).
+ * runs [n_runs] = {first token, tokens, slot, 1 if the state starts at zero}: the consecutive tokens of one sequence.  o [T][n_head * vdim] fp32.
+ * pi_k_linear_step walks every run token by token; front (optional) and prep (optional, the queries and cells of a grouped-query attention
+ * beside it) run in the same launch.
  * pi_k_linear_prep + pi_k_linear_chunks (bf16) do the same for long runs in chunks of pi_k_linear_chunk() tokens: q, k [T][n_head][dim_ld] and
  * v [T][n_head][vdim_ld] in bf16 (dim_ld a multiple of 32, vdim_ld of 64), then the states before every chunk (as sums of two bf16) into
  * states (pi_k_linear_states_bytes) and the outputs.  chunks [n_chunks] = {first token, tokens, 1 if nothing lies before it}, a run's chunks
- * behind one another; run r of `runs` begins with chunk first_chunk[r].  powers [n_head][chunk + 1]: decay^0 .. decay^chunk. */
+ * behind one another; run r of `runs` begins with chunk first_chunk[r].  powers [n_head][chunk + 1]: decay^0 .. decay^chunk.  gates: room for
+ * pi_k_linear_gate_floats numbers - the sums of log2 decays since the chunk's start [T][n_head][dim_ld], or per token and head
+ * what the exponential gates come to, and the running maximum ahead of every chunk. */
+enum { PI_DECAY_CONST = 0, PI_DECAY_KEYED = 1, PI_DECAY_GATED = 2 };
 typedef struct pi_linear {
     const float * z; int32_t ldz, T, n_head, dim, vdim, off_k, off_v;
     const float * decay, * powers; float * state; const int32_t * runs; int32_t n_runs; float * o;
     void * q, * k, * v, * states; int32_t dim_ld, vdim_ld, n_chunks; const int32_t * chunks, * first_chunk;
+    int32_t decay_kind, off_q, plain; float q_scale; size_t slot_ld;
+    const void * a2; const float * a2_b; int32_t off_a, rank, rank_ld; float tau;
+    const float * i_b, * f_b; int32_t off_i, off_f; float cap; float * den;
+    float * gates;
 } pi_linear;
 PI_API int    pi_k_linear_chunk(void);
 PI_API int    pi_k_linear_supported(int dim, int vdim);
+PI_API int    pi_k_linear_copies(int vdim);
+PI_API size_t pi_k_linear_slot_floats(int decay_kind, int n_head, int dim, int vdim);
 PI_API size_t pi_k_linear_states_bytes(int n_chunks, int n_head, int dim_ld, int vdim_ld);
+PI_API size_t pi_k_linear_gate_floats(int decay_kind, int T, int n_chunks, int n_head, int dim_ld);
 PI_API int    pi_k_linear_step(int type, const pi_linear * p, const pi_ffn_front * front, pi_stream_t stream);
+PI_API int    pi_k_linear_step_beside(int type, const pi_linear * p, const pi_gqa_prep * prep, pi_stream_t stream);
 PI_API int    pi_k_linear_prep(int type, const pi_linear * p, const pi_ffn_front * front, pi_stream_t stream);
 PI_API int    pi_k_linear_chunks(const pi_linear * p, pi_stream_t stream);
-/* att[t][0 .. n) = rms_norm(o[t]) * w * sigmoid(z[t][off_gate ..]), o [T][n] */
-typedef struct pi_gate_norm { const float * o, * z, * w; int32_t ldz, off_gate, n, T; float eps; void * att; int32_t ld_att; } pi_gate_norm;
+/* att[t][0 .. n) = scale * rms_norm(o[t]) * w * sigmoid(z[t][off_gate ..]), o [T][n]; heads > 0: the norm is taken over each of `heads` equal parts of
+ * o[t] by itself (up to 256 values a part), divided by den [T][heads] before (optional); silu: silu of the gate instead of its sigmoid */
+typedef struct pi_gate_norm {
+    const float * o, * z, * w; int32_t ldz, off_gate, n, T; float eps; void * att; int32_t ld_att;
+    float scale; int32_t heads, silu; const float * den;
+} pi_gate_norm;
 PI_API int pi_k_gate_norm(int type, const pi_gate_norm * p, pi_stream_t stream);
 /* expert choice of T tokens from router logits z [T][n_expert] (see PI_FFN_MOE): ids, weights [T][n_top] by falling choice score */
 PI_API int pi_k_route(const float * z, int T, int n_expert, int n_top, int n_group, int n_keep, const float * bias, int32_t * ids, float * weights,
@@ -719,6 +751,8 @@ typedef struct pi_layer_out {
     const float * x; const void * wo, * att; int32_t rows, ld_att, T;
     const void * down, * act; const int32_t * ids; int32_t ld_act, top, n_expert;
     float * out, * keep;
+    int32_t scaled; float alpha;                                 /* scaled != 0: out = alpha x + .. */
+    const float * gate_z, * gate_b; int32_t ld_gate, off_gate;   /* gate_z (optional): what is added is multiplied by sigmoid(gate_z[t][off_gate + row] + gate_b[row]) */
 } pi_layer_out;
 PI_API int pi_k_layer_step_supported(int T, int n_expert, int n_top);
 PI_API int pi_k_latent_step(const pi_latent_prep * p, const void * uk_t, const float * z_router, int n_expert, int n_top, int n_group, int n_keep, const float * bias,
@@ -732,6 +766,18 @@ PI_API int pi_k_layer_out_step(const pi_layer_out * a, pi_stream_t stream);
  * turn) for every (token, choice), in one launch. */
 PI_API int pi_k_mix_up_step(const pi_gqa_attn * attn, const pi_gate_norm * gate, const void * up, int n_expert, int ff, int cols, float limit, float gain,
                             const void * x_ol, int T, const int32_t * ids, const float * weights, int top, void * act, int ld_act, pi_stream_t stream);
+/* What closes a sublayer whose norm comes after the sum: s = alpha x[t] + g * mix[t] with g = sigmoid(gate_z[t][off_gate ..] + gate_b) (gate_z NULL: 1),
+ * or s = x[t] (mix NULL); out[t] = rms_norm(s) * w (w NULL: s); h (optional): the same as the next product's operand, rows of ld values or
+ * (ol, BF16, T <= 16) in the operand layout of pi_k_gemm_bf16_ol; keep (optional) receives a copy.  out may be x. */
+typedef struct pi_res_norm {
+    const float * x, * mix, * gate_z, * gate_b, * w; int32_t ld_gate, off_gate, T, cols; float alpha, eps;
+    float * out, * keep; void * h; int32_t ld, ol;
+} pi_res_norm;
+PI_API int pi_k_res_norm(int type, const pi_res_norm * p, pi_stream_t stream);
+/* Steps of up to 16 tokens (bf16), one launch over activations in the operand layout: act [T][ld_act] = g * sigmoid(gain g) * (u + one) with gate and up
+ * rows of W [2 ff][cols] in turn (clamped to limit as pi_ffn_front does), and (W2 != NULL) y2 [T][rows2] = W2 x; cols % 256 == 0 */
+PI_API int pi_k_gemm_bf16_ol_glu(const void * W, int ff, const void * xn_ol, float limit, float gain, float one, void * act, int ld_act, const void * W2, int rows2, float * y2,
+                                 int cols, int T, pi_stream_t stream);
 /* BF16 matrices: out [rows][ld] = in [rows][cols] padded with zeros; out [n_mat][cols][ld] = each in [rows][cols] transposed, padded with zeros */
 PI_API int pi_k_pad_cols_bf16(const void * in, int64_t rows, int cols, void * out, int ld, pi_stream_t stream);
 /* row r of in [rows][cols] becomes columns col0 .. col0 + width - 1 (zeros behind cols) of row row0 + r * row_step of out [..][ld] */
@@ -742,7 +788,7 @@ PI_API int pi_k_cells_advance(int T, const int32_t * seq, const int32_t * lists,
 
 /* ---- decode loop with resident weights ------------------------------------------------------------- */
 
-enum { PI_ARCH_LLAMA = 0, PI_ARCH_FALCON = 1, PI_ARCH_LERASUN = 2, PI_ARCH_PIBALORN = 3 };
+enum { PI_ARCH_LLAMA = 0, PI_ARCH_FALCON = 1, PI_ARCH_LERASUN = 2, PI_ARCH_PIBALORN = 3, PI_ARCH_FIKEVIK = 4 };
 
 /* the llama_hparams fields this path reads (llama.cpp:1207-1270) */
 typedef struct pi_hparams {
@@ -770,6 +816,12 @@ enum {
     PI_T_BIGRAM, PI_T_LOOP_STEP,
     PI_T_MIX_K, PI_T_MIX_V, PI_T_MIX_G, PI_T_MIX_NORM, PI_T_MIX_DECAY,
     PI_T_EXPERT_GATE, PI_T_GLU_GATE, PI_T_GLU_UP, PI_T_GLU_DOWN, PI_T_SHARED_SCORE,
+    /* gates on what a sublayer adds (matrix and bias, mixer and feed-forward); norms of queries and keys, factors of the heads' scores; low-rank
+     * decays of a keyed linear attention; the matrix memory beside an attention (projections, norm, gate rows and their biases) */
+    PI_T_RES_GATE, PI_T_RES_GATE_B, PI_T_RES_GATE_FFN, PI_T_RES_GATE_FFN_B,
+    PI_T_MIX_Q_NORM, PI_T_MIX_K_NORM, PI_T_MIX_TEMP,
+    PI_T_MIX_A1, PI_T_MIX_A2, PI_T_MIX_A2_B,
+    PI_T_MEM_Q, PI_T_MEM_K, PI_T_MEM_V, PI_T_MEM_G, PI_T_MEM_O, PI_T_MEM_NORM, PI_T_MEM_I, PI_T_MEM_I_B, PI_T_MEM_F, PI_T_MEM_F_B,
     PI_T_COUNT
 };
 
@@ -777,6 +829,11 @@ enum {
  * Models whose layers are described one by one.  A layer is  x + (mixer(norm_a(x)) + ffn(norm_b(x)))  (both of the same x; tensors
  * PI_T_ATTN_NORM and PI_T_FFN_NORM), or without the second part (PI_FFN_NONE).  PI_MIXER_LATENT layers have two RMS norms, layers with
  * the other mixers one layer norm (weight, no bias) that both parts share; a model has layers of one of the two families.
+ * With post_norm the arrangement is another one: x = rms_norm(residual_alpha x + g * mixer(x)) * PI_T_ATTN_NORM, then the same with the feed-forward and
+ * PI_T_FFN_NORM (without a feed-forward only the first), where g = sigmoid(W x + b) of the sublayer's input if the layer has gated_residual
+ * (PI_T_RES_GATE [n_embd][n_embd], PI_T_RES_GATE_B; PI_T_RES_GATE_FFN, PI_T_RES_GATE_FFN_B), else 1; mixers PI_MIXER_GROUPED and PI_MIXER_KEYED,
+ * feed-forwards PI_FFN_NONE and PI_FFN_GLU.  A layer with weights_of = j + 1 has no tensors and uses those of layer j, with a cache and states of
+ * its own.
  *
  * Layers loop_start .. loop_stop - 1 run loop_times times in a row (each pass with a cache or state of its own).  Before every pass but the
  * first the embedding is added to the residual stream, before every pass row t of PI_T_LOOP_STEP [loop_times][n_embd].
@@ -797,13 +854,22 @@ enum {
  *   or, values_are_keys, the keys as projected).  Rotation of the first rot_dim values of a head, value i paired with i + rot_dim / 2,
  *   frequency rot_base^(-2i / rot_dim); unit_qk: queries and keys are divided by their root mean square afterwards; scores times
  *   `scale`; sink: the soft-max has one more entry, of this score and without a value (-INFINITY: none).
+ *   rot_pairs: value 2 i paired with 2 i + 1; qk_norm: RMS norms PI_T_MIX_Q_NORM, _K_NORM [dim] of every head ahead of the rotation; unit_v: values
+ *   divided by their root mean square; head_temp: scores also times PI_T_MIX_TEMP [n_head]; window > 0: a token sees itself and the
+ *   window - 1 positions before it.
+ *   mem_heads > 0 (post_norm): beside it, from the same input, a matrix memory with exponential gates (PI_DECAY_GATED; PI_T_MEM_*, mem_heads heads of
+ *   mem_dim x mem_vdim, cap mem_cap), its heads divided by their root mean square, times PI_T_MEM_NORM [mem_heads * mem_vdim] and
+ *   sigmoid(PI_T_MEM_G h), through PI_T_MEM_O; the mixer is out_scale * attention + mem_scale * memory.
+ * PI_MIXER_KEYED (post_norm): linear attention with a decay per key channel (PI_DECAY_KEYED; PI_T_MIX_Q, _K, _V, _A1 [decay_rank][n_embd],
+ *   _A2 [n_head * dim][decay_rank], _A2_B, decay_tau), queries times dim^-1/2, every head RMS-normed with its part of PI_T_MIX_NORM [n_head * vdim], times
+ *   silu(PI_T_MIX_G h), through PI_T_WO.
  * PI_MIXER_LINEAR: linear attention with the decay PI_T_MIX_DECAY [n_head] (pi_linear; PI_T_MIX_Q, _K [n_head * dim], _V [n_head * vdim]), its output
  *   RMS-normed over all heads with PI_T_MIX_NORM, times sigmoid(PI_T_MIX_G h), through PI_T_WO.
- * PI_FFN_GLU: PI_T_GLU_GATE, _UP [glu_ff][n_embd], _DOWN [n_embd][glu_ff], the clamped GLU with glu_limit and glu_gain (pi_ffn_front).
+ * PI_FFN_GLU: PI_T_GLU_GATE, _UP [glu_ff][n_embd], _DOWN [n_embd][glu_ff], the clamped GLU with glu_limit and glu_gain (pi_ffn_front; glu_plain_up: plain_up).
  * PI_FFN_GLU_MOE: PI_T_ROUTER; the n_top largest logits, weights their soft-max; PI_T_EXPERT_GATE, _UP, _DOWN as above with expert_limit;
  *   glu_ff > 0: beside them a shared one (PI_T_GLU_*, glu_limit) that every token uses times sigmoid(PI_T_SHARED_SCORE [1][n_embd] h).
  */
-enum { PI_MIXER_LATENT = 0, PI_MIXER_GROUPED = 1, PI_MIXER_LINEAR = 2 };
+enum { PI_MIXER_LATENT = 0, PI_MIXER_GROUPED = 1, PI_MIXER_LINEAR = 2, PI_MIXER_KEYED = 3 };
 enum { PI_FFN_NONE = 0, PI_FFN_MOE = 1, PI_FFN_GLU = 2, PI_FFN_GLU_MOE = 3 };
 typedef struct pi_layer_desc {
     int32_t mixer, n_head, dim, rot_dim, vdim, kv_rank, kv_from;
@@ -812,6 +878,10 @@ typedef struct pi_layer_desc {
     int32_t ffn, n_expert, n_top, n_group, n_group_keep, expert_ff;
     int32_t n_kv_head, values_are_keys, unit_qk; float sink;
     int32_t glu_ff; float glu_limit, expert_limit, glu_gain;
+    int32_t weights_of, gated_residual, glu_plain_up;
+    int32_t rot_pairs, qk_norm, unit_v, head_temp, window; float out_scale;
+    int32_t mem_heads, mem_dim, mem_vdim; float mem_cap, mem_scale;
+    int32_t decay_rank; float decay_tau;
 } pi_layer_desc;
 typedef struct pi_layers_opts {
     int32_t compute;         /* PI_TYPE_BF16: activations and caches in bf16, fp32 accumulation (residual, norms, router, scores in fp32);
@@ -825,6 +895,7 @@ typedef struct pi_layers_opts {
     int32_t bigram_buckets; int64_t bigram_mul_prev, bigram_mul_cur;
     int32_t loop_start, loop_stop, loop_times;
     int32_t n_slots;         /* sequences whose recurrent states there is room for at the start (0: 4; grows when more are live) */
+    int32_t post_norm; float residual_alpha;
 } pi_layers_opts;
 
 /* The ggml_cuda_* boundary (include/ggml_backend_abi.h) keeps single-token nodes in a window until it knows whether they form a block

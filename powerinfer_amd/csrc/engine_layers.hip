@@ -25,20 +25,34 @@ constexpr int kLinearChunked = 17;       // tokens from which a run of linear at
 
 int up_to(int v, int m) { return (v + m - 1) / m * m; }
 
+// the recurrent part of a layer's mixer: rows of the joint projection, sizes and weights
+struct Rec {
+    int kind = -1, n_head = 0, dim = 0, vdim = 0, dim_ld = 0, vdim_ld = 0, rank = 0, rank_ld = 0;
+    int off_q = 0, off_k = 0, off_v = 0, off_g = 0, off_a = 0, off_i = 0, off_f = 0, off_att = 0;      // off_att: column of the mixer's result
+    float tau = 0.0f, cap = 0.0f, q_scale = 1.0f, scale = 1.0f;
+    bool plain = false, silu = false, per_head = false;           // projections without an activation; gate; norm over every head by itself
+    const float *decay = nullptr, *powers = nullptr, *norm = nullptr, *a2_b = nullptr, *i_b = nullptr, *f_b = nullptr;
+    const void * a2 = nullptr;
+    bool on() const { return kind >= 0; }
+};
+
 struct Layer {
     pi_layer_desc d{};
+    Rec rec;
     int nq = 0, z_rows = 0, dim_ld = 0, rank_ld = 0, kd = 0, hv_ld = 0, ff_ld = 0, rot = 0, hc = 0;      // rot, hc: index among the model's rotations / kinds of heads
-    int off_k = 0, off_v = 0, off_g = 0, off_glu = 0, off_score = -1, off_router = 0;      // rows of the joint projection (layers with one norm)
-    int hd = 0, vdim_ld = 0, glu_ld = 0, close_ld = 0;
+    int off_k = 0, off_v = 0, off_glu = 0, off_score = -1, off_router = 0;      // rows of the joint projection (layers with one norm)
+    int off_gate = 0, off_gate_ffn = 0, z2_rows = 0;              // norm after the sum: rows of the residual gates, rows of the feed-forward's projection
+    int hd = 0, glu_ld = 0, close_ld = 0;
     bool own_kv = true;
     const void *w_z = nullptr, *uk = nullptr, *uk_t = nullptr, *uv = nullptr, *wo = nullptr, *router = nullptr, *up = nullptr, *down = nullptr;
     const float *norm_a = nullptr, *norm_b = nullptr, *dkv_norm = nullptr, *sink = nullptr, *bias = nullptr;
-    const float *mix_norm = nullptr, *decay = nullptr, *powers = nullptr;
+    const void * w_ffn = nullptr;                                 // norm after the sum: [gate and up rows in turn | residual gate]
+    const float *q_norm = nullptr, *k_norm = nullptr, *temp = nullptr, *gate_b = nullptr, *gate_ffn_b = nullptr;
     // one per pass of the loop the layer is part of
     std::vector<void *> cache;                         // cells
-    std::vector<float *> state;                        // [slots][n_head][dim][vdim]
+    std::vector<float *> state;                        // [slots][state_floats()]
     size_t cell_values() const { return d.mixer == PI_MIXER_GROUPED ? (size_t)d.n_kv_head * 2 * hd : d.mixer == PI_MIXER_LATENT && own_kv ? (size_t)kd : 0; }
-    size_t state_floats() const { return d.mixer == PI_MIXER_LINEAR ? (size_t)d.n_head * d.dim * d.vdim : 0; }
+    size_t state_floats() const { return rec.on() ? pi_k_linear_slot_floats(rec.kind, rec.n_head, rec.dim, rec.vdim) : 0; }
     bool moe() const { return d.ffn == PI_FFN_MOE || d.ffn == PI_FFN_GLU_MOE; }
 };
 
@@ -46,7 +60,9 @@ struct LayerRun { int layer, pass; bool starts; };     // starts: a pass of the 
 
 struct Rotation { int dims; double base; };
 // n_head: of a work item's rows - all heads on a latent, the heads of a group otherwise (n_kv groups, kd values of a key row)
-struct HeadKind { int mixer, n_head, n_kv, dim, rot_dim, vdim, rank_ld, kd; };
+// window > 0: cells a token sees
+struct HeadKind { int mixer, n_head, n_kv, dim, rot_dim, vdim, rank_ld, kd, window; };
+enum Family { kTwoNorms, kOneNorm, kPostNorm };
 
 // where a pass finds its tokens
 struct Step {
@@ -61,6 +77,7 @@ struct Step {
     // grouped-query attention: the long runs as wide work items (per kind); linear attention: the runs walked token by token and in chunks;
     // prev: each token's predecessor (carry: the embedding moves it on, for a captured step)
     std::vector<Work> wide;
+    std::vector<const int32_t *> first;                // per kind: the first cell of each token's window (null: counted back from its last)
     int32_t * prev = nullptr; bool carry = false;
     const int32_t *lin = nullptr, *lin_long = nullptr, *lin_first = nullptr, *lin_chunks = nullptr;
     int n_lin = 0, n_lin_long = 0, n_lin_chunks = 0;
@@ -80,7 +97,8 @@ struct LayerState {
     const void *embed = nullptr, *head = nullptr, *bigram = nullptr;
     const float * loop_step = nullptr;                 // [loop_times][n_embd]
     std::vector<LayerRun> order;                       // the layer runs of a step
-    bool one_norm = false, recurrent = false;
+    Family family = kTwoNorms;
+    bool recurrent = false;
     int n_slots = 0, slot_of[32];                      // slots of recurrent states; -1: the sequence has none
     KvCells kv;
     std::vector<int32_t> cell_tok;                     // the token of every cell
@@ -91,7 +109,7 @@ struct LayerState {
     // step buffers for `cap` tokens (one allocation)
     int cap = 0;
     unsigned char * arena = nullptr;
-    float *x = nullptr, *x2 = nullptr, *x0 = nullptr, *z = nullptr, *mix = nullptr, *rl = nullptr, *wts = nullptr, *lin_o = nullptr;
+    float *x = nullptr, *x2 = nullptr, *x0 = nullptr, *z = nullptr, *mix = nullptr, *rl = nullptr, *wts = nullptr, *lin_o = nullptr, *lin_den = nullptr, *lin_gates = nullptr;
     void *lin_q = nullptr, *lin_k = nullptr, *lin_v = nullptr, *lin_states = nullptr;
     void *h_a = nullptr, *h_b = nullptr, *q_un = nullptr, *q_lat = nullptr, *o_lat = nullptr, *att = nullptr, *act = nullptr, *y_exp = nullptr;
     int32_t *ids = nullptr, *perm = nullptr, *inv = nullptr, *off = nullptr, *tiles = nullptr, *n_tiles = nullptr;
@@ -177,6 +195,13 @@ uint16_t * zeroed(pi_model * m, size_t n) {
     return p && pi_memset(p, 0, n * 2) == PI_OK ? p : nullptr;
 }
 
+// a vector of n floats
+int vec(pi_model * m, int il, int kind, int64_t n, const char * what, const float ** out) {
+    PI_TRY(want_tensor(m->L(il, kind), PI_TYPE_F32, n, 1, what));
+    *out = (const float *)m->L(il, kind).dev;
+    return PI_OK;
+}
+
 // A layer with one norm: everything that reads the normed input is one matrix - the mixer's projections, gate and up rows of the dense or
 // shared feed-forward (in turn), its score row, the router - and what closes the layer is one as well, [W_o | W_down].
 int one_norm_weights(pi_model * m, int il) {
@@ -195,17 +220,18 @@ int one_norm_weights(pi_model * m, int il) {
         return place(m, m->L(il, kind), z, s->d_ld, 0, s->d_ld, off, step);
     };
     PI_TRY(rows(PI_T_MIX_Q, (int64_t)d.n_head * d.dim, 0, 1, "mix_q"));
-    PI_TRY(rows(PI_T_MIX_K, (int64_t)(d.mixer == PI_MIXER_GROUPED ? d.n_kv_head : d.n_head) * d.dim, L.off_k, 1, "mix_k"));
-    if (L.off_v != L.off_k) PI_TRY(rows(PI_T_MIX_V, (int64_t)(d.mixer == PI_MIXER_GROUPED ? d.n_kv_head : d.n_head) * d.vdim, L.off_v, 1, "mix_v"));
-    if (d.mixer == PI_MIXER_LINEAR) {
-        PI_TRY(rows(PI_T_MIX_G, hv, L.off_g, 1, "mix_g"));
-        PI_TRY(want_tensor(m->L(il, PI_T_MIX_NORM), PI_TYPE_F32, hv, 1, "mix_norm"));
-        PI_TRY(want_tensor(m->L(il, PI_T_MIX_DECAY), PI_TYPE_F32, d.n_head, 1, "mix_decay"));
-        L.mix_norm = (const float *)m->L(il, PI_T_MIX_NORM).dev;
-        L.decay = (const float *)m->L(il, PI_T_MIX_DECAY).dev;
+    const bool grouped = d.mixer == PI_MIXER_GROUPED;
+    const int64_t n_kv = grouped ? d.n_kv_head : d.n_head;
+    PI_TRY(rows(PI_T_MIX_K, n_kv * d.dim, grouped ? L.off_k : L.rec.off_k, 1, "mix_k"));
+    if (!grouped || L.off_v != L.off_k) PI_TRY(rows(PI_T_MIX_V, n_kv * d.vdim, grouped ? L.off_v : L.rec.off_v, 1, "mix_v"));
+    if (L.rec.on()) {
+        Rec & r = L.rec;
+        PI_TRY(rows(PI_T_MIX_G, hv, r.off_g, 1, "mix_g"));
+        PI_TRY(vec(m, il, PI_T_MIX_NORM, hv, "mix_norm", &r.norm));
+        PI_TRY(vec(m, il, PI_T_MIX_DECAY, d.n_head, "mix_decay", &r.decay));
         const int C = pi_k_linear_chunk();
         std::vector<float> dec(d.n_head), pw((size_t)d.n_head * (C + 1));
-        PI_TRY(pi_memcpy_d2h(dec.data(), L.decay, sizeof(float) * dec.size()));
+        PI_TRY(pi_memcpy_d2h(dec.data(), r.decay, sizeof(float) * dec.size()));
         for (int h = 0; h < d.n_head; ++h) {
             double v = 1.0;
             for (int k = 0; k <= C; ++k, v *= dec[h]) pw[(size_t)h * (C + 1) + k] = (float)v;
@@ -213,7 +239,7 @@ int one_norm_weights(pi_model * m, int il) {
         float * p = m->alloc<float>(pw.size());
         if (!p) return PI_E_HIP;
         PI_TRY(pi_memcpy_h2d(p, pw.data(), sizeof(float) * pw.size()));
-        L.powers = p;
+        r.powers = p;
     }
     uint16_t * close = zeroed(m, (size_t)D * L.close_ld);
     if (!close) return PI_E_HIP;
@@ -251,10 +277,10 @@ void one_norm_sizes(Layer & L) {
         L.off_k = take(d.n_kv_head * d.dim);
         L.off_v = d.values_are_keys ? L.off_k : take(d.n_kv_head * d.vdim);
     } else {
-        L.off_k = take(d.n_head * d.dim);
-        L.off_v = take(d.n_head * d.vdim);
-        L.off_g = take(d.n_head * d.vdim);
-        L.dim_ld = up_to(d.dim, 32); L.vdim_ld = up_to(d.vdim, 64);
+        Rec & r = L.rec;
+        r.off_k = take(d.n_head * d.dim);
+        r.off_v = take(d.n_head * d.vdim);
+        r.off_g = take(d.n_head * d.vdim);
     }
     if (d.glu_ff > 0) {
         L.off_glu = take(2 * d.glu_ff);
@@ -264,6 +290,125 @@ void one_norm_sizes(Layer & L) {
     L.z_rows = at;
     L.hv_ld = up_to(d.n_head * d.vdim, 128); L.glu_ld = d.glu_ff > 0 ? up_to(d.glu_ff, 128) : 0; L.close_ld = L.hv_ld + L.glu_ld;
     L.ff_ld = d.ffn == PI_FFN_GLU_MOE ? up_to(d.expert_ff, 64) : 0;
+}
+
+// A layer whose norms come after the sums: what the mixer projects and the gate of its residual are one matrix, what closes the mixer is one
+// ([W_o | W_o of the memory]), gate and up rows of the feed-forward and the gate of its residual are one.
+int post_norm_weights(pi_model * m, int il) {
+    LayerState * s = m->lay;
+    Layer & L = s->layers[il];
+    const pi_layer_desc & d = L.d;
+    Rec & r = L.rec;
+    const int D = m->hp.n_embd, hv = d.n_head * d.vdim;
+    const auto want = [&](int kind, int64_t ne0, int64_t ne1, const char * what) { return want_tensor(m->L(il, kind), PI_TYPE_BF16, ne0, ne1, what); };
+    PI_TRY(want_tensor(m->L(il, PI_T_ATTN_NORM), PI_TYPE_F32, D, 1, "attn_norm"));
+    PI_TRY(norm_weights(m, m->L(il, PI_T_ATTN_NORM), s->opts.norm_offset, 1.0f, &L.norm_a));
+    uint16_t * z = zeroed(m, (size_t)L.z_rows * s->d_ld), * close = zeroed(m, (size_t)D * L.close_ld);
+    if (!z || !close) return PI_E_HIP;
+    L.w_z = z; L.wo = close;
+    const auto rows = [&](uint16_t * to, int kind, int64_t n, int off, int step, const char * what) -> int {
+        PI_TRY(want(kind, D, n, what));
+        return place(m, m->L(il, kind), to, s->d_ld, 0, s->d_ld, off, step);
+    };
+    const bool grouped = d.mixer == PI_MIXER_GROUPED;
+    PI_TRY(rows(z, PI_T_MIX_Q, (int64_t)d.n_head * d.dim, 0, 1, "mix_q"));
+    if (grouped) {
+        PI_TRY(rows(z, PI_T_MIX_K, (int64_t)d.n_kv_head * d.dim, L.off_k, 1, "mix_k"));
+        if (L.off_v != L.off_k) PI_TRY(rows(z, PI_T_MIX_V, (int64_t)d.n_kv_head * d.vdim, L.off_v, 1, "mix_v"));
+        if (d.qk_norm) { PI_TRY(vec(m, il, PI_T_MIX_Q_NORM, d.dim, "mix_q_norm", &L.q_norm)); PI_TRY(vec(m, il, PI_T_MIX_K_NORM, d.dim, "mix_k_norm", &L.k_norm)); }
+        if (d.head_temp) PI_TRY(vec(m, il, PI_T_MIX_TEMP, d.n_head, "mix_temp", &L.temp));
+    } else {
+        PI_TRY(rows(z, PI_T_MIX_K, (int64_t)d.n_head * d.dim, r.off_k, 1, "mix_k"));
+        PI_TRY(rows(z, PI_T_MIX_V, hv, r.off_v, 1, "mix_v"));
+        PI_TRY(rows(z, PI_T_MIX_G, hv, r.off_g, 1, "mix_g"));
+        PI_TRY(rows(z, PI_T_MIX_A1, r.rank, r.off_a, 1, "mix_a1"));
+        PI_TRY(want(PI_T_MIX_A2, r.rank, (int64_t)d.n_head * d.dim, "mix_a2"));
+        PI_TRY(padded(m, m->L(il, PI_T_MIX_A2), r.rank_ld, &r.a2));
+        PI_TRY(vec(m, il, PI_T_MIX_A2_B, (int64_t)d.n_head * d.dim, "mix_a2_b", &r.a2_b));
+        PI_TRY(vec(m, il, PI_T_MIX_NORM, hv, "mix_norm", &r.norm));
+    }
+    PI_TRY(want(PI_T_WO, hv, D, "wo"));
+    PI_TRY(place(m, m->L(il, PI_T_WO), close, L.close_ld, 0, L.hv_ld, 0, 1));
+    if (grouped && r.on()) {
+        const int64_t hk = (int64_t)r.n_head * r.dim, mv = (int64_t)r.n_head * r.vdim;
+        PI_TRY(rows(z, PI_T_MEM_Q, hk, r.off_q, 1, "mem_q"));
+        PI_TRY(rows(z, PI_T_MEM_K, hk, r.off_k, 1, "mem_k"));
+        PI_TRY(rows(z, PI_T_MEM_V, mv, r.off_v, 1, "mem_v"));
+        PI_TRY(rows(z, PI_T_MEM_G, mv, r.off_g, 1, "mem_g"));
+        PI_TRY(rows(z, PI_T_MEM_I, r.n_head, r.off_i, 1, "mem_i"));
+        PI_TRY(rows(z, PI_T_MEM_F, r.n_head, r.off_f, 1, "mem_f"));
+        PI_TRY(vec(m, il, PI_T_MEM_I_B, r.n_head, "mem_i_b", &r.i_b));
+        PI_TRY(vec(m, il, PI_T_MEM_F_B, r.n_head, "mem_f_b", &r.f_b));
+        PI_TRY(vec(m, il, PI_T_MEM_NORM, mv, "mem_norm", &r.norm));
+        PI_TRY(want(PI_T_MEM_O, mv, D, "mem_o"));
+        PI_TRY(place(m, m->L(il, PI_T_MEM_O), close, L.close_ld, r.off_att, L.close_ld - r.off_att, 0, 1));
+    }
+    if (d.gated_residual) {
+        PI_TRY(rows(z, PI_T_RES_GATE, D, L.off_gate, 1, "res_gate"));
+        PI_TRY(vec(m, il, PI_T_RES_GATE_B, D, "res_gate_b", &L.gate_b));
+    }
+    if (d.ffn == PI_FFN_NONE) return PI_OK;
+    PI_TRY(want_tensor(m->L(il, PI_T_FFN_NORM), PI_TYPE_F32, D, 1, "ffn_norm"));
+    PI_TRY(norm_weights(m, m->L(il, PI_T_FFN_NORM), s->opts.norm_offset, 1.0f, &L.norm_b));
+    uint16_t * f = zeroed(m, (size_t)L.z2_rows * s->d_ld);
+    if (!f) return PI_E_HIP;
+    L.w_ffn = f;
+    PI_TRY(rows(f, PI_T_GLU_GATE, d.glu_ff, 0, 2, "glu_gate"));
+    PI_TRY(rows(f, PI_T_GLU_UP, d.glu_ff, 1, 2, "glu_up"));
+    if (d.gated_residual) {
+        PI_TRY(rows(f, PI_T_RES_GATE_FFN, D, L.off_gate_ffn, 1, "res_gate_ffn"));
+        PI_TRY(vec(m, il, PI_T_RES_GATE_FFN_B, D, "res_gate_ffn_b", &L.gate_ffn_b));
+    }
+    PI_TRY(want(PI_T_GLU_DOWN, d.glu_ff, D, "glu_down"));
+    return padded(m, m->L(il, PI_T_GLU_DOWN), L.glu_ld, &L.down);
+}
+
+void post_norm_sizes(Layer & L, int D) {
+    const pi_layer_desc & d = L.d;
+    Rec & r = L.rec;
+    int at = 0;
+    const auto take = [&](int n) { const int o = at; at = up_to(at + n, 16); return o; };
+    take(d.n_head * d.dim);
+    L.hv_ld = up_to(d.n_head * d.vdim, 128); L.close_ld = L.hv_ld;
+    if (d.mixer == PI_MIXER_GROUPED) {
+        L.off_k = take(d.n_kv_head * d.dim);
+        L.off_v = d.values_are_keys ? L.off_k : take(d.n_kv_head * d.vdim);
+        if (r.on()) r.off_q = take(r.n_head * r.dim);
+        r.off_att = L.hv_ld;
+        if (r.on()) L.close_ld += up_to(r.n_head * r.vdim, 128);
+    }
+    if (r.on()) {
+        r.off_k = take(r.n_head * r.dim);
+        r.off_v = take(r.n_head * r.vdim);
+        r.off_g = take(r.n_head * r.vdim);
+        if (r.kind == PI_DECAY_KEYED) r.off_a = take(r.rank);
+        else { r.off_i = take(r.n_head); r.off_f = take(r.n_head); }
+    }
+    if (d.gated_residual) L.off_gate = take(D);
+    L.z_rows = at;
+    if (d.ffn == PI_FFN_NONE) return;
+    L.off_gate_ffn = up_to(2 * d.glu_ff, 16);
+    L.z2_rows = L.off_gate_ffn + (d.gated_residual ? up_to(D, 16) : 0);
+    L.glu_ld = up_to(d.glu_ff, 128);
+}
+
+// the recurrent part that a description asks for
+Rec recurrent_part(const pi_layer_desc & d) {
+    Rec r;
+    if (d.mixer == PI_MIXER_LINEAR || d.mixer == PI_MIXER_KEYED) { r.n_head = d.n_head; r.dim = d.dim; r.vdim = d.vdim; }
+    if (d.mixer == PI_MIXER_LINEAR) r.kind = PI_DECAY_CONST;
+    if (d.mixer == PI_MIXER_KEYED) {
+        r.kind = PI_DECAY_KEYED;
+        r.rank = d.decay_rank; r.rank_ld = up_to(d.decay_rank, 8); r.tau = d.decay_tau; r.silu = true;
+    }
+    if (d.mixer == PI_MIXER_GROUPED && d.mem_heads > 0) {
+        r.kind = PI_DECAY_GATED;
+        r.n_head = d.mem_heads; r.dim = d.mem_dim; r.vdim = d.mem_vdim; r.cap = d.mem_cap; r.scale = d.mem_scale;
+    }
+    r.plain = r.per_head = r.kind > PI_DECAY_CONST;
+    if (r.plain) r.q_scale = 1.0f / sqrtf((float)r.dim);
+    r.dim_ld = up_to(r.dim, 32); r.vdim_ld = up_to(r.vdim, 64);
+    return r;
 }
 
 int layer_weights(pi_model * m, int il) {
@@ -325,18 +470,21 @@ int ensure_capacity(pi_model * m, int T) {
     int cap = 64;
     while (cap < T) cap *= 2;
     const size_t es = s->es, D = m->hp.n_embd;
-    size_t z = 0, qu = 0, ql = 0, ol = 0, at = 0, E = 0, top = 0, ff = 0, lq = 0, lv = 0, lo = 0, ls = 0;
+    size_t z = 0, qu = 0, ql = 0, ol = 0, at = 0, E = 0, top = 0, ff = 0, lq = 0, lv = 0, lo = 0, ls = 0, ln = 0, lg = 0;
     const size_t chunks = s->recurrent && bf16_mode(s) ? (size_t)cap / pi_k_linear_chunk() + 32 : 0;        // every run of a pass ends with a part of one
     for (const Layer & L : s->layers) {
         const pi_layer_desc & d = L.d;
-        if (s->one_norm) {
-            z = std::max(z, (size_t)L.z_rows); at = std::max(at, (size_t)L.close_ld);
+        if (s->family != kTwoNorms) {
+            z = std::max({z, (size_t)L.z_rows, (size_t)L.z2_rows}); at = std::max({at, (size_t)L.close_ld, (size_t)L.glu_ld});
             if (d.mixer == PI_MIXER_GROUPED) ql = std::max(ql, (size_t)d.n_head * L.hd);
-            else {
-                lo = std::max(lo, (size_t)d.n_head * d.vdim);
+            const Rec & r = L.rec;
+            if (r.on()) {
+                lo = std::max(lo, (size_t)r.n_head * r.vdim);
+                if (r.kind == PI_DECAY_GATED) ln = std::max(ln, (size_t)r.n_head);
                 if (chunks) {
-                    lq = std::max(lq, (size_t)d.n_head * L.dim_ld); lv = std::max(lv, (size_t)d.n_head * L.vdim_ld);
-                    ls = std::max(ls, pi_k_linear_states_bytes((int)chunks, d.n_head, L.dim_ld, L.vdim_ld));
+                    lq = std::max(lq, (size_t)r.n_head * r.dim_ld); lv = std::max(lv, (size_t)r.n_head * r.vdim_ld);
+                    ls = std::max(ls, pi_k_linear_states_bytes((int)chunks, r.n_head, r.dim_ld, r.vdim_ld));
+                    lg = std::max(lg, pi_k_linear_gate_floats(r.kind, cap, (int)chunks, r.n_head, r.dim_ld));
                 }
             }
             if (L.moe()) { E = std::max(E, (size_t)d.n_expert); top = std::max(top, (size_t)d.n_top); ff = std::max(ff, (size_t)d.n_top * L.ff_ld); }
@@ -367,6 +515,7 @@ int ensure_capacity(pi_model * m, int T) {
         carve(s->tiles, (n * top / 64 + E + 1) * 8); carve(s->n_tiles, 4);
         carve(s->x0, s->opts.loop_times > 0 ? n * D * 4 : 0);
         carve(s->lin_o, n * lo * 4); carve(s->lin_q, n * lq * 2); carve(s->lin_k, n * lq * 2); carve(s->lin_v, n * lv * 2); carve(s->lin_states, ls);
+        carve(s->lin_den, n * ln * 4); carve(s->lin_gates, lg * 4);
         s->cs.resize(s->rots.size());
         for (size_t r = 0; r < s->rots.size(); ++r) carve(s->cs[r], n * s->rots[r].dims * 4);
     };
@@ -548,18 +697,70 @@ pi_gqa_attn gqa_args(pi_model * m, const Layer & L, int pass, const Step & in, c
     pi_gqa_attn a{};
     a.q = s->q_lat; a.cache = L.cache[pass]; a.lists = s->lists; a.list_ld = s->kv.n; a.work = bf16_mode(s) ? w.items : in.seq; a.n_vis = in.n_vis; a.n_work = w.n; a.T = in.T;
     a.n_head = d.n_head; a.n_kv = d.n_kv_head; a.dim = d.dim; a.vdim = d.vdim; a.hd = L.hd; a.n_parts = w.parts; a.wide = wide; a.scale = d.scale; a.sink = d.sink;
-    a.scratch = s->scratch; a.att = s->att; a.ld_att = L.close_ld;
+    a.scratch = s->scratch; a.att = s->att; a.ld_att = L.close_ld; a.out_scale = s->family == kPostNorm ? d.out_scale : 1.0f; a.window = d.window; a.first = in.first[L.hc];
     return a;
+}
+
+pi_gqa_prep gqa_prep_args(pi_model * m, const Layer & L, int pass, const Step & in) {
+    LayerState * s = m->lay;
+    const pi_layer_desc & d = L.d;
+    pi_gqa_prep p{};
+    p.z = s->z; p.ldz = L.z_rows; p.T = in.T; p.n_head = d.n_head; p.n_kv = d.n_kv_head; p.dim = d.dim; p.vdim = d.vdim; p.rot_dim = d.rot_dim; p.off_k = L.off_k; p.off_v = L.off_v;
+    p.hd = L.hd; p.unit = d.unit_qk; p.cs = L.rot >= 0 ? s->cs[L.rot] : s->x; p.eps = m->hp.norm_eps; p.q = s->q_lat; p.cache = L.cache[pass]; p.cell = in.cell;
+    p.rot_pairs = d.rot_pairs; p.unit_v = d.unit_v; p.q_norm = L.q_norm; p.k_norm = L.k_norm; p.temp = L.temp;
+    return p;
+}
+
+// step: the parts of a split attention stay unmerged (parts says which)
+int attend_grouped(pi_model * m, const Layer & L, int pass, const Step & in, bool step, pi_gqa_attn & parts) {
+    LayerState * s = m->lay;
+    const int type = s->opts.compute;
+    if (bf16_mode(s) && in.wide[L.hc].n > 0) {
+        const pi_gqa_attn a = gqa_args(m, L, pass, in, in.wide[L.hc], 1);
+        PI_TRY(pi_k_gqa_attn(type, &a, m->stream));
+    }
+    if (in.work[L.hc].n == 0) return PI_OK;
+    const pi_gqa_attn a = gqa_args(m, L, pass, in, in.work[L.hc], 0);
+    if (!step) return pi_k_gqa_attn(type, &a, m->stream);
+    if (a.n_parts > 1) parts = a;
+    return pi_k_gqa_attn_parts(&a, m->stream);
 }
 
 pi_linear linear_args(pi_model * m, const Layer & L, int pass, const Step & in) {
     LayerState * s = m->lay;
-    const pi_layer_desc & d = L.d;
+    const Rec & r = L.rec;
     pi_linear p{};
-    p.z = s->z; p.ldz = L.z_rows; p.T = in.T; p.n_head = d.n_head; p.dim = d.dim; p.vdim = d.vdim; p.off_k = L.off_k; p.off_v = L.off_v; p.decay = L.decay; p.powers = L.powers;
+    p.z = s->z; p.ldz = L.z_rows; p.T = in.T; p.n_head = r.n_head; p.dim = r.dim; p.vdim = r.vdim; p.off_q = r.off_q; p.off_k = r.off_k; p.off_v = r.off_v; p.decay = r.decay; p.powers = r.powers;
     p.state = L.state[pass]; p.runs = in.lin; p.n_runs = in.n_lin; p.o = s->lin_o; p.q = s->lin_q; p.k = s->lin_k; p.v = s->lin_v; p.states = s->lin_states;
-    p.dim_ld = L.dim_ld; p.vdim_ld = L.vdim_ld;
+    p.dim_ld = r.dim_ld; p.vdim_ld = r.vdim_ld; p.decay_kind = r.kind; p.plain = r.plain; p.q_scale = r.q_scale; p.slot_ld = L.state_floats();
+    p.a2 = r.a2; p.a2_b = r.a2_b; p.off_a = r.off_a; p.rank = r.rank; p.rank_ld = r.rank_ld; p.tau = r.tau;
+    p.i_b = r.i_b; p.f_b = r.f_b; p.off_i = r.off_i; p.off_f = r.off_f; p.cap = r.cap; p.den = s->lin_den; p.gates = s->lin_gates;
+    p.n_chunks = in.n_lin_chunks; p.chunks = in.lin_chunks; p.first_chunk = in.lin_first;
     return p;
+}
+
+// the recurrent part of a mixer, short runs token by token and long ones in chunks; front or beside in a launch of it where there is one
+int recur(pi_model * m, const Layer & L, int pass, const Step & in, const pi_ffn_front * front, const pi_gqa_prep * beside) {
+    LayerState * s = m->lay;
+    const int type = s->opts.compute;
+    hipStream_t st = m->stream;
+    pi_linear p = linear_args(m, L, pass, in);
+    if (in.n_lin_long == 0) return beside ? pi_k_linear_step_beside(type, &p, beside, st) : pi_k_linear_step(type, &p, front, st);
+    PI_TRY(pi_k_linear_prep(type, &p, front, st));
+    if (beside) PI_TRY(pi_k_gqa_prep(type, beside, nullptr, st));
+    if (in.n_lin > 0) PI_TRY(pi_k_linear_step(type, &p, nullptr, st));
+    p.runs = in.lin_long; p.n_runs = in.n_lin_long;
+    return pi_k_linear_chunks(&p, st);
+}
+
+pi_gate_norm gate_norm_args(pi_model * m, const Layer & L, int T) {
+    LayerState * s = m->lay;
+    const Rec & r = L.rec;
+    pi_gate_norm g{};
+    g.o = s->lin_o; g.z = s->z; g.w = r.norm; g.ldz = L.z_rows; g.off_gate = r.off_g; g.n = r.n_head * r.vdim; g.T = T; g.eps = m->hp.norm_eps;
+    g.att = (unsigned char *)s->att + (size_t)r.off_att * s->es; g.ld_att = L.close_ld; g.scale = r.scale; g.heads = r.per_head ? r.n_head : 0; g.silu = r.silu;
+    g.den = r.kind == PI_DECAY_GATED ? s->lin_den : nullptr;
+    return g;
 }
 
 // A layer with one norm.  Steps of up to 16 tokens (bf16): norm, joint projection, what lies behind it (queries and cells or the state's step,
@@ -582,31 +783,13 @@ int one_norm_layer(pi_model * m, Layer & L, const LayerRun & r, const Step & in,
     pi_gqa_attn parts{};
     pi_gate_norm gate{};
     if (linear) {
-        pi_linear p = linear_args(m, L, r.pass, in);
-        if (in.n_lin_long == 0) PI_TRY(pi_k_linear_step(type, &p, &f, st));
-        else {
-            PI_TRY(pi_k_linear_prep(type, &p, &f, st));
-            if (in.n_lin > 0) PI_TRY(pi_k_linear_step(type, &p, nullptr, st));
-            p.runs = in.lin_long; p.n_runs = in.n_lin_long; p.chunks = in.lin_chunks; p.n_chunks = in.n_lin_chunks; p.first_chunk = in.lin_first;
-            PI_TRY(pi_k_linear_chunks(&p, st));
-        }
-        gate.o = s->lin_o; gate.z = s->z; gate.w = L.mix_norm; gate.ldz = L.z_rows; gate.off_gate = L.off_g; gate.n = d.n_head * d.vdim; gate.T = T; gate.eps = m->hp.norm_eps;
-        gate.att = s->att; gate.ld_att = L.close_ld;
+        PI_TRY(recur(m, L, r.pass, in, &f, nullptr));
+        gate = gate_norm_args(m, L, T);
         if (!step) PI_TRY(pi_k_gate_norm(type, &gate, st));
     } else {
-        pi_gqa_prep p{};
-        p.z = s->z; p.ldz = L.z_rows; p.T = T; p.n_head = d.n_head; p.n_kv = d.n_kv_head; p.dim = d.dim; p.vdim = d.vdim; p.rot_dim = d.rot_dim; p.off_k = L.off_k; p.off_v = L.off_v;
-        p.hd = L.hd; p.unit = d.unit_qk; p.cs = L.rot >= 0 ? s->cs[L.rot] : s->x; p.eps = m->hp.norm_eps; p.q = s->q_lat; p.cache = L.cache[r.pass]; p.cell = in.cell;
+        const pi_gqa_prep p = gqa_prep_args(m, L, r.pass, in);
         PI_TRY(pi_k_gqa_prep(type, &p, &f, st));
-        if (bf16_mode(s) && in.wide[L.hc].n > 0) {
-            const pi_gqa_attn a = gqa_args(m, L, r.pass, in, in.wide[L.hc], 1);
-            PI_TRY(pi_k_gqa_attn(type, &a, st));
-        }
-        if (in.work[L.hc].n > 0) {
-            const pi_gqa_attn a = gqa_args(m, L, r.pass, in, in.work[L.hc], 0);
-            if (step) { PI_TRY(pi_k_gqa_attn_parts(&a, st)); if (a.n_parts > 1) parts = a; }
-            else PI_TRY(pi_k_gqa_attn(type, &a, st));
-        }
+        PI_TRY(attend_grouped(m, L, r.pass, in, step, parts));
     }
     if (step) {
         if (moe || linear || parts.n_parts > 1)
@@ -620,6 +803,61 @@ int one_norm_layer(pi_model * m, Layer & L, const LayerRun & r, const Step & in,
     PI_TRY(dense(m, L.wo, D, L.close_ld, s->att, T, s->mix));
     if (moe) PI_TRY(experts(m, L, s->h_a, in));
     return pi_k_moe_combine(type, s->x, s->mix, s->y_exp, s->inv, moe ? s->wts : nullptr, moe ? d.n_top : 0, T, D, s->x2, keep, st);
+}
+
+// A layer whose norms come after the sums.  Steps of up to 16 tokens (bf16): joint projection, what lies behind it (queries and cells beside the
+// state's step), attention, merge and gated norm, the mixer's closing product with the gated sum, norm; gate and up rows with their
+// GLU beside the second residual gate, closing product with the gated sum, norm.
+int post_norm_layer(pi_model * m, Layer & L, const LayerRun & r, const Step & in, float * keep) {
+    LayerState * s = m->lay;
+    const pi_layer_desc & d = L.d;
+    const int T = in.T, D = m->hp.n_embd, type = s->opts.compute;
+    const bool step = bf16_mode(s) && pi_k_layer_step_supported(T, 0, 0), grouped = d.mixer == PI_MIXER_GROUPED;
+    hipStream_t st = m->stream;
+    if (step) PI_TRY(pi_k_gemm_bf16_ol(L.w_z, L.z_rows, s->d_ld, s->h_a, T, PI_EPI_NONE, nullptr, nullptr, s->z, nullptr, st));
+    else PI_TRY(dense(m, L.w_z, L.z_rows, s->d_ld, s->h_a, T, s->z));
+    pi_gqa_attn parts{};
+    if (grouped) {
+        const pi_gqa_prep p = gqa_prep_args(m, L, r.pass, in);
+        if (L.rec.on()) PI_TRY(recur(m, L, r.pass, in, nullptr, &p));
+        else PI_TRY(pi_k_gqa_prep(type, &p, nullptr, st));
+        PI_TRY(attend_grouped(m, L, r.pass, in, step, parts));
+    } else PI_TRY(recur(m, L, r.pass, in, nullptr, nullptr));
+    const pi_gate_norm gate = L.rec.on() ? gate_norm_args(m, L, T) : pi_gate_norm{};
+    if (step) {
+        if (L.rec.on() || parts.n_parts > 1)
+            PI_TRY(pi_k_mix_up_step(parts.n_parts > 1 ? &parts : nullptr, L.rec.on() ? &gate : nullptr, nullptr, 0, 0, 0, 0.0f, 0.0f, nullptr, T, nullptr, nullptr, 0, nullptr, 0, st));
+    } else if (L.rec.on()) PI_TRY(pi_k_gate_norm(type, &gate, st));
+    // x = norm(alpha x + gate * W att), with the next product's operand
+    const auto close = [&](const void * W, int ld, const float * gz, int ld_gate, int off_gate, const float * gb, const float * w, float * kept) -> int {
+        pi_res_norm n{};
+        n.w = w; n.T = T; n.cols = D; n.alpha = s->opts.residual_alpha; n.eps = m->hp.norm_eps; n.out = s->x; n.keep = kept; n.h = s->h_a; n.ld = s->d_ld; n.ol = step;
+        if (step) {
+            pi_layer_out o{};
+            o.x = s->x; o.wo = W; o.att = s->att; o.rows = D; o.ld_att = ld; o.T = T; o.out = s->x2; o.scaled = 1; o.alpha = n.alpha;
+            o.gate_z = gz; o.ld_gate = ld_gate; o.off_gate = off_gate; o.gate_b = gb;
+            PI_TRY(pi_k_layer_out_step(&o, st));
+            n.x = s->x2;
+        } else {
+            PI_TRY(dense(m, W, D, ld, s->att, T, s->mix));
+            n.x = s->x; n.mix = s->mix; n.gate_z = gz; n.ld_gate = ld_gate; n.off_gate = off_gate; n.gate_b = gb;
+        }
+        return pi_k_res_norm(type, &n, st);
+    };
+    const bool gated = d.gated_residual != 0, ffn = d.ffn == PI_FFN_GLU;
+    PI_TRY(close(L.wo, L.close_ld, gated ? s->z : nullptr, L.z_rows, L.off_gate, L.gate_b, L.norm_a, ffn ? nullptr : keep));
+    if (!ffn) return PI_OK;
+    if (step) {
+        const uint16_t * W = (const uint16_t *)L.w_ffn;
+        PI_TRY(pi_k_gemm_bf16_ol_glu(W, d.glu_ff, s->h_a, d.glu_limit, d.glu_gain, d.glu_plain_up ? 0.0f : 1.0f, s->att, L.glu_ld, gated ? W + (size_t)L.off_gate_ffn * s->d_ld : nullptr, D,
+                                     s->z, s->d_ld, T, st));
+        return close(L.down, L.glu_ld, gated ? s->z : nullptr, D, 0, L.gate_ffn_b, L.norm_b, keep);
+    }
+    PI_TRY(dense(m, L.w_ffn, L.z2_rows, s->d_ld, s->h_a, T, s->z));
+    pi_ffn_front f{};
+    f.ff = d.glu_ff; f.ff_ld = L.glu_ld; f.off_score = -1; f.limit = d.glu_limit; f.gain = d.glu_gain; f.plain_up = d.glu_plain_up; f.act = s->att; f.ld_act = L.glu_ld;
+    PI_TRY(pi_k_ffn_front(type, s->z, L.z2_rows, T, &f, st));
+    return close(L.down, L.glu_ld, gated ? s->z : nullptr, L.z2_rows, L.off_gate_ffn, L.gate_ffn_b, L.norm_b, keep);
 }
 
 // a layer of a step of up to 16 tokens (bf16): six launches
@@ -648,15 +886,24 @@ int pass_layers(pi_model * m, const Step & in) {
     LayerState * s = m->lay;
     const int type = s->opts.compute, T = in.T, D = m->hp.n_embd;
     hipStream_t st = m->stream;
-    if (s->one_norm) PI_TRY(pi_k_embed_bigram(s->embed, D, in.tokens, in.prev, T, s->opts.embed_scale, s->bigram, s->opts.bigram_buckets, s->opts.bigram_mul_prev, s->opts.bigram_mul_cur,
+    if (s->family != kTwoNorms) PI_TRY(pi_k_embed_bigram(s->embed, D, in.tokens, in.prev, T, s->opts.embed_scale, s->bigram, s->opts.bigram_buckets, s->opts.bigram_mul_prev, s->opts.bigram_mul_cur,
                                               in.carry, s->x, s->opts.loop_times > 0 ? s->x0 : nullptr, st));
     else PI_TRY(pi_k_embed_norm(s->embed, D, in.tokens, T, s->embd_norm, m->hp.norm_eps, s->x, st));
+    if (s->family == kPostNorm) {                      // the first product's operand
+        pi_res_norm n{};
+        n.x = n.out = s->x; n.T = T; n.cols = D; n.h = s->h_a; n.ld = s->d_ld; n.ol = bf16_mode(s) && pi_k_layer_step_supported(T, 0, 0);
+        PI_TRY(pi_k_res_norm(type, &n, st));
+    }
     for (size_t r = 0; r < s->rots.size(); ++r) PI_TRY(pi_k_rope_angles(in.pos, T, s->rots[r].dims, s->rots[r].base, s->cs[r], st));
     for (size_t k = 0; k < s->order.size(); ++k) {
         Layer & L = s->layers[s->order[k].layer];
         const bool moe = L.moe();
         float * keep = s->streams_T ? s->streams + k * (size_t)s->streams_T * D : nullptr;
-        if (s->one_norm) {
+        if (s->family == kPostNorm) {
+            PI_TRY(post_norm_layer(m, L, s->order[k], in, keep));
+            continue;
+        }
+        if (s->family == kOneNorm) {
             PI_TRY(one_norm_layer(m, L, s->order[k], in, keep));
             std::swap(s->x, s->x2);
             continue;
@@ -680,7 +927,7 @@ int pass_head(pi_model * m, const int32_t * rows, int n) {
     LayerState * s = m->lay;
     const int D = m->hp.n_embd;
     const bool ol = bf16_mode(s) && n <= 16;
-    if (s->one_norm) PI_TRY(pi_k_layer_norm(s->opts.compute, s->x, rows, n, D, m->hp.norm_eps, s->out_norm, nullptr, nullptr, s->h_head, s->d_ld, ol, m->stream));
+    if (s->family == kOneNorm) PI_TRY(pi_k_layer_norm(s->opts.compute, s->x, rows, n, D, m->hp.norm_eps, s->out_norm, nullptr, nullptr, s->h_head, s->d_ld, ol, m->stream));
     else PI_TRY(pi_k_norm_pair(s->opts.compute, s->x, rows, n, D, m->hp.norm_eps, s->out_norm, s->h_head, nullptr, nullptr, s->d_ld, ol, m->stream));
     if (ol) return pi_k_gemm_bf16_ol(s->head, m->hp.n_vocab, s->d_ld, s->h_head, n, PI_EPI_NONE, nullptr, nullptr, s->logits, nullptr, m->stream);
     return dense(m, s->head, m->hp.n_vocab, s->d_ld, s->h_head, n, s->logits);
@@ -730,6 +977,8 @@ void gqa_items(const int32_t * seq, const int32_t * n_vis, int n, int per, std::
     }
 }
 
+// span: the most cells a work item sees
+int gqa_span(const HeadKind & h, int n_vis_max, bool wide) { return h.window > 0 ? std::min(n_vis_max, h.window + pi_k_gqa_rows(wide)) : n_vis_max; }
 int gqa_parts(int n_groups, int n_vis_max, int cells) { return n_groups <= 0 ? 1 : std::max(1, std::min({kAttnItems / n_groups, (n_vis_max + cells - 1) / cells, 64})); }
 
 // how many workgroups share one work item's cells
@@ -780,7 +1029,7 @@ int apply_shift(pi_model * m) {
     PI_TRY(pi_memcpy_h2d(s->d_delta, s->kv.delta.data(), sizeof(int32_t) * s->kv.n));
     for (Layer & L : s->layers) {
         if (L.d.mixer == PI_MIXER_GROUPED)
-            for (void * c : L.cache) PI_TRY(pi_k_gqa_shift(s->opts.compute, c, s->kv.n, L.d.n_kv_head, L.hd, L.d.rot_dim, L.d.rot_base, s->d_delta, m->stream));
+            for (void * c : L.cache) PI_TRY(pi_k_gqa_shift(s->opts.compute, c, s->kv.n, L.d.n_kv_head, L.hd, L.d.rot_dim, L.d.rot_base, L.d.rot_pairs, s->d_delta, m->stream));
         else if (L.cell_values()) PI_TRY(pi_k_latent_shift(s->opts.compute, L.cache[0], s->kv.n, L.kd, L.rank_ld, L.d.rot_dim, L.d.rot_base, s->d_delta, m->stream));
     }
     PI_HIP_TRY(hipStreamSynchronize(m->stream));
@@ -905,7 +1154,7 @@ int layers_finalize(pi_model * m) {
     PI_TRY(want_tensor(m->glob[PI_T_OUTPUT_NORM], PI_TYPE_F32, D, 1, "output_norm"));
     s->embed = m->glob[PI_T_TOK_EMBD].dev;
     PI_TRY(padded(m, m->glob[PI_T_OUTPUT], s->d_ld, &s->head));
-    if (!s->one_norm) {
+    if (s->family == kTwoNorms) {
         PI_TRY(want_tensor(m->embd_norm, PI_TYPE_F32, D, 1, "embd_norm"));
         PI_TRY(norm_weights(m, m->embd_norm, s->opts.norm_offset, 1.0f, &s->embd_norm));
     }
@@ -934,18 +1183,18 @@ int layers_finalize(pi_model * m) {
             if (h == s->kinds.size()) s->kinds.push_back(hk);
             L.hc = (int)h;
         };
-        if (s->one_norm) {
-            one_norm_sizes(L);
+        if (s->family != kTwoNorms) {
+            if (s->family == kOneNorm) one_norm_sizes(L); else post_norm_sizes(L, D);
             if (d.mixer == PI_MIXER_GROUPED) {
                 L.hd = pi_k_gqa_head_ld(s->opts.compute, d.dim, d.vdim);
                 if (!L.hd) return fail(PI_E_UNSUPPORTED, "pi_model_finalize: head sizes outside the attention kernels (up to 256)");
                 if (d.rot_dim > 0) rotation(); else L.rot = -1;
-                kind(HeadKind{d.mixer, d.n_head / d.n_kv_head, d.n_kv_head, 0, 0, 0, 0, L.hd});
+                kind(HeadKind{d.mixer, d.n_head / d.n_kv_head, d.n_kv_head, 0, 0, 0, 0, L.hd, d.window});
                 scratch = std::max(scratch, pi_k_gqa_scratch_floats(kAttnItems, 1, 1, L.hd, 2) / 2);      // items x groups x parts <= kAttnItems
-            } else if (!pi_k_linear_supported(d.dim, d.vdim)) {
-                return fail(PI_E_UNSUPPORTED, "pi_model_finalize: head sizes outside the linear attention's kernels (up to 256)");
             }
-            PI_TRY(one_norm_weights(m, (int)il));
+            if (L.rec.on() && !pi_k_linear_supported(L.rec.dim, L.rec.vdim)) return fail(PI_E_UNSUPPORTED, "pi_model_finalize: head sizes outside the linear attention's kernels (up to 256)");
+            if (d.weights_of) continue;
+            PI_TRY(s->family == kOneNorm ? one_norm_weights(m, (int)il) : post_norm_weights(m, (int)il));
             continue;
         }
         L.own_kv = d.kv_from < 0;
@@ -955,9 +1204,15 @@ int layers_finalize(pi_model * m) {
         L.hv_ld = up_to(d.n_head * d.vdim, 128); L.ff_ld = d.ffn == PI_FFN_MOE ? up_to(d.expert_ff, 64) : 0;
         if (!pi_k_latent_attn_supported(s->opts.compute, L.rank_ld, L.kd)) return fail(PI_E_UNSUPPORTED, "pi_model_finalize: latent sizes outside the attention kernels (rank up to 1024)");
         rotation();
-        kind(HeadKind{d.mixer, d.n_head, 1, d.dim, d.rot_dim, d.vdim, L.rank_ld, L.kd});
+        kind(HeadKind{d.mixer, d.n_head, 1, d.dim, d.rot_dim, d.vdim, L.rank_ld, L.kd, 0});
         scratch = std::max(scratch, pi_k_latent_attn_scratch_floats(kItemRows * kAttnItems / 2, L.rank_ld, 2));      // items x parts <= kAttnItems
         PI_TRY(layer_weights(m, (int)il));
+    }
+    for (Layer & L : s->layers) {                      // another layer's weights, caches and states of its own
+        if (!L.d.weights_of) continue;
+        Layer own = s->layers[L.d.weights_of - 1];
+        own.cache = L.cache; own.state = L.state;
+        L = own;
     }
     if (bf16_mode(s)) {
         s->scratch = m->alloc<float>(scratch);
@@ -1078,6 +1333,16 @@ int layers_step(pi_model * m, const int32_t * tokens, const int32_t * positions,
             items.insert(items.end(), first.begin(), first.end());
             items.insert(items.end(), chunks.begin(), chunks.end());
         }
+        std::vector<long long> at_first;                          // kinds with a window over positions that are not 0, 1, 2 ..: first cells by position
+        for (const HeadKind & h : s->kinds) {
+            bool gaps = false;
+            for (int t = 0; t < T && h.window > 0; ++t) gaps = gaps || s->list_pos[seq[t0 + t]][vis[t0 + t] - 1] != vis[t0 + t] - 1;
+            at_first.push_back(gaps ? (long long)items.size() : -1);
+            for (int t = 0; t < T && gaps; ++t) {
+                const auto & lp = s->list_pos[seq[t0 + t]];
+                items.push_back((int32_t)(std::upper_bound(lp.begin(), lp.end(), positions[t0 + t] - h.window) - lp.begin()));
+            }
+        }
         const size_t n_in = (size_t)8 * T + items.size() + rows.size();
         PI_TRY(ensure_inputs(m, n_in));
         PI_HIP_TRY(hipStreamSynchronize(m->stream));
@@ -1095,13 +1360,14 @@ int layers_step(pi_model * m, const int32_t * tokens, const int32_t * positions,
             w.items = s->d_in + 8 * T + begin[k];
             w.n = bf16_mode(s) ? (int)(begin[k + 1] - begin[k]) / 4 : T;
             const HeadKind & hk = s->kinds[k];
-            w.parts = hk.mixer == PI_MIXER_GROUPED ? (bf16_mode(s) ? gqa_parts(w.n * hk.n_kv, vmax, 128) : 1) : choose_parts(s, w.n, vmax);
+            w.parts = hk.mixer == PI_MIXER_GROUPED ? (bf16_mode(s) ? gqa_parts(w.n * hk.n_kv, gqa_span(hk, vmax, false), 128) : 1) : choose_parts(s, w.n, vmax);
             in.work.push_back(w);
             Step::Work wd;
             wd.items = s->d_in + 8 * T + begin.back() + begin_wide[k];
             wd.n = (int)(begin_wide[k + 1] - begin_wide[k]) / 4;
-            wd.parts = gqa_parts(wd.n * hk.n_kv, vmax, 512);
+            wd.parts = gqa_parts(wd.n * hk.n_kv, gqa_span(hk, vmax, true), 512);
             in.wide.push_back(wd);
+            in.first.push_back(at_first[k] < 0 ? nullptr : s->d_in + 8 * T + at_first[k]);
         }
         s->streams_T = 0;
         if (m->capture) {
@@ -1245,9 +1511,10 @@ int layers_generate(pi_model * m, int own, int n_steps, int32_t * out_tokens, fl
         if (bf16_mode(s)) { if (h.mixer == PI_MIXER_GROUPED) gqa_items(seq.data(), vis.data(), T, h.n_head, items, nullptr); else work_items(seq.data(), vis.data(), T, h, items, nullptr); }
         w.items = s->g_work + at;
         w.n = bf16_mode(s) ? (int)(items.size() - at) / 4 : T;
-        w.parts = h.mixer == PI_MIXER_GROUPED ? (bf16_mode(s) ? gqa_parts(w.n * h.n_kv, vmax, 128) : 1) : choose_parts(s, w.n, vmax);
+        w.parts = h.mixer == PI_MIXER_GROUPED ? (bf16_mode(s) ? gqa_parts(w.n * h.n_kv, gqa_span(h, vmax, false), 128) : 1) : choose_parts(s, w.n, vmax);
         in.work.push_back(w);
         in.wide.emplace_back();
+        in.first.push_back(nullptr);                           // (the positions are 0, 1, 2 ..)
         parts.push_back(w.parts);
     }
     PI_HIP_TRY(hipStreamSynchronize(m->stream));
@@ -1352,18 +1619,29 @@ extern "C" {
 
 pi_model * pi_model_create_layers(const pi_hparams * hp, const pi_layers_opts * opts, const pi_layer_desc * layers, int n_layer) {
     const auto bad = [](const char * why) -> pi_model * { pi::set_error(why); return nullptr; };
-    if (!hp || !opts || !layers || n_layer <= 0 || hp->n_embd <= 0 || hp->n_vocab <= 0 || hp->n_ctx <= 0 || (hp->arch != PI_ARCH_LERASUN && hp->arch != PI_ARCH_PIBALORN) ||
+    if (!hp || !opts || !layers || n_layer <= 0 || hp->n_embd <= 0 || hp->n_vocab <= 0 || hp->n_ctx <= 0 || (hp->arch != PI_ARCH_LERASUN && hp->arch != PI_ARCH_PIBALORN && hp->arch != PI_ARCH_FIKEVIK) ||
         (opts->compute != PI_TYPE_BF16 && opts->compute != PI_TYPE_F32) || opts->max_batch < 0)
         return bad("pi_model_create_layers: inconsistent hyper-parameters");
-    const bool one_norm = layers[0].mixer != PI_MIXER_LATENT;
+    const Family family = opts->post_norm ? kPostNorm : layers[0].mixer != PI_MIXER_LATENT ? kOneNorm : kTwoNorms;
     for (int il = 0; il < n_layer; ++il) {
         const pi_layer_desc & d = layers[il];
-        if ((d.mixer != PI_MIXER_LATENT) != one_norm) return bad("pi_model_create_layers: layers of one and of two norms in one model");
-        if (one_norm) {
-            if ((d.mixer != PI_MIXER_GROUPED && d.mixer != PI_MIXER_LINEAR) || d.n_head <= 0 || d.dim <= 0 || d.vdim <= 0) return bad("pi_model_create_layers: a layer's mixer");
+        if ((d.mixer == PI_MIXER_LATENT) != (family == kTwoNorms)) return bad("pi_model_create_layers: layers of several families in one model");
+        if (family != kPostNorm && (d.weights_of || d.gated_residual || d.mem_heads)) return bad("pi_model_create_layers: shared weights, gated residuals and memories need post_norm");
+        if (family != kTwoNorms) {
+            if ((d.mixer != PI_MIXER_GROUPED && d.mixer != (family == kOneNorm ? PI_MIXER_LINEAR : PI_MIXER_KEYED)) || d.n_head <= 0 || d.dim <= 0 || d.vdim <= 0)
+                return bad("pi_model_create_layers: a layer's mixer");
             if (d.mixer == PI_MIXER_GROUPED && (d.n_kv_head <= 0 || d.n_head % d.n_kv_head || d.rot_dim < 0 || d.rot_dim % 2 || d.rot_dim > d.dim || (d.rot_dim && !(d.rot_base > 0.0)) ||
-                                                (d.values_are_keys && d.vdim != d.dim)))
+                                                (d.values_are_keys && d.vdim != d.dim) || d.window < 0 || (d.qk_norm && d.unit_qk)))
                 return bad("pi_model_create_layers: a layer's grouped-query attention");
+            if (d.mixer == PI_MIXER_KEYED && (d.decay_rank <= 0 || d.decay_rank > 512 || !(d.decay_tau > 0.0f))) return bad("pi_model_create_layers: a layer's key decays (rank up to 512)");
+            if (d.mem_heads < 0 || (d.mem_heads > 0 && (d.mixer != PI_MIXER_GROUPED || d.mem_dim <= 0 || d.mem_vdim <= 0 || !(d.mem_cap > 0.0f)))) return bad("pi_model_create_layers: a layer's memory");
+            if (d.weights_of) {
+                pi_layer_desc same = d;
+                same.weights_of = 0;
+                if (d.weights_of < 0 || d.weights_of > n_layer || memcmp(&same, &layers[d.weights_of - 1], sizeof same))
+                    return bad("pi_model_create_layers: weights_of must name a layer with weights of its own and the same description");
+            }
+            if (family == kPostNorm && d.ffn == PI_FFN_GLU_MOE) return bad("pi_model_create_layers: a layer's feed-forward");
             if (d.ffn != PI_FFN_NONE && d.ffn != PI_FFN_GLU && d.ffn != PI_FFN_GLU_MOE) return bad("pi_model_create_layers: a layer's feed-forward");
             if (d.glu_ff < 0 || (d.ffn == PI_FFN_GLU) > (d.glu_ff > 0) || (d.ffn == PI_FFN_NONE && d.glu_ff) ||
                 (d.ffn == PI_FFN_GLU_MOE && (d.n_expert <= 0 || d.n_expert > 4096 || d.n_top <= 0 || d.n_top > d.n_expert || d.expert_ff <= 0)))
@@ -1382,8 +1660,8 @@ pi_model * pi_model_create_layers(const pi_hparams * hp, const pi_layers_opts * 
                                      d.n_top <= 0 || d.n_top > d.n_group_keep * (d.n_expert / d.n_group) || d.expert_ff <= 0))
             return bad("pi_model_create_layers: a layer's experts");
     }
-    if (opts->loop_times < 0 || (opts->loop_times > 0 && (!one_norm || opts->loop_start < 0 || opts->loop_start >= opts->loop_stop || opts->loop_stop > n_layer)) || opts->bigram_buckets < 0 ||
-        (opts->bigram_buckets && (!one_norm || opts->bigram_mul_prev < 0 || opts->bigram_mul_cur < 0)))
+    if (opts->loop_times < 0 || (opts->loop_times > 0 && (family != kOneNorm || opts->loop_start < 0 || opts->loop_start >= opts->loop_stop || opts->loop_stop > n_layer)) || opts->bigram_buckets < 0 ||
+        (opts->bigram_buckets && (family == kTwoNorms || opts->bigram_mul_prev < 0 || opts->bigram_mul_cur < 0)))
         return bad("pi_model_create_layers: the loop or the bigram table");
     if (pi_init(0) != PI_OK) return nullptr;
     pi_model * m = new pi_model();
@@ -1393,15 +1671,16 @@ pi_model * pi_model_create_layers(const pi_hparams * hp, const pi_layers_opts * 
     m->lay = new LayerState();
     m->lay->opts = *opts;
     LayerState * s = m->lay;
-    s->one_norm = one_norm;
+    s->family = family;
     std::fill(s->slot_of, s->slot_of + 32, -1);
     const int lo = opts->loop_times > 0 ? opts->loop_start : n_layer, hi = opts->loop_times > 0 ? opts->loop_stop : n_layer;
     for (int il = 0; il < n_layer; ++il) {
         Layer L;
         L.d = layers[il];
         const int passes = il >= lo && il < hi ? opts->loop_times : 1;
-        if (L.d.mixer == PI_MIXER_LINEAR) { L.state.resize(passes, nullptr); s->recurrent = true; }
-        else if (L.d.mixer == PI_MIXER_GROUPED || L.d.kv_from < 0) L.cache.resize(passes, nullptr);
+        L.rec = recurrent_part(L.d);
+        if (L.rec.on()) { L.state.resize(passes, nullptr); s->recurrent = true; }
+        if (L.d.mixer == PI_MIXER_GROUPED || (L.d.mixer == PI_MIXER_LATENT && L.d.kv_from < 0)) L.cache.resize(passes, nullptr);
         s->layers.push_back(L);
     }
     for (int il = 0; il < lo; ++il) s->order.push_back({il, 0, false});

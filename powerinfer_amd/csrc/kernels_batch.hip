@@ -1,6 +1,7 @@
 // Steps of several tokens: 2..16 sequences in lockstep or a prompt chunk of one sequence.  Dense and sparse mat-muls on the matrix
 // cores, the union of the tokens' active rows, norm + rounding passes, Q4_0 expansion and row assembly for prompt chunks.
 #include "gemm_tile.hpp"
+#include "mixers.hpp"
 
 namespace {
 
@@ -186,15 +187,18 @@ __global__ __launch_bounds__(kBlock) void gemm_t16_kernel(const EL * __restrict_
 constexpr int kGlStride = 512 + 16;               // bytes per LDS row: 256 fp16 + one 16-byte pad
 // a second matrix of the same width with its own input and output (no epilogue) in the same launch; rows 0: none
 struct SecondGemm { const void * W; const void * x; int rows; float * y; };
+// rows of the first matrix are gate and up rows in turn: out [T][ld] = clamped GLU (instead of y)
+constexpr int kEpiGlu = PI_EPI_ADD2 + 1;
+struct GluOut { void * out; int ld; float limit, gain, one; };
 template <typename EL, int RT, int NW>
 __global__ __launch_bounds__(64 * NW) void gemm_t16_lds_kernel(const EL * __restrict__ W, const EL * __restrict__ xn, int T, int rows, int cols,
                                                                   int epi, const float * __restrict__ add1, const float * __restrict__ add2, float * __restrict__ y,
-                                                                  EL * __restrict__ y16, float thr, unsigned char * __restrict__ row_any, int lay, SecondGemm two) {
+                                                                  EL * __restrict__ y16, float thr, unsigned char * __restrict__ row_any, int lay, SecondGemm two, GluOut glu) {
     const int n_first = (rows + 16 * RT - 1) / (16 * RT);
     int bx = blockIdx.x;
     if (bx >= n_first) {                                // the workgroups behind the first matrix take the second one
         bx -= n_first;
-        W = (const EL *)two.W; xn = (const EL *)two.x; rows = two.rows; y = two.y;
+        W = (const EL *)two.W; xn = (const EL *)two.x; rows = two.rows; y = two.y; epi = PI_EPI_NONE;
     }
     __shared__ __align__(16) unsigned char tile[NW][16 * kGlStride];
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
@@ -263,6 +267,14 @@ __global__ __launch_bounds__(64 * NW) void gemm_t16_lds_kernel(const EL * __rest
             float sum = cs(0, rr, t);
 #pragma unroll
             for (int w = 1; w < NW; ++w) sum += cs(w, rr, t);
+            if (epi == kEpiGlu) {
+                if (rr & 1) continue;
+                float up = cs(0, rr + 1, t);
+#pragma unroll
+                for (int w = 1; w < NW; ++w) up += cs(w, rr + 1, t);
+                ((EL *)glu.out)[(size_t)t * glu.ld + row / 2] = to_el<EL>(clamped_glu(sum, up, glu.limit, glu.gain, glu.one));
+                continue;
+            }
             const size_t o = (size_t)t * rows + row;
             if (epi == PI_EPI_RELU) sum = fmaxf(sum, 0.0f);
             else if (epi == PI_EPI_ADD) sum = __fadd_rn(sum, add1[o]);
@@ -1029,17 +1041,18 @@ int pi_k_norm_q8_round_f16(const float * x, int T, int cols, const pi_norm * nor
 // lay bit 0: xn_f16 in the operand layout of the step's activations (pi_ol_index), bit 1: y_f16 written in it
 template <typename EL>
 static int gemm_launch(const char * who, const void * W, int rows, int cols, const void * xn_f16, int T, int epilogue, const float * add1, const float * add2,
-                       float * y, void * y_f16, float thr, unsigned char * row_any, pi_stream_t stream, int lay = 0, SecondGemm two = {nullptr, nullptr, 0, nullptr}) {
-    if (!W || !xn_f16 || !y || rows <= 0) return pi::fail(PI_E_ARG, who);
+                       float * y, void * y_f16, float thr, unsigned char * row_any, pi_stream_t stream, int lay = 0, SecondGemm two = {nullptr, nullptr, 0, nullptr}, GluOut glu = {nullptr, 0, 0.0f, 0.0f, 0.0f}) {
+    if (!W || !xn_f16 || (!y && !glu.out) || rows <= 0) return pi::fail(PI_E_ARG, who);
     if (T < 1 || T > kBtMaxT || cols <= 0 || cols % 128) return pi::fail(PI_E_ARG, "batched mat-mul: 1 <= T <= 16 and cols % 128 == 0 required");
     if (epilogue < 0 || epilogue > PI_EPI_ADD2 || (epilogue >= PI_EPI_ADD && !add1) || (epilogue == PI_EPI_ADD2 && !add2))
         return pi::fail(PI_E_ARG, "batched mat-mul: bad epilogue arguments");
+    if (glu.out) epilogue = kEpiGlu;
     // row tiles per wave: enough workgroups to fill the chip first, then as few reads of the activations as possible
     const int rt = rows >= 16384 ? 4 : rows >= 5120 ? 2 : 1;      // (two tiles already at 5120 rows: the activations, re-read per row tile, are what limits one tile per wave)
 #define PI_GEMM_T16(RT) hipLaunchKernelGGL((gemm_t16_kernel<EL, RT>), dim3((rows + 16 * RT - 1) / (16 * RT)), dim3(kBlock), 0, (hipStream_t)stream, \
                        (const EL *)W, (const EL *)xn_f16, T, rows, cols, epilogue, add1, add2, y, (EL *)y_f16, thr, row_any, lay)
 #define PI_GEMM_LDS(RT, NW) hipLaunchKernelGGL((gemm_t16_lds_kernel<EL, RT, NW>), dim3((rows + 16 * RT - 1) / (16 * RT) + (two.rows + 16 * RT - 1) / (16 * RT)), dim3(64 * NW), 0, (hipStream_t)stream, \
-                       (const EL *)W, (const EL *)xn_f16, T, rows, cols, epilogue, add1, add2, y, (EL *)y_f16, thr, row_any, lay, two)
+                       (const EL *)W, (const EL *)xn_f16, T, rows, cols, epilogue, add1, add2, y, (EL *)y_f16, thr, row_any, lay, two, glu)
     if (cols % 256 == 0) {
         // waves per workgroup: when every workgroup has a compute unit to itself (at most one per unit), eight waves keep twice
         // the loads in flight per unit; with more workgroups than units the chip is full with four
@@ -1084,6 +1097,13 @@ int pi_k_gemm_bf16_ol_two(const void * W, int rows, const void * xn_ol, float * 
     if (!W2 || !xn2_ol || !y2 || rows2 <= 0 || cols % 256) return pi::fail(PI_E_ARG, "pi_k_gemm_bf16_ol_two: bad arguments (cols % 256 == 0)");
     return gemm_launch<__bf16>("pi_k_gemm_bf16_ol_two", W, rows, cols, xn_ol, T, PI_EPI_NONE, nullptr, nullptr, y, nullptr, 0.0f, nullptr, stream, 3,
                                SecondGemm{W2, xn2_ol, rows2, y2});
+}
+
+int pi_k_gemm_bf16_ol_glu(const void * W, int ff, const void * xn_ol, float limit, float gain, float one, void * act, int ld_act, const void * W2, int rows2, float * y2,
+                          int cols, int T, pi_stream_t stream) {
+    if (ff <= 0 || !act || ld_act < ff || cols % 256 || (W2 && (!y2 || rows2 <= 0))) return pi::fail(PI_E_ARG, "pi_k_gemm_bf16_ol_glu: bad arguments (cols % 256 == 0)");
+    return gemm_launch<__bf16>("pi_k_gemm_bf16_ol_glu", W, 2 * ff, cols, xn_ol, T, PI_EPI_NONE, nullptr, nullptr, nullptr, nullptr, 0.0f, nullptr, stream, 1,
+                               SecondGemm{W2, xn_ol, W2 ? rows2 : 0, y2}, GluOut{act, ld_act, limit, gain, one});
 }
 
 }  // extern "C"

@@ -4,47 +4,16 @@
 
 namespace {
 
-// ---------------------------------------------------------------------------------------------------------------------------------
-// behind the joint projection: a wave per head - rotation, division by the root mean square, query row or cell
-// ---------------------------------------------------------------------------------------------------------------------------------
-constexpr int kGqaMaxDim = 256;
 template <typename ST>
 __global__ __launch_bounds__(256) void gqa_prep_kernel(pi_gqa_prep p, pi_ffn_front f, int n_heads4, int per) {
     extern __shared__ __align__(16) float sm[];
     const int t = blockIdx.x / per, b = blockIdx.x % per;
-    if (b >= n_heads4) { front_block<ST>(f, p.z, p.ldz, t, b - n_heads4, sm); return; }
-    const int head = b * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63, half = p.rot_dim / 2;
-    if (head >= p.n_head + p.n_kv) return;
-    const bool key = head >= p.n_head;
-    const int g = head - p.n_head;
-    const float * z = p.z + (size_t)t * p.ldz, * src = key ? z + p.off_k + g * p.dim : z + head * p.dim;
-    const float2 * cs = (const float2 *)p.cs + (size_t)t * half;
-    constexpr int J = kGqaMaxDim / 64;
-    float x[J];
-    float ss = 0.0f;
-#pragma unroll
-    for (int j = 0; j < J; ++j) {
-        const int e = lane + 64 * j;
-        float v = 0.0f;
-        if (e < p.dim) {
-            v = src[e];
-            if (e < half) { const float2 c = cs[e]; v = v * c.x - src[e + half] * c.y; }
-            else if (e < 2 * half) { const float2 c = cs[e - half]; v = v * c.x + src[e - half] * c.y; }
-        }
-        x[j] = v;
-        ss = fmaf(v, v, ss);
-    }
-    float sc = 1.0f;
-    if (p.unit) sc = pi_inv_sqrt(pi_wave_sum(ss) / (float)p.dim + p.eps);
-    ST * row = key ? (ST *)p.cache + ((size_t)p.cell[t] * p.n_kv + g) * 2 * p.hd : (ST *)p.q + ((size_t)t * p.n_head + head) * p.hd;
-#pragma unroll
-    for (int j = 0; j < J; ++j) { const int e = lane + 64 * j; if (e < p.hd) row[e] = to_st<ST>(x[j] * sc); }      // (zeros behind dim)
-    if (key) {
-        const float * v = z + p.off_v + g * p.vdim;
-#pragma unroll
-        for (int j = 0; j < J; ++j) { const int e = lane + 64 * j; if (e < p.hd) row[p.hd + e] = to_st<ST>(e < p.vdim ? v[e] : 0.0f); }
-    }
+    if (b >= n_heads4) front_block<ST>(f, p.z, p.ldz, t, b - n_heads4, sm);
+    else gqa_prep_heads<ST>(p, t, b);
 }
+
+// the first cell a token sees
+__device__ __forceinline__ int first_cell(const pi_gqa_attn & p, int t) { return p.first ? p.first[t] : p.window > 0 ? max(p.n_vis[t] - p.window, 0) : 0; }
 
 // ---------------------------------------------------------------------------------------------------------------------------------
 // bf16 attention on the matrix cores.  Scores are formed transposed (keys x query rows), so that a lane's scores belong to one row, its
@@ -71,9 +40,11 @@ __global__ __launch_bounds__(256, WIDE && KS <= 4 ? 2 : 1) void gqa_attn_kernel(
     const int tok0 = item.x, first = item.y, rows = min(item.z, R), per = p.n_head / p.n_kv;
     const int32_t * list = p.lists + (size_t)item.w * p.list_ld;
     const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, i = lane & 15, gq = lane >> 4;
-    const int n_keys = p.n_vis[tok0 + (first + rows - 1) / per], n_all = p.n_vis[tok0 + first / per];       // the most and the fewest cells a row here sees
-    const int tiles = (n_keys + NK - 1) / NK;
-    const int c0 = (int)((long long)tiles * part / p.n_parts) * NK, c1 = min((int)((long long)tiles * (part + 1) / p.n_parts) * NK, n_keys);
+    const int tok_a = tok0 + first / per, tok_z = tok0 + (first + rows - 1) / per;
+    const int n_keys = p.n_vis[tok_z], n_all = p.n_vis[tok_a];       // the most and the fewest cells a row here sees
+    const int lo_a = first_cell(p, tok_a), lo_z = first_cell(p, tok_z);      // the first cell of the rows' windows: the earliest and the latest
+    const int tiles = (n_keys - lo_a + NK - 1) / NK;
+    const int c0 = lo_a + (int)((long long)tiles * part / p.n_parts) * NK, c1 = min(lo_a + (int)((long long)tiles * (part + 1) / p.n_parts) * NK, n_keys);
     // the thread's pieces of a tile: eight threads share a cell's row
     const int sub = tid % 8, key0 = tid / 8;
     const uint16_t * cache = (const uint16_t *)p.cache + (size_t)g * 2 * HD + sub * 8;
@@ -90,7 +61,7 @@ __global__ __launch_bounds__(256, WIDE && KS <= 4 ? 2 : 1) void gqa_attn_kernel(
             for (int j = 0; j < KS; ++j) pre[k][j] = pi_ld16(cache + (size_t)idx[k] * p.n_kv * 2 * HD + j * 64);
     };
     if (c0 < c1) look_up(c0);
-    int row[U], tok[U], head[U], nv[U];
+    int row[U], tok[U], head[U], nv[U], lo[U];
     pi_u32x4 qf[U][KS];
 #pragma unroll
     for (int u = 0; u < U; ++u) {
@@ -99,6 +70,7 @@ __global__ __launch_bounds__(256, WIDE && KS <= 4 ? 2 : 1) void gqa_attn_kernel(
         tok[u] = tok0 + rr / per;
         head[u] = g * per + rr % per;
         nv[u] = row[u] < rows ? p.n_vis[tok[u]] : 0;
+        lo[u] = first_cell(p, tok[u]);
 #pragma unroll
         for (int s = 0; s < KS; ++s) qf[u][s] = pi_ld16((const uint16_t *)p.q + ((size_t)tok[u] * p.n_head + head[u]) * HD + s * 32 + gq * 8);
     }
@@ -137,7 +109,7 @@ __global__ __launch_bounds__(256, WIDE && KS <= 4 ? 2 : 1) void gqa_attn_kernel(
             }
         }
         pi_u32x4 pb[U][KT / 2];                                  // weights as the column operand
-        const bool edge = cb + NK > n_all;
+        const bool edge = cb + NK > n_all || cb < lo_z;
 #pragma unroll
         for (int u = 0; u < U; ++u) {
             float mx = -INFINITY;
@@ -146,7 +118,8 @@ __global__ __launch_bounds__(256, WIDE && KS <= 4 ? 2 : 1) void gqa_attn_kernel(
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
                     float v = s[u][kt][r] * p.scale;
-                    if (edge && cb + kb + kt * 16 + 4 * gq + r >= nv[u]) v = -INFINITY;
+                    const int c = cb + kb + kt * 16 + 4 * gq + r;
+                    if (edge && (c >= nv[u] || c < lo[u])) v = -INFINITY;
                     s[u][kt][r] = v;
                     mx = fmaxf(mx, v);
                 }
@@ -200,7 +173,7 @@ __global__ __launch_bounds__(256, WIDE && KS <= 4 ? 2 : 1) void gqa_attn_kernel(
                 if (gq == 0) ml[(srow0 + row[u]) * p.n_parts + part] = make_float2(m[u], l[u]);
                 continue;
             }
-            const float mf = fmaxf(m[u], p.sink), a = m[u] == -INFINITY ? 0.0f : expf(m[u] - mf), f = a / (l[u] * a + expf(p.sink - mf));
+            const float mf = fmaxf(m[u], p.sink), a = m[u] == -INFINITY ? 0.0f : expf(m[u] - mf), f = a / (l[u] * a + expf(p.sink - mf)) * p.out_scale;
             bf16 * out = (bf16 *)p.att + (size_t)tok[u] * p.ld_att + head[u] * p.vdim;
 #pragma unroll
             for (int v = 0; v < VT; ++v) {
@@ -230,7 +203,7 @@ __global__ __launch_bounds__(256, WIDE && KS <= 4 ? 2 : 1) void gqa_attn_kernel(
     float fin = 1.0f;
     if (whole) {
         const float mf = fmaxf(mm, p.sink), a = mm == -INFINITY ? 0.0f : expf(mm - mf);
-        fin = a / (sum * a + expf(p.sink - mf));
+        fin = a / (sum * a + expf(p.sink - mf)) * p.out_scale;
     } else if (cl == 0) ml[(srow0 + r) * p.n_parts + part] = make_float2(mm, sum);
     const int rr = first + r;
     bf16 * out = (bf16 *)p.att + (size_t)(tok0 + rr / per) * p.ld_att + (g * per + rr % per) * p.vdim;
@@ -271,7 +244,7 @@ __global__ __launch_bounds__(256) void gqa_attn_f32_kernel(pi_gqa_attn p) {
     for (int k = tid; k < p.dim; k += 256) q[k] = ((const float *)p.q)[(size_t)blockIdx.x * p.hd + k];
     const bool sink = p.sink != -INFINITY;
     float m = p.sink, l = sink ? 1.0f : 0.0f, acc = 0.0f;              // the sink is the soft-max's first entry: weight exp(0), no value
-    for (int c0 = 0; c0 < n; c0 += kGfCells) {
+    for (int c0 = first_cell(p, t); c0 < n; c0 += kGfCells) {
         const int nc = min(kGfCells, n - c0);
         __syncthreads();
         for (int c = tid; c < nc; c += 256) idx[c] = list[c0 + c];
@@ -296,21 +269,21 @@ __global__ __launch_bounds__(256) void gqa_attn_f32_kernel(pi_gqa_attn p) {
         }
         m = mn;
     }
-    if (tid < p.vdim) ((float *)p.att)[(size_t)t * p.ld_att + h * p.vdim + tid] = acc / l;
+    if (tid < p.vdim) ((float *)p.att)[(size_t)t * p.ld_att + h * p.vdim + tid] = acc / l * p.out_scale;
 }
 
 template <typename ST>
-__global__ void gqa_shift_kernel(ST * __restrict__ cache, int n_kv, int hd, int rot_dim, double base, const int32_t * __restrict__ delta) {
+__global__ void gqa_shift_kernel(ST * __restrict__ cache, int n_kv, int hd, int rot_dim, double base, int pairs, const int32_t * __restrict__ delta) {
     const int c = blockIdx.x, d = delta[c], half = rot_dim / 2;
     if (d == 0) return;
     for (int e = threadIdx.x; e < n_kv * half; e += blockDim.x) {
         const int g = e / half, i = e % half;
         double sn, cn;
         sincos((double)d * pow(base, -2.0 * (double)i / (double)rot_dim), &sn, &cn);
-        ST * r = cache + ((size_t)c * n_kv + g) * 2 * hd + i;
-        const float u = from_st(r[0]), v = from_st(r[half]);
-        r[0] = to_st<ST>(u * (float)cn - v * (float)sn);
-        r[half] = to_st<ST>(v * (float)cn + u * (float)sn);
+        ST * r = cache + ((size_t)c * n_kv + g) * 2 * hd + (pairs ? 2 * i : i), * o = r + (pairs ? 1 : half);
+        const float u = from_st(*r), v = from_st(*o);
+        *r = to_st<ST>(u * (float)cn - v * (float)sn);
+        *o = to_st<ST>(v * (float)cn + u * (float)sn);
     }
 }
 
@@ -327,7 +300,7 @@ template <int KS, bool WIDE> int launch_gqa(const pi_gqa_attn * p, hipStream_t s
 
 int gqa_check(int type, const pi_gqa_attn * p) {
     if (!p || !p->q || !p->cache || !p->lists || !p->work || !p->n_vis || !p->att || p->T <= 0 || p->n_head <= 0 || p->n_kv <= 0 || p->n_head % p->n_kv || p->dim <= 0 || p->vdim <= 0 ||
-        p->hd < p->dim || p->hd < p->vdim || p->ld_att < p->n_head * p->vdim || p->hd != pi_k_gqa_head_ld(type, p->dim, p->vdim) || p->n_parts <= 0)
+        p->hd < p->dim || p->hd < p->vdim || p->ld_att < p->n_head * p->vdim || p->hd != pi_k_gqa_head_ld(type, p->dim, p->vdim) || p->n_parts <= 0 || p->window < 0)
         return pi::fail(PI_E_ARG, "pi_k_gqa_attn: bad arguments");
     if (type == PI_TYPE_BF16 && (p->n_work <= 0 || (long long)p->n_work * p->n_kv > (1 << 30) || p->n_parts > 64 || (p->n_parts > 1 && !p->scratch)))
         return pi::fail(PI_E_ARG, "pi_k_gqa_attn: bad work arguments");
@@ -358,11 +331,9 @@ int pi_k_gqa_head_ld(int type, int dim, int vdim) {
 
 int pi_k_gqa_prep(int type, const pi_gqa_prep * p, const pi_ffn_front * front, pi_stream_t stream) {
     const pi_ffn_front f = front ? *front : pi_ffn_front{};
-    if (!p || !p->z || !p->cs || !p->q || !p->cache || !p->cell || p->T <= 0 || p->n_head <= 0 || p->n_kv <= 0 || p->n_head % p->n_kv || p->rot_dim < 0 || p->rot_dim % 2 || p->rot_dim > p->dim ||
-        p->hd != pi_k_gqa_head_ld(type, p->dim, p->vdim) || p->hd <= 0 || p->off_k < p->n_head * p->dim || p->off_k + p->n_kv * p->dim > p->ldz || p->off_v < 0 ||
-        p->off_v + p->n_kv * p->vdim > p->ldz || !front_ok(f, p->ldz))
+    if (!p || !gqa_prep_ok(type, *p) || !front_ok(f, p->ldz))
         return pi::fail(PI_E_ARG, "pi_k_gqa_prep: bad arguments");
-    const int n4 = (p->n_head + p->n_kv + 3) / 4, per = n4 + front_blocks(f);
+    const int n4 = gqa_prep_blocks(*p), per = n4 + front_blocks(f);
     if ((long long)per * p->T > (1 << 30)) return pi::fail(PI_E_ARG, "pi_k_gqa_prep: too many tokens");
     if (type == PI_TYPE_BF16) hipLaunchKernelGGL(gqa_prep_kernel<bf16>, dim3(per * p->T), dim3(256), front_lds_bytes(f), (hipStream_t)stream, *p, f, n4, per);
     else if (type == PI_TYPE_F32) hipLaunchKernelGGL(gqa_prep_kernel<float>, dim3(per * p->T), dim3(256), front_lds_bytes(f), (hipStream_t)stream, *p, f, n4, per);
@@ -396,11 +367,11 @@ int pi_k_gqa_attn(int type, const pi_gqa_attn * p, pi_stream_t stream) {
     return pi::check_launch("pi_k_gqa_attn merge");
 }
 
-int pi_k_gqa_shift(int type, void * cache, int n_cells, int n_kv, int hd, int rot_dim, double base, const int32_t * delta, pi_stream_t stream) {
+int pi_k_gqa_shift(int type, void * cache, int n_cells, int n_kv, int hd, int rot_dim, double base, int pairs, const int32_t * delta, pi_stream_t stream) {
     if (!cache || !delta || n_cells <= 0 || n_kv <= 0 || hd <= 0 || rot_dim < 0 || rot_dim % 2 || rot_dim > hd) return pi::fail(PI_E_ARG, "pi_k_gqa_shift: bad arguments");
     if (rot_dim == 0) return PI_OK;
-    if (type == PI_TYPE_BF16) hipLaunchKernelGGL(gqa_shift_kernel<bf16>, dim3(n_cells), dim3(64), 0, (hipStream_t)stream, (bf16 *)cache, n_kv, hd, rot_dim, base, delta);
-    else if (type == PI_TYPE_F32) hipLaunchKernelGGL(gqa_shift_kernel<float>, dim3(n_cells), dim3(64), 0, (hipStream_t)stream, (float *)cache, n_kv, hd, rot_dim, base, delta);
+    if (type == PI_TYPE_BF16) hipLaunchKernelGGL(gqa_shift_kernel<bf16>, dim3(n_cells), dim3(64), 0, (hipStream_t)stream, (bf16 *)cache, n_kv, hd, rot_dim, base, pairs, delta);
+    else if (type == PI_TYPE_F32) hipLaunchKernelGGL(gqa_shift_kernel<float>, dim3(n_cells), dim3(64), 0, (hipStream_t)stream, (float *)cache, n_kv, hd, rot_dim, base, pairs, delta);
     else return pi::fail(PI_E_UNSUPPORTED, "pi_k_gqa_shift: type");
     return pi::check_launch("pi_k_gqa_shift");
 }

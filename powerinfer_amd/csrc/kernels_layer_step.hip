@@ -284,12 +284,12 @@ __global__ __launch_bounds__(256) void value_and_up_kernel(pi_latent_attn p, con
     else expert_up(u, (b - n_value) % n_up_tiles, (b - n_value) / n_up_tiles, smem);
 }
 
-// the merge of a split grouped-query attention (four rows a workgroup) or the gated norm of a linear attention (a token a workgroup) beside
-// the experts' first matrices
+// the merge of a split grouped-query attention (four rows a workgroup) and the gated norm of a linear attention (a token or four heads a
+// workgroup) beside the experts' first matrices
 __global__ __launch_bounds__(256) void mix_and_up_kernel(pi_gqa_attn p, pi_gate_norm gn, int n_merge, int n_gate, ExpertUp u, int n_up_tiles) {
     extern __shared__ __align__(16) unsigned char smem[];
     int b = blockIdx.x;
-    if (b < n_gate) { gate_norm_token<bf16>(gn, b, reinterpret_cast<double *>(smem)); return; }
+    if (b < n_gate) { gate_norm_block<bf16>(gn, b, reinterpret_cast<double *>(smem)); return; }
     b -= n_gate;
     if (b < n_merge) {
         const int r4 = gqa_rows(p.wide) / 4;
@@ -300,7 +300,8 @@ __global__ __launch_bounds__(256) void mix_and_up_kernel(pi_gqa_attn p, pi_gate_
 }
 
 // ---------------------------------------------------------------------------------------------------------------------------------
-// what closes a layer: out[t] = x[t] + (W_o att[t] + sum over the token's experts of W_down[e] act[pair]), 16 rows a workgroup.  The
+// what closes a layer: out[t] = x[t] + (W_o att[t] + sum over the token's experts of W_down[e] act[pair]), 16 rows a workgroup (or, what closes a
+// sublayer in front of its norm: out[t] = alpha x[t] + gate * W att[t]).  The
 // pieces of 256 columns of W_o and of every expert of the step form one list that the waves take in turn.
 // ---------------------------------------------------------------------------------------------------------------------------------
 template <int NW>
@@ -355,7 +356,9 @@ __global__ __launch_bounds__(64 * NW) void layer_out_step_kernel(pi_layer_out a)
     float v = 0.0f;
 #pragma unroll
     for (int w = 0; w < NW; ++w) v += reinterpret_cast<float (*)[17]>(tiles[w])[tid & 15][t];
-    v += a.x[(size_t)t * a.rows + row];
+    if (a.gate_z) v *= sigmoid_f32(a.gate_z[(size_t)t * a.ld_gate + a.off_gate + row] + a.gate_b[row]);
+    const float x = a.x[(size_t)t * a.rows + row];
+    v += a.scaled ? a.alpha * x : x;
     a.out[(size_t)t * a.rows + row] = v;
     if (a.keep) a.keep[(size_t)t * a.rows + row] = v;
 }
@@ -407,7 +410,7 @@ int pi_k_mix_up_step(const pi_gqa_attn * attn, const pi_gate_norm * gate, const 
         return pi::fail(PI_E_ARG, "pi_k_mix_up_step: bad arguments");
     if (ids && (!up || !x_ol || !weights || !act || n_expert <= 0 || ff <= 0 || cols <= 0 || cols % 32 || top <= 0 || T * top > kStepPairs || ld_act < ff))
         return pi::fail(PI_E_ARG, "pi_k_mix_up_step: bad expert arguments");
-    const int n_merge = attn ? p.n_work * p.n_kv * (gqa_rows(p.wide) / 4) : 0, n_gate = gate ? g.T : 0, n_up_tiles = ids ? (2 * ff + 15) / 16 : 1, n_up = ids ? n_up_tiles * T * top : 0;
+    const int n_merge = attn ? p.n_work * p.n_kv * (gqa_rows(p.wide) / 4) : 0, n_gate = gate ? gate_norm_blocks(g) : 0, n_up_tiles = ids ? (2 * ff + 15) / 16 : 1, n_up = ids ? n_up_tiles * T * top : 0;
     if (n_merge + n_gate + n_up == 0) return PI_OK;
     ExpertUp u{(const bf16 *)up, 2 * ff, cols, (const bf16 *)x_ol, ids, weights, T, top, (bf16 *)act, ld_act};
     u.glu = 1; u.limit = limit; u.gain = gain;
@@ -416,7 +419,7 @@ int pi_k_mix_up_step(const pi_gqa_attn * attn, const pi_gate_norm * gate, const 
 }
 
 int pi_k_layer_out_step(const pi_layer_out * a, pi_stream_t stream) {
-    if (!a || !a->x || !a->wo || !a->att || !a->out || a->rows <= 0 || a->T <= 0 || a->T > kBtMaxT || a->ld_att <= 0 || a->ld_att % 32 ||
+    if (!a || !a->x || !a->wo || !a->att || !a->out || (a->gate_z && (!a->gate_b || a->off_gate < 0 || a->off_gate + a->rows > a->ld_gate)) || a->rows <= 0 || a->T <= 0 || a->T > kBtMaxT || a->ld_att <= 0 || a->ld_att % 32 ||
         (a->ids && (!a->down || !a->act || a->ld_act <= 0 || a->ld_act % 32 || a->top <= 0 || a->T * a->top > kStepPairs || a->n_expert <= 0 || a->n_expert > kStepExperts)))
         return pi::fail(PI_E_ARG, "pi_k_layer_out_step: bad arguments");
     // eight waves a workgroup when every workgroup has a compute unit to itself, four (and several workgroups a unit) beyond

@@ -172,6 +172,78 @@ __global__ __launch_bounds__(1024) void layer_norm_kernel(float * __restrict__ x
     for (int i = threadIdx.x; i < cols; i += blockDim.x) out[at(i)] = to_st<ST>((xt[i] - mean) * sc * w[i]);
 }
 
+// what closes a sublayer whose norm comes after the sum (pi_res_norm): Q quads of columns per thread in registers, one trip over the row
+template <typename ST, int Q>
+__global__ void res_norm_kernel(pi_res_norm p) {
+    __shared__ double red[16];
+    const int t = blockIdx.x, tid = threadIdx.x, nt = blockDim.x;
+    const size_t base = (size_t)t * p.cols;
+    const float * gz = p.gate_z ? p.gate_z + (size_t)t * p.ld_gate + p.off_gate : nullptr;
+    float v[Q][4], wv[Q][4];
+    double s = 0.0;
+    const bool quads = ((p.cols | p.ld_gate | p.off_gate) & 3) == 0;
+    auto load = [&](const float * a, int c, float (&o)[4]) {      // columns c .. c + 3 of a row (past its end: zeros)
+        if (quads && c < p.cols) { const float4 q = *reinterpret_cast<const float4 *>(a + c); o[0] = q.x; o[1] = q.y; o[2] = q.z; o[3] = q.w; }
+        else for (int j = 0; j < 4; ++j) o[j] = c + j < p.cols ? a[c + j] : 0.0f;
+    };
+#pragma unroll
+    for (int q = 0; q < Q; ++q) {
+        const int c = (tid + q * nt) * 4;
+        load(p.x + base, c, v[q]);
+        if (p.w) load(p.w, c, wv[q]);
+        if (p.mix) {
+            float m[4];
+            load(p.mix + base, c, m);
+            if (gz) {
+                float g[4], b[4];
+                load(gz, c, g);
+                load(p.gate_b, c, b);
+#pragma unroll
+                for (int j = 0; j < 4; ++j) m[j] *= sigmoid_f32(g[j] + b[j]);
+            }
+#pragma unroll
+            for (int j = 0; j < 4; ++j) v[q][j] = fmaf(p.alpha, v[q][j], m[j]);
+        }
+#pragma unroll
+        for (int j = 0; j < 4; ++j) if (c + j < p.cols) s += (double)v[q][j] * (double)v[q][j];
+    }
+    float sc = 1.0f;
+    if (p.w) sc = pi_inv_sqrt((float)(block_sum_f64(s, red) / p.cols) + p.eps);
+    ST * h = (ST *)p.h;
+#pragma unroll
+    for (int q = 0; q < Q; ++q) {
+        const int c = (tid + q * nt) * 4;
+        if (c >= p.cols) break;
+        if (p.w) {
+#pragma unroll
+            for (int j = 0; j < 4; ++j) v[q][j] *= sc * wv[q][j];
+        }
+        const bool whole = quads && c + 4 <= p.cols;
+        store4(p.out + base + c, v[q], whole, p.cols - c);
+        if (p.keep) store4(p.keep + base + c, v[q], whole, p.cols - c);
+        if (h) {                                       // (four columns from a multiple of four on lie together in both layouts)
+            ST * o = h + (p.ol ? pi_ol_index(t, c) : (size_t)t * p.ld + c);
+            store4(o, v[q], ((uintptr_t)o & (4 * sizeof(ST) - 1)) == 0 && c + 4 <= p.cols, p.cols - c);
+        }
+    }
+}
+template <typename ST> int launch_res_norm(const pi_res_norm & p, hipStream_t st) {
+    const int quads = (p.cols + 3) / 4;
+    if (quads <= 256) hipLaunchKernelGGL((res_norm_kernel<ST, 1>), dim3(p.T), dim3(256), 0, st, p);
+    else if (quads <= 512) hipLaunchKernelGGL((res_norm_kernel<ST, 1>), dim3(p.T), dim3(512), 0, st, p);
+    else if (quads <= 1024) hipLaunchKernelGGL((res_norm_kernel<ST, 2>), dim3(p.T), dim3(512), 0, st, p);
+    else if (quads <= 2048) hipLaunchKernelGGL((res_norm_kernel<ST, 4>), dim3(p.T), dim3(512), 0, st, p);
+    else if (quads <= 8192) hipLaunchKernelGGL((res_norm_kernel<ST, 8>), dim3(p.T), dim3(1024), 0, st, p);
+    else return pi::fail(PI_E_UNSUPPORTED, "pi_k_res_norm: up to 32768 columns");
+    return pi::check_launch("pi_k_res_norm");
+}
+
+template <typename ST>
+__global__ __launch_bounds__(256) void ffn_front_kernel(pi_ffn_front f, const float * __restrict__ z, int ldz, int per) {
+    extern __shared__ __align__(16) float sm[];
+    front_block<ST>(f, z, ldz, blockIdx.x / per, blockIdx.x % per, sm);
+}
+
 // ---------------------------------------------------------------------------------------------------------------------------------
 // grouped mat-mul.  A workgroup of four waves owns 64 rows of one group's matrix x 32 of the group's tokens; each wave holds 16 rows in
 // the matrix cores' operand layout (lane l: row l % 16, eight consecutive columns 8 * (l / 16) of a 32-column step) against two token
@@ -469,6 +541,26 @@ int pi_k_layer_norm(int type, float * x, const int32_t * rows, int T, int cols, 
     else if (type == PI_TYPE_F32) hipLaunchKernelGGL(layer_norm_kernel<float>, dim3(T), dim3(block), 0, (hipStream_t)stream, x, rows, cols, eps, w, x0, step, (float *)out, ld, 0);
     else return pi::fail(PI_E_UNSUPPORTED, "pi_k_layer_norm: type");
     return pi::check_launch("pi_k_layer_norm");
+}
+
+int pi_k_res_norm(int type, const pi_res_norm * p, pi_stream_t stream) {
+    if (!p || !p->x || !p->out || p->T <= 0 || p->cols <= 0 || (p->mix && p->gate_z && (!p->gate_b || p->off_gate < 0 || p->off_gate + p->cols > p->ld_gate)) || (p->h && p->ld < p->cols))
+        return pi::fail(PI_E_ARG, "pi_k_res_norm: bad arguments");
+    if (p->h && p->ol && (type != PI_TYPE_BF16 || p->T > kBtMaxT || p->ld % 8)) return pi::fail(PI_E_ARG, "pi_k_res_norm: operand layout needs BF16, T <= 16, ld % 8 == 0");
+    if (type == PI_TYPE_BF16) return launch_res_norm<bf16>(*p, (hipStream_t)stream);
+    if (type == PI_TYPE_F32) return launch_res_norm<float>(*p, (hipStream_t)stream);
+    return pi::fail(PI_E_UNSUPPORTED, "pi_k_res_norm: type");
+}
+
+int pi_k_ffn_front(int type, const float * z, int ldz, int T, const pi_ffn_front * front, pi_stream_t stream) {
+    if (!z || !front || T <= 0 || !front_ok(*front, ldz)) return pi::fail(PI_E_ARG, "pi_k_ffn_front: bad arguments");
+    const int per = front_blocks(*front);
+    if (per == 0) return PI_OK;
+    if ((long long)per * T > (1 << 30)) return pi::fail(PI_E_ARG, "pi_k_ffn_front: too many tokens");
+    if (type == PI_TYPE_BF16) hipLaunchKernelGGL(ffn_front_kernel<bf16>, dim3(per * T), dim3(256), front_lds_bytes(*front), (hipStream_t)stream, *front, z, ldz, per);
+    else if (type == PI_TYPE_F32) hipLaunchKernelGGL(ffn_front_kernel<float>, dim3(per * T), dim3(256), front_lds_bytes(*front), (hipStream_t)stream, *front, z, ldz, per);
+    else return pi::fail(PI_E_UNSUPPORTED, "pi_k_ffn_front: type");
+    return pi::check_launch("pi_k_ffn_front");
 }
 
 int pi_k_norm_pair(int type, const float * x, const int32_t * rows, int T, int cols, float eps, const float * wa, void * out_a,

@@ -1,5 +1,5 @@
 // Pieces of a layer that several launches hold: the clamped GLU, what a layer with one norm computes of its feed-forward straight from the
-// joint projection, the merge of a split grouped-query attention, and the gated norm behind a linear attention.
+// joint projection, queries and cells of a grouped-query attention, the merge of a split one, and the gated norm behind a linear attention.
 #pragma once
 #include "layer_types.hpp"
 #include "route.hpp"
@@ -8,10 +8,10 @@ namespace {
 
 __device__ __forceinline__ float sigmoid_f32(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float silu_f32(float z) { return z * sigmoid_f32(z); }
-__device__ __forceinline__ float clamped_glu(float g, float u, float limit, float gain) {
+__device__ __forceinline__ float clamped_glu(float g, float u, float limit, float gain, float one = 1.0f) {
     g = fminf(g, limit);
     u = fminf(fmaxf(u, -limit), limit);
-    return g * sigmoid_f32(gain * g) * (u + 1.0f);
+    return g * sigmoid_f32(gain * g) * (u + one);
 }
 
 // four values of activation storage in one store where the place allows it
@@ -50,11 +50,75 @@ template <typename ST> __device__ void front_block(const pi_ffn_front & f, const
 #pragma unroll
         for (int k = 0; k < 8; ++k) w[k] = j0 + k / 2 < f.ff ? g[k] : 0.0f;
     }
-    const float s = f.off_score >= 0 ? sigmoid_f32(row[f.off_score]) : 1.0f;
+    const float s = f.off_score >= 0 ? sigmoid_f32(row[f.off_score]) : 1.0f, one = f.plain_up ? 0.0f : 1.0f;
 #pragma unroll
-    for (int k = 0; k < 4; ++k) v[k] = j0 + k < f.ff ? s * clamped_glu(w[2 * k], w[2 * k + 1], f.limit, f.gain) : 0.0f;
+    for (int k = 0; k < 4; ++k) v[k] = j0 + k < f.ff ? s * clamped_glu(w[2 * k], w[2 * k + 1], f.limit, f.gain, one) : 0.0f;
     ST * o = (ST *)f.act + (size_t)t * f.ld_act + j0;
     store4(o, v, ((uintptr_t)o & (4 * sizeof(ST) - 1)) == 0, 4);
+}
+
+// ---- grouped-query attention, behind the joint projection: a wave per head (four heads a block) - norm, rotation, division by the root
+// mean square, query row or cell --------------------------------------------------------------------------------------------------------
+constexpr int kGqaMaxDim = 256;
+__host__ __device__ inline int gqa_prep_blocks(const pi_gqa_prep & p) { return (p.n_head + p.n_kv + 3) / 4; }
+template <typename ST> __device__ void gqa_prep_heads(const pi_gqa_prep & p, int t, int b) {
+    const int head = b * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63, half = p.rot_dim / 2;
+    if (head >= p.n_head + p.n_kv) return;
+    const bool key = head >= p.n_head;
+    const int g = head - p.n_head;
+    const float * z = p.z + (size_t)t * p.ldz, * src = key ? z + p.off_k + g * p.dim : z + head * p.dim;
+    const float * w = key ? p.k_norm : p.q_norm;
+    const float2 * cs = (const float2 *)p.cs + (size_t)t * half;
+    constexpr int J = kGqaMaxDim / 64;
+    float x[J], y[J];                                    // the lane's values and what each is paired with
+    float ss = 0.0f;
+#pragma unroll
+    for (int j = 0; j < J; ++j) {
+        const int e = lane + 64 * j, o = e >= 2 * half ? e : p.rot_pairs ? e ^ 1 : e < half ? e + half : e - half;
+        const float f = w && e < p.dim ? w[e] : 1.0f, fo = w && e < p.dim ? w[o] : 1.0f;
+        x[j] = e < p.dim ? src[e] : 0.0f;
+        y[j] = e < p.dim ? src[o] * fo : 0.0f;
+        ss = fmaf(x[j], x[j], ss);
+        x[j] *= f;
+    }
+    float sc = w ? pi_inv_sqrt(pi_wave_sum(ss) / (float)p.dim + p.eps) : 1.0f;
+    ss = 0.0f;
+#pragma unroll
+    for (int j = 0; j < J; ++j) {
+        const int e = lane + 64 * j;
+        float v = x[j];
+        if (e < 2 * half) {
+            const float2 c = cs[p.rot_pairs ? e >> 1 : e < half ? e : e - half];
+            const bool second = p.rot_pairs ? e & 1 : e >= half;
+            v = second ? v * c.x + y[j] * c.y : v * c.x - y[j] * c.y;
+        }
+        x[j] = v;
+        ss = fmaf(v, v, ss);
+    }
+    if (p.unit) sc = pi_inv_sqrt(pi_wave_sum(ss) / (float)p.dim + p.eps);
+    if (!key && p.temp) sc *= p.temp[head];
+    ST * row = key ? (ST *)p.cache + ((size_t)p.cell[t] * p.n_kv + g) * 2 * p.hd : (ST *)p.q + ((size_t)t * p.n_head + head) * p.hd;
+#pragma unroll
+    for (int j = 0; j < J; ++j) { const int e = lane + 64 * j; if (e < p.hd) row[e] = to_st<ST>(x[j] * sc); }      // (zeros behind dim)
+    if (key) {
+        const float * v = z + p.off_v + g * p.vdim;
+        float sv = 1.0f;
+#pragma unroll
+        for (int j = 0; j < J; ++j) { const int e = lane + 64 * j; x[j] = e < p.vdim ? v[e] : 0.0f; }
+        if (p.unit_v) {
+            ss = 0.0f;
+#pragma unroll
+            for (int j = 0; j < J; ++j) ss = fmaf(x[j], x[j], ss);
+            sv = pi_inv_sqrt(pi_wave_sum(ss) / (float)p.vdim + p.eps);
+        }
+#pragma unroll
+        for (int j = 0; j < J; ++j) { const int e = lane + 64 * j; if (e < p.hd) row[p.hd + e] = to_st<ST>(x[j] * sv); }
+    }
+}
+inline bool gqa_prep_ok(int type, const pi_gqa_prep & p) {
+    return p.z && p.cs && p.q && p.cache && p.cell && p.T > 0 && p.n_head > 0 && p.n_kv > 0 && p.n_head % p.n_kv == 0 && p.rot_dim >= 0 && p.rot_dim % 2 == 0 && p.rot_dim <= p.dim &&
+           p.hd == pi_k_gqa_head_ld(type, p.dim, p.vdim) && p.hd > 0 && p.off_k >= p.n_head * p.dim && p.off_k + p.n_kv * p.dim <= p.ldz && p.off_v >= 0 &&
+           p.off_v + p.n_kv * p.vdim <= p.ldz && !p.q_norm == !p.k_norm && !(p.q_norm && p.unit);
 }
 
 // ---- grouped-query attention: the parts of one row of a work item, by one wave (fixed order, the sink in the denominator) -------------
@@ -70,7 +134,7 @@ __device__ void gqa_merge_row(const pi_gqa_attn & p, int item_index, int g, int 
     const float m = fmaxf(pi_wave_max(ml.x), p.sink);
     const float e = ml.x == -INFINITY ? 0.0f : expf(ml.x - m);
     const float l = pi_wave_sum(e * ml.y) + expf(p.sink - m);
-    const float f = e / l;
+    const float f = e / l * p.out_scale;
     const int rr = item.y + r, head = g * per + rr % per;
     bf16 * out = (bf16 *)p.att + (size_t)(item.x + rr / per) * p.ld_att + head * p.vdim;
     for (int c0 = 0; c0 < p.vdim; c0 += 64) {            // (every lane stays in the loop: the factors are passed between lanes)
@@ -90,12 +154,41 @@ __device__ void gqa_merge_row(const pi_gqa_attn & p, int item_index, int g, int 
     }
 }
 
-// ---- gated norm of one token by one workgroup ------------------------------------------------------------------------------------------
-template <typename ST> __device__ void gate_norm_token(const pi_gate_norm & p, int t, double * red) {
+// ---- gated norm by a block of 256 threads: of one token, or (heads) of four of a token's heads, a wave each ------------------------------
+__host__ __device__ inline int gate_norm_blocks(const pi_gate_norm & p) { return p.heads > 0 ? p.T * ((p.heads + 3) / 4) : p.T; }
+template <typename ST> __device__ void gate_norm_heads(const pi_gate_norm & p, int t, int h) {
+    if (h >= p.heads) return;
+    const int vd = p.n / p.heads, lane = threadIdx.x & 63;
+    const float * o = p.o + (size_t)t * p.n + h * vd, * g = p.z + (size_t)t * p.ldz + p.off_gate + h * vd, * w = p.w + h * vd;
+    ST * out = (ST *)p.att + (size_t)t * p.ld_att + h * vd;
+    constexpr int J = 4;
+    const float den = p.den ? p.den[(size_t)t * p.heads + h] : 1.0f;
+    float v[J], gv[J], wv[J], ss = 0.0f;
+#pragma unroll
+    for (int j = 0; j < J; ++j) {
+        const int e = min(lane + 64 * j, vd - 1);
+        v[j] = o[e]; gv[j] = g[e]; wv[j] = w[e];
+    }
+#pragma unroll
+    for (int j = 0; j < J; ++j) {
+        v[j] /= den;
+        if (lane + 64 * j < vd) ss = fmaf(v[j], v[j], ss);
+    }
+    const float sc = pi_inv_sqrt(pi_wave_sum(ss) / (float)vd + p.eps) * p.scale;
+#pragma unroll
+    for (int j = 0; j < J; ++j) {
+        const int e = lane + 64 * j;
+        if (e < vd) out[e] = to_st<ST>(v[j] * sc * wv[j] * (p.silu ? silu_f32(gv[j]) : sigmoid_f32(gv[j])));
+    }
+}
+template <typename ST> __device__ void gate_norm_block(const pi_gate_norm & p, int b, double * red) {
+    if (p.heads > 0) { const int per = (p.heads + 3) / 4; gate_norm_heads<ST>(p, b / per, b % per * 4 + (threadIdx.x >> 6)); return; }
+    const int t = b;
     const float * o = p.o + (size_t)t * p.n, * g = p.z + (size_t)t * p.ldz + p.off_gate;
     ST * out = (ST *)p.att + (size_t)t * p.ld_att;
     constexpr int K = 16;
     const int nt = blockDim.x;
+    const auto gate = [&](float z) { return p.silu ? silu_f32(z) : sigmoid_f32(z); };
     if (p.n <= K * nt) {                              // one memory round trip: everything requested together, kept in registers
         float v[K], gv[K], wv[K];
         double s = 0.0;
@@ -107,22 +200,23 @@ template <typename ST> __device__ void gate_norm_token(const pi_gate_norm & p, i
 #pragma unroll
         for (int k = 0; k < K; ++k) if ((int)threadIdx.x + k * nt < p.n) s += (double)v[k] * (double)v[k];
         s = block_sum_f64(s, red);
-        const float sc = pi_inv_sqrt((float)(s / p.n) + p.eps);
+        const float sc = pi_inv_sqrt((float)(s / p.n) + p.eps) * p.scale;
 #pragma unroll
         for (int k = 0; k < K; ++k) {
             const int i = threadIdx.x + k * nt;
-            if (i < p.n) out[i] = to_st<ST>(v[k] * sc * wv[k] * sigmoid_f32(gv[k]));
+            if (i < p.n) out[i] = to_st<ST>(v[k] * sc * wv[k] * gate(gv[k]));
         }
         return;
     }
     double s = 0.0;
     for (int i = threadIdx.x; i < p.n; i += nt) s += (double)o[i] * (double)o[i];
     s = block_sum_f64(s, red);
-    const float sc = pi_inv_sqrt((float)(s / p.n) + p.eps);
-    for (int i = threadIdx.x; i < p.n; i += nt) out[i] = to_st<ST>(o[i] * sc * p.w[i] * sigmoid_f32(g[i]));
+    const float sc = pi_inv_sqrt((float)(s / p.n) + p.eps) * p.scale;
+    for (int i = threadIdx.x; i < p.n; i += nt) out[i] = to_st<ST>(o[i] * sc * p.w[i] * gate(g[i]));
 }
 inline bool gate_norm_ok(const pi_gate_norm & p) {
-    return p.o && p.z && p.w && p.att && p.n > 0 && p.T > 0 && p.off_gate >= 0 && p.off_gate + p.n <= p.ldz && p.ld_att >= p.n;
+    return p.o && p.z && p.w && p.att && p.n > 0 && p.T > 0 && p.off_gate >= 0 && p.off_gate + p.n <= p.ldz && p.ld_att >= p.n && p.heads >= 0 &&
+           (p.heads == 0 ? !p.den : p.n % p.heads == 0 && p.n / p.heads <= 256);
 }
 
 }  // namespace

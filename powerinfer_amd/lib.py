@@ -12,7 +12,8 @@ HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(HERE, "libpowerinfer_hip.so")
 
 F32, F16, Q4_0, I32, BF16 = 0, 1, 2, 18, 30
-MIXER_LATENT, MIXER_GROUPED, MIXER_LINEAR = 0, 1, 2
+MIXER_LATENT, MIXER_GROUPED, MIXER_LINEAR, MIXER_KEYED = 0, 1, 2, 3
+DECAY_CONST, DECAY_KEYED, DECAY_GATED = 0, 1, 2
 FFN_NONE, FFN_MOE, FFN_GLU, FFN_GLU_MOE = 0, 1, 2, 3
 EPI_NONE, EPI_RELU, EPI_ADD, EPI_ADD2 = 0, 1, 2, 3
 NORM_NONE, NORM_RMS, NORM_LAYER = 0, 1, 2
@@ -50,34 +51,41 @@ class LatentExpanded(C.Structure):
 
 class FfnFront(C.Structure):
     _fields_ = [(n, C.c_int32) for n in ("off_glu", "ff", "ff_ld", "off_score")] + [("limit", _f), ("gain", _f), ("act", _vp)] + [
-        (n, C.c_int32) for n in ("ld_act", "off_router", "n_expert", "n_top")] + [("ids", _vp), ("weights", _vp)]
+        (n, C.c_int32) for n in ("ld_act", "off_router", "n_expert", "n_top")] + [("ids", _vp), ("weights", _vp), ("plain_up", C.c_int32)]
 
 
 class GqaPrep(C.Structure):
     _fields_ = [("z", _vp)] + [(n, C.c_int32) for n in ("ldz", "T", "n_head", "n_kv", "dim", "vdim", "rot_dim", "off_k", "off_v", "hd", "unit")] + [
-        ("cs", _vp), ("eps", _f), ("q", _vp), ("cache", _vp), ("cell", _vp)]
+        ("cs", _vp), ("eps", _f), ("q", _vp), ("cache", _vp), ("cell", _vp), ("rot_pairs", C.c_int32), ("unit_v", C.c_int32), ("q_norm", _vp), ("k_norm", _vp), ("temp", _vp)]
 
 
 class GqaAttn(C.Structure):
     _fields_ = [("q", _vp), ("cache", _vp), ("lists", _vp), ("list_ld", _sz), ("work", _vp), ("n_vis", _vp)] + [
         (n, C.c_int32) for n in ("n_work", "T", "n_head", "n_kv", "dim", "vdim", "hd", "n_parts", "wide")] + [
-        ("scale", _f), ("sink", _f), ("scratch", _vp), ("att", _vp), ("ld_att", C.c_int32)]
+        ("scale", _f), ("sink", _f), ("scratch", _vp), ("att", _vp), ("ld_att", C.c_int32), ("out_scale", _f), ("window", C.c_int32), ("first", _vp)]
 
 
 class Linear(C.Structure):
     _fields_ = [("z", _vp)] + [(n, C.c_int32) for n in ("ldz", "T", "n_head", "dim", "vdim", "off_k", "off_v")] + [
         ("decay", _vp), ("powers", _vp), ("state", _vp), ("runs", _vp), ("n_runs", C.c_int32), ("o", _vp), ("q", _vp), ("k", _vp), ("v", _vp), ("states", _vp)] + [
-        (n, C.c_int32) for n in ("dim_ld", "vdim_ld", "n_chunks")] + [("chunks", _vp), ("first_chunk", _vp)]
+        (n, C.c_int32) for n in ("dim_ld", "vdim_ld", "n_chunks")] + [("chunks", _vp), ("first_chunk", _vp)] + [
+        (n, C.c_int32) for n in ("decay_kind", "off_q", "plain")] + [("q_scale", _f), ("slot_ld", _sz), ("a2", _vp), ("a2_b", _vp)] + [
+        (n, C.c_int32) for n in ("off_a", "rank", "rank_ld")] + [("tau", _f), ("i_b", _vp), ("f_b", _vp), ("off_i", C.c_int32), ("off_f", C.c_int32), ("cap", _f), ("den", _vp), ("gates", _vp)]
 
 
 class GateNorm(C.Structure):
-    _fields_ = [("o", _vp), ("z", _vp), ("w", _vp)] + [(n, C.c_int32) for n in ("ldz", "off_gate", "n", "T")] + [("eps", _f), ("att", _vp), ("ld_att", C.c_int32)]
+    _fields_ = [("o", _vp), ("z", _vp), ("w", _vp)] + [(n, C.c_int32) for n in ("ldz", "off_gate", "n", "T")] + [("eps", _f), ("att", _vp), ("ld_att", C.c_int32), ("scale", _f), ("heads", C.c_int32), ("silu", C.c_int32), ("den", _vp)]
 
 
 class LayerOut(C.Structure):
     _fields_ = [("x", _vp), ("wo", _vp), ("att", _vp), ("rows", C.c_int32), ("ld_att", C.c_int32), ("T", C.c_int32),
                 ("down", _vp), ("act", _vp), ("ids", _vp), ("ld_act", C.c_int32), ("top", C.c_int32), ("n_expert", C.c_int32),
-                ("out", _vp), ("keep", _vp)]
+                ("out", _vp), ("keep", _vp), ("scaled", C.c_int32), ("alpha", _f), ("gate_z", _vp), ("gate_b", _vp), ("ld_gate", C.c_int32), ("off_gate", C.c_int32)]
+
+
+class ResNorm(C.Structure):
+    _fields_ = [(n, _vp) for n in ("x", "mix", "gate_z", "gate_b", "w")] + [(n, C.c_int32) for n in ("ld_gate", "off_gate", "T", "cols")] + [
+        ("alpha", _f), ("eps", _f), ("out", _vp), ("keep", _vp), ("h", _vp), ("ld", C.c_int32), ("ol", C.c_int32)]
 
 
 class PiError(RuntimeError):
@@ -235,10 +243,17 @@ _SIGS = {
     "pi_k_gqa_scratch_floats": (_sz, [_i, _i, _i, _i, _i]),
     "pi_k_gqa_attn": (_i, [_i, C.POINTER(GqaAttn), _vp]),
     "pi_k_gqa_attn_parts": (_i, [C.POINTER(GqaAttn), _vp]),
-    "pi_k_gqa_shift": (_i, [_i, _vp, _i, _i, _i, _i, C.c_double, _vp, _vp]),
+    "pi_k_gqa_shift": (_i, [_i, _vp, _i, _i, _i, _i, C.c_double, _i, _vp, _vp]),
     "pi_k_linear_chunk": (_i, []),
     "pi_k_linear_supported": (_i, [_i, _i]),
     "pi_k_linear_states_bytes": (_sz, [_i, _i, _i, _i]),
+    "pi_k_linear_copies": (_i, [_i]),
+    "pi_k_linear_slot_floats": (_sz, [_i, _i, _i, _i]),
+    "pi_k_linear_gate_floats": (_sz, [_i, _i, _i, _i, _i]),
+    "pi_k_ffn_front": (_i, [_i, _vp, _i, _i, C.POINTER(FfnFront), _vp]),
+    "pi_k_linear_step_beside": (_i, [_i, C.POINTER(Linear), C.POINTER(GqaPrep), _vp]),
+    "pi_k_res_norm": (_i, [_i, C.POINTER(ResNorm), _vp]),
+    "pi_k_gemm_bf16_ol_glu": (_i, [_vp, _i, _vp, _f, _f, _f, _vp, _i, _vp, _i, _vp, _i, _i, _vp]),
     "pi_k_linear_step": (_i, [_i, C.POINTER(Linear), C.POINTER(FfnFront), _vp]),
     "pi_k_linear_prep": (_i, [_i, C.POINTER(Linear), C.POINTER(FfnFront), _vp]),
     "pi_k_linear_chunks": (_i, [C.POINTER(Linear), _vp]),

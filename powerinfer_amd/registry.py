@@ -20,7 +20,12 @@ def _pibalorn(config, tensors, **kw):
     return pibalorn.build(config, tensors, **kw)
 
 
-FOLDERS = {"Lerasun": _lerasun, "Pibalorn": _pibalorn}
+def _fikevik(config, tensors, **kw):
+    from . import fikevik
+    return fikevik.build(config, tensors, **kw)
+
+
+FOLDERS = {"Lerasun": _lerasun, "Pibalorn": _pibalorn, "Fikevik": _fikevik}
 
 
 def load_model(path, dtype="bfloat16", n_ctx=4096, max_batch=0):

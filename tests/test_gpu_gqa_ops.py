@@ -178,7 +178,7 @@ def attend(t, rng, seqs, H, G, dim, vdim, parts, wide, scale, sink, spike=()):
     qb, cb, lb, vb, att = store(qp, t), store(pad, t), i32(lists), i32(vis), pl.DevBuf.zeros(4 * T * ld)
     wb = i32(work if t == pl.BF16 else seq_of)
     scratch = pl.DevBuf(4 * max(L.pi_k_gqa_scratch_floats(len(work), wide, G, hd, parts), 1))
-    a = filled(pl.GqaAttn, q=qb, cache=cb, lists=lb, list_ld=list_ld, work=wb, n_vis=vb, n_work=len(work), T=T, n_head=H, n_kv=G, dim=dim, vdim=vdim, hd=hd, n_parts=parts, wide=wide,
+    a = filled(pl.GqaAttn, out_scale=1.0, q=qb, cache=cb, lists=lb, list_ld=list_ld, work=wb, n_vis=vb, n_work=len(work), T=T, n_head=H, n_kv=G, dim=dim, vdim=vdim, hd=hd, n_parts=parts, wide=wide,
                scale=scale, sink=sink, scratch=scratch, att=att, ld_att=ld)
     pl.check(L.pi_k_gqa_attn(t, C.byref(a), None))
     pl.sync()
@@ -240,7 +240,7 @@ def test_shifted_keys(t):
     cells[:, :, 0, :dim] = o.unit(o.rotate_halves(k, pos, rot, 800.0), 1e-5)
     cells[:, :, 1, :dim] = k
     cb, db = store(cells, t), i32(delta)
-    pl.check(L.pi_k_gqa_shift(t, cb.ptr, n, G, hd, rot, 800.0, db.ptr, None))
+    pl.check(L.pi_k_gqa_shift(t, cb.ptr, n, G, hd, rot, 800.0, 0, db.ptr, None))
     pl.sync()
     got = fetch(cb, t, cells.shape)
     assert np.abs(got[:, :, 0, :dim] - o.unit(o.rotate_halves(k, pos + delta, rot, 800.0), 1e-5)).max() < (2e-2 if t == pl.BF16 else 1e-5)
@@ -268,7 +268,7 @@ def test_step_launch_beside_the_experts(T, E, top, ff, cols, what):
     acc, ml = rng.standard_normal((T, 16, P, hd)).astype(np.float32), np.stack([3 * rng.standard_normal((T, 16, P)), 1 + rng.random((T, 16, P))], -1).astype(np.float32)
     ml[:, :, 2], acc[:, :, 2] = [-np.inf, 0], 0
     sb, kb, attm = dev(np.concatenate([acc.ravel(), ml.ravel()])), i32(work), pl.DevBuf.zeros(2 * T * (hv + 2))
-    merge = filled(pl.GqaAttn, work=kb, n_work=T, T=T, n_head=3, n_kv=1, dim=20, vdim=20, hd=hd, n_parts=P, wide=0, scale=1.0, sink=0.0, scratch=sb, att=attm, ld_att=hv + 2)
+    merge = filled(pl.GqaAttn, out_scale=1.0, work=kb, n_work=T, T=T, n_head=3, n_kv=1, dim=20, vdim=20, hd=hd, n_parts=P, wide=0, scale=1.0, sink=0.0, scratch=sb, att=attm, ld_att=hv + 2)
     with_gate, with_merge = what in ("gate", "both"), what in ("merge", "both")
     pl.check(L.pi_k_mix_up_step(C.byref(merge) if with_merge else None, C.byref(gate) if with_gate else None, ub.ptr, E, ff, cols, 0.9, 1.702, hb.ptr, T, ib.ptr if E else None, wb.ptr,
                                 top, act.ptr, ld, None))
@@ -301,7 +301,7 @@ def test_place():
 def test_bad_arguments_are_errors():
     L = pl.init()
     buf = pl.DevBuf.zeros(1 << 16)
-    a = filled(pl.GqaAttn, q=buf, cache=buf, lists=buf, list_ld=8, work=buf, n_vis=buf, n_work=1, T=1, n_head=3, n_kv=2, dim=32, vdim=32, hd=32, n_parts=1, scale=1.0, att=buf, ld_att=96)
+    a = filled(pl.GqaAttn, out_scale=1.0, q=buf, cache=buf, lists=buf, list_ld=8, work=buf, n_vis=buf, n_work=1, T=1, n_head=3, n_kv=2, dim=32, vdim=32, hd=32, n_parts=1, scale=1.0, att=buf, ld_att=96)
     assert L.pi_k_gqa_attn(pl.BF16, C.byref(a), None) != 0                 # heads are no multiple of the groups
     a.n_kv, a.hd = 3, 64
     assert L.pi_k_gqa_attn(pl.BF16, C.byref(a), None) != 0                 # not the row length of this head size

@@ -122,7 +122,7 @@ def test_gate_norm(t, T, n):
     L, rng = pl.init(), np.random.default_rng(n)
     x, z, w = rng.standard_normal((T, n)).astype(np.float32) * 4, rng.standard_normal((T, n + 9)).astype(np.float32), rng.random(n).astype(np.float32)
     xb, zb, wb, att = dev(x), dev(z), dev(w), pl.DevBuf.zeros(4 * T * (n + 4))
-    g = filled(pl.GateNorm, o=xb, z=zb, w=wb, ldz=n + 9, off_gate=4, n=n, T=T, eps=1e-5, att=att, ld_att=n + 4)
+    g = filled(pl.GateNorm, scale=1.0, o=xb, z=zb, w=wb, ldz=n + 9, off_gate=4, n=n, T=T, eps=1e-5, att=att, ld_att=n + 4)
     pl.check(L.pi_k_gate_norm(t, C.byref(g), None))
     pl.sync()
     want = o.unit(x.astype(np.float64), 1e-5) * w * o.sigmoid(z[:, 4:4 + n].astype(np.float64))
