@@ -686,8 +686,8 @@ PI_API int    pi_k_gqa_attn_parts(const pi_gqa_attn * p, pi_stream_t stream);
 /* rotates the key parts of cells by delta[cell] positions (pairs != 0: neighbouring values are a pair) */
 PI_API int pi_k_gqa_shift(int type, void * cache, int n_cells, int n_kv, int hd, int rot_dim, double base, int pairs, const int32_t * delta, pi_stream_t stream);
 /* Linear attention over a fp32 state [slot][n_head][dim][vdim] (slot_ld floats per slot, 0: exactly these), behind the joint projection
- * z [T][ldz]: q at off_q (n_head x dim), k at off_k, v at off_v (n_head x vdim); silu of each, or with plain != 0 the projections themselves and
- * q times q_scale.  decay_kind says what becomes of the state:
+ * z [T][ldz]: q at off_q (n_head x dim), k at off_k, v at off_v (n_head x vdim); silu of each, or with plain != 0 the projections themselves
+ * (pi_k_linear_step: unrounded) and q times q_scale.  decay_kind says what becomes of the state:
  *   PI_DECAY_CONST  S = d S + k v^T with d = decay[head], o = S^T q
  *   PI_DECAY_KEYED  S = diag(a) S + k v^T with a decay per key channel and token, a = sigmoid(u)^(1 / tau), u = a2 z[off_a ..] + a2_b;
  *                   a2 [n_head * dim][rank_ld] bf16, rank_ld a multiple of 8

@@ -22,6 +22,7 @@ constexpr int kItemRows = 32;             // query rows of an attention work ite
 constexpr int kAttnItems = 512;          // (work item, part) pairs a split attention aims at: two workgroups per compute unit
 constexpr int kWideRows = 64;            // query rows from which a run of grouped-query attention takes the wide work items
 constexpr int kLinearChunked = 17;       // tokens from which a run of linear attention is worked in chunks
+constexpr int kFreshSteps = 4;           // first tokens of a sequence that a norm over every head's sums is sensitive to (see layers_step)
 
 int up_to(int v, int m) { return (v + m - 1) / m * m; }
 
@@ -1316,6 +1317,9 @@ int layers_step(pi_model * m, const int32_t * tokens, const int32_t * positions,
             for (int a = 0; a < T;) {
                 int b = a + 1;
                 while (b < T && seq[t0 + b] == seq[t0 + a]) ++b;
+                // A sequence's first results are few products (q . k) v, of which a norm over the head leaves the direction: the less of q . k is
+                // rounded the better.  They are walked with unrounded projections, and the chunks begin behind them.
+                if (s->family == kPostNorm && bf16_mode(s) && (fresh >> seq[t0 + a] & 1u) && b - a >= kLinearChunked + kFreshSteps) b = a + kFreshSteps;
                 const int q = seq[t0 + a], new_state = fresh >> q & 1u;
                 const int32_t run[4] = {a, b - a, s->slot_of[q], new_state};
                 fresh &= ~(1u << q);                              // a later pass of this step goes on

@@ -21,8 +21,12 @@ __device__ __forceinline__ float keyed_log2(float u, float tau) { return log_sig
 __device__ __forceinline__ float soft_cap(float z, float cap) { return cap * tanhf(z / cap); }
 __device__ __forceinline__ float log_input_gate(const pi_linear & p, const float * z, int h) { return soft_cap(z[p.off_i + h] + p.i_b[h], p.cap); }
 __device__ __forceinline__ float log_forget_gate(const pi_linear & p, const float * z, int h) { return log_sigmoid_f32(soft_cap(z[p.off_f + h] + p.f_b[h], p.cap)); }
-// the value of a projection as the recurrence takes it
+// the value of a projection as the recurrence takes it; walked token by token it is rounded to the activations' storage only behind an activation
 __device__ __forceinline__ float lin_value(const pi_linear & p, float z, bool query) { return p.plain ? (query ? z * p.q_scale : z) : silu_f32(z); }
+template <typename ST> __device__ __forceinline__ float lin_operand(const pi_linear & p, float z, bool query) {
+    const float v = lin_value(p, z, query);
+    return p.plain ? v : from_st(to_st<ST>(v));
+}
 __device__ __forceinline__ float lin_den(float nq, float m) { return fmaxf(fabsf(nq), expf(-m)) + 1e-6f; }
 // places of the sum of keys and of the copies of the running maximum inside a slot
 __host__ __device__ inline int lin_copies(int vdim) { return (vdim + kLinCols - 1) / kLinCols; }
@@ -73,8 +77,8 @@ __global__ __launch_bounds__(256) void linear_step_kernel(pi_linear p, pi_ffn_fr
         for (int e = tid; e < n * D; e += 256) {
             const int t = e / D, r = e % D;
             const float * zt = p.z + (size_t)(run.x + t0 + t) * p.ldz, * z = zt + h * p.dim + r;
-            qs[e] = r < p.dim ? from_st(to_st<ST>(lin_value(p, z[p.off_q], true))) : 0.0f;
-            ks[e] = r < p.dim ? from_st(to_st<ST>(lin_value(p, z[p.off_k], false))) : 0.0f;
+            qs[e] = r < p.dim ? lin_operand<ST>(p, z[p.off_q], true) : 0.0f;
+            ks[e] = r < p.dim ? lin_operand<ST>(p, z[p.off_k], false) : 0.0f;
             if constexpr (MODE == kKeyed) {
                 float a = 0.0f;
                 if (r < p.dim) {
@@ -93,7 +97,7 @@ __global__ __launch_bounds__(256) void linear_step_kernel(pi_linear p, pi_ffn_fr
         }
         for (int e = tid; e < n * kLinCols; e += 256) {
             const int t = e / kLinCols, v = slice * kLinCols + e % kLinCols;
-            vs[e] = v < p.vdim ? from_st(to_st<ST>(lin_value(p, p.z[(size_t)(run.x + t0 + t) * p.ldz + p.off_v + h * p.vdim + v], false))) : 0.0f;
+            vs[e] = v < p.vdim ? lin_operand<ST>(p, p.z[(size_t)(run.x + t0 + t) * p.ldz + p.off_v + h * p.vdim + v], false) : 0.0f;
         }
         if (MODE == kGated && tid < n) {
             const float * z = p.z + (size_t)(run.x + t0 + tid) * p.ldz;
@@ -202,6 +206,9 @@ __device__ __forceinline__ float * lin_chunk_tops(const pi_linear & p) { return 
 // sums of keys ahead of every chunk, behind the states: [chunk][head][hi, lo][dim_ld]
 __device__ __forceinline__ bf16 * lin_chunk_keys(const pi_linear & p) { return (bf16 *)p.states + (size_t)p.n_chunks * p.n_head * 2 * p.vdim_ld * p.dim_ld; }
 
+// log2 of the smallest decay of one token: what it leaves is far below fp32's last place, and the sums stay small enough to tell the
+// decays of the tokens behind it apart
+constexpr float kLinForgotten = -100.0f;
 // a workgroup per (chunk, 256 key channels of all heads): the second factor of the low-rank projection, 16 tokens at a time
 __global__ __launch_bounds__(256) void linear_decays_kernel(pi_linear p, int n_blocks) {
     extern __shared__ __align__(16) float us[];              // [64][rank_ld]
@@ -235,7 +242,7 @@ __global__ __launch_bounds__(256) void linear_decays_kernel(pi_linear p, int n_b
         }
 #pragma unroll
         for (int t = 0; t < 16; ++t) {
-            sum += keyed_log2(acc[t], p.tau);
+            sum += fmaxf(keyed_log2(acc[t], p.tau), kLinForgotten);
             if (t0 + t < n) out[(size_t)(t0 + t) * all] = real ? sum : 0.0f;
         }
     }

@@ -131,9 +131,10 @@ def empty_memory(m):
 
 
 def memory_reads(q, k, v, i, f, memory):
-    """q, k [n, H, dim], v [n, H, vdim], i, f [n, H], memory (S [H, dim, vdim], sum of keys [H, dim], running maximum [H])."""
+    """q, k [n, H, dim], v [n, H, vdim], i, f [n, H], memory (S [H, dim, vdim], sum of keys [H, dim], running maximum [H]).
+    memory_reads.den: what each read was divided by."""
     s, z, m = memory
-    out = []
+    out, dens = [], []
     for t in range(q.shape[0]):
         top = np.maximum(f[t] + m, i[t])
         keep, add = np.exp(f[t] + m - top), np.exp(i[t] - top)
@@ -141,7 +142,9 @@ def memory_reads(q, k, v, i, f, memory):
         z = keep[:, None] * z + add[:, None] * k[t]
         m = top
         den = np.maximum(np.abs((z * q[t]).sum(-1)), np.exp(-m)) + 1e-6
+        dens.append(den)
         out.append(np.einsum("hdv,hd->hv", s, q[t]) / den[:, None])
+    memory_reads.den = np.asarray(dens)
     return np.asarray(out).reshape(q.shape[0], *v.shape[1:]), (s, z, m)
 
 
@@ -194,6 +197,10 @@ class PlainModel:
         right, self.state[i] = matrix_memory(h, self.sub(p + "right."), m["right"], eps, self.state.get(i, empty_memory(m["right"])))
         return side_by_side(left, right, m)
 
+    def operand(self, x):
+        """What the sublayers read of the residual stream."""
+        return x
+
     def feed(self, tokens):
         """Logits [n, vocab] of the next tokens of the sequence; self.streams: the residual stream after every layer."""
         eps, alpha, t = self.c["norm"]["eps"], self.c["postln_alpha"], self.t
@@ -204,9 +211,11 @@ class PlainModel:
         self.streams = []
         for i, ly in enumerate(self.c["layers"]):
             p = f"l{self.owner(i)}."
-            x = norm_after_sum(x, gated(self.mix(i, x, pos), x, t[p + "rg1"], t[p + "rg1.b"]), alpha, t[p + "norm1"], eps)
+            h = self.operand(x)
+            x = norm_after_sum(x, gated(self.mix(i, h, pos), h, t[p + "rg1"], t[p + "rg1.b"]), alpha, t[p + "norm1"], eps)
             if ly["mlp"] is not None:
-                y = swiglu(x, t[p + "mlp.gate"], t[p + "mlp.up"], t[p + "mlp.down"])
-                x = norm_after_sum(x, gated(y, x, t[p + "rg2"], t[p + "rg2.b"]), alpha, t[p + "norm2"], eps)
+                h = self.operand(x)
+                y = swiglu(h, t[p + "mlp.gate"], t[p + "mlp.up"], t[p + "mlp.down"])
+                x = norm_after_sum(x, gated(y, h, t[p + "rg2"], t[p + "rg2.b"]), alpha, t[p + "norm2"], eps)
             self.streams.append(x)
         return rms_norm(x, t["final.norm"], eps) @ t["head"].T

@@ -139,9 +139,10 @@ def test_gqa_prep_and_front(t, H, G, dim, vdim, rot, unit, ff, E, top):
     check_front(z, t, f, bufs)
 
 
-def attend(t, rng, seqs, H, G, dim, vdim, parts, wide, scale, sink, spike=()):
+def attend(t, rng, seqs, H, G, dim, vdim, parts, wide, scale, sink, spike=(), window=0, first=None, out_scale=1.0):
     """seqs: (tokens of the step, cells before them) per sequence.  Runs pi_k_gqa_attn on scattered cells; returns (got, want) [T, H, vdim].
-    spike: (sequence, token, cell, head) whose score is made to stand out."""
+    spike: (sequence, token, cell, head) whose score is made to stand out.  window, first (a function of sequence and token): what the tokens
+    see (without the soft-max's own entry)."""
     L = pl.init()
     hd, per, T = L.pi_k_gqa_head_ld(t, dim, vdim), H // G, sum(n for n, _ in seqs)
     pool = sum(n + b for n, b in seqs) + 7
@@ -164,7 +165,8 @@ def attend(t, rng, seqs, H, G, dim, vdim, parts, wide, scale, sink, spike=()):
         k, v = cache[cells][:, :, 0, :dim].astype(np.float64), cache[cells][:, :, 1, :vdim].astype(np.float64)
         if sink == -np.inf:
             for a in range(H):
-                sc = np.where(np.arange(n + b)[None] <= np.arange(b, b + n)[:, None], q[at:at + n, a].astype(np.float64) @ k[:, a // per].T * scale, -np.inf)
+                lo = np.array([first(s, i) if first else max(b + i + 1 - window, 0) if window else 0 for i in range(n)])[:, None]
+                sc = np.where((np.arange(n + b)[None] <= np.arange(b, b + n)[:, None]) & (np.arange(n + b)[None] >= lo), q[at:at + n, a].astype(np.float64) @ k[:, a // per].T * scale, -np.inf)
                 e = np.exp(sc - sc.max(1, keepdims=True))
                 want[at:at + n, a] = e / e.sum(1, keepdims=True) @ v[:, a // per]
         else:
@@ -177,14 +179,15 @@ def attend(t, rng, seqs, H, G, dim, vdim, parts, wide, scale, sink, spike=()):
     ld = H * vdim + 5
     qb, cb, lb, vb, att = store(qp, t), store(pad, t), i32(lists), i32(vis), pl.DevBuf.zeros(4 * T * ld)
     wb = i32(work if t == pl.BF16 else seq_of)
+    fb = i32([first(s, i) for s, (n, _) in enumerate(seqs) for i in range(n)]) if first else None
     scratch = pl.DevBuf(4 * max(L.pi_k_gqa_scratch_floats(len(work), wide, G, hd, parts), 1))
-    a = filled(pl.GqaAttn, out_scale=1.0, q=qb, cache=cb, lists=lb, list_ld=list_ld, work=wb, n_vis=vb, n_work=len(work), T=T, n_head=H, n_kv=G, dim=dim, vdim=vdim, hd=hd, n_parts=parts, wide=wide,
+    a = filled(pl.GqaAttn, out_scale=out_scale, window=window, first=fb, q=qb, cache=cb, lists=lb, list_ld=list_ld, work=wb, n_vis=vb, n_work=len(work), T=T, n_head=H, n_kv=G, dim=dim, vdim=vdim, hd=hd, n_parts=parts, wide=wide,
                scale=scale, sink=sink, scratch=scratch, att=att, ld_att=ld)
     pl.check(L.pi_k_gqa_attn(t, C.byref(a), None))
     pl.sync()
     got = fetch(att, t, (T, ld))
     assert not got[:, H * vdim:].any()
-    return got[:, :H * vdim].reshape(T, H, vdim), want
+    return got[:, :H * vdim].reshape(T, H, vdim), want * out_scale
 
 
 SHAPES = [(6, 2, 96, 96), (5, 1, 17, 17), (4, 4, 32, 20), (8, 1, 64, 64), (16, 2, 128, 128), (3, 3, 130, 130), (40, 2, 40, 64), (2, 1, 256, 250)]
@@ -261,7 +264,7 @@ def test_step_launch_beside_the_experts(T, E, top, ff, cols, what):
     n, hv = 90, 3 * 20
     og, zg, wg, attg = rng.standard_normal((T, n)).astype(np.float32), rng.standard_normal((T, n + 7)).astype(np.float32), rng.random(n).astype(np.float32), pl.DevBuf.zeros(2 * T * (n + 6))
     ob, zb, nb = dev(og), dev(zg), dev(wg)
-    gate = filled(pl.GateNorm, o=ob, z=zb, w=nb, ldz=n + 7, off_gate=5, n=n, T=T, eps=1e-5, att=attg, ld_att=n + 6)
+    gate = filled(pl.GateNorm, scale=1.0, o=ob, z=zb, w=nb, ldz=n + 7, off_gate=5, n=n, T=T, eps=1e-5, att=attg, ld_att=n + 6)
     # parts of an attention: 3 heads of one group, 5 parts, one of them empty
     P, hd = 5, 32
     work = np.array([[t, 0, 3, 0] for t in range(T)], np.int32)
