@@ -416,6 +416,78 @@ def build_pibalorn_on_device(width, sh, n_ctx, keep):
     return m
 
 
+# shapes of --design fikevik: eight layers, gated linear attention and attention beside a matrix memory in turn, the last two on the weights of the
+# two before them, beside Pibalorn of equal width and depth (eight layer runs)
+FIKEVIK_SHAPES = {
+    2048: dict(heads=16, kv_heads=4, dim=128, window=1024, lin_heads=16, lin_dim=128, rank=16, mem_heads=16, mem_dim=128, ff=5632, beside=2048),
+    4096: dict(heads=32, kv_heads=8, dim=128, window=1024, lin_heads=32, lin_dim=128, rank=16, mem_heads=32, mem_dim=128, ff=11008, beside=4096),
+    5120: dict(heads=40, kv_heads=8, dim=128, window=1024, lin_heads=40, lin_dim=128, rank=16, mem_heads=40, mem_dim=128, ff=13824, beside=5120),
+}
+
+
+def build_fikevik_on_device(width, sh, n_ctx, keep):
+    """Random-init weights of a Fikevik shape generated in HBM."""
+    from powerinfer_amd import lib as pl, fikevik
+    from powerinfer_amd.model import LayerModel
+    L = pl.init()
+    V, dim, f32 = 32000, sh["dim"], np.float32
+    mlp = {"kind": "dense", "ff": sh["ff"]}
+    lin = {"type": "gla", "mixer": {"heads": sh["lin_heads"], "dim": sh["lin_dim"], "vdim": sh["lin_dim"], "tau": 16.0}, "mlp": mlp}
+    par = {"type": "parallel", "mlp": mlp, "mixer": {
+        "left": {"heads": sh["heads"], "kv_heads": sh["kv_heads"], "dim": dim, "vdim": dim, "rot": {"dims": dim, "base": 10000.0}, "scale": dim ** -0.5, "mask": {"size": sh["window"]}},
+        "right": {"heads": sh["mem_heads"], "dim": sh["mem_dim"], "vdim": sh["mem_dim"], "gate_cap": 15.0}, "left_scale": 0.7, "right_scale": 0.7}}
+    cfg = {"width": width, "vocab": V, "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0}, "postln_alpha": 2.0,
+           "layers": [lin, par, lin, par, lin, par, dict(lin, weights_of=4), dict(par, weights_of=5)]}
+    ranks = {f"l{i}.mix.a1": np.empty((sh["rank"], width), f32) for i in range(0, 8, 2)}
+    descs = fikevik.layer_descs(cfg, ranks)
+    m = LayerModel("fikevik", descs, n_embd=width, n_vocab=V, n_ctx=n_ctx, norm_eps=1e-6, **fikevik.model_opts(cfg))
+    seed = [7]
+
+    def put(layer, kind, rows, cols):
+        seed[0] += 1
+        buf = pl.DevBuf(rows * cols * 2)
+        pl.check(L.pi_fill_normal_bf16(buf.ptr, rows * cols, seed[0], 0.02, None), "fill")
+        m.set_tensor_device(layer, kind, buf.ptr, pl.BF16, cols, rows)
+        keep.append(buf)
+
+    one, zero = np.ones(width, f32), np.zeros(width, f32)
+    put(-1, "tok_embd", V, width)
+    put(-1, "output", V, width)
+    m.set_tensor(-1, "output_norm", one)
+    for i, d in enumerate(descs):
+        if d["weights_of"]:
+            continue
+        H, hv = d["n_head"], d["n_head"] * d["vdim"]
+        for part, norm in (("res_gate", "attn_norm"), ("res_gate_ffn", "ffn_norm")):
+            m.set_tensor(i, norm, one)
+            put(i, part, width, width)
+            m.set_tensor(i, part + "_b", zero)
+        put(i, "mix_q", H * d["dim"], width)
+        if d["mixer"] == pl.MIXER_GROUPED:
+            put(i, "mix_k", d["n_kv_head"] * d["dim"], width)
+            put(i, "mix_v", d["n_kv_head"] * d["vdim"], width)
+            for k, n in (("mix_q_norm", d["dim"]), ("mix_k_norm", d["dim"]), ("mix_temp", H), ("mem_norm", d["mem_heads"] * d["mem_vdim"])):
+                m.set_tensor(i, k, np.ones(n, f32))
+            M = d["mem_heads"]
+            for k, rows in (("mem_q", M * d["mem_dim"]), ("mem_k", M * d["mem_dim"]), ("mem_v", M * d["mem_vdim"]), ("mem_g", M * d["mem_vdim"]), ("mem_i", M), ("mem_f", M)):
+                put(i, k, rows, width)
+            m.set_tensor(i, "mem_i_b", np.zeros(M, f32))
+            m.set_tensor(i, "mem_f_b", np.full(M, 4, f32))
+            put(i, "mem_o", width, M * d["mem_vdim"])
+        else:
+            for k, rows in (("mix_k", H * d["dim"]), ("mix_v", hv), ("mix_g", hv), ("mix_a1", sh["rank"])):
+                put(i, k, rows, width)
+            put(i, "mix_a2", H * d["dim"], sh["rank"])
+            m.set_tensor(i, "mix_a2_b", np.zeros(H * d["dim"], f32))
+            m.set_tensor(i, "mix_norm", np.ones(hv, f32))
+        put(i, "wo", width, hv)
+        for k, rows, cols in (("glu_gate", sh["ff"], width), ("glu_up", sh["ff"], width), ("glu_down", width, sh["ff"])):
+            put(i, k, rows, cols)
+    pl.sync()
+    m.finalize()
+    return m
+
+
 def time_prefill_and_decode(m, n_prompt, steps, warmup):
     """(prompt seconds, seconds per decoded token) of one sequence: the prompt through Model.decode (second pass timed), then the greedy loop."""
     from powerinfer_amd import lib as pl
@@ -451,12 +523,12 @@ def time_lockstep(m, n_seq, n_prompt, steps, warmup):
 
 def bench_design(args):
     """Prefill and decode of a design described layer by layer at sizes like a real model's, beside the closest existing model at equal width
-    and depth: the sparse LLaMA engine for Lerasun, Lerasun for Pibalorn."""
+    and depth: the sparse LLaMA engine for Lerasun, Lerasun for Pibalorn, Pibalorn for Fikevik."""
     from powerinfer_amd import lib as pl, synth
     pl.init()
     n_prompt, steps, lock_prompt = (2048 if args.prompt == 64 else args.prompt), min(args.steps, 128), 128
     n_ctx = n_prompt + steps + args.warmup + 8
-    shapes = DESIGN_SHAPES if args.design == "lerasun" else PIBALORN_SHAPES
+    shapes = {"lerasun": DESIGN_SHAPES, "pibalorn": PIBALORN_SHAPES, "fikevik": FIKEVIK_SHAPES}[args.design]
     rows = []
     for width in ([args.design_width] if args.design_width else sorted(shapes)):
         sh = shapes[width]
@@ -465,7 +537,11 @@ def bench_design(args):
             if args.design_only and who != args.design_only:
                 continue
             keep = []
-            if who == "pibalorn":
+            if who == "fikevik":
+                m = build_fikevik_on_device(width, sh, n_ctx, keep)
+            elif args.design == "fikevik":
+                m = build_pibalorn_on_device(width, PIBALORN_SHAPES[sh["beside"]], n_ctx, keep)
+            elif who == "pibalorn":
                 m = build_pibalorn_on_device(width, sh, n_ctx, keep)
             elif who == "lerasun":
                 m = build_lerasun_on_device(width, sh, n_ctx, keep)
@@ -493,9 +569,9 @@ def bench_design(args):
 
 def main():
     ap = argparse.ArgumentParser()
-    ap.add_argument("--design", choices=["lerasun", "pibalorn"], default=None, help="instead of the default workload: prefill and decode of this design beside the closest existing model")
+    ap.add_argument("--design", choices=["lerasun", "pibalorn", "fikevik"], default=None, help="instead of the default workload: prefill and decode of this design beside the closest existing model")
     ap.add_argument("--design-width", type=int, default=None, choices=sorted(DESIGN_SHAPES), help="one size of --design only")
-    ap.add_argument("--design-only", choices=["lerasun", "pibalorn", "beside"], default=None, help="one side of --design only")
+    ap.add_argument("--design-only", choices=["lerasun", "pibalorn", "fikevik", "beside"], default=None, help="one side of --design only")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=256)
     ap.add_argument("--warmup", type=int, default=8)

@@ -690,7 +690,7 @@ PI_API int pi_k_gqa_shift(int type, void * cache, int n_cells, int n_kv, int hd,
  * (pi_k_linear_step: unrounded) and q times q_scale.  decay_kind says what becomes of the state:
  *   PI_DECAY_CONST  S = d S + k v^T with d = decay[head], o = S^T q
  *   PI_DECAY_KEYED  S = diag(a) S + k v^T with a decay per key channel and token, a = sigmoid(u)^(1 / tau), u = a2 z[off_a ..] + a2_b;
- *                   a2 [n_head * dim][rank_ld] bf16, rank_ld a multiple of 8
+ *                   a2 [n_head * dim][rank_ld] bf16, rank_ld a multiple of 8 (zeros behind the rank, where z is read as well)
  *   PI_DECAY_GATED  exponential gates per head with a running maximum: i = cap tanh((z[off_i + head] + i_b) / cap),
  *                   f = log sigmoid(cap tanh((z[off_f + head] + f_b) / cap)), m' = max(f + m, i), S = exp(f + m - m') S + exp(i - m') k v^T, the sum n of
  *                   keys likewise, o = S^T q and den [T][n_head] = max(|n . q|, exp(-m')) + 1e-6, by which o has still to be divided.

@@ -9,7 +9,7 @@ __global__ __launch_bounds__(256) void gqa_prep_kernel(pi_gqa_prep p, pi_ffn_fro
     extern __shared__ __align__(16) float sm[];
     const int t = blockIdx.x / per, b = blockIdx.x % per;
     if (b >= n_heads4) front_block<ST>(f, p.z, p.ldz, t, b - n_heads4, sm);
-    else gqa_prep_heads<ST>(p, t, b);
+    else gqa_prep_block<ST>(p, t, b);
 }
 
 // the first cell a token sees

@@ -16,8 +16,13 @@ constexpr int kLinMaxRank = 512;         // of the projection that key decays co
 constexpr float kLog2E = 1.44269504088896340736f;
 
 __device__ __forceinline__ float log_sigmoid_f32(float z) { return fminf(z, 0.0f) - log1pf(expf(-fabsf(z))); }
-// log2 of the decay of a key channel
+__device__ __forceinline__ float lin_exp2(float v) { return __builtin_amdgcn_exp2f(v); }
+// log2 of the decay of a key channel; the quick form's error is of the order of fp32's last place of one, not of the result
 __device__ __forceinline__ float keyed_log2(float u, float tau) { return log_sigmoid_f32(u) / tau * kLog2E; }
+__device__ __forceinline__ float keyed_log2_quick(float u, float per_tau) {
+    const float a = u * kLog2E;
+    return (fminf(a, 0.0f) - __builtin_amdgcn_logf(1.0f + lin_exp2(-fabsf(a)))) * per_tau;
+}
 __device__ __forceinline__ float soft_cap(float z, float cap) { return cap * tanhf(z / cap); }
 __device__ __forceinline__ float log_input_gate(const pi_linear & p, const float * z, int h) { return soft_cap(z[p.off_i + h] + p.i_b[h], p.cap); }
 __device__ __forceinline__ float log_forget_gate(const pi_linear & p, const float * z, int h) { return log_sigmoid_f32(soft_cap(z[p.off_f + h] + p.f_b[h], p.cap)); }
@@ -51,7 +56,7 @@ __global__ __launch_bounds__(256) void linear_step_kernel(pi_linear p, pi_ffn_fr
     if ((int)blockIdx.x >= n_state) {
         const int b = blockIdx.x - n_state;
         if (b < n_front) front_block<ST>(f, p.z, p.ldz, b / per, b % per, sm);
-        else gqa_prep_heads<ST>(beside, (b - n_front) / per_beside, (b - n_front) % per_beside);
+        else gqa_prep_block<ST>(beside, (b - n_front) / per_beside, (b - n_front) % per_beside);
         return;
     }
     float * qs = sm, * ks = qs + kLinBlock * D, * vs = ks + kLinBlock * D, * part = vs + kLinBlock * kLinCols;      // [16][D], [16][D], [16][32], [4][16][32]
@@ -66,9 +71,15 @@ __global__ __launch_bounds__(256) void linear_step_kernel(pi_linear p, pi_ffn_fr
     const bool sums = MODE == kGated && slice == 0;
 #pragma unroll
     for (int j = 0; j < J; ++j) {
+        const int r = min(rg * J + j, p.dim - 1);              // (no guard around a load)
+        s[j] = S[(size_t)r * p.vdim + min(col, p.vdim - 1)];
+        if constexpr (MODE == kGated) nk[j] = lin_keys(p, slot, h)[r];
+    }
+#pragma unroll
+    for (int j = 0; j < J; ++j) {
         const int r = rg * J + j;
-        s[j] = !run.w && r < p.dim && col < p.vdim ? S[(size_t)r * p.vdim + col] : 0.0f;
-        if constexpr (MODE == kGated) nk[j] = sums && !run.w && r < p.dim ? lin_keys(p, slot, h)[r] : 0.0f;
+        if (run.w || r >= p.dim || col >= p.vdim) s[j] = 0.0f;
+        if constexpr (MODE == kGated) if (run.w || r >= p.dim || !sums) nk[j] = 0.0f;
     }
     if constexpr (MODE == kGated) top = run.w ? 0.0f : lin_tops(p, slot, h)[slice];
     for (int t0 = 0; t0 < run.y; t0 += kLinBlock) {
@@ -88,7 +99,7 @@ __global__ __launch_bounds__(256) void linear_step_kernel(pi_linear p, pi_ffn_fr
                     for (int k = 0; k < p.rank_ld; k += 8) {
                         const Frag<float> wf = frag_weights<float>(w + k);
 #pragma unroll
-                        for (int i = 0; i < 8; ++i) b = fmaf(wf.v[i], k + i < p.rank ? u[k + i] : 0.0f, b);
+                        for (int i = 0; i < 8; ++i) b = fmaf(wf.v[i], u[k + i], b);        // (behind the rank: zeros of a2)
                     }
                     a = exp2f(keyed_log2(b, p.tau));
                 }
@@ -199,8 +210,9 @@ __global__ __launch_bounds__(256) void linear_prep_kernel(pi_linear p, pi_ffn_fr
 // ---------------------------------------------------------------------------------------------------------------------------------
 constexpr int kLinC = 64;                // tokens of a chunk
 // what pi_linear::gates holds.  Keyed: [T][n_head][dim_ld] sums of log2 decays from the chunk's start on (fp32).  Gated: with F the sum of log
-// forget gates from the chunk's start on, i the log input gate and m the running maximum, per (token, head) {F - m, i - F, m, -}, and
-// behind them m ahead of every chunk [n_chunks][n_head].
+// forget gates from the chunk's start on and i the log input gate, per (token, head) {F, i - F, largest i - F since the chunk's start, -},
+// and behind them the running maximum m ahead of every chunk [n_chunks][n_head].  With m0 ahead of the chunk the maximum at a token is
+// m = F + max(m0, largest i - F), so that only the few numbers per chunk depend on what came before it.
 __device__ __forceinline__ const float4 * lin_gates(const pi_linear & p) { return (const float4 *)p.gates; }
 __device__ __forceinline__ float * lin_chunk_tops(const pi_linear & p) { return p.gates + (size_t)4 * p.T * p.n_head; }
 // sums of keys ahead of every chunk, behind the states: [chunk][head][hi, lo][dim_ld]
@@ -223,7 +235,7 @@ __global__ __launch_bounds__(256) void linear_decays_kernel(pi_linear p, int n_b
     const bool real = r < p.dim;
     const int row = h * p.dim + (real ? r : 0);
     const uint16_t * w = (const uint16_t *)p.a2 + (size_t)row * p.rank_ld;
-    const float bias = p.a2_b[row];
+    const float bias = p.a2_b[row], per_tau = 1.0f / p.tau;
     float * out = p.gates + (size_t)tok0 * all + ch;
     float sum = 0.0f;
     for (int t0 = 0; t0 < n; t0 += 16) {
@@ -242,44 +254,32 @@ __global__ __launch_bounds__(256) void linear_decays_kernel(pi_linear p, int n_b
         }
 #pragma unroll
         for (int t = 0; t < 16; ++t) {
-            sum += fmaxf(keyed_log2(acc[t], p.tau), kLinForgotten);
+            sum += fmaxf(keyed_log2_quick(acc[t], per_tau), kLinForgotten);
             if (t0 + t < n) out[(size_t)(t0 + t) * all] = real ? sum : 0.0f;
         }
     }
 }
 
-// a wave per (run, head) walks the run's chunks, a lane per token
-__global__ __launch_bounds__(256) void linear_gates_kernel(pi_linear p) {
-    const int h = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63, ri = blockIdx.y;
-    if (h >= p.n_head) return;
-    const int4 run = reinterpret_cast<const int4 *>(p.runs)[ri];
-    const int n_chunk = (run.y + kLinC - 1) / kLinC, last = run.x + run.y - 1;
-    float * tops = lin_tops(p, lin_slot(p, run.z), h);
-    float top = run.w ? 0.0f : tops[0];
-    float zi, zf;
-    const float ib = p.i_b[h], fb = p.f_b[h];
-    auto fetch = [&](int ck) {
-        const float * z = p.z + (size_t)min(run.x + ck * kLinC + lane, last) * p.ldz + h;
-        zi = z[p.off_i]; zf = z[p.off_f];
-    };
-    fetch(0);
-    for (int ck = 0; ck < n_chunk; ++ck) {
-        const int t = run.x + ck * kLinC + lane;
-        const bool real = t <= last;
-        const float i = real ? soft_cap(zi + ib, p.cap) : -INFINITY;
-        float F = real ? log_sigmoid_f32(soft_cap(zf + fb, p.cap)) : 0.0f;
-        fetch(ck + 1);                                       // past the last chunk: the last token again, not used
-#pragma unroll
-        for (int o = 1; o < PI_WAVE; o <<= 1) { const float v = __shfl_up(F, o, PI_WAVE); if (lane >= o) F += v; }
-        float best = i - F;
-#pragma unroll
-        for (int o = 1; o < PI_WAVE; o <<= 1) { const float v = __shfl_up(best, o, PI_WAVE); if (lane >= o) best = fmaxf(best, v); }
-        const float m = F + fmaxf(top, best);
-        if (real) reinterpret_cast<float4 *>(p.gates)[(size_t)t * p.n_head + h] = make_float4(F - m, i - F, m, 0.0f);
-        if (lane == 0) lin_chunk_tops(p)[(size_t)(p.first_chunk[ri] + ck) * p.n_head + h] = top;
-        top = __shfl(m, min(last - run.x - ck * kLinC, PI_WAVE - 1), PI_WAVE);
+// a wave per (chunk, head), a lane per token; the workgroups behind them hand the slots' maxima to their runs' first chunks
+__global__ __launch_bounds__(256) void linear_gates_kernel(pi_linear p, int h4) {
+    const int lane = threadIdx.x & 63;
+    if ((int)blockIdx.x >= p.n_chunks * h4) {
+        const int ri = blockIdx.x - p.n_chunks * h4;
+        const int4 run = reinterpret_cast<const int4 *>(p.runs)[ri];
+        for (int h = threadIdx.x; h < p.n_head; h += 256) lin_chunk_tops(p)[(size_t)p.first_chunk[ri] * p.n_head + h] = run.w ? 0.0f : lin_tops(p, lin_slot(p, run.z), h)[0];
+        return;
     }
-    for (int k = lane; k < lin_copies(p.vdim); k += PI_WAVE) tops[k] = top;
+    const int ck = blockIdx.x / h4, h = blockIdx.x % h4 * 4 + (int)(threadIdx.x >> 6), tok0 = p.chunks[3 * ck], n = p.chunks[3 * ck + 1];
+    if (h >= p.n_head) return;
+    const float * z = p.z + (size_t)(tok0 + min(lane, n - 1)) * p.ldz;
+    const float i = log_input_gate(p, z, h);
+    float F = log_forget_gate(p, z, h);
+#pragma unroll
+    for (int o = 1; o < PI_WAVE; o <<= 1) { const float v = __shfl_up(F, o, PI_WAVE); if (lane >= o) F += v; }
+    float best = i - F;
+#pragma unroll
+    for (int o = 1; o < PI_WAVE; o <<= 1) { const float v = __shfl_up(best, o, PI_WAVE); if (lane >= o) best = fmaxf(best, v); }
+    if (lane < n) reinterpret_cast<float4 *>(p.gates)[(size_t)(tok0 + lane) * p.n_head + h] = make_float4(F, i - F, best, 0.0f);
 }
 
 // ---------------------------------------------------------------------------------------------------------------------------------
@@ -307,7 +307,6 @@ __device__ __forceinline__ void lin_split8(const pi_u32x4 & x, const float (&f)[
     hi = __builtin_bit_cast(pi_u32x4, h);
     lo = __builtin_bit_cast(pi_u32x4, l);
 }
-__device__ __forceinline__ float lin_exp2(float v) { return __builtin_amdgcn_exp2f(v); }
 
 // states: per (chunk, head) the state before the chunk, transposed, as two bf16 matrices [vdim_ld][dim_ld].  A workgroup owns 32 rows x 64
 // value columns of one head's state and walks the run's chunks; the next chunk's keys and values are requested while one is multiplied.
@@ -324,6 +323,7 @@ __global__ __launch_bounds__(256) void linear_states_kernel(pi_linear p, int til
     float * slot = lin_slot(p, run.z), * S = slot + (size_t)h * p.dim * p.vdim;
     const int vcol = v0 + wave * 16 + i;
     const bool sums = MODE == kGated && v0 == 0 && wave == 0;      // this wave keeps the sums of keys of its rows as well (all of its columns alike)
+    const bool keeps = MODE == kGated && v0 == 0 && d0 == 0 && tid == 0;      // this thread reports the running maximum
     pi_f4 acc[2], accn[2];
 #pragma unroll
     for (int m = 0; m < 2; ++m)
@@ -341,7 +341,7 @@ __global__ __launch_bounds__(256) void linear_states_kernel(pi_linear p, int til
     pi_u32x4 rk, rv[2];
     float4 gk[2], ge[2], gr[2];                                  // keyed: sums of the key's channels, of the chunk's last token, and of the rows of acc
     float4 tk, te;                                               // gated: the key's and the last token's numbers
-    float t0v = 0.0f;
+    float top = MODE == kGated ? lin_chunk_tops(p)[(size_t)chunk0 * p.n_head + h] : 0.0f;      // the running maximum ahead of the chunk
     auto fetch = [&](int ck) {
         const int t0 = run.x + ck * kLinC, end = min(t0 + kLinC - 1, last);
         rk = pi_ld16(kp + (size_t)min(t0 + kt, last) * ldk);
@@ -356,7 +356,6 @@ __global__ __launch_bounds__(256) void linear_states_kernel(pi_linear p, int til
         if constexpr (MODE == kGated) {
             tk = lin_gates(p)[(size_t)min(t0 + kt, last) * p.n_head + h];
             te = lin_gates(p)[(size_t)end * p.n_head + h];
-            t0v = lin_chunk_tops(p)[(size_t)(chunk0 + min(ck, n_chunk - 1)) * p.n_head + h];
         }
     };
     fetch(0);
@@ -373,7 +372,12 @@ __global__ __launch_bounds__(256) void linear_states_kernel(pi_linear p, int til
 #pragma unroll
                 for (int m = 0; m < 2; ++m) { dn[m][0] = lin_exp2(gr[m].x); dn[m][1] = lin_exp2(gr[m].y); dn[m][2] = lin_exp2(gr[m].z); dn[m][3] = lin_exp2(gr[m].w); }
             } else {
-                const float one = kt < n ? (MODE == kGated ? expf(te.x + tk.y) : pw[max(n - 1 - kt, 0)]) : 0.0f, all = MODE == kGated ? expf(te.x + t0v) : pw[n];
+                const float most = MODE == kGated ? fmaxf(top, te.z) : 0.0f;
+                const float one = kt < n ? (MODE == kGated ? expf(tk.y - most) : pw[max(n - 1 - kt, 0)]) : 0.0f, all = MODE == kGated ? expf(top - most) : pw[n];
+                if constexpr (MODE == kGated) {
+                    if (keeps && ck) lin_chunk_tops(p)[(size_t)(chunk0 + ck) * p.n_head + h] = top;
+                    top = te.x + most;
+                }
 #pragma unroll
                 for (int j = 0; j < 8; ++j) { w[j] = one; dn[j >> 2][j & 3] = all; }
             }
@@ -424,6 +428,7 @@ __global__ __launch_bounds__(256) void linear_states_kernel(pi_linear p, int til
             if (row < p.dim && vcol < p.vdim) S[(size_t)row * p.vdim + vcol] = acc[m][r];
             if (sums && i == 0 && row < p.dim) lin_keys(p, slot, h)[row] = accn[m][r];
         }
+    if (keeps) for (int k = 0; k < lin_copies(p.vdim); ++k) lin_tops(p, slot, h)[k] = top;
 }
 
 // ---- outputs of one chunk of one head.  Wave w forms the decayed scores of tokens 16 w .. (as columns, keys x tokens) and leaves them in LDS in
@@ -529,7 +534,8 @@ __global__ __launch_bounds__(256) void linear_out_kernel(pi_linear p) {
         top = lin_chunk_tops(p)[(size_t)ck * p.n_head + h];
         if (tid < kLinC) {
             const float4 v = lin_gates(p)[(size_t)(tok0 + min(tid, n - 1)) * p.n_head + h];
-            fa[tid] = v.x; fb[tid] = v.y; ft[tid] = v.z;
+            const float most = fmaxf(top, v.z);
+            fa[tid] = -most; fb[tid] = v.y; ft[tid] = v.x + most;
         }
     } else for (int e = tid; e <= kLinC; e += 256) pw[e] = p.powers[(size_t)h * (kLinC + 1) + e];
     const int qp = p.dim_ld / 8, vp = p.vdim_ld / 8;
@@ -774,7 +780,7 @@ bool linear_ok(const pi_linear * p, const pi_ffn_front & f) {
         return false;
     if (p->decay_kind == kKeyed)
         return p->a2 && p->a2_b && p->rank > 0 && p->rank <= kLinMaxRank && p->rank_ld >= p->rank && p->rank_ld % 8 == 0 && p->rank_ld <= kLinMaxRank && p->off_a >= 0 &&
-               p->off_a + p->rank <= p->ldz && p->tau > 0.0f;
+               p->off_a + p->rank_ld <= p->ldz && p->tau > 0.0f;
     if (p->decay_kind == kGated) return p->i_b && p->f_b && p->den && p->off_i >= 0 && p->off_i + p->n_head <= p->ldz && p->off_f >= 0 && p->off_f + p->n_head <= p->ldz && p->cap > 0.0f;
     return p->decay_kind == kConst;
 }
@@ -815,7 +821,8 @@ template <int VPW> int launch_out(const pi_linear * p, hipStream_t st) {
 }
 int launch_decays(const pi_linear * p, hipStream_t st) {
     if (p->decay_kind == kGated) {
-        hipLaunchKernelGGL(linear_gates_kernel, dim3((p->n_head + 3) / 4, p->n_runs), dim3(256), 0, st, *p);
+        const int h4 = (p->n_head + 3) / 4;
+        hipLaunchKernelGGL(linear_gates_kernel, dim3(p->n_chunks * h4 + p->n_runs), dim3(256), 0, st, *p, h4);
         return pi::check_launch("pi_k_linear_chunks gates");
     }
     if (p->decay_kind != kKeyed) return PI_OK;

@@ -60,21 +60,20 @@ template <typename ST> __device__ void front_block(const pi_ffn_front & f, const
 // ---- grouped-query attention, behind the joint projection: a wave per head (four heads a block) - norm, rotation, division by the root
 // mean square, query row or cell --------------------------------------------------------------------------------------------------------
 constexpr int kGqaMaxDim = 256;
-__host__ __device__ inline int gqa_prep_blocks(const pi_gqa_prep & p) { return (p.n_head + p.n_kv + 3) / 4; }
 template <typename ST> __device__ void gqa_prep_heads(const pi_gqa_prep & p, int t, int b) {
     const int head = b * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63, half = p.rot_dim / 2;
     if (head >= p.n_head + p.n_kv) return;
     const bool key = head >= p.n_head;
     const int g = head - p.n_head;
     const float * z = p.z + (size_t)t * p.ldz, * src = key ? z + p.off_k + g * p.dim : z + head * p.dim;
-    const float * w = key ? p.k_norm : p.q_norm;
+    const float * w = key ? p.k_norm : p.q_norm;             // (pairs i, i + half of the rotation's dimensions)
     const float2 * cs = (const float2 *)p.cs + (size_t)t * half;
     constexpr int J = kGqaMaxDim / 64;
     float x[J], y[J];                                    // the lane's values and what each is paired with
     float ss = 0.0f;
 #pragma unroll
     for (int j = 0; j < J; ++j) {
-        const int e = lane + 64 * j, o = e >= 2 * half ? e : p.rot_pairs ? e ^ 1 : e < half ? e + half : e - half;
+        const int e = lane + 64 * j, o = e >= 2 * half ? e : e < half ? e + half : e - half;
         const float f = w && e < p.dim ? w[e] : 1.0f, fo = w && e < p.dim ? w[o] : 1.0f;
         x[j] = e < p.dim ? src[e] : 0.0f;
         y[j] = e < p.dim ? src[o] * fo : 0.0f;
@@ -88,9 +87,8 @@ template <typename ST> __device__ void gqa_prep_heads(const pi_gqa_prep & p, int
         const int e = lane + 64 * j;
         float v = x[j];
         if (e < 2 * half) {
-            const float2 c = cs[p.rot_pairs ? e >> 1 : e < half ? e : e - half];
-            const bool second = p.rot_pairs ? e & 1 : e >= half;
-            v = second ? v * c.x + y[j] * c.y : v * c.x - y[j] * c.y;
+            const float2 c = cs[e < half ? e : e - half];
+            v = e >= half ? v * c.x + y[j] * c.y : v * c.x - y[j] * c.y;
         }
         x[j] = v;
         ss = fmaf(v, v, ss);
@@ -114,6 +112,93 @@ template <typename ST> __device__ void gqa_prep_heads(const pi_gqa_prep & p, int
 #pragma unroll
         for (int j = 0; j < J; ++j) { const int e = lane + 64 * j; if (e < p.hd) row[p.hd + e] = to_st<ST>(x[j] * sv); }
     }
+}
+// The same for neighbouring pairs, which one lane holds: pairs lane and lane + 64 of N heads of a wave, 4 N heads a block, everything requested
+// together and without guards (past the end of a row: its last values again, not used).  EVEN: no row starts or ends in the middle of a pair.
+template <typename ST, int N, bool EVEN> __device__ void gqa_prep_pairs(const pi_gqa_prep & p, int t, int b) {
+    const int lane = threadIdx.x & 63, half = p.rot_dim / 2, all = p.n_head + p.n_kv, h0 = (b * 4 + (int)(threadIdx.x >> 6)) * N;
+    if (h0 >= all) return;
+    const float * z = p.z + (size_t)t * p.ldz, * qn = p.q_norm ? p.q_norm : z, * kn = p.k_norm ? p.k_norm : z;
+    const float2 * cs = (const float2 *)p.cs + (size_t)t * half;
+    const int cell = p.cell[t];
+    constexpr int J = kGqaMaxDim / 128;
+    const auto load = [](const float * a, int e, int n) {
+        if constexpr (EVEN) return *reinterpret_cast<const float2 *>(a + min(e, n - 2));
+        else return make_float2(a[min(e, n - 1)], a[min(e + 1, n - 1)]);
+    };
+    const auto store = [](ST * o, float a, float b) {
+        struct alignas(2 * sizeof(ST)) Pair { ST v[2]; } q{{to_st<ST>(a), to_st<ST>(b)}};
+        *reinterpret_cast<Pair *>(o) = q;
+    };
+    float2 x[N][J], v[N][J], wq[J], wk[J], c[J];
+#pragma unroll
+    for (int j = 0; j < J; ++j) {
+        const int e = 2 * (lane + 64 * j);
+        wq[j] = load(qn, e, p.dim);
+        wk[j] = load(kn, e, p.dim);
+        c[j] = cs[min(lane + 64 * j, max(half - 1, 0))];
+#pragma unroll
+        for (int n = 0; n < N; ++n) {
+            const int h = min(h0 + n, all - 1), g = h - p.n_head;
+            x[n][j] = load(g >= 0 ? z + p.off_k + g * p.dim : z + h * p.dim, e, p.dim);
+        }
+    }
+    const bool keys = h0 + N > p.n_head;
+    if (keys) {
+#pragma unroll
+        for (int j = 0; j < J; ++j)
+#pragma unroll
+            for (int n = 0; n < N; ++n) v[n][j] = load(z + p.off_v + max(min(h0 + n, all - 1) - p.n_head, 0) * p.vdim, 2 * (lane + 64 * j), p.vdim);
+    }
+#pragma unroll
+    for (int n = 0; n < N; ++n) {
+        const int h = h0 + n, g = h - p.n_head;
+        if (h >= all) break;
+        const bool key = g >= 0;
+        float ss = 0.0f;
+#pragma unroll
+        for (int j = 0; j < J; ++j) {
+            const int e = 2 * (lane + 64 * j);
+            if (e >= p.dim) x[n][j].x = 0.0f;
+            if (e + 1 >= p.dim) x[n][j].y = 0.0f;
+            ss = fmaf(x[n][j].x, x[n][j].x, fmaf(x[n][j].y, x[n][j].y, ss));
+        }
+        float sc = p.q_norm || p.unit ? pi_inv_sqrt(pi_wave_sum(ss) / (float)p.dim + p.eps) : 1.0f;      // (a rotation changes no sum of squares)
+        if (!key && p.temp) sc *= p.temp[h];
+        ST * row = key ? (ST *)p.cache + ((size_t)cell * p.n_kv + g) * 2 * p.hd : (ST *)p.q + ((size_t)t * p.n_head + h) * p.hd;
+#pragma unroll
+        for (int j = 0; j < J; ++j) {
+            const int e = 2 * (lane + 64 * j);
+            const float2 f = !p.q_norm ? make_float2(1.0f, 1.0f) : key ? wk[j] : wq[j], r = e < p.rot_dim ? c[j] : make_float2(1.0f, 0.0f);
+            const float a = x[n][j].x * f.x * sc, o = x[n][j].y * f.y * sc;
+            if (e < p.hd) store(row + e, a * r.x - o * r.y, o * r.x + a * r.y);
+        }
+        if (!key) continue;
+        float sv = 0.0f;
+#pragma unroll
+        for (int j = 0; j < J; ++j) {
+            const int e = 2 * (lane + 64 * j);
+            if (e >= p.vdim) v[n][j].x = 0.0f;
+            if (e + 1 >= p.vdim) v[n][j].y = 0.0f;
+            sv = fmaf(v[n][j].x, v[n][j].x, fmaf(v[n][j].y, v[n][j].y, sv));
+        }
+        const float s2 = p.unit_v ? pi_inv_sqrt(pi_wave_sum(sv) / (float)p.vdim + p.eps) : 1.0f;
+#pragma unroll
+        for (int j = 0; j < J; ++j) { const int e = 2 * (lane + 64 * j); if (e < p.hd) store(row + p.hd + e, v[n][j].x * s2, v[n][j].y * s2); }
+    }
+}
+// heads of a block: neighbouring pairs of long steps several a wave
+constexpr int kGqaPrepHeads = 4;
+__host__ __device__ inline int gqa_prep_blocks(const pi_gqa_prep & p) {
+    const int per = p.rot_pairs && p.T > 16 ? 4 * kGqaPrepHeads : 4;
+    return (p.n_head + p.n_kv + per - 1) / per;
+}
+template <typename ST> __device__ void gqa_prep_block(const pi_gqa_prep & p, int t, int b) {
+    const bool even = ((p.dim | p.vdim | p.ldz | p.off_k | p.off_v) & 1) == 0;
+    if (!p.rot_pairs) gqa_prep_heads<ST>(p, t, b);
+    else if (p.T > 16) { if (even) gqa_prep_pairs<ST, kGqaPrepHeads, true>(p, t, b); else gqa_prep_pairs<ST, kGqaPrepHeads, false>(p, t, b); }
+    else if (even) gqa_prep_pairs<ST, 1, true>(p, t, b);
+    else gqa_prep_pairs<ST, 1, false>(p, t, b);
 }
 inline bool gqa_prep_ok(int type, const pi_gqa_prep & p) {
     return p.z && p.cs && p.q && p.cache && p.cell && p.T > 0 && p.n_head > 0 && p.n_kv > 0 && p.n_head % p.n_kv == 0 && p.rot_dim >= 0 && p.rot_dim % 2 == 0 && p.rot_dim <= p.dim &&
@@ -154,35 +239,44 @@ __device__ void gqa_merge_row(const pi_gqa_attn & p, int item_index, int g, int 
     }
 }
 
-// ---- gated norm by a block of 256 threads: of one token, or (heads) of four of a token's heads, a wave each ------------------------------
-__host__ __device__ inline int gate_norm_blocks(const pi_gate_norm & p) { return p.heads > 0 ? p.T * ((p.heads + 3) / 4) : p.T; }
-template <typename ST> __device__ void gate_norm_heads(const pi_gate_norm & p, int t, int h) {
-    if (h >= p.heads) return;
-    const int vd = p.n / p.heads, lane = threadIdx.x & 63;
+// ---- gated norm by a block of 256 threads: of one token, or (heads) of as many of a token's heads as there are groups of lanes in it,
+// four values a lane ----------------------------------------------------------------------------------------------------------------------
+__host__ __device__ inline int gate_norm_lanes(const pi_gate_norm & p) { const int q = (p.n / p.heads + 3) / 4; return q <= 8 ? 8 : q <= 16 ? 16 : q <= 32 ? 32 : 64; }
+__host__ __device__ inline int gate_norm_per_token(const pi_gate_norm & p) { const int per = 256 / gate_norm_lanes(p); return (p.heads + per - 1) / per; }
+__host__ __device__ inline int gate_norm_blocks(const pi_gate_norm & p) { return p.heads > 0 ? p.T * gate_norm_per_token(p) : p.T; }
+template <typename ST> __device__ void gate_norm_heads(const pi_gate_norm & p, int t, int b) {
+    const int vd = p.n / p.heads, lanes = gate_norm_lanes(p), h = min(b * (256 / lanes) + (int)threadIdx.x / lanes, p.heads - 1), c = (int)(threadIdx.x % lanes) * 4;      // (behind the last head: it again)
     const float * o = p.o + (size_t)t * p.n + h * vd, * g = p.z + (size_t)t * p.ldz + p.off_gate + h * vd, * w = p.w + h * vd;
-    ST * out = (ST *)p.att + (size_t)t * p.ld_att + h * vd;
-    constexpr int J = 4;
+    ST * out = (ST *)p.att + (size_t)t * p.ld_att + h * vd + c;
+    const bool quads = ((vd | p.ldz | p.off_gate) & 3) == 0;
+    float v[4] = {0.0f, 0.0f, 0.0f, 0.0f}, gv[4], wv[4];
     const float den = p.den ? p.den[(size_t)t * p.heads + h] : 1.0f;
-    float v[J], gv[J], wv[J], ss = 0.0f;
+    if (quads) {
+        const int e = min(c, vd - 4);
+        const float4 a = *reinterpret_cast<const float4 *>(o + e), q = *reinterpret_cast<const float4 *>(g + e), f = *reinterpret_cast<const float4 *>(w + e);
+        if (c < vd) { v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w; }
+        gv[0] = q.x; gv[1] = q.y; gv[2] = q.z; gv[3] = q.w;
+        wv[0] = f.x; wv[1] = f.y; wv[2] = f.z; wv[3] = f.w;
+    } else {
 #pragma unroll
-    for (int j = 0; j < J; ++j) {
-        const int e = min(lane + 64 * j, vd - 1);
-        v[j] = o[e]; gv[j] = g[e]; wv[j] = w[e];
+        for (int j = 0; j < 4; ++j) {
+            const int e = min(c + j, vd - 1);
+            if (c + j < vd) v[j] = o[e];
+            gv[j] = g[e]; wv[j] = w[e];
+        }
     }
+    const float per = 1.0f / den;
+    float ss = 0.0f;
 #pragma unroll
-    for (int j = 0; j < J; ++j) {
-        v[j] /= den;
-        if (lane + 64 * j < vd) ss = fmaf(v[j], v[j], ss);
-    }
-    const float sc = pi_inv_sqrt(pi_wave_sum(ss) / (float)vd + p.eps) * p.scale;
+    for (int j = 0; j < 4; ++j) { v[j] *= per; ss = fmaf(v[j], v[j], ss); }
+    for (int k = 1; k < lanes; k <<= 1) ss += __shfl_xor(ss, k, PI_WAVE);
+    const float sc = pi_inv_sqrt(ss / (float)vd + p.eps) * p.scale;
 #pragma unroll
-    for (int j = 0; j < J; ++j) {
-        const int e = lane + 64 * j;
-        if (e < vd) out[e] = to_st<ST>(v[j] * sc * wv[j] * (p.silu ? silu_f32(gv[j]) : sigmoid_f32(gv[j])));
-    }
+    for (int j = 0; j < 4; ++j) v[j] *= sc * wv[j] * (p.silu ? silu_f32(gv[j]) : sigmoid_f32(gv[j]));
+    if (c < vd) store4(out, v, quads && ((uintptr_t)out & (4 * sizeof(ST) - 1)) == 0, vd - c);
 }
 template <typename ST> __device__ void gate_norm_block(const pi_gate_norm & p, int b, double * red) {
-    if (p.heads > 0) { const int per = (p.heads + 3) / 4; gate_norm_heads<ST>(p, b / per, b % per * 4 + (threadIdx.x >> 6)); return; }
+    if (p.heads > 0) { const int per = gate_norm_per_token(p); gate_norm_heads<ST>(p, b / per, b % per); return; }
     const int t = b;
     const float * o = p.o + (size_t)t * p.n, * g = p.z + (size_t)t * p.ldz + p.off_gate;
     ST * out = (ST *)p.att + (size_t)t * p.ld_att;
