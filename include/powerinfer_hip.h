@@ -696,8 +696,8 @@ PI_API int pi_k_gqa_shift(int type, void * cache, int n_cells, int n_kv, int hd,
  *                   keys likewise, o = S^T q and den [T][n_head] = max(|n . q|, exp(-m')) + 1e-6, by which o has still to be divided.
  *                   Behind a slot's S follow n [n_head][dim] and pi_k_linear_copies(vdim) copies of m per head (pi_k_linear_slot_floats).
  * runs [n_runs] = {first token, tokens, slot, 1 if the state starts at zero}: the consecutive tokens of one sequence.  o [T][n_head * vdim] fp32.
- * pi_k_linear_step walks every run token by token; front (optional) and prep (optional, the queries and cells of a grouped-query attention
- * beside it) run in the same launch.
+ * pi_k_linear_step walks every run token by token; front (optional) runs in the same launch, in pi_k_linear_step_beside (keyed and gated)
+ * the queries and cells of a grouped-query attention.
  * pi_k_linear_prep + pi_k_linear_chunks (bf16) do the same for long runs in chunks of pi_k_linear_chunk() tokens: q, k [T][n_head][dim_ld] and
  * v [T][n_head][vdim_ld] in bf16 (dim_ld a multiple of 32, vdim_ld of 64), then the states before every chunk (as sums of two bf16) into
  * states (pi_k_linear_states_bytes) and the outputs.  chunks [n_chunks] = {first token, tokens, 1 if nothing lies before it}, a run's chunks

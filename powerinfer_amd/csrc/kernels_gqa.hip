@@ -4,12 +4,16 @@
 
 namespace {
 
-template <typename ST>
+template <typename ST, bool PAIRS>
 __global__ __launch_bounds__(256) void gqa_prep_kernel(pi_gqa_prep p, pi_ffn_front f, int n_heads4, int per) {
     extern __shared__ __align__(16) float sm[];
     const int t = blockIdx.x / per, b = blockIdx.x % per;
     if (b >= n_heads4) front_block<ST>(f, p.z, p.ldz, t, b - n_heads4, sm);
-    else gqa_prep_block<ST>(p, t, b);
+    else gqa_prep_block<ST, PAIRS>(p, t, b);
+}
+template <typename ST> void launch_prep(const pi_gqa_prep & p, const pi_ffn_front & f, int n4, int per, hipStream_t st) {
+    if (p.rot_pairs) hipLaunchKernelGGL((gqa_prep_kernel<ST, true>), dim3(per * p.T), dim3(256), front_lds_bytes(f), st, p, f, n4, per);
+    else hipLaunchKernelGGL((gqa_prep_kernel<ST, false>), dim3(per * p.T), dim3(256), front_lds_bytes(f), st, p, f, n4, per);
 }
 
 // the first cell a token sees
@@ -61,7 +65,8 @@ __global__ __launch_bounds__(256, WIDE && KS <= 4 ? 2 : 1) void gqa_attn_kernel(
             for (int j = 0; j < KS; ++j) pre[k][j] = pi_ld16(cache + (size_t)idx[k] * p.n_kv * 2 * HD + j * 64);
     };
     if (c0 < c1) look_up(c0);
-    int row[U], tok[U], head[U], nv[U], lo[U];
+    int row[U], tok[U], head[U], lo[U];
+    unsigned nv[U];                                              // cells the row sees, from lo on
     pi_u32x4 qf[U][KS];
 #pragma unroll
     for (int u = 0; u < U; ++u) {
@@ -69,8 +74,8 @@ __global__ __launch_bounds__(256, WIDE && KS <= 4 ? 2 : 1) void gqa_attn_kernel(
         const int rr = first + min(row[u], rows - 1);
         tok[u] = tok0 + rr / per;
         head[u] = g * per + rr % per;
-        nv[u] = row[u] < rows ? p.n_vis[tok[u]] : 0;
         lo[u] = first_cell(p, tok[u]);
+        nv[u] = row[u] < rows ? p.n_vis[tok[u]] - lo[u] : 0;
 #pragma unroll
         for (int s = 0; s < KS; ++s) qf[u][s] = pi_ld16((const uint16_t *)p.q + ((size_t)tok[u] * p.n_head + head[u]) * HD + s * 32 + gq * 8);
     }
@@ -118,8 +123,7 @@ __global__ __launch_bounds__(256, WIDE && KS <= 4 ? 2 : 1) void gqa_attn_kernel(
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
                     float v = s[u][kt][r] * p.scale;
-                    const int c = cb + kb + kt * 16 + 4 * gq + r;
-                    if (edge && (c >= nv[u] || c < lo[u])) v = -INFINITY;
+                    if (edge && (unsigned)(cb + kb + kt * 16 + 4 * gq + r - lo[u]) >= nv[u]) v = -INFINITY;
                     s[u][kt][r] = v;
                     mx = fmaxf(mx, v);
                 }
@@ -335,8 +339,8 @@ int pi_k_gqa_prep(int type, const pi_gqa_prep * p, const pi_ffn_front * front, p
         return pi::fail(PI_E_ARG, "pi_k_gqa_prep: bad arguments");
     const int n4 = gqa_prep_blocks(*p), per = n4 + front_blocks(f);
     if ((long long)per * p->T > (1 << 30)) return pi::fail(PI_E_ARG, "pi_k_gqa_prep: too many tokens");
-    if (type == PI_TYPE_BF16) hipLaunchKernelGGL(gqa_prep_kernel<bf16>, dim3(per * p->T), dim3(256), front_lds_bytes(f), (hipStream_t)stream, *p, f, n4, per);
-    else if (type == PI_TYPE_F32) hipLaunchKernelGGL(gqa_prep_kernel<float>, dim3(per * p->T), dim3(256), front_lds_bytes(f), (hipStream_t)stream, *p, f, n4, per);
+    if (type == PI_TYPE_BF16) launch_prep<bf16>(*p, f, n4, per, (hipStream_t)stream);
+    else if (type == PI_TYPE_F32) launch_prep<float>(*p, f, n4, per, (hipStream_t)stream);
     else return pi::fail(PI_E_UNSUPPORTED, "pi_k_gqa_prep: type");
     return pi::check_launch("pi_k_gqa_prep");
 }

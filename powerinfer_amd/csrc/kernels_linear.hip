@@ -56,7 +56,9 @@ __global__ __launch_bounds__(256) void linear_step_kernel(pi_linear p, pi_ffn_fr
     if ((int)blockIdx.x >= n_state) {
         const int b = blockIdx.x - n_state;
         if (b < n_front) front_block<ST>(f, p.z, p.ldz, b / per, b % per, sm);
-        else gqa_prep_block<ST>(beside, (b - n_front) / per_beside, (b - n_front) % per_beside);
+        else if (MODE == kConst) return;                         // (asks for nothing beside it: checked by the launcher)
+        else if (beside.rot_pairs) gqa_prep_block<ST, true>(beside, (b - n_front) / per_beside, (b - n_front) % per_beside);
+        else gqa_prep_block<ST, false>(beside, (b - n_front) / per_beside, (b - n_front) % per_beside);
         return;
     }
     float * qs = sm, * ks = qs + kLinBlock * D, * vs = ks + kLinBlock * D, * part = vs + kLinBlock * kLinCols;      // [16][D], [16][D], [16][32], [4][16][32]
@@ -850,7 +852,7 @@ int pi_k_linear_step(int type, const pi_linear * p, const pi_ffn_front * front, 
     return linear_step(type, p, front ? *front : pi_ffn_front{}, nullptr, (hipStream_t)stream);
 }
 int pi_k_linear_step_beside(int type, const pi_linear * p, const pi_gqa_prep * prep, pi_stream_t stream) {
-    if (!prep) return pi::fail(PI_E_ARG, "pi_k_linear_step_beside: bad arguments");
+    if (!p || !prep || p->decay_kind == kConst) return pi::fail(PI_E_ARG, "pi_k_linear_step_beside: bad arguments (a recurrence with gates)");
     return linear_step(type, p, pi_ffn_front{}, prep, (hipStream_t)stream);
 }
 

@@ -60,7 +60,7 @@ template <typename ST> __device__ void front_block(const pi_ffn_front & f, const
 // ---- grouped-query attention, behind the joint projection: a wave per head (four heads a block) - norm, rotation, division by the root
 // mean square, query row or cell --------------------------------------------------------------------------------------------------------
 constexpr int kGqaMaxDim = 256;
-template <typename ST> __device__ void gqa_prep_heads(const pi_gqa_prep & p, int t, int b) {
+template <typename ST, bool NORM> __device__ void gqa_prep_heads(const pi_gqa_prep & p, int t, int b) {      // NORM: q_norm and k_norm are given
     const int head = b * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63, half = p.rot_dim / 2;
     if (head >= p.n_head + p.n_kv) return;
     const bool key = head >= p.n_head;
@@ -68,47 +68,51 @@ template <typename ST> __device__ void gqa_prep_heads(const pi_gqa_prep & p, int
     const float * z = p.z + (size_t)t * p.ldz, * src = key ? z + p.off_k + g * p.dim : z + head * p.dim;
     const float * w = key ? p.k_norm : p.q_norm;             // (pairs i, i + half of the rotation's dimensions)
     const float2 * cs = (const float2 *)p.cs + (size_t)t * half;
+    ST * row = key ? (ST *)p.cache + ((size_t)p.cell[t] * p.n_kv + g) * 2 * p.hd : (ST *)p.q + ((size_t)t * p.n_head + head) * p.hd;
     constexpr int J = kGqaMaxDim / 64;
-    float x[J], y[J];                                    // the lane's values and what each is paired with
+    float x[J], y[J];                                    // the lane's values and what each is paired with (no guard around a load)
+    float2 c[J];
     float ss = 0.0f;
 #pragma unroll
     for (int j = 0; j < J; ++j) {
-        const int e = lane + 64 * j, o = e >= 2 * half ? e : e < half ? e + half : e - half;
-        const float f = w && e < p.dim ? w[e] : 1.0f, fo = w && e < p.dim ? w[o] : 1.0f;
-        x[j] = e < p.dim ? src[e] : 0.0f;
-        y[j] = e < p.dim ? src[o] * fo : 0.0f;
-        ss = fmaf(x[j], x[j], ss);
-        x[j] *= f;
+        const int e = min(lane + 64 * j, p.dim - 1), o = e >= 2 * half ? e : e < half ? e + half : e - half;
+        x[j] = src[e]; y[j] = src[o];
+        c[j] = cs[min(e < half ? e : e - half, max(half - 1, 0))];
     }
-    float sc = w ? pi_inv_sqrt(pi_wave_sum(ss) / (float)p.dim + p.eps) : 1.0f;
+#pragma unroll
+    for (int j = 0; j < J; ++j) {
+        if (lane + 64 * j >= p.dim) x[j] = 0.0f;
+        ss = fmaf(x[j], x[j], ss);
+    }
+    float sc = 1.0f;
+    if constexpr (NORM) {
+        sc = pi_inv_sqrt(pi_wave_sum(ss) / (float)p.dim + p.eps);
+#pragma unroll
+        for (int j = 0; j < J; ++j) {
+            const int e = min(lane + 64 * j, p.dim - 1), o = e >= 2 * half ? e : e < half ? e + half : e - half;
+            x[j] *= w[e]; y[j] *= w[o];
+        }
+    }
     ss = 0.0f;
 #pragma unroll
     for (int j = 0; j < J; ++j) {
         const int e = lane + 64 * j;
-        float v = x[j];
-        if (e < 2 * half) {
-            const float2 c = cs[e < half ? e : e - half];
-            v = e >= half ? v * c.x + y[j] * c.y : v * c.x - y[j] * c.y;
-        }
-        x[j] = v;
-        ss = fmaf(v, v, ss);
+        if (e < 2 * half) x[j] = e >= half ? x[j] * c[j].x + y[j] * c[j].y : x[j] * c[j].x - y[j] * c[j].y;
+        ss = fmaf(x[j], x[j], ss);
     }
     if (p.unit) sc = pi_inv_sqrt(pi_wave_sum(ss) / (float)p.dim + p.eps);
     if (!key && p.temp) sc *= p.temp[head];
-    ST * row = key ? (ST *)p.cache + ((size_t)p.cell[t] * p.n_kv + g) * 2 * p.hd : (ST *)p.q + ((size_t)t * p.n_head + head) * p.hd;
 #pragma unroll
     for (int j = 0; j < J; ++j) { const int e = lane + 64 * j; if (e < p.hd) row[e] = to_st<ST>(x[j] * sc); }      // (zeros behind dim)
     if (key) {
         const float * v = z + p.off_v + g * p.vdim;
         float sv = 1.0f;
 #pragma unroll
-        for (int j = 0; j < J; ++j) { const int e = lane + 64 * j; x[j] = e < p.vdim ? v[e] : 0.0f; }
-        if (p.unit_v) {
-            ss = 0.0f;
+        for (int j = 0; j < J; ++j) x[j] = v[min(lane + 64 * j, p.vdim - 1)];
+        ss = 0.0f;
 #pragma unroll
-            for (int j = 0; j < J; ++j) ss = fmaf(x[j], x[j], ss);
-            sv = pi_inv_sqrt(pi_wave_sum(ss) / (float)p.vdim + p.eps);
-        }
+        for (int j = 0; j < J; ++j) { if (lane + 64 * j >= p.vdim) x[j] = 0.0f; ss = fmaf(x[j], x[j], ss); }
+        if (p.unit_v) sv = pi_inv_sqrt(pi_wave_sum(ss) / (float)p.vdim + p.eps);
 #pragma unroll
         for (int j = 0; j < J; ++j) { const int e = lane + 64 * j; if (e < p.hd) row[p.hd + e] = to_st<ST>(x[j] * sv); }
     }
@@ -193,9 +197,10 @@ __host__ __device__ inline int gqa_prep_blocks(const pi_gqa_prep & p) {
     const int per = p.rot_pairs && p.T > 16 ? 4 * kGqaPrepHeads : 4;
     return (p.n_head + p.n_kv + per - 1) / per;
 }
-template <typename ST> __device__ void gqa_prep_block(const pi_gqa_prep & p, int t, int b) {
+template <typename ST, bool PAIRS> __device__ void gqa_prep_block(const pi_gqa_prep & p, int t, int b) {
     const bool even = ((p.dim | p.vdim | p.ldz | p.off_k | p.off_v) & 1) == 0;
-    if (!p.rot_pairs) gqa_prep_heads<ST>(p, t, b);
+    if (!PAIRS && !p.q_norm) gqa_prep_heads<ST, false>(p, t, b);
+    else if (!PAIRS) gqa_prep_heads<ST, true>(p, t, b);
     else if (p.T > 16) { if (even) gqa_prep_pairs<ST, kGqaPrepHeads, true>(p, t, b); else gqa_prep_pairs<ST, kGqaPrepHeads, false>(p, t, b); }
     else if (even) gqa_prep_pairs<ST, 1, true>(p, t, b);
     else gqa_prep_pairs<ST, 1, false>(p, t, b);

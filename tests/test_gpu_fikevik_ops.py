@@ -6,6 +6,7 @@ import numpy as np
 import pytest
 
 import plain_fikevik as o
+from plain_pibalorn import rotate_halves
 from powerinfer_amd import lib as pl
 from test_gpu_gqa_ops import attend, filled
 from test_gpu_latent_ops import TYPES, as_stored, dev, fetch, i32, padded, rounded, store, tol
@@ -179,8 +180,8 @@ def test_state_far_back_decides(kind, chunked):
 PREPS = [(6, 2, 96, 130, 96), (5, 1, 17, 9, 6), (4, 2, 128, 64, 32), (3, 3, 256, 256, 0), (8, 2, 40, 72, 40)]
 
 
-def prepared(L, t, z, ldz, T, at, H, G, dim, vdim, rot, rng, n_cells=40):
-    """(pi_gqa_prep with every option, its buffers, what it should leave as a function of z)."""
+def prepared(L, t, z, ldz, T, at, H, G, dim, vdim, rot, rng, n_cells=40, pairs=1):
+    """(pi_gqa_prep with every option, a check of what it should leave given z)."""
     off_k, off_v, hd = at + H * dim + 1, at + H * dim + 1 + G * dim + 2, L.pi_k_gqa_head_ld(t, dim, vdim)
     pos, cells = rng.integers(0, 5000, T).astype(np.int32), rng.permutation(n_cells)[:T]
     qn, kn = (1 + 0.3 * rng.standard_normal((2, dim))).astype(np.float32)
@@ -191,7 +192,7 @@ def prepared(L, t, z, ldz, T, at, H, G, dim, vdim, rot, rng, n_cells=40):
     if rot:
         pl.check(L.pi_k_rope_angles(pb.ptr, T, rot, 700.0, b["cs"].ptr, None))
         pl.sync()
-    p = filled(pl.GqaPrep, z=z, ldz=ldz, T=T, n_head=H, n_kv=G, dim=dim, vdim=vdim, rot_dim=rot, off_k=off_k, off_v=off_v, hd=hd, eps=1e-5, rot_pairs=1, unit_v=1, **b)
+    p = filled(pl.GqaPrep, z=z, ldz=ldz, T=T, n_head=H, n_kv=G, dim=dim, vdim=vdim, rot_dim=rot, off_k=off_k, off_v=off_v, hd=hd, eps=1e-5, rot_pairs=pairs, unit_v=1, **b)
 
     def check(z64):
         tail = {"q": np.eye(H * dim), "k": np.eye(G * dim), "v": np.eye(G * vdim)}
@@ -213,13 +214,17 @@ def prepared(L, t, z, ldz, T, at, H, G, dim, vdim, rot, rng, n_cells=40):
 
 
 @pytest.mark.parametrize("t", TYPES)
+@pytest.mark.parametrize("T,pairs", [(6, 1), (33, 1), (6, 0)])
 @pytest.mark.parametrize("H,G,dim,vdim,rot", PREPS)
-def test_queries_and_cells(t, H, G, dim, vdim, rot):
+def test_queries_and_cells(monkeypatch, t, T, pairs, H, G, dim, vdim, rot):
+    """In steps and in prompts (several heads a wave), and for the rotation of the other designs."""
+    if not pairs:
+        monkeypatch.setattr(o, "rotate_neighbours", rotate_halves)
     L, rng = pl.init(), np.random.default_rng(dim)
-    T, ldz = 6, (H * dim + G * (dim + vdim) + 20) // 16 * 16
+    ldz = (H * dim + G * (dim + vdim) + 20) // 16 * 16
     z = (2 * rng.standard_normal((T, ldz))).astype(np.float32)
     zb = dev(z)
-    p, check = prepared(L, t, zb, ldz, T, 0, H, G, dim, vdim, rot, rng)
+    p, check = prepared(L, t, zb, ldz, T, 0, H, G, dim, vdim, rot, rng, pairs=pairs)
     pl.check(L.pi_k_gqa_prep(t, C.byref(p), None, None))
     pl.sync()
     check(z.astype(np.float64))
