@@ -594,7 +594,8 @@ PI_API int pi_k_layer_norm(int type, float * x, const int32_t * rows, int T, int
  * the T rows x + g * x_gs + t * ldx into y + g * y_gs + t * ldy.  off != NULL (n_group + 1 offsets on the device): group g takes the
  * places s in [off[g], off[g + 1]) of a list; input row = gather ? gather[s] / gather_div : s, output row = s; T bounds the places of one group.
  * relu2: y = relu(.)^2.  glu: rows 2 j and 2 j + 1 of W are gate and up row j, y has rows / 2 columns: the clamped GLU
- * (pi_ffn_front).  y_f32: y is fp32 whatever `type` is.  Strides count elements. */
+ * (pi_ffn_front; glu_plain_up: plain_up).  pair_w (optional, with gather): the products of place s are multiplied by pair_w[gather[s]] ahead of the
+ * activation, as if the input were.  y_f32: y is fp32 whatever `type` is.  Strides count elements. */
 typedef struct pi_group_gemm {
     const void * W; size_t w_gs; int32_t rows, cols, ldw, n_group;
     const void * x; size_t x_gs; int32_t ldx, T;
@@ -603,12 +604,15 @@ typedef struct pi_group_gemm {
     const int32_t * off, * gather; int32_t gather_div;
     const int32_t * tiles, * n_tiles; int32_t max_tiles;      /* pi_k_group_gemm_tile with off: pi_k_moe_sort's list and an upper bound of its length */
     int32_t glu; float glu_limit, glu_gain;
+    const float * pair_w; int32_t glu_plain_up;
 } pi_group_gemm;
 PI_API int pi_k_group_gemm(int type, const pi_group_gemm * g, pi_stream_t stream);
 /* the same for many tokens, bf16, both operands tiled through LDS (cols % 64 == 0); tile_n 64 or 128 tokens per tile, as given to pi_k_moe_sort */
 PI_API int pi_k_group_gemm_tile(const pi_group_gemm * g, int tile_n, pi_stream_t stream);
 /* (cos, sin)[t][i] of the angles pos[t] * base^(-2i / dims), i < dims / 2 */
 PI_API int pi_k_rope_angles(const int32_t * pos, int T, int dims, double base, void * cs_float2, pi_stream_t stream);
+/* the same with given frequencies (dims / 2 of them), cosine and sine times length */
+PI_API int pi_k_rope_angles_table(const int32_t * pos, int T, int dims, const double * freq, double length, void * cs_float2, pi_stream_t stream);
 /* Behind the joint projection of a latent-attention layer, z [T][ldz] = per head [dim | rot_dim], then (own cells) [kv_rank | rot_dim]:
  * the unrotated query parts to q_un [T][n_head][dim_ld], the rotated ones to q_lat [T][n_head][kd] behind rank_ld values, and
  * (cache != NULL) the token's cell: normed latent, rotated key part behind rank_ld values, rows of kd values. */
@@ -659,12 +663,14 @@ PI_API int pi_k_ffn_front(int type, const float * z, int ldz, int T, const pi_ff
  * first rot_dim values, with rot_pairs != 0 pairs 2 i, 2 i + 1; cs as pi_k_rope_angles makes it) and, with unit != 0, divided by their root
  * mean square; queries go to q [T][n_head][hd], the token's cell is n_kv rows [key | value] of hd values each, padded with zeros
  * (pi_k_gqa_head_ld).  q_norm, k_norm (optional, [dim], both or none; unit 0): RMS norm of every head with these weights ahead of the
- * rotation; unit_v: values are divided by their root mean square; temp (optional, [n_head]): factor of a head's queries.  front (optional) runs in the
- * same launch. */
+ * rotation; unit_v: values are divided by their root mean square; temp (optional, [n_head]): factor of a head's queries.  v_keep (optional): the
+ * projected values [T][ld_first] for layers behind this one, which give them back as v_first and mix (1 - v_mix[0]) v + v_mix[0] v_first ahead of
+ * anything else.  front (optional) runs in the same launch. */
 typedef struct pi_gqa_prep {
     const float * z; int32_t ldz, T, n_head, n_kv, dim, vdim, rot_dim, off_k, off_v, hd, unit;
     const void * cs; float eps; void * q, * cache; const int32_t * cell;
     int32_t rot_pairs, unit_v; const float * q_norm, * k_norm, * temp;
+    const float * v_first, * v_mix; float * v_keep; int32_t ld_first;
 } pi_gqa_prep;
 PI_API int pi_k_gqa_head_ld(int type, int dim, int vdim);                    /* hd for a head size, 0: not supported */
 PI_API int pi_k_gqa_prep(int type, const pi_gqa_prep * p, const pi_ffn_front * front, pi_stream_t stream);
@@ -673,18 +679,28 @@ PI_API int pi_k_gqa_prep(int type, const pi_gqa_prep * p, const pi_ffn_front * f
  * workgroups, partial sums in scratch (pi_k_gqa_scratch_floats).  fp32: work [T] = each token's sequence.  sink: score of an entry of the
  * soft-max without a value (-INFINITY: none).  window > 0: a token sees the last `window` of those cells only; first (optional, [T]): it sees
  * the cells from first[token] on instead (ascending along a run).  att [T][ld_att] gets n_head x vdim values per token, times out_scale.
- * pi_k_gqa_attn merges the parts, pi_k_gqa_attn_parts leaves them to pi_k_mix_up_step. */
+ * softcap > 0: scores become softcap * tanh(score / softcap).  sinks (optional, [n_head]): a sink per head instead of `sink`.  all_values != 0: every
+ * head's weights meet the values of every key / value head, att is fp32 [T][n_head][n_kv][vdim] (for pi_k_gqa_mix) and there are n_kv * n_kv groups
+ * where n_kv counts them.  pi_k_gqa_attn merges the parts, pi_k_gqa_attn_parts leaves them to pi_k_mix_up_step. */
 typedef struct pi_gqa_attn {
     const void * q, * cache; const int32_t * lists; size_t list_ld; const int32_t * work, * n_vis;
     int32_t n_work, T, n_head, n_kv, dim, vdim, hd, n_parts, wide; float scale, sink; float * scratch; void * att; int32_t ld_att;
     float out_scale; int32_t window; const int32_t * first;
+    float softcap; const float * sinks; int32_t all_values;
 } pi_gqa_attn;
 PI_API int    pi_k_gqa_rows(int wide);
 PI_API size_t pi_k_gqa_scratch_floats(int n_work, int wide, int n_kv, int hd, int n_parts);
 PI_API int    pi_k_gqa_attn(int type, const pi_gqa_attn * p, pi_stream_t stream);
 PI_API int    pi_k_gqa_attn_parts(const pi_gqa_attn * p, pi_stream_t stream);
+/* Heads mixed behind an attention with all_values: att[t][h] = sigmoid(z[t][off_gate + h]) * sum over g of talk[h][g] * a[t][g][h's key / value head]
+ * (talk NULL: a[t][h][..]; off_gate < 0: no gate). */
+typedef struct pi_gqa_mix {
+    const float * a, * talk, * z; int32_t ldz, off_gate, T, n_head, n_kv, vdim; void * att; int32_t ld_att;
+} pi_gqa_mix;
+PI_API int    pi_k_gqa_mix(int type, const pi_gqa_mix * p, pi_stream_t stream);
 /* rotates the key parts of cells by delta[cell] positions (pairs != 0: neighbouring values are a pair) */
 PI_API int pi_k_gqa_shift(int type, void * cache, int n_cells, int n_kv, int hd, int rot_dim, double base, int pairs, const int32_t * delta, pi_stream_t stream);
+PI_API int pi_k_gqa_shift_table(int type, void * cache, int n_cells, int n_kv, int hd, int rot_dim, const double * freq, int pairs, const int32_t * delta, pi_stream_t stream);
 /* Linear attention over a fp32 state [slot][n_head][dim][vdim] (slot_ld floats per slot, 0: exactly these), behind the joint projection
  * z [T][ldz]: q at off_q (n_head x dim), k at off_k, v at off_v (n_head x vdim); silu of each, or with plain != 0 the projections themselves
  * (pi_k_linear_step: unrounded) and q times q_scale.  decay_kind says what becomes of the state:
@@ -734,6 +750,8 @@ PI_API int pi_k_gate_norm(int type, const pi_gate_norm * p, pi_stream_t stream);
 /* expert choice of T tokens from router logits z [T][n_expert] (see PI_FFN_MOE): ids, weights [T][n_top] by falling choice score */
 PI_API int pi_k_route(const float * z, int T, int n_expert, int n_top, int n_group, int n_keep, const float * bias, int32_t * ids, float * weights,
                       pi_stream_t stream);
+/* the experts with the largest sigmoid scores, their weights the scores themselves */
+PI_API int pi_k_route_scores(const float * z, int T, int n_expert, int n_top, int32_t * ids, float * weights, pi_stream_t stream);
 /* pairs (token, choice) in expert order: off [n_expert + 1], perm[place] = pair, inv[pair] = place.  tiles (optional): {expert, first
  * place} of every group of up to tile_n pairs of one expert; *n_tiles of them, at most n_pairs / tile_n + n_expert */
 PI_API int pi_k_moe_sort(const int32_t * ids, int n_pairs, int n_expert, int32_t * off, int32_t * perm, int32_t * inv, int tile_n, int32_t * tiles,
@@ -746,7 +764,7 @@ PI_API int pi_k_moe_combine(int type, const float * x, const float * mix, const 
  * [n_head][kv_rank][dim_ld]; p->q_un is not used) and, with ids != NULL, pi_k_route in one launch.  pi_k_value_up_step: the merge of
  * a split attention (or its whole result) and the value expansion, att [T][ld_att] - pi_k_latent_attn_parts leaves the parts unmerged -
  * and, with ids != NULL, act [T * top][ld_act] = weight * relu(up[e] x)^2 for every (token, choice).  pi_k_layer_out_step: what closes the
- * layer, out = x + (wo att + sum over the pairs of a token of down[e] act[pair]); ids == NULL: no experts. */
+ * layer, out = x + (wo att + sum over the pairs of a token of down[e] act[pair]); ids == NULL: no experts; x == NULL: zeros; wo == NULL: experts only. */
 typedef struct pi_layer_out {
     const float * x; const void * wo, * att; int32_t rows, ld_att, T;
     const void * down, * act; const int32_t * ids; int32_t ld_act, top, n_expert;
@@ -766,6 +784,29 @@ PI_API int pi_k_layer_out_step(const pi_layer_out * a, pi_stream_t stream);
  * turn) for every (token, choice), in one launch. */
 PI_API int pi_k_mix_up_step(const pi_gqa_attn * attn, const pi_gate_norm * gate, const void * up, int n_expert, int ff, int cols, float limit, float gain,
                             const void * x_ol, int T, const int32_t * ids, const float * weights, int top, void * act, int ld_act, pi_stream_t stream);
+/* The experts' first matrices alone; weigh_input: act = clamped GLU of (weight * up[e] x) instead of weight * clamped GLU; plain_up as in pi_ffn_front. */
+PI_API int pi_k_expert_up_step(const void * up, int n_expert, int ff, int cols, float limit, float gain, int plain_up, int weigh_input, const void * x_ol, int T, const int32_t * ids,
+                               const float * weights, int top, void * act, int ld_act, pi_stream_t stream);
+/* Norms in groups: a row falls into `groups` equal consecutive parts, each divided by its own root mean square, the whole times w.
+ * pi_k_sum_norm closes a sublayer with a norm on its result: x[t] += mult * norm(s) * w with s = mix[t], or (y != NULL) the sum over k < top of
+ * y[inv[t * top + k]] (y of the given type, rows of cols values; y_w (optional): each times y_w[t * top + k]); w NULL: x stays.  keep (optional) receives a copy of the new x; h (optional): norm(x) *
+ * w_next as the next product's operand, rows of ld values or (ol, BF16, T <= 16) in the operand layout of pi_k_gemm_bf16_ol; rows (optional, w NULL): row t of
+ * h is made of x[rows[t]]. */
+typedef struct pi_sum_norm {
+    float * x; const float * mix; const void * y; const int32_t * inv; int32_t top; const float * y_w, * w; float mult;
+    const float * w_next; const int32_t * rows; int32_t T, cols, groups; float eps; float * keep; void * h; int32_t ld, ol;
+} pi_sum_norm;
+PI_API int pi_k_sum_norm(int type, const pi_sum_norm * p, pi_stream_t stream);
+/* A norm in groups and behind it a causal convolution over time on every channel: u = norm(x[t]) * w, h[t] = u_t + sum over j of taps_w[c][j] *
+ * u_(t - taps + 1 + j) along the token's sequence, zeros ahead of it.  items [n_items] of eight integers: {first token, tokens, tokens of the run ahead of
+ * them, tokens of the run, slot, 1 if nothing lies before the run, 0, 0}; a run's first item holds at least min(taps - 1, all) of its tokens, reads the last
+ * taps - 1 inputs before the run from state + slot * slot_ld ([taps - 1][cols] fp32) and leaves those before the run's end there. */
+typedef struct pi_conv_norm {
+    const float * x, * w, * taps_w; int32_t T, cols, groups, taps; float eps; float * state; size_t slot_ld; const int32_t * items; int32_t n_items;
+    void * h; int32_t ld, ol;
+} pi_conv_norm;
+PI_API int pi_k_conv_norm(int type, const pi_conv_norm * p, pi_stream_t stream);
+PI_API int pi_k_conv_tokens(int T, int taps);                                 /* tokens of an item of a step of T tokens */
 /* What closes a sublayer whose norm comes after the sum: s = alpha x[t] + g * mix[t] with g = sigmoid(gate_z[t][off_gate ..] + gate_b) (gate_z NULL: 1),
  * or s = x[t] (mix NULL); out[t] = rms_norm(s) * w (w NULL: s); h (optional): the same as the next product's operand, rows of ld values or
  * (ol, BF16, T <= 16) in the operand layout of pi_k_gemm_bf16_ol; keep (optional) receives a copy.  out may be x. */
@@ -788,7 +829,7 @@ PI_API int pi_k_cells_advance(int T, const int32_t * seq, const int32_t * lists,
 
 /* ---- decode loop with resident weights ------------------------------------------------------------- */
 
-enum { PI_ARCH_LLAMA = 0, PI_ARCH_FALCON = 1, PI_ARCH_LERASUN = 2, PI_ARCH_PIBALORN = 3, PI_ARCH_FIKEVIK = 4 };
+enum { PI_ARCH_LLAMA = 0, PI_ARCH_FALCON = 1, PI_ARCH_LERASUN = 2, PI_ARCH_PIBALORN = 3, PI_ARCH_FIKEVIK = 4, PI_ARCH_PUFIVIK = 5 };
 
 /* the llama_hparams fields this path reads (llama.cpp:1207-1270) */
 typedef struct pi_hparams {
@@ -822,6 +863,8 @@ enum {
     PI_T_MIX_Q_NORM, PI_T_MIX_K_NORM, PI_T_MIX_TEMP,
     PI_T_MIX_A1, PI_T_MIX_A2, PI_T_MIX_A2_B,
     PI_T_MEM_Q, PI_T_MEM_K, PI_T_MEM_V, PI_T_MEM_G, PI_T_MEM_O, PI_T_MEM_NORM, PI_T_MEM_I, PI_T_MEM_I_B, PI_T_MEM_F, PI_T_MEM_F_B,
+    /* norms before and after every sublayer, convolution of a mixer's input, mixed values, heads and gates of grouped-query attention */
+    PI_T_ATTN_NORM_AFTER, PI_T_FFN_NORM_AFTER, PI_T_MIX_CONV, PI_T_MIX_VALUE, PI_T_MIX_TALK, PI_T_MIX_HEAD_GATE,
     PI_T_COUNT
 };
 
@@ -868,9 +911,21 @@ enum {
  * PI_FFN_GLU: PI_T_GLU_GATE, _UP [glu_ff][n_embd], _DOWN [n_embd][glu_ff], the clamped GLU with glu_limit and glu_gain (pi_ffn_front; glu_plain_up: plain_up).
  * PI_FFN_GLU_MOE: PI_T_ROUTER; the n_top largest logits, weights their soft-max; PI_T_EXPERT_GATE, _UP, _DOWN as above with expert_limit;
  *   glu_ff > 0: beside them a shared one (PI_T_GLU_*, glu_limit) that every token uses times sigmoid(PI_T_SHARED_SCORE [1][n_embd] h).
+ *
+ * both_norms: a layer is x = x + residual_mult * norm(mixer(conv(norm(x)))), then the same with the feed-forward and without the convolution; norms in
+ * norm_groups groups (PI_T_ATTN_NORM, _ATTN_NORM_AFTER, PI_T_FFN_NORM, _FFN_NORM_AFTER), conv_taps > 0: PI_T_MIX_CONV [n_embd][conv_taps] (pi_conv_norm; the
+ * last conv_taps - 1 inputs are a state of the sequence); mixer PI_MIXER_GROUPED, feed-forwards PI_FFN_NONE and PI_FFN_GLU_MOE without a shared one.
+ * With it grouped-query attention may have: softcap (pi_gqa_attn); head_sinks: PI_T_MIX_SINK [n_head]; head_mix: PI_T_MIX_TALK [n_head][n_head], soft-max
+ *   weights mixed over the heads (pi_gqa_mix); head_gate: heads times sigmoid(PI_T_MIX_HEAD_GATE [n_head][n_embd] h); value_mix: all layers that have it but the
+ *   first mix that one's values of the same token into their own by PI_T_MIX_VALUE [1] (n_kv_head * vdim alike in all of them).
+ *   rot_scaling of frequencies: PI_ROT_WAVES divides those with fewer than rot_low turns in rot_original positions by rot_factor, keeps those with
+ *   more than rot_high and blends between; PI_ROT_RAMP divides and keeps along a ramp over the pairs, between the pairs that make rot_low and rot_high
+ *   turns, and lengthens the rotated part by 0.1 ln(rot_factor) + 1.
+ * PI_FFN_GLU_MOE with route_scores: weights are the sigmoids of the chosen logits; weigh_input: they multiply the experts' input; glu_plain_up as above.
  */
 enum { PI_MIXER_LATENT = 0, PI_MIXER_GROUPED = 1, PI_MIXER_LINEAR = 2, PI_MIXER_KEYED = 3 };
 enum { PI_FFN_NONE = 0, PI_FFN_MOE = 1, PI_FFN_GLU = 2, PI_FFN_GLU_MOE = 3 };
+enum { PI_ROT_PLAIN = 0, PI_ROT_WAVES = 1, PI_ROT_RAMP = 2 };
 typedef struct pi_layer_desc {
     int32_t mixer, n_head, dim, rot_dim, vdim, kv_rank, kv_from;
     float   scale;
@@ -882,6 +937,9 @@ typedef struct pi_layer_desc {
     int32_t rot_pairs, qk_norm, unit_v, head_temp, window; float out_scale;
     int32_t mem_heads, mem_dim, mem_vdim; float mem_cap, mem_scale;
     int32_t decay_rank; float decay_tau;
+    float   softcap; int32_t head_sinks, head_mix, head_gate, value_mix;
+    int32_t rot_scaling; double rot_factor, rot_original, rot_low, rot_high;
+    int32_t route_scores, weigh_input;
 } pi_layer_desc;
 typedef struct pi_layers_opts {
     int32_t compute;         /* PI_TYPE_BF16: activations and caches in bf16, fp32 accumulation (residual, norms, router, scores in fp32);
@@ -896,6 +954,7 @@ typedef struct pi_layers_opts {
     int32_t loop_start, loop_stop, loop_times;
     int32_t n_slots;         /* sequences whose recurrent states there is room for at the start (0: 4; grows when more are live) */
     int32_t post_norm; float residual_alpha;
+    int32_t both_norms; float residual_mult; int32_t norm_groups, conv_taps;
 } pi_layers_opts;
 
 /* The ggml_cuda_* boundary (include/ggml_backend_abi.h) keeps single-token nodes in a window until it knows whether they form a block

@@ -49,21 +49,52 @@ struct Layer {
     const float *norm_a = nullptr, *norm_b = nullptr, *dkv_norm = nullptr, *sink = nullptr, *bias = nullptr;
     const void * w_ffn = nullptr;                                 // norm after the sum: [gate and up rows in turn | residual gate]
     const float *q_norm = nullptr, *k_norm = nullptr, *temp = nullptr, *gate_b = nullptr, *gate_ffn_b = nullptr;
+    // norms around the sublayers, convolution of the mixer's input, heads mixed and gated, mixed values
+    const float *norm_a_after = nullptr, *norm_b_after = nullptr, *conv = nullptr, *talk = nullptr, *v_mix = nullptr;
+    int off_head_gate = -1; size_t conv_floats = 0; bool first_values = false;
     // one per pass of the loop the layer is part of
     std::vector<void *> cache;                         // cells
     std::vector<float *> state;                        // [slots][state_floats()]
     size_t cell_values() const { return d.mixer == PI_MIXER_GROUPED ? (size_t)d.n_kv_head * 2 * hd : d.mixer == PI_MIXER_LATENT && own_kv ? (size_t)kd : 0; }
-    size_t state_floats() const { return rec.on() ? pi_k_linear_slot_floats(rec.kind, rec.n_head, rec.dim, rec.vdim) : 0; }
+    // a slot: the recurrent part's state, then the last inputs of the convolution
+    size_t rec_floats() const { return rec.on() ? pi_k_linear_slot_floats(rec.kind, rec.n_head, rec.dim, rec.vdim) : 0; }
+    size_t state_floats() const { return rec_floats() + conv_floats; }
+    bool heads_apart() const { return d.head_mix || d.head_gate; }      // the heads' results are mixed or gated behind the attention
     bool moe() const { return d.ffn == PI_FFN_MOE || d.ffn == PI_FFN_GLU_MOE; }
 };
 
 struct LayerRun { int layer, pass; bool starts; };     // starts: a pass of the loop begins with it
 
-struct Rotation { int dims; double base; };
-// n_head: of a work item's rows - all heads on a latent, the heads of a group otherwise (n_kv groups, kd values of a key row)
+struct Rotation {
+    int dims; double base;
+    int scaling; double factor, original, low, high;
+    const double * freq;                               // device, with a scaling
+    bool same(const pi_layer_desc & d) const {
+        return dims == d.rot_dim && base == d.rot_base && scaling == d.rot_scaling && (!scaling || (factor == d.rot_factor && original == d.rot_original && low == d.rot_low && high == d.rot_high));
+    }
+    double length() const { return scaling == PI_ROT_RAMP ? 0.1 * log(factor) + 1.0 : 1.0; }
+    // what becomes of base^(-2 i / dims)
+    std::vector<double> frequencies() const {
+        std::vector<double> f(dims / 2);
+        const auto pair_of = [&](double turns) { return dims * log(original / (2.0 * M_PI * turns)) / (2.0 * log(base)); };      // the pair that makes so many turns
+        const double first = std::max(floor(pair_of(high)), 0.0), last = std::min(ceil(pair_of(low)), dims - 1.0);
+        for (int i = 0; i < dims / 2; ++i) {
+            f[i] = pow(base, -2.0 * i / dims);
+            double kept = 1.0;                         // share of the frequency that stays as it is
+            if (scaling == PI_ROT_WAVES) {
+                const double turns = original * f[i] / (2.0 * M_PI);
+                kept = turns > high ? 1.0 : turns < low ? 0.0 : (turns - low) / (high - low);
+            } else if (scaling == PI_ROT_RAMP) kept = 1.0 - std::min(std::max((i - first) / std::max(last - first, 0.001), 0.0), 1.0);
+            f[i] = f[i] * kept + f[i] / factor * (1.0 - kept);
+        }
+        return f;
+    }
+};
+// n_head: of a work item's rows - all heads on a latent, the heads of a group otherwise (n_kv groups, with pi_gqa_attn's all_values pairs of them; kd
+// values of a key row)
 // window > 0: cells a token sees
 struct HeadKind { int mixer, n_head, n_kv, dim, rot_dim, vdim, rank_ld, kd, window; };
-enum Family { kTwoNorms, kOneNorm, kPostNorm };
+enum Family { kTwoNorms, kOneNorm, kPostNorm, kBothNorms };
 
 // where a pass finds its tokens
 struct Step {
@@ -82,6 +113,7 @@ struct Step {
     int32_t * prev = nullptr; bool carry = false;
     const int32_t *lin = nullptr, *lin_long = nullptr, *lin_first = nullptr, *lin_chunks = nullptr;
     int n_lin = 0, n_lin_long = 0, n_lin_chunks = 0;
+    const int32_t * conv = nullptr; int n_conv = 0;    // items of the convolutions
 };
 
 }  // namespace
@@ -114,6 +146,7 @@ struct LayerState {
     void *lin_q = nullptr, *lin_k = nullptr, *lin_v = nullptr, *lin_states = nullptr;
     void *h_a = nullptr, *h_b = nullptr, *q_un = nullptr, *q_lat = nullptr, *o_lat = nullptr, *att = nullptr, *act = nullptr, *y_exp = nullptr;
     int32_t *ids = nullptr, *perm = nullptr, *inv = nullptr, *off = nullptr, *tiles = nullptr, *n_tiles = nullptr;
+    float *heads = nullptr, *v_first = nullptr;        // the heads' results ahead of their mixture, the first values of the step's tokens
     std::vector<float *> cs;                           // per rotation [cap][dims / 2] (cos, sin)
     bf16_t * expanded = nullptr; size_t expanded_cap = 0;      // keys and values of a long run's cells
     float * scratch = nullptr;                         // partial sums of a split attention
@@ -123,7 +156,7 @@ struct LayerState {
     // lockstep decoding and the greedy loop
     int n_seq = 0;
     int32_t last_tok[32], last_pos[32];
-    int32_t *g_tok = nullptr, *g_pos = nullptr, *g_cell = nullptr, *g_vis = nullptr, *g_seq = nullptr, *g_work = nullptr, *g_step = nullptr, *g_out = nullptr, *g_prev = nullptr, *g_lin = nullptr;
+    int32_t *g_tok = nullptr, *g_pos = nullptr, *g_cell = nullptr, *g_vis = nullptr, *g_seq = nullptr, *g_work = nullptr, *g_step = nullptr, *g_out = nullptr, *g_prev = nullptr, *g_lin = nullptr, *g_conv = nullptr;
     int max_steps = 4096;
     hipGraph_t graph = nullptr; hipGraphExec_t exec = nullptr;
     int graph_T = 0, graph_seq0 = -1; std::vector<int> graph_parts;
@@ -203,6 +236,25 @@ int vec(pi_model * m, int il, int kind, int64_t n, const char * what, const floa
     return PI_OK;
 }
 
+// the experts of a layer: gate and up rows in turn
+int expert_weights(pi_model * m, int il) {
+    LayerState * s = m->lay;
+    Layer & L = s->layers[il];
+    const pi_layer_desc & d = L.d;
+    const int D = m->hp.n_embd;
+    const auto want = [&](int kind, int64_t ne0, int64_t ne1, const char * what) { return want_tensor(m->L(il, kind), PI_TYPE_BF16, ne0, ne1, what); };
+    const int64_t ne = (int64_t)d.n_expert * d.expert_ff;
+    uint16_t * up = zeroed(m, (size_t)2 * ne * s->d_ld);
+    if (!up) return PI_E_HIP;
+    PI_TRY(want(PI_T_EXPERT_GATE, D, ne, "expert_gate"));
+    PI_TRY(want(PI_T_EXPERT_UP, D, ne, "expert_up"));
+    PI_TRY(want(PI_T_EXPERT_DOWN, d.expert_ff, (int64_t)d.n_expert * D, "expert_down"));
+    PI_TRY(place(m, m->L(il, PI_T_EXPERT_GATE), up, s->d_ld, 0, s->d_ld, 0, 2));
+    PI_TRY(place(m, m->L(il, PI_T_EXPERT_UP), up, s->d_ld, 0, s->d_ld, 1, 2));
+    L.up = up;
+    return padded(m, m->L(il, PI_T_EXPERT_DOWN), L.ff_ld, &L.down);
+}
+
 // A layer with one norm: everything that reads the normed input is one matrix - the mixer's projections, gate and up rows of the dense or
 // shared feed-forward (in turn), its score row, the router - and what closes the layer is one as well, [W_o | W_down].
 int one_norm_weights(pi_model * m, int il) {
@@ -256,16 +308,7 @@ int one_norm_weights(pi_model * m, int il) {
     }
     if (d.ffn != PI_FFN_GLU_MOE) return PI_OK;
     PI_TRY(rows(PI_T_ROUTER, d.n_expert, L.off_router, 1, "router"));
-    const int64_t ne = (int64_t)d.n_expert * d.expert_ff;
-    uint16_t * up = zeroed(m, (size_t)2 * ne * s->d_ld);
-    if (!up) return PI_E_HIP;
-    PI_TRY(want(PI_T_EXPERT_GATE, D, ne, "expert_gate"));
-    PI_TRY(want(PI_T_EXPERT_UP, D, ne, "expert_up"));
-    PI_TRY(want(PI_T_EXPERT_DOWN, d.expert_ff, (int64_t)d.n_expert * D, "expert_down"));
-    PI_TRY(place(m, m->L(il, PI_T_EXPERT_GATE), up, s->d_ld, 0, s->d_ld, 0, 2));
-    PI_TRY(place(m, m->L(il, PI_T_EXPERT_UP), up, s->d_ld, 0, s->d_ld, 1, 2));
-    L.up = up;
-    return padded(m, m->L(il, PI_T_EXPERT_DOWN), L.ff_ld, &L.down);
+    return expert_weights(m, il);
 }
 
 // sizes and places that follow from the description of a layer with one norm
@@ -393,6 +436,65 @@ void post_norm_sizes(Layer & L, int D) {
     L.glu_ld = up_to(d.glu_ff, 128);
 }
 
+// A layer with norms before and after its sublayers: what the mixer projects and the gates of its heads are one matrix.
+int both_norms_weights(pi_model * m, int il) {
+    LayerState * s = m->lay;
+    Layer & L = s->layers[il];
+    const pi_layer_desc & d = L.d;
+    const int D = m->hp.n_embd, hv = d.n_head * d.vdim;
+    const auto want = [&](int kind, int64_t ne0, int64_t ne1, const char * what) { return want_tensor(m->L(il, kind), PI_TYPE_BF16, ne0, ne1, what); };
+    const auto norm = [&](int kind, const char * what, const float ** out) -> int {
+        PI_TRY(want_tensor(m->L(il, kind), PI_TYPE_F32, D, 1, what));
+        return norm_weights(m, m->L(il, kind), s->opts.norm_offset, 1.0f, out);
+    };
+    PI_TRY(norm(PI_T_ATTN_NORM, "attn_norm", &L.norm_a));
+    PI_TRY(norm(PI_T_ATTN_NORM_AFTER, "attn_norm_after", &L.norm_a_after));
+    if (s->opts.conv_taps > 0) {
+        PI_TRY(want_tensor(m->L(il, PI_T_MIX_CONV), PI_TYPE_F32, s->opts.conv_taps, D, "mix_conv"));
+        L.conv = (const float *)m->L(il, PI_T_MIX_CONV).dev;
+    }
+    uint16_t * z = zeroed(m, (size_t)L.z_rows * s->d_ld);
+    if (!z) return PI_E_HIP;
+    L.w_z = z;
+    const auto rows = [&](int kind, int64_t n, int off, const char * what) -> int {
+        PI_TRY(want(kind, D, n, what));
+        return place(m, m->L(il, kind), z, s->d_ld, 0, s->d_ld, off, 1);
+    };
+    PI_TRY(rows(PI_T_MIX_Q, (int64_t)d.n_head * d.dim, 0, "mix_q"));
+    PI_TRY(rows(PI_T_MIX_K, (int64_t)d.n_kv_head * d.dim, L.off_k, "mix_k"));
+    if (L.off_v != L.off_k) PI_TRY(rows(PI_T_MIX_V, (int64_t)d.n_kv_head * d.vdim, L.off_v, "mix_v"));
+    if (d.head_gate) PI_TRY(rows(PI_T_MIX_HEAD_GATE, d.n_head, L.off_head_gate, "mix_head_gate"));
+    if (d.qk_norm) { PI_TRY(vec(m, il, PI_T_MIX_Q_NORM, d.dim, "mix_q_norm", &L.q_norm)); PI_TRY(vec(m, il, PI_T_MIX_K_NORM, d.dim, "mix_k_norm", &L.k_norm)); }
+    if (d.head_temp) PI_TRY(vec(m, il, PI_T_MIX_TEMP, d.n_head, "mix_temp", &L.temp));
+    if (d.head_sinks) PI_TRY(vec(m, il, PI_T_MIX_SINK, d.n_head, "mix_sink", &L.sink));
+    if (d.head_mix) {
+        PI_TRY(want_tensor(m->L(il, PI_T_MIX_TALK), PI_TYPE_F32, d.n_head, d.n_head, "mix_talk"));
+        L.talk = (const float *)m->L(il, PI_T_MIX_TALK).dev;
+    }
+    if (d.value_mix && !L.first_values) PI_TRY(vec(m, il, PI_T_MIX_VALUE, 1, "mix_value", &L.v_mix));
+    PI_TRY(want(PI_T_WO, hv, D, "wo"));
+    PI_TRY(padded(m, m->L(il, PI_T_WO), L.close_ld, &L.wo));
+    if (d.ffn == PI_FFN_NONE) return PI_OK;
+    PI_TRY(norm(PI_T_FFN_NORM, "ffn_norm", &L.norm_b));
+    PI_TRY(norm(PI_T_FFN_NORM_AFTER, "ffn_norm_after", &L.norm_b_after));
+    PI_TRY(want(PI_T_ROUTER, D, d.n_expert, "router"));
+    PI_TRY(padded(m, m->L(il, PI_T_ROUTER), s->d_ld, &L.router));
+    return expert_weights(m, il);
+}
+
+void both_norms_sizes(Layer & L) {
+    const pi_layer_desc & d = L.d;
+    int at = 0;
+    const auto take = [&](int n) { const int o = at; at = up_to(at + n, 16); return o; };
+    take(d.n_head * d.dim);
+    L.off_k = take(d.n_kv_head * d.dim);
+    L.off_v = d.values_are_keys ? L.off_k : take(d.n_kv_head * d.vdim);
+    if (d.head_gate) L.off_head_gate = take(d.n_head);
+    L.z_rows = at;
+    L.hv_ld = L.close_ld = up_to(d.n_head * d.vdim, 128);
+    L.ff_ld = d.ffn == PI_FFN_GLU_MOE ? up_to(d.expert_ff, 64) : 0;
+}
+
 // the recurrent part that a description asks for
 Rec recurrent_part(const pi_layer_desc & d) {
     Rec r;
@@ -471,13 +573,15 @@ int ensure_capacity(pi_model * m, int T) {
     int cap = 64;
     while (cap < T) cap *= 2;
     const size_t es = s->es, D = m->hp.n_embd;
-    size_t z = 0, qu = 0, ql = 0, ol = 0, at = 0, E = 0, top = 0, ff = 0, lq = 0, lv = 0, lo = 0, ls = 0, ln = 0, lg = 0;
+    size_t z = 0, qu = 0, ql = 0, ol = 0, at = 0, E = 0, top = 0, ff = 0, lq = 0, lv = 0, lo = 0, ls = 0, ln = 0, lg = 0, hr = 0, vf = 0;
     const size_t chunks = s->recurrent && bf16_mode(s) ? (size_t)cap / pi_k_linear_chunk() + 32 : 0;        // every run of a pass ends with a part of one
     for (const Layer & L : s->layers) {
         const pi_layer_desc & d = L.d;
         if (s->family != kTwoNorms) {
             z = std::max({z, (size_t)L.z_rows, (size_t)L.z2_rows}); at = std::max({at, (size_t)L.close_ld, (size_t)L.glu_ld});
             if (d.mixer == PI_MIXER_GROUPED) ql = std::max(ql, (size_t)d.n_head * L.hd);
+            if (L.heads_apart()) hr = std::max(hr, (size_t)d.n_head * d.n_kv_head * d.vdim);
+            if (d.value_mix) vf = std::max(vf, (size_t)d.n_kv_head * d.vdim);
             const Rec & r = L.rec;
             if (r.on()) {
                 lo = std::max(lo, (size_t)r.n_head * r.vdim);
@@ -516,7 +620,7 @@ int ensure_capacity(pi_model * m, int T) {
         carve(s->tiles, (n * top / 64 + E + 1) * 8); carve(s->n_tiles, 4);
         carve(s->x0, s->opts.loop_times > 0 ? n * D * 4 : 0);
         carve(s->lin_o, n * lo * 4); carve(s->lin_q, n * lq * 2); carve(s->lin_k, n * lq * 2); carve(s->lin_v, n * lv * 2); carve(s->lin_states, ls);
-        carve(s->lin_den, n * ln * 4); carve(s->lin_gates, lg * 4);
+        carve(s->lin_den, n * ln * 4); carve(s->lin_gates, lg * 4); carve(s->heads, n * hr * 4); carve(s->v_first, n * vf * 4);
         s->cs.resize(s->rots.size());
         for (size_t r = 0; r < s->rots.size(); ++r) carve(s->cs[r], n * s->rots[r].dims * 4);
     };
@@ -672,10 +776,11 @@ int experts(pi_model * m, Layer & L, const void * h, const Step & in) {
     PI_TRY(pi_k_moe_sort(s->ids, T * d.n_top, d.n_expert, s->off, s->perm, s->inv, tile_n, s->tiles, s->n_tiles, st));
     pi_group_gemm g{};
     g.W = L.up; g.w_gs = (size_t)per * d.expert_ff * s->d_ld; g.rows = per * d.expert_ff; g.cols = s->d_ld; g.ldw = s->d_ld; g.n_group = d.n_expert; g.alpha = 1.0f;
-    if (per == 2) { g.glu = 1; g.glu_limit = d.expert_limit; g.glu_gain = d.glu_gain; }
+    if (per == 2) { g.glu = 1; g.glu_limit = d.expert_limit; g.glu_gain = d.glu_gain; g.glu_plain_up = d.glu_plain_up; }
     else g.relu2 = 1;
     g.x = h; g.ldx = s->d_ld; g.T = T; g.y = s->act; g.ldy = L.ff_ld; g.off = s->off; g.gather = s->perm; g.gather_div = d.n_top;
     g.tiles = s->tiles; g.n_tiles = s->n_tiles; g.max_tiles = T * d.n_top / tile_n + d.n_expert;
+    g.pair_w = d.weigh_input ? s->wts : nullptr;
     PI_TRY(grouped(s, g, tile_n, st));
     pi_group_gemm w{};
     w.W = L.down; w.w_gs = (size_t)D * L.ff_ld; w.rows = D; w.cols = L.ff_ld; w.ldw = L.ff_ld; w.n_group = d.n_expert; w.alpha = 1.0f;
@@ -699,6 +804,8 @@ pi_gqa_attn gqa_args(pi_model * m, const Layer & L, int pass, const Step & in, c
     a.q = s->q_lat; a.cache = L.cache[pass]; a.lists = s->lists; a.list_ld = s->kv.n; a.work = bf16_mode(s) ? w.items : in.seq; a.n_vis = in.n_vis; a.n_work = w.n; a.T = in.T;
     a.n_head = d.n_head; a.n_kv = d.n_kv_head; a.dim = d.dim; a.vdim = d.vdim; a.hd = L.hd; a.n_parts = w.parts; a.wide = wide; a.scale = d.scale; a.sink = d.sink;
     a.scratch = s->scratch; a.att = s->att; a.ld_att = L.close_ld; a.out_scale = s->family == kPostNorm ? d.out_scale : 1.0f; a.window = d.window; a.first = in.first[L.hc];
+    a.softcap = d.softcap; a.sinks = d.head_sinks ? L.sink : nullptr;
+    if (L.heads_apart()) { a.all_values = 1; a.att = s->heads; }
     return a;
 }
 
@@ -709,6 +816,7 @@ pi_gqa_prep gqa_prep_args(pi_model * m, const Layer & L, int pass, const Step & 
     p.z = s->z; p.ldz = L.z_rows; p.T = in.T; p.n_head = d.n_head; p.n_kv = d.n_kv_head; p.dim = d.dim; p.vdim = d.vdim; p.rot_dim = d.rot_dim; p.off_k = L.off_k; p.off_v = L.off_v;
     p.hd = L.hd; p.unit = d.unit_qk; p.cs = L.rot >= 0 ? s->cs[L.rot] : s->x; p.eps = m->hp.norm_eps; p.q = s->q_lat; p.cache = L.cache[pass]; p.cell = in.cell;
     p.rot_pairs = d.rot_pairs; p.unit_v = d.unit_v; p.q_norm = L.q_norm; p.k_norm = L.k_norm; p.temp = L.temp;
+    if (d.value_mix) { p.ld_first = d.n_kv_head * d.vdim; if (L.first_values) p.v_keep = s->v_first; else { p.v_first = s->v_first; p.v_mix = L.v_mix; } }
     return p;
 }
 
@@ -861,6 +969,63 @@ int post_norm_layer(pi_model * m, Layer & L, const LayerRun & r, const Step & in
     return close(L.down, L.glu_ld, gated ? s->z : nullptr, L.z2_rows, L.off_gate_ffn, L.gate_ffn_b, L.norm_b, keep);
 }
 
+// A layer with norms before and after its sublayers.  Steps of up to 16 tokens (bf16) stream the weights past operands in the matrix cores' layout; the
+// sum that closes a sublayer and the norm ahead of the feed-forward are one launch, the norm ahead of the mixer and its convolution another.
+int both_norms_layer(pi_model * m, Layer & L, const LayerRun & r, const Step & in, float * keep) {
+    LayerState * s = m->lay;
+    const pi_layer_desc & d = L.d;
+    const int T = in.T, D = m->hp.n_embd, type = s->opts.compute;
+    const bool moe = L.moe(), step = bf16_mode(s) && pi_k_layer_step_supported(T, moe ? d.n_expert : 0, moe ? d.n_top : 0);
+    hipStream_t st = m->stream;
+    if (L.conv) {
+        pi_conv_norm c{};
+        c.x = s->x; c.w = L.norm_a; c.taps_w = L.conv; c.T = T; c.cols = D; c.groups = s->opts.norm_groups; c.taps = s->opts.conv_taps; c.eps = m->hp.norm_eps;
+        c.state = L.conv_floats ? L.state[r.pass] + L.rec_floats() : nullptr; c.slot_ld = L.state_floats(); c.items = in.conv; c.n_items = in.n_conv; c.h = s->h_a; c.ld = s->d_ld; c.ol = step;
+        PI_TRY(pi_k_conv_norm(type, &c, st));
+    } else {
+        pi_sum_norm n{};
+        n.x = s->x; n.w_next = L.norm_a; n.T = T; n.cols = D; n.groups = s->opts.norm_groups; n.eps = m->hp.norm_eps; n.h = s->h_a; n.ld = s->d_ld; n.ol = step;
+        PI_TRY(pi_k_sum_norm(type, &n, st));
+    }
+    const auto product = [&](const void * W, int rows, const void * h, float * y) -> int {
+        return step ? pi_k_gemm_bf16_ol(W, rows, s->d_ld, h, T, PI_EPI_NONE, nullptr, nullptr, y, nullptr, st) : dense(m, W, rows, s->d_ld, h, T, y);
+    };
+    PI_TRY(product(L.w_z, L.z_rows, s->h_a, s->z));
+    const pi_gqa_prep p = gqa_prep_args(m, L, r.pass, in);
+    PI_TRY(pi_k_gqa_prep(type, &p, nullptr, st));
+    pi_gqa_attn parts{};
+    PI_TRY(attend_grouped(m, L, r.pass, in, step, parts));
+    if (parts.n_parts > 1) PI_TRY(pi_k_mix_up_step(&parts, nullptr, nullptr, 0, 0, 0, 0.0f, 0.0f, nullptr, T, nullptr, nullptr, 0, nullptr, 0, st));
+    if (L.heads_apart()) {
+        pi_gqa_mix x{};
+        x.a = s->heads; x.talk = L.talk; x.z = s->z; x.ldz = L.z_rows; x.off_gate = L.off_head_gate; x.T = T; x.n_head = d.n_head; x.n_kv = d.n_kv_head; x.vdim = d.vdim;
+        x.att = s->att; x.ld_att = L.close_ld;
+        PI_TRY(pi_k_gqa_mix(type, &x, st));
+    }
+    pi_layer_out o{};
+    o.rows = D; o.T = T; o.out = s->mix;
+    if (step) { o.wo = L.wo; o.att = s->att; o.ld_att = L.close_ld; PI_TRY(pi_k_layer_out_step(&o, st)); }
+    else PI_TRY(dense(m, L.wo, D, L.close_ld, s->att, T, s->mix));
+    pi_sum_norm n{};
+    n.x = s->x; n.mix = s->mix; n.w = L.norm_a_after; n.mult = s->opts.residual_mult; n.T = T; n.cols = D; n.groups = s->opts.norm_groups; n.eps = m->hp.norm_eps;
+    n.ld = s->d_ld; n.ol = step;
+    if (moe) { n.h = s->h_b; n.w_next = L.norm_b; } else n.keep = keep;
+    PI_TRY(pi_k_sum_norm(type, &n, st));
+    if (!moe) return PI_OK;
+    PI_TRY(product(L.router, d.n_expert, s->h_b, s->rl));
+    PI_TRY(pi_k_route_scores(s->rl, T, d.n_expert, d.n_top, s->ids, s->wts, st));
+    n.w = L.norm_b_after; n.w_next = nullptr; n.h = nullptr; n.keep = keep;
+    if (step) {
+        PI_TRY(pi_k_expert_up_step(L.up, d.n_expert, d.expert_ff, s->d_ld, d.expert_limit, d.glu_gain, d.glu_plain_up, d.weigh_input, s->h_b, T, s->ids, s->wts, d.n_top, s->act, L.ff_ld, st));
+        o.wo = nullptr; o.down = L.down; o.act = s->act; o.ids = s->ids; o.ld_act = L.ff_ld; o.top = d.n_top; o.n_expert = d.n_expert;
+        PI_TRY(pi_k_layer_out_step(&o, st));
+    } else {
+        PI_TRY(experts(m, L, s->h_b, in));
+        n.mix = nullptr; n.y = s->y_exp; n.inv = s->inv; n.top = d.n_top; n.y_w = d.weigh_input ? nullptr : s->wts;
+    }
+    return pi_k_sum_norm(type, &n, st);
+}
+
 // a layer of a step of up to 16 tokens (bf16): six launches
 int step_layer(pi_model * m, Layer & L, const Step & in, float * keep) {
     LayerState * s = m->lay;
@@ -895,11 +1060,18 @@ int pass_layers(pi_model * m, const Step & in) {
         n.x = n.out = s->x; n.T = T; n.cols = D; n.h = s->h_a; n.ld = s->d_ld; n.ol = bf16_mode(s) && pi_k_layer_step_supported(T, 0, 0);
         PI_TRY(pi_k_res_norm(type, &n, st));
     }
-    for (size_t r = 0; r < s->rots.size(); ++r) PI_TRY(pi_k_rope_angles(in.pos, T, s->rots[r].dims, s->rots[r].base, s->cs[r], st));
+    for (size_t k = 0; k < s->rots.size(); ++k) {
+        const Rotation & r = s->rots[k];
+        PI_TRY(r.scaling ? pi_k_rope_angles_table(in.pos, T, r.dims, r.freq, r.length(), s->cs[k], st) : pi_k_rope_angles(in.pos, T, r.dims, r.base, s->cs[k], st));
+    }
     for (size_t k = 0; k < s->order.size(); ++k) {
         Layer & L = s->layers[s->order[k].layer];
         const bool moe = L.moe();
         float * keep = s->streams_T ? s->streams + k * (size_t)s->streams_T * D : nullptr;
+        if (s->family == kBothNorms) {
+            PI_TRY(both_norms_layer(m, L, s->order[k], in, keep));
+            continue;
+        }
         if (s->family == kPostNorm) {
             PI_TRY(post_norm_layer(m, L, s->order[k], in, keep));
             continue;
@@ -928,7 +1100,11 @@ int pass_head(pi_model * m, const int32_t * rows, int n) {
     LayerState * s = m->lay;
     const int D = m->hp.n_embd;
     const bool ol = bf16_mode(s) && n <= 16;
-    if (s->family == kOneNorm) PI_TRY(pi_k_layer_norm(s->opts.compute, s->x, rows, n, D, m->hp.norm_eps, s->out_norm, nullptr, nullptr, s->h_head, s->d_ld, ol, m->stream));
+    if (s->family == kBothNorms) {
+        pi_sum_norm h{};
+        h.x = s->x; h.w_next = s->out_norm; h.rows = rows; h.T = n; h.cols = D; h.groups = s->opts.norm_groups; h.eps = m->hp.norm_eps; h.h = s->h_head; h.ld = s->d_ld; h.ol = ol;
+        PI_TRY(pi_k_sum_norm(s->opts.compute, &h, m->stream));
+    } else if (s->family == kOneNorm) PI_TRY(pi_k_layer_norm(s->opts.compute, s->x, rows, n, D, m->hp.norm_eps, s->out_norm, nullptr, nullptr, s->h_head, s->d_ld, ol, m->stream));
     else PI_TRY(pi_k_norm_pair(s->opts.compute, s->x, rows, n, D, m->hp.norm_eps, s->out_norm, s->h_head, nullptr, nullptr, s->d_ld, ol, m->stream));
     if (ol) return pi_k_gemm_bf16_ol(s->head, m->hp.n_vocab, s->d_ld, s->h_head, n, PI_EPI_NONE, nullptr, nullptr, s->logits, nullptr, m->stream);
     return dense(m, s->head, m->hp.n_vocab, s->d_ld, s->h_head, n, s->logits);
@@ -1030,7 +1206,9 @@ int apply_shift(pi_model * m) {
     PI_TRY(pi_memcpy_h2d(s->d_delta, s->kv.delta.data(), sizeof(int32_t) * s->kv.n));
     for (Layer & L : s->layers) {
         if (L.d.mixer == PI_MIXER_GROUPED)
-            for (void * c : L.cache) PI_TRY(pi_k_gqa_shift(s->opts.compute, c, s->kv.n, L.d.n_kv_head, L.hd, L.d.rot_dim, L.d.rot_base, L.d.rot_pairs, s->d_delta, m->stream));
+            for (void * c : L.cache)
+                PI_TRY(L.d.rot_scaling ? pi_k_gqa_shift_table(s->opts.compute, c, s->kv.n, L.d.n_kv_head, L.hd, L.d.rot_dim, s->rots[L.rot].freq, L.d.rot_pairs, s->d_delta, m->stream)
+                                       : pi_k_gqa_shift(s->opts.compute, c, s->kv.n, L.d.n_kv_head, L.hd, L.d.rot_dim, L.d.rot_base, L.d.rot_pairs, s->d_delta, m->stream));
         else if (L.cell_values()) PI_TRY(pi_k_latent_shift(s->opts.compute, L.cache[0], s->kv.n, L.kd, L.rank_ld, L.d.rot_dim, L.d.rot_base, s->d_delta, m->stream));
     }
     PI_HIP_TRY(hipStreamSynchronize(m->stream));
@@ -1172,11 +1350,21 @@ int layers_finalize(pi_model * m) {
     for (size_t il = 0; il < s->layers.size(); ++il) {
         Layer & L = s->layers[il];
         const pi_layer_desc & d = L.d;
-        const auto rotation = [&]() {
+        const auto rotation = [&]() -> int {
             size_t r = 0;
-            while (r < s->rots.size() && (s->rots[r].dims != d.rot_dim || s->rots[r].base != d.rot_base)) ++r;
-            if (r == s->rots.size()) s->rots.push_back({d.rot_dim, d.rot_base});
+            while (r < s->rots.size() && !s->rots[r].same(d)) ++r;
             L.rot = (int)r;
+            if (r < s->rots.size()) return PI_OK;
+            Rotation n{d.rot_dim, d.rot_base, d.rot_scaling, d.rot_factor, d.rot_original, d.rot_low, d.rot_high, nullptr};
+            if (n.scaling) {
+                const std::vector<double> f = n.frequencies();
+                double * p = m->alloc<double>(f.size());
+                if (!p) return PI_E_HIP;
+                PI_TRY(pi_memcpy_h2d(p, f.data(), sizeof(double) * f.size()));
+                n.freq = p;
+            }
+            s->rots.push_back(n);
+            return PI_OK;
         };
         const auto kind = [&](const HeadKind & hk) {
             size_t h = 0;
@@ -1185,17 +1373,17 @@ int layers_finalize(pi_model * m) {
             L.hc = (int)h;
         };
         if (s->family != kTwoNorms) {
-            if (s->family == kOneNorm) one_norm_sizes(L); else post_norm_sizes(L, D);
+            if (s->family == kOneNorm) one_norm_sizes(L); else if (s->family == kBothNorms) both_norms_sizes(L); else post_norm_sizes(L, D);
             if (d.mixer == PI_MIXER_GROUPED) {
                 L.hd = pi_k_gqa_head_ld(s->opts.compute, d.dim, d.vdim);
                 if (!L.hd) return fail(PI_E_UNSUPPORTED, "pi_model_finalize: head sizes outside the attention kernels (up to 256)");
-                if (d.rot_dim > 0) rotation(); else L.rot = -1;
-                kind(HeadKind{d.mixer, d.n_head / d.n_kv_head, d.n_kv_head, 0, 0, 0, 0, L.hd, d.window});
+                if (d.rot_dim > 0) PI_TRY(rotation()); else L.rot = -1;
+                kind(HeadKind{d.mixer, d.n_head / d.n_kv_head, d.n_kv_head * (L.heads_apart() ? d.n_kv_head : 1), 0, 0, 0, 0, L.hd, d.window});
                 scratch = std::max(scratch, pi_k_gqa_scratch_floats(kAttnItems, 1, 1, L.hd, 2) / 2);      // items x groups x parts <= kAttnItems
             }
             if (L.rec.on() && !pi_k_linear_supported(L.rec.dim, L.rec.vdim)) return fail(PI_E_UNSUPPORTED, "pi_model_finalize: head sizes outside the linear attention's kernels (up to 256)");
             if (d.weights_of) continue;
-            PI_TRY(s->family == kOneNorm ? one_norm_weights(m, (int)il) : post_norm_weights(m, (int)il));
+            PI_TRY(s->family == kOneNorm ? one_norm_weights(m, (int)il) : s->family == kBothNorms ? both_norms_weights(m, (int)il) : post_norm_weights(m, (int)il));
             continue;
         }
         L.own_kv = d.kv_from < 0;
@@ -1204,7 +1392,7 @@ int layers_finalize(pi_model * m) {
         L.dim_ld = up_to(d.dim, 64); L.rank_ld = up_to(d.kv_rank, 64); L.kd = L.rank_ld + up_to(d.rot_dim, 32);
         L.hv_ld = up_to(d.n_head * d.vdim, 128); L.ff_ld = d.ffn == PI_FFN_MOE ? up_to(d.expert_ff, 64) : 0;
         if (!pi_k_latent_attn_supported(s->opts.compute, L.rank_ld, L.kd)) return fail(PI_E_UNSUPPORTED, "pi_model_finalize: latent sizes outside the attention kernels (rank up to 1024)");
-        rotation();
+        PI_TRY(rotation());
         kind(HeadKind{d.mixer, d.n_head, 1, d.dim, d.rot_dim, d.vdim, L.rank_ld, L.kd, 0});
         scratch = std::max(scratch, pi_k_latent_attn_scratch_floats(kItemRows * kAttnItems / 2, L.rank_ld, 2));      // items x parts <= kAttnItems
         PI_TRY(layer_weights(m, (int)il));
@@ -1222,7 +1410,8 @@ int layers_finalize(pi_model * m) {
     PI_TRY(head_buffers(m));
     if (s->recurrent) PI_TRY(resize_slots(m, s->opts.n_slots > 0 ? s->opts.n_slots : 4));
     s->g_lin = m->alloc<int32_t>(4 * kMaxLockstep);
-    if (!s->g_lin) return PI_E_HIP;
+    s->g_conv = m->alloc<int32_t>(8 * kMaxLockstep);
+    if (!s->g_lin || !s->g_conv) return PI_E_HIP;
     for (int32_t ** p : {&s->g_tok, &s->g_pos, &s->g_cell, &s->g_vis, &s->g_seq, &s->g_step, &s->g_prev}) {
         *p = m->alloc<int32_t>(kMaxLockstep);
         if (!*p) return PI_E_HIP;
@@ -1310,6 +1499,23 @@ int layers_step(pi_model * m, const int32_t * tokens, const int32_t * positions,
         begin.push_back(items.size());
         begin_wide.push_back(wide.size());
         items.insert(items.end(), wide.begin(), wide.end());
+        const size_t at_conv = items.size();
+        if (s->opts.conv_taps > 0) {
+            const int back = s->opts.conv_taps - 1, per = pi_k_conv_tokens(T, s->opts.conv_taps);
+            for (int a = 0; a < T;) {
+                int b = a + 1;
+                while (b < T && seq[t0 + b] == seq[t0 + a]) ++b;
+                const int q = seq[t0 + a];
+                for (int c = a; c < b;) {
+                    const int n = std::min(c == a ? std::max(per, back) : per, b - c);
+                    const int32_t item[8] = {c, n, c - a, b - a, std::max(s->slot_of[q], 0), (int32_t)(fresh >> q & 1u), 0, 0};
+                    items.insert(items.end(), item, item + 8);
+                    c += n;
+                }
+                a = b;
+            }
+            in.n_conv = (int)(items.size() - at_conv) / 8;
+        }
         const size_t at_lin = items.size();
         if (s->recurrent) {                                       // runs walked token by token, long runs, their first chunks, the chunks
             std::vector<int32_t> lng, first, chunks;
@@ -1358,6 +1564,7 @@ int layers_step(pi_model * m, const int32_t * tokens, const int32_t * positions,
         if (!rows.empty()) memcpy(h + 8 * T + items.size(), rows.data(), 4 * rows.size());
         PI_HIP_TRY(hipMemcpyAsync(s->d_in, h, 4 * n_in, hipMemcpyHostToDevice, m->stream));
         in.tokens = s->d_in; in.pos = s->d_in + T; in.cell = s->d_in + 2 * T; in.n_vis = s->d_in + 3 * T; in.seq = s->d_in + 4 * T; in.prev = s->d_in + 5 * T;
+        in.conv = s->d_in + 8 * T + at_conv;
         in.lin = s->d_in + 8 * T + at_lin; in.lin_long = in.lin + 4 * in.n_lin; in.lin_first = in.lin_long + 4 * in.n_lin_long; in.lin_chunks = in.lin_first + in.n_lin_long;
         for (size_t k = 0; k < s->kinds.size(); ++k) {
             Step::Work w;
@@ -1527,6 +1734,12 @@ int layers_generate(pi_model * m, int own, int n_steps, int32_t * out_tokens, fl
         in.lin = s->g_lin; in.n_lin = T;
         PI_TRY(pi_memcpy_h2d(s->g_lin, lin.data(), 16 * T));
     }
+    if (s->opts.conv_taps > 0) {
+        std::vector<int32_t> conv;
+        for (int t = 0; t < T; ++t) { const int32_t item[8] = {t, 1, 0, 1, std::max(s->slot_of[q0 + t], 0), 0, 0, 0}; conv.insert(conv.end(), item, item + 8); }
+        in.conv = s->g_conv; in.n_conv = T;
+        PI_TRY(pi_memcpy_h2d(s->g_conv, conv.data(), 4 * conv.size()));
+    }
     in.prev = s->g_prev; in.carry = true;
     PI_TRY(pi_memcpy_h2d(s->g_prev, prev.data(), 4 * T));
     const int32_t zero = 0;
@@ -1623,16 +1836,31 @@ extern "C" {
 
 pi_model * pi_model_create_layers(const pi_hparams * hp, const pi_layers_opts * opts, const pi_layer_desc * layers, int n_layer) {
     const auto bad = [](const char * why) -> pi_model * { pi::set_error(why); return nullptr; };
-    if (!hp || !opts || !layers || n_layer <= 0 || hp->n_embd <= 0 || hp->n_vocab <= 0 || hp->n_ctx <= 0 || (hp->arch != PI_ARCH_LERASUN && hp->arch != PI_ARCH_PIBALORN && hp->arch != PI_ARCH_FIKEVIK) ||
+    if (!hp || !opts || !layers || n_layer <= 0 || hp->n_embd <= 0 || hp->n_vocab <= 0 || hp->n_ctx <= 0 || (hp->arch != PI_ARCH_LERASUN && hp->arch != PI_ARCH_PIBALORN && hp->arch != PI_ARCH_FIKEVIK && hp->arch != PI_ARCH_PUFIVIK) ||
         (opts->compute != PI_TYPE_BF16 && opts->compute != PI_TYPE_F32) || opts->max_batch < 0)
         return bad("pi_model_create_layers: inconsistent hyper-parameters");
-    const Family family = opts->post_norm ? kPostNorm : layers[0].mixer != PI_MIXER_LATENT ? kOneNorm : kTwoNorms;
+    const Family family = opts->both_norms ? kBothNorms : opts->post_norm ? kPostNorm : layers[0].mixer != PI_MIXER_LATENT ? kOneNorm : kTwoNorms;
+    if (opts->both_norms && (opts->post_norm || opts->norm_groups <= 0 || hp->n_embd % opts->norm_groups || opts->norm_groups > 1024 || opts->conv_taps < 0 || opts->conv_taps > 64))
+        return bad("pi_model_create_layers: norm_groups parts of n_embd (up to 1024) and up to 64 conv_taps");
+    if (!opts->both_norms && opts->conv_taps) return bad("pi_model_create_layers: conv_taps needs both_norms");
+    const pi_layer_desc * first_values = nullptr;      // the first layer with value_mix
     for (int il = 0; il < n_layer; ++il) {
         const pi_layer_desc & d = layers[il];
+        if (family != kBothNorms && (d.softcap != 0.0f || d.head_sinks || d.head_mix || d.head_gate || d.value_mix || d.rot_scaling || d.route_scores || d.weigh_input))
+            return bad("pi_model_create_layers: soft caps, mixed heads and values, scaled rotations and scores of experts need both_norms");
+        if (family == kBothNorms) {
+            if (d.mixer != PI_MIXER_GROUPED || (d.ffn != PI_FFN_NONE && (d.ffn != PI_FFN_GLU_MOE || d.glu_ff || !d.route_scores))) return bad("pi_model_create_layers: a layer's mixer or feed-forward");
+            if (!(d.softcap >= 0.0f) || (d.head_mix && d.n_head > 128)) return bad("pi_model_create_layers: a layer's soft cap or its heads (up to 128 are mixed)");
+            if (d.rot_scaling < PI_ROT_PLAIN || d.rot_scaling > PI_ROT_RAMP || (d.rot_scaling && (!(d.rot_factor > 0.0) || !(d.rot_original > 0.0) || !(d.rot_low > 0.0) || !(d.rot_high > 0.0) ||
+                (d.rot_scaling == PI_ROT_RAMP && !(d.rot_base > 1.0)))))
+                return bad("pi_model_create_layers: a layer's rotation");
+            if (d.value_mix && !first_values) first_values = &d;
+            if (d.value_mix && (d.values_are_keys || d.n_kv_head * d.vdim != first_values->n_kv_head * first_values->vdim)) return bad("pi_model_create_layers: layers that mix values need as many of them");
+        }
         if ((d.mixer == PI_MIXER_LATENT) != (family == kTwoNorms)) return bad("pi_model_create_layers: layers of several families in one model");
         if (family != kPostNorm && (d.weights_of || d.gated_residual || d.mem_heads)) return bad("pi_model_create_layers: shared weights, gated residuals and memories need post_norm");
         if (family != kTwoNorms) {
-            if ((d.mixer != PI_MIXER_GROUPED && d.mixer != (family == kOneNorm ? PI_MIXER_LINEAR : PI_MIXER_KEYED)) || d.n_head <= 0 || d.dim <= 0 || d.vdim <= 0)
+            if ((d.mixer != PI_MIXER_GROUPED && d.mixer != (family == kPostNorm ? PI_MIXER_KEYED : PI_MIXER_LINEAR)) || d.n_head <= 0 || d.dim <= 0 || d.vdim <= 0)
                 return bad("pi_model_create_layers: a layer's mixer");
             if (d.mixer == PI_MIXER_GROUPED && (d.n_kv_head <= 0 || d.n_head % d.n_kv_head || d.rot_dim < 0 || d.rot_dim % 2 || d.rot_dim > d.dim || (d.rot_dim && !(d.rot_base > 0.0)) ||
                                                 (d.values_are_keys && d.vdim != d.dim) || d.window < 0 || (d.qk_norm && d.unit_qk)))
@@ -1683,7 +1911,9 @@ pi_model * pi_model_create_layers(const pi_hparams * hp, const pi_layers_opts * 
         L.d = layers[il];
         const int passes = il >= lo && il < hi ? opts->loop_times : 1;
         L.rec = recurrent_part(L.d);
-        if (L.rec.on()) { L.state.resize(passes, nullptr); s->recurrent = true; }
+        if (opts->conv_taps > 1) L.conv_floats = (size_t)(opts->conv_taps - 1) * hp->n_embd;
+        L.first_values = &layers[il] == first_values;
+        if (L.state_floats()) { L.state.resize(passes, nullptr); s->recurrent = true; }
         if (L.d.mixer == PI_MIXER_GROUPED || (L.d.mixer == PI_MIXER_LATENT && L.d.kv_from < 0)) L.cache.resize(passes, nullptr);
         s->layers.push_back(L);
     }

@@ -34,12 +34,19 @@ __device__ __forceinline__ pi_s4 tr_read(const unsigned char * q) {
 
 template <int KS, bool WIDE> constexpr size_t gqa_lds() { return (size_t)2 * (WIDE ? 64 : 128) * (KS * 64 + 16); }
 
-template <int KS, bool WIDE>      // 32-column steps of a key or value row
+// EXT: soft caps, a sink per head, every head against the values of every key / value head (all_values)
+__device__ __forceinline__ int gqa_groups(const pi_gqa_attn & p) { return p.all_values ? p.n_kv * p.n_kv : p.n_kv; }
+// cap * tanh(v * k / (2 log2 e)): k = 2 log2 e / cap
+__device__ __forceinline__ float soft_cap(float v, float k, float cap) { return fmaf(-2.0f * cap, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(v * k) + 1.0f), cap); }
+constexpr float kTwoLog2E = 2.8853900817779268f;
+
+template <int KS, bool WIDE, bool EXT>      // 32-column steps of a key or value row
 __global__ __launch_bounds__(256, WIDE && KS <= 4 ? 2 : 1) void gqa_attn_kernel(pi_gqa_attn p) {
     constexpr int VT = 2 * KS, NK = WIDE ? 64 : 128, R = WIDE ? 128 : 16, U = WIDE ? 2 : 1, KT = WIDE ? 4 : 2, ROW = KS * 64 + 16, NKK = NK / 32, HD = KS * 32;
     extern __shared__ __align__(16) unsigned char smem[];
     unsigned char * ks = smem, * vs = smem + NK * ROW;
-    const int g = blockIdx.x % p.n_kv, item_index = p.n_work - 1 - (int)blockIdx.x / p.n_kv, part = blockIdx.y;      // the last items see the most cells
+    const int n_groups = EXT ? gqa_groups(p) : p.n_kv, vg = blockIdx.x % n_groups, item_index = p.n_work - 1 - (int)blockIdx.x / n_groups, part = blockIdx.y;      // the last items see the most cells
+    const int g = EXT && p.all_values ? vg / p.n_kv : vg, gv = EXT && p.all_values ? vg % p.n_kv : vg;      // the group's keys and whose values
     const int4 item = reinterpret_cast<const int4 *>(p.work)[item_index];
     const int tok0 = item.x, first = item.y, rows = min(item.z, R), per = p.n_head / p.n_kv;
     const int32_t * list = p.lists + (size_t)item.w * p.list_ld;
@@ -62,7 +69,7 @@ __global__ __launch_bounds__(256, WIDE && KS <= 4 ? 2 : 1) void gqa_attn_kernel(
 #pragma unroll
         for (int k = 0; k < NKK; ++k)
 #pragma unroll
-            for (int j = 0; j < KS; ++j) pre[k][j] = pi_ld16(cache + (size_t)idx[k] * p.n_kv * 2 * HD + j * 64);
+            for (int j = 0; j < KS; ++j) pre[k][j] = pi_ld16(cache + (size_t)idx[k] * p.n_kv * 2 * HD + j * 64 + (EXT && sub + 8 * j >= 4 * KS ? (gv - g) * 2 * HD : 0));
     };
     if (c0 < c1) look_up(c0);
     int row[U], tok[U], head[U], lo[U];
@@ -89,6 +96,7 @@ __global__ __launch_bounds__(256, WIDE && KS <= 4 ? 2 : 1) void gqa_attn_kernel(
         for (int v = 0; v < VT; ++v) o[u][v] = pi_f4{0, 0, 0, 0};
     }
     const int kb = WIDE ? 0 : wave * 32;                         // this wave's cells of a tile
+    const float cap_k = EXT && p.softcap > 0.0f ? kTwoLog2E / p.softcap : 0.0f;
     for (int cb = c0; cb < c1; cb += NK) {
         __syncthreads();
 #pragma unroll
@@ -123,6 +131,7 @@ __global__ __launch_bounds__(256, WIDE && KS <= 4 ? 2 : 1) void gqa_attn_kernel(
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
                     float v = s[u][kt][r] * p.scale;
+                    if (EXT && p.softcap > 0.0f) v = soft_cap(v, cap_k, p.softcap);
                     if (edge && (unsigned)(cb + kb + kt * 16 + 4 * gq + r - lo[u]) >= nv[u]) v = -INFINITY;
                     s[u][kt][r] = v;
                     mx = fmaxf(mx, v);
@@ -164,8 +173,8 @@ __global__ __launch_bounds__(256, WIDE && KS <= 4 ? 2 : 1) void gqa_attn_kernel(
 #pragma unroll
     for (int u = 0; u < U; ++u) { l[u] += __shfl_xor(l[u], 16, PI_WAVE); l[u] += __shfl_xor(l[u], 32, PI_WAVE); }
     const bool whole = p.n_parts == 1, quads = ((p.vdim | p.ld_att) & 3) == 0;
-    const size_t srow0 = ((size_t)item_index * p.n_kv + g) * R;
-    float2 * ml = reinterpret_cast<float2 *>(p.scratch + (size_t)p.n_work * p.n_kv * R * p.n_parts * HD);
+    const size_t srow0 = ((size_t)item_index * n_groups + vg) * R;
+    float2 * ml = reinterpret_cast<float2 *>(p.scratch + (size_t)p.n_work * n_groups * R * p.n_parts * HD);
     if (WIDE) {
 #pragma unroll
         for (int u = 0; u < U; ++u) {
@@ -177,7 +186,18 @@ __global__ __launch_bounds__(256, WIDE && KS <= 4 ? 2 : 1) void gqa_attn_kernel(
                 if (gq == 0) ml[(srow0 + row[u]) * p.n_parts + part] = make_float2(m[u], l[u]);
                 continue;
             }
-            const float mf = fmaxf(m[u], p.sink), a = m[u] == -INFINITY ? 0.0f : expf(m[u] - mf), f = a / (l[u] * a + expf(p.sink - mf)) * p.out_scale;
+            const float sink = EXT && p.sinks ? p.sinks[head[u]] : p.sink;
+            const float mf = fmaxf(m[u], sink), a = m[u] == -INFINITY ? 0.0f : expf(m[u] - mf), f = a / (l[u] * a + expf(sink - mf)) * p.out_scale;
+            if (EXT && p.all_values) {
+                float * out = (float *)p.att + (((size_t)tok[u] * p.n_head + head[u]) * p.n_kv + gv) * p.vdim;
+#pragma unroll
+                for (int v = 0; v < VT; ++v) {
+                    const int c = v * 16 + 4 * gq;
+                    const float w[4] = {o[u][v][0] * f, o[u][v][1] * f, o[u][v][2] * f, o[u][v][3] * f};
+                    if (c < p.vdim) store4(out + c, w, (p.vdim & 3) == 0, p.vdim - c);
+                }
+                continue;
+            }
             bf16 * out = (bf16 *)p.att + (size_t)tok[u] * p.ld_att + head[u] * p.vdim;
 #pragma unroll
             for (int v = 0; v < VT; ++v) {
@@ -206,8 +226,9 @@ __global__ __launch_bounds__(256, WIDE && KS <= 4 ? 2 : 1) void gqa_attn_kernel(
     for (int w = 0; w < 4; ++w) { const float2 x = wm[w * 16 + r]; f[w] = x.x == -INFINITY ? 0.0f : expf(x.x - mm); sum += f[w] * x.y; }
     float fin = 1.0f;
     if (whole) {
-        const float mf = fmaxf(mm, p.sink), a = mm == -INFINITY ? 0.0f : expf(mm - mf);
-        fin = a / (sum * a + expf(p.sink - mf)) * p.out_scale;
+        const float sink = EXT && p.sinks ? p.sinks[g * per + (first + r) % per] : p.sink;
+        const float mf = fmaxf(mm, sink), a = mm == -INFINITY ? 0.0f : expf(mm - mf);
+        fin = a / (sum * a + expf(sink - mf)) * p.out_scale;
     } else if (cl == 0) ml[(srow0 + r) * p.n_parts + part] = make_float2(mm, sum);
     const int rr = first + r;
     bf16 * out = (bf16 *)p.att + (size_t)(tok0 + rr / per) * p.ld_att + (g * per + rr % per) * p.vdim;
@@ -223,7 +244,9 @@ __global__ __launch_bounds__(256, WIDE && KS <= 4 ? 2 : 1) void gqa_attn_kernel(
         if (whole) {
 #pragma unroll
             for (int k = 0; k < 4; ++k) v[k] *= fin;
-            if (c < p.vdim) store4(out + c, v, quads && c + 4 <= p.vdim, p.vdim - c);
+            if (EXT && p.all_values) {
+                if (c < p.vdim) store4((float *)p.att + (((size_t)(tok0 + rr / per) * p.n_head + g * per + rr % per) * p.n_kv + gv) * p.vdim + c, v, (p.vdim & 3) == 0, p.vdim - c);
+            } else if (c < p.vdim) store4(out + c, v, quads && c + 4 <= p.vdim, p.vdim - c);
         } else {
             *reinterpret_cast<float4 *>(acc + c) = make_float4(v[0], v[1], v[2], v[3]);
         }
@@ -231,8 +254,8 @@ __global__ __launch_bounds__(256, WIDE && KS <= 4 ? 2 : 1) void gqa_attn_kernel(
 }
 
 __global__ __launch_bounds__(256) void gqa_merge_kernel(pi_gqa_attn p) {
-    const int R4 = gqa_rows(p.wide) / 4, wg = blockIdx.x;
-    gqa_merge_row(p, wg / R4 / p.n_kv, wg / R4 % p.n_kv, (wg % R4) * 4 + (threadIdx.x >> 6));
+    const int R4 = gqa_rows(p.wide) / 4, wg = blockIdx.x, n = p.all_values ? p.n_kv * p.n_kv : p.n_kv;
+    gqa_merge_row(p, wg / R4 / n, wg / R4 % n, (wg % R4) * 4 + (threadIdx.x >> 6));
 }
 
 // fp32: one workgroup per (token, head), 64 cells at a time (a wave per cell for the scores, a thread per column for the sum)
@@ -240,14 +263,17 @@ constexpr int kGfCells = 64;
 __global__ __launch_bounds__(256) void gqa_attn_f32_kernel(pi_gqa_attn p) {
     __shared__ float q[kGqaMaxDim], s[kGfCells];
     __shared__ int idx[kGfCells];
-    const int t = blockIdx.x / p.n_head, h = blockIdx.x % p.n_head, g = h / (p.n_head / p.n_kv), tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+    const int vals = p.all_values ? p.n_kv : 1, th = blockIdx.x / vals;
+    const int t = th / p.n_head, h = th % p.n_head, g = h / (p.n_head / p.n_kv), gv = p.all_values ? blockIdx.x % vals : g, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
     const int n = p.n_vis[t];
     const int32_t * list = p.lists + (size_t)p.work[t] * p.list_ld;
     const float * cache = (const float *)p.cache + (size_t)g * 2 * p.hd;
+    const float * values = (const float *)p.cache + (size_t)gv * 2 * p.hd + p.hd;
     const size_t cell_ld = (size_t)p.n_kv * 2 * p.hd;
-    for (int k = tid; k < p.dim; k += 256) q[k] = ((const float *)p.q)[(size_t)blockIdx.x * p.hd + k];
-    const bool sink = p.sink != -INFINITY;
-    float m = p.sink, l = sink ? 1.0f : 0.0f, acc = 0.0f;              // the sink is the soft-max's first entry: weight exp(0), no value
+    for (int k = tid; k < p.dim; k += 256) q[k] = ((const float *)p.q)[(size_t)th * p.hd + k];
+    const float own_sink = p.sinks ? p.sinks[h] : p.sink;
+    const bool sink = own_sink != -INFINITY;
+    float m = own_sink, l = sink ? 1.0f : 0.0f, acc = 0.0f;              // the sink is the soft-max's first entry: weight exp(0), no value
     for (int c0 = first_cell(p, t); c0 < n; c0 += kGfCells) {
         const int nc = min(kGfCells, n - c0);
         __syncthreads();
@@ -258,7 +284,7 @@ __global__ __launch_bounds__(256) void gqa_attn_f32_kernel(pi_gqa_attn p) {
             float d = 0.0f;
             for (int k = lane; k < p.dim; k += 64) d = fmaf(q[k], row[k], d);
             d = pi_wave_sum(d);
-            if (lane == 0) s[c] = d * p.scale;
+            if (lane == 0) s[c] = p.softcap > 0.0f ? p.softcap * tanhf(d * p.scale / p.softcap) : d * p.scale;
         }
         __syncthreads();
         float mn = m;
@@ -269,21 +295,56 @@ __global__ __launch_bounds__(256) void gqa_attn_f32_kernel(pi_gqa_attn p) {
         for (int c = 0; c < nc; ++c) {
             const float w = expf(s[c] - mn);
             l += w;
-            if (tid < p.vdim) acc = fmaf(w, cache[idx[c] * cell_ld + p.hd + tid], acc);
+            if (tid < p.vdim) acc = fmaf(w, values[idx[c] * cell_ld + tid], acc);
         }
         m = mn;
     }
-    if (tid < p.vdim) ((float *)p.att)[(size_t)t * p.ld_att + h * p.vdim + tid] = acc / l * p.out_scale;
+    if (tid < p.vdim) ((float *)p.att)[p.all_values ? (size_t)blockIdx.x * p.vdim + tid : (size_t)t * p.ld_att + h * p.vdim + tid] = acc / l * p.out_scale;
+}
+
+// heads mixed behind an attention with all_values: a thread per value of a key / value head, its query heads eight at a time
+template <typename ST>
+__global__ __launch_bounds__(256) void gqa_mix_kernel(pi_gqa_mix p) {
+    extern __shared__ __align__(16) float talk[];
+    const int t = blockIdx.x, per = p.n_head / p.n_kv, n = p.n_kv * p.vdim;
+    if (p.talk) {
+        for (int i = threadIdx.x; i < p.n_head * p.n_head; i += 256) talk[i] = p.talk[i];
+        __syncthreads();
+    }
+    const int e = blockIdx.y * 256 + threadIdx.x;
+    if (e >= n) return;
+    const int kv = e / p.vdim, c = e % p.vdim;
+    const float * a = p.a + (size_t)t * p.n_head * n + e;
+    const float * gate = p.off_gate >= 0 ? p.z + (size_t)t * p.ldz + p.off_gate : nullptr;
+    ST * out = (ST *)p.att + (size_t)t * p.ld_att;
+    for (int h0 = 0; h0 < per; h0 += 8) {
+        float s[8] = {0, 0, 0, 0, 0, 0, 0, 0};
+        if (p.talk) {
+            for (int g = 0; g < p.n_head; ++g) {
+                const float v = a[(size_t)g * n];
+#pragma unroll
+                for (int k = 0; k < 8; ++k) s[k] = fmaf(talk[(kv * per + min(h0 + k, per - 1)) * p.n_head + g], v, s[k]);
+            }
+        } else {
+#pragma unroll
+            for (int k = 0; k < 8; ++k) s[k] = a[(size_t)(kv * per + min(h0 + k, per - 1)) * n];
+        }
+#pragma unroll
+        for (int k = 0; k < 8; ++k) {
+            const int h = kv * per + h0 + k;
+            if (h0 + k < per) out[h * p.vdim + c] = to_st<ST>(gate ? s[k] * sigmoid_f32(gate[h]) : s[k]);
+        }
+    }
 }
 
 template <typename ST>
-__global__ void gqa_shift_kernel(ST * __restrict__ cache, int n_kv, int hd, int rot_dim, double base, int pairs, const int32_t * __restrict__ delta) {
+__global__ void gqa_shift_kernel(ST * __restrict__ cache, int n_kv, int hd, int rot_dim, double base, const double * __restrict__ freq, int pairs, const int32_t * __restrict__ delta) {
     const int c = blockIdx.x, d = delta[c], half = rot_dim / 2;
     if (d == 0) return;
     for (int e = threadIdx.x; e < n_kv * half; e += blockDim.x) {
         const int g = e / half, i = e % half;
         double sn, cn;
-        sincos((double)d * pow(base, -2.0 * (double)i / (double)rot_dim), &sn, &cn);
+        sincos((double)d * (freq ? freq[i] : pow(base, -2.0 * (double)i / (double)rot_dim)), &sn, &cn);
         ST * r = cache + ((size_t)c * n_kv + g) * 2 * hd + (pairs ? 2 * i : i), * o = r + (pairs ? 1 : half);
         const float u = from_st(*r), v = from_st(*o);
         *r = to_st<ST>(u * (float)cn - v * (float)sn);
@@ -291,22 +352,25 @@ __global__ void gqa_shift_kernel(ST * __restrict__ cache, int n_kv, int hd, int 
     }
 }
 
-template <int KS, bool WIDE> int launch_gqa(const pi_gqa_attn * p, hipStream_t st) {
+template <int KS, bool WIDE, bool EXT> int launch_gqa_as(const pi_gqa_attn * p, hipStream_t st) {
     constexpr size_t tile = gqa_lds<KS, WIDE>(), merge = WIDE ? 0 : sizeof(float) * (4 * 16 * (KS * 32 + 4) + 2 * 4 * 16), lds = tile > merge ? tile : merge;
     static bool raised = false;
     if (!raised && lds > 64 * 1024) {
-        PI_HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void *>(&gqa_attn_kernel<KS, WIDE>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
+        PI_HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void *>(&gqa_attn_kernel<KS, WIDE, EXT>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
         raised = true;
     }
-    hipLaunchKernelGGL((gqa_attn_kernel<KS, WIDE>), dim3(p->n_work * p->n_kv, p->n_parts), dim3(256), lds, st, *p);
+    hipLaunchKernelGGL((gqa_attn_kernel<KS, WIDE, EXT>), dim3(p->n_work * p->n_kv * (p->all_values ? p->n_kv : 1), p->n_parts), dim3(256), lds, st, *p);
     return pi::check_launch("pi_k_gqa_attn");
+}
+template <int KS, bool WIDE> int launch_gqa(const pi_gqa_attn * p, hipStream_t st) {
+    return p->softcap > 0.0f || p->sinks || p->all_values ? launch_gqa_as<KS, WIDE, true>(p, st) : launch_gqa_as<KS, WIDE, false>(p, st);
 }
 
 int gqa_check(int type, const pi_gqa_attn * p) {
     if (!p || !p->q || !p->cache || !p->lists || !p->work || !p->n_vis || !p->att || p->T <= 0 || p->n_head <= 0 || p->n_kv <= 0 || p->n_head % p->n_kv || p->dim <= 0 || p->vdim <= 0 ||
-        p->hd < p->dim || p->hd < p->vdim || p->ld_att < p->n_head * p->vdim || p->hd != pi_k_gqa_head_ld(type, p->dim, p->vdim) || p->n_parts <= 0 || p->window < 0)
+        p->hd < p->dim || p->hd < p->vdim || (!p->all_values && p->ld_att < p->n_head * p->vdim) || p->hd != pi_k_gqa_head_ld(type, p->dim, p->vdim) || p->n_parts <= 0 || p->window < 0)
         return pi::fail(PI_E_ARG, "pi_k_gqa_attn: bad arguments");
-    if (type == PI_TYPE_BF16 && (p->n_work <= 0 || (long long)p->n_work * p->n_kv > (1 << 30) || p->n_parts > 64 || (p->n_parts > 1 && !p->scratch)))
+    if (type == PI_TYPE_BF16 && (p->n_work <= 0 || (long long)p->n_work * p->n_kv * (p->all_values ? p->n_kv : 1) > (1 << 30) || p->n_parts > 64 || (p->n_parts > 1 && !p->scratch)))
         return pi::fail(PI_E_ARG, "pi_k_gqa_attn: bad work arguments");
     return PI_OK;
 }
@@ -361,23 +425,45 @@ int pi_k_gqa_attn(int type, const pi_gqa_attn * p, pi_stream_t stream) {
     if (type == PI_TYPE_F32) {
         const int rc = gqa_check(type, p);
         if (rc != PI_OK) return rc;
-        hipLaunchKernelGGL(gqa_attn_f32_kernel, dim3(p->T * p->n_head), dim3(256), 0, (hipStream_t)stream, *p);
+        hipLaunchKernelGGL(gqa_attn_f32_kernel, dim3(p->T * p->n_head * (p->all_values ? p->n_kv : 1)), dim3(256), 0, (hipStream_t)stream, *p);
         return pi::check_launch("pi_k_gqa_attn");
     }
     if (type != PI_TYPE_BF16) return pi::fail(PI_E_UNSUPPORTED, "pi_k_gqa_attn: type");
     const int rc = pi_k_gqa_attn_parts(p, stream);
     if (rc != PI_OK || p->n_parts == 1) return rc;
-    hipLaunchKernelGGL(gqa_merge_kernel, dim3(p->n_work * p->n_kv * (gqa_rows(p->wide) / 4)), dim3(256), 0, (hipStream_t)stream, *p);
+    hipLaunchKernelGGL(gqa_merge_kernel, dim3(p->n_work * p->n_kv * (p->all_values ? p->n_kv : 1) * (gqa_rows(p->wide) / 4)), dim3(256), 0, (hipStream_t)stream, *p);
     return pi::check_launch("pi_k_gqa_attn merge");
 }
 
-int pi_k_gqa_shift(int type, void * cache, int n_cells, int n_kv, int hd, int rot_dim, double base, int pairs, const int32_t * delta, pi_stream_t stream) {
+int pi_k_gqa_mix(int type, const pi_gqa_mix * p, pi_stream_t stream) {
+    if (!p || !p->a || !p->att || p->T <= 0 || p->n_head <= 0 || p->n_kv <= 0 || p->n_head % p->n_kv || p->vdim <= 0 || p->ld_att < p->n_head * p->vdim ||
+        (p->off_gate >= 0 && (!p->z || p->off_gate + p->n_head > p->ldz)))
+        return pi::fail(PI_E_ARG, "pi_k_gqa_mix: bad arguments");
+    const size_t lds = p->talk ? sizeof(float) * p->n_head * p->n_head : 0;
+    const dim3 grid(p->T, (p->n_kv * p->vdim + 255) / 256);
+    if (lds > 64 * 1024 || grid.y > 65535) return pi::fail(PI_E_UNSUPPORTED, "pi_k_gqa_mix: up to 128 heads");
+    if (type == PI_TYPE_BF16) hipLaunchKernelGGL(gqa_mix_kernel<bf16>, grid, dim3(256), lds, (hipStream_t)stream, *p);
+    else if (type == PI_TYPE_F32) hipLaunchKernelGGL(gqa_mix_kernel<float>, grid, dim3(256), lds, (hipStream_t)stream, *p);
+    else return pi::fail(PI_E_UNSUPPORTED, "pi_k_gqa_mix: type");
+    return pi::check_launch("pi_k_gqa_mix");
+}
+
+static int gqa_shift(int type, void * cache, int n_cells, int n_kv, int hd, int rot_dim, double base, const double * freq, int pairs, const int32_t * delta, pi_stream_t stream) {
     if (!cache || !delta || n_cells <= 0 || n_kv <= 0 || hd <= 0 || rot_dim < 0 || rot_dim % 2 || rot_dim > hd) return pi::fail(PI_E_ARG, "pi_k_gqa_shift: bad arguments");
     if (rot_dim == 0) return PI_OK;
-    if (type == PI_TYPE_BF16) hipLaunchKernelGGL(gqa_shift_kernel<bf16>, dim3(n_cells), dim3(64), 0, (hipStream_t)stream, (bf16 *)cache, n_kv, hd, rot_dim, base, pairs, delta);
-    else if (type == PI_TYPE_F32) hipLaunchKernelGGL(gqa_shift_kernel<float>, dim3(n_cells), dim3(64), 0, (hipStream_t)stream, (float *)cache, n_kv, hd, rot_dim, base, pairs, delta);
+    if (type == PI_TYPE_BF16) hipLaunchKernelGGL(gqa_shift_kernel<bf16>, dim3(n_cells), dim3(64), 0, (hipStream_t)stream, (bf16 *)cache, n_kv, hd, rot_dim, base, freq, pairs, delta);
+    else if (type == PI_TYPE_F32) hipLaunchKernelGGL(gqa_shift_kernel<float>, dim3(n_cells), dim3(64), 0, (hipStream_t)stream, (float *)cache, n_kv, hd, rot_dim, base, freq, pairs, delta);
     else return pi::fail(PI_E_UNSUPPORTED, "pi_k_gqa_shift: type");
     return pi::check_launch("pi_k_gqa_shift");
+}
+
+int pi_k_gqa_shift(int type, void * cache, int n_cells, int n_kv, int hd, int rot_dim, double base, int pairs, const int32_t * delta, pi_stream_t stream) {
+    return gqa_shift(type, cache, n_cells, n_kv, hd, rot_dim, base, nullptr, pairs, delta, stream);
+}
+
+int pi_k_gqa_shift_table(int type, void * cache, int n_cells, int n_kv, int hd, int rot_dim, const double * freq, int pairs, const int32_t * delta, pi_stream_t stream) {
+    if (!freq) return pi::fail(PI_E_ARG, "pi_k_gqa_shift_table: bad arguments");
+    return gqa_shift(type, cache, n_cells, n_kv, hd, rot_dim, 1.0, freq, pairs, delta, stream);
 }
 
 }  // extern "C"

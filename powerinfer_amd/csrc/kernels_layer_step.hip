@@ -219,9 +219,10 @@ __device__ int step_experts(StepExperts & s, int * first, const int32_t * __rest
 
 // ---------------------------------------------------------------------------------------------------------------------------------
 // first matrices of the step's experts: workgroup (row tile, pair) works for the pair's expert if no earlier pair has the same one, for
-// every token that chose it; act[pair] = weight * relu(z)^2, or (glu: rows of gate and up in turn, ff of both together) weight * clamped GLU
+// every token that chose it; act[pair] = weight * relu(z)^2, or (glu: rows of gate and up in turn, ff of both together) weight * clamped GLU (weigh_input:
+// the clamped GLU of the weighted rows)
 // ---------------------------------------------------------------------------------------------------------------------------------
-struct ExpertUp { const bf16 * up; int ff, cols; const bf16 * x_ol; const int32_t * ids; const float * weights; int T, top; bf16 * act; int ld_act; int glu = 0; float limit = 0.0f, gain = 0.0f; };
+struct ExpertUp { const bf16 * up; int ff, cols; const bf16 * x_ol; const int32_t * ids; const float * weights; int T, top; bf16 * act; int ld_act; int glu = 0; float limit = 0.0f, gain = 0.0f, one = 1.0f; int weigh_input = 0; };
 constexpr int kUpLds = 4 * 16 * kWsStride;
 __device__ void expert_up(const ExpertUp & a, int tile, int p, unsigned char * smem) {
     constexpr int NW = 4;
@@ -262,9 +263,12 @@ __device__ void expert_up(const ExpertUp & a, int tile, int p, unsigned char * s
         float g = 0.0f, u = 0.0f;
 #pragma unroll
         for (int w = 0; w < NW; ++w) { g += reinterpret_cast<float (*)[17]>(tiles[w])[rr][t]; u += reinterpret_cast<float (*)[17]>(tiles[w])[rr + 1][t]; }
-        const float y = clamped_glu(g, u, a.limit, a.gain);
-        for (int k = 0; k < top; ++k)
-            if (ids[t * top + k] == e) a.act[(size_t)(t * top + k) * a.ld_act + row / 2] = (bf16)(a.weights[t * top + k] * y);
+        for (int k = 0; k < top; ++k) {
+            if (ids[t * top + k] != e) continue;
+            const float w = a.weights[t * top + k];
+            const float y = a.weigh_input ? clamped_glu(w * g, w * u, a.limit, a.gain, a.one) : w * clamped_glu(g, u, a.limit, a.gain, a.one);
+            a.act[(size_t)(t * top + k) * a.ld_act + row / 2] = (bf16)y;
+        }
         return;
     }
     float v = 0.0f;
@@ -293,7 +297,8 @@ __global__ __launch_bounds__(256) void mix_and_up_kernel(pi_gqa_attn p, pi_gate_
     b -= n_gate;
     if (b < n_merge) {
         const int r4 = gqa_rows(p.wide) / 4;
-        gqa_merge_row(p, b / r4 / p.n_kv, b / r4 % p.n_kv, (b % r4) * 4 + (threadIdx.x >> 6));
+        const int n = p.all_values ? p.n_kv * p.n_kv : p.n_kv;
+        gqa_merge_row(p, b / r4 / n, b / r4 % n, (b % r4) * 4 + (threadIdx.x >> 6));
         return;
     }
     expert_up(u, (b - n_merge) % n_up_tiles, (b - n_merge) / n_up_tiles, smem);
@@ -313,7 +318,7 @@ __global__ __launch_bounds__(64 * NW) void layer_out_step_kernel(pi_layer_out a)
     static_assert(NW < 8 || sizeof(tiles) + sizeof(se) + sizeof(first) > 80 * 1024, "one workgroup per compute unit");
     const int tid = threadIdx.x, wave = tid >> 6;
     const WaveStream ws(tiles[wave]);
-    const int row0 = blockIdx.x * 16, n_o = (a.ld_att + 255) / 256, n_e = a.ids ? (a.ld_act + 255) / 256 : 1;
+    const int row0 = blockIdx.x * 16, n_o = a.wo ? (a.ld_att + 255) / 256 : 0, n_e = a.ids ? (a.ld_act + 255) / 256 : 1;
     const int tok = min(ws.i, a.T - 1);
     const bf16 * wo = (const bf16 *)a.wo, * down = (const bf16 *)a.down;
     pi_u32x4 ld[2][8];
@@ -357,7 +362,7 @@ __global__ __launch_bounds__(64 * NW) void layer_out_step_kernel(pi_layer_out a)
 #pragma unroll
     for (int w = 0; w < NW; ++w) v += reinterpret_cast<float (*)[17]>(tiles[w])[tid & 15][t];
     if (a.gate_z) v *= sigmoid_f32(a.gate_z[(size_t)t * a.ld_gate + a.off_gate + row] + a.gate_b[row]);
-    const float x = a.x[(size_t)t * a.rows + row];
+    const float x = a.x ? a.x[(size_t)t * a.rows + row] : 0.0f;
     v += a.scaled ? a.alpha * x : x;
     a.out[(size_t)t * a.rows + row] = v;
     if (a.keep) a.keep[(size_t)t * a.rows + row] = v;
@@ -410,7 +415,7 @@ int pi_k_mix_up_step(const pi_gqa_attn * attn, const pi_gate_norm * gate, const 
         return pi::fail(PI_E_ARG, "pi_k_mix_up_step: bad arguments");
     if (ids && (!up || !x_ol || !weights || !act || n_expert <= 0 || ff <= 0 || cols <= 0 || cols % 32 || top <= 0 || T * top > kStepPairs || ld_act < ff))
         return pi::fail(PI_E_ARG, "pi_k_mix_up_step: bad expert arguments");
-    const int n_merge = attn ? p.n_work * p.n_kv * (gqa_rows(p.wide) / 4) : 0, n_gate = gate ? gate_norm_blocks(g) : 0, n_up_tiles = ids ? (2 * ff + 15) / 16 : 1, n_up = ids ? n_up_tiles * T * top : 0;
+    const int n_merge = attn ? p.n_work * p.n_kv * (p.all_values ? p.n_kv : 1) * (gqa_rows(p.wide) / 4) : 0, n_gate = gate ? gate_norm_blocks(g) : 0, n_up_tiles = ids ? (2 * ff + 15) / 16 : 1, n_up = ids ? n_up_tiles * T * top : 0;
     if (n_merge + n_gate + n_up == 0) return PI_OK;
     ExpertUp u{(const bf16 *)up, 2 * ff, cols, (const bf16 *)x_ol, ids, weights, T, top, (bf16 *)act, ld_act};
     u.glu = 1; u.limit = limit; u.gain = gain;
@@ -418,8 +423,19 @@ int pi_k_mix_up_step(const pi_gqa_attn * attn, const pi_gate_norm * gate, const 
     return pi::check_launch("pi_k_mix_up_step");
 }
 
+int pi_k_expert_up_step(const void * up, int n_expert, int ff, int cols, float limit, float gain, int plain_up, int weigh_input, const void * x_ol, int T, const int32_t * ids,
+                        const float * weights, int top, void * act, int ld_act, pi_stream_t stream) {
+    if (!up || !x_ol || !ids || !weights || !act || T <= 0 || T > kBtMaxT || n_expert <= 0 || ff <= 0 || cols <= 0 || cols % 32 || top <= 0 || T * top > kStepPairs || ld_act < ff)
+        return pi::fail(PI_E_ARG, "pi_k_expert_up_step: bad arguments");
+    ExpertUp u{(const bf16 *)up, 2 * ff, cols, (const bf16 *)x_ol, ids, weights, T, top, (bf16 *)act, ld_act};
+    u.glu = 1; u.limit = limit; u.gain = gain; u.one = plain_up ? 0.0f : 1.0f; u.weigh_input = weigh_input;
+    const int tiles = (2 * ff + 15) / 16;
+    hipLaunchKernelGGL(mix_and_up_kernel, dim3(tiles * T * top), dim3(256), kUpLds, (hipStream_t)stream, pi_gqa_attn{}, pi_gate_norm{}, 0, 0, u, tiles);
+    return pi::check_launch("pi_k_expert_up_step");
+}
+
 int pi_k_layer_out_step(const pi_layer_out * a, pi_stream_t stream) {
-    if (!a || !a->x || !a->wo || !a->att || !a->out || (a->gate_z && (!a->gate_b || a->off_gate < 0 || a->off_gate + a->rows > a->ld_gate)) || a->rows <= 0 || a->T <= 0 || a->T > kBtMaxT || a->ld_att <= 0 || a->ld_att % 32 ||
+    if (!a || (a->wo ? !a->att || a->ld_att <= 0 || a->ld_att % 32 : !a->ids) || !a->out || (a->gate_z && (!a->gate_b || a->off_gate < 0 || a->off_gate + a->rows > a->ld_gate)) || a->rows <= 0 || a->T <= 0 || a->T > kBtMaxT ||
         (a->ids && (!a->down || !a->act || a->ld_act <= 0 || a->ld_act % 32 || a->top <= 0 || a->T * a->top > kStepPairs || a->n_expert <= 0 || a->n_expert > kStepExperts)))
         return pi::fail(PI_E_ARG, "pi_k_layer_out_step: bad arguments");
     // eight waves a workgroup when every workgroup has a compute unit to itself, four (and several workgroups a unit) beyond

@@ -278,13 +278,14 @@ __global__ __launch_bounds__(256) void group_gemm_kernel(pi_group_gemm g) {
     for (int u = 0; u < 2; ++u) {
         const int t = t0 + u * 16 + i;
         if (t >= n) continue;
+        const float alpha = g.pair_w ? g.alpha * g.pair_w[g.gather[lo + t]] : g.alpha, one = g.glu_plain_up ? 0.0f : 1.0f;
         const size_t yr = g.off ? (size_t)(lo + t) * g.ldy : (size_t)grp * g.y_gs + (size_t)t * g.ldy;
         if (g.glu) {                                   // rows in (gate, up) pairs: a lane holds two of them
 #pragma unroll
             for (int r = 0; r < 4; r += 2) {
                 const int row = row0 + 4 * q + r;
                 if (row >= g.rows) continue;
-                const float v = clamped_glu(acc[u][r] * g.alpha, acc[u][r + 1] * g.alpha, g.glu_limit, g.glu_gain);
+                const float v = clamped_glu(acc[u][r] * alpha, acc[u][r + 1] * alpha, g.glu_limit, g.glu_gain, one);
                 if (g.y_f32) ((float *)g.y)[yr + row / 2] = v;
                 else ((ST *)g.y)[yr + row / 2] = to_st<ST>(v);
             }
@@ -294,7 +295,7 @@ __global__ __launch_bounds__(256) void group_gemm_kernel(pi_group_gemm g) {
         for (int r = 0; r < 4; ++r) {
             const int row = row0 + 4 * q + r;
             if (row >= g.rows) continue;
-            float v = acc[u][r] * g.alpha;
+            float v = acc[u][r] * alpha;
             if (g.relu2) { v = fmaxf(v, 0.0f); v *= v; }
             if (g.y_f32) ((float *)g.y)[yr + row] = v;
             else ((ST *)g.y)[yr + row] = to_st<ST>(v);
@@ -312,6 +313,14 @@ __global__ void rope_angles_kernel(const int32_t * __restrict__ pos, int T, int 
     double s, c;
     sincos((double)pos[t] * pow(base, -2.0 * (double)i / (double)dims), &s, &c);
     cs[idx] = make_float2((float)c, (float)s);
+}
+
+__global__ void rope_table_kernel(const int32_t * __restrict__ pos, int T, int half, const double * __restrict__ freq, double length, float2 * __restrict__ cs) {
+    const int idx = blockIdx.x * blockDim.x + threadIdx.x;
+    if (idx >= T * half) return;
+    double s, c;
+    sincos((double)pos[idx / half] * freq[idx % half], &s, &c);
+    cs[idx] = make_float2((float)(length * c), (float)(length * s));
 }
 
 // expert choice, one workgroup per token
@@ -398,10 +407,11 @@ __global__ __launch_bounds__(64 * WGM * WGN, (WGM * WGN > 4 ? 1 : BM + BN <= 192
         for (int nn = 0; nn < NT; ++nn) {
             const int row = row0 + wm * WM + m * 16 + 4 * q, tok = wn * WN + nn * 16 + i;
             if (tok >= n || row >= g.rows) continue;
+            const float alpha = g.pair_w ? g.alpha * g.pair_w[g.gather[lo + tok]] : g.alpha;
             if (g.glu) {                               // rows in (gate, up) pairs: a lane holds two of them
                 const size_t o = (g.off ? 0 : (size_t)grp * g.y_gs) + (size_t)(lo + tok) * g.ldy + row / 2;
-                const float a = clamped_glu(acc[m][nn][0] * g.alpha, acc[m][nn][1] * g.alpha, g.glu_limit, g.glu_gain);
-                const float b = clamped_glu(acc[m][nn][2] * g.alpha, acc[m][nn][3] * g.alpha, g.glu_limit, g.glu_gain);
+                const float one = g.glu_plain_up ? 0.0f : 1.0f, a = clamped_glu(acc[m][nn][0] * alpha, acc[m][nn][1] * alpha, g.glu_limit, g.glu_gain, one);
+                const float b = clamped_glu(acc[m][nn][2] * alpha, acc[m][nn][3] * alpha, g.glu_limit, g.glu_gain, one);
                 const bool two = row + 4 <= g.rows;
                 if (g.y_f32) {
                     ((float *)g.y)[o] = a;
@@ -419,7 +429,7 @@ __global__ __launch_bounds__(64 * WGM * WGN, (WGM * WGN > 4 ? 1 : BM + BN <= 192
             float v[4];
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
-                v[r] = acc[m][nn][r] * g.alpha;
+                v[r] = acc[m][nn][r] * alpha;
                 if (g.relu2) { v[r] = fmaxf(v[r], 0.0f); v[r] *= v[r]; }
             }
             const bool quad = row + 4 <= g.rows && (o & 3) == 0;
@@ -578,7 +588,7 @@ int pi_k_norm_pair(int type, const float * x, const int32_t * rows, int T, int c
 
 int pi_k_group_gemm(int type, const pi_group_gemm * g, pi_stream_t stream) {
     if (!g || !g->W || !g->x || !g->y || g->rows <= 0 || g->cols <= 0 || g->cols % 32 || g->ldw < g->cols || g->ldw % 8 || g->ldx < g->cols || g->ldx % 8 ||
-        g->ldy < (g->glu ? g->rows / 2 : g->rows) || (g->glu && (g->rows % 2 || g->relu2)) || g->T <= 0 || g->n_group <= 0 || g->n_group > 65535 || (g->gather && g->gather_div <= 0) || g->w_gs % 8 || g->x_gs % 8)
+        g->ldy < (g->glu ? g->rows / 2 : g->rows) || (g->glu && (g->rows % 2 || g->relu2)) || g->T <= 0 || g->n_group <= 0 || g->n_group > 65535 || (g->gather && g->gather_div <= 0) || (g->pair_w && (!g->gather || !g->off)) || g->w_gs % 8 || g->x_gs % 8)
         return pi::fail(PI_E_ARG, "pi_k_group_gemm: bad arguments");
     const dim3 grid((g->rows + 63) / 64, (g->T + 31) / 32, g->n_group);
     if (grid.y > 65535) return pi::fail(PI_E_ARG, "pi_k_group_gemm: too many tokens");
@@ -592,6 +602,20 @@ int pi_k_rope_angles(const int32_t * pos, int T, int dims, double base, void * c
     if (!pos || !cs || T <= 0 || dims <= 0 || dims % 2 || !(base > 0.0)) return pi::fail(PI_E_ARG, "pi_k_rope_angles: bad arguments");
     hipLaunchKernelGGL(rope_angles_kernel, dim3((T * (dims / 2) + 63) / 64), dim3(64), 0, (hipStream_t)stream, pos, T, dims, base, (float2 *)cs);
     return pi::check_launch("pi_k_rope_angles");
+}
+
+int pi_k_rope_angles_table(const int32_t * pos, int T, int dims, const double * freq, double length, void * cs, pi_stream_t stream) {
+    if (!pos || !cs || !freq || T <= 0 || dims <= 0 || dims % 2) return pi::fail(PI_E_ARG, "pi_k_rope_angles_table: bad arguments");
+    hipLaunchKernelGGL(rope_table_kernel, dim3((T * (dims / 2) + 63) / 64), dim3(64), 0, (hipStream_t)stream, pos, T, dims / 2, freq, length, (float2 *)cs);
+    return pi::check_launch("pi_k_rope_angles_table");
+}
+
+int pi_k_route_scores(const float * z, int T, int n_expert, int n_top, int32_t * ids, float * weights, pi_stream_t stream) {
+    if (!z || !ids || !weights || T <= 0 || n_expert <= 0 || n_expert > 4096 || n_top <= 0 || n_top > n_expert) return pi::fail(PI_E_ARG, "pi_k_route_scores: bad arguments");
+    RouteArgs r{z, n_expert, n_top, 1, 1, nullptr, ids, weights};
+    r.raw = true;
+    hipLaunchKernelGGL(route_kernel, dim3(T), dim3(n_expert > 128 ? 256 : n_expert > 64 ? 128 : 64), route_lds_bytes(n_expert, 1, n_top), (hipStream_t)stream, r);
+    return pi::check_launch("pi_k_route_scores");
 }
 
 int pi_k_route(const float * z, int T, int n_expert, int n_top, int n_group, int n_keep, const float * bias, int32_t * ids, float * weights, pi_stream_t stream) {
@@ -611,7 +635,7 @@ int pi_k_moe_sort(const int32_t * ids, int n_pairs, int n_expert, int32_t * off,
 
 int pi_k_group_gemm_tile(const pi_group_gemm * g, int tile_n, pi_stream_t stream) {
     if (!g || !g->W || !g->x || !g->y || g->rows <= 0 || g->cols <= 0 || g->cols % kGtBK || g->ldw < g->cols || g->ldw % 8 || g->ldx < g->cols || g->ldx % 8 ||
-        g->ldy < (g->glu ? g->rows / 2 : g->rows) || (g->glu && (g->rows % 2 || g->relu2)) || g->T <= 0 || g->n_group <= 0 || (g->gather && g->gather_div <= 0) || g->w_gs % 8 || g->x_gs % 8 || (g->off && (!g->tiles || !g->n_tiles || g->max_tiles <= 0)))
+        g->ldy < (g->glu ? g->rows / 2 : g->rows) || (g->glu && (g->rows % 2 || g->relu2)) || g->T <= 0 || g->n_group <= 0 || (g->gather && g->gather_div <= 0) || (g->pair_w && (!g->gather || !g->off)) || g->w_gs % 8 || g->x_gs % 8 || (g->off && (!g->tiles || !g->n_tiles || g->max_tiles <= 0)))
         return pi::fail(PI_E_ARG, "pi_k_group_gemm_tile: bad arguments");
     if ((((uintptr_t)g->W | (uintptr_t)g->x | (uintptr_t)g->y) & 15) != 0) return pi::fail(PI_E_ARG, "pi_k_group_gemm_tile: operands must be 16-byte aligned");
     hipStream_t st = (hipStream_t)stream;

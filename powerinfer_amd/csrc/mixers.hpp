@@ -60,6 +60,12 @@ template <typename ST> __device__ void front_block(const pi_ffn_front & f, const
 // ---- grouped-query attention, behind the joint projection: a wave per head (four heads a block) - norm, rotation, division by the root
 // mean square, query row or cell --------------------------------------------------------------------------------------------------------
 constexpr int kGqaMaxDim = 256;
+// value e of a token's heads: kept for the layers behind, or mixed with the one an earlier layer kept
+__device__ __forceinline__ float mixed_value(const pi_gqa_prep & p, float v, int t, int e) {
+    if (p.v_keep) p.v_keep[(size_t)t * p.ld_first + e] = v;
+    if (p.v_first) { const float l = p.v_mix[0]; v = (1.0f - l) * v + l * p.v_first[(size_t)t * p.ld_first + e]; }
+    return v;
+}
 template <typename ST, bool NORM> __device__ void gqa_prep_heads(const pi_gqa_prep & p, int t, int b) {      // NORM: q_norm and k_norm are given
     const int head = b * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63, half = p.rot_dim / 2;
     if (head >= p.n_head + p.n_kv) return;
@@ -108,7 +114,7 @@ template <typename ST, bool NORM> __device__ void gqa_prep_heads(const pi_gqa_pr
         const float * v = z + p.off_v + g * p.vdim;
         float sv = 1.0f;
 #pragma unroll
-        for (int j = 0; j < J; ++j) x[j] = v[min(lane + 64 * j, p.vdim - 1)];
+        for (int j = 0; j < J; ++j) x[j] = mixed_value(p, v[min(lane + 64 * j, p.vdim - 1)], t, g * p.vdim + min(lane + 64 * j, p.vdim - 1));
         ss = 0.0f;
 #pragma unroll
         for (int j = 0; j < J; ++j) { if (lane + 64 * j >= p.vdim) x[j] = 0.0f; ss = fmaf(x[j], x[j], ss); }
@@ -178,6 +184,14 @@ template <typename ST, int N, bool EVEN> __device__ void gqa_prep_pairs(const pi
             if (e < p.hd) store(row + e, a * r.x - o * r.y, o * r.x + a * r.y);
         }
         if (!key) continue;
+        if (p.v_keep || p.v_first) {
+#pragma unroll
+            for (int j = 0; j < J; ++j) {
+                const int e = 2 * (lane + 64 * j);
+                if (e < p.vdim) v[n][j].x = mixed_value(p, v[n][j].x, t, g * p.vdim + e);
+                if (e + 1 < p.vdim) v[n][j].y = mixed_value(p, v[n][j].y, t, g * p.vdim + e + 1);
+            }
+        }
         float sv = 0.0f;
 #pragma unroll
         for (int j = 0; j < J; ++j) {
@@ -208,25 +222,28 @@ template <typename ST, bool PAIRS> __device__ void gqa_prep_block(const pi_gqa_p
 inline bool gqa_prep_ok(int type, const pi_gqa_prep & p) {
     return p.z && p.cs && p.q && p.cache && p.cell && p.T > 0 && p.n_head > 0 && p.n_kv > 0 && p.n_head % p.n_kv == 0 && p.rot_dim >= 0 && p.rot_dim % 2 == 0 && p.rot_dim <= p.dim &&
            p.hd == pi_k_gqa_head_ld(type, p.dim, p.vdim) && p.hd > 0 && p.off_k >= p.n_head * p.dim && p.off_k + p.n_kv * p.dim <= p.ldz && p.off_v >= 0 &&
-           p.off_v + p.n_kv * p.vdim <= p.ldz && !p.q_norm == !p.k_norm && !(p.q_norm && p.unit);
+           p.off_v + p.n_kv * p.vdim <= p.ldz && !p.q_norm == !p.k_norm && !(p.q_norm && p.unit) && (!(p.v_first || p.v_keep) || p.ld_first >= p.n_kv * p.vdim) && (!p.v_first || p.v_mix);
 }
 
 // ---- grouped-query attention: the parts of one row of a work item, by one wave (fixed order, the sink in the denominator) -------------
 __host__ __device__ inline int gqa_rows(int wide) { return wide ? 128 : 16; }
-__device__ void gqa_merge_row(const pi_gqa_attn & p, int item_index, int g, int r) {
+// vg: the group, or (all_values) the pair of a group and whose values its rows met
+__device__ void gqa_merge_row(const pi_gqa_attn & p, int item_index, int vg, int r) {
+    const int n_groups = p.all_values ? p.n_kv * p.n_kv : p.n_kv, g = p.all_values ? vg / p.n_kv : vg;
     const int lane = threadIdx.x & 63, per = p.n_head / p.n_kv, R = gqa_rows(p.wide);
     const int4 item = reinterpret_cast<const int4 *>(p.work)[item_index];
     if (r >= item.z) return;
-    const size_t srow = ((size_t)item_index * p.n_kv + g) * R + r;
+    const size_t srow = ((size_t)item_index * n_groups + vg) * R + r;
     const float * acc = p.scratch + srow * p.n_parts * p.hd;
-    const float2 ml = lane < p.n_parts ? reinterpret_cast<const float2 *>(p.scratch + (size_t)p.n_work * p.n_kv * R * p.n_parts * p.hd)[srow * p.n_parts + lane]
+    const float2 ml = lane < p.n_parts ? reinterpret_cast<const float2 *>(p.scratch + (size_t)p.n_work * n_groups * R * p.n_parts * p.hd)[srow * p.n_parts + lane]
                                        : make_float2(-INFINITY, 0.0f);
-    const float m = fmaxf(pi_wave_max(ml.x), p.sink);
-    const float e = ml.x == -INFINITY ? 0.0f : expf(ml.x - m);
-    const float l = pi_wave_sum(e * ml.y) + expf(p.sink - m);
-    const float f = e / l * p.out_scale;
     const int rr = item.y + r, head = g * per + rr % per;
+    const float sink = p.sinks ? p.sinks[head] : p.sink, m = fmaxf(pi_wave_max(ml.x), sink);
+    const float e = ml.x == -INFINITY ? 0.0f : expf(ml.x - m);
+    const float l = pi_wave_sum(e * ml.y) + expf(sink - m);
+    const float f = e / l * p.out_scale;
     bf16 * out = (bf16 *)p.att + (size_t)(item.x + rr / per) * p.ld_att + head * p.vdim;
+    float * all = p.all_values ? (float *)p.att + (((size_t)(item.x + rr / per) * p.n_head + head) * p.n_kv + vg % p.n_kv) * p.vdim : nullptr;
     for (int c0 = 0; c0 < p.vdim; c0 += 64) {            // (every lane stays in the loop: the factors are passed between lanes)
         const int c = min(c0 + lane, p.hd - 1);
         float v = 0.0f;
@@ -240,7 +257,7 @@ __device__ void gqa_merge_row(const pi_gqa_attn & p, int item_index, int g, int 
                 if (s0 + u < p.n_parts) v = fmaf(w, a[u], v);
             }
         }
-        if (c0 + lane < p.vdim) out[c0 + lane] = (bf16)v;
+        if (c0 + lane < p.vdim) { if (all) all[c0 + lane] = v; else out[c0 + lane] = (bf16)v; }
     }
 }
 

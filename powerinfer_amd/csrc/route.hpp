@@ -4,9 +4,10 @@
 
 namespace {
 
-// soft: the experts with the largest logits, their weights the soft-max over them; else sigmoid scores, a bias on the choice and groups.
+// soft: the experts with the largest logits, their weights the soft-max over them; else sigmoid scores, a bias on the choice (optional) and groups,
+// weights over their sum or (raw) as they are.
 // ldz: values between the tokens' rows of z (0: E)
-struct RouteArgs { const float * z; int E, top, G, keep; const float * bias; int32_t * ids; float * weights; int ldz = 0; bool soft = false; };
+struct RouteArgs { const float * z; int E, top, G, keep; const float * bias; int32_t * ids; float * weights; int ldz = 0; bool soft = false, raw = false; };
 
 __host__ __device__ inline size_t route_lds_bytes(int E, int G, int top) { return sizeof(float) * (size_t)(2 * ((E + 3) / 4 * 4) + (G > top ? G : top)); }
 
@@ -20,7 +21,7 @@ __device__ void route_token(const RouteArgs & r, int t, float * sm) {
         float s = 0.0f, c = -INFINITY;
         if (e < E) {
             s = r.soft ? z[e] : 1.0f / (1.0f + expf(-z[e]));
-            c = r.soft ? s : s + r.bias[e];
+            c = r.soft || !r.bias ? s : s + r.bias[e];
             if (!(c == c)) c = -INFINITY;                      // not a number: never chosen over a number
         }
         sc[e] = s;
@@ -72,7 +73,7 @@ __device__ void route_token(const RouteArgs & r, int t, float * sm) {
         return;
     }
     for (int k = 0; k < r.top; ++k) total += gs[k];
-    for (int k = tid; k < r.top; k += nt) r.weights[(size_t)t * r.top + k] = gs[k] / (total + 1e-20f);
+    for (int k = tid; k < r.top; k += nt) r.weights[(size_t)t * r.top + k] = r.raw ? gs[k] : gs[k] / (total + 1e-20f);
 }
 
 }  // namespace

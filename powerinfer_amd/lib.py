@@ -15,6 +15,7 @@ F32, F16, Q4_0, I32, BF16 = 0, 1, 2, 18, 30
 MIXER_LATENT, MIXER_GROUPED, MIXER_LINEAR, MIXER_KEYED = 0, 1, 2, 3
 DECAY_CONST, DECAY_KEYED, DECAY_GATED = 0, 1, 2
 FFN_NONE, FFN_MOE, FFN_GLU, FFN_GLU_MOE = 0, 1, 2, 3
+ROT_PLAIN, ROT_WAVES, ROT_RAMP = 0, 1, 2
 EPI_NONE, EPI_RELU, EPI_ADD, EPI_ADD2 = 0, 1, 2, 3
 NORM_NONE, NORM_RMS, NORM_LAYER = 0, 1, 2
 
@@ -30,7 +31,8 @@ class GroupGemm(C.Structure):
                 ("x", _vp), ("x_gs", _sz), ("ldx", C.c_int32), ("T", C.c_int32),
                 ("y", _vp), ("y_gs", _sz), ("ldy", C.c_int32), ("y_f32", C.c_int32), ("relu2", C.c_int32),
                 ("alpha", _f), ("off", _vp), ("gather", _vp), ("gather_div", C.c_int32),
-                ("tiles", _vp), ("n_tiles", _vp), ("max_tiles", C.c_int32), ("glu", C.c_int32), ("glu_limit", _f), ("glu_gain", _f)]
+                ("tiles", _vp), ("n_tiles", _vp), ("max_tiles", C.c_int32), ("glu", C.c_int32), ("glu_limit", _f), ("glu_gain", _f),
+                ("pair_w", _vp), ("glu_plain_up", C.c_int32)]
 
 
 class LatentPrep(C.Structure):
@@ -56,13 +58,19 @@ class FfnFront(C.Structure):
 
 class GqaPrep(C.Structure):
     _fields_ = [("z", _vp)] + [(n, C.c_int32) for n in ("ldz", "T", "n_head", "n_kv", "dim", "vdim", "rot_dim", "off_k", "off_v", "hd", "unit")] + [
-        ("cs", _vp), ("eps", _f), ("q", _vp), ("cache", _vp), ("cell", _vp), ("rot_pairs", C.c_int32), ("unit_v", C.c_int32), ("q_norm", _vp), ("k_norm", _vp), ("temp", _vp)]
+        ("cs", _vp), ("eps", _f), ("q", _vp), ("cache", _vp), ("cell", _vp), ("rot_pairs", C.c_int32), ("unit_v", C.c_int32), ("q_norm", _vp), ("k_norm", _vp), ("temp", _vp),
+        ("v_first", _vp), ("v_mix", _vp), ("v_keep", _vp), ("ld_first", C.c_int32)]
 
 
 class GqaAttn(C.Structure):
     _fields_ = [("q", _vp), ("cache", _vp), ("lists", _vp), ("list_ld", _sz), ("work", _vp), ("n_vis", _vp)] + [
         (n, C.c_int32) for n in ("n_work", "T", "n_head", "n_kv", "dim", "vdim", "hd", "n_parts", "wide")] + [
-        ("scale", _f), ("sink", _f), ("scratch", _vp), ("att", _vp), ("ld_att", C.c_int32), ("out_scale", _f), ("window", C.c_int32), ("first", _vp)]
+        ("scale", _f), ("sink", _f), ("scratch", _vp), ("att", _vp), ("ld_att", C.c_int32), ("out_scale", _f), ("window", C.c_int32), ("first", _vp),
+        ("softcap", _f), ("sinks", _vp), ("all_values", C.c_int32)]
+
+
+class GqaMix(C.Structure):
+    _fields_ = [("a", _vp), ("talk", _vp), ("z", _vp)] + [(n, C.c_int32) for n in ("ldz", "off_gate", "T", "n_head", "n_kv", "vdim")] + [("att", _vp), ("ld_att", C.c_int32)]
 
 
 class Linear(C.Structure):
@@ -86,6 +94,16 @@ class LayerOut(C.Structure):
 class ResNorm(C.Structure):
     _fields_ = [(n, _vp) for n in ("x", "mix", "gate_z", "gate_b", "w")] + [(n, C.c_int32) for n in ("ld_gate", "off_gate", "T", "cols")] + [
         ("alpha", _f), ("eps", _f), ("out", _vp), ("keep", _vp), ("h", _vp), ("ld", C.c_int32), ("ol", C.c_int32)]
+
+
+class SumNorm(C.Structure):
+    _fields_ = [("x", _vp), ("mix", _vp), ("y", _vp), ("inv", _vp), ("top", C.c_int32), ("y_w", _vp), ("w", _vp), ("mult", _f), ("w_next", _vp), ("rows", _vp)] + [
+        (n, C.c_int32) for n in ("T", "cols", "groups")] + [("eps", _f), ("keep", _vp), ("h", _vp), ("ld", C.c_int32), ("ol", C.c_int32)]
+
+
+class ConvNorm(C.Structure):
+    _fields_ = [("x", _vp), ("w", _vp), ("taps_w", _vp)] + [(n, C.c_int32) for n in ("T", "cols", "groups", "taps")] + [
+        ("eps", _f), ("state", _vp), ("slot_ld", _sz), ("items", _vp), ("n_items", C.c_int32), ("h", _vp), ("ld", C.c_int32), ("ol", C.c_int32)]
 
 
 class PiError(RuntimeError):
@@ -244,6 +262,14 @@ _SIGS = {
     "pi_k_gqa_attn": (_i, [_i, C.POINTER(GqaAttn), _vp]),
     "pi_k_gqa_attn_parts": (_i, [C.POINTER(GqaAttn), _vp]),
     "pi_k_gqa_shift": (_i, [_i, _vp, _i, _i, _i, _i, C.c_double, _i, _vp, _vp]),
+    "pi_k_gqa_shift_table": (_i, [_i, _vp, _i, _i, _i, _i, _vp, _i, _vp, _vp]),
+    "pi_k_gqa_mix": (_i, [_i, C.POINTER(GqaMix), _vp]),
+    "pi_k_rope_angles_table": (_i, [_vp, _i, _i, _vp, C.c_double, _vp, _vp]),
+    "pi_k_route_scores": (_i, [_vp, _i, _i, _i, _vp, _vp, _vp]),
+    "pi_k_expert_up_step": (_i, [_vp, _i, _i, _i, _f, _f, _i, _i, _vp, _i, _vp, _vp, _i, _vp, _i, _vp]),
+    "pi_k_sum_norm": (_i, [_i, C.POINTER(SumNorm), _vp]),
+    "pi_k_conv_norm": (_i, [_i, C.POINTER(ConvNorm), _vp]),
+    "pi_k_conv_tokens": (_i, [_i, _i]),
     "pi_k_linear_chunk": (_i, []),
     "pi_k_linear_supported": (_i, [_i, _i]),
     "pi_k_linear_states_bytes": (_sz, [_i, _i, _i, _i]),

@@ -7,7 +7,7 @@ import numpy as np
 from . import lib as pl
 from .lib import check
 
-ARCH = {"llama": 0, "falcon": 1, "lerasun": 2, "pibalorn": 3, "fikevik": 4}
+ARCH = {"llama": 0, "falcon": 1, "lerasun": 2, "pibalorn": 3, "fikevik": 4, "pufivik": 5}
 
 # tensor roles, same order as the enum in include/powerinfer_hip.h
 KINDS = ["tok_embd", "output_norm", "output_norm_b", "output",
@@ -20,7 +20,8 @@ KINDS = ["tok_embd", "output_norm", "output_norm_b", "output",
          "bigram", "loop_step", "mix_k", "mix_v", "mix_g", "mix_norm", "mix_decay",
          "expert_gate", "glu_gate", "glu_up", "glu_down", "shared_score",
          "res_gate", "res_gate_b", "res_gate_ffn", "res_gate_ffn_b", "mix_q_norm", "mix_k_norm", "mix_temp", "mix_a1", "mix_a2", "mix_a2_b",
-         "mem_q", "mem_k", "mem_v", "mem_g", "mem_o", "mem_norm", "mem_i", "mem_i_b", "mem_f", "mem_f_b"]
+         "mem_q", "mem_k", "mem_v", "mem_g", "mem_o", "mem_norm", "mem_i", "mem_i_b", "mem_f", "mem_f_b",
+         "attn_norm_after", "ffn_norm_after", "mix_conv", "mix_value", "mix_talk", "mix_head_gate"]
 KIND = {k: i for i, k in enumerate(KINDS)}
 
 
@@ -37,13 +38,16 @@ class LayerDescC(C.Structure):
         ("sink", C.c_float), ("glu_ff", C.c_int32), ("glu_limit", C.c_float), ("expert_limit", C.c_float), ("glu_gain", C.c_float)] + [
         (n, C.c_int32) for n in ("weights_of", "gated_residual", "glu_plain_up", "rot_pairs", "qk_norm", "unit_v", "head_temp", "window")] + [
         ("out_scale", C.c_float), ("mem_heads", C.c_int32), ("mem_dim", C.c_int32), ("mem_vdim", C.c_int32), ("mem_cap", C.c_float), ("mem_scale", C.c_float),
-        ("decay_rank", C.c_int32), ("decay_tau", C.c_float)]
+        ("decay_rank", C.c_int32), ("decay_tau", C.c_float), ("softcap", C.c_float)] + [
+        (n, C.c_int32) for n in ("head_sinks", "head_mix", "head_gate", "value_mix", "rot_scaling")] + [
+        (n, C.c_double) for n in ("rot_factor", "rot_original", "rot_low", "rot_high")] + [("route_scores", C.c_int32), ("weigh_input", C.c_int32)]
 
 
 class LayersOptsC(C.Structure):
     _fields_ = [("compute", C.c_int32), ("logit_scale", C.c_float), ("norm_offset", C.c_float), ("max_batch", C.c_int32),
                 ("embed_scale", C.c_float), ("bigram_buckets", C.c_int32), ("bigram_mul_prev", C.c_int64), ("bigram_mul_cur", C.c_int64),
-                ("loop_start", C.c_int32), ("loop_stop", C.c_int32), ("loop_times", C.c_int32), ("n_slots", C.c_int32), ("post_norm", C.c_int32), ("residual_alpha", C.c_float)]
+                ("loop_start", C.c_int32), ("loop_stop", C.c_int32), ("loop_times", C.c_int32), ("n_slots", C.c_int32), ("post_norm", C.c_int32), ("residual_alpha", C.c_float),
+                ("both_norms", C.c_int32), ("residual_mult", C.c_float), ("norm_groups", C.c_int32), ("conv_taps", C.c_int32)]
 
 
 def _declare(L):

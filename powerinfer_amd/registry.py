@@ -25,7 +25,12 @@ def _fikevik(config, tensors, **kw):
     return fikevik.build(config, tensors, **kw)
 
 
-FOLDERS = {"Lerasun": _lerasun, "Pibalorn": _pibalorn, "Fikevik": _fikevik}
+def _pufivik(config, tensors, **kw):
+    from . import pufivik
+    return pufivik.build(config, tensors, **kw)
+
+
+FOLDERS = {"Lerasun": _lerasun, "Pibalorn": _pibalorn, "Fikevik": _fikevik, "Pufivik": _pufivik}
 
 
 def load_model(path, dtype="bfloat16", n_ctx=4096, max_batch=0):
