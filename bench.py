@@ -488,6 +488,62 @@ def build_fikevik_on_device(width, sh, n_ctx, keep):
     return m
 
 
+# shapes of --design pufivik: eight layers, the two kinds of attention in turn, experts everywhere, beside Pibalorn of equal width, depth (eight layer runs)
+# and experts
+PUFIVIK_SHAPES = {
+    2048: dict(heads=16, kv_heads=4, dim=128, experts=64, top=6, ff=1408, beside=2048),
+    4096: dict(heads=32, kv_heads=8, dim=128, experts=64, top=6, ff=1408, beside=4096),
+    5120: dict(heads=40, kv_heads=8, dim=128, experts=160, top=6, ff=1536, beside=5120),
+}
+
+
+def build_pufivik_on_device(width, sh, n_ctx, keep):
+    """Random-init weights of a Pufivik shape generated in HBM."""
+    from powerinfer_amd import lib as pl, pufivik
+    from powerinfer_amd.model import LayerModel
+    L = pl.init()
+    V, H, dim, f32 = 32000, sh["heads"], sh["dim"], np.float32
+    mix = {"heads": H, "kv_heads": sh["kv_heads"], "dim": dim, "vdim": dim, "scale": dim ** -0.5, "v_mix": True}
+    mlp = {"kind": "moe", "router": {"experts": sh["experts"], "top": sh["top"]}, "expert": {"ff": sh["ff"]}}
+    waves = {"type": "attention", "mlp": mlp, "mixer": dict(mix, rot={"dims": dim // 2, "base": 500000.0, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}})}
+    capped = {"type": "attention_2", "mlp": mlp, "mixer": dict(mix, softcap=50.0, rot={"dims": dim // 2, "base": 10000.0, "scaling": {"factor": 4.0, "slow": 1.0, "fast": 32.0, "original": 4096}})}
+    cfg = {"width": width, "vocab": V, "norm": {"eps": 1e-6, "groups": 8}, "embedding": {"scale": 1.0}, "residual_mult": 0.5, "canon": {"taps": 4}, "layers": [waves, capped] * 4}
+    descs = pufivik.layer_descs(cfg)
+    m = LayerModel("pufivik", descs, n_embd=width, n_vocab=V, n_ctx=n_ctx, norm_eps=1e-6, **pufivik.model_opts(cfg))
+    seed = [7]
+
+    def put(layer, kind, rows, cols):
+        seed[0] += 1
+        buf = pl.DevBuf(rows * cols * 2)
+        pl.check(L.pi_fill_normal_bf16(buf.ptr, rows * cols, seed[0], 0.02, None), "fill")
+        m.set_tensor_device(layer, kind, buf.ptr, pl.BF16, cols, rows)
+        keep.append(buf)
+
+    one = np.ones(width, f32)
+    put(-1, "tok_embd", V, width)
+    put(-1, "output", V, width)
+    m.set_tensor(-1, "output_norm", one)
+    for i, d in enumerate(descs):
+        for k in ("attn_norm", "attn_norm_after", "ffn_norm", "ffn_norm_after"):
+            m.set_tensor(i, k, one)
+        m.set_tensor(i, "mix_conv", np.full((4, width), 0.2, f32))
+        G, E, ff = d["n_kv_head"], d["n_expert"], d["expert_ff"]
+        for k, rows in (("mix_q", H * dim), ("mix_k", G * dim), ("mix_v", G * dim), ("router", E)):
+            put(i, k, rows, width)
+        put(i, "wo", width, H * dim)
+        if i:
+            m.set_tensor(i, "mix_value", np.full(1, 0.4, f32))
+        if d.get("head_mix"):
+            m.set_tensor(i, "mix_sink", np.zeros(H, f32))
+            m.set_tensor(i, "mix_talk", np.eye(H, dtype=f32) + f32(0.1) / H)
+            put(i, "mix_head_gate", H, width)
+        for k, rows, cols in (("expert_gate", E * ff, width), ("expert_up", E * ff, width), ("expert_down", E * width, ff)):
+            put(i, k, rows, cols)
+    pl.sync()
+    m.finalize()
+    return m
+
+
 def time_prefill_and_decode(m, n_prompt, steps, warmup):
     """(prompt seconds, seconds per decoded token) of one sequence: the prompt through Model.decode (second pass timed), then the greedy loop."""
     from powerinfer_amd import lib as pl
@@ -523,12 +579,12 @@ def time_lockstep(m, n_seq, n_prompt, steps, warmup):
 
 def bench_design(args):
     """Prefill and decode of a design described layer by layer at sizes like a real model's, beside the closest existing model at equal width
-    and depth: the sparse LLaMA engine for Lerasun, Lerasun for Pibalorn, Pibalorn for Fikevik."""
+    and depth: the sparse LLaMA engine for Lerasun, Lerasun for Pibalorn, Pibalorn for Fikevik and Pufivik."""
     from powerinfer_amd import lib as pl, synth
     pl.init()
     n_prompt, steps, lock_prompt = (2048 if args.prompt == 64 else args.prompt), min(args.steps, 128), 128
     n_ctx = n_prompt + steps + args.warmup + 8
-    shapes = {"lerasun": DESIGN_SHAPES, "pibalorn": PIBALORN_SHAPES, "fikevik": FIKEVIK_SHAPES}[args.design]
+    shapes = {"lerasun": DESIGN_SHAPES, "pibalorn": PIBALORN_SHAPES, "fikevik": FIKEVIK_SHAPES, "pufivik": PUFIVIK_SHAPES}[args.design]
     rows = []
     for width in ([args.design_width] if args.design_width else sorted(shapes)):
         sh = shapes[width]
@@ -539,7 +595,9 @@ def bench_design(args):
             keep = []
             if who == "fikevik":
                 m = build_fikevik_on_device(width, sh, n_ctx, keep)
-            elif args.design == "fikevik":
+            elif who == "pufivik":
+                m = build_pufivik_on_device(width, sh, n_ctx, keep)
+            elif args.design in ("fikevik", "pufivik"):
                 m = build_pibalorn_on_device(width, PIBALORN_SHAPES[sh["beside"]], n_ctx, keep)
             elif who == "pibalorn":
                 m = build_pibalorn_on_device(width, sh, n_ctx, keep)
@@ -569,9 +627,9 @@ def bench_design(args):
 
 def main():
     ap = argparse.ArgumentParser()
-    ap.add_argument("--design", choices=["lerasun", "pibalorn", "fikevik"], default=None, help="instead of the default workload: prefill and decode of this design beside the closest existing model")
+    ap.add_argument("--design", choices=["lerasun", "pibalorn", "fikevik", "pufivik"], default=None, help="instead of the default workload: prefill and decode of this design beside the closest existing model")
     ap.add_argument("--design-width", type=int, default=None, choices=sorted(DESIGN_SHAPES), help="one size of --design only")
-    ap.add_argument("--design-only", choices=["lerasun", "pibalorn", "fikevik", "beside"], default=None, help="one side of --design only")
+    ap.add_argument("--design-only", choices=["lerasun", "pibalorn", "fikevik", "pufivik", "beside"], default=None, help="one side of --design only")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=256)
     ap.add_argument("--warmup", type=int, default=8)

@@ -696,8 +696,16 @@ PI_API int    pi_k_gqa_attn_parts(const pi_gqa_attn * p, pi_stream_t stream);
  * (talk NULL: a[t][h][..]; off_gate < 0: no gate). */
 typedef struct pi_gqa_mix {
     const float * a, * talk, * z; int32_t ldz, off_gate, T, n_head, n_kv, vdim; void * att; int32_t ld_att;
+    const int32_t * tokens; int32_t n_tokens;                    /* optional: these tokens only */
 } pi_gqa_mix;
 PI_API int    pi_k_gqa_mix(int type, const pi_gqa_mix * p, pi_stream_t stream);
+/* The same for long runs (bf16) without a result per pair of heads: pi_k_gqa_stats leaves every row's log2 of its soft-max denominator in stats [T][n_head]
+ * (attn: wide work items, its sinks, soft cap and window), pi_k_gqa_talk forms the weights again, mixes them (mix: talk, gate and att) and applies them.  items
+ * [n_items] of four integers: {first token, tokens, sequence, 0}, consecutive tokens of one sequence, at most pi_k_gqa_talk_tokens (0: sizes that are
+ * not supported).  talk is rounded to bf16. */
+PI_API int    pi_k_gqa_talk_tokens(int n_head, int n_kv, int dim, int vdim);
+PI_API int    pi_k_gqa_stats(const pi_gqa_attn * attn, float * stats, pi_stream_t stream);
+PI_API int    pi_k_gqa_talk(const pi_gqa_attn * attn, const pi_gqa_mix * mix, const float * stats, const int32_t * items, int n_items, pi_stream_t stream);
 /* rotates the key parts of cells by delta[cell] positions (pairs != 0: neighbouring values are a pair) */
 PI_API int pi_k_gqa_shift(int type, void * cache, int n_cells, int n_kv, int hd, int rot_dim, double base, int pairs, const int32_t * delta, pi_stream_t stream);
 PI_API int pi_k_gqa_shift_table(int type, void * cache, int n_cells, int n_kv, int hd, int rot_dim, const double * freq, int pairs, const int32_t * delta, pi_stream_t stream);
@@ -797,7 +805,7 @@ typedef struct pi_sum_norm {
     const float * w_next; const int32_t * rows; int32_t T, cols, groups; float eps; float * keep; void * h; int32_t ld, ol;
 } pi_sum_norm;
 PI_API int pi_k_sum_norm(int type, const pi_sum_norm * p, pi_stream_t stream);
-/* A norm in groups and behind it a causal convolution over time on every channel: u = norm(x[t]) * w, h[t] = u_t + sum over j of taps_w[c][j] *
+/* A norm in groups and behind it a causal convolution over time on every channel: u = norm(x[t]) * w, h[t] = u_t + sum over j of taps_w[j][c] *
  * u_(t - taps + 1 + j) along the token's sequence, zeros ahead of it.  items [n_items] of eight integers: {first token, tokens, tokens of the run ahead of
  * them, tokens of the run, slot, 1 if nothing lies before the run, 0, 0}; a run's first item holds at least min(taps - 1, all) of its tokens, reads the last
  * taps - 1 inputs before the run from state + slot * slot_ld ([taps - 1][cols] fp32) and leaves those before the run's end there. */
@@ -913,7 +921,7 @@ enum {
  *   glu_ff > 0: beside them a shared one (PI_T_GLU_*, glu_limit) that every token uses times sigmoid(PI_T_SHARED_SCORE [1][n_embd] h).
  *
  * both_norms: a layer is x = x + residual_mult * norm(mixer(conv(norm(x)))), then the same with the feed-forward and without the convolution; norms in
- * norm_groups groups (PI_T_ATTN_NORM, _ATTN_NORM_AFTER, PI_T_FFN_NORM, _FFN_NORM_AFTER), conv_taps > 0: PI_T_MIX_CONV [n_embd][conv_taps] (pi_conv_norm; the
+ * norm_groups groups (PI_T_ATTN_NORM, _ATTN_NORM_AFTER, PI_T_FFN_NORM, _FFN_NORM_AFTER), conv_taps > 0: PI_T_MIX_CONV [conv_taps][n_embd] (pi_conv_norm; the
  * last conv_taps - 1 inputs are a state of the sequence); mixer PI_MIXER_GROUPED, feed-forwards PI_FFN_NONE and PI_FFN_GLU_MOE without a shared one.
  * With it grouped-query attention may have: softcap (pi_gqa_attn); head_sinks: PI_T_MIX_SINK [n_head]; head_mix: PI_T_MIX_TALK [n_head][n_head], soft-max
  *   weights mixed over the heads (pi_gqa_mix); head_gate: heads times sigmoid(PI_T_MIX_HEAD_GATE [n_head][n_embd] h); value_mix: all layers that have it but the

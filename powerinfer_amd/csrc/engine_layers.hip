@@ -21,6 +21,7 @@ constexpr long long kExpandedValues = 1LL << 29;      // most expanded key and v
 constexpr int kItemRows = 32;             // query rows of an attention work item
 constexpr int kAttnItems = 512;          // (work item, part) pairs a split attention aims at: two workgroups per compute unit
 constexpr int kWideRows = 64;            // query rows from which a run of grouped-query attention takes the wide work items
+constexpr int kTalkItems = 32;           // items from which pi_k_gqa_talk fills enough of the device (fewer: the cells of an item are split)
 constexpr int kLinearChunked = 17;       // tokens from which a run of linear attention is worked in chunks
 constexpr int kFreshSteps = 4;           // first tokens of a sequence that a norm over every head's sums is sensitive to (see layers_step)
 
@@ -93,7 +94,8 @@ struct Rotation {
 // n_head: of a work item's rows - all heads on a latent, the heads of a group otherwise (n_kv groups, with pi_gqa_attn's all_values pairs of them; kd
 // values of a key row)
 // window > 0: cells a token sees
-struct HeadKind { int mixer, n_head, n_kv, dim, rot_dim, vdim, rank_ld, kd, window; };
+// talk_tokens: tokens of an item of pi_k_gqa_talk (0: that does not serve these heads)
+struct HeadKind { int mixer, n_head, n_kv, dim, rot_dim, vdim, rank_ld, kd, window, talk_tokens; };
 enum Family { kTwoNorms, kOneNorm, kPostNorm, kBothNorms };
 
 // where a pass finds its tokens
@@ -109,6 +111,9 @@ struct Step {
     // grouped-query attention: the long runs as wide work items (per kind); linear attention: the runs walked token by token and in chunks;
     // prev: each token's predecessor (carry: the embedding moves it on, for a captured step)
     std::vector<Work> wide;
+    // heads mixed behind their attention: the tokens of the long runs for pi_k_gqa_talk (then the wide items are its first pass's), and the others
+    std::vector<Work> talk;
+    std::vector<Work> apart;
     std::vector<const int32_t *> first;                // per kind: the first cell of each token's window (null: counted back from its last)
     int32_t * prev = nullptr; bool carry = false;
     const int32_t *lin = nullptr, *lin_long = nullptr, *lin_first = nullptr, *lin_chunks = nullptr;
@@ -146,7 +151,7 @@ struct LayerState {
     void *lin_q = nullptr, *lin_k = nullptr, *lin_v = nullptr, *lin_states = nullptr;
     void *h_a = nullptr, *h_b = nullptr, *q_un = nullptr, *q_lat = nullptr, *o_lat = nullptr, *att = nullptr, *act = nullptr, *y_exp = nullptr;
     int32_t *ids = nullptr, *perm = nullptr, *inv = nullptr, *off = nullptr, *tiles = nullptr, *n_tiles = nullptr;
-    float *heads = nullptr, *v_first = nullptr;        // the heads' results ahead of their mixture, the first values of the step's tokens
+    float *heads = nullptr, *v_first = nullptr, *stats = nullptr;        // the heads' results ahead of their mixture, the first values of the step's tokens
     std::vector<float *> cs;                           // per rotation [cap][dims / 2] (cos, sin)
     bf16_t * expanded = nullptr; size_t expanded_cap = 0;      // keys and values of a long run's cells
     float * scratch = nullptr;                         // partial sums of a split attention
@@ -450,7 +455,7 @@ int both_norms_weights(pi_model * m, int il) {
     PI_TRY(norm(PI_T_ATTN_NORM, "attn_norm", &L.norm_a));
     PI_TRY(norm(PI_T_ATTN_NORM_AFTER, "attn_norm_after", &L.norm_a_after));
     if (s->opts.conv_taps > 0) {
-        PI_TRY(want_tensor(m->L(il, PI_T_MIX_CONV), PI_TYPE_F32, s->opts.conv_taps, D, "mix_conv"));
+        PI_TRY(want_tensor(m->L(il, PI_T_MIX_CONV), PI_TYPE_F32, D, s->opts.conv_taps, "mix_conv"));
         L.conv = (const float *)m->L(il, PI_T_MIX_CONV).dev;
     }
     uint16_t * z = zeroed(m, (size_t)L.z_rows * s->d_ld);
@@ -573,7 +578,7 @@ int ensure_capacity(pi_model * m, int T) {
     int cap = 64;
     while (cap < T) cap *= 2;
     const size_t es = s->es, D = m->hp.n_embd;
-    size_t z = 0, qu = 0, ql = 0, ol = 0, at = 0, E = 0, top = 0, ff = 0, lq = 0, lv = 0, lo = 0, ls = 0, ln = 0, lg = 0, hr = 0, vf = 0;
+    size_t z = 0, qu = 0, ql = 0, ol = 0, at = 0, E = 0, top = 0, ff = 0, lq = 0, lv = 0, lo = 0, ls = 0, ln = 0, lg = 0, hr = 0, vf = 0, sh = 0;
     const size_t chunks = s->recurrent && bf16_mode(s) ? (size_t)cap / pi_k_linear_chunk() + 32 : 0;        // every run of a pass ends with a part of one
     for (const Layer & L : s->layers) {
         const pi_layer_desc & d = L.d;
@@ -581,6 +586,7 @@ int ensure_capacity(pi_model * m, int T) {
             z = std::max({z, (size_t)L.z_rows, (size_t)L.z2_rows}); at = std::max({at, (size_t)L.close_ld, (size_t)L.glu_ld});
             if (d.mixer == PI_MIXER_GROUPED) ql = std::max(ql, (size_t)d.n_head * L.hd);
             if (L.heads_apart()) hr = std::max(hr, (size_t)d.n_head * d.n_kv_head * d.vdim);
+            if (L.heads_apart()) sh = std::max(sh, (size_t)d.n_head);
             if (d.value_mix) vf = std::max(vf, (size_t)d.n_kv_head * d.vdim);
             const Rec & r = L.rec;
             if (r.on()) {
@@ -620,7 +626,7 @@ int ensure_capacity(pi_model * m, int T) {
         carve(s->tiles, (n * top / 64 + E + 1) * 8); carve(s->n_tiles, 4);
         carve(s->x0, s->opts.loop_times > 0 ? n * D * 4 : 0);
         carve(s->lin_o, n * lo * 4); carve(s->lin_q, n * lq * 2); carve(s->lin_k, n * lq * 2); carve(s->lin_v, n * lv * 2); carve(s->lin_states, ls);
-        carve(s->lin_den, n * ln * 4); carve(s->lin_gates, lg * 4); carve(s->heads, n * hr * 4); carve(s->v_first, n * vf * 4);
+        carve(s->lin_den, n * ln * 4); carve(s->lin_gates, lg * 4); carve(s->heads, n * hr * 4); carve(s->v_first, n * vf * 4); carve(s->stats, n * sh * 4);
         s->cs.resize(s->rots.size());
         for (size_t r = 0; r < s->rots.size(); ++r) carve(s->cs[r], n * s->rots[r].dims * 4);
     };
@@ -824,7 +830,7 @@ pi_gqa_prep gqa_prep_args(pi_model * m, const Layer & L, int pass, const Step & 
 int attend_grouped(pi_model * m, const Layer & L, int pass, const Step & in, bool step, pi_gqa_attn & parts) {
     LayerState * s = m->lay;
     const int type = s->opts.compute;
-    if (bf16_mode(s) && in.wide[L.hc].n > 0) {
+    if (bf16_mode(s) && in.wide[L.hc].n > 0 && in.talk[L.hc].n == 0) {
         const pi_gqa_attn a = gqa_args(m, L, pass, in, in.wide[L.hc], 1);
         PI_TRY(pi_k_gqa_attn(type, &a, m->stream));
     }
@@ -997,10 +1003,17 @@ int both_norms_layer(pi_model * m, Layer & L, const LayerRun & r, const Step & i
     PI_TRY(attend_grouped(m, L, r.pass, in, step, parts));
     if (parts.n_parts > 1) PI_TRY(pi_k_mix_up_step(&parts, nullptr, nullptr, 0, 0, 0, 0.0f, 0.0f, nullptr, T, nullptr, nullptr, 0, nullptr, 0, st));
     if (L.heads_apart()) {
+        const Step::Work & talk = in.talk[L.hc], & apart = in.apart[L.hc];
         pi_gqa_mix x{};
         x.a = s->heads; x.talk = L.talk; x.z = s->z; x.ldz = L.z_rows; x.off_gate = L.off_head_gate; x.T = T; x.n_head = d.n_head; x.n_kv = d.n_kv_head; x.vdim = d.vdim;
         x.att = s->att; x.ld_att = L.close_ld;
-        PI_TRY(pi_k_gqa_mix(type, &x, st));
+        if (talk.n > 0) {
+            const pi_gqa_attn a = gqa_args(m, L, r.pass, in, in.wide[L.hc], 1);
+            PI_TRY(pi_k_gqa_stats(&a, s->stats, st));
+            PI_TRY(pi_k_gqa_talk(&a, &x, s->stats, talk.items, talk.n, st));
+            x.tokens = apart.items; x.n_tokens = apart.n;
+        }
+        if (talk.n == 0 || apart.n > 0) PI_TRY(pi_k_gqa_mix(type, &x, st));
     }
     pi_layer_out o{};
     o.rows = D; o.T = T; o.out = s->mix;
@@ -1150,6 +1163,19 @@ void gqa_items(const int32_t * seq, const int32_t * n_vis, int n, int per, std::
         const bool w = wide && rows >= kWideRows;
         const int step = pi_k_gqa_rows(w);
         for (int r = 0; r < rows; r += step) { const int32_t item[4] = {t0, r, std::min(step, rows - r), seq[t0]}; (w ? *wide : narrow).insert((w ? *wide : narrow).end(), item, item + 4); }
+        t0 = t1;
+    }
+}
+
+// the tokens of the runs that gqa_items takes as wide ones, as items of pi_k_gqa_talk, and all others
+void talk_items(const int32_t * seq, const int32_t * n_vis, int n, const HeadKind & h, std::vector<int32_t> & items, std::vector<int32_t> & others) {
+    for (int t0 = 0; t0 < n;) {
+        int t1 = t0 + 1;
+        while (t1 < n && seq[t1] == seq[t0] && n_vis[t1] >= n_vis[t1 - 1]) ++t1;
+        if ((t1 - t0) * h.n_head >= kWideRows)
+            for (int t = t0; t < t1; t += h.talk_tokens) { const int32_t item[4] = {t, std::min(h.talk_tokens, t1 - t), seq[t0], 0}; items.insert(items.end(), item, item + 4); }
+        else
+            for (int t = t0; t < t1; ++t) others.push_back(t);
         t0 = t1;
     }
 }
@@ -1378,7 +1404,8 @@ int layers_finalize(pi_model * m) {
                 L.hd = pi_k_gqa_head_ld(s->opts.compute, d.dim, d.vdim);
                 if (!L.hd) return fail(PI_E_UNSUPPORTED, "pi_model_finalize: head sizes outside the attention kernels (up to 256)");
                 if (d.rot_dim > 0) PI_TRY(rotation()); else L.rot = -1;
-                kind(HeadKind{d.mixer, d.n_head / d.n_kv_head, d.n_kv_head * (L.heads_apart() ? d.n_kv_head : 1), 0, 0, 0, 0, L.hd, d.window});
+                kind(HeadKind{d.mixer, d.n_head / d.n_kv_head, d.n_kv_head * (L.heads_apart() ? d.n_kv_head : 1), 0, 0, 0, 0, L.hd, d.window,
+                              L.heads_apart() && bf16_mode(s) ? pi_k_gqa_talk_tokens(d.n_head, d.n_kv_head, d.dim, d.vdim) : 0});
                 scratch = std::max(scratch, pi_k_gqa_scratch_floats(kAttnItems, 1, 1, L.hd, 2) / 2);      // items x groups x parts <= kAttnItems
             }
             if (L.rec.on() && !pi_k_linear_supported(L.rec.dim, L.rec.vdim)) return fail(PI_E_UNSUPPORTED, "pi_model_finalize: head sizes outside the linear attention's kernels (up to 256)");
@@ -1393,7 +1420,7 @@ int layers_finalize(pi_model * m) {
         L.hv_ld = up_to(d.n_head * d.vdim, 128); L.ff_ld = d.ffn == PI_FFN_MOE ? up_to(d.expert_ff, 64) : 0;
         if (!pi_k_latent_attn_supported(s->opts.compute, L.rank_ld, L.kd)) return fail(PI_E_UNSUPPORTED, "pi_model_finalize: latent sizes outside the attention kernels (rank up to 1024)");
         PI_TRY(rotation());
-        kind(HeadKind{d.mixer, d.n_head, 1, d.dim, d.rot_dim, d.vdim, L.rank_ld, L.kd, 0});
+        kind(HeadKind{d.mixer, d.n_head, 1, d.dim, d.rot_dim, d.vdim, L.rank_ld, L.kd, 0, 0});
         scratch = std::max(scratch, pi_k_latent_attn_scratch_floats(kItemRows * kAttnItems / 2, L.rank_ld, 2));      // items x parts <= kAttnItems
         PI_TRY(layer_weights(m, (int)il));
     }
@@ -1499,6 +1526,16 @@ int layers_step(pi_model * m, const int32_t * tokens, const int32_t * positions,
         begin.push_back(items.size());
         begin_wide.push_back(wide.size());
         items.insert(items.end(), wide.begin(), wide.end());
+        std::vector<size_t> at_talk, at_apart;
+        std::vector<int> n_talk, n_apart;
+        std::vector<int32_t> others;
+        for (const HeadKind & h : s->kinds) {
+            at_talk.push_back(items.size()); at_apart.push_back(others.size());
+            if (h.talk_tokens > 0 && T > 16) talk_items(seq.data() + t0, vis.data() + t0, T, h, items, others);
+            n_talk.push_back((int)(items.size() - at_talk.back()) / 4);
+            if (n_talk.back() < kTalkItems) { items.resize(at_talk.back()); others.resize(at_apart.back()); n_talk.back() = 0; }
+            n_apart.push_back((int)(others.size() - at_apart.back()));
+        }
         const size_t at_conv = items.size();
         if (s->opts.conv_taps > 0) {
             const int back = s->opts.conv_taps - 1, per = pi_k_conv_tokens(T, s->opts.conv_taps);
@@ -1553,6 +1590,8 @@ int layers_step(pi_model * m, const int32_t * tokens, const int32_t * positions,
                 items.push_back((int32_t)(std::upper_bound(lp.begin(), lp.end(), positions[t0 + t] - h.window) - lp.begin()));
             }
         }
+        const size_t at_others = items.size();
+        items.insert(items.end(), others.begin(), others.end());
         const size_t n_in = (size_t)8 * T + items.size() + rows.size();
         PI_TRY(ensure_inputs(m, n_in));
         PI_HIP_TRY(hipStreamSynchronize(m->stream));
@@ -1578,6 +1617,10 @@ int layers_step(pi_model * m, const int32_t * tokens, const int32_t * positions,
             wd.n = (int)(begin_wide[k + 1] - begin_wide[k]) / 4;
             wd.parts = gqa_parts(wd.n * hk.n_kv, gqa_span(hk, vmax, true), 512);
             in.wide.push_back(wd);
+            Step::Work talk, apart;
+            talk.items = s->d_in + 8 * T + at_talk[k]; talk.n = n_talk[k];
+            apart.items = s->d_in + 8 * T + at_others + at_apart[k]; apart.n = n_apart[k];
+            in.talk.push_back(talk); in.apart.push_back(apart);
             in.first.push_back(at_first[k] < 0 ? nullptr : s->d_in + 8 * T + at_first[k]);
         }
         s->streams_T = 0;
@@ -1724,7 +1767,7 @@ int layers_generate(pi_model * m, int own, int n_steps, int32_t * out_tokens, fl
         w.n = bf16_mode(s) ? (int)(items.size() - at) / 4 : T;
         w.parts = h.mixer == PI_MIXER_GROUPED ? (bf16_mode(s) ? gqa_parts(w.n * h.n_kv, gqa_span(h, vmax, false), 128) : 1) : choose_parts(s, w.n, vmax);
         in.work.push_back(w);
-        in.wide.emplace_back();
+        in.wide.emplace_back(); in.talk.emplace_back(); in.apart.emplace_back();
         in.first.push_back(nullptr);                           // (the positions are 0, 1, 2 ..)
         parts.push_back(w.parts);
     }

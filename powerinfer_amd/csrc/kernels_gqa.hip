@@ -253,6 +253,269 @@ __global__ __launch_bounds__(256, WIDE && KS <= 4 ? 2 : 1) void gqa_attn_kernel(
     }
 }
 
+// ---------------------------------------------------------------------------------------------------------------------------------
+// Long runs whose heads' weights are mixed, in two passes over the cells.  The first leaves the soft-max denominator of every (token, head).
+// The second has a wave per key / value head: it forms its heads' weights from the denominators, hands them to the others through LDS, mixes those
+// of all heads into its own and applies them to its values.  A tile's 16 rows are (token, head of the group) pairs, so the mixture is a product with a
+// matrix that is zero between different tokens; the scores come out with rows as the inner dimension of that product, and its result with cells
+// as the inner dimension of the product with the values.  Weights are mixed as sums of two bf16.
+// ---------------------------------------------------------------------------------------------------------------------------------
+constexpr float kLog2E = 1.4426950408889634f;
+template <int KS>
+__global__ __launch_bounds__(256) void gqa_stats_kernel(pi_gqa_attn p, float * __restrict__ stats) {
+    constexpr int NK = 64, ROW = KS * 64 + 16, HD = KS * 32, C = 4 * KS, LD = (NK * C + 255) / 256;      // pieces of 16 bytes of a tile, per thread
+    __shared__ __align__(16) unsigned char ks[NK * ROW];
+    const int g = blockIdx.x % p.n_kv, item_index = p.n_work - 1 - (int)blockIdx.x / p.n_kv;
+    const int4 item = reinterpret_cast<const int4 *>(p.work)[item_index];
+    const int tok0 = item.x, first = item.y, rows = min(item.z, 128), per = p.n_head / p.n_kv;
+    const int32_t * list = p.lists + (size_t)item.w * p.list_ld;
+    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, i = lane & 15, gq = lane >> 4;
+    const int tok_a = tok0 + first / per, tok_z = tok0 + (first + rows - 1) / per, n_keys = p.n_vis[tok_z], n_all = p.n_vis[tok_a], lo_a = first_cell(p, tok_a), lo_z = first_cell(p, tok_z);
+    const uint16_t * cache = (const uint16_t *)p.cache + (size_t)g * 2 * HD;
+    pi_u32x4 pre[LD];
+    auto fetch = [&](int cb) {
+#pragma unroll
+        for (int k = 0; k < LD; ++k) {
+            const int e = min(tid + 256 * k, NK * C - 1);
+            pre[k] = pi_ld16(cache + (size_t)list[min(cb + e / C, n_keys - 1)] * p.n_kv * 2 * HD + (e % C) * 8);
+        }
+    };
+    fetch(lo_a);
+    int lo[2], tok[2], head[2], row[2];
+    unsigned nv[2];
+    pi_u32x4 qf[2][KS];
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+        row[u] = wave * 32 + u * 16 + i;
+        const int rr = first + min(row[u], rows - 1);
+        tok[u] = tok0 + rr / per;
+        head[u] = g * per + rr % per;
+        lo[u] = first_cell(p, tok[u]);
+        nv[u] = row[u] < rows ? p.n_vis[tok[u]] - lo[u] : 0;
+#pragma unroll
+        for (int s = 0; s < KS; ++s) qf[u][s] = pi_ld16((const uint16_t *)p.q + ((size_t)tok[u] * p.n_head + head[u]) * HD + s * 32 + gq * 8);
+    }
+    const float cap_k = p.softcap > 0.0f ? kTwoLog2E / p.softcap : 0.0f;
+    float m[2] = {-INFINITY, -INFINITY}, l[2] = {0.0f, 0.0f};      // of this lane's cells, scores times log2 e
+    for (int cb = lo_a; cb < n_keys; cb += NK) {
+        __syncthreads();
+#pragma unroll
+        for (int k = 0; k < LD; ++k) {
+            const int e = tid + 256 * k;
+            if (e < NK * C) *reinterpret_cast<pi_u32x4 *>(ks + (e / C) * ROW + (e % C) * 16) = pre[k];
+        }
+        __syncthreads();
+        fetch(cb + NK);                                          // past the last tile: rows of the last cell, not used
+        pi_f4 s[2][4];
+#pragma unroll
+        for (int kt = 0; kt < 4; ++kt) {
+            s[0][kt] = s[1][kt] = pi_f4{0, 0, 0, 0};
+#pragma unroll
+            for (int c = 0; c < KS; ++c) {
+                const pi_u32x4 a = *reinterpret_cast<const pi_u32x4 *>(ks + (kt * 16 + i) * ROW + c * 64 + gq * 16);
+#pragma unroll
+                for (int u = 0; u < 2; ++u) s[u][kt] = mfma_bf16(a, qf[u][c], s[u][kt]);
+            }
+        }
+        const bool edge = cb + NK > n_all || cb < lo_z;
+#pragma unroll
+        for (int u = 0; u < 2; ++u) {
+            float mx = m[u];
+#pragma unroll
+            for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    float v = s[u][kt][r] * p.scale;
+                    if (p.softcap > 0.0f) v = soft_cap(v, cap_k, p.softcap);
+                    v *= kLog2E;
+                    if (edge && (unsigned)(cb + kt * 16 + 4 * gq + r - lo[u]) >= nv[u]) v = -INFINITY;
+                    s[u][kt][r] = v;
+                    mx = fmaxf(mx, v);
+                }
+            const float base = mx == -INFINITY ? 0.0f : mx;
+            float sum = l[u] * __builtin_amdgcn_exp2f(m[u] - base);
+#pragma unroll
+            for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) sum += __builtin_amdgcn_exp2f(s[u][kt][r] - base);
+            m[u] = mx; l[u] = sum;
+        }
+    }
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+        float mm = fmaxf(m[u], __shfl_xor(m[u], 16, PI_WAVE));
+        mm = fmaxf(mm, __shfl_xor(mm, 32, PI_WAVE));
+        const float sink = (p.sinks ? p.sinks[head[u]] : p.sink) * kLog2E;
+        mm = fmaxf(mm, sink);
+        float sum = m[u] == -INFINITY ? 0.0f : l[u] * __builtin_amdgcn_exp2f(m[u] - mm);
+        sum += __shfl_xor(sum, 16, PI_WAVE);
+        sum += __shfl_xor(sum, 32, PI_WAVE);
+        if (row[u] < rows && gq == 0) stats[(size_t)tok[u] * p.n_head + head[u]] = mm + log2f(sum + __builtin_amdgcn_exp2f(sink - mm));
+    }
+}
+
+constexpr int kTalkTiles = 2, kTalkGroups = 8;      // tiles of 16 rows a wave has; most key / value heads
+template <int KS> constexpr size_t talk_values_bytes() { return (size_t)32 * (KS * 64 + 16); }
+inline int talk_pairs(int n_kv) { return (n_kv + 1) / 2; }
+inline size_t talk_weights_bytes(int n_kv) { return (size_t)2 * kTalkTiles * 2 * talk_pairs(n_kv) * 64 * 16; }
+
+template <int KS>
+__global__ __launch_bounds__(64 * kTalkGroups) void gqa_talk_kernel(pi_gqa_attn p, pi_gqa_mix x, const float * __restrict__ stats, const int4 * __restrict__ items, int n_items) {
+    constexpr int U = kTalkTiles, VT = 2 * KS, ROW = KS * 64 + 16, HD = KS * 32, C = 4 * KS, LD = 32 * C / 64, MAXP = kTalkGroups / 2;
+    extern __shared__ __align__(16) unsigned char smem[];
+    const int pairs = (p.n_kv + 1) / 2, groups = 2 * pairs;
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, i = lane & 15, gq = lane >> 4, g = wave;
+    pi_u32x4 * ws = reinterpret_cast<pi_u32x4 *>(smem);           // [2 cell tiles][U][groups][64]: four weights as bf16, and what is left of them
+    unsigned char * vs = smem + (size_t)2 * U * groups * 64 * 16 + (size_t)wave * talk_values_bytes<KS>();
+    const int4 item = items[n_items - 1 - (int)blockIdx.x];       // the last items see the most cells
+    const int tok0 = item.x, n_tok = item.y, per = p.n_head / p.n_kv, tpt = 16 / per;      // tokens of a tile
+    const int32_t * list = p.lists + (size_t)item.z * p.list_ld;
+    const int n_keys = p.n_vis[tok0 + n_tok - 1], n_all = p.n_vis[tok0], lo_a = first_cell(p, tok0), lo_z = first_cell(p, tok0 + n_tok - 1);
+    const uint16_t * cache = (const uint16_t *)p.cache + (size_t)g * 2 * HD;
+    if (p.n_kv & 1)                                               // the missing group of the last pair: zeros
+        for (int k = threadIdx.x; k < 2 * U * 64; k += blockDim.x) ws[((k >> 6) * groups + p.n_kv) * 64 + (k & 63)] = pi_u32x4{0, 0, 0, 0};
+    // rows 4 gq + r of the wave's tiles
+    float c[U][4];
+    int lo[U][4];
+    unsigned nv[U][4];
+    pi_u32x4 qf[U][KS];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int row = 4 * gq + r, tl = u * tpt + row / per;
+            const bool in = row < tpt * per && tl < n_tok;
+            const int t = tok0 + (in ? tl : 0);
+            lo[u][r] = first_cell(p, t);
+            nv[u][r] = in ? p.n_vis[t] - lo[u][r] : 0;
+            c[u][r] = in ? stats[(size_t)t * p.n_head + g * per + row % per] : 0.0f;
+        }
+        const int tq = tok0 + (i < tpt * per ? min(u * tpt + i / per, n_tok - 1) : 0), hq = g * per + i % per;
+#pragma unroll
+        for (int s = 0; s < KS; ++s) qf[u][s] = pi_ld16((const uint16_t *)p.q + ((size_t)tq * p.n_head + hq) * HD + s * 32 + gq * 8);
+    }
+    // column operand of the mixture: slot (gq, j) is row 4 gq + j of the pair's first group or row 4 gq + j - 4 of its second
+    pi_u32x4 tf[MAXP];
+#pragma unroll
+    for (int q = 0; q < MAXP; ++q) {
+        bf16 b[8];
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+            const int row = 4 * gq + (j & 3), from = 2 * q + (j >> 2);
+            const bool in = from < p.n_kv && row < tpt * per && i < tpt * per && row / per == i / per;
+            const int at = in ? (g * per + i % per) * p.n_head + from * per + row % per : 0;
+            b[j] = (bf16)(in ? (x.talk ? x.talk[at] : (float)(at / p.n_head == at % p.n_head)) : 0.0f);
+        }
+        tf[q] = __builtin_bit_cast(pi_u32x4, b);
+    }
+    pi_f4 o[U][VT];
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+#pragma unroll
+        for (int v = 0; v < VT; ++v) o[u][v] = pi_f4{0, 0, 0, 0};
+    const float cap_k = p.softcap > 0.0f ? kTwoLog2E / p.softcap : 0.0f;
+    pi_u32x4 kf[2][KS], vf[LD];
+    int cell = list[min(lo_a + (lane & 31), n_keys - 1)];
+    auto fetch = [&]() {
+#pragma unroll
+        for (int kt = 0; kt < 2; ++kt) {
+            const uint16_t * k = cache + (size_t)__shfl(cell, kt * 16 + i, PI_WAVE) * p.n_kv * 2 * HD + gq * 8;
+#pragma unroll
+            for (int s = 0; s < KS; ++s) kf[kt][s] = pi_ld16(k + s * 32);
+        }
+#pragma unroll
+        for (int k = 0; k < LD; ++k) {
+            const int e = lane + 64 * k;
+            vf[k] = pi_ld16(cache + (size_t)__shfl(cell, e / C, PI_WAVE) * p.n_kv * 2 * HD + HD + (e % C) * 8);
+        }
+    };
+    fetch();
+    cell = list[min(lo_a + 32 + (lane & 31), n_keys - 1)];
+    for (int cb = lo_a; cb < n_keys; cb += 32) {
+        const bool edge = cb + 32 > n_all || cb < lo_z;
+        __syncthreads();                                         // the last tile's weights and values have been read
+#pragma unroll
+        for (int k = 0; k < LD; ++k) { const int e = lane + 64 * k; *reinterpret_cast<pi_u32x4 *>(vs + (e / C) * ROW + (e % C) * 16) = vf[k]; }
+#pragma unroll
+        for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+                pi_f4 s = pi_f4{0, 0, 0, 0};
+#pragma unroll
+                for (int k = 0; k < KS; ++k) s = mfma_bf16(qf[u][k], kf[kt][k], s);
+                bf16 w[8];
+                const bool all_rows = !edge;
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    float v = s[r] * p.scale;
+                    if (p.softcap > 0.0f) v = soft_cap(v, cap_k, p.softcap);
+                    float e = __builtin_amdgcn_exp2f(fmaf(v, kLog2E, -c[u][r]));
+                    if (all_rows ? nv[u][r] == 0 : (unsigned)(cb + kt * 16 + i - lo[u][r]) >= nv[u][r]) e = 0.0f;
+                    w[r] = (bf16)e;
+                    w[4 + r] = (bf16)(e - (float)w[r]);
+                }
+                ws[((kt * U + u) * groups + g) * 64 + lane] = __builtin_bit_cast(pi_u32x4, w);
+            }
+        fetch();                                                 // past the last tile: rows of the last cell, not used
+        cell = list[min(cb + 64 + (lane & 31), n_keys - 1)];
+        __syncthreads();
+        pi_u32x4 pb[U];
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            bf16 b[8];
+#pragma unroll
+            for (int kt = 0; kt < 2; ++kt) {
+                pi_f4 mix = pi_f4{0, 0, 0, 0};
+                const pi_u32x4 * wp = ws + (size_t)(kt * U + u) * groups * 64 + lane;
+#pragma unroll
+                for (int q = 0; q < MAXP; ++q) {
+                    if (q >= pairs) break;
+                    const pi_u32x4 a = wp[(2 * q) * 64], d = wp[(2 * q + 1) * 64];
+                    mix = mfma_bf16(pi_u32x4{a.x, a.y, d.x, d.y}, tf[q], mix);
+                    mix = mfma_bf16(pi_u32x4{a.z, a.w, d.z, d.w}, tf[q], mix);
+                }
+#pragma unroll
+                for (int r = 0; r < 4; ++r) b[kt * 4 + r] = (bf16)mix[r];
+            }
+            pb[u] = __builtin_bit_cast(pi_u32x4, b);
+        }
+#pragma unroll
+        for (int v = 0; v < VT; ++v) {
+            const unsigned char * a = vs + (4 * gq + (i >> 2)) * ROW + (v * 16 + (i & 3) * 4) * 2;
+            const pi_u32x2 l = __builtin_bit_cast(pi_u32x2, tr_read(a)), h = __builtin_bit_cast(pi_u32x2, tr_read(a + 16 * ROW));
+            const pi_u32x4 fr{l.x, l.y, h.x, h.y};
+#pragma unroll
+            for (int u = 0; u < U; ++u) o[u][v] = mfma_bf16(fr, pb[u], o[u][v]);
+        }
+    }
+    const bool quads = ((x.vdim | x.ld_att) & 3) == 0;
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+        const int tl = u * tpt + i / per, head = g * per + i % per;
+        if (i >= tpt * per || tl >= n_tok) continue;
+        const int t = tok0 + tl;
+        const float f = x.off_gate >= 0 ? sigmoid_f32(x.z[(size_t)t * x.ldz + x.off_gate + head]) : 1.0f;
+        bf16 * out = (bf16 *)x.att + (size_t)t * x.ld_att + head * x.vdim;
+#pragma unroll
+        for (int v = 0; v < VT; ++v) {
+            const int col = v * 16 + 4 * gq;
+            const float w[4] = {o[u][v][0] * f, o[u][v][1] * f, o[u][v][2] * f, o[u][v][3] * f};
+            if (col < x.vdim) store4(out + col, w, quads && col + 4 <= x.vdim, x.vdim - col);
+        }
+    }
+}
+
+template <int KS> int launch_talk(const pi_gqa_attn * p, const pi_gqa_mix * x, const float * stats, const int32_t * items, int n, hipStream_t st) {
+    const size_t lds = talk_weights_bytes(p->n_kv) + talk_values_bytes<KS>() * p->n_kv;
+    static bool raised = false;
+    if (!raised) {
+        PI_HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void *>(&gqa_talk_kernel<KS>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)(talk_weights_bytes(kTalkGroups) + talk_values_bytes<KS>() * kTalkGroups)));
+        raised = true;
+    }
+    hipLaunchKernelGGL(gqa_talk_kernel<KS>, dim3(n), dim3(64 * p->n_kv), lds, st, *p, *x, stats, (const int4 *)items, n);
+    return pi::check_launch("pi_k_gqa_talk");
+}
+
 __global__ __launch_bounds__(256) void gqa_merge_kernel(pi_gqa_attn p) {
     const int R4 = gqa_rows(p.wide) / 4, wg = blockIdx.x, n = p.all_values ? p.n_kv * p.n_kv : p.n_kv;
     gqa_merge_row(p, wg / R4 / n, wg / R4 % n, (wg % R4) * 4 + (threadIdx.x >> 6));
@@ -306,7 +569,7 @@ __global__ __launch_bounds__(256) void gqa_attn_f32_kernel(pi_gqa_attn p) {
 template <typename ST>
 __global__ __launch_bounds__(256) void gqa_mix_kernel(pi_gqa_mix p) {
     extern __shared__ __align__(16) float talk[];
-    const int t = blockIdx.x, per = p.n_head / p.n_kv, n = p.n_kv * p.vdim;
+    const int t = p.tokens ? p.tokens[blockIdx.x] : blockIdx.x, per = p.n_head / p.n_kv, n = p.n_kv * p.vdim;
     if (p.talk) {
         for (int i = threadIdx.x; i < p.n_head * p.n_head; i += 256) talk[i] = p.talk[i];
         __syncthreads();
@@ -320,10 +583,16 @@ __global__ __launch_bounds__(256) void gqa_mix_kernel(pi_gqa_mix p) {
     for (int h0 = 0; h0 < per; h0 += 8) {
         float s[8] = {0, 0, 0, 0, 0, 0, 0, 0};
         if (p.talk) {
-            for (int g = 0; g < p.n_head; ++g) {
-                const float v = a[(size_t)g * n];
+            for (int g0 = 0; g0 < p.n_head; g0 += 8) {          // eight heads requested together
+                float v[8];
 #pragma unroll
-                for (int k = 0; k < 8; ++k) s[k] = fmaf(talk[(kv * per + min(h0 + k, per - 1)) * p.n_head + g], v, s[k]);
+                for (int j = 0; j < 8; ++j) v[j] = a[(size_t)min(g0 + j, p.n_head - 1) * n];
+#pragma unroll
+                for (int j = 0; j < 8; ++j) {
+                    if (g0 + j >= p.n_head) break;
+#pragma unroll
+                    for (int k = 0; k < 8; ++k) s[k] = fmaf(talk[(kv * per + min(h0 + k, per - 1)) * p.n_head + g0 + j], v[j], s[k]);
+                }
             }
         } else {
 #pragma unroll
@@ -435,12 +704,48 @@ int pi_k_gqa_attn(int type, const pi_gqa_attn * p, pi_stream_t stream) {
     return pi::check_launch("pi_k_gqa_attn merge");
 }
 
+int pi_k_gqa_talk_tokens(int n_head, int n_kv, int dim, int vdim) {
+    const int hd = pi_k_gqa_head_ld(PI_TYPE_BF16, dim, vdim);
+    if (!hd || hd > 128 || n_head <= 0 || n_kv <= 0 || n_kv > kTalkGroups || n_head % n_kv || n_head / n_kv > 16) return 0;
+    return kTalkTiles * (16 / (n_head / n_kv));
+}
+
+int pi_k_gqa_stats(const pi_gqa_attn * p, float * stats, pi_stream_t stream) {
+    if (!p || !p->q || !p->cache || !p->lists || !p->work || !p->n_vis || !stats || p->n_work <= 0 || p->window < 0 || !p->wide || !pi_k_gqa_talk_tokens(p->n_head, p->n_kv, p->dim, p->vdim) ||
+        p->hd != pi_k_gqa_head_ld(PI_TYPE_BF16, p->dim, p->vdim))
+        return pi::fail(PI_E_ARG, "pi_k_gqa_stats: bad arguments");
+    hipStream_t st = (hipStream_t)stream;
+    const dim3 grid(p->n_work * p->n_kv);
+    switch (p->hd) {
+        case 32: hipLaunchKernelGGL(gqa_stats_kernel<1>, grid, dim3(256), 0, st, *p, stats); break;
+        case 64: hipLaunchKernelGGL(gqa_stats_kernel<2>, grid, dim3(256), 0, st, *p, stats); break;
+        case 96: hipLaunchKernelGGL(gqa_stats_kernel<3>, grid, dim3(256), 0, st, *p, stats); break;
+        default: hipLaunchKernelGGL(gqa_stats_kernel<4>, grid, dim3(256), 0, st, *p, stats);
+    }
+    return pi::check_launch("pi_k_gqa_stats");
+}
+
+int pi_k_gqa_talk(const pi_gqa_attn * p, const pi_gqa_mix * x, const float * stats, const int32_t * items, int n_items, pi_stream_t stream) {
+    if (!p || !x || !p->q || !p->cache || !p->lists || !p->n_vis || !stats || !items || n_items <= 0 || p->window < 0 || !pi_k_gqa_talk_tokens(p->n_head, p->n_kv, p->dim, p->vdim) ||
+        p->hd != pi_k_gqa_head_ld(PI_TYPE_BF16, p->dim, p->vdim) || !x->att || x->vdim != p->vdim || x->ld_att < p->n_head * p->vdim ||
+        (x->off_gate >= 0 && (!x->z || x->off_gate + p->n_head > x->ldz)))
+        return pi::fail(PI_E_ARG, "pi_k_gqa_talk: bad arguments");
+    hipStream_t st = (hipStream_t)stream;
+    switch (p->hd) {
+        case 32: return launch_talk<1>(p, x, stats, items, n_items, st);
+        case 64: return launch_talk<2>(p, x, stats, items, n_items, st);
+        case 96: return launch_talk<3>(p, x, stats, items, n_items, st);
+        default: return launch_talk<4>(p, x, stats, items, n_items, st);
+    }
+}
+
 int pi_k_gqa_mix(int type, const pi_gqa_mix * p, pi_stream_t stream) {
     if (!p || !p->a || !p->att || p->T <= 0 || p->n_head <= 0 || p->n_kv <= 0 || p->n_head % p->n_kv || p->vdim <= 0 || p->ld_att < p->n_head * p->vdim ||
         (p->off_gate >= 0 && (!p->z || p->off_gate + p->n_head > p->ldz)))
         return pi::fail(PI_E_ARG, "pi_k_gqa_mix: bad arguments");
     const size_t lds = p->talk ? sizeof(float) * p->n_head * p->n_head : 0;
-    const dim3 grid(p->T, (p->n_kv * p->vdim + 255) / 256);
+    if (p->tokens && p->n_tokens <= 0) return pi::fail(PI_E_ARG, "pi_k_gqa_mix: bad arguments");
+    const dim3 grid(p->tokens ? p->n_tokens : p->T, (p->n_kv * p->vdim + 255) / 256);
     if (lds > 64 * 1024 || grid.y > 65535) return pi::fail(PI_E_UNSUPPORTED, "pi_k_gqa_mix: up to 128 heads");
     if (type == PI_TYPE_BF16) hipLaunchKernelGGL(gqa_mix_kernel<bf16>, grid, dim3(256), lds, (hipStream_t)stream, *p);
     else if (type == PI_TYPE_F32) hipLaunchKernelGGL(gqa_mix_kernel<float>, grid, dim3(256), lds, (hipStream_t)stream, *p);

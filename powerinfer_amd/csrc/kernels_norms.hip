@@ -109,7 +109,7 @@ __global__ void sum_norm_kernel(pi_sum_norm p) {
 }
 
 // An item of consecutive tokens of one run a workgroup: first the groups' scales of every row the item touches, then column by column the normed
-// inputs of those rows and their convolution.  N: columns of a thread that are worked together.
+// inputs of those rows and their convolution.
 __host__ __device__ inline int conv_rows(int tokens, int taps) { return tokens + 2 * taps; }
 template <typename ST>
 __global__ __launch_bounds__(256) void conv_norm_kernel(pi_conv_norm p, int max_rows) {
@@ -128,7 +128,7 @@ __global__ __launch_bounds__(256) void conv_norm_kernel(pi_conv_norm p, int max_
     ST * h = (ST *)p.h;
     for (int c = threadIdx.x; c < p.cols; c += 256) {
         const int g = c / size;
-        const float w = p.w[c], * tw = p.taps_w + (size_t)c * p.taps;
+        const float w = p.w[c], * tw = p.taps_w + c;
         auto input = [&](int i) -> float {             // the normed input at place i of the item (negative: before it)
             const int r = i + before;
             if (r >= 0) return p.x[(size_t)(t0 + i) * p.cols + c] * scale[r * p.groups + g] * w;
@@ -138,8 +138,8 @@ __global__ __launch_bounds__(256) void conv_norm_kernel(pi_conv_norm p, int max_
         for (int i = 0; i < n; ++i) {
             const float own = input(i);
             float v = 0.0f;
-            for (int j = 0; j < back; ++j) v = fmaf(tw[j], input(i - back + j), v);
-            v = fmaf(tw[back], own, v) + own;
+            for (int j = 0; j < back; ++j) v = fmaf(tw[(size_t)j * p.cols], input(i - back + j), v);
+            v = fmaf(tw[(size_t)back * p.cols], own, v) + own;
             h[p.ol ? pi_ol_index(t0 + i, c) : (size_t)(t0 + i) * p.ld + c] = to_st<ST>(v);
         }
         if (!head || back == 0) continue;
@@ -152,6 +152,83 @@ __global__ __launch_bounds__(256) void conv_norm_kernel(pi_conv_norm p, int max_
             state[(size_t)s * p.cols + c] = v;
         }
     }
+}
+
+// The same, four columns a thread, for up to BACK inputs ahead of a token and N >= BACK tokens of an item: a thread's inputs lie in registers, all requested together.
+template <typename ST, int BACK, int N>
+__global__ __launch_bounds__(1024) void conv_norm_quads_kernel(pi_conv_norm p, int max_rows) {
+    extern __shared__ __align__(16) float sm[];
+    const int4 a = reinterpret_cast<const int4 *>(p.items)[2 * blockIdx.x], b = reinterpret_cast<const int4 *>(p.items)[2 * blockIdx.x + 1];
+    const int t0 = a.x, n = min(a.y, N), off = a.z, len = a.w, slot = b.x, size = p.cols / p.groups;
+    const bool head = off == 0, fresh = b.y != 0;
+    const int before = min(off, BACK), run0 = t0 - off, n_a = n + before, tail = head ? max(n, len - BACK) : len, rows = n_a + (head ? len - tail : 0);
+    if (rows > max_rows) return;                       // (the launcher's bound)
+    float * scale = sm, * part = sm + max_rows * p.groups;
+    group_scales(part, scale, rows, p.groups, p.cols, p.eps, [&](int r) { return p.x + (size_t)(r < n_a ? t0 - before + r : run0 + tail + (r - n_a)) * p.cols; });
+    float * state = p.state ? p.state + slot * p.slot_ld : nullptr;
+    ST * h = (ST *)p.h;
+    for (int c = threadIdx.x * 4; c < p.cols; c += blockDim.x * 4) {
+        const int g = c / size;
+        const auto quad = [&](const float * q) { return *reinterpret_cast<const float4 *>(q + c); };
+        float4 u[BACK + N], tw[BACK + 1];              // inputs: place k - BACK of the item
+        const float4 w = quad(p.w);
+#pragma unroll
+        for (int j = 0; j <= BACK; ++j) tw[j] = quad(p.taps_w + (size_t)j * p.cols);
+#pragma unroll
+        for (int k = 0; k < BACK + N; ++k) {
+            const int i = k - BACK;
+            u[k] = make_float4(0, 0, 0, 0);
+            if (i >= n) continue;
+            if (i + before >= 0) u[k] = quad(p.x + (size_t)(t0 + i) * p.cols);
+            else if (head && !fresh) u[k] = quad(state + (size_t)k * p.cols);
+        }
+#pragma unroll
+        for (int k = 0; k < BACK + N; ++k) {
+            const int r = k - BACK + before;
+            if (r < 0 || r >= n_a) continue;
+            const float f = scale[r * p.groups + g];
+            u[k] = make_float4(u[k].x * f * w.x, u[k].y * f * w.y, u[k].z * f * w.z, u[k].w * f * w.w);
+        }
+#pragma unroll
+        for (int i = 0; i < N; ++i) {
+            if (i >= n) break;
+            float4 v = u[BACK + i];
+#pragma unroll
+            for (int j = 0; j <= BACK; ++j) {
+                const float4 q = u[i + j];
+                v = make_float4(fmaf(tw[j].x, q.x, v.x), fmaf(tw[j].y, q.y, v.y), fmaf(tw[j].z, q.z, v.z), fmaf(tw[j].w, q.w, v.w));
+            }
+            const float o[4] = {v.x, v.y, v.z, v.w};
+            store4(h + (p.ol ? pi_ol_index(t0 + i, c) : (size_t)(t0 + i) * p.ld + c), o, true, 4);
+        }
+        if (!head || BACK == 0) continue;
+#pragma unroll
+        for (int s = 0; s < BACK; ++s) {
+            const int i = len - BACK + s;              // place in the run
+            float4 v = make_float4(0, 0, 0, 0);
+            if (i >= n) {
+                const float f = scale[(n_a + i - tail) * p.groups + g];
+                const float4 q = quad(p.x + (size_t)(run0 + i) * p.cols);
+                v = make_float4(q.x * f * w.x, q.y * f * w.y, q.z * f * w.z, q.w * f * w.w);
+            } else {
+#pragma unroll
+                for (int k = 0; k < BACK + N; ++k) if (k == BACK + i) v = u[k];
+            }
+            *reinterpret_cast<float4 *>(state + (size_t)s * p.cols + c) = v;
+        }
+    }
+}
+template <typename ST> bool launch_conv_quads(const pi_conv_norm & p, int rows, size_t lds, hipStream_t st) {
+    if ((p.cols / p.groups) % 4 || p.ld % 4 || p.slot_ld % 4 || p.taps > 5) return false;
+    const dim3 grid(p.n_items), block(p.cols > 2048 ? 1024 : p.cols > 1024 ? 512 : 256);
+    switch (p.taps) {
+        case 1: hipLaunchKernelGGL((conv_norm_quads_kernel<ST, 0, 4>), grid, block, lds, st, p, rows); break;
+        case 2: hipLaunchKernelGGL((conv_norm_quads_kernel<ST, 1, 4>), grid, block, lds, st, p, rows); break;
+        case 3: hipLaunchKernelGGL((conv_norm_quads_kernel<ST, 2, 4>), grid, block, lds, st, p, rows); break;
+        case 4: hipLaunchKernelGGL((conv_norm_quads_kernel<ST, 3, 4>), grid, block, lds, st, p, rows); break;
+        default: hipLaunchKernelGGL((conv_norm_quads_kernel<ST, 4, 4>), grid, block, lds, st, p, rows);
+    }
+    return true;
 }
 
 }  // namespace
@@ -186,11 +263,13 @@ int pi_k_conv_norm(int type, const pi_conv_norm * p, pi_stream_t stream) {
         return pi::fail(PI_E_ARG, "pi_k_conv_norm: bad arguments");
     if (p->ol && (type != PI_TYPE_BF16 || p->T > kBtMaxT || p->ld % 8)) return pi::fail(PI_E_ARG, "pi_k_conv_norm: operand layout needs BF16, T <= 16, ld % 8 == 0");
     const int rows = conv_rows(pi_k_conv_tokens(p->T, p->taps), p->taps);
-    const size_t lds = sizeof(float) * ((size_t)rows * p->groups + group_parts(rows, p->groups, 4) + 4);
+    const size_t lds = sizeof(float) * ((size_t)rows * p->groups + group_parts(rows, p->groups, 16) + 16);
     if (lds > 64 * 1024) return pi::fail(PI_E_UNSUPPORTED, "pi_k_conv_norm: taps x groups");
-    if (type == PI_TYPE_BF16) hipLaunchKernelGGL(conv_norm_kernel<bf16>, dim3(p->n_items), dim3(256), lds, (hipStream_t)stream, *p, rows);
-    else if (type == PI_TYPE_F32) hipLaunchKernelGGL(conv_norm_kernel<float>, dim3(p->n_items), dim3(256), lds, (hipStream_t)stream, *p, rows);
-    else return pi::fail(PI_E_UNSUPPORTED, "pi_k_conv_norm: type");
+    if (type != PI_TYPE_BF16 && type != PI_TYPE_F32) return pi::fail(PI_E_UNSUPPORTED, "pi_k_conv_norm: type");
+    hipStream_t st = (hipStream_t)stream;
+    if (type == PI_TYPE_BF16 ? launch_conv_quads<bf16>(*p, rows, lds, st) : launch_conv_quads<float>(*p, rows, lds, st)) return pi::check_launch("pi_k_conv_norm");
+    if (type == PI_TYPE_BF16) hipLaunchKernelGGL(conv_norm_kernel<bf16>, dim3(p->n_items), dim3(256), lds, st, *p, rows);
+    else hipLaunchKernelGGL(conv_norm_kernel<float>, dim3(p->n_items), dim3(256), lds, st, *p, rows);
     return pi::check_launch("pi_k_conv_norm");
 }
 

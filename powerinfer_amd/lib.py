@@ -70,7 +70,7 @@ class GqaAttn(C.Structure):
 
 
 class GqaMix(C.Structure):
-    _fields_ = [("a", _vp), ("talk", _vp), ("z", _vp)] + [(n, C.c_int32) for n in ("ldz", "off_gate", "T", "n_head", "n_kv", "vdim")] + [("att", _vp), ("ld_att", C.c_int32)]
+    _fields_ = [("a", _vp), ("talk", _vp), ("z", _vp)] + [(n, C.c_int32) for n in ("ldz", "off_gate", "T", "n_head", "n_kv", "vdim")] + [("att", _vp), ("ld_att", C.c_int32), ("tokens", _vp), ("n_tokens", C.c_int32)]
 
 
 class Linear(C.Structure):
@@ -264,6 +264,9 @@ _SIGS = {
     "pi_k_gqa_shift": (_i, [_i, _vp, _i, _i, _i, _i, C.c_double, _i, _vp, _vp]),
     "pi_k_gqa_shift_table": (_i, [_i, _vp, _i, _i, _i, _i, _vp, _i, _vp, _vp]),
     "pi_k_gqa_mix": (_i, [_i, C.POINTER(GqaMix), _vp]),
+    "pi_k_gqa_talk_tokens": (_i, [_i, _i, _i, _i]),
+    "pi_k_gqa_stats": (_i, [C.POINTER(GqaAttn), _vp, _vp]),
+    "pi_k_gqa_talk": (_i, [C.POINTER(GqaAttn), C.POINTER(GqaMix), _vp, _vp, _i, _vp]),
     "pi_k_rope_angles_table": (_i, [_vp, _i, _i, _vp, C.c_double, _vp, _vp]),
     "pi_k_route_scores": (_i, [_vp, _i, _i, _i, _vp, _vp, _vp]),
     "pi_k_expert_up_step": (_i, [_vp, _i, _i, _i, _f, _f, _i, _i, _vp, _i, _vp, _vp, _i, _vp, _i, _vp]),

@@ -54,7 +54,7 @@ def layer_tensors(d, t, i, keeps_values):
     p, x, bf, f32 = f"l{i}.", f"l{i}.mix.", as_bf16, as_f32
     yield "attn_norm", f32(t[p + "norm1"])
     yield "attn_norm_after", f32(t[p + "norm1b"])
-    yield "mix_conv", f32(t[p + "canon1"])
+    yield "mix_conv", np.ascontiguousarray(f32(t[p + "canon1"]).T)
     for role in ("q", "k", "v"):
         yield "mix_" + role, bf(t[x + role])
     if d.get("head_mix"):

@@ -181,6 +181,8 @@ class PlainModel:
         return {k[len(prefix):]: v for k, v in self.t.items() if k.startswith(prefix)}
 
     def turn(self, kind, x, pos, rot):
+        if not rot:
+            return x
         s = rot.get("scaling")
         if kind == "attention":
             return rotate_halves(x, pos, wavelength_frequencies(rot["dims"], rot["base"], s) if s else plain_frequencies(rot["dims"], rot["base"]))
