@@ -697,12 +697,13 @@ PI_API int    pi_k_gqa_attn_parts(const pi_gqa_attn * p, pi_stream_t stream);
 typedef struct pi_gqa_mix {
     const float * a, * talk, * z; int32_t ldz, off_gate, T, n_head, n_kv, vdim; void * att; int32_t ld_att;
     const int32_t * tokens; int32_t n_tokens;                    /* optional: these tokens only */
+    float * parts; int32_t n_parts;                              /* pi_k_gqa_talk with items in up to n_parts parts: [n_parts][T][n_head][vdim] */
 } pi_gqa_mix;
 PI_API int    pi_k_gqa_mix(int type, const pi_gqa_mix * p, pi_stream_t stream);
 /* The same for long runs (bf16) without a result per pair of heads: pi_k_gqa_stats leaves every row's log2 of its soft-max denominator in stats [T][n_head]
  * (attn: wide work items, its sinks, soft cap and window), pi_k_gqa_talk forms the weights again, mixes them (mix: talk, gate and att) and applies them.  items
- * [n_items] of four integers: {first token, tokens, sequence, 0}, consecutive tokens of one sequence, at most pi_k_gqa_talk_tokens (0: sizes that are
- * not supported).  talk is rounded to bf16. */
+ * [n_items] of four integers: {first token, tokens, sequence, part + 65536 * parts}, consecutive tokens of one sequence, at most pi_k_gqa_talk_tokens (0:
+ * sizes that are not supported), with the given part of their cells; the later items start first.  talk is rounded to bf16. */
 PI_API int    pi_k_gqa_talk_tokens(int n_head, int n_kv, int dim, int vdim);
 PI_API int    pi_k_gqa_stats(const pi_gqa_attn * attn, float * stats, pi_stream_t stream);
 PI_API int    pi_k_gqa_talk(const pi_gqa_attn * attn, const pi_gqa_mix * mix, const float * stats, const int32_t * items, int n_items, pi_stream_t stream);

@@ -21,6 +21,7 @@ constexpr long long kExpandedValues = 1LL << 29;      // most expanded key and v
 constexpr int kItemRows = 32;             // query rows of an attention work item
 constexpr int kAttnItems = 512;          // (work item, part) pairs a split attention aims at: two workgroups per compute unit
 constexpr int kWideRows = 64;            // query rows from which a run of grouped-query attention takes the wide work items
+constexpr int kTalkCells = 256;          // fewest cells of a part of such an item
 constexpr int kTalkItems = 32;           // items from which pi_k_gqa_talk fills enough of the device (fewer: the cells of an item are split)
 constexpr int kLinearChunked = 17;       // tokens from which a run of linear attention is worked in chunks
 constexpr int kFreshSteps = 4;           // first tokens of a sequence that a norm over every head's sums is sensitive to (see layers_step)
@@ -95,7 +96,11 @@ struct Rotation {
 // values of a key row)
 // window > 0: cells a token sees
 // talk_tokens: tokens of an item of pi_k_gqa_talk (0: that does not serve these heads)
-struct HeadKind { int mixer, n_head, n_kv, dim, rot_dim, vdim, rank_ld, kd, window, talk_tokens; };
+// (grouped-query attention: n_head query heads per group, n_kv groups, or pairs of a group and whose values its heads meet)
+struct HeadKind {
+    int mixer, n_head, n_kv, dim, rot_dim, vdim, rank_ld, kd, window, talk_tokens;
+    int value_groups() const { int g = 1; while ((g + 1) * (g + 1) <= n_kv) ++g; return g; }      // (where n_kv counts pairs)
+};
 enum Family { kTwoNorms, kOneNorm, kPostNorm, kBothNorms };
 
 // where a pass finds its tokens
@@ -1007,13 +1012,15 @@ int both_norms_layer(pi_model * m, Layer & L, const LayerRun & r, const Step & i
         pi_gqa_mix x{};
         x.a = s->heads; x.talk = L.talk; x.z = s->z; x.ldz = L.z_rows; x.off_gate = L.off_head_gate; x.T = T; x.n_head = d.n_head; x.n_kv = d.n_kv_head; x.vdim = d.vdim;
         x.att = s->att; x.ld_att = L.close_ld;
+        if (talk.n > 0) { x.tokens = apart.items; x.n_tokens = apart.n; }
+        if (talk.n == 0 || apart.n > 0) PI_TRY(pi_k_gqa_mix(type, &x, st));
         if (talk.n > 0) {
+            if (talk.parts > d.n_kv_head) return pi::fail(PI_E_ARG, "attention: more parts than there is room for");
             const pi_gqa_attn a = gqa_args(m, L, r.pass, in, in.wide[L.hc], 1);
+            x.tokens = nullptr; x.n_tokens = 0; x.parts = s->heads; x.n_parts = talk.parts;      // (s->heads has room for n_kv parts, and is free again)
             PI_TRY(pi_k_gqa_stats(&a, s->stats, st));
             PI_TRY(pi_k_gqa_talk(&a, &x, s->stats, talk.items, talk.n, st));
-            x.tokens = apart.items; x.n_tokens = apart.n;
         }
-        if (talk.n == 0 || apart.n > 0) PI_TRY(pi_k_gqa_mix(type, &x, st));
     }
     pi_layer_out o{};
     o.rows = D; o.T = T; o.out = s->mix;
@@ -1178,6 +1185,27 @@ void talk_items(const int32_t * seq, const int32_t * n_vis, int n, const HeadKin
             for (int t = t0; t < t1; ++t) others.push_back(t);
         t0 = t1;
     }
+}
+
+// Items {first token, tokens, sequence, 0} of pi_k_gqa_talk from place `at` on, in up to max_parts parts each, so that none has much more than a compute unit's
+// share of the cells; by falling cells from the end, where the device begins.  Returns the most parts of an item.
+int split_talk_items(std::vector<int32_t> & items, size_t at, const int32_t * n_vis, int max_parts) {
+    struct Item { int32_t v[4]; long long cells; };
+    std::vector<Item> all;
+    long long total = 0;
+    for (size_t k = at; k < items.size(); k += 4) total += n_vis[items[k] + items[k + 1] - 1];
+    const long long share = std::max<long long>(kTalkCells, total / std::max(pi::compute_units(), 1) + 1);
+    int most = 1;
+    for (size_t k = at; k < items.size(); k += 4) {
+        const long long n = n_vis[items[k] + items[k + 1] - 1];
+        const int parts = (int)std::max<long long>(1, std::min<long long>((n + share - 1) / share, max_parts));
+        most = std::max(most, parts);
+        for (int j = 0; j < parts; ++j) all.push_back({{items[k], items[k + 1], items[k + 2], parts > 1 ? parts << 16 | j : 0}, n / parts});
+    }
+    std::stable_sort(all.begin(), all.end(), [](const Item & a, const Item & b) { return a.cells < b.cells; });
+    items.resize(at);
+    for (const Item & i : all) items.insert(items.end(), i.v, i.v + 4);
+    return most;
 }
 
 // span: the most cells a work item sees
@@ -1527,13 +1555,15 @@ int layers_step(pi_model * m, const int32_t * tokens, const int32_t * positions,
         begin_wide.push_back(wide.size());
         items.insert(items.end(), wide.begin(), wide.end());
         std::vector<size_t> at_talk, at_apart;
-        std::vector<int> n_talk, n_apart;
+        std::vector<int> n_talk, n_apart, talk_parts;
         std::vector<int32_t> others;
         for (const HeadKind & h : s->kinds) {
             at_talk.push_back(items.size()); at_apart.push_back(others.size());
             if (h.talk_tokens > 0 && T > 16) talk_items(seq.data() + t0, vis.data() + t0, T, h, items, others);
             n_talk.push_back((int)(items.size() - at_talk.back()) / 4);
             if (n_talk.back() < kTalkItems) { items.resize(at_talk.back()); others.resize(at_apart.back()); n_talk.back() = 0; }
+            talk_parts.push_back(n_talk.back() > 0 ? split_talk_items(items, at_talk.back(), vis.data() + t0, h.value_groups()) : 1);
+            n_talk.back() = (int)(items.size() - at_talk.back()) / 4;
             n_apart.push_back((int)(others.size() - at_apart.back()));
         }
         const size_t at_conv = items.size();
@@ -1618,7 +1648,7 @@ int layers_step(pi_model * m, const int32_t * tokens, const int32_t * positions,
             wd.parts = gqa_parts(wd.n * hk.n_kv, gqa_span(hk, vmax, true), 512);
             in.wide.push_back(wd);
             Step::Work talk, apart;
-            talk.items = s->d_in + 8 * T + at_talk[k]; talk.n = n_talk[k];
+            talk.items = s->d_in + 8 * T + at_talk[k]; talk.n = n_talk[k]; talk.parts = talk_parts[k];
             apart.items = s->d_in + 8 * T + at_others + at_apart[k]; apart.n = n_apart[k];
             in.talk.push_back(talk); in.apart.push_back(apart);
             in.first.push_back(at_first[k] < 0 ? nullptr : s->d_in + 8 * T + at_first[k]);

@@ -370,7 +370,13 @@ __global__ __launch_bounds__(64 * kTalkGroups) void gqa_talk_kernel(pi_gqa_attn 
     const int4 item = items[n_items - 1 - (int)blockIdx.x];       // the last items see the most cells
     const int tok0 = item.x, n_tok = item.y, per = p.n_head / p.n_kv, tpt = 16 / per;      // tokens of a tile
     const int32_t * list = p.lists + (size_t)item.z * p.list_ld;
-    const int n_keys = p.n_vis[tok0 + n_tok - 1], n_all = p.n_vis[tok0], lo_a = first_cell(p, tok0), lo_z = first_cell(p, tok0 + n_tok - 1);
+    const int n_all = p.n_vis[tok0], lo_z = first_cell(p, tok0 + n_tok - 1), parts = min(item.w >> 16, x.n_parts), part = item.w & 0xffff;
+    int lo_a = first_cell(p, tok0), n_keys = p.n_vis[tok0 + n_tok - 1];
+    if (parts > 1) {                                              // this part's cells
+        const int each = ((n_keys - lo_a + parts - 1) / parts + 31) / 32 * 32;
+        lo_a = min(lo_a + part * each, n_keys);
+        n_keys = min(lo_a + each, n_keys);
+    }
     const uint16_t * cache = (const uint16_t *)p.cache + (size_t)g * 2 * HD;
     if (p.n_kv & 1)                                               // the missing group of the last pair: zeros
         for (int k = threadIdx.x; k < 2 * U * 64; k += blockDim.x) ws[((k >> 6) * groups + p.n_kv) * 64 + (k & 63)] = pi_u32x4{0, 0, 0, 0};
@@ -494,6 +500,17 @@ __global__ __launch_bounds__(64 * kTalkGroups) void gqa_talk_kernel(pi_gqa_attn 
         const int tl = u * tpt + i / per, head = g * per + i % per;
         if (i >= tpt * per || tl >= n_tok) continue;
         const int t = tok0 + tl;
+        if (parts > 1) {                                          // (gated by gqa_talk_sum_kernel)
+            if (part >= parts) continue;
+            float * out = x.parts + (((size_t)part * x.T + t) * p.n_head + head) * x.vdim;
+#pragma unroll
+            for (int v = 0; v < VT; ++v) {
+                const int col = v * 16 + 4 * gq;
+                const float w[4] = {o[u][v][0], o[u][v][1], o[u][v][2], o[u][v][3]};
+                if (col < x.vdim) store4(out + col, w, (x.vdim & 3) == 0, x.vdim - col);
+            }
+            continue;
+        }
         const float f = x.off_gate >= 0 ? sigmoid_f32(x.z[(size_t)t * x.ldz + x.off_gate + head]) : 1.0f;
         bf16 * out = (bf16 *)x.att + (size_t)t * x.ld_att + head * x.vdim;
 #pragma unroll
@@ -501,6 +518,31 @@ __global__ __launch_bounds__(64 * kTalkGroups) void gqa_talk_kernel(pi_gqa_attn 
             const int col = v * 16 + 4 * gq;
             const float w[4] = {o[u][v][0] * f, o[u][v][1] * f, o[u][v][2] * f, o[u][v][3] * f};
             if (col < x.vdim) store4(out + col, w, quads && col + 4 <= x.vdim, x.vdim - col);
+        }
+    }
+}
+
+// the sum of the parts of split items, with the heads' gates: a workgroup per (item, token of it)
+__global__ __launch_bounds__(256) void gqa_talk_sum_kernel(pi_gqa_mix x, const int4 * __restrict__ items) {
+    const int4 item = items[blockIdx.x];
+    const int parts = min(item.w >> 16, x.n_parts), n = x.n_head * x.vdim;
+    if (parts <= 1 || (item.w & 0xffff) != 0 || (int)blockIdx.y >= item.y) return;
+    const int t = item.x + blockIdx.y;
+    const float * a = x.parts + (size_t)t * n, * gate = x.off_gate >= 0 ? x.z + (size_t)t * x.ldz + x.off_gate : nullptr;
+    bf16 * out = (bf16 *)x.att + (size_t)t * x.ld_att;
+    const size_t step = (size_t)x.T * n;
+    if (((x.vdim | x.ld_att) & 3) == 0) {
+        for (int e = threadIdx.x * 4; e < n; e += 1024) {
+            float4 s = make_float4(0, 0, 0, 0);
+            for (int k = 0; k < parts; ++k) { const float4 v = *reinterpret_cast<const float4 *>(a + k * step + e); s.x += v.x; s.y += v.y; s.z += v.z; s.w += v.w; }
+            const float f = gate ? sigmoid_f32(gate[e / x.vdim]) : 1.0f, w[4] = {s.x * f, s.y * f, s.z * f, s.w * f};
+            store4(out + e, w, true, 4);
+        }
+    } else {
+        for (int e = threadIdx.x; e < n; e += 256) {
+            float s = 0.0f;
+            for (int k = 0; k < parts; ++k) s += a[k * step + e];
+            out[e] = (bf16)(gate ? s * sigmoid_f32(gate[e / x.vdim]) : s);
         }
     }
 }
@@ -513,6 +555,7 @@ template <int KS> int launch_talk(const pi_gqa_attn * p, const pi_gqa_mix * x, c
         raised = true;
     }
     hipLaunchKernelGGL(gqa_talk_kernel<KS>, dim3(n), dim3(64 * p->n_kv), lds, st, *p, *x, stats, (const int4 *)items, n);
+    if (x->n_parts > 1) hipLaunchKernelGGL(gqa_talk_sum_kernel, dim3(n, kTalkTiles * (16 / (p->n_head / p->n_kv))), dim3(256), 0, st, *x, (const int4 *)items);
     return pi::check_launch("pi_k_gqa_talk");
 }
 
@@ -565,43 +608,57 @@ __global__ __launch_bounds__(256) void gqa_attn_f32_kernel(pi_gqa_attn p) {
     if (tid < p.vdim) ((float *)p.att)[p.all_values ? (size_t)blockIdx.x * p.vdim + tid : (size_t)t * p.ld_att + h * p.vdim + tid] = acc / l * p.out_scale;
 }
 
-// heads mixed behind an attention with all_values: a thread per value of a key / value head, its query heads eight at a time
+// heads mixed behind an attention with all_values: 64 values of the key / value heads a workgroup, a quarter of the heads a wave, the query heads of a value's
+// group eight at a time
+constexpr int kMixAhead = 8, kMixHeads = 128;          // heads a wave requests together; most heads
+__host__ __device__ inline int mix_groups(int n_kv, int vdim) { return min(n_kv, 63 / vdim + 2); }      // groups that 64 values can belong to
 template <typename ST>
 __global__ __launch_bounds__(256) void gqa_mix_kernel(pi_gqa_mix p) {
-    extern __shared__ __align__(16) float talk[];
-    const int t = p.tokens ? p.tokens[blockIdx.x] : blockIdx.x, per = p.n_head / p.n_kv, n = p.n_kv * p.vdim;
-    if (p.talk) {
-        for (int i = threadIdx.x; i < p.n_head * p.n_head; i += 256) talk[i] = p.talk[i];
-        __syncthreads();
-    }
-    const int e = blockIdx.y * 256 + threadIdx.x;
-    if (e >= n) return;
-    const int kv = e / p.vdim, c = e % p.vdim;
+    extern __shared__ __align__(16) float talk[];      // the rows of the heads of those groups
+    __shared__ float sum[4][8][64];
+    const int t = p.tokens ? p.tokens[blockIdx.x] : blockIdx.x, per = p.n_head / p.n_kv, n = p.n_kv * p.vdim, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int e0 = blockIdx.y * 64, e = min(e0 + lane, n - 1), kv = e / p.vdim, c = e % p.vdim, kv0 = e0 / p.vdim, each = (p.n_head + 3) / 4;
+    const int lo = min(wave * each, p.n_head), hi = min(lo + each, p.n_head);
     const float * a = p.a + (size_t)t * p.n_head * n + e;
+    float v[kMixAhead];
+    const auto fetch = [&](int g0) {
+#pragma unroll
+        for (int j = 0; j < kMixAhead; ++j) v[j] = g0 + j < hi ? a[(size_t)(g0 + j) * n] : 0.0f;
+    };
+    if (p.talk) {
+        fetch(lo);
+        const int rows = (min(e0 + 63, n - 1) / p.vdim - kv0 + 1) * per;
+        for (int i = threadIdx.x; i < rows * p.n_head; i += 256) talk[i] = p.talk[kv0 * per * p.n_head + i];
+    }
+    __syncthreads();
     const float * gate = p.off_gate >= 0 ? p.z + (size_t)t * p.ldz + p.off_gate : nullptr;
     ST * out = (ST *)p.att + (size_t)t * p.ld_att;
     for (int h0 = 0; h0 < per; h0 += 8) {
         float s[8] = {0, 0, 0, 0, 0, 0, 0, 0};
         if (p.talk) {
-            for (int g0 = 0; g0 < p.n_head; g0 += 8) {          // eight heads requested together
-                float v[8];
+            for (int g0 = lo; g0 < hi; g0 += kMixAhead) {
+                if (h0 > 0 || g0 > lo) fetch(g0);
 #pragma unroll
-                for (int j = 0; j < 8; ++j) v[j] = a[(size_t)min(g0 + j, p.n_head - 1) * n];
+                for (int k = 0; k < 8; ++k) {
+                    const float * row = talk + (size_t)((kv - kv0) * per + min(h0 + k, per - 1)) * p.n_head + g0;
 #pragma unroll
-                for (int j = 0; j < 8; ++j) {
-                    if (g0 + j >= p.n_head) break;
-#pragma unroll
-                    for (int k = 0; k < 8; ++k) s[k] = fmaf(talk[(kv * per + min(h0 + k, per - 1)) * p.n_head + g0 + j], v[j], s[k]);
+                    for (int j = 0; j < kMixAhead; ++j) s[k] = g0 + j < hi ? fmaf(row[j], v[j], s[k]) : s[k];
                 }
             }
-        } else {
+        } else if (wave == 0) {
 #pragma unroll
             for (int k = 0; k < 8; ++k) s[k] = a[(size_t)(kv * per + min(h0 + k, per - 1)) * n];
         }
+        if (h0 > 0) __syncthreads();                   // the last eight heads' sums have been read
 #pragma unroll
-        for (int k = 0; k < 8; ++k) {
-            const int h = kv * per + h0 + k;
-            if (h0 + k < per) out[h * p.vdim + c] = to_st<ST>(gate ? s[k] * sigmoid_f32(gate[h]) : s[k]);
+        for (int k = 0; k < 8; ++k) sum[wave][k][lane] = s[k];
+        __syncthreads();
+#pragma unroll
+        for (int q = 0; q < 2; ++q) {
+            const int k = wave + 4 * q, h = kv * per + h0 + k;
+            if (h0 + k >= per || e0 + lane >= n) continue;
+            const float r = (sum[0][k][lane] + sum[1][k][lane]) + (sum[2][k][lane] + sum[3][k][lane]);
+            out[h * p.vdim + c] = to_st<ST>(gate ? r * sigmoid_f32(gate[h]) : r);
         }
     }
 }
@@ -728,7 +785,7 @@ int pi_k_gqa_stats(const pi_gqa_attn * p, float * stats, pi_stream_t stream) {
 int pi_k_gqa_talk(const pi_gqa_attn * p, const pi_gqa_mix * x, const float * stats, const int32_t * items, int n_items, pi_stream_t stream) {
     if (!p || !x || !p->q || !p->cache || !p->lists || !p->n_vis || !stats || !items || n_items <= 0 || p->window < 0 || !pi_k_gqa_talk_tokens(p->n_head, p->n_kv, p->dim, p->vdim) ||
         p->hd != pi_k_gqa_head_ld(PI_TYPE_BF16, p->dim, p->vdim) || !x->att || x->vdim != p->vdim || x->ld_att < p->n_head * p->vdim ||
-        (x->off_gate >= 0 && (!x->z || x->off_gate + p->n_head > x->ldz)))
+        (x->off_gate >= 0 && (!x->z || x->off_gate + p->n_head > x->ldz)) || x->n_head != p->n_head || x->n_kv != p->n_kv || x->n_parts < 0 || (x->n_parts > 1 && (!x->parts || x->T != p->T)))
         return pi::fail(PI_E_ARG, "pi_k_gqa_talk: bad arguments");
     hipStream_t st = (hipStream_t)stream;
     switch (p->hd) {
@@ -743,10 +800,16 @@ int pi_k_gqa_mix(int type, const pi_gqa_mix * p, pi_stream_t stream) {
     if (!p || !p->a || !p->att || p->T <= 0 || p->n_head <= 0 || p->n_kv <= 0 || p->n_head % p->n_kv || p->vdim <= 0 || p->ld_att < p->n_head * p->vdim ||
         (p->off_gate >= 0 && (!p->z || p->off_gate + p->n_head > p->ldz)))
         return pi::fail(PI_E_ARG, "pi_k_gqa_mix: bad arguments");
-    const size_t lds = p->talk ? sizeof(float) * p->n_head * p->n_head : 0;
+    const size_t lds = p->talk ? sizeof(float) * mix_groups(p->n_kv, p->vdim) * (p->n_head / p->n_kv) * p->n_head : 0;
     if (p->tokens && p->n_tokens <= 0) return pi::fail(PI_E_ARG, "pi_k_gqa_mix: bad arguments");
-    const dim3 grid(p->tokens ? p->n_tokens : p->T, (p->n_kv * p->vdim + 255) / 256);
-    if (lds > 64 * 1024 || grid.y > 65535) return pi::fail(PI_E_UNSUPPORTED, "pi_k_gqa_mix: up to 128 heads");
+    const dim3 grid(p->tokens ? p->n_tokens : p->T, (p->n_kv * p->vdim + 63) / 64);
+    if (p->n_head > kMixHeads || grid.y > 65535) return pi::fail(PI_E_UNSUPPORTED, "pi_k_gqa_mix: up to 128 heads");
+    static bool raised = false;
+    if (!raised) {
+        PI_HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void *>(&gqa_mix_kernel<bf16>), hipFuncAttributeMaxDynamicSharedMemorySize, kMixHeads * kMixHeads * (int)sizeof(float)));
+        PI_HIP_TRY(hipFuncSetAttribute(reinterpret_cast<const void *>(&gqa_mix_kernel<float>), hipFuncAttributeMaxDynamicSharedMemorySize, kMixHeads * kMixHeads * (int)sizeof(float)));
+        raised = true;
+    }
     if (type == PI_TYPE_BF16) hipLaunchKernelGGL(gqa_mix_kernel<bf16>, grid, dim3(256), lds, (hipStream_t)stream, *p);
     else if (type == PI_TYPE_F32) hipLaunchKernelGGL(gqa_mix_kernel<float>, grid, dim3(256), lds, (hipStream_t)stream, *p);
     else return pi::fail(PI_E_UNSUPPORTED, "pi_k_gqa_mix: type");

@@ -70,7 +70,8 @@ class GqaAttn(C.Structure):
 
 
 class GqaMix(C.Structure):
-    _fields_ = [("a", _vp), ("talk", _vp), ("z", _vp)] + [(n, C.c_int32) for n in ("ldz", "off_gate", "T", "n_head", "n_kv", "vdim")] + [("att", _vp), ("ld_att", C.c_int32), ("tokens", _vp), ("n_tokens", C.c_int32)]
+    _fields_ = [("a", _vp), ("talk", _vp), ("z", _vp)] + [(n, C.c_int32) for n in ("ldz", "off_gate", "T", "n_head", "n_kv", "vdim")] + [("att", _vp), ("ld_att", C.c_int32), ("tokens", _vp), ("n_tokens", C.c_int32),
+        ("parts", _vp), ("n_parts", C.c_int32)]
 
 
 class Linear(C.Structure):

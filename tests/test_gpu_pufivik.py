@@ -210,6 +210,25 @@ def test_a_decoded_token_beside_a_long_prompt(make, compute):
     m.close()
 
 
+@pytest.mark.parametrize("groups", [1, 2, 4])
+def test_prompts_of_many_cells(groups):
+    """Prompts whose later tokens' cells are shared out between workgroups, in one step and with a start that has been read already."""
+    def make():
+        f = moe(6, 2, 32)
+        return config(96, 120, [talking(4, groups, 32, 24, f, original=300), capped(4, groups, 32, 24, 20.0, f), talking(4, groups, 40, 24)], groups=3)
+
+    make.__name__ = f"many_cells_{groups}"
+    orc = Oracle(make, pl.BF16)
+    toks = tokens(orc.cfg, 1100, 3)
+    m = model(orc, pl.BF16, n_ctx=1200)
+    st = serve.Stepper(m, 1200)
+    for cuts in ([0, 1100], [0, 300, 1099, 1100]):
+        got = np.vstack([st.run([("r", toks[a:b], list(range(b - a)))])[0] for a, b in zip(cuts, cuts[1:])])
+        check(got, orc, toks, pl.BF16)
+        st.end("r")
+    m.close()
+
+
 def looking_model(layer):
     """One layer whose attention makes token 32 + k look for token 42 + k and for nothing else."""
     rng = np.random.default_rng(0)

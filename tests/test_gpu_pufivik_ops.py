@@ -197,10 +197,10 @@ def test_queries_cells_and_mixed_values(t, T, pairs, H, G, dim, vdim, rot):
 
 
 # ---- attention ----------------------------------------------------------------------------------------------------------------------
-def attend(t, seqs, H, G, dim, vdim, route, parts=1, wide=0, scale=None, cap=0.0, sinks=None, talk=None, gate=True, spike=(), seed=0, blind=False):
+def attend(t, seqs, H, G, dim, vdim, route, parts=1, wide=0, scale=None, cap=0.0, sinks=None, talk=None, gate=True, spike=(), seed=0, blind=False, split=1):
     """seqs: (tokens of the step, cells before them) per sequence, on scattered cells.  route: "own" (a head meets its own group's values), "all" (every
     group's, then the mixture) or "passes" (soft-max denominators first, then weights mixed as they are formed).  spike: (sequence, token,
-    cell, head) whose score stands out.  Returns (got, want) [T, H, vdim]; blind: the oracle does not see the spikes' keys."""
+    cell, head) whose score stands out.  split: parts of an item's cells, for the passes.  Returns (got, want) [T, H, vdim]; blind: the oracle does not see the spikes' keys."""
     L, rng = pl.init(), np.random.default_rng(seed)
     hd, per, T = L.pi_k_gqa_head_ld(t, dim, vdim), H // G, sum(n for n, _ in seqs)
     scale = dim ** -0.5 if scale is None else scale
@@ -220,7 +220,7 @@ def attend(t, seqs, H, G, dim, vdim, route, parts=1, wide=0, scale=None, cap=0.0
         rows, step = n * per, L.pi_k_gqa_rows(wide)
         work += [[at, r, min(step, rows - r), s] for r in range(0, rows, step)]
         if route == "passes":
-            items += [[at + i, min(most, n - i), s, 0] for i in range(0, n, most)]
+            items += [[at + i, min(most, n - i), s, split << 16 | j if split > 1 and i % (2 * most) == 0 else 0] for i in range(0, n, most) for j in range(split if i % (2 * most) == 0 else 1)]
         seq_of += [s] * n
         vis += list(range(b + 1, b + n + 1))
         k, v = cache[cells][:, :, 0, :dim].astype(np.float64), cache[cells][:, :, 1, :vdim].astype(np.float64)
@@ -245,7 +245,8 @@ def attend(t, seqs, H, G, dim, vdim, route, parts=1, wide=0, scale=None, cap=0.0
     m = filled(pl.GqaMix, a=heads, talk=tb, z=zb, ldz=H + 9, off_gate=4 if gate else -1, T=T, n_head=H, n_kv=G, vdim=vdim, att=att, ld_att=ld)
     if route == "passes":
         assert most > 0
-        stats, ib = pl.DevBuf.zeros(4 * T * H), i32(items)
+        stats, ib, some = pl.DevBuf.zeros(4 * T * H), i32(items), pl.DevBuf(4 * split * T * H * vdim)
+        m.parts, m.n_parts = some.ptr, split
         pl.check(L.pi_k_gqa_stats(C.byref(a), stats.ptr, None))
         pl.check(L.pi_k_gqa_talk(C.byref(a), C.byref(m), stats.ptr, ib.ptr, len(items), None))
     else:
@@ -289,18 +290,18 @@ def test_a_sink_per_head(t, parts, wide):
 
 
 @pytest.mark.parametrize("t,parts,wide", WAYS)
-@pytest.mark.parametrize("H,G,dim,vdim", SHAPES + [(2, 2, 256, 250), (18, 9, 32, 32)])
+@pytest.mark.parametrize("H,G,dim,vdim", SHAPES + [(2, 2, 256, 250), (18, 9, 32, 32), (128, 1, 16, 10), (100, 50, 8, 2)])
 def test_mixed_heads(t, parts, wide, H, G, dim, vdim):
     talk, sinks = mixture(H)
     near(*attend(t, LONG if wide else SHORT, H, G, dim, vdim, "all", parts, wide, sinks=sinks, talk=talk), t)
 
 
-@pytest.mark.parametrize("cap,sink,gate", [(0.0, True, True), (0.0, False, False), (1.5, True, True)])
+@pytest.mark.parametrize("cap,sink,gate,split", [(0.0, True, True, 1), (0.0, False, False, 2), (1.5, True, True, 5)])
 @pytest.mark.parametrize("H,G,dim,vdim", SHAPES)
-def test_mixed_heads_in_two_passes(H, G, dim, vdim, cap, sink, gate):
+def test_mixed_heads_in_two_passes(H, G, dim, vdim, cap, sink, gate, split):
     talk, sinks = mixture(H)
     seqs = LONG + [(2, 0), (1, 0), (33, 500), (1, 31), (5, 32)]
-    near(*attend(pl.BF16, seqs, H, G, dim, vdim, "passes", 1, 1, cap=cap, sinks=sinks if sink else None, talk=talk, gate=gate), pl.BF16, 2)
+    near(*attend(pl.BF16, seqs, H, G, dim, vdim, "passes", 1, 1, cap=cap, sinks=sinks if sink else None, talk=talk, gate=gate, split=split), pl.BF16, 2)
 
 
 def test_sizes_two_passes_do_not_take():
@@ -319,6 +320,8 @@ def test_one_key_among_hundreds(t, parts, wide, route):
     kw = dict(scale=64 ** -0.5, sinks=sinks, talk=talk, spike=spike)
     got, want = attend(t, [(n, 400)], 4, 2, 64, 64, route, parts, wide, **kw)
     near(got, want, t, 2)
+    if route == "passes":
+        near(attend(t, [(n, 400)], 4, 2, 64, 64, route, parts, wide, split=3, **kw)[0], want, t, 2)
     _, blind = attend(t, [(n, 400)], 4, 2, 64, 64, route, parts, wide, blind=True, **kw)
     assert (np.abs(blind - want)[:6].max(axis=(1, 2)) > 0.3).all()
 
