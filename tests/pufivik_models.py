@@ -44,9 +44,9 @@ def odd_config():
 
 # sizes like those of larger models
 def even_config():
-    f = moe(16, 4, 64)
-    t, c = talking(8, 2, 64, 64, f, base=50000.0, original=128), capped(8, 2, 64, 64, 30.0, f, original=256)
-    return config(192, 200, [t, c, c, t, dict(c, mlp=None)], groups=4, taps=4, mult=0.7)
+    f = moe(12, 4, 64)
+    t, c = talking(16, 4, 64, 64, f, base=50000.0, original=128), capped(16, 4, 64, 64, 25.0, f, original=256)
+    return config(256, 200, [t, c, c, t, dict(c, mlp=None)], groups=8, taps=4, mult=0.6)
 
 
 # the remaining head sizes of the kernels, one group of keys for many heads and one for each, a long convolution

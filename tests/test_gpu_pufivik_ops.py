@@ -162,7 +162,7 @@ def test_shifted_keys_with_given_frequencies(t, pairs):
 @pytest.mark.parametrize("t", TYPES)
 @pytest.mark.parametrize("T", [6, 33])
 @pytest.mark.parametrize("pairs", [0, 1])
-@pytest.mark.parametrize("H,G,dim,vdim,rot", [(6, 2, 40, 24, 24), (5, 1, 17, 33, 6), (4, 4, 128, 128, 64), (3, 3, 2, 1, 2), (8, 2, 96, 32, 48), (2, 1, 256, 200, 256)])
+@pytest.mark.parametrize("H,G,dim,vdim,rot", [(6, 2, 40, 24, 24), (5, 1, 17, 33, 6), (4, 4, 128, 128, 64), (3, 3, 2, 1, 2), (8, 4, 96, 40, 32), (2, 1, 256, 200, 256)])
 def test_queries_cells_and_mixed_values(t, T, pairs, H, G, dim, vdim, rot):
     """A layer that keeps its values, then one that mixes them into its own; rotations longer than one."""
     L, rng = pl.init(), np.random.default_rng(dim + T)
